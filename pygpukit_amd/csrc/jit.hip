@@ -111,6 +111,7 @@ pgk_status pgk_jit_compile(const char* source, const char* name, const char* con
         opts.push_back(options[i]);
     }
     if (!has_arch) opts.push_back("--offload-arch=gfx950");
+    for (const char* o : {"-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops"}) opts.push_back(o);   // as the Makefile: no packed fp32
     r = rtc().compile(prog, (int)opts.size(), opts.data());
     Program* p = new Program();
     size_t n = 0;

@@ -352,10 +352,9 @@ pgk_status pgk_fill(void* dst, double value, size_t n, pgk_dtype dt, pgk_stream 
 // ------------------------------------------------------------ streams / events / graphs ----
 pgk_status pgk_stream_create(pgk_stream* out, int high_priority) {
     PGK_REQUIRE(out, "pgk_stream_create: null output");
-    int lo = 0, hi = 0;
-    PGK_CHECK_HIP(hipDeviceGetStreamPriorityRange(&lo, &hi));
+    (void)high_priority;   // a scheduling hint only: every stream is created at the default priority (streams of different priorities can stall each other here)
     hipStream_t s = nullptr;
-    PGK_CHECK_HIP(hipStreamCreateWithPriority(&s, hipStreamNonBlocking, high_priority ? hi : lo));
+    PGK_CHECK_HIP(hipStreamCreateWithFlags(&s, hipStreamNonBlocking));
     {
         Pool& P = pool();
         std::lock_guard<std::mutex> lk(P.mu);
