@@ -346,6 +346,24 @@ pgk_status pgk_sdpa_fixed_cache(const void* q, const void* k_cache, const void* 
                                 int q_len, int max_seq, int d, float scale, int h_context_len,
                                 const int32_t* ctx_buf, void* workspace, pgk_dtype dt, pgk_stream s);
 
+/* ---------------------------------------------- layer-list operators (ops_latent.hip) */
+/* out[row] = x / sqrt(mean(x^2) + eps) * weight: fp32 rows and weight, result in out_dt */
+pgk_status pgk_rmsnorm_f32(const float* x, const float* weight, void* out, int rows, int cols, float eps, pgk_dtype out_dt,
+                           pgk_stream s);
+/* x[row] += mult * y / sqrt(mean(y^2) + eps) * weight: fp32 stream, sublayer output y in y_dt */
+pgk_status pgk_rmsnorm_add_f32(float* x, const void* y, const float* weight, int rows, int cols, float eps, float mult,
+                               pgk_dtype y_dt, pgk_stream s);
+/* Sliding-window causal attention: q [q_len, hq, dk], k [kv_len, hkv, dk], v [kv_len, hkv, dv] -> out [q_len, hq, dv]; query i is
+ * position kv_len - q_len + i and sees the `window` positions that end with its own.  gate (or NULL): [q_len rows of gate_stride
+ * elements][hq], the head's output is multiplied by sigmoid(gate). */
+pgk_status pgk_window_attention(const void* q, const void* k, const void* v, void* out, int hq, int hkv, int q_len, int kv_len,
+                                int dk, int dv, float scale, int window, const void* gate, int64_t gate_stride, pgk_dtype dt,
+                                pgk_stream s);
+/* x[row][head][:] *= sigmoid(gate[row][head]) in place */
+pgk_status pgk_head_gate(void* x, const void* gate, int rows, int heads, int d, int64_t gate_stride, pgk_dtype dt, pgk_stream s);
+/* dst [dst_rows, dst_cols] = src [rows, cols] with zeros around it */
+pgk_status pgk_pad_2d(const void* src, void* dst, int rows, int cols, int dst_rows, int dst_cols, pgk_dtype dt, pgk_stream s);
+
 /* ---------------------------------------------------------------------- engine ------ */
 /* Native decode/prefill launcher: one C call (or one hipGraph launch) per token step instead of
  * ~21 Python-dispatched launches per layer.  Replaces the device-dispatch half
@@ -376,6 +394,31 @@ typedef struct {
 
 pgk_status pgk_engine_create(const pgk_model_config_t* cfg, const void* embed, const void* lm_head,
                              const void* final_norm, const pgk_layer_weights_t* layers, pgk_engine* out);
+/* Layer-list decoders (csrc/engine_stack.hip): fp32 residual stream, norm before and after each sublayer, sliding-window latent
+ * attention with a per-head output gate, dense SwiGLU or no feed-forward; every layer has its own sizes.  dtype PGK_BF16 or PGK_F32
+ * is the element type of the tables, matrices, activations and the latent cache; norm weights are fp32 with any offset applied.
+ * Caller pads with zeros: Wp = width up to a multiple of 64, head_pad >= dim and vdim (64, 128 or a larger multiple of 64),
+ * rank_pad and ff_pad multiples of 64 (ff_pad 0: the layer has no feed-forward), n_in a multiple of 64. */
+typedef struct {
+    int vocab_size, width, num_layers, max_positions, max_seq_len, max_batch;
+    float norm_eps, residual_mult;
+    pgk_dtype dtype;
+} pgk_stack_config_t;
+typedef struct {
+    int heads, dim, vdim, rank, window;            /* true sizes; window: keys a query sees, itself included */
+    int head_pad, rank_pad, n_in, ff_pad;
+    float scale;
+    const float *norm1, *norm1b, *norm2, *norm2b;  /* [Wp] */
+    const void* w_in;                              /* [n_in, Wp]: heads x head_pad query rows, rank_pad latent rows, heads gate rows */
+    const float* c_norm;                           /* [rank_pad] */
+    const void* w_ukv;                             /* [2 heads head_pad, rank_pad]: key rows, then value rows */
+    const void* w_o;                               /* [Wp, heads head_pad] */
+    const void* w_gate_up;                         /* [2 ff_pad, Wp] */
+    const void* w_down;                            /* [Wp, ff_pad] */
+} pgk_stack_layer_t;
+/* embed [vocab, width], pos_embed [max_positions, width] or NULL, head [vocab, Wp], final_norm [Wp] */
+pgk_status pgk_engine_create_stack(const pgk_stack_config_t* cfg, const void* embed, const void* pos_embed, const void* head,
+                                   const float* final_norm, const pgk_stack_layer_t* layers, pgk_engine* out);
 pgk_status pgk_engine_destroy(pgk_engine e);
 /* bytes the engine allocated from the pool (KV caches, activations, rope tables) */
 pgk_status pgk_engine_bytes(pgk_engine e, size_t* kv_bytes, size_t* workspace_bytes);
@@ -384,6 +427,12 @@ pgk_status pgk_engine_bytes(pgk_engine e, size_t* kv_bytes, size_t* workspace_by
  * [n,V]) may be NULL. */
 pgk_status pgk_engine_prefill(pgk_engine e, int seq, const int32_t* h_tokens, int n, int start_pos,
                               void* all_logits, float* h_last_logits, pgk_stream s);
+/* Several sequences in one call: sequence i brings h_lens[i] tokens for slot h_slots[i] from position h_starts[i] on (tokens
+ * concatenated in that order).  h_want: ascending row indices into the concatenation whose fp32 logits are copied to h_logits
+ * [n_want][V].  QKV + RoPE engines run the sequences one after another and give last rows only; layer-list engines run all
+ * rows as one ragged batch and give any row. */
+pgk_status pgk_engine_prefill_batch(pgk_engine e, int n_seqs, const int32_t* h_slots, const int32_t* h_lens, const int32_t* h_starts,
+                                    const int32_t* h_tokens, int n_want, const int32_t* h_want, float* h_logits, pgk_stream s);
 /* Set the per-sequence decode state (token to feed, its position) for `batch` sequences. */
 pgk_status pgk_engine_set_state(pgk_engine e, const int32_t* h_tokens, const int32_t* h_positions, int batch,
                                 pgk_stream s);

@@ -46,6 +46,16 @@ class LayerWeights(C.Structure):
                                           "mlp_norm", "w_gate_up", "s_gate_up", "w_down", "s_down")]
 
 
+class StackConfig(C.Structure):
+    _fields_ = [(n, C.c_int) for n in ("vocab_size", "width", "num_layers", "max_positions", "max_seq_len", "max_batch")] + \
+               [("norm_eps", C.c_float), ("residual_mult", C.c_float), ("dtype", C.c_int)]
+
+
+class StackLayer(C.Structure):
+    _fields_ = [(n, C.c_int) for n in ("heads", "dim", "vdim", "rank", "window", "head_pad", "rank_pad", "n_in", "ff_pad")] + [("scale", C.c_float)] + \
+               [(n, C.c_void_p) for n in ("norm1", "norm1b", "norm2", "norm2b", "w_in", "c_norm", "w_ukv", "w_o", "w_gate_up", "w_down")]
+
+
 # name -> (argtypes); every function returns pgk_status (int) unless listed in _NON_STATUS
 _V, _I, _F, _Z, _D, _I64 = C.c_void_p, C.c_int, C.c_float, C.c_size_t, C.c_double, C.c_int64
 _PROTOS = {
@@ -101,6 +111,11 @@ _PROTOS = {
     "pgk_engine_create": [C.POINTER(ModelConfig), _V, _V, _V, C.POINTER(LayerWeights), c_void_pp],
     "pgk_engine_destroy": [_V], "pgk_engine_bytes": [_V, C.POINTER(_Z), C.POINTER(_Z)],
     "pgk_engine_prefill": [_V, _I, c_i32_p, _I, _I, _V, C.POINTER(_F), _V],
+    "pgk_engine_prefill_batch": [_V, _I, c_i32_p, c_i32_p, c_i32_p, c_i32_p, _I, c_i32_p, C.POINTER(_F), _V],
+    "pgk_engine_create_stack": [C.POINTER(StackConfig), _V, _V, _V, _V, C.POINTER(StackLayer), c_void_pp],
+    "pgk_rmsnorm_f32": [_V, _V, _V, _I, _I, _F, _I, _V], "pgk_rmsnorm_add_f32": [_V, _V, _V, _I, _I, _F, _F, _I, _V],
+    "pgk_window_attention": [_V, _V, _V, _V, _I, _I, _I, _I, _I, _I, _F, _I, _V, _I64, _I, _V],
+    "pgk_head_gate": [_V, _V, _I, _I, _I, _I64, _I, _V], "pgk_pad_2d": [_V, _V, _I, _I, _I, _I, _I, _V],
     "pgk_engine_set_state": [_V, c_i32_p, c_i32_p, _I, _V], "pgk_engine_decode_step": [_V, _I, _V],
     "pgk_engine_profile_step": [_V, _I, _I, C.POINTER(_F), C.POINTER(_I), _V],
     "pgk_engine_timeline": [_V, _I, _I, C.POINTER(C.c_uint64), _I, C.POINTER(_I), _V],
@@ -137,14 +152,17 @@ def load():
             f"libpgk_hip.so not found at {LIB_PATH}: build it with `python -c 'import __graft_entry__ as g; g.build()'` "
             "(or `make -C pygpukit_amd/csrc`). pygpukit_amd has no CPU fallback.")
     lib = C.CDLL(LIB_PATH)
+    # a library built from a subset of the sources (`make serve-stack`) lacks some entry points: calling one of those raises
     for name, argtypes in _PROTOS.items():
-        fn = getattr(lib, name)
-        fn.argtypes = argtypes
-        fn.restype = C.c_int
+        fn = getattr(lib, name, None)
+        if fn is not None:
+            fn.argtypes = argtypes
+            fn.restype = C.c_int
     for name, (argtypes, restype) in _NON_STATUS.items():
-        fn = getattr(lib, name)
-        fn.argtypes = argtypes
-        fn.restype = restype
+        fn = getattr(lib, name, None)
+        if fn is not None:
+            fn.argtypes = argtypes
+            fn.restype = restype
     _lib = lib
     return lib
 
@@ -152,7 +170,10 @@ def load():
 def call(name: str, *args):
     """Invoke a status-returning entry point; raise PgkError with the library's message on failure."""
     lib = load()
-    st = getattr(lib, name)(*args)
+    fn = getattr(lib, name, None)
+    if fn is None:
+        raise PgkError(f"{name} is not in {LIB_PATH}: this library was built from a subset of the sources; build the whole one")
+    st = fn(*args)
     if st != 0:
         msg = lib.pgk_last_error()
         raise PgkError(f"{name} failed (status {st}): {msg.decode(errors='replace') if msg else ''}")

@@ -22,20 +22,12 @@
 //
 // Prefill runs the MFMA GEMM / flash-attention kernels on bf16 activations with an fp32 residual stream.
 
-#include <cstdlib>
-#include <type_traits>
-#include <vector>
-
 #include "attn_core.hip.h"
-#include "engine_common.hip.h"
+#include "engine_state.hip.h"
 #include "gemm_epilogues.hip.h"
 #include "pkgemm.hip.h"
 
 namespace pgk {
-
-constexpr int SHORT_CTX = 512;   // contexts up to here take the whole-context attention kernels (direct batch attention); one sequence: SHORT_CTX_B1
-constexpr int SHORT_CTX_B1 = 384; // a single sequence's fused attention + o_proj kernel walks the context in chunks of 192 rows (AM_CHUNK) in EVERY one of its
-                                  // 256 workgroups: two chunks still beat the split-KV sequence (context 300: 0.616 vs 0.625 ms per step), three do not (400: 0.678 vs 0.627)
 
 pgk_status engine_gemm_nt(const bf16* A, const void* W, const bf16* wscale, bool fp8, void* C, bool accum_f32, int M,
                           int N, int K, hipStream_t st, bool packed = false);      // packed: W = the fragment-major bf16 copy
@@ -414,91 +406,6 @@ __global__ void embed_kernel(const bf16* embed, const int32_t* tokens, float* h,
         cur_cos[(size_t)b * half + i] = rope_cos[(size_t)pos * half + i];
         cur_sin[(size_t)b * half + i] = rope_sin[(size_t)pos * half + i];
     }
-}
-
-// token[b] = argmax over workgroup partials (ties -> lowest index); position[b] += 1; log the token;
-// h[b] = E[token] for the next step; the last workgroup of the step's last chunk bumps the step counter.
-// One workgroup per sequence (grid = M).  Every workgroup reads the step counter before it takes an arrival ticket
-// (step_counter[1]); the bump is made by whoever draws the last ticket, so it cannot overtake a read.  (One workgroup
-// for the whole chunk, a wave per sequence, took 25 us at M = 8 and 57 us at M = 16 - a dependent walk per sequence.)
-__global__ __launch_bounds__(256) void finalize_kernel(unsigned long long* tl, const float* amax_val, const int* amax_idx, int nblk,
-                                                       int32_t* tokens, int32_t* positions, int32_t* token_log,
-                                                       int32_t* step_counter, int log_width, int log_cap,
-                                                       const bf16* embed, float* h, int H, int bump,
-                                                       unsigned long long* clk_log, const float* rope_cos,
-                                                       const float* rope_sin, float* cur_cos, float* cur_sin, int half,
-                                                       int max_seq, int M, const int32_t* sampled) {
-    const TLStamp tls(tl);
-    __shared__ float sv[4];
-    __shared__ int si[4];
-    __shared__ int s_tok, s_pos;
-    const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6, b = blockIdx.x;
-    const int step = step_counter[0];
-    int bi;
-    if (sampled) {
-        bi = sampled[b];                                  // temperature / top-k / top-p draw (ops_sampling.hip)
-    } else {
-        float bv = -INFINITY;
-        bi = 0x7FFFFFFF;
-        for (int i = threadIdx.x; i < nblk; i += 256) {
-            const float v = amax_val[(size_t)b * nblk + i];
-            const int ix = amax_idx[(size_t)b * nblk + i];
-            if (v > bv || (v == bv && ix < bi)) { bv = v; bi = ix; }
-        }
-#pragma unroll
-        for (int off = 32; off >= 1; off >>= 1) {
-            const float ov = __shfl_xor(bv, off, 64);
-            const int oi = __shfl_xor(bi, off, 64);
-            if (ov > bv || (ov == bv && oi < bi)) { bv = ov; bi = oi; }
-        }
-        if (lane == 0) { sv[wid] = bv; si[wid] = bi; }
-        __syncthreads();
-        bv = sv[0]; bi = si[0];
-#pragma unroll
-        for (int w = 1; w < 4; ++w)
-            if (sv[w] > bv || (sv[w] == bv && si[w] < bi)) { bv = sv[w]; bi = si[w]; }
-        if (bi == 0x7FFFFFFF) bi = 0;
-    }
-    if (threadIdx.x == 0) {
-        s_tok = bi;
-        tokens[b] = bi;
-        const int npos = positions[b] + 1;
-        positions[b] = npos;
-        s_pos = min(npos, max_seq - 1);
-        if (step < log_cap) token_log[(size_t)step * log_width + b] = bi;
-        if (b == 0 && step < log_cap && clk_log) {  // shader-clock / 100 MHz wall-clock stamps (diagnostic only)
-            clk_log[2 * (size_t)step] = __builtin_amdgcn_s_memtime();
-            clk_log[2 * (size_t)step + 1] = __builtin_amdgcn_s_memrealtime();
-        }
-    }
-    __syncthreads();
-    // next step's inputs of this sequence: its embedding row (8 bf16 per lane) and the RoPE row of its next position
-    const bf16* erow = embed + (size_t)s_tok * H;
-    float* hrow = h + (size_t)b * H;
-    if ((H & 7) == 0) {
-        for (int v = threadIdx.x; v < (H >> 3); v += 256) {
-            const uint4 raw = *reinterpret_cast<const uint4*>(erow + v * 8);
-            float f[8];
-            WTraits<bf16>::decode(raw, f);
-            *reinterpret_cast<float4*>(hrow + v * 8) = make_float4(f[0], f[1], f[2], f[3]);
-            *reinterpret_cast<float4*>(hrow + v * 8 + 4) = make_float4(f[4], f[5], f[6], f[7]);
-        }
-    } else {
-        for (int i = threadIdx.x; i < H; i += 256) hrow[i] = to_f(erow[i]);
-    }
-    for (int i = threadIdx.x; i < half; i += 256) {
-        cur_cos[(size_t)b * half + i] = rope_cos[(size_t)s_pos * half + i];
-        cur_sin[(size_t)b * half + i] = rope_sin[(size_t)s_pos * half + i];
-    }
-    if (bump && threadIdx.x == 0) {
-        if (M == 1) {
-            step_counter[0] = step + 1;
-        } else if (atomicAdd(&step_counter[1], 1) == M - 1) {   // every workgroup has read `step` before its own ticket
-            atomicExch(&step_counter[1], 0);
-            step_counter[0] = step + 1;
-        }
-    }
-    tls.end();
 }
 
 // --------------------------------------------------------------------------------------------
@@ -1530,81 +1437,6 @@ __global__ void bf16_rows_to_f32_kernel(const bf16* in, float* out, size_t n) {
     for (size_t i = blockIdx.x * (size_t)blockDim.x + threadIdx.x; i < n; i += stride) out[i] = to_f(in[i]);
 }
 
-// --------------------------------------------------------------------------------------------
-thread_local Probe* g_probe = nullptr;   // measurement hooks: engine_common.hip.h
-
-struct Engine {
-    pgk_model_config_t cfg;
-    const bf16 *embed, *lm_head, *final_norm;
-    std::vector<pgk_layer_weights_t> layers;
-    int nsplit = 1, lm_blocks = 1, lm_cap = 1, log_cap = 4096;
-    bool batched_mfma = true;   // chunks of 3 and 5..16 sequences use engine_batched.hip.h (PGK_BATCHED_MFMA=0: GEMV kernels only, =2: from 3 up)
-    int batched_min = 5, batched_max = 64;   // PGK_BATCHED_MAX=16: chunks of at most 16 sequences (one weight pass per chunk), the A/B switch of the tiled kernels
-    int cu_count = 256;
-    bool short_path = true;     // contexts <= SHORT_CTX take the whole-context attention kernels (PGK_FUSED_ATTN=0: the split-KV sequence at every context)
-    int pos_hi = -1;            // host-side upper bound of the largest position the next step sees (-1: unknown); selects the sequence, see step_is_short
-    // in-graph stochastic sampling (pgk_engine_set_sampling): temperature <= 0 keeps greedy argmax
-    float sample_temperature = 0.f, sample_top_p = 1.f;
-    int sample_top_k = 0, u_cap = 0, u_alloc_rows = 0;   // u_cap: rows in use (ring length); u_alloc_rows: rows allocated
-    float* u_ring = nullptr;       // [u_cap][max_batch] uniforms, row = step counter % u_cap
-    void* sample_scratch = nullptr;   // top-k candidate keys (ops_sampling.hip), sized for max_batch rows
-    size_t sample_scratch_cap = 0;
-    int32_t* sampled = nullptr;    // [max_batch]
-    bool fused_attn = false;   // one sequence at short context: attn + o_proj in one kernel (bf16 W_o, shapes that tile)
-    bool attn_mfma = false;    // ... with Q.K^T and P.V on the matrix pipe from LDS-staged K/V (head_dim 128; PGK_ATTN_MFMA=0: the dot2 kernels); also the whole-context
-                               // batch attention while its workgroups (96 KB of LDS: one per CU) fit one round - batch x Hkv <= CUs (beyond: attn_decode_kernel, batch 64 1.258 vs 1.316 ms)
-    bool merged_oproj = false; // long contexts / fp8 W_o, one or two sequences: split-KV merge + o_proj in one kernel (PGK_MERGED_OPROJ=0: merge kernel + GEMV)
-    int moproj_rows = 32;
-    int oproj_rows = 32;       // W_o rows per workgroup on the fused path
-    // device state
-    bf16 *kcache = nullptr, *vcache = nullptr;
-    float *rope_cos = nullptr, *rope_sin = nullptr, *cur_cos = nullptr, *cur_sin = nullptr;
-    int32_t *tokens = nullptr, *positions = nullptr, *token_log = nullptr, *step_counter = nullptr;
-    bf16 *act16 = nullptr, *attnv16 = nullptr;   // batched MFMA path: bf16 hand-off of SwiGLU output and attention output
-    bf16* x16 = nullptr;                         // 17..64 sequences: the next RMSNorm's input rows in bf16 (layer 0: normalised by norm_rows_bf16; then un-normalised, written by o_proj / down)
-    float* ss_part = nullptr;                    // ... and its statistic: per-workgroup sums of squares [64][1024]
-    float *h = nullptr, *h2 = nullptr, *qkv = nullptr, *part = nullptr, *opart = nullptr, *attnv = nullptr, *act = nullptr, *logits = nullptr,
-          *amax_val = nullptr;
-    int* amax_idx = nullptr;
-    unsigned long long* clk_log = nullptr;
-    size_t kv_bytes = 0, ws_bytes = 0;
-    // fragment-major copies of the layer weights for prompts of <= 128 tokens (ops_pkgemm.hip); PGK_PACKED_PREFILL=0: none
-    struct PackedLayer { bf16 *qkv = nullptr, *o = nullptr, *gate_up = nullptr, *down = nullptr; };
-    std::vector<PackedLayer> packed;
-    bool packed_ok = false;     // the skinny-GEMM kernels of ops_pkgemm.hip can use the copy (their shape limits)
-    bool packed_have = false;   // the copy exists (w8a16 engines: also for shapes beyond those kernels - the long-prompt GEMMs read it)
-    size_t packed_bytes = 0;
-    bool packed_resid = false;      // o_proj / down_proj without K split, carrying the next RMSNorm (pkgemm_resid_nt); PGK_PACKED_RESID=0: split-K slabs + norm launches
-    float* pk_ss = nullptr;         // its sum-of-squares table [128][PK_SS_LD]
-    bf16* packed_lm = nullptr;      // fragment-major lm_head for the batched (3..64 sequences) lm_head kernels; PGK_PACKED_LMHEAD=0: none
-    float* dec_slabs = nullptr;     // 17..64 sequences on the packed kernels: split-K slabs of o_proj / down_proj [splits][M][H] (PGK_PACKED_DECODE=0: engine_batched kernels)
-    bool packed_decode = false;
-    // prefill workspace (grown on demand, outside capture)
-    void* pf = nullptr;
-    size_t pf_bytes = 0;
-    int32_t* pf_tokens = nullptr;
-    int pf_tokens_cap = 0;
-    // captured step: [0] the long-context launch sequence, [1] the short-context one (when the engine has both)
-    // captured steps: tier 0 = the short-context sequence (span 0); the others = the split-KV sequence with its slices cut for
-    // contexts up to `span` positions (1024, 2048, ... and the cache length).  pgk_engine_replay picks per step (pick_tier).
-    struct Tier { int span = 0; hipGraph_t graph = nullptr; hipGraphExec_t exec = nullptr; int launches = 0; };
-    std::vector<Tier> tiers;
-    int graph_batch = 0;
-    int step_span = 0;          // the split-KV slicing of the step being enqueued (launch_attn); 0: the whole cache
-    int launches_per_step = 0;
-    std::vector<void*> allocs;
-
-    size_t kv_layer_elems() const { return (size_t)cfg.max_batch * cfg.num_kv_heads * cfg.max_seq_len * cfg.head_dim; }
-    int qkv_dim() const { return (cfg.num_heads + 2 * cfg.num_kv_heads) * cfg.head_dim; }
-};
-
-static pgk_status dev_alloc(Engine* e, void** p, size_t bytes, size_t* acct) {
-    pgk_status r = pgk_malloc(p, bytes);
-    if (r != PGK_OK) return r;
-    e->allocs.push_back(*p);
-    if (acct) *acct += bytes;
-    return PGK_OK;
-}
 
 
 template <class WT, class XT, int M, int R, int PRO, int EPI, int C>
@@ -1779,18 +1611,6 @@ static pgk_status launch_attn(Engine* e, int layer, int b0, int m, bool fused, b
     return PGK_OK;
 }
 
-// One decode step for sequences [b0, b0+M); `last` = this is the step's last chunk (bumps the step counter)
-pgk_status sample_rows_ring(const float* logits, int rows, int vocab, float temperature, int top_k, float top_p, const float* u_ring,
-                            int u_cap, int u_stride, const int32_t* step_counter, int32_t* out, void* scratch, hipStream_t st);
-size_t sample_scratch_bytes(int rows, int vocab, int top_k, float top_p);
-
-// one draw per sequence of the chunk from the fp32 logits the lm_head kernel just wrote; the uniform numbers come from
-// the device ring row (step counter % u_cap), so a captured graph replays with fresh randomness the host queued up
-static pgk_status engine_sample(Engine* e, int b0, int M, hipStream_t st) {
-    return sample_rows_ring(e->logits + (size_t)b0 * e->cfg.vocab_size, M, e->cfg.vocab_size, e->sample_temperature, e->sample_top_k,
-                            e->sample_top_p, e->u_ring + b0, e->u_cap, e->cfg.max_batch, e->step_counter, e->sampled + b0, e->sample_scratch, st);
-}
-
 // One decode step for sequences [b0, b0+M); `last` = this is the step's last chunk (bumps the step counter).
 // `short_ctx`: every sequence of the step has at most SHORT_CTX positions - a single sequence then takes the fused
 // attention + o_proj kernel (4 L + 2 launches); otherwise split-KV slices + merge/o_proj (5 L + 2).  Both are correct at
@@ -1877,11 +1697,11 @@ static pgk_status decode_chunk(Engine* e, int b0, bool last, hipStream_t st, int
         sampled = e->sampled + b0;
         *launches += 1;
     }
-    PGK_CHECK_HIP(launch_k(finalize_kernel, dim3(M), dim3(256), 0, st, e->amax_val + (size_t)b0 * e->lm_blocks, e->amax_idx + (size_t)b0 * e->lm_blocks,
+    PGK_CHECK_HIP(launch_k(finalize_kernel<bf16>, dim3(M), dim3(256), 0, st, e->amax_val + (size_t)b0 * e->lm_blocks, e->amax_idx + (size_t)b0 * e->lm_blocks,
                                        e->lm_blocks, e->tokens + b0, e->positions + b0, e->token_log + b0, e->step_counter,
                                        e->cfg.max_batch, e->log_cap, e->embed, h, H, last ? 1 : 0, b0 == 0 ? e->clk_log : nullptr,
                                        e->rope_cos, e->rope_sin, e->cur_cos + (size_t)b0 * (D / 2), e->cur_sin + (size_t)b0 * (D / 2),
-                                       D / 2, c.max_seq_len, M, sampled));
+                                       D / 2, c.max_seq_len, M, sampled, (const bf16*)nullptr, H));
     *launches += 2;
     return PGK_OK;
 }
@@ -1974,10 +1794,10 @@ static pgk_status decode_chunk_batched(Engine* e, int b0, int M, bool last, hipS
         sampled = e->sampled + b0;
         *launches += 1;
     }
-    PGK_CHECK_HIP(launch_k(finalize_kernel, dim3(M), dim3(256), 0, st, a.amax_val, a.amax_idx, nblk, e->tokens + b0, e->positions + b0, e->token_log + b0, e->step_counter,
+    PGK_CHECK_HIP(launch_k(finalize_kernel<bf16>, dim3(M), dim3(256), 0, st, a.amax_val, a.amax_idx, nblk, e->tokens + b0, e->positions + b0, e->token_log + b0, e->step_counter,
                                        e->cfg.max_batch, e->log_cap, e->embed, h, H, last ? 1 : 0, b0 == 0 ? e->clk_log : nullptr,
                                        e->rope_cos, e->rope_sin, e->cur_cos + (size_t)b0 * (D / 2), e->cur_sin + (size_t)b0 * (D / 2),
-                                       D / 2, c.max_seq_len, M, sampled));
+                                       D / 2, c.max_seq_len, M, sampled, (const bf16*)nullptr, H));
     *launches += 2;
     return PGK_OK;
 }
@@ -2066,10 +1886,10 @@ static pgk_status decode_chunk_packed(Engine* e, int b0, int M, bool last, hipSt
         sampled = e->sampled + b0;
         *launches += 1;
     }
-    PGK_CHECK_HIP(launch_k(finalize_kernel, dim3(M), dim3(256), 0, st, a.amax_val, a.amax_idx, nblk, e->tokens + b0, e->positions + b0, e->token_log + b0, e->step_counter,
+    PGK_CHECK_HIP(launch_k(finalize_kernel<bf16>, dim3(M), dim3(256), 0, st, a.amax_val, a.amax_idx, nblk, e->tokens + b0, e->positions + b0, e->token_log + b0, e->step_counter,
                                        e->cfg.max_batch, e->log_cap, e->embed, h, H, last ? 1 : 0, b0 == 0 ? e->clk_log : nullptr,
                                        e->rope_cos, e->rope_sin, e->cur_cos + (size_t)b0 * (D / 2), e->cur_sin + (size_t)b0 * (D / 2),
-                                       D / 2, c.max_seq_len, M, sampled));
+                                       D / 2, c.max_seq_len, M, sampled, (const bf16*)nullptr, H));
     *launches += 3;
     return PGK_OK;
 }
@@ -2106,254 +1926,12 @@ static pgk_status decode_step(Engine* e, int batch, hipStream_t st, int* launche
     return decode_step_impl<bf16>(e, batch, st, launches, short_ctx);
 }
 
-// Which launch sequence the NEXT step takes: the short-context one while the host-side bound on the step's largest
-// position (set by pgk_engine_set_state, advanced by every step this library enqueues) stays below SHORT_CTX.  The bound
-// is a speed hint only - both sequences are correct at any context - so a caller that rewrites the device-resident
-// positions behind the library's back loses speed, never correctness; an unknown bound selects the long sequence.
-static int short_limit(int batch) { return batch == 1 ? SHORT_CTX_B1 : SHORT_CTX; }
-static bool step_is_short(const Engine* e, int batch) { return e->short_path && e->pos_hi >= 0 && e->pos_hi + 1 <= short_limit(batch); }
-
-static void drop_graphs(Engine* e) {
-    for (auto& t : e->tiers) {
-        if (t.exec) (void)hipGraphExecDestroy(t.exec);
-        if (t.graph) (void)hipGraphDestroy(t.graph);
-    }
-    e->tiers.clear();
-    e->graph_batch = 0;
-}
-
-// The split-KV slicing a step at the host-side position bound needs: the smallest of 1024, 2048, ... that covers the context, capped at
-// the cache length (an unknown bound: the cache length).
-static int span_for(const Engine* e) {
-    const int cap = e->cfg.max_seq_len;
-    if (e->pos_hi < 0) return cap;
-    int span = 1024;
-    while (span < e->pos_hi + 1 && span < cap) span *= 2;
-    return span < cap ? span : cap;
-}
-
-// The captured step the next replay takes: the short-context sequence while the position bound allows it (and it was captured),
-// otherwise the split-KV tier whose slices cover the context; both kinds are correct at any context they cover.
-static size_t pick_tier(const Engine* e) {
-    const bool has_short = !e->tiers.empty() && e->tiers[0].span == 0;
-    if (has_short && (e->tiers.size() == 1 || step_is_short(e, e->graph_batch))) return 0;
-    const int want = span_for(e);
-    for (size_t i = has_short ? 1 : 0; i < e->tiers.size(); ++i)
-        if (e->tiers[i].span >= want) return i;
-    return e->tiers.size() - 1;
-}
-
-}  // namespace pgk
-
-using namespace pgk;
-
-extern "C" {
-
-pgk_status pgk_engine_create(const pgk_model_config_t* cfg, const void* embed, const void* lm_head,
-                             const void* final_norm, const pgk_layer_weights_t* layers, pgk_engine* out) {
-    PGK_REQUIRE(cfg && embed && final_norm && layers && out, "pgk_engine_create: null argument");
-    const auto& c = *cfg;
-    PGK_REQUIRE(c.head_dim == 128 || c.head_dim == 64, "pgk_engine_create: head_dim %d not in {64,128}", c.head_dim);
-    PGK_REQUIRE(c.num_heads % c.num_kv_heads == 0, "pgk_engine_create: Hq %d %% Hkv %d", c.num_heads, c.num_kv_heads);
-    const int G = c.num_heads / c.num_kv_heads;
-    PGK_REQUIRE(G >= 1, "pgk_engine_create: GQA group %d", G);
-    PGK_REQUIRE(c.hidden_size % 16 == 0 && c.intermediate_size % 16 == 0, "pgk_engine_create: sizes must be multiples of 16");
-    PGK_REQUIRE(c.weight_format == 0 || (c.hidden_size % 128 == 0 && c.intermediate_size % 128 == 0),
-                "pgk_engine_create: fp8 weights need 128-multiple dims");
-    PGK_REQUIRE(c.max_batch >= 1 && c.max_seq_len >= 1 && c.num_layers >= 1, "pgk_engine_create: bad sizes");
-    Engine* e = new Engine();
-    e->cfg = c;
-    e->embed = (const bf16*)embed;
-    e->lm_head = (const bf16*)(lm_head ? lm_head : embed);
-    e->final_norm = (const bf16*)final_norm;
-    e->layers.assign(layers, layers + c.num_layers);
-    int nsplit = (c.max_seq_len + 63) / 64;   // ~64 cached positions per workgroup: one KV batch per wave
-    {
-        int dev = 0;
-        hipDeviceProp_t prop;
-        if (hipGetDevice(&dev) == hipSuccess && hipGetDeviceProperties(&prop, dev) == hipSuccess && prop.multiProcessorCount > 0)
-            e->cu_count = prop.multiProcessorCount;
-    }
-    e->nsplit = nsplit < 1 ? 1 : (nsplit > 64 ? 64 : nsplit);
-    e->lm_blocks = 1024;
-    // fused attention + o_proj: short contexts, bf16 W_o, and a row slicing that tiles the workgroup
-    {
-        const int gd = G * c.head_dim, rpp = 256 / (gd / 8);
-        int rows = c.hidden_size / 32;
-        while (rows > 4 * rpp && rows % 2 == 0) rows /= 2;   // <= 4 preloaded passes per workgroup
-        while (rows < rpp) rows *= 2;
-        const bool tiles = rows % rpp == 0 && c.hidden_size % rows == 0 && gd / 8 <= 64;
-        // PGK_FUSED_ATTN=0: no short-context launch sequence at all (the split-KV sequence at every context; A/B and tests)
-        const char* env = getenv("PGK_FUSED_ATTN");
-        e->short_path = env ? atoi(env) != 0 : true;
-        e->fused_attn = tiles && c.weight_format == 0 && (G == 1 || G == 2 || G == 4);
-        e->oproj_rows = rows;
-        {
-            const char* am = getenv("PGK_ATTN_MFMA");
-            e->attn_mfma = c.head_dim == 128 && !(am && atoi(am) == 0);
-        }
-        // merged o_proj (long contexts, fp8 W_o): same slicing rule with 16 codes per lane for fp8
-        const int nwt = c.weight_format != 0 ? 16 : 8, lpw = gd / nwt, rpp2 = lpw > 0 ? 256 / lpw : 256;
-        int rows2 = c.hidden_size / 32;
-        while (rows2 > 4 * rpp2 && rows2 % 2 == 0) rows2 /= 2;
-        while (rows2 < rpp2) rows2 *= 2;
-        const char* emo = getenv("PGK_MERGED_OPROJ");
-        e->merged_oproj = !(emo && atoi(emo) == 0) && (G == 1 || G == 2 || G == 4) && lpw >= 8 && lpw <= 64 && 256 % lpw == 0 &&
-                          rows2 % rpp2 == 0 && c.hidden_size % rows2 == 0 && (c.weight_format == 0 || (gd % 128 == 0 || 128 % gd == 0));
-        e->moproj_rows = rows2;
-    }
-    const int B = c.max_batch, H = c.hidden_size, D = c.head_dim;
-    pgk_status r = PGK_OK;
-    auto A = [&](void** p, size_t bytes, size_t* acct) { if (r == PGK_OK) r = dev_alloc(e, p, bytes, acct); };
-    const size_t kvb = (size_t)c.num_layers * e->kv_layer_elems() * sizeof(bf16);
-    A((void**)&e->kcache, kvb, &e->kv_bytes);
-    A((void**)&e->vcache, kvb, &e->kv_bytes);
-    A((void**)&e->rope_cos, (size_t)c.max_seq_len * (D / 2) * 4, &e->ws_bytes);
-    A((void**)&e->rope_sin, (size_t)c.max_seq_len * (D / 2) * 4, &e->ws_bytes);
-    A((void**)&e->cur_cos, (size_t)B * (D / 2) * 4, &e->ws_bytes);
-    A((void**)&e->cur_sin, (size_t)B * (D / 2) * 4, &e->ws_bytes);
-    A((void**)&e->tokens, (size_t)B * 4, &e->ws_bytes);
-    A((void**)&e->positions, (size_t)B * 4, &e->ws_bytes);
-    A((void**)&e->token_log, (size_t)e->log_cap * B * 4, &e->ws_bytes);
-    A((void**)&e->step_counter, 16, &e->ws_bytes);
-    A((void**)&e->h, (size_t)B * H * 4, &e->ws_bytes);
-    A((void**)&e->h2, (size_t)B * H * 4, &e->ws_bytes);
-    A((void**)&e->qkv, (size_t)B * e->qkv_dim() * 4, &e->ws_bytes);
-    A((void**)&e->part, (size_t)B * c.num_heads * e->nsplit * (D + 2) * 4, &e->ws_bytes);
-    A((void**)&e->opart, (size_t)B * c.num_kv_heads * H * 4, &e->ws_bytes);
-    A((void**)&e->act16, (size_t)B * c.intermediate_size * 2, &e->ws_bytes);
-    A((void**)&e->attnv16, (size_t)B * c.num_heads * c.head_dim * 2, &e->ws_bytes);
-    A((void**)&e->x16, (size_t)B * H * 2, &e->ws_bytes);
-    A((void**)&e->ss_part, (size_t)64 * 1024 * 4, &e->ws_bytes);
-    A((void**)&e->attnv, (size_t)B * c.num_heads * D * 4, &e->ws_bytes);
-    A((void**)&e->act, (size_t)B * c.intermediate_size * 4, &e->ws_bytes);
-    A((void**)&e->logits, (size_t)B * c.vocab_size * 4, &e->ws_bytes);
-    e->lm_cap = e->lm_blocks > ceil_div(c.vocab_size, 16) ? e->lm_blocks : ceil_div(c.vocab_size, 16);   // per-sequence argmax partial slots
-    {
-        const char* ev = getenv("PGK_BATCHED_MFMA");
-        e->batched_min = (ev && atoi(ev) == 2) ? 3 : 5;   // 2: from 3 up
-        // every projection's K must suit the MFMA decode kernels: K = 128 S with S in {8, 16, 24, 32} (activation
-        // fragments in registers) or an LDS image of K x 16 bf16 that fits (K <= 4096); Llama-3-8B's down_proj
-        // (K = 14336) does neither, so such models decode batches in GEMV chunks of 8 / 4 / 2 / 1
-        auto k_ok = [](int K) { return K % 128 == 0 && K <= 4096; };
-        e->batched_mfma = !(ev && atoi(ev) == 0) && k_ok(c.hidden_size) && k_ok(c.intermediate_size) && k_ok(c.num_heads * c.head_dim);
-        // 17..64 sequences in one weight pass (batched_mt_kernel) need K = 128 S with S instantiated; otherwise chunks of 16
-        auto k_tiled = [](int K) { const int s = K / 128; return K % 128 == 0 && (s == 2 || s == 4 || s == 8 || s == 16 || s == 24 || s == 32); };
-        e->batched_max = (k_tiled(c.hidden_size) && k_tiled(c.intermediate_size) && k_tiled(c.num_heads * c.head_dim)) ? 64 : 16;
-        if (const char* em = getenv("PGK_BATCHED_MAX")) { const int v = atoi(em); if (v >= 16 && v < e->batched_max) e->batched_max = v; }
-    }
-    A((void**)&e->amax_val, (size_t)B * e->lm_cap * 4, &e->ws_bytes);
-    A((void**)&e->amax_idx, (size_t)B * e->lm_cap * 4, &e->ws_bytes);
-    A((void**)&e->clk_log, (size_t)e->log_cap * 16, &e->ws_bytes);
-    {
-        // Second, fragment-major copy of the bf16 layer weights: what the short-prompt prefill streams (ops_pkgemm.hip).
-        // Costs the layers' bytes again; skipped when that is more than a quarter of the device's free memory.
-        const int QDp = c.num_heads * D, NQ = e->qkv_dim(), I = c.intermediate_size;
-        const char* ep = getenv("PGK_PACKED_PREFILL");
-        const size_t per_layer = ((size_t)NQ * H + (size_t)H * QDp + (size_t)2 * I * H + (size_t)H * I) * 2;
-        size_t free_b = 0, total_b = 0;
-        const bool fits = hipMemGetInfo(&free_b, &total_b) == hipSuccess && per_layer * c.num_layers < free_b / 4;
-        const bool shapes = pkgemm_shape_ok(NQ, H, false) && pkgemm_shape_ok(H, QDp, true) && pkgemm_shape_ok(2 * I, H, false) && pkgemm_shape_ok(H, I, true) && I % 64 == 0;
-        // bf16 layers, or fp8 codes + block scales (w8a16): the copy is bf16 either way (ops_pkgemm.hip)
-        const bool f8w = c.weight_format == 1;
-        // w8a16 engines keep the copy also where the skinny kernels cannot use it (Llama-3-8B: K = 4096 / 14336 is beyond them):
-        // their long-prompt GEMMs read it (packed_have), instead of dequantising every weight again in front of every call
-        const bool long_only = f8w && !shapes && NQ % 16 == 0 && H % 64 == 0 && QDp % 64 == 0 && I % 64 == 0;
-        if (r == PGK_OK && (c.weight_format == 0 || f8w) && (shapes || long_only) && fits && !(ep && atoi(ep) == 0)) {
-            e->packed.resize(c.num_layers);
-            hipStream_t st = resolve_stream(nullptr);
-            for (int l = 0; l < c.num_layers && r == PGK_OK; ++l) {
-                auto& P = e->packed[l];
-                const auto& L = e->layers[l];
-                A((void**)&P.qkv, (size_t)NQ * H * 2, &e->packed_bytes);
-                A((void**)&P.o, (size_t)H * QDp * 2, &e->packed_bytes);
-                A((void**)&P.gate_up, (size_t)2 * I * H * 2, &e->packed_bytes);
-                A((void**)&P.down, (size_t)H * I * 2, &e->packed_bytes);
-                if (r == PGK_OK) r = f8w ? pack_weights_fp8(L.w_qkv, L.s_qkv, P.qkv, NQ, H, st) : pack_weights_bf16(L.w_qkv, P.qkv, NQ, H, st);
-                if (r == PGK_OK) r = f8w ? pack_weights_fp8(L.w_o, L.s_o, P.o, H, QDp, st) : pack_weights_bf16(L.w_o, P.o, H, QDp, st);
-                if (r == PGK_OK) r = f8w ? pack_weights_fp8(L.w_gate_up, L.s_gate_up, P.gate_up, 2 * I, H, st) : pack_weights_bf16(L.w_gate_up, P.gate_up, 2 * I, H, st);
-                if (r == PGK_OK) r = f8w ? pack_weights_fp8(L.w_down, L.s_down, P.down, H, I, st) : pack_weights_bf16(L.w_down, P.down, H, I, st);
-            }
-            if (r == PGK_OK && hipStreamSynchronize(st) != hipSuccess) r = set_error(PGK_ERR_HIP, "pgk_engine_create: packing the prefill weights failed");
-            e->packed_have = r == PGK_OK;
-            e->packed_ok = e->packed_have && shapes;
-            if (e->packed_ok && pkgemm_resid_ok(H, QDp) && pkgemm_resid_ok(H, I)) {
-                A((void**)&e->pk_ss, (size_t)128 * PK_SS_LD * 4, &e->ws_bytes);
-                e->packed_resid = r == PGK_OK;
-            }
-            if (e->packed_ok && c.max_batch >= 3 && c.vocab_size % 16 == 0 && H % 32 == 0) {
-                A((void**)&e->packed_lm, (size_t)c.vocab_size * H * 2, &e->packed_bytes);
-                if (r == PGK_OK) r = pack_weights_bf16(e->lm_head, e->packed_lm, c.vocab_size, H, st);
-                if (r == PGK_OK && hipStreamSynchronize(st) != hipSuccess) r = set_error(PGK_ERR_HIP, "pgk_engine_create: packing the lm_head failed");
-            }
-            const char* pd = getenv("PGK_PACKED_DECODE");
-            if (e->packed_ok && c.max_batch > 16 && !(pd && atoi(pd) == 0)) {
-                A((void**)&e->dec_slabs, (size_t)16 * 64 * H * 4, &e->ws_bytes);
-                e->packed_decode = r == PGK_OK;
-            }
-        }
-    }
-    if (r != PGK_OK) { pgk_engine_destroy(e); return r; }
-    // RoPE tables in fp32, same formula as the reference (src/pygpukit/llm/layers/rope.py:13-24):
-    // freqs = 1/theta^(2i/D) in fp32, angle = float(t) * freq in fp32, cos/sin of that.
-    {
-        std::vector<float> hc((size_t)c.max_seq_len * (D / 2)), hs(hc.size());
-        for (int i = 0; i < D / 2; ++i) {
-            const float expo = (float)(2 * i) / (float)D;
-            const float freq = 1.0f / powf(c.rope_theta, expo);
-            for (int t = 0; t < c.max_seq_len; ++t) {
-                const float ang = (float)t * freq;
-                hc[(size_t)t * (D / 2) + i] = (float)cos((double)ang);
-                hs[(size_t)t * (D / 2) + i] = (float)sin((double)ang);
-            }
-        }
-        hipStream_t st = resolve_stream(nullptr);
-        hipError_t he = hipMemcpyAsync(e->rope_cos, hc.data(), hc.size() * 4, hipMemcpyHostToDevice, st);
-        if (he == hipSuccess) he = hipMemcpyAsync(e->rope_sin, hs.data(), hs.size() * 4, hipMemcpyHostToDevice, st);
-        if (he == hipSuccess) he = hipMemsetAsync(e->kcache, 0, kvb, st);
-        if (he == hipSuccess) he = hipMemsetAsync(e->vcache, 0, kvb, st);
-        if (he == hipSuccess) he = hipMemsetAsync(e->tokens, 0, (size_t)B * 4, st);
-        if (he == hipSuccess) he = hipMemsetAsync(e->positions, 0, (size_t)B * 4, st);
-        if (he == hipSuccess) he = hipMemsetAsync(e->step_counter, 0, 16, st);
-        if (he == hipSuccess) he = hipMemsetAsync(e->h, 0, (size_t)B * H * 4, st);
-        if (he == hipSuccess) he = hipStreamSynchronize(st);
-        if (he != hipSuccess) { pgk_engine_destroy(e); return set_error(PGK_ERR_HIP, "pgk_engine_create: %s", hipGetErrorString(he)); }
-    }
-    *out = e;
-    return PGK_OK;
-}
-
-pgk_status pgk_engine_destroy(pgk_engine eh) {
-    if (!eh) return PGK_OK;
-    Engine* e = (Engine*)eh;
-    drop_graphs(e);
-    for (void* p : e->allocs) (void)pgk_free(p);
-    if (e->pf) (void)pgk_free(e->pf);
-    if (e->pf_tokens) (void)pgk_free(e->pf_tokens);
-    if (e->u_ring) (void)pgk_free(e->u_ring);
-    if (e->sampled) (void)pgk_free(e->sampled);
-    if (e->sample_scratch) (void)pgk_free(e->sample_scratch);
-    delete e;
-    return PGK_OK;
-}
-
-pgk_status pgk_engine_bytes(pgk_engine eh, size_t* kv_bytes, size_t* workspace_bytes) {
-    PGK_REQUIRE(eh, "pgk_engine_bytes: null engine");
-    Engine* e = (Engine*)eh;
-    if (kv_bytes) *kv_bytes = e->kv_bytes;
-    if (workspace_bytes) *workspace_bytes = e->ws_bytes + e->pf_bytes + e->packed_bytes;
-    return PGK_OK;
-}
-
-pgk_status pgk_engine_prefill(pgk_engine eh, int seq, const int32_t* h_tokens, int n, int start_pos, void* all_logits,
-                              float* h_last_logits, pgk_stream s) {
-    PGK_REQUIRE(eh && h_tokens, "pgk_engine_prefill: null argument");
-    Engine* e = (Engine*)eh;
+static pgk_status dense_prefill(Engine* e, int seq, const int32_t* h_tokens, int n, int start_pos, void* all_logits,
+                                float* h_last_logits, hipStream_t st) {
     const auto& c = e->cfg;
     PGK_REQUIRE(seq >= 0 && seq < c.max_batch, "pgk_engine_prefill: sequence slot %d outside [0,%d)", seq, c.max_batch);
     PGK_REQUIRE(n >= 1 && start_pos >= 0 && start_pos + n <= c.max_seq_len, "pgk_engine_prefill: positions %d..%d outside cache of %d",
                 start_pos, start_pos + n, c.max_seq_len);
-    hipStream_t st = resolve_stream(s);
     // (prompts of 129..256 tokens used to run as two chunks of <= 128 through the packed-weight kernels; since the staged 128-tile
     // GEMM and the epilogue fusions of round 3 the long-prompt path is faster at every such length: 144 tokens 1.94 vs 2.38 ms,
     // 256 tokens 2.27 vs 2.62)
@@ -2590,326 +2168,215 @@ pgk_status pgk_engine_prefill(pgk_engine eh, int seq, const int32_t* h_tokens, i
     return PGK_OK;
 }
 
-pgk_status pgk_engine_set_state(pgk_engine eh, const int32_t* h_tokens, const int32_t* h_positions, int batch, pgk_stream s) {
-    PGK_REQUIRE(eh && h_tokens && h_positions, "pgk_engine_set_state: null argument");
-    Engine* e = (Engine*)eh;
-    PGK_REQUIRE(batch >= 1 && batch <= e->cfg.max_batch, "pgk_engine_set_state: batch %d outside [1,%d]", batch, e->cfg.max_batch);
-    for (int b = 0; b < batch; ++b) {
-        PGK_REQUIRE(h_tokens[b] >= 0 && h_tokens[b] < e->cfg.vocab_size, "pgk_engine_set_state: token %d out of range", h_tokens[b]);
-        PGK_REQUIRE(h_positions[b] >= 0 && h_positions[b] < e->cfg.max_seq_len, "pgk_engine_set_state: position %d outside cache of %d",
-                    h_positions[b], e->cfg.max_seq_len);
+// A sequence at a time: the prompt kernels below take one sequence's rows; logits only of a sequence's last row.
+static pgk_status dense_prefill_batch(Engine* e, int n_seqs, const int32_t* h_slots, const int32_t* h_lens, const int32_t* h_starts, const int32_t* h_tokens,
+                                      int n_want, const int32_t* h_want, float* h_logits, hipStream_t st) {
+    int row0 = 0, w = 0;
+    for (int i = 0; i < n_seqs; ++i) {
+        const int last = row0 + h_lens[i] - 1;
+        PGK_REQUIRE(w >= n_want || h_want[w] >= last, "pgk_engine_prefill_batch: this model gives the logits of a sequence's last row only");
+        float* out = (w < n_want && h_want[w] == last) ? h_logits + (size_t)w * e->cfg.vocab_size : nullptr;
+        if (pgk_status r = dense_prefill(e, h_slots[i], h_tokens + row0, h_lens[i], h_starts[i], nullptr, out, st)) return r;
+        if (out) ++w;
+        row0 += h_lens[i];
     }
-    hipStream_t st = resolve_stream(s);
-    e->pos_hi = 0;
-    for (int b = 0; b < batch; ++b) e->pos_hi = h_positions[b] > e->pos_hi ? h_positions[b] : e->pos_hi;
-    PGK_CHECK_HIP(hipMemcpyAsync(e->tokens, h_tokens, (size_t)batch * 4, hipMemcpyHostToDevice, st));
-    PGK_CHECK_HIP(hipMemcpyAsync(e->positions, h_positions, (size_t)batch * 4, hipMemcpyHostToDevice, st));
-    // the residual stream enters a step already holding the embeddings of the state tokens
+    PGK_REQUIRE(w == n_want, "pgk_engine_prefill_batch: wanted rows must be ascending last rows");
+    return PGK_OK;
+}
+
+static pgk_status dense_embed_state(Engine* e, int batch, hipStream_t st) {
     embed_kernel<<<batch, 256, 0, st>>>(e->embed, e->tokens, e->h, e->cfg.hidden_size, e->positions, e->rope_cos, e->rope_sin,
                                         e->cur_cos, e->cur_sin, e->cfg.head_dim / 2, e->cfg.max_seq_len);
     PGK_LAUNCH_CHECK();
-    PGK_CHECK_HIP(hipStreamSynchronize(st));
     return PGK_OK;
 }
 
-pgk_status pgk_engine_decode_step(pgk_engine eh, int batch, pgk_stream s) {
-    PGK_REQUIRE(eh, "pgk_engine_decode_step: null engine");
-    Engine* e = (Engine*)eh;
-    PGK_REQUIRE(batch >= 1 && batch <= e->cfg.max_batch, "pgk_engine_decode_step: batch %d outside [1,%d]", batch, e->cfg.max_batch);
-    int launches = 0;
-    e->step_span = span_for(e);
-    pgk_status r = decode_step(e, batch, resolve_stream(s), &launches, step_is_short(e, batch));
-    e->launches_per_step = launches;
-    if (e->pos_hi >= 0) ++e->pos_hi;
-    return r;
-}
-
-pgk_status pgk_engine_profile_step(pgk_engine eh, int batch, int n_iters, float* h_ms_sum, int* h_count, pgk_stream s) {
-    PGK_REQUIRE(eh && h_ms_sum && h_count, "pgk_engine_profile_step: null argument");
-    Engine* e = (Engine*)eh;
-    PGK_REQUIRE(batch >= 1 && batch <= e->cfg.max_batch && n_iters >= 1, "pgk_engine_profile_step: bad arguments");
-    hipStream_t st = resolve_stream(s);
-    for (int i = 0; i < KC_COUNT; ++i) { h_ms_sum[i] = 0.f; h_count[i] = 0; }
-    // Eager steps whose every launch carries its own start / stop event (hipExtLaunchKernelGGL): the elapsed time of a
-    // pair is the dispatch's begin -> end interval, the quantity rocprofv3 --kernel-trace reports - no launch gap, nothing
-    // subtracted.
-    Probe probe;
-    probe.timing = true;
-    pgk_status r = PGK_OK;
-    for (int it = 0; it < n_iters && r == PGK_OK; ++it) {
-        probe.used = 0;
-        probe.info.clear();
-        g_probe = &probe;
-        int launches = 0;
-        e->step_span = span_for(e);
-        r = decode_step(e, batch, st, &launches, step_is_short(e, batch));
-        g_probe = nullptr;
-        if (e->pos_hi >= 0) ++e->pos_hi;
-        if (r != PGK_OK) break;
-        hipError_t he = hipStreamSynchronize(st);
-        if (he != hipSuccess) { r = set_error(PGK_ERR_HIP, "pgk_engine_profile_step: %s", hipGetErrorString(he)); break; }
-        for (size_t i = 0; i < probe.used; ++i) {
-            float ms = 0.f;
-            const int cls = probe.cls[i];
-            if (cls >= 0 && cls < KC_COUNT && hipEventElapsedTime(&ms, probe.ev[2 * i], probe.ev[2 * i + 1]) == hipSuccess) {
-                h_ms_sum[cls] += ms;
-                h_count[cls] += 1;
-            }
-        }
-    }
-    for (hipEvent_t ev : probe.ev) (void)hipEventDestroy(ev);
-    return r;
-}
-
-// Timeline of ONE replayed step (diagnostic): the step is captured into a temporary graph with every kernel's `tl` slot
-// set, replayed `warm` times and then once more; per launch the host gets
-//   h_out[6 i .. 6 i + 5] = { kernel class (KC_*), workgroups, first start, last start, first end, last end }
-// with the four times in ticks of the 100 MHz s_memrealtime counter relative to the step's first start.  The engine's
-// own captured graph is left alone; the sequence state advances by warm + 1 real steps.
-pgk_status pgk_engine_timeline(pgk_engine eh, int batch, int warm, uint64_t* h_out, int max_launches, int* n_launches, pgk_stream s) {
-    PGK_REQUIRE(eh && h_out && n_launches && max_launches >= 1 && warm >= 0, "pgk_engine_timeline: bad arguments");
-    Engine* e = (Engine*)eh;
-    PGK_REQUIRE(batch >= 1 && batch <= e->cfg.max_batch, "pgk_engine_timeline: batch %d outside [1,%d]", batch, e->cfg.max_batch);
-    hipStream_t st = resolve_stream(s);
-    const int cap = 16 * e->cfg.num_layers + 64;
-    Probe probe;
-    probe.tl_cap = cap;
-    const size_t bytes = (size_t)cap * TL_MAXWG * 2 * sizeof(unsigned long long);
-    if (pgk_status r = pgk_malloc((void**)&probe.tl, bytes)) return r;
-    pgk_status r = PGK_OK;
-    hipGraph_t g = nullptr;
-    hipGraphExec_t ex = nullptr;
-    hipError_t he = hipMemsetAsync(probe.tl, 0, bytes, st);
-    if (he == hipSuccess) he = hipStreamSynchronize(st);
-    if (he == hipSuccess) he = hipStreamBeginCapture(st, hipStreamCaptureModeRelaxed);
-    if (he == hipSuccess) {
-        g_probe = &probe;
-        int launches = 0;
-        e->step_span = span_for(e);
-        r = decode_step(e, batch, st, &launches, step_is_short(e, batch));
-        g_probe = nullptr;
-        he = hipStreamEndCapture(st, &g);
-    }
-    if (r == PGK_OK && he == hipSuccess) he = hipGraphInstantiate(&ex, g, nullptr, nullptr, 0);
-    for (int i = 0; r == PGK_OK && he == hipSuccess && i <= warm; ++i) he = hipGraphLaunch(ex, st);
-    if (e->pos_hi >= 0) e->pos_hi += warm + 1;
-    if (r == PGK_OK && he == hipSuccess) he = hipStreamSynchronize(st);
-    const int n = (int)probe.info.size() < cap ? (int)probe.info.size() : cap;
-    if (r == PGK_OK && he == hipSuccess) {
-        std::vector<unsigned long long> host((size_t)n * TL_MAXWG * 2);
-        he = hipMemcpy(host.data(), probe.tl, host.size() * sizeof(unsigned long long), hipMemcpyDeviceToHost);
-        if (he == hipSuccess) {
-            unsigned long long origin = ~0ull;
-            std::vector<unsigned long long> agg((size_t)n * 4);
-            for (int i = 0; i < n; ++i) {
-                const int nwg = probe.info[i].nwg < TL_MAXWG ? probe.info[i].nwg : TL_MAXWG;
-                unsigned long long s0 = ~0ull, s1 = 0, e0 = ~0ull, e1 = 0;
-                for (int w = 0; w < nwg; ++w) {
-                    const unsigned long long a = host[((size_t)i * TL_MAXWG + w) * 2], b = host[((size_t)i * TL_MAXWG + w) * 2 + 1];
-                    if (a == 0 && b == 0) continue;   // slot never written
-                    s0 = a < s0 ? a : s0; s1 = a > s1 ? a : s1; e0 = b < e0 ? b : e0; e1 = b > e1 ? b : e1;
-                }
-                agg[4 * i] = s0; agg[4 * i + 1] = s1; agg[4 * i + 2] = e0; agg[4 * i + 3] = e1;
-                if (s0 < origin) origin = s0;
-            }
-#ifdef PGK_PHASE_STAMPS
-            {
-                double sum[KC_COUNT][8] = {}, cnt[KC_COUNT][8] = {}, dur[KC_COUNT] = {};
-                for (int i = 0; i < n; ++i) {
-                    const int cls = probe.info[i].cls, nwg = probe.info[i].nwg;
-                    if (cls < 0 || cls >= KC_COUNT || nwg > 256) continue;
-                    for (int w = 0; w < nwg; ++w) {
-                        const unsigned long long t0 = host[((size_t)i * TL_MAXWG + w) * 2], t1 = host[((size_t)i * TL_MAXWG + w) * 2 + 1];
-                        dur[cls] += (double)(t1 - t0);
-                        for (int k = 0; k < 8; ++k) {
-                            const unsigned long long v = host[((size_t)i * TL_MAXWG + 256 + 4 * w) * 2 + k];
-                            if (v) { sum[cls][k] += (double)(v - t0); cnt[cls][k] += 1; }
-                        }
-                    }
-                }
-                for (int cls = 0; cls < KC_COUNT; ++cls)
-                    for (int k = 0; k < 8; ++k)
-                        if (cnt[cls][k] > 0) fprintf(stderr, "phase stamps: class %d phase %d at %.2f us after its workgroup's start (n=%.0f)\n", cls, k, sum[cls][k] / cnt[cls][k] / 100.0, cnt[cls][k]);
-            }
-#endif
-            *n_launches = n < max_launches ? n : max_launches;
-            for (int i = 0; i < *n_launches; ++i) {
-                h_out[6 * i] = (uint64_t)probe.info[i].cls;
-                h_out[6 * i + 1] = (uint64_t)probe.info[i].nwg;
-                for (int k = 0; k < 4; ++k) h_out[6 * i + 2 + k] = agg[4 * i] == ~0ull ? 0 : agg[4 * i + k] - origin;
-            }
-        }
-    }
-    if (ex) (void)hipGraphExecDestroy(ex);
-    if (g) (void)hipGraphDestroy(g);
-    (void)pgk_free(probe.tl);
-    if (r != PGK_OK) return r;
-    if (he != hipSuccess) return set_error(PGK_ERR_HIP, "pgk_engine_timeline: %s", hipGetErrorString(he));
-    return PGK_OK;
-}
-
-pgk_status pgk_engine_capture(pgk_engine eh, int batch, pgk_stream s) {
-    PGK_REQUIRE(eh, "pgk_engine_capture: null engine");
-    Engine* e = (Engine*)eh;
-    PGK_REQUIRE(batch >= 1 && batch <= e->cfg.max_batch, "pgk_engine_capture: batch %d outside [1,%d]", batch, e->cfg.max_batch);
-    hipStream_t st = resolve_stream(s);
-    drop_graphs(e);
-    // tier 0: the short-context sequence; then the split-KV sequence once per context tier (1024, 2048, ... positions and the
-    // cache length) - needed whenever a context can exceed the short limit (or the short sequences are switched off)
-    std::vector<int> spans;
-    if (e->short_path) spans.push_back(0);
-    if (!e->short_path || e->cfg.max_seq_len > short_limit(batch)) {
-        for (int sp = 1024; sp < e->cfg.max_seq_len; sp *= 2) spans.push_back(sp);
-        spans.push_back(e->cfg.max_seq_len);
-    }
-    for (int span : spans) {
-        PGK_CHECK_HIP(hipStreamBeginCapture(st, hipStreamCaptureModeRelaxed));
-        int launches = 0;
-        e->step_span = span;
-        pgk_status r = decode_step(e, batch, st, &launches, span == 0);
-        hipGraph_t g = nullptr;
-        hipError_t he = hipStreamEndCapture(st, &g);
-        if (r != PGK_OK) { if (g) (void)hipGraphDestroy(g); drop_graphs(e); return r; }
-        if (he != hipSuccess || !g) { drop_graphs(e); return set_error(PGK_ERR_HIP, "pgk_engine_capture: hipStreamEndCapture: %s", hipGetErrorString(he)); }
-        Engine::Tier t;
-        t.span = span; t.graph = g; t.launches = launches;
-        he = hipGraphInstantiate(&t.exec, g, nullptr, nullptr, 0);
-        e->tiers.push_back(t);      // owned from here on (drop_graphs)
-        if (he != hipSuccess) { drop_graphs(e); return set_error(PGK_ERR_HIP, "pgk_engine_capture: hipGraphInstantiate: %s", hipGetErrorString(he)); }
-    }
-    e->graph_batch = batch;
-    e->launches_per_step = e->tiers[pick_tier(e)].launches;
-    return PGK_OK;
-}
-
-pgk_status pgk_engine_replay(pgk_engine eh, int n_steps, pgk_stream s) {
-    PGK_REQUIRE(eh, "pgk_engine_replay: null engine");
-    Engine* e = (Engine*)eh;
-    PGK_REQUIRE(!e->tiers.empty(), "pgk_engine_replay: no captured graph (call pgk_engine_capture first)");
-    hipStream_t st = resolve_stream(s);
-    for (int i = 0; i < n_steps; ++i) {
-        const auto& t = e->tiers[pick_tier(e)];
-        PGK_CHECK_HIP(hipGraphLaunch(t.exec, st));
-        e->launches_per_step = t.launches;
-        if (e->pos_hi >= 0) ++e->pos_hi;
-    }
-    return PGK_OK;
-}
-
-pgk_status pgk_engine_logits_ptr(pgk_engine eh, void** logits_f32) {
-    PGK_REQUIRE(eh && logits_f32, "pgk_engine_logits_ptr: null argument");
-    *logits_f32 = ((Engine*)eh)->logits;
-    return PGK_OK;
-}
-
-pgk_status pgk_engine_read_tokens(pgk_engine eh, int32_t* h_out, int batch, int n_steps, pgk_stream s) {
-    PGK_REQUIRE(eh && h_out, "pgk_engine_read_tokens: null argument");
-    Engine* e = (Engine*)eh;
-    PGK_REQUIRE(n_steps >= 0 && n_steps <= e->log_cap, "pgk_engine_read_tokens: %d steps exceed the log capacity %d", n_steps, e->log_cap);
-    PGK_REQUIRE(batch >= 1 && batch <= e->cfg.max_batch, "pgk_engine_read_tokens: bad batch %d", batch);
-    hipStream_t st = resolve_stream(s);
-    // log rows are max_batch wide; return the first `batch` columns, step-major
-    std::vector<int32_t> tmp((size_t)n_steps * e->cfg.max_batch);
-    if (n_steps) PGK_CHECK_HIP(hipMemcpyAsync(tmp.data(), e->token_log, tmp.size() * 4, hipMemcpyDeviceToHost, st));
-    PGK_CHECK_HIP(hipStreamSynchronize(st));
-    for (int t = 0; t < n_steps; ++t)
-        for (int b = 0; b < batch; ++b) h_out[(size_t)t * batch + b] = tmp[(size_t)t * e->cfg.max_batch + b];
-    return PGK_OK;
-}
-
-pgk_status pgk_engine_read_clock(pgk_engine eh, uint64_t* h_out, int n_steps, pgk_stream s) {
-    PGK_REQUIRE(eh && h_out, "pgk_engine_read_clock: null argument");
-    Engine* e = (Engine*)eh;
-    PGK_REQUIRE(n_steps >= 0 && n_steps <= e->log_cap, "pgk_engine_read_clock: %d steps exceed the log capacity %d", n_steps, e->log_cap);
-    hipStream_t st = resolve_stream(s);
-    if (n_steps) {
-        PGK_CHECK_HIP(hipMemcpyAsync(h_out, e->clk_log, (size_t)n_steps * 16, hipMemcpyDeviceToHost, st));
-        PGK_CHECK_HIP(hipStreamSynchronize(st));
-    }
-    return PGK_OK;
-}
-
-// In-graph stochastic sampling.  temperature <= 0 restores greedy argmax.  `h_uniforms` [n_rows][max_batch] floats in
-// [0,1) are copied into the device ring: step s of the log uses row s % n_rows.  The sampling node and its arguments
-// (ring pointer and length, scratch pointer, temperature, top-k, top-p) are baked into a captured graph, so ANY change
-// of them - switching sampling on or off, another temperature / top-k / top-p, another n_rows, a scratch buffer that had
-// to grow - drops the engine's captured graph: pgk_engine_replay then fails with "no captured graph" until
-// pgk_engine_capture is called again.  A refill with the same n_rows and the same parameters only overwrites the ring's
-// contents and keeps the graph.
-pgk_status pgk_engine_set_sampling(pgk_engine eh, float temperature, int top_k, float top_p, const float* h_uniforms, int n_rows,
-                                   pgk_stream s) {
-    PGK_REQUIRE(eh, "pgk_engine_set_sampling: null engine");
-    Engine* e = (Engine*)eh;
-    hipStream_t st = resolve_stream(s);
-    auto drop_graph = [&]() {
-        if (!e->tiers.empty()) (void)hipStreamSynchronize(st);
-        drop_graphs(e);
-    };
-    if (temperature <= 0.f) {
-        if (e->sample_temperature > 0.f) drop_graph();          // a captured sampling node must not be replayed as "greedy"
-        e->sample_temperature = 0.f;
-        return PGK_OK;
-    }
-    PGK_REQUIRE(top_k >= 0 && top_p > 0.f && top_p <= 1.f, "pgk_engine_set_sampling: need top_k >= 0 and 0 < top_p <= 1");
-    PGK_REQUIRE(h_uniforms && n_rows >= 1, "pgk_engine_set_sampling: uniforms missing");
-    const int B = e->cfg.max_batch;
-    bool changed = e->sample_temperature != temperature || e->sample_top_k != top_k || e->sample_top_p != top_p || n_rows != e->u_cap;
-    if (n_rows > e->u_alloc_rows) {
-        drop_graph();                                           // its nodes hold the old ring pointer
-        PGK_CHECK_HIP(hipStreamSynchronize(st));
-        if (e->u_ring) pgk_free(e->u_ring);
-        e->u_ring = nullptr;
-        e->u_alloc_rows = 0;
-        if (pgk_status r = pgk_malloc((void**)&e->u_ring, (size_t)n_rows * B * 4)) return r;
-        e->u_alloc_rows = n_rows;
-    }
-    if (!e->sampled) {
-        if (pgk_status r = pgk_malloc((void**)&e->sampled, (size_t)B * 4)) return r;
-    }
-    if (const size_t need = sample_scratch_bytes(B, e->cfg.vocab_size, top_k, top_p); need > e->sample_scratch_cap) {
-        drop_graph();
-        PGK_CHECK_HIP(hipStreamSynchronize(st));
-        if (e->sample_scratch) pgk_free(e->sample_scratch);
-        e->sample_scratch = nullptr;
-        e->sample_scratch_cap = 0;
-        if (pgk_status r = pgk_malloc(&e->sample_scratch, need)) return r;
-        e->sample_scratch_cap = need;
-    }
-    if (changed) drop_graph();
-    PGK_CHECK_HIP(hipMemcpyAsync(e->u_ring, h_uniforms, (size_t)n_rows * B * 4, hipMemcpyHostToDevice, st));
-    PGK_CHECK_HIP(hipStreamSynchronize(st));
-    e->u_cap = n_rows;                                          // ring length = rows queued: row index is step % n_rows
-    e->sample_temperature = temperature;
-    e->sample_top_k = top_k;
-    e->sample_top_p = top_p;
-    return PGK_OK;
-}
-
-pgk_status pgk_engine_reset_log(pgk_engine eh, pgk_stream s) {
-    PGK_REQUIRE(eh, "pgk_engine_reset_log: null engine");
-    PGK_CHECK_HIP(hipMemsetAsync(((Engine*)eh)->step_counter, 0, 16, resolve_stream(s)));
-    return PGK_OK;
-}
-
-pgk_status pgk_engine_kv_ptr(pgk_engine eh, int layer, void** k, void** v) {
-    PGK_REQUIRE(eh && k && v, "pgk_engine_kv_ptr: null argument");
-    Engine* e = (Engine*)eh;
-    PGK_REQUIRE(layer >= 0 && layer < e->cfg.num_layers, "pgk_engine_kv_ptr: layer %d", layer);
+static pgk_status dense_kv_ptr(Engine* e, int layer, void** k, void** v) {
     *k = e->kcache + (size_t)layer * e->kv_layer_elems();
     *v = e->vcache + (size_t)layer * e->kv_layer_elems();
     return PGK_OK;
 }
 
-pgk_status pgk_engine_state_ptr(pgk_engine eh, void** tokens, void** positions) {
-    PGK_REQUIRE(eh && tokens && positions, "pgk_engine_state_ptr: null argument");
-    *tokens = ((Engine*)eh)->tokens;
-    *positions = ((Engine*)eh)->positions;
-    return PGK_OK;
-}
+static const EngineKind DENSE_KIND = {decode_step, dense_prefill_batch, dense_prefill, dense_embed_state, nullptr, nullptr, dense_kv_ptr, nullptr};
 
-pgk_status pgk_engine_launches_per_step(pgk_engine eh, int* n) {
-    PGK_REQUIRE(eh && n, "pgk_engine_launches_per_step: null argument");
-    *n = ((Engine*)eh)->launches_per_step;
+}  // namespace pgk
+
+using namespace pgk;
+
+extern "C" {
+
+pgk_status pgk_engine_create(const pgk_model_config_t* cfg, const void* embed, const void* lm_head,
+                             const void* final_norm, const pgk_layer_weights_t* layers, pgk_engine* out) {
+    PGK_REQUIRE(cfg && embed && final_norm && layers && out, "pgk_engine_create: null argument");
+    const auto& c = *cfg;
+    PGK_REQUIRE(c.head_dim == 128 || c.head_dim == 64, "pgk_engine_create: head_dim %d not in {64,128}", c.head_dim);
+    PGK_REQUIRE(c.num_heads % c.num_kv_heads == 0, "pgk_engine_create: Hq %d %% Hkv %d", c.num_heads, c.num_kv_heads);
+    const int G = c.num_heads / c.num_kv_heads;
+    PGK_REQUIRE(G >= 1, "pgk_engine_create: GQA group %d", G);
+    PGK_REQUIRE(c.hidden_size % 16 == 0 && c.intermediate_size % 16 == 0, "pgk_engine_create: sizes must be multiples of 16");
+    PGK_REQUIRE(c.weight_format == 0 || (c.hidden_size % 128 == 0 && c.intermediate_size % 128 == 0),
+                "pgk_engine_create: fp8 weights need 128-multiple dims");
+    PGK_REQUIRE(c.max_batch >= 1 && c.max_seq_len >= 1 && c.num_layers >= 1, "pgk_engine_create: bad sizes");
+    Engine* e = new Engine();
+    e->kind = &DENSE_KIND;
+    e->cfg = c;
+    e->embed = (const bf16*)embed;
+    e->lm_head = (const bf16*)(lm_head ? lm_head : embed);
+    e->final_norm = (const bf16*)final_norm;
+    e->layers.assign(layers, layers + c.num_layers);
+    int nsplit = (c.max_seq_len + 63) / 64;   // ~64 cached positions per workgroup: one KV batch per wave
+    {
+        int dev = 0;
+        hipDeviceProp_t prop;
+        if (hipGetDevice(&dev) == hipSuccess && hipGetDeviceProperties(&prop, dev) == hipSuccess && prop.multiProcessorCount > 0)
+            e->cu_count = prop.multiProcessorCount;
+    }
+    e->nsplit = nsplit < 1 ? 1 : (nsplit > 64 ? 64 : nsplit);
+    e->lm_blocks = 1024;
+    // fused attention + o_proj: short contexts, bf16 W_o, and a row slicing that tiles the workgroup
+    {
+        const int gd = G * c.head_dim, rpp = 256 / (gd / 8);
+        int rows = c.hidden_size / 32;
+        while (rows > 4 * rpp && rows % 2 == 0) rows /= 2;   // <= 4 preloaded passes per workgroup
+        while (rows < rpp) rows *= 2;
+        const bool tiles = rows % rpp == 0 && c.hidden_size % rows == 0 && gd / 8 <= 64;
+        // PGK_FUSED_ATTN=0: no short-context launch sequence at all (the split-KV sequence at every context; A/B and tests)
+        const char* env = getenv("PGK_FUSED_ATTN");
+        e->short_path = env ? atoi(env) != 0 : true;
+        e->fused_attn = tiles && c.weight_format == 0 && (G == 1 || G == 2 || G == 4);
+        e->oproj_rows = rows;
+        {
+            const char* am = getenv("PGK_ATTN_MFMA");
+            e->attn_mfma = c.head_dim == 128 && !(am && atoi(am) == 0);
+        }
+        // merged o_proj (long contexts, fp8 W_o): same slicing rule with 16 codes per lane for fp8
+        const int nwt = c.weight_format != 0 ? 16 : 8, lpw = gd / nwt, rpp2 = lpw > 0 ? 256 / lpw : 256;
+        int rows2 = c.hidden_size / 32;
+        while (rows2 > 4 * rpp2 && rows2 % 2 == 0) rows2 /= 2;
+        while (rows2 < rpp2) rows2 *= 2;
+        const char* emo = getenv("PGK_MERGED_OPROJ");
+        e->merged_oproj = !(emo && atoi(emo) == 0) && (G == 1 || G == 2 || G == 4) && lpw >= 8 && lpw <= 64 && 256 % lpw == 0 &&
+                          rows2 % rpp2 == 0 && c.hidden_size % rows2 == 0 && (c.weight_format == 0 || (gd % 128 == 0 || 128 % gd == 0));
+        e->moproj_rows = rows2;
+    }
+    const int B = c.max_batch, H = c.hidden_size, D = c.head_dim;
+    pgk_status r = PGK_OK;
+    auto A = [&](void** p, size_t bytes, size_t* acct) { if (r == PGK_OK) r = dev_alloc(e, p, bytes, acct); };
+    const size_t kvb = (size_t)c.num_layers * e->kv_layer_elems() * sizeof(bf16);
+    A((void**)&e->kcache, kvb, &e->kv_bytes);
+    A((void**)&e->vcache, kvb, &e->kv_bytes);
+    A((void**)&e->rope_cos, (size_t)c.max_seq_len * (D / 2) * 4, &e->ws_bytes);
+    A((void**)&e->rope_sin, (size_t)c.max_seq_len * (D / 2) * 4, &e->ws_bytes);
+    A((void**)&e->cur_cos, (size_t)B * (D / 2) * 4, &e->ws_bytes);
+    A((void**)&e->cur_sin, (size_t)B * (D / 2) * 4, &e->ws_bytes);
+    A((void**)&e->tokens, (size_t)B * 4, &e->ws_bytes);
+    A((void**)&e->positions, (size_t)B * 4, &e->ws_bytes);
+    A((void**)&e->token_log, (size_t)e->log_cap * B * 4, &e->ws_bytes);
+    A((void**)&e->step_counter, 16, &e->ws_bytes);
+    A((void**)&e->h, (size_t)B * H * 4, &e->ws_bytes);
+    A((void**)&e->h2, (size_t)B * H * 4, &e->ws_bytes);
+    A((void**)&e->qkv, (size_t)B * e->qkv_dim() * 4, &e->ws_bytes);
+    A((void**)&e->part, (size_t)B * c.num_heads * e->nsplit * (D + 2) * 4, &e->ws_bytes);
+    A((void**)&e->opart, (size_t)B * c.num_kv_heads * H * 4, &e->ws_bytes);
+    A((void**)&e->act16, (size_t)B * c.intermediate_size * 2, &e->ws_bytes);
+    A((void**)&e->attnv16, (size_t)B * c.num_heads * c.head_dim * 2, &e->ws_bytes);
+    A((void**)&e->x16, (size_t)B * H * 2, &e->ws_bytes);
+    A((void**)&e->ss_part, (size_t)64 * 1024 * 4, &e->ws_bytes);
+    A((void**)&e->attnv, (size_t)B * c.num_heads * D * 4, &e->ws_bytes);
+    A((void**)&e->act, (size_t)B * c.intermediate_size * 4, &e->ws_bytes);
+    A((void**)&e->logits, (size_t)B * c.vocab_size * 4, &e->ws_bytes);
+    e->lm_cap = e->lm_blocks > ceil_div(c.vocab_size, 16) ? e->lm_blocks : ceil_div(c.vocab_size, 16);   // per-sequence argmax partial slots
+    {
+        const char* ev = getenv("PGK_BATCHED_MFMA");
+        e->batched_min = (ev && atoi(ev) == 2) ? 3 : 5;   // 2: from 3 up
+        // every projection's K must suit the MFMA decode kernels: K = 128 S with S in {8, 16, 24, 32} (activation
+        // fragments in registers) or an LDS image of K x 16 bf16 that fits (K <= 4096); Llama-3-8B's down_proj
+        // (K = 14336) does neither, so such models decode batches in GEMV chunks of 8 / 4 / 2 / 1
+        auto k_ok = [](int K) { return K % 128 == 0 && K <= 4096; };
+        e->batched_mfma = !(ev && atoi(ev) == 0) && k_ok(c.hidden_size) && k_ok(c.intermediate_size) && k_ok(c.num_heads * c.head_dim);
+        // 17..64 sequences in one weight pass (batched_mt_kernel) need K = 128 S with S instantiated; otherwise chunks of 16
+        auto k_tiled = [](int K) { const int s = K / 128; return K % 128 == 0 && (s == 2 || s == 4 || s == 8 || s == 16 || s == 24 || s == 32); };
+        e->batched_max = (k_tiled(c.hidden_size) && k_tiled(c.intermediate_size) && k_tiled(c.num_heads * c.head_dim)) ? 64 : 16;
+        if (const char* em = getenv("PGK_BATCHED_MAX")) { const int v = atoi(em); if (v >= 16 && v < e->batched_max) e->batched_max = v; }
+    }
+    A((void**)&e->amax_val, (size_t)B * e->lm_cap * 4, &e->ws_bytes);
+    A((void**)&e->amax_idx, (size_t)B * e->lm_cap * 4, &e->ws_bytes);
+    A((void**)&e->clk_log, (size_t)e->log_cap * 16, &e->ws_bytes);
+    {
+        // Second, fragment-major copy of the bf16 layer weights: what the short-prompt prefill streams (ops_pkgemm.hip).
+        // Costs the layers' bytes again; skipped when that is more than a quarter of the device's free memory.
+        const int QDp = c.num_heads * D, NQ = e->qkv_dim(), I = c.intermediate_size;
+        const char* ep = getenv("PGK_PACKED_PREFILL");
+        const size_t per_layer = ((size_t)NQ * H + (size_t)H * QDp + (size_t)2 * I * H + (size_t)H * I) * 2;
+        size_t free_b = 0, total_b = 0;
+        const bool fits = hipMemGetInfo(&free_b, &total_b) == hipSuccess && per_layer * c.num_layers < free_b / 4;
+        const bool shapes = pkgemm_shape_ok(NQ, H, false) && pkgemm_shape_ok(H, QDp, true) && pkgemm_shape_ok(2 * I, H, false) && pkgemm_shape_ok(H, I, true) && I % 64 == 0;
+        // bf16 layers, or fp8 codes + block scales (w8a16): the copy is bf16 either way (ops_pkgemm.hip)
+        const bool f8w = c.weight_format == 1;
+        // w8a16 engines keep the copy also where the skinny kernels cannot use it (Llama-3-8B: K = 4096 / 14336 is beyond them):
+        // their long-prompt GEMMs read it (packed_have), instead of dequantising every weight again in front of every call
+        const bool long_only = f8w && !shapes && NQ % 16 == 0 && H % 64 == 0 && QDp % 64 == 0 && I % 64 == 0;
+        if (r == PGK_OK && (c.weight_format == 0 || f8w) && (shapes || long_only) && fits && !(ep && atoi(ep) == 0)) {
+            e->packed.resize(c.num_layers);
+            hipStream_t st = resolve_stream(nullptr);
+            for (int l = 0; l < c.num_layers && r == PGK_OK; ++l) {
+                auto& P = e->packed[l];
+                const auto& L = e->layers[l];
+                A((void**)&P.qkv, (size_t)NQ * H * 2, &e->packed_bytes);
+                A((void**)&P.o, (size_t)H * QDp * 2, &e->packed_bytes);
+                A((void**)&P.gate_up, (size_t)2 * I * H * 2, &e->packed_bytes);
+                A((void**)&P.down, (size_t)H * I * 2, &e->packed_bytes);
+                if (r == PGK_OK) r = f8w ? pack_weights_fp8(L.w_qkv, L.s_qkv, P.qkv, NQ, H, st) : pack_weights_bf16(L.w_qkv, P.qkv, NQ, H, st);
+                if (r == PGK_OK) r = f8w ? pack_weights_fp8(L.w_o, L.s_o, P.o, H, QDp, st) : pack_weights_bf16(L.w_o, P.o, H, QDp, st);
+                if (r == PGK_OK) r = f8w ? pack_weights_fp8(L.w_gate_up, L.s_gate_up, P.gate_up, 2 * I, H, st) : pack_weights_bf16(L.w_gate_up, P.gate_up, 2 * I, H, st);
+                if (r == PGK_OK) r = f8w ? pack_weights_fp8(L.w_down, L.s_down, P.down, H, I, st) : pack_weights_bf16(L.w_down, P.down, H, I, st);
+            }
+            if (r == PGK_OK && hipStreamSynchronize(st) != hipSuccess) r = set_error(PGK_ERR_HIP, "pgk_engine_create: packing the prefill weights failed");
+            e->packed_have = r == PGK_OK;
+            e->packed_ok = e->packed_have && shapes;
+            if (e->packed_ok && pkgemm_resid_ok(H, QDp) && pkgemm_resid_ok(H, I)) {
+                A((void**)&e->pk_ss, (size_t)128 * PK_SS_LD * 4, &e->ws_bytes);
+                e->packed_resid = r == PGK_OK;
+            }
+            if (e->packed_ok && c.max_batch >= 3 && c.vocab_size % 16 == 0 && H % 32 == 0) {
+                A((void**)&e->packed_lm, (size_t)c.vocab_size * H * 2, &e->packed_bytes);
+                if (r == PGK_OK) r = pack_weights_bf16(e->lm_head, e->packed_lm, c.vocab_size, H, st);
+                if (r == PGK_OK && hipStreamSynchronize(st) != hipSuccess) r = set_error(PGK_ERR_HIP, "pgk_engine_create: packing the lm_head failed");
+            }
+            const char* pd = getenv("PGK_PACKED_DECODE");
+            if (e->packed_ok && c.max_batch > 16 && !(pd && atoi(pd) == 0)) {
+                A((void**)&e->dec_slabs, (size_t)16 * 64 * H * 4, &e->ws_bytes);
+                e->packed_decode = r == PGK_OK;
+            }
+        }
+    }
+    if (r != PGK_OK) { pgk_engine_destroy(e); return r; }
+    // RoPE tables in fp32, same formula as the reference (src/pygpukit/llm/layers/rope.py:13-24):
+    // freqs = 1/theta^(2i/D) in fp32, angle = float(t) * freq in fp32, cos/sin of that.
+    {
+        std::vector<float> hc((size_t)c.max_seq_len * (D / 2)), hs(hc.size());
+        for (int i = 0; i < D / 2; ++i) {
+            const float expo = (float)(2 * i) / (float)D;
+            const float freq = 1.0f / powf(c.rope_theta, expo);
+            for (int t = 0; t < c.max_seq_len; ++t) {
+                const float ang = (float)t * freq;
+                hc[(size_t)t * (D / 2) + i] = (float)cos((double)ang);
+                hs[(size_t)t * (D / 2) + i] = (float)sin((double)ang);
+            }
+        }
+        hipStream_t st = resolve_stream(nullptr);
+        hipError_t he = hipMemcpyAsync(e->rope_cos, hc.data(), hc.size() * 4, hipMemcpyHostToDevice, st);
+        if (he == hipSuccess) he = hipMemcpyAsync(e->rope_sin, hs.data(), hs.size() * 4, hipMemcpyHostToDevice, st);
+        if (he == hipSuccess) he = hipMemsetAsync(e->kcache, 0, kvb, st);
+        if (he == hipSuccess) he = hipMemsetAsync(e->vcache, 0, kvb, st);
+        if (he == hipSuccess) he = hipMemsetAsync(e->tokens, 0, (size_t)B * 4, st);
+        if (he == hipSuccess) he = hipMemsetAsync(e->positions, 0, (size_t)B * 4, st);
+        if (he == hipSuccess) he = hipMemsetAsync(e->step_counter, 0, 16, st);
+        if (he == hipSuccess) he = hipMemsetAsync(e->h, 0, (size_t)B * H * 4, st);
+        if (he == hipSuccess) he = hipStreamSynchronize(st);
+        if (he != hipSuccess) { pgk_engine_destroy(e); return set_error(PGK_ERR_HIP, "pgk_engine_create: %s", hipGetErrorString(he)); }
+    }
+    *out = e;
     return PGK_OK;
 }
 

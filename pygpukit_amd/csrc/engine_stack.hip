@@ -1,0 +1,1030 @@
+// Native engine for layer-list decoders: an fp32 residual stream, RMSNorm before AND after each sublayer, latent attention over a
+// sliding window (the cache holds one normalised latent row per token, not keys and values), dense SwiGLU or no feed-forward.
+// Every layer has its own sizes.  Elements are bf16 (fp32 stream, norms, scores and softmax) or fp32 throughout.
+//
+//   x   <- x + m * rho(O (sigmoid(G h) * attention(Q h, c)); n1b),  h = rho(x; n1),  c = rms(D h) * w_c,  k = U_k c,  v = U_v c
+//   x   <- x + m * rho(W_d (silu(W_g h) * W_u h); n2b),             h = rho(x; n2)
+//
+// Cache: per layer [slot][R][rank] latents, R = min(window, max_seq_len); position p lives in row p mod R, so a full ring IS the
+// window and a decode step needs no mask.  Keys and values are never stored: decode folds U_k into the query (q_lat = U_k^T q, scores
+// q_lat . c) and applies U_v to the probability-weighted latent sum, prefill expands the latents it needs into a scratch K | V.
+//
+// Decode, one sequence (fp32 between kernels):
+//   in_proj    [pending: x += m rho(y; n2b)] q | latent | gate = W_in . rho(x; n1)
+//   absorb     q_lat = scale log2e U_k^T q per head;  the new latent row -> ring
+//   attn       split over the ring: scores, softmax, sum p c  -> partial records
+//   merge_uv   combine the records, U_v, head gate
+//   oproj      y = O a
+//   gateup     x += m rho(y; n1b);  act = silu(g) * u of rho(x; n2)
+//   down       y = W_d act
+// The reduction a post-norm needs over the whole sublayer output is done in the NEXT kernel's prologue, by every workgroup for itself
+// (one row: a few KB from L2), so it costs no launch.
+// Several sequences and prompts: the same kernels on rows, the norms as a launch of their own and the projections on the GEMM family
+// (pgk_gemm_nt: GEMV up to 8 rows, weight-streaming MFMA up to 128, tiled MFMA beyond).
+// All widths are padded with zeros by the caller: every K is a multiple of 64, head widths are 64, 128 or a larger multiple of 64.
+
+#include <cstring>
+
+#include "engine_state.hip.h"
+#include "latent.hip.h"
+
+namespace pgk {
+
+pgk_status wsgemm_nt(const bf16* a, int lda, const void* w, const bf16* wscale, bool fp8, void* c, const bf16* bias, int mode,
+                     int splits, int M, int N, int K, hipStream_t st);
+bool engine_gemm_swiglu_ok(int M, int I, int K, bool fp8);     // ops_gemm.hip
+pgk_status engine_gemm_swiglu_nt(const bf16* A, const void* W, const bf16* wscale, bool fp8, bf16* act, int M, int I, int K, hipStream_t st, bool packed = false);
+
+constexpr float LOG2E = 1.4426950408889634f;
+
+// -------------------------------------------------------------------------------------------- one-row projection
+enum { SP_NORM = 0, SP_PLAIN = 1 };
+enum { SE_STORE = 0, SE_SWIGLU = 1, SE_LOGITS = 2 };
+
+struct StackGemvArgs {
+    const void* w;            // [N][K] (SE_SWIGLU: [2 N][K], gate rows then up rows)
+    int N, K, W;              // W: true width of the normalised row (columns W..K are zero padding)
+    const float* x;           // SP_NORM: residual row; SP_PLAIN: input row  [K]
+    const float* y;           // SP_NORM: pending sublayer output (null: none)
+    const float* g_post;      // its post-norm weight
+    float* x_out;             // where workgroup 0 writes the updated residual row (another buffer than x; null: nowhere)
+    const float* gamma;
+    float eps, mult;
+    float* out;               // [N]
+    float* amax_val; int* amax_idx;
+};
+
+// 256 threads; a wave owns R weight rows per trip.  C > 0: the first trip's C chunks of every row are requested before the prologue
+// touches the activations (which were requested before them: vector memory returns in order), K <= C * 64 * NW; C == 0: any K.
+// Chunks beyond K are clamped in the weight row and zero in the LDS image.
+template <class WT, int R, int PRO, int EPI, int C>
+__global__ __launch_bounds__(256) void stack_gemv_kernel(unsigned long long* tl, StackGemvArgs a) {
+    const TLStamp tls(tl);
+    constexpr int NW = WTraits<WT>::NW, CH = 64 * NW;
+    extern __shared__ __attribute__((aligned(16))) char smem[];
+    WT* xs = reinterpret_cast<WT*>(smem);                         // [round_up(K, CH)]
+    __shared__ float red[16], s_bv[4];
+    __shared__ int s_bi[4];
+    const int K = a.K, N = a.N, lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
+    constexpr int OUT = EPI == SE_SWIGLU ? R / 2 : R;
+    const int wave = blockIdx.x * 4 + wid, nwaves = gridDim.x * 4;
+    const WT* w = reinterpret_cast<const WT*>(a.w);
+    auto row_of = [&](int n0, int r) -> int {
+        if constexpr (EPI == SE_SWIGLU) return r < R / 2 ? min(n0 + r, N - 1) : N + min(n0 + r - R / 2, N - 1);
+        else return min(n0 + r, N - 1);
+    };
+    uint4 pre[R][C > 0 ? C : 1];
+    if constexpr (C > 0) {
+        constexpr int NT = (C * CH + 1023) / 1024;                // float4 per thread
+        float4 v[NT], y[NT], gp[NT], gm[NT];
+#pragma unroll
+        for (int t = 0; t < NT; ++t) {
+            const int i = min((int)(threadIdx.x + 256 * t) * 4, K - 4);
+            v[t] = *reinterpret_cast<const float4*>(a.x + i);
+            if constexpr (PRO == SP_NORM) {
+                const float* yp = a.y ? a.y : a.x;                // unconditional loads; masked below
+                const float* pp = a.y ? a.g_post : a.gamma;
+                y[t] = *reinterpret_cast<const float4*>(yp + i);
+                gp[t] = *reinterpret_cast<const float4*>(pp + i);
+                gm[t] = *reinterpret_cast<const float4*>(a.gamma + i);
+            }
+        }
+        __builtin_amdgcn_sched_barrier(0);
+        const int nf = min(wave * OUT, N - 1);
+#pragma unroll
+        for (int r = 0; r < R; ++r)
+#pragma unroll
+            for (int c = 0; c < C; ++c) pre[r][c] = load_nt16(w + (size_t)row_of(nf, r) * K + min(c * CH + lane * NW, K - NW));
+        __builtin_amdgcn_sched_barrier(0);
+        float ss = 0.f;
+        if constexpr (PRO == SP_NORM) {
+            if (a.y) {
+#pragma unroll
+                for (int t = 0; t < NT; ++t)
+                    if ((int)(threadIdx.x + 256 * t) * 4 < K) ss += y[t].x * y[t].x + y[t].y * y[t].y + y[t].z * y[t].z + y[t].w * y[t].w;
+                ss = block_sum(ss, red);
+                const float inv = a.mult / sqrtf(ss / a.W + a.eps);
+#pragma unroll
+                for (int t = 0; t < NT; ++t) {
+                    const int i = (threadIdx.x + 256 * t) * 4;
+                    v[t].x = fmaf(y[t].x * inv, gp[t].x, v[t].x); v[t].y = fmaf(y[t].y * inv, gp[t].y, v[t].y);
+                    v[t].z = fmaf(y[t].z * inv, gp[t].z, v[t].z); v[t].w = fmaf(y[t].w * inv, gp[t].w, v[t].w);
+                    if (a.x_out && blockIdx.x == 0 && i < K) *reinterpret_cast<float4*>(a.x_out + i) = v[t];
+                }
+            }
+            ss = 0.f;
+#pragma unroll
+            for (int t = 0; t < NT; ++t)
+                if ((int)(threadIdx.x + 256 * t) * 4 < K) ss += v[t].x * v[t].x + v[t].y * v[t].y + v[t].z * v[t].z + v[t].w * v[t].w;
+            ss = block_sum(ss, red);
+            const float inv = 1.0f / sqrtf(ss / a.W + a.eps);
+#pragma unroll
+            for (int t = 0; t < NT; ++t) {
+                v[t].x *= inv * gm[t].x; v[t].y *= inv * gm[t].y; v[t].z *= inv * gm[t].z; v[t].w *= inv * gm[t].w;
+            }
+        }
+#pragma unroll
+        for (int t = 0; t < NT; ++t) {
+            const int i = (threadIdx.x + 256 * t) * 4;
+            if (i < C * CH) store4<WT>(xs + i, i < K ? v[t] : make_float4(0.f, 0.f, 0.f, 0.f));
+        }
+    } else {
+        if constexpr (PRO == SP_NORM) {
+            float inv_y = 0.f;
+            if (a.y) {
+                float ss = 0.f;
+                for (int i = threadIdx.x; i < K; i += 256) ss = fmaf(a.y[i], a.y[i], ss);
+                inv_y = a.mult / sqrtf(block_sum(ss, red) / a.W + a.eps);
+            }
+            auto xin = [&](int i) -> float { return a.y ? fmaf(a.y[i] * inv_y, a.g_post[i], a.x[i]) : a.x[i]; };
+            float ss = 0.f;
+            for (int i = threadIdx.x; i < K; i += 256) {
+                const float v = xin(i);
+                if (a.y && a.x_out && blockIdx.x == 0) a.x_out[i] = v;
+                ss = fmaf(v, v, ss);
+            }
+            const float inv = 1.0f / sqrtf(block_sum(ss, red) / a.W + a.eps);
+            for (int i = threadIdx.x; i < K; i += 256) xs[i] = from_f<WT>(xin(i) * inv * a.gamma[i]);
+        } else {
+            for (int i = threadIdx.x; i < K; i += 256) xs[i] = from_f<WT>(a.x[i]);
+        }
+    }
+    __syncthreads();
+    float best_v = -INFINITY;
+    int best_i = 0x7FFFFFFF;
+    for (int g = wave; g * OUT < N; g += nwaves) {
+        const int n0 = g * OUT;
+        float acc[R][1];
+#pragma unroll
+        for (int r = 0; r < R; ++r) acc[r][0] = 0.f;
+        auto dot = [&](const uint4& raw, const WT* xp, float s) -> float {
+            if constexpr (std::is_same<WT, bf16>::value) return dot8_bf16(raw, *reinterpret_cast<const uint4*>(xp), s);
+            else {
+                const float4 x4 = *reinterpret_cast<const float4*>(xp);
+                s = fmaf(__uint_as_float(raw.x), x4.x, s); s = fmaf(__uint_as_float(raw.y), x4.y, s);
+                s = fmaf(__uint_as_float(raw.z), x4.z, s); return fmaf(__uint_as_float(raw.w), x4.w, s);
+            }
+        };
+        if (C > 0) {
+            if (g != wave) {
+#pragma unroll
+                for (int r = 0; r < R; ++r)
+#pragma unroll
+                    for (int c = 0; c < C; ++c) pre[r][c] = load_nt16(w + (size_t)row_of(n0, r) * K + min(c * CH + lane * NW, K - NW));
+            }
+#pragma unroll
+            for (int c = 0; c < (C > 0 ? C : 1); ++c)
+#pragma unroll
+                for (int r = 0; r < R; ++r) acc[r][0] = dot(pre[r][c], xs + c * CH + lane * NW, acc[r][0]);
+        } else {
+            const WT* wrow[R];
+#pragma unroll
+            for (int r = 0; r < R; ++r) wrow[r] = w + (size_t)row_of(n0, r) * K;
+            gemv_rows<WT, WT, 1, R>(wrow, xs, K, K, lane, acc);
+        }
+#pragma unroll
+        for (int r = 0; r < R; ++r) acc[r][0] = wave_sum(acc[r][0]);
+        if (lane == 0) {
+#pragma unroll
+            for (int r = 0; r < OUT; ++r)
+                if (n0 + r < N) {
+                    float o = acc[r][0];
+                    if constexpr (EPI == SE_SWIGLU) o = o / (1.0f + (std::is_same<WT, float>::value ? expf(-o) : __expf(-o))) * acc[r + R / 2][0];
+                    a.out[n0 + r] = o;
+                    if constexpr (EPI == SE_LOGITS) { if (o > best_v) { best_v = o; best_i = n0 + r; } }
+                }
+        }
+    }
+    if constexpr (EPI == SE_LOGITS) {
+        if (lane == 0) { s_bv[wid] = best_v; s_bi[wid] = best_i; }
+        __syncthreads();
+        if (threadIdx.x == 0) {
+            float bv = s_bv[0];
+            int bi = s_bi[0];
+            for (int i = 1; i < 4; ++i)
+                if (s_bv[i] > bv || (s_bv[i] == bv && s_bi[i] < bi)) { bv = s_bv[i]; bi = s_bi[i]; }
+            a.amax_val[blockIdx.x] = bv;
+            a.amax_idx[blockIdx.x] = bi;
+        }
+    }
+    tls.end();
+}
+
+template <class WT, int R, int PRO, int EPI, int C>
+static pgk_status stack_gemv_c(const StackGemvArgs& a, int grid, hipStream_t st) {
+    constexpr int CH = 64 * WTraits<WT>::NW;
+    const size_t lds = (size_t)ceil_div(a.K, CH) * CH * sizeof(WT) > (size_t)C * CH * sizeof(WT) ? (size_t)ceil_div(a.K, CH) * CH * sizeof(WT) : (size_t)C * CH * sizeof(WT);
+    auto kfn = &stack_gemv_kernel<WT, R, PRO, EPI, C>;
+    PGK_REQUIRE(lds <= 156 * 1024, "engine: a row of %d does not fit LDS", a.K);
+    static bool attr_done = false;
+    if (lds > 48 * 1024 && !attr_done) {
+        PGK_CHECK_HIP(hipFuncSetAttribute(reinterpret_cast<const void*>(kfn), hipFuncAttributeMaxDynamicSharedMemorySize, 156 * 1024));
+        attr_done = true;
+    }
+    PGK_CHECK_HIP(launch_k(kfn, dim3(grid), dim3(256), lds, st, a));
+    return PGK_OK;
+}
+
+template <class WT, int R, int PRO, int EPI>
+static pgk_status stack_gemv_r(const StackGemvArgs& a, hipStream_t st, int force_grid = 0) {
+    constexpr int OUT = EPI == SE_SWIGLU ? R / 2 : R;
+    int grid = force_grid ? force_grid : ceil_div(a.N, OUT * 4);
+    if (grid > 1024) grid = 1024;
+    if constexpr (std::is_same<WT, bf16>::value) {
+        const int c = ceil_div(a.K, 512);
+        if constexpr (R * 2 <= 16) { if (c <= 2) return stack_gemv_c<WT, R, PRO, EPI, 2>(a, grid, st); }
+        if constexpr (R * 4 <= 16) { if (c <= 4) return stack_gemv_c<WT, R, PRO, EPI, 4>(a, grid, st); }
+        if constexpr (R * 8 <= 16) { if (c <= 8) return stack_gemv_c<WT, R, PRO, EPI, 8>(a, grid, st); }
+    }
+    return stack_gemv_c<WT, R, PRO, EPI, 0>(a, grid, st);
+}
+
+template <class WT, int PRO, int EPI>
+static pgk_status stack_gemv(const StackGemvArgs& a, hipStream_t st, int force_grid = 0) {
+    if constexpr (std::is_same<WT, float>::value) return stack_gemv_r<WT, EPI == SE_STORE ? 1 : 2, PRO, EPI>(a, st, force_grid);
+    else if constexpr (EPI == SE_SWIGLU) {
+        if (a.N >= 4096) return stack_gemv_r<WT, 4, PRO, EPI>(a, st);
+        return stack_gemv_r<WT, 2, PRO, EPI>(a, st);
+    } else if constexpr (EPI == SE_LOGITS) return stack_gemv_r<WT, 4, PRO, EPI>(a, st, force_grid);
+    else {
+        if (a.N >= 4096) return stack_gemv_r<WT, 4, PRO, EPI>(a, st);
+        if (a.N >= 2048) return stack_gemv_r<WT, 2, PRO, EPI>(a, st);
+        return stack_gemv_r<WT, 1, PRO, EPI>(a, st);
+    }
+}
+
+// -------------------------------------------------------------------------------------------- latent attention, decode
+struct LatentArgs {
+    const void* in;           // [B][ld_in] (IT): q at h * D, latent at qn, head gates at qn + rank
+    int ld_in, qn, g_off;
+    const void *w_uk, *w_uv;  // [H * D][rank] (T)
+    const float* c_norm;      // [rank]
+    void* cache;              // [slots][R][rank] (T)
+    const int32_t* positions; // [B]
+    int B, H, D, dim, vdim, rank, rank_true, R, nsplit;
+    float eps, scale;         // scale already times log2e
+    float* qlat;              // [B][H][rank]
+    float* po;                // [B][H][nsplit][rank]
+    float* pml;               // [B][H][nsplit][2]
+    void* out;                // [B][ld_out] (IT): head h at h * D
+    int ld_out;
+};
+
+// q_lat[b][h][r] = scale * sum_d U_k[h D + d][r] q[b][h][d]: workgroup = (head, 128 columns) x MB sequences, the four waves split d.
+// The last workgroup column normalises the MB new latent rows into the ring instead.
+template <class T, class IT, int MB>
+__global__ __launch_bounds__(256) void latent_absorb_kernel(unsigned long long* tl, LatentArgs a) {
+    const TLStamp tls(tl);
+    const int nt = (a.rank + 127) / 128, lane = threadIdx.x & 63, wid = threadIdx.x >> 6, b0 = blockIdx.y * MB;
+    const IT* in = reinterpret_cast<const IT*>(a.in);
+    if ((int)blockIdx.x == a.H * nt) {
+        for (int m = wid; m < MB && b0 + m < a.B; m += 4) {        // a wave per sequence
+            const int b = b0 + m;
+            const IT* c = in + (size_t)b * a.ld_in + a.qn;
+            float ss = 0.f;
+            for (int r = lane; r < a.rank; r += 64) { const float v = to_f(c[r]); ss = fmaf(v, v, ss); }
+            const float inv = 1.0f / sqrtf(wave_sum(ss) / a.rank_true + a.eps);
+            T* row = reinterpret_cast<T*>(a.cache) + ((size_t)b * a.R + max(a.positions[b], 0) % a.R) * a.rank;
+            for (int r = lane; r < a.rank; r += 64) row[r] = from_f<T>(to_f(c[r]) * inv * a.c_norm[r]);
+        }
+        tls.end();
+        return;
+    }
+    __shared__ float qs[MB][512], part[4][MB][128];
+    const int h = blockIdx.x / nt, r0 = (blockIdx.x % nt) * 128 + 2 * lane;
+    const bool live = r0 < a.rank;                                 // rank is a multiple of 64: both columns or none
+    float acc[MB][2];
+#pragma unroll
+    for (int m = 0; m < MB; ++m) acc[m][0] = acc[m][1] = 0.f;
+    for (int d0 = 0; d0 < a.dim; d0 += 512) {
+        const int dn = min(512, a.dim - d0);
+        __syncthreads();
+        for (int i = threadIdx.x; i < MB * dn; i += 256) {
+            const int m = i / dn, d = i % dn;
+            qs[m][d] = to_f(in[(size_t)min(b0 + m, a.B - 1) * a.ld_in + h * a.D + d0 + d]);
+        }
+        __syncthreads();
+        const T* u = reinterpret_cast<const T*>(a.w_uk) + (size_t)(h * a.D + d0) * a.rank + (live ? r0 : 0);
+#pragma unroll 8
+        for (int d = wid; d < dn; d += 4) {
+            float w0, w1;
+            if constexpr (std::is_same<T, bf16>::value) {
+                const uint32_t x = *reinterpret_cast<const uint32_t*>(u + (size_t)d * a.rank);
+                w0 = __uint_as_float(x << 16); w1 = __uint_as_float(x & 0xFFFF0000u);
+            } else {
+                const float2 x = *reinterpret_cast<const float2*>(u + (size_t)d * a.rank);
+                w0 = x.x; w1 = x.y;
+            }
+#pragma unroll
+            for (int m = 0; m < MB; ++m) { acc[m][0] = fmaf(w0, qs[m][d], acc[m][0]); acc[m][1] = fmaf(w1, qs[m][d], acc[m][1]); }
+        }
+    }
+#pragma unroll
+    for (int m = 0; m < MB; ++m) { part[wid][m][2 * lane] = acc[m][0]; part[wid][m][2 * lane + 1] = acc[m][1]; }
+    __syncthreads();
+    for (int i = threadIdx.x; i < MB * 128; i += 256) {
+        const int m = i >> 7, c = i & 127, r = (blockIdx.x % nt) * 128 + c;
+        if (b0 + m < a.B && r < a.rank)
+            a.qlat[((size_t)(b0 + m) * a.H + h) * a.rank + r] = a.scale * (part[0][m][c] + part[1][m][c] + part[2][m][c] + part[3][m][c]);
+    }
+    tls.end();
+}
+
+// the ring rows [k0, k1) of split s out of n occupied rows
+__device__ __forceinline__ void split_range(int n, int nsplit, int s, int& k0, int& k1) {
+    int per = (n + nsplit - 1) / nsplit;
+    per = (per + 31) / 32 * 32;
+    k0 = min(s * per, n);
+    k1 = min(k0 + per, n);
+}
+
+// Any rank up to 2048, any element type: a wave walks every fourth key, one strided element per lane and 64 columns.
+template <class T, int RC, int HB>
+__global__ __launch_bounds__(256) void latent_attn_kernel(unsigned long long* tl, LatentArgs a) {
+    const TLStamp tls(tl);
+    __shared__ float sm[4][HB][2];
+    extern __shared__ float so[];                                  // [HB][rank]
+    const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6, s = blockIdx.x, h0 = blockIdx.y * HB, b = blockIdx.z;
+    const int n = min(max(a.positions[b], 0) + 1, a.R);
+    int k0, k1;
+    split_range(n, a.nsplit, s, k0, k1);
+    float q[HB][RC], o[HB][RC], m[HB], l[HB];
+#pragma unroll
+    for (int i = 0; i < HB; ++i) {
+        m[i] = -INFINITY; l[i] = 0.f;
+        const float* qp = a.qlat + ((size_t)b * a.H + min(h0 + i, a.H - 1)) * a.rank;
+#pragma unroll
+        for (int j = 0; j < RC; ++j) { const int r = 64 * j + lane; q[i][j] = r < a.rank ? qp[r] : 0.f; o[i][j] = 0.f; }
+    }
+    const T* cb = reinterpret_cast<const T*>(a.cache) + (size_t)b * a.R * a.rank;
+    for (int k = k0 + wid; k < k1; k += 4) {
+        float c[RC];
+#pragma unroll
+        for (int j = 0; j < RC; ++j) { const int r = 64 * j + lane; c[j] = r < a.rank ? to_f(cb[(size_t)k * a.rank + r]) : 0.f; }
+#pragma unroll
+        for (int i = 0; i < HB; ++i) {
+            float t = 0.f;
+#pragma unroll
+            for (int j = 0; j < RC; ++j) t = fmaf(q[i][j], c[j], t);
+            t = wave_sum(t);
+            const float mn = fmaxf(m[i], t), al = exp2f(m[i] - mn), p = exp2f(t - mn);
+            m[i] = mn;
+            l[i] = fmaf(l[i], al, p);
+#pragma unroll
+            for (int j = 0; j < RC; ++j) o[i][j] = fmaf(o[i][j], al, p * c[j]);
+        }
+    }
+    if (lane == 0) {
+#pragma unroll
+        for (int i = 0; i < HB; ++i) { sm[wid][i][0] = m[i]; sm[wid][i][1] = l[i]; }
+    }
+    for (int i = threadIdx.x; i < HB * a.rank; i += 256) so[i] = 0.f;
+    __syncthreads();
+    for (int w = 0; w < 4; ++w) {                                  // waves add their share in turn: a fixed order
+        if (wid == w) {
+#pragma unroll
+            for (int i = 0; i < HB; ++i) {
+                const float mm = fmaxf(fmaxf(sm[0][i][0], sm[1][i][0]), fmaxf(sm[2][i][0], sm[3][i][0]));
+                const float f = l[i] > 0.f ? exp2f(m[i] - mm) : 0.f;
+#pragma unroll
+                for (int j = 0; j < RC; ++j) { const int r = 64 * j + lane; if (r < a.rank) so[i * a.rank + r] += f * o[i][j]; }
+            }
+        }
+        __syncthreads();
+    }
+    for (int i = threadIdx.x; i < HB * a.rank; i += 256) {
+        const int hh = h0 + i / a.rank;
+        if (hh < a.H) a.po[(((size_t)b * a.H + hh) * a.nsplit + s) * a.rank + i % a.rank] = so[i];
+    }
+    if (threadIdx.x < HB && h0 + (int)threadIdx.x < a.H) {
+        const int i = threadIdx.x;
+        float mm = -INFINITY, ll = 0.f;
+        for (int w = 0; w < 4; ++w) mm = fmaxf(mm, sm[w][i][0]);
+        for (int w = 0; w < 4; ++w) if (sm[w][i][1] > 0.f) ll += sm[w][i][1] * exp2f(sm[w][i][0] - mm);
+        float* ml = a.pml + (((size_t)b * a.H + h0 + i) * a.nsplit + s) * 2;
+        ml[0] = mm; ml[1] = ll;
+    }
+    tls.end();
+}
+
+// Combine the split records of (sequence, head), apply U_v (rows v of the workgroup's 32) and the head's gate.
+template <class T, class IT, int MB>
+__global__ __launch_bounds__(256) void latent_merge_uv_kernel(unsigned long long* tl, LatentArgs a) {
+    const TLStamp tls(tl);
+    extern __shared__ __attribute__((aligned(16))) float ol[];     // [MB][rank]
+    __shared__ float sw[MB][64];
+    const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6, h = blockIdx.x, v0 = blockIdx.y * 32, b0 = blockIdx.z * MB;
+    for (int m = wid; m < MB; m += 4) {
+        const size_t rec = ((size_t)min(b0 + m, a.B - 1) * a.H + h) * a.nsplit;
+        const float mm = lane < a.nsplit ? a.pml[(rec + lane) * 2] : -INFINITY, ll = lane < a.nsplit ? a.pml[(rec + lane) * 2 + 1] : 0.f;
+        const float top = wave_max(ll > 0.f ? mm : -INFINITY), f = ll > 0.f ? exp2f(mm - top) : 0.f;
+        const float den = wave_sum(f * ll);
+        sw[m][lane] = f / den;
+    }
+    __syncthreads();
+    for (int i = threadIdx.x; i < MB * a.rank; i += 256) {
+        const int m = i / a.rank, r = i % a.rank;
+        const float* p = a.po + ((size_t)min(b0 + m, a.B - 1) * a.H + h) * a.nsplit * a.rank + r;
+        float t = 0.f;
+        for (int s = 0; s < a.nsplit; ++s) {
+            const float f = sw[m][s];                              // empty splits hold zeros or nothing of this step
+            t = fmaf(f, f > 0.f ? p[(size_t)s * a.rank] : 0.f, t);
+        }
+        ol[i] = t;
+    }
+    __syncthreads();
+    constexpr int NW = WTraits<T>::NW;
+    const T* u = reinterpret_cast<const T*>(a.w_uv) + (size_t)h * a.D * a.rank;
+    for (int v = v0 + wid; v < min(v0 + 32, a.vdim); v += 4) {
+        float acc[MB];
+#pragma unroll
+        for (int m = 0; m < MB; ++m) acc[m] = 0.f;
+        for (int r = lane * NW; r < a.rank; r += 64 * NW) {
+            float w[NW];
+            WTraits<T>::decode(*reinterpret_cast<const uint4*>(u + (size_t)v * a.rank + r), w);
+#pragma unroll
+            for (int m = 0; m < MB; ++m)
+#pragma unroll
+                for (int j = 0; j < NW; ++j) acc[m] = fmaf(w[j], ol[m * a.rank + r + j], acc[m]);
+        }
+#pragma unroll
+        for (int m = 0; m < MB; ++m) {
+            const float y = wave_sum(acc[m]);
+            if (lane == 0 && b0 + m < a.B) {
+                const float g = to_f(reinterpret_cast<const IT*>(a.in)[(size_t)(b0 + m) * a.ld_in + a.g_off + h]);
+                reinterpret_cast<IT*>(a.out)[(size_t)(b0 + m) * a.ld_out + h * a.D + v] = from_f<IT>(y / (1.0f + expf(-g)));
+            }
+        }
+    }
+    tls.end();
+}
+
+// -------------------------------------------------------------------------------------------- rows (prompts, batches)
+template <class T>
+__global__ void stack_embed_kernel(const T* embed, const T* pos, const int32_t* tok, const int32_t* position, float* h, int W, int ld, int npos) {
+    const size_t row = blockIdx.x;
+    const T* e = embed + (size_t)tok[row] * W;
+    const T* p = pos ? pos + (size_t)min(max(position[row], 0), npos - 1) * W : nullptr;
+    for (int i = threadIdx.x; i < ld; i += blockDim.x) h[row * ld + i] = i < W ? to_f(e[i]) + (p ? to_f(p[i]) : 0.f) : 0.f;
+}
+
+// A prompt row's place: position, cache slot, row in the latent scratch, and whether it is one of the last R of its sequence (the ones the ring keeps)
+struct RowPlace { int32_t pos, slot, kv, store; };
+
+// latents of positions already in the ring -> scratch rows (a portion that continues a sequence)
+template <class T>
+__global__ void latent_gather_kernel(const RowPlace* pl, const T* cache, T* c_all, int R, int rank) {
+    const RowPlace p = pl[blockIdx.x];
+    const T* src = cache + ((size_t)p.slot * R + p.pos % R) * rank;
+    for (int r = threadIdx.x; r < rank; r += blockDim.x) c_all[(size_t)p.kv * rank + r] = src[r];
+}
+
+// new rows: normalise the latent part of the in-projection -> scratch row and, for the last R positions of a sequence, ring row
+template <class T>
+__global__ __launch_bounds__(256) void latent_rows_kernel(const RowPlace* pl, const T* in, int ld_in, int off, const float* c_norm, T* cache, T* c_all, int n,
+                                                          int R, int rank, int rank_true, float eps) {
+    const int i = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
+    if (i >= n) return;
+    const T* c = in + (size_t)i * ld_in + off;
+    float ss = 0.f;
+    for (int r = lane; r < rank; r += 64) { const float v = to_f(c[r]); ss = fmaf(v, v, ss); }
+    const float inv = 1.0f / sqrtf(wave_sum(ss) / rank_true + eps);
+    const RowPlace p = pl[i];
+    T* ring = cache + ((size_t)p.slot * R + p.pos % R) * rank;
+    for (int r = lane; r < rank; r += 64) {
+        const T v = from_f<T>(to_f(c[r]) * inv * c_norm[r]);
+        c_all[(size_t)p.kv * rank + r] = v;
+        if (p.store) ring[r] = v;
+    }
+}
+
+// argmax partials of fp32 logit rows: grid (nblk, rows)
+__global__ __launch_bounds__(256) void rows_argmax_kernel(unsigned long long* tl, const float* logits, int V, float* amax_val, int* amax_idx) {
+    const TLStamp tls(tl);
+    __shared__ float sv[4];
+    __shared__ int si[4];
+    const float* l = logits + (size_t)blockIdx.y * V;
+    float bv = -INFINITY;
+    int bi = 0x7FFFFFFF;
+    for (int i = blockIdx.x * 256 + threadIdx.x; i < V; i += gridDim.x * 256) if (l[i] > bv) { bv = l[i]; bi = i; }
+#pragma unroll
+    for (int off = 32; off >= 1; off >>= 1) {
+        const float ov = __shfl_xor(bv, off, 64);
+        const int oi = __shfl_xor(bi, off, 64);
+        if (ov > bv || (ov == bv && oi < bi)) { bv = ov; bi = oi; }
+    }
+    if ((threadIdx.x & 63) == 0) { sv[threadIdx.x >> 6] = bv; si[threadIdx.x >> 6] = bi; }
+    __syncthreads();
+    if (threadIdx.x == 0) {
+        for (int w = 1; w < 4; ++w)
+            if (sv[w] > bv || (sv[w] == bv && si[w] < bi)) { bv = sv[w]; bi = si[w]; }
+        amax_val[(size_t)blockIdx.y * gridDim.x + blockIdx.x] = bv;
+        amax_idx[(size_t)blockIdx.y * gridDim.x + blockIdx.x] = bi;
+    }
+    tls.end();
+}
+
+// -------------------------------------------------------------------------------------------- engine state
+struct Stack {
+    pgk_stack_config_t cfg;
+    std::vector<pgk_stack_layer_t> layers;
+    const void *embed = nullptr, *pos = nullptr, *head = nullptr;
+    const float* final_norm = nullptr;
+    int Wp = 0, max_in = 0, max_att = 0, max_ff = 0, max_heads_rank = 0, max_heads = 0;
+    std::vector<void*> cache;              // per layer [max_batch][R][rank]
+    std::vector<int> ring;                 // R per layer
+    std::vector<int32_t> len;              // per slot: positions held (host side; advanced with every step enqueued)
+    // decode buffers (rows = max_batch)
+    float *in32 = nullptr, *a32 = nullptr, *y32 = nullptr, *act32 = nullptr, *qlat = nullptr, *po = nullptr, *pml = nullptr;
+    void *x16 = nullptr, *in16 = nullptr, *a16 = nullptr, *y16 = nullptr, *gu16 = nullptr, *act16 = nullptr;
+    int max_split = 64;
+    // prompt buffers, grown on demand outside capture
+    void* pf = nullptr; size_t pf_bytes = 0;
+    void* tab = nullptr; size_t tab_bytes = 0;
+    size_t esize() const { return cfg.dtype == PGK_F32 ? 4 : 2; }
+};
+static Stack* stack_of(const Engine* e) { return (Stack*)e->kind_state; }
+
+static int pick_nsplit(const Engine* e, int B, const pgk_stack_layer_t& L, int R) {
+    const int htiles = ceil_div(L.heads, 16);
+    int s = ceil_div(R, 32);
+    const int want = 2 * e->cu_count / (B * htiles) > 0 ? 2 * e->cu_count / (B * htiles) : 1;
+    if (s > want) s = want;
+    return s > 64 ? 64 : (s < 1 ? 1 : s);
+}
+
+template <class T, int HB>
+static hipError_t launch_latent_attn(const LatentArgs& a, hipStream_t st) {
+    const dim3 grid(a.nsplit, ceil_div(a.H, HB), a.B);
+    const size_t lds = (size_t)HB * a.rank * 4;
+#define PGK_RC(N) if (a.rank <= 64 * N) return launch_k(&latent_attn_kernel<T, N, HB>, grid, dim3(256), lds, st, a);
+    PGK_RC(1) PGK_RC(2) PGK_RC(4) PGK_RC(8) PGK_RC(16)
+#undef PGK_RC
+    return launch_k(&latent_attn_kernel<T, 32, HB>, grid, dim3(256), lds, st, a);
+}
+
+// absorb -> attention over the ring -> merge + U_v + gate for B sequences whose in-projection rows are in `in`
+template <class T, class IT>
+static pgk_status latent_decode(Engine* e, int l, int B, const void* in, void* out, hipStream_t st, int* launches) {
+    Stack* s = stack_of(e);
+    const auto& L = s->layers[l];
+    LatentArgs a{};
+    a.in = in; a.ld_in = L.n_in; a.qn = L.heads * L.head_pad; a.g_off = a.qn + L.rank_pad;
+    a.w_uk = L.w_ukv; a.w_uv = (const char*)L.w_ukv + (size_t)L.heads * L.head_pad * L.rank_pad * sizeof(T);
+    a.c_norm = L.c_norm; a.cache = s->cache[l]; a.positions = e->positions;
+    a.B = B; a.H = L.heads; a.D = L.head_pad; a.dim = L.dim; a.vdim = L.vdim; a.rank = L.rank_pad; a.rank_true = L.rank; a.R = s->ring[l];
+    a.nsplit = pick_nsplit(e, B, L, a.R);
+    a.eps = s->cfg.norm_eps; a.scale = L.scale * LOG2E;
+    a.qlat = s->qlat; a.po = s->po; a.pml = s->pml; a.out = out; a.ld_out = L.heads * L.head_pad;
+    const int nx = L.heads * ceil_div(a.rank, 128) + 1;
+    if (B == 1) PGK_CHECK_HIP((launch_k(&latent_absorb_kernel<T, IT, 1>, dim3(nx, 1), dim3(256), 0, st, a)));
+    else PGK_CHECK_HIP((launch_k(&latent_absorb_kernel<T, IT, 4>, dim3(nx, ceil_div(B, 4)), dim3(256), 0, st, a)));
+    PGK_CHECK_HIP((launch_latent_attn<T, 4>(a, st)));
+    const int nv = ceil_div(a.vdim, 32);
+    if (B == 1) PGK_CHECK_HIP((launch_k(&latent_merge_uv_kernel<T, IT, 1>, dim3(a.H, nv, 1), dim3(256), (size_t)a.rank * 4, st, a)));
+    else PGK_CHECK_HIP((launch_k(&latent_merge_uv_kernel<T, IT, 4>, dim3(a.H, nv, ceil_div(B, 4)), dim3(256), (size_t)4 * a.rank * 4, st, a)));
+    *launches += 3;
+    return PGK_OK;
+}
+
+// ---- one sequence: fused steps, fp32 between kernels ----
+template <class T>
+static pgk_status step_one(Engine* e, hipStream_t st, int* launches) {
+    Stack* s = stack_of(e);
+    const auto& c = s->cfg;
+    float *x = e->h, *xn = e->h2;
+    const float* pend = nullptr;              // post-norm weight of the sublayer output waiting in y32
+    auto norm_in = [&](StackGemvArgs& a, const float* gamma) {
+        a.K = s->Wp; a.W = c.width; a.x = x; a.gamma = gamma; a.eps = c.norm_eps; a.mult = c.residual_mult;
+        if (pend) { a.y = s->y32; a.g_post = pend; a.x_out = xn; }
+    };
+    auto settle = [&]() { if (pend) { float* t = x; x = xn; xn = t; } pend = nullptr; };
+    for (int l = 0; l < c.num_layers; ++l) {
+        const auto& L = s->layers[l];
+        StackGemvArgs a{};
+        mark(KC_NORM_QKV);
+        norm_in(a, L.norm1);
+        a.w = L.w_in; a.N = L.n_in; a.out = s->in32;
+        if (pgk_status r = stack_gemv<T, SP_NORM, SE_STORE>(a, st)) return r;
+        settle();
+        mark(KC_ATTN);
+        if (pgk_status r = latent_decode<T, float>(e, l, 1, s->in32, s->a32, st, launches)) return r;
+        mark(KC_OPROJ);
+        a = StackGemvArgs{};
+        a.w = L.w_o; a.N = s->Wp; a.K = L.heads * L.head_pad; a.x = s->a32; a.out = s->y32;
+        if (pgk_status r = stack_gemv<T, SP_PLAIN, SE_STORE>(a, st)) return r;
+        pend = L.norm1b;
+        *launches += 2;
+        if (!L.ff_pad) continue;
+        mark(KC_GATEUP);
+        a = StackGemvArgs{};
+        norm_in(a, L.norm2);
+        a.w = L.w_gate_up; a.N = L.ff_pad; a.out = s->act32;
+        if (pgk_status r = stack_gemv<T, SP_NORM, SE_SWIGLU>(a, st)) return r;
+        settle();
+        mark(KC_DOWN);
+        a = StackGemvArgs{};
+        a.w = L.w_down; a.N = s->Wp; a.K = L.ff_pad; a.x = s->act32; a.out = s->y32;
+        if (pgk_status r = stack_gemv<T, SP_PLAIN, SE_STORE>(a, st)) return r;
+        pend = L.norm2b;
+        *launches += 2;
+    }
+    mark(KC_LMHEAD);
+    StackGemvArgs a{};
+    norm_in(a, s->final_norm);
+    a.x_out = nullptr;
+    a.w = s->head; a.N = c.vocab_size; a.out = e->logits; a.amax_val = e->amax_val; a.amax_idx = e->amax_idx;
+    if (pgk_status r = stack_gemv<T, SP_NORM, SE_LOGITS>(a, st, e->lm_blocks)) return r;
+    *launches += 1;
+    return PGK_OK;
+}
+
+// fp32 logits of `n` normalised rows (element type T, row stride Wp)
+template <class T>
+static pgk_status head_rows(Stack* s, const T* x, float* logits, int n, hipStream_t st) {
+    const int V = s->cfg.vocab_size;
+    if constexpr (std::is_same<T, float>::value) return pgk_gemm_nt(x, s->head, nullptr, logits, n, V, s->Wp, PGK_F32, st);
+    for (int r = 0; r < n; r += 128) {
+        const int m = n - r < 128 ? n - r : 128;
+        if (pgk_status q = wsgemm_nt((const bf16*)x + (size_t)r * s->Wp, s->Wp, s->head, nullptr, false, logits + (size_t)r * V, nullptr, 1, 1, m, V, s->Wp, st)) return q;
+    }
+    return PGK_OK;
+}
+
+struct RowBufs { float* h; void *x, *in, *a, *y, *gu, *act; };
+
+// feed-forward of n rows: act = silu(x W_g) * (x W_u), y = act W_d
+template <class T>
+static pgk_status rows_mlp(Stack* s, const pgk_stack_layer_t& L, const RowBufs& b, int n, hipStream_t st) {
+    constexpr pgk_dtype DT = std::is_same<T, float>::value ? PGK_F32 : PGK_BF16;
+    if (DT == PGK_BF16 && engine_gemm_swiglu_ok(n, L.ff_pad, s->Wp, false)) {
+        if (pgk_status r = engine_gemm_swiglu_nt((const bf16*)b.x, L.w_gate_up, nullptr, false, (bf16*)b.act, n, L.ff_pad, s->Wp, st)) return r;
+    } else {
+        if (pgk_status r = pgk_gemm_nt(b.x, L.w_gate_up, nullptr, b.gu, n, 2 * L.ff_pad, s->Wp, DT, st)) return r;
+        if (pgk_status r = pgk_glu_packed(b.gu, b.act, n, L.ff_pad, 0, DT, st)) return r;
+    }
+    return pgk_gemm_nt(b.act, L.w_down, nullptr, b.y, n, s->Wp, L.ff_pad, DT, st);
+}
+
+// The layers on n rows of b.h; `mix(l)` turns in-projection rows b.in into attention rows b.a.  Returns the pending post-norm.
+template <class T, class Mix>
+static pgk_status rows_layers(Stack* s, const RowBufs& b, int n, hipStream_t st, const float** pend_out, Mix mix) {
+    constexpr pgk_dtype DT = std::is_same<T, float>::value ? PGK_F32 : PGK_BF16;
+    const auto& c = s->cfg;
+    const float* pend = nullptr;
+    auto norm = [&](const float* gamma) -> pgk_status {
+        RowsNormArgs a{b.h, pend ? b.y : nullptr, s->Wp, pend, c.residual_mult, gamma, b.x, c.width, s->Wp, c.norm_eps, nullptr, 1};
+        return rows_norm(a, n, DT, st);
+    };
+    for (int l = 0; l < c.num_layers; ++l) {
+        const auto& L = s->layers[l];
+        mark(KC_NORM_QKV);
+        if (pgk_status r = norm(L.norm1)) return r;
+        if (pgk_status r = pgk_gemm_nt(b.x, L.w_in, nullptr, b.in, n, L.n_in, s->Wp, DT, st)) return r;
+        mark(KC_ATTN);
+        if (pgk_status r = mix(l)) return r;
+        mark(KC_OPROJ);
+        if (pgk_status r = pgk_gemm_nt(b.a, L.w_o, nullptr, b.y, n, s->Wp, L.heads * L.head_pad, DT, st)) return r;
+        pend = L.norm1b;
+        if (!L.ff_pad) continue;
+        mark(KC_GATEUP);
+        if (pgk_status r = norm(L.norm2)) return r;
+        if (pgk_status r = rows_mlp<T>(s, L, b, n, st)) return r;
+        pend = L.norm2b;
+    }
+    *pend_out = pend;
+    return PGK_OK;
+}
+
+constexpr int ROWS_ARGMAX_BLOCKS = 64;
+
+template <class T>
+static pgk_status step_rows(Engine* e, int B, hipStream_t st, int* launches) {
+    Stack* s = stack_of(e);
+    constexpr pgk_dtype DT = std::is_same<T, float>::value ? PGK_F32 : PGK_BF16;
+    const auto& c = s->cfg;
+    const RowBufs b{e->h, s->x16, s->in16, s->a16, s->y16, s->gu16, s->act16};
+    const float* pend = nullptr;
+    if (pgk_status r = rows_layers<T>(s, b, B, st, &pend, [&](int l) { return latent_decode<T, T>(e, l, B, b.in, b.a, st, launches); })) return r;
+    mark(KC_LMHEAD);
+    RowsNormArgs a{b.h, pend ? b.y : nullptr, s->Wp, pend, c.residual_mult, s->final_norm, b.x, c.width, s->Wp, c.norm_eps, nullptr, 1};
+    if (pgk_status r = rows_norm(a, B, DT, st)) return r;
+    if (pgk_status r = head_rows<T>(s, (const T*)b.x, e->logits, B, st)) return r;
+    PGK_CHECK_HIP(launch_k(rows_argmax_kernel, dim3(ROWS_ARGMAX_BLOCKS, B), dim3(256), 0, st, e->logits, c.vocab_size, e->amax_val, e->amax_idx));
+    *launches += 3;
+    for (const auto& L : s->layers) *launches += 3 + (L.ff_pad ? 4 : 0);
+    return PGK_OK;
+}
+
+template <class T>
+static pgk_status stack_step(Engine* e, int batch, hipStream_t st, int* launches) {
+    Stack* s = stack_of(e);
+    int nblk = ROWS_ARGMAX_BLOCKS;
+    if (batch == 1) {
+        nblk = e->lm_blocks;
+        if (pgk_status r = step_one<T>(e, st, launches)) return r;
+    } else if (pgk_status r = step_rows<T>(e, batch, st, launches)) return r;
+    mark(KC_ARGMAX);
+    const int32_t* sampled = nullptr;
+    if (e->sample_temperature > 0.f) {
+        if (pgk_status r = engine_sample(e, 0, batch, st)) return r;
+        sampled = e->sampled;
+        *launches += 1;
+    }
+    PGK_CHECK_HIP(launch_k(&finalize_kernel<T>, dim3(batch), dim3(256), 0, st, e->amax_val, e->amax_idx, nblk, e->tokens, e->positions, e->token_log,
+                           e->step_counter, e->cfg.max_batch, e->log_cap, (const T*)s->embed, e->h, s->cfg.width, 1, e->clk_log, (const float*)nullptr,
+                           (const float*)nullptr, (float*)nullptr, (float*)nullptr, 0, e->cfg.max_seq_len, batch, sampled, (const T*)s->pos, s->Wp));
+    *launches += 1;
+    return PGK_OK;
+}
+
+static pgk_status stack_decode_step(Engine* e, int batch, hipStream_t st, int* launches, bool) {
+    return stack_of(e)->cfg.dtype == PGK_F32 ? stack_step<float>(e, batch, st, launches) : stack_step<bf16>(e, batch, st, launches);
+}
+
+static pgk_status stack_embed_state(Engine* e, int batch, hipStream_t st) {
+    Stack* s = stack_of(e);
+    const auto& c = s->cfg;
+    if (c.dtype == PGK_F32) stack_embed_kernel<float><<<batch, 256, 0, st>>>((const float*)s->embed, (const float*)s->pos, e->tokens, e->positions, e->h, c.width, s->Wp, c.max_positions);
+    else stack_embed_kernel<bf16><<<batch, 256, 0, st>>>((const bf16*)s->embed, (const bf16*)s->pos, e->tokens, e->positions, e->h, c.width, s->Wp, c.max_positions);
+    PGK_LAUNCH_CHECK();
+    return PGK_OK;
+}
+
+// May slot `slot` go on at `pos`?  Position 0 starts a new sequence; otherwise the rows its windows reach must still be in the rings
+// (a ring row is overwritten by the position `R` later).
+static pgk_status check_position(const Engine* e, int slot, int pos) {
+    const Stack* s = stack_of(e);
+    const int len = s->len[slot];
+    PGK_REQUIRE(pos <= len, "engine: slot %d holds %d positions, cannot go on at position %d", slot, len, pos);
+    if (pos == 0 || pos == len) return PGK_OK;
+    for (int l = 0; l < s->cfg.num_layers; ++l) {
+        const int R = s->ring[l], first = pos - s->layers[l].window + 1 > 0 ? pos - s->layers[l].window + 1 : 0;
+        PGK_REQUIRE(first + R >= len, "engine: slot %d has moved on to position %d; the window of position %d is no longer in its ring", slot, len, pos);
+    }
+    return PGK_OK;
+}
+
+static pgk_status stack_check_state(Engine* e, const int32_t* h_positions, int batch) {
+    for (int b = 0; b < batch; ++b)
+        if (pgk_status r = check_position(e, b, h_positions[b])) return r;
+    for (int b = 0; b < batch; ++b) stack_of(e)->len[b] = h_positions[b];      // the step that follows writes position h_positions[b]
+    return PGK_OK;
+}
+
+static void stack_advance(Engine* e, int batch, int steps) {
+    for (int b = 0; b < batch; ++b) stack_of(e)->len[b] += steps;
+}
+
+template <class T>
+static pgk_status stack_prefill_t(Engine* e, int n_seqs, const int32_t* slots, const int32_t* lens, const int32_t* starts, const int32_t* tokens, int n_want,
+                                  const int32_t* want, float* h_logits, hipStream_t st) {
+    Stack* s = stack_of(e);
+    constexpr pgk_dtype DT = std::is_same<T, float>::value ? PGK_F32 : PGK_BF16;
+    const auto& c = s->cfg;
+    for (int i = 0; i < n_seqs; ++i)
+        if (pgk_status r = check_position(e, slots[i], starts[i])) return r;
+    int n = 0;
+    for (int i = 0; i < n_seqs; ++i) n += lens[i];
+    // per layer: which latent rows a sequence's queries reach (its own rows and up to window - 1 before them)
+    struct LayerRows { size_t past0 = 0; int n_past = 0, n_kv = 0; };
+    std::vector<LayerRows> lr(c.num_layers);
+    std::vector<RowPlace> place;                        // per layer: n_past gathered rows, then n new rows (equal layers share them)
+    std::vector<int> share(c.num_layers, -1);
+    int max_kv = 0;
+    for (int l = 0; l < c.num_layers; ++l) {
+        for (int k = 0; k < l && share[l] < 0; ++k)
+            if (share[k] < 0 && s->ring[k] == s->ring[l] && s->layers[k].window == s->layers[l].window) share[l] = k;
+        if (share[l] >= 0) { lr[l] = lr[share[l]]; continue; }
+        lr[l].past0 = place.size();
+        int kv = 0;
+        std::vector<RowPlace> fresh;
+        for (int i = 0; i < n_seqs; ++i) {
+            const int past = starts[i] < s->layers[l].window - 1 ? starts[i] : s->layers[l].window - 1, end = starts[i] + lens[i];
+            for (int p = starts[i] - past; p < starts[i]; ++p) place.push_back(RowPlace{p, slots[i], kv++, 0});
+            for (int p = starts[i]; p < end; ++p) fresh.push_back(RowPlace{p, slots[i], kv++, p >= end - s->ring[l] ? 1 : 0});
+            lr[l].n_past += past;
+        }
+        lr[l].n_kv = kv;
+        if (kv > max_kv) max_kv = kv;
+        place.insert(place.end(), fresh.begin(), fresh.end());
+    }
+    size_t kv_elems = 0, c_elems = 0;
+    for (int l = 0; l < c.num_layers; ++l) {
+        const auto& L = s->layers[l];
+        const size_t ke = (size_t)lr[l].n_kv * 2 * L.heads * L.head_pad, ce = (size_t)lr[l].n_kv * L.rank_pad;
+        if (ke > kv_elems) kv_elems = ke;
+        if (ce > c_elems) c_elems = ce;
+    }
+    const int wrows = n_want < 128 ? n_want : 128;
+    auto up = [](size_t v) { return (v + 255) & ~(size_t)255; };
+    const size_t E = sizeof(T);
+    const size_t sizes[] = {(size_t)n * s->Wp * 4, (size_t)n * s->Wp * E, (size_t)n * s->max_in * E, (size_t)n * s->max_att * E, (size_t)n * s->Wp * E,
+                            (size_t)n * 2 * s->max_ff * E, (size_t)n * s->max_ff * E, c_elems * E, kv_elems * E, (size_t)wrows * s->Wp * E, (size_t)wrows * c.vocab_size * 4};
+    size_t need = 0;
+    for (size_t z : sizes) need += up(z);
+    const size_t tab_need = up((size_t)n * 4) * 2 + up(place.size() * sizeof(RowPlace)) + up((size_t)n_want * 4);
+    auto grow = [&](void** p, size_t* have, size_t want_bytes) -> pgk_status {
+        if (want_bytes <= *have) return PGK_OK;
+        if (*p) { PGK_CHECK_HIP(hipStreamSynchronize(st)); pgk_free(*p); }
+        *p = nullptr; *have = 0;
+        if (pgk_status r = pgk_malloc(p, want_bytes)) return r;
+        *have = want_bytes;
+        return PGK_OK;
+    };
+    const size_t before = s->pf_bytes + s->tab_bytes;
+    if (pgk_status r = grow(&s->pf, &s->pf_bytes, need)) return r;
+    if (pgk_status r = grow(&s->tab, &s->tab_bytes, tab_need)) return r;
+    e->ws_bytes += s->pf_bytes + s->tab_bytes - before;
+    char* p = (char*)s->pf;
+    auto take = [&](size_t bytes) { char* q = p; p += up(bytes); return (void*)q; };
+    RowBufs b;
+    b.h = (float*)take(sizes[0]); b.x = take(sizes[1]); b.in = take(sizes[2]); b.a = take(sizes[3]); b.y = take(sizes[4]); b.gu = take(sizes[5]); b.act = take(sizes[6]);
+    T* c_all = (T*)take(sizes[7]);
+    T* kv = (T*)take(sizes[8]);
+    void* xw = take(sizes[9]);
+    float* lg = (float*)take(sizes[10]);
+    // one host image of the index tables, one copy
+    std::vector<char> img(tab_need, 0);
+    const size_t o_pos = up((size_t)n * 4), o_place = 2 * o_pos, o_want = o_place + up(place.size() * sizeof(RowPlace));
+    memcpy(img.data(), tokens, (size_t)n * 4);
+    for (int i = 0, row = 0; i < n_seqs; ++i)
+        for (int j = 0; j < lens[i]; ++j, ++row) ((int32_t*)(img.data() + o_pos))[row] = starts[i] + j;
+    if (!place.empty()) memcpy(img.data() + o_place, place.data(), place.size() * sizeof(RowPlace));
+    if (n_want) memcpy(img.data() + o_want, want, (size_t)n_want * 4);
+    PGK_CHECK_HIP(hipMemcpyAsync(s->tab, img.data(), tab_need, hipMemcpyHostToDevice, st));
+    PGK_CHECK_HIP(hipStreamSynchronize(st));      // the image is pageable host memory
+    const int32_t* d_tok = (const int32_t*)s->tab;
+    const int32_t* d_pos = (const int32_t*)((char*)s->tab + o_pos);
+    const RowPlace* d_place = (const RowPlace*)((char*)s->tab + o_place);
+    const int32_t* d_want = (const int32_t*)((char*)s->tab + o_want);
+    stack_embed_kernel<T><<<n, 256, 0, st>>>((const T*)s->embed, (const T*)s->pos, d_tok, d_pos, b.h, c.width, s->Wp, c.max_positions);
+    PGK_LAUNCH_CHECK();
+    auto mix = [&](int l) -> pgk_status {
+        const auto& L = s->layers[l];
+        const LayerRows& w = lr[l];
+        const int HD = L.heads * L.head_pad, R = s->ring[l];
+        if (w.n_past) {
+            latent_gather_kernel<T><<<w.n_past, 64, 0, st>>>(d_place + w.past0, (const T*)s->cache[l], c_all, R, L.rank_pad);
+            PGK_LAUNCH_CHECK();
+        }
+        latent_rows_kernel<T><<<ceil_div(n, 4), 256, 0, st>>>(d_place + w.past0 + w.n_past, (const T*)b.in, L.n_in, HD, L.c_norm, (T*)s->cache[l], c_all, n, R,
+                                                              L.rank_pad, L.rank, c.norm_eps);
+        PGK_LAUNCH_CHECK();
+        if (pgk_status r = pgk_gemm_nt(c_all, L.w_ukv, nullptr, kv, w.n_kv, 2 * HD, L.rank_pad, DT, st)) return r;
+        int row = 0, kv0 = 0;
+        const WindowStrides sd{L.head_pad, L.n_in, L.head_pad, 2 * HD, L.head_pad, 2 * HD, L.head_pad, HD};
+        for (int i = 0; i < n_seqs; ++i) {
+            const int past = starts[i] < L.window - 1 ? starts[i] : L.window - 1, klen = past + lens[i];
+            const T* q = (const T*)b.in + (size_t)row * L.n_in;
+            const T* k = kv + (size_t)kv0 * 2 * HD;
+            if (pgk_status r = window_attention(q, k, k + HD, (T*)b.a + (size_t)row * HD, L.heads, L.heads, lens[i], klen, L.head_pad, L.head_pad, L.scale, L.window, sd,
+                                                q + HD + L.rank_pad, L.n_in, DT, st))
+                return r;
+            row += lens[i];
+            kv0 += klen;
+        }
+        return PGK_OK;
+    };
+    const float* pend = nullptr;
+    if (pgk_status r = rows_layers<T>(s, b, n, st, &pend, mix)) return r;
+    for (int i = 0; i < n_seqs; ++i) s->len[slots[i]] = starts[i] + lens[i];
+    for (int w0 = 0; w0 < n_want; w0 += 128) {
+        const int m = n_want - w0 < 128 ? n_want - w0 : 128;
+        RowsNormArgs a{b.h, pend ? b.y : nullptr, s->Wp, pend, c.residual_mult, s->final_norm, xw, c.width, s->Wp, c.norm_eps, d_want + w0, 0};
+        if (pgk_status r = rows_norm(a, m, DT, st)) return r;
+        if (pgk_status r = head_rows<T>(s, (const T*)xw, lg, m, st)) return r;
+        PGK_CHECK_HIP(hipMemcpyAsync(h_logits + (size_t)w0 * c.vocab_size, lg, (size_t)m * c.vocab_size * 4, hipMemcpyDeviceToHost, st));
+        PGK_CHECK_HIP(hipStreamSynchronize(st));
+    }
+    return PGK_OK;
+}
+
+static pgk_status stack_prefill(Engine* e, int n_seqs, const int32_t* slots, const int32_t* lens, const int32_t* starts, const int32_t* tokens, int n_want,
+                                const int32_t* want, float* h_logits, hipStream_t st) {
+    if (stack_of(e)->cfg.dtype == PGK_F32) return stack_prefill_t<float>(e, n_seqs, slots, lens, starts, tokens, n_want, want, h_logits, st);
+    return stack_prefill_t<bf16>(e, n_seqs, slots, lens, starts, tokens, n_want, want, h_logits, st);
+}
+
+// layer l's latent ring [max_batch][R][rank_pad]; there is no value cache
+static pgk_status stack_kv_ptr(Engine* e, int layer, void** k, void** v) {
+    *k = stack_of(e)->cache[layer];
+    *v = nullptr;
+    return PGK_OK;
+}
+
+static void stack_destroy(Engine* e) {
+    Stack* s = stack_of(e);
+    if (s->pf) (void)pgk_free(s->pf);
+    if (s->tab) (void)pgk_free(s->tab);
+    delete s;
+    e->kind_state = nullptr;
+}
+
+static const EngineKind STACK_KIND = {stack_decode_step, stack_prefill, nullptr, stack_embed_state, stack_check_state, stack_advance, stack_kv_ptr, stack_destroy};
+
+}  // namespace pgk
+
+using namespace pgk;
+
+extern "C" {
+
+pgk_status pgk_engine_create_stack(const pgk_stack_config_t* cfg, const void* embed, const void* pos_embed, const void* head, const float* final_norm,
+                                   const pgk_stack_layer_t* layers, pgk_engine* out) {
+    PGK_REQUIRE(cfg && embed && head && final_norm && layers && out, "pgk_engine_create_stack: null argument");
+    const auto& c = *cfg;
+    PGK_REQUIRE(c.dtype == PGK_BF16 || c.dtype == PGK_F32, "pgk_engine_create_stack: dtype %d (bf16 or f32)", (int)c.dtype);
+    PGK_REQUIRE(c.vocab_size >= 1 && c.width >= 1 && c.num_layers >= 1 && c.max_batch >= 1 && c.max_seq_len >= 1, "pgk_engine_create_stack: bad sizes");
+    PGK_REQUIRE(!pos_embed || c.max_seq_len <= c.max_positions, "pgk_engine_create_stack: %d positions of cache but %d learned positions", c.max_seq_len, c.max_positions);
+    const int Wp = ceil_div(c.width, 64) * 64;
+    for (int l = 0; l < c.num_layers; ++l) {
+        const auto& L = layers[l];
+        PGK_REQUIRE(L.heads >= 1 && L.dim >= 1 && L.vdim >= 1 && L.rank >= 1 && L.window >= 1, "pgk_engine_create_stack: layer %d: bad mixer sizes", l);
+        PGK_REQUIRE(L.head_pad % 64 == 0 && L.head_pad >= L.dim && L.head_pad >= L.vdim, "pgk_engine_create_stack: layer %d: head pad %d for widths %d / %d", l, L.head_pad, L.dim, L.vdim);
+        PGK_REQUIRE(L.rank_pad % 64 == 0 && L.rank_pad >= L.rank && L.rank_pad <= 2048, "pgk_engine_create_stack: layer %d: latent size %d padded to %d (at most 2048)", l, L.rank, L.rank_pad);
+        PGK_REQUIRE(L.n_in % 64 == 0 && L.n_in >= L.heads * L.head_pad + L.rank_pad + L.heads, "pgk_engine_create_stack: layer %d: in-projection rows %d", l, L.n_in);
+        PGK_REQUIRE(L.ff_pad % 64 == 0 && L.ff_pad >= 0, "pgk_engine_create_stack: layer %d: feed-forward pad %d", l, L.ff_pad);
+        PGK_REQUIRE(L.norm1 && L.norm1b && L.w_in && L.c_norm && L.w_ukv && L.w_o && (!L.ff_pad || (L.norm2 && L.norm2b && L.w_gate_up && L.w_down)),
+                    "pgk_engine_create_stack: layer %d: missing weights", l);
+    }
+    Engine* e = new Engine();
+    Stack* s = new Stack();
+    e->kind = &STACK_KIND;
+    e->kind_state = s;
+    e->one_sequence = true;
+    s->cfg = c;
+    s->layers.assign(layers, layers + c.num_layers);
+    s->embed = embed; s->pos = pos_embed; s->head = head; s->final_norm = final_norm;
+    s->Wp = Wp;
+    s->len.assign(c.max_batch, 0);
+    e->cfg = pgk_model_config_t{};
+    e->cfg.vocab_size = c.vocab_size; e->cfg.hidden_size = c.width; e->cfg.num_layers = c.num_layers;
+    e->cfg.max_seq_len = c.max_seq_len; e->cfg.max_batch = c.max_batch; e->cfg.norm_eps = c.norm_eps;
+    {
+        int dev = 0;
+        hipDeviceProp_t prop;
+        if (hipGetDevice(&dev) == hipSuccess && hipGetDeviceProperties(&prop, dev) == hipSuccess && prop.multiProcessorCount > 0) e->cu_count = prop.multiProcessorCount;
+    }
+    e->lm_blocks = ceil_div(c.vocab_size, 16) < 1024 ? ceil_div(c.vocab_size, 16) : 1024;
+    e->lm_cap = e->lm_blocks > ROWS_ARGMAX_BLOCKS ? e->lm_blocks : ROWS_ARGMAX_BLOCKS;
+    pgk_status r = PGK_OK;
+    std::vector<std::pair<void*, size_t>> clear;
+    auto A = [&](void** p, size_t bytes, size_t* acct, bool zero = false) {
+        if (r == PGK_OK) r = dev_alloc(e, p, bytes, acct);
+        if (r == PGK_OK && zero) clear.push_back({*p, bytes});
+    };
+    const size_t B = c.max_batch, E = s->esize();
+    size_t part = 0, ml = 0, ql = 0;
+    for (int l = 0; l < c.num_layers; ++l) {
+        const auto& L = s->layers[l];
+        const int R = L.window < c.max_seq_len ? L.window : c.max_seq_len;
+        s->ring.push_back(R);
+        void* p = nullptr;
+        A(&p, B * R * L.rank_pad * E, &e->kv_bytes, true);
+        s->cache.push_back(p);
+        if (L.n_in > s->max_in) s->max_in = L.n_in;
+        if (L.heads * L.head_pad > s->max_att) s->max_att = L.heads * L.head_pad;
+        if (L.ff_pad > s->max_ff) s->max_ff = L.ff_pad;
+        for (int m = 1; m <= c.max_batch; ++m) {
+            const size_t ns = (size_t)pick_nsplit(e, m, L, R) * m * L.heads;
+            if (ns * L.rank_pad > part) part = ns * L.rank_pad;
+            if (ns * 2 > ml) ml = ns * 2;
+        }
+        if (B * L.heads * L.rank_pad > ql) ql = B * L.heads * L.rank_pad;
+    }
+    A((void**)&e->tokens, B * 4, &e->ws_bytes, true);
+    A((void**)&e->positions, B * 4, &e->ws_bytes, true);
+    A((void**)&e->token_log, (size_t)e->log_cap * B * 4, &e->ws_bytes);
+    A((void**)&e->step_counter, 16, &e->ws_bytes, true);
+    A((void**)&e->h, B * Wp * 4, &e->ws_bytes, true);
+    A((void**)&e->h2, B * Wp * 4, &e->ws_bytes, true);
+    A((void**)&e->logits, B * c.vocab_size * 4, &e->ws_bytes);
+    A((void**)&e->amax_val, B * e->lm_cap * 4, &e->ws_bytes);
+    A((void**)&e->amax_idx, B * e->lm_cap * 4, &e->ws_bytes);
+    A((void**)&e->clk_log, (size_t)e->log_cap * 16, &e->ws_bytes);
+    A((void**)&s->in32, (size_t)s->max_in * 4, &e->ws_bytes);
+    A((void**)&s->a32, (size_t)s->max_att * 4, &e->ws_bytes, true);     // padding columns of a head are never written: zero
+    A((void**)&s->y32, (size_t)Wp * 4, &e->ws_bytes, true);
+    A((void**)&s->act32, (size_t)(s->max_ff ? s->max_ff : 64) * 4, &e->ws_bytes);
+    A((void**)&s->qlat, ql * 4, &e->ws_bytes);
+    A((void**)&s->po, part * 4, &e->ws_bytes);
+    A((void**)&s->pml, ml * 4, &e->ws_bytes);
+    A(&s->x16, B * Wp * E, &e->ws_bytes);
+    A(&s->in16, B * s->max_in * E, &e->ws_bytes);
+    A(&s->a16, B * s->max_att * E, &e->ws_bytes, true);
+    A(&s->y16, B * Wp * E, &e->ws_bytes);
+    A(&s->gu16, B * 2 * (s->max_ff ? s->max_ff : 64) * E, &e->ws_bytes);
+    A(&s->act16, B * (s->max_ff ? s->max_ff : 64) * E, &e->ws_bytes);
+    if (r == PGK_OK) {
+        hipStream_t st = resolve_stream(nullptr);
+        hipError_t he = hipSuccess;
+        for (const auto& z : clear) if (he == hipSuccess) he = hipMemsetAsync(z.first, 0, z.second, st);
+        if (he == hipSuccess) he = hipStreamSynchronize(st);
+        if (he != hipSuccess) r = set_error(PGK_ERR_HIP, "pgk_engine_create_stack: %s", hipGetErrorString(he));
+    }
+    if (r != PGK_OK) { pgk_engine_destroy(e); return r; }
+    *out = e;
+    return PGK_OK;
+}
+
+}  // extern "C"

@@ -1,0 +1,49 @@
+// Shared by ops_latent.hip (operators) and engine_stack.hip (engine): fp32-stream norms and sliding-window attention.
+#pragma once
+
+#include "gemv_core.hip.h"
+#include "pgk_device.hip.h"
+#include "pgk_internal.h"
+
+namespace pgk {
+
+template <class T> __device__ __forceinline__ float4 load4(const T* p);
+template <> __device__ __forceinline__ float4 load4<float>(const float* p) { return *reinterpret_cast<const float4*>(p); }
+template <> __device__ __forceinline__ float4 load4<bf16>(const bf16* p) {
+    const uint2 g = *reinterpret_cast<const uint2*>(p);
+    return make_float4(__uint_as_float(g.x << 16), __uint_as_float(g.x & 0xFFFF0000u), __uint_as_float(g.y << 16), __uint_as_float(g.y & 0xFFFF0000u));
+}
+template <class T> __device__ __forceinline__ void store4(T* p, const float4& v);
+template <> __device__ __forceinline__ void store4<float>(float* p, const float4& v) { *reinterpret_cast<float4*>(p) = v; }
+template <> __device__ __forceinline__ void store4<bf16>(bf16* p, const float4& v) {
+    *reinterpret_cast<uint2*>(p) = make_uint2(pack_bf16x2(v.x, v.y), pack_bf16x2(v.z, v.w));
+}
+
+// One sandwich step on rows of the fp32 stream h [*][ld] (columns W..ld are zero padding):
+//   y given:    h += mult * y / rms(y) * g_post       (y rows in the engine's element type, row stride ldy; store_h: write h back)
+//   out given:  out[i] = h / rms(h) * gamma           (rows of stride ld in the engine's element type)
+// Workgroup i works on row rows[i] (null: row i) and writes out row i.  The norm weights are fp32, offsets already applied.
+struct RowsNormArgs {
+    float* h;
+    const void* y;
+    int ldy;
+    const float* g_post;
+    float mult;
+    const float* gamma;
+    void* out;
+    int W, ld;
+    float eps;
+    const int32_t* rows;
+    int store_h;
+};
+pgk_status rows_norm(const RowsNormArgs& a, int n, pgk_dtype dt, hipStream_t st);
+
+struct WindowStrides { long long qh, qs, kh, ks, vh, vs, oh, os; };   // elements: per head, per row
+// out[i] = sigmoid(gate[i][head]) * softmax over keys i' with 0 <= i - i' < window (queries are the last q_len of kv_len positions)
+pgk_status window_attention(const void* q, const void* k, const void* v, void* out, int hq, int hkv, int q_len, int kv_len, int dk, int dv, float scale,
+                            int window, const WindowStrides& sd, const void* gate, long long gs, pgk_dtype dt, hipStream_t st);
+pgk_status flash_window(const void* q, const void* k, const void* v, void* out, int hq, int hkv, int q_len, int kv_len, int d, float scale,
+                        int window, const void* gate, long long gs, long long qh, long long qs, long long kh, long long ks, long long oh,
+                        long long os, hipStream_t st);   // ops_flash.hip
+
+}  // namespace pgk

@@ -69,10 +69,23 @@ struct FlashSplit {
     float* q8s;
 };
 
-template <class T, int D>
+// Sliding window (WIN instantiations): query i sees keys i - window + 1 .. i, tiles left of a workgroup's first window are never
+// loaded.  `gate` (may be null): one value per (query row, head) at gate[row * gs + head]; the head's output row is multiplied by
+// its sigmoid.  The scores are scaled in fp32 after the product (scale > 0: the running maximum is kept on unscaled scores).
+struct FlashWindow {
+    int window;
+    const void* gate;
+    long long gs;
+};
+template <class T> __device__ __forceinline__ float flash_gate(const FlashWindow& w, int qrow, int head) {
+    if (!w.gate) return 1.f;
+    return 1.0f / (1.0f + __expf(-to_f(reinterpret_cast<const T*>(w.gate)[(long long)qrow * w.gs + head])));
+}
+
+template <class T, int D, bool WIN = false>
 __global__ __launch_bounds__(FL_THREADS, 2) void flash_fwd_kernel(const T* q, const T* k, const T* vt, T* out, int hq, int hkv,
                                                               int q_len, int kv_len, int kv_pad, float scale_log2e, FlashStrides sd,
-                                                              FlashSplit sp) {
+                                                              FlashSplit sp, FlashWindow win) {
     constexpr int NC = D / 8;            // 16-byte chunks per K row
     constexpr int KS = D / 16;           // k-steps of Q.K^T
     constexpr int DT = D / 32;           // 32-row tiles of O^T
@@ -117,7 +130,7 @@ __global__ __launch_bounds__(FL_THREADS, 2) void flash_fwd_kernel(const T* q, co
             float f[8];
             v.to_float(f);
 #pragma unroll
-            for (int j = 0; j < 8; ++j) f[j] *= scale_log2e;
+            for (int j = 0; j < 8; ++j) f[j] *= WIN ? 1.f : scale_log2e;
             v.from_float(f);
             qf[ks] = v.raw;
         }
@@ -133,7 +146,9 @@ __global__ __launch_bounds__(FL_THREADS, 2) void flash_fwd_kernel(const T* q, co
     const int kv_end = min(kv_len, causal_off + q_last + 1);
     const int nt_all = (kv_end + FL_BKV - 1) / FL_BKV;
     // this workgroup's run of KV tiles [t0, t1)
-    const int t0 = (int)((long long)nt_all * split / sp.nsplit), t1 = (int)((long long)nt_all * (split + 1) / sp.nsplit);
+    const int first_kv = WIN ? causal_off + qt * FL_BQ - win.window + 1 : 0;
+    const int tb = WIN && first_kv > 0 ? first_kv / FL_BKV : 0;            // tiles before it are outside every row's window
+    const int t0 = tb + (int)((long long)(nt_all - tb) * split / sp.nsplit), t1 = tb + (int)((long long)(nt_all - tb) * (split + 1) / sp.nsplit);
 
     // staging in NAMED registers (an array here ends up in scratch memory at this register pressure, see
     // ops_fp8_gemm.hip): chunk i of this thread is c = tid + 256 i; KCH = VCH = D / 32 chunks each
@@ -212,7 +227,9 @@ __global__ __launch_bounds__(FL_THREADS, 2) void flash_fwd_kernel(const T* q, co
         }
     };
     // tiles entirely above this wave's diagonal contribute nothing (wave-uniform)
-    auto live = [&](int t) -> bool { return t < t1 && t * FL_BKV <= causal_off + qw0 + 31; };
+    auto live = [&](int t) -> bool {
+        return t < t1 && t * FL_BKV <= causal_off + qw0 + 31 && (!WIN || t * FL_BKV + FL_BKV - 1 > causal_off + qw0 - win.window);
+    };
 
     // One KV tile per iteration: S = K . Q^T, softmax, O += V . P; the global loads of tile t + 1 are issued before the MFMAs of
     // tile t and parked in the other LDS buffer after them: one barrier per tile.  (Tried in round 3: multiplying S(t + 1) under
@@ -240,15 +257,17 @@ __global__ __launch_bounds__(FL_THREADS, 2) void flash_fwd_kernel(const T* q, co
         if (cur) qk(buf, sc0, sc1);
         if (cur) {
             // ---- mask, online softmax (this lane: query qw0 + ql, kv rows (r&3) + 8(r>>2) + 4h of each sub-tile) ----
-            const bool need_mask = kv0 + FL_BKV - 1 > causal_off + qw0 || kv0 + FL_BKV > kv_len;   // wave-uniform
+            const bool need_mask = kv0 + FL_BKV - 1 > causal_off + qw0 || kv0 + FL_BKV > kv_len ||
+                                   (WIN && kv0 <= causal_off + qw0 + 31 - win.window);   // wave-uniform
             const int lim = min(causal_off + qw0 + ql, kv_len - 1) - kv0 - 4 * h;                  // local kv row <= lim is visible
+            const int low = WIN ? causal_off + qw0 + ql - win.window + 1 - kv0 - 4 * h : 0;       // ... and >= low with a window
             float mx = -INFINITY;
             if (need_mask) {   // diagonal / ragged tiles only: a real wave-uniform branch, not 32 predicated selects per tile
 #pragma unroll
                 for (int r = 0; r < 16; ++r) {
                     const int kvl = (r & 3) + 8 * (r >> 2);
-                    sc0[r] = kvl <= lim ? sc0[r] : -INFINITY;
-                    sc1[r] = 32 + kvl <= lim ? sc1[r] : -INFINITY;
+                    sc0[r] = kvl <= lim && (!WIN || kvl >= low) ? sc0[r] : -INFINITY;
+                    sc1[r] = 32 + kvl <= lim && (!WIN || 32 + kvl >= low) ? sc1[r] : -INFINITY;
                 }
             }
             // (this file is built with -fno-honor-nans: without it every operand of a max is first canonicalised with a
@@ -256,6 +275,7 @@ __global__ __launch_bounds__(FL_THREADS, 2) void flash_fwd_kernel(const T* q, co
 #pragma unroll
             for (int r = 0; r < 16; r += 2) mx = fmaxf(fmaxf(fmaxf(sc0[r], sc1[r]), fmaxf(sc0[r + 1], sc1[r + 1])), mx);
             mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
+            if constexpr (WIN) mx *= scale_log2e;                        // -inf stays -inf (scale > 0)
             // Deferred rescale: the reference point of a row only moves when its maximum grew by more than 6 (log2
             // domain), so probabilities stay <= 64 (exact in fp32 sums, fine in 16-bit P) and on most tiles - for the whole
             // wave - alpha is exactly 1 and the 64-multiply rescale of O is skipped.
@@ -266,8 +286,13 @@ __global__ __launch_bounds__(FL_THREADS, 2) void flash_fwd_kernel(const T* q, co
             float ls = 0.f;
 #pragma unroll
             for (int r = 0; r < 16; ++r) {
-                sc0[r] = __builtin_amdgcn_exp2f(sc0[r] - m_use);
-                sc1[r] = __builtin_amdgcn_exp2f(sc1[r] - m_use);
+                if constexpr (WIN) {
+                    sc0[r] = __builtin_amdgcn_exp2f(fmaf(sc0[r], scale_log2e, -m_use));
+                    sc1[r] = __builtin_amdgcn_exp2f(fmaf(sc1[r], scale_log2e, -m_use));
+                } else {
+                    sc0[r] = __builtin_amdgcn_exp2f(sc0[r] - m_use);
+                    sc1[r] = __builtin_amdgcn_exp2f(sc1[r] - m_use);
+                }
                 ls += sc0[r] + sc1[r];
             }
             l_run = l_run * alpha + ls;
@@ -312,8 +337,9 @@ __global__ __launch_bounds__(FL_THREADS, 2) void flash_fwd_kernel(const T* q, co
 
     // ---- normalise and store: lane = query row, registers 4g..4g+3 of tile i are d = 32i + 8g + 4h .. +3 ----
     const float l_tot = l_run + __shfl_xor(l_run, 32, 64);
-    const float inv = l_tot > 0.f ? 1.f / l_tot : 0.f;
+    float inv = l_tot > 0.f ? 1.f / l_tot : 0.f;
     const int qrow = qw0 + ql;
+    if constexpr (WIN) { if (sp.nsplit == 1) inv *= flash_gate<T>(win, min(qrow, q_len - 1), head); }
     if constexpr (std::is_same<T, bf16>::value && D == 128) {
         if (sp.q8 != nullptr && sp.nsplit == 1) {       // workgroup-uniform
             // the lane's 64 dims (the partner lane ^ 32 holds the other 64), rounded to bf16 as the plain store would
@@ -363,7 +389,7 @@ __global__ __launch_bounds__(FL_THREADS, 2) void flash_fwd_kernel(const T* q, co
 // out[q][head][:] = sum_s w_s o_s / sum_s w_s,  w_s = l_s 2^(m_s - max m): one thread per 8 output elements
 template <class T, int D>
 __global__ __launch_bounds__(256) void flash_merge_kernel(const float* ml, const T* po, T* out, int hq, int q_len, int nsplit, long long oh, long long os,
-                                                          uint8_t* q8 = nullptr, float* q8s = nullptr) {
+                                                          uint8_t* q8 = nullptr, float* q8s = nullptr, FlashWindow win = FlashWindow{}) {
     constexpr int CPR = D / 8;
     const size_t gid = (size_t)blockIdx.x * 256 + threadIdx.x;
     const size_t nrow = (size_t)q_len * hq;
@@ -386,7 +412,7 @@ __global__ __launch_bounds__(256) void flash_merge_kernel(const float* ml, const
             den += w;
         }
     }
-    const float inv = den > 0.f ? 1.f / den : 0.f;
+    const float inv = (den > 0.f ? 1.f / den : 0.f) * flash_gate<T>(win, qrow, head);
 #pragma unroll
     for (int j = 0; j < 8; ++j) acc[j] *= inv;
     Vec<T> v;
@@ -440,9 +466,9 @@ __global__ __launch_bounds__(256) void transpose_v_kernel(const T* v, T* vt, int
     }
 }
 
-template <class T, int D>
+template <class T, int D, bool WIN = false>
 static pgk_status flash_launch(const T* q, const T* k, const T* v, T* out, int hq, int hkv, int q_len, int kv_len, float scale,
-                               const FlashStrides& sd, hipStream_t st, uint8_t* q8 = nullptr, float* q8s = nullptr) {
+                               const FlashStrides& sd, hipStream_t st, uint8_t* q8 = nullptr, float* q8s = nullptr, const FlashWindow& win = FlashWindow{}) {
     const int kv_pad = ceil_div(kv_len, 64) * 64;
     const int nqt = ceil_div(q_len, FL_BQ);
     // KV runs per query tile: enough workgroups for two per CU (the kernel's occupancy), never more runs than the
@@ -453,7 +479,8 @@ static pgk_status flash_launch(const T* q, const T* k, const T* v, T* out, int h
         hipDeviceProp_t prop;
         if (hipGetDevice(&dev) == hipSuccess && hipGetDeviceProperties(&prop, dev) == hipSuccess && prop.multiProcessorCount > 0) cus = prop.multiProcessorCount;
         const long long wgs = (long long)nqt * hq;
-        while (nsplit < 4 && wgs * nsplit < 2LL * cus && ceil_div(kv_len, FL_BKV) >= 4 * (nsplit * 2)) nsplit *= 2;
+        const int span = WIN && (long long)win.window + FL_BQ < kv_len ? win.window + FL_BQ : kv_len;    // keys the heaviest query tile walks
+        while (nsplit < 4 && wgs * nsplit < 2LL * cus && ceil_div(span, FL_BKV) >= 4 * (nsplit * 2)) nsplit *= 2;
     }
     const size_t vt_bytes = (size_t)hkv * D * kv_pad * sizeof(T);
     const size_t po_bytes = nsplit > 1 ? (size_t)nsplit * q_len * hq * D * sizeof(T) : 0;
@@ -471,16 +498,16 @@ static pgk_status flash_launch(const T* q, const T* k, const T* v, T* out, int h
     constexpr size_t LDS = 2 * (size_t)(64 * D * 2) + 2 * (size_t)(D * 128);
     static bool attr_done = false;
     if (LDS > 48 * 1024 && !attr_done) {
-        PGK_CHECK_HIP(hipFuncSetAttribute(reinterpret_cast<const void*>(&flash_fwd_kernel<T, D>),
+        PGK_CHECK_HIP(hipFuncSetAttribute(reinterpret_cast<const void*>(&flash_fwd_kernel<T, D, WIN>),
                                           hipFuncAttributeMaxDynamicSharedMemorySize, (int)LDS));
         attr_done = true;
     }
-    flash_fwd_kernel<T, D><<<nqt * hq * nsplit, FL_THREADS, LDS, st>>>(q, k, (const T*)vt, out, hq, hkv, q_len, kv_len, kv_pad,
-                                                                      scale * 1.4426950408889634f, sd, sp);
+    flash_fwd_kernel<T, D, WIN><<<nqt * hq * nsplit, FL_THREADS, LDS, st>>>(q, k, (const T*)vt, out, hq, hkv, q_len, kv_len, kv_pad,
+                                                                      scale * 1.4426950408889634f, sd, sp, win);
     hipError_t e = hipGetLastError();
     if (e == hipSuccess && nsplit > 1) {
         const size_t work = (size_t)q_len * hq * (D / 8);
-        flash_merge_kernel<T, D><<<(unsigned)((work + 255) / 256), 256, 0, st>>>(sp.ml, (const T*)sp.o, out, hq, q_len, nsplit, sd.oh, sd.os, q8, q8s);
+        flash_merge_kernel<T, D><<<(unsigned)((work + 255) / 256), 256, 0, st>>>(sp.ml, (const T*)sp.o, out, hq, q_len, nsplit, sd.oh, sd.os, q8, q8s, win);
         e = hipGetLastError();
     }
     pgk_free(ws);   // stream-ordered reuse: later work on this stream runs after the kernels above
@@ -499,6 +526,18 @@ pgk_status flash_prefill(const void* q, const void* k, const void* v, void* out,
     }
     if (d == 128) return flash_launch<f16, 128>((const f16*)q, (const f16*)k, (const f16*)v, (f16*)out, hq, hkv, q_len, kv_len, scale, sd, st);
     return flash_launch<f16, 64>((const f16*)q, (const f16*)k, (const f16*)v, (f16*)out, hq, hkv, q_len, kv_len, scale, sd, st);
+}
+
+// sliding-window causal attention with an optional per-head output gate (bf16, head_dim 64 / 128, one key head per query head or
+// a divisor, scale > 0): ops_latent.hip, engine_stack.hip
+pgk_status flash_window(const void* q, const void* k, const void* v, void* out, int hq, int hkv, int q_len, int kv_len, int d, float scale,
+                        int window, const void* gate, long long gs, long long qh, long long qs, long long kh, long long ks, long long oh,
+                        long long os, hipStream_t st) {
+    PGK_REQUIRE((d == 64 || d == 128) && window >= 1 && scale > 0.f && kv_len >= q_len, "flash_window: d=%d window=%d q_len=%d kv_len=%d", d, window, q_len, kv_len);
+    const FlashStrides sd{qh, qs, kh, ks, oh, os};
+    const FlashWindow win{window, gate, gs};
+    if (d == 128) return flash_launch<bf16, 128, true>((const bf16*)q, (const bf16*)k, (const bf16*)v, (bf16*)out, hq, hkv, q_len, kv_len, scale, sd, st, nullptr, nullptr, win);
+    return flash_launch<bf16, 64, true>((const bf16*)q, (const bf16*)k, (const bf16*)v, (bf16*)out, hq, hkv, q_len, kv_len, scale, sd, st, nullptr, nullptr, win);
 }
 
 // engine entry (fp8 x fp8 prefill, bf16, head_dim 128, q_len > 128): causal attention whose result leaves as the o_proj's fp8

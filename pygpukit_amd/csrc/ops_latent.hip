@@ -1,0 +1,236 @@
+// Operators of the layer-list models (llm/layers/latent_attention.py, engine_stack.hip): RMSNorm of an fp32 stream with fp32 weights,
+// normalised residual add, sliding-window attention with separate key / value widths, per-head sigmoid gate, zero padding.
+
+#include "latent.hip.h"
+
+namespace pgk {
+
+// One workgroup per row; see latent.hip.h.  NT float4 per thread keep the row in registers between the two reductions.
+template <class T, class YT, int NT>
+__global__ __launch_bounds__(256) void rows_norm_kernel(RowsNormArgs a) {
+    __shared__ float red[16];
+    const int row = a.rows ? a.rows[blockIdx.x] : blockIdx.x;
+    float* hr = a.h + (size_t)row * a.ld;
+    float4 v[NT];
+    const int nt = a.ld;
+#pragma unroll
+    for (int t = 0; t < NT; ++t) {
+        const int i = (threadIdx.x + 256 * t) * 4;
+        v[t] = i < nt ? *reinterpret_cast<const float4*>(hr + i) : make_float4(0.f, 0.f, 0.f, 0.f);
+    }
+    if (a.y) {
+        const YT* yr = reinterpret_cast<const YT*>(a.y) + (size_t)row * a.ldy;
+        float4 y[NT];
+        float ss = 0.f;
+#pragma unroll
+        for (int t = 0; t < NT; ++t) {
+            const int i = (threadIdx.x + 256 * t) * 4;
+            y[t] = i < nt ? load4<YT>(yr + i) : make_float4(0.f, 0.f, 0.f, 0.f);
+            ss += y[t].x * y[t].x + y[t].y * y[t].y + y[t].z * y[t].z + y[t].w * y[t].w;
+        }
+        ss = block_sum(ss, red);
+        const float inv = a.mult / sqrtf(ss / a.W + a.eps);
+#pragma unroll
+        for (int t = 0; t < NT; ++t) {
+            const int i = (threadIdx.x + 256 * t) * 4;
+            if (i < nt) {
+                const float4 g = *reinterpret_cast<const float4*>(a.g_post + i);
+                v[t].x = fmaf(y[t].x * inv, g.x, v[t].x); v[t].y = fmaf(y[t].y * inv, g.y, v[t].y);
+                v[t].z = fmaf(y[t].z * inv, g.z, v[t].z); v[t].w = fmaf(y[t].w * inv, g.w, v[t].w);
+                if (a.store_h) *reinterpret_cast<float4*>(hr + i) = v[t];
+            }
+        }
+    }
+    if (!a.out) return;
+    float ss = 0.f;
+#pragma unroll
+    for (int t = 0; t < NT; ++t) ss += v[t].x * v[t].x + v[t].y * v[t].y + v[t].z * v[t].z + v[t].w * v[t].w;
+    ss = block_sum(ss, red);
+    const float inv = 1.0f / sqrtf(ss / a.W + a.eps);
+    T* o = reinterpret_cast<T*>(a.out) + (size_t)blockIdx.x * a.ld;
+#pragma unroll
+    for (int t = 0; t < NT; ++t) {
+        const int i = (threadIdx.x + 256 * t) * 4;
+        if (i < nt) {
+            const float4 g = *reinterpret_cast<const float4*>(a.gamma + i);
+            store4<T>(o + i, make_float4(v[t].x * inv * g.x, v[t].y * inv * g.y, v[t].z * inv * g.z, v[t].w * inv * g.w));
+        }
+    }
+}
+
+template <class T, class YT>
+static pgk_status rows_norm_t(const RowsNormArgs& a, int n, hipStream_t st) {
+    PGK_REQUIRE(a.ld % 4 == 0 && a.W <= a.ld, "rows_norm: row stride %d / width %d", a.ld, a.W);
+    if (a.ld <= 1024) rows_norm_kernel<T, YT, 1><<<n, 256, 0, st>>>(a);
+    else if (a.ld <= 2048) rows_norm_kernel<T, YT, 2><<<n, 256, 0, st>>>(a);
+    else if (a.ld <= 4096) rows_norm_kernel<T, YT, 4><<<n, 256, 0, st>>>(a);
+    else if (a.ld <= 16384) rows_norm_kernel<T, YT, 16><<<n, 256, 0, st>>>(a);
+    else return set_error(PGK_ERR_UNSUPPORTED, "rows_norm: width %d beyond 16384", a.W);
+    PGK_LAUNCH_CHECK();
+    return PGK_OK;
+}
+
+pgk_status rows_norm(const RowsNormArgs& a, int n, pgk_dtype dt, hipStream_t st) {
+    if (dt == PGK_BF16) return rows_norm_t<bf16, bf16>(a, n, st);
+    if (dt == PGK_F32) return rows_norm_t<float, float>(a, n, st);
+    return set_error(PGK_ERR_UNSUPPORTED, "rows_norm: dtype %d", (int)dt);
+}
+
+// ---- any width (not a multiple of 4, any row stride): the operator form of the same two steps ----
+template <class T>
+__global__ __launch_bounds__(256) void rmsnorm_f32_kernel(const float* x, const float* w, T* out, int cols, float eps) {
+    __shared__ float red[16];
+    const float* xr = x + (size_t)blockIdx.x * cols;
+    float ss = 0.f;
+    for (int i = threadIdx.x; i < cols; i += 256) ss = fmaf(xr[i], xr[i], ss);
+    ss = block_sum(ss, red);
+    const float inv = 1.0f / sqrtf(ss / cols + eps);
+    for (int i = threadIdx.x; i < cols; i += 256) out[(size_t)blockIdx.x * cols + i] = from_f<T>(xr[i] * inv * w[i]);
+}
+template <class T>
+__global__ __launch_bounds__(256) void rmsnorm_add_kernel(float* x, const T* y, const float* w, int cols, float eps, float mult) {
+    __shared__ float red[16];
+    const T* yr = y + (size_t)blockIdx.x * cols;
+    float* xr = x + (size_t)blockIdx.x * cols;
+    float ss = 0.f;
+    for (int i = threadIdx.x; i < cols; i += 256) { const float v = to_f(yr[i]); ss = fmaf(v, v, ss); }
+    ss = block_sum(ss, red);
+    const float inv = mult / sqrtf(ss / cols + eps);
+    for (int i = threadIdx.x; i < cols; i += 256) xr[i] = fmaf(to_f(yr[i]) * inv, w[i], xr[i]);
+}
+
+template <class T>
+__global__ __launch_bounds__(256) void head_gate_kernel(T* x, const T* gate, size_t total, int heads, int d, long long gs) {
+    for (size_t i = blockIdx.x * (size_t)256 + threadIdx.x; i < total; i += (size_t)gridDim.x * 256) {
+        const size_t rh = i / d;
+        const float g = to_f(gate[(long long)(rh / heads) * gs + (long long)(rh % heads)]);
+        x[i] = from_f<T>(to_f(x[i]) / (1.0f + expf(-g)));
+    }
+}
+
+template <class E>
+__global__ __launch_bounds__(256) void pad_2d_kernel(const E* src, E* dst, int rows, int cols, int dcols, size_t total) {
+    for (size_t i = blockIdx.x * (size_t)256 + threadIdx.x; i < total; i += (size_t)gridDim.x * 256) {
+        const size_t r = i / dcols, c = i % dcols;
+        dst[i] = r < (size_t)rows && c < (size_t)cols ? src[r * cols + c] : E(0);
+    }
+}
+
+// Sliding-window attention for any widths and for fp32: one workgroup per (query row, head), each wave takes every fourth block of
+// 64 keys (a lane per key for the scores, a lane per value column for the sum), the four partial softmaxes meet in LDS.
+template <class T>
+__global__ __launch_bounds__(256) void window_attn_simple_kernel(const T* q, const T* k, const T* v, T* out, int rep, int q_len, int kv_len, int dk, int dv,
+                                                                 float scale, int window, WindowStrides sd, const T* gate, long long gs) {
+    extern __shared__ float wsm[];
+    const int row = blockIdx.x, head = blockIdx.y, kvh = head / rep, lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
+    float* qs = wsm;                          // [dk]
+    float* acc = wsm + dk + wid * dv;         // [4][dv]
+    float* ps = wsm + dk + 4 * dv + wid * 64; // [4][64]
+    float* ml = wsm + dk + 4 * dv + 4 * 64;   // [4][2]
+    const T* qr = q + head * sd.qh + row * sd.qs;
+    for (int i = threadIdx.x; i < dk; i += 256) qs[i] = to_f(qr[i]);
+    for (int i = lane; i < dv; i += 64) acc[i] = 0.f;
+    __syncthreads();
+    const int qpos = kv_len - q_len + row, lo = max(0, qpos - window + 1);
+    const T* kh = k + kvh * sd.kh;
+    const T* vh = v + kvh * sd.vh;
+    float m = -INFINITY, l = 0.f;
+    for (int k0 = lo + 64 * wid; k0 <= qpos; k0 += 256) {          // wave-uniform
+        const int key = k0 + lane, kn = min(64, qpos + 1 - k0);
+        float s = 0.f;
+        const T* kr = kh + (long long)min(key, qpos) * sd.ks;
+        for (int d = 0; d < dk; ++d) s = fmaf(qs[d], to_f(kr[d]), s);
+        s = lane < kn ? s * scale : -INFINITY;
+        const float mn = fmaxf(m, wave_max(s)), alpha = expf(m - mn), p = expf(s - mn);      // mn is finite: kn >= 1
+        m = mn;
+        l = l * alpha + wave_sum(p);
+        ps[lane] = p;
+        __builtin_amdgcn_wave_barrier();
+        for (int c = lane; c < dv; c += 64) {
+            float t = acc[c] * alpha;
+            const T* vc = vh + (long long)k0 * sd.vs + c;
+            for (int j = 0; j < kn; ++j) t = fmaf(ps[j], to_f(vc[(long long)j * sd.vs]), t);
+            acc[c] = t;
+        }
+        __builtin_amdgcn_wave_barrier();
+    }
+    if (lane == 0) { ml[2 * wid] = m; ml[2 * wid + 1] = l; }
+    __syncthreads();
+    float mm = -INFINITY, den = 0.f, w[4];
+    for (int i = 0; i < 4; ++i) mm = fmaxf(mm, ml[2 * i]);
+    for (int i = 0; i < 4; ++i) { w[i] = ml[2 * i + 1] > 0.f ? expf(ml[2 * i] - mm) : 0.f; den += w[i] * ml[2 * i + 1]; }
+    float f = 1.f / den;
+    if (gate) f /= 1.0f + expf(-to_f(gate[(long long)row * gs + head]));
+    const float* a0 = wsm + dk;
+    T* o = out + head * sd.oh + row * sd.os;
+    for (int c = threadIdx.x; c < dv; c += 256) o[c] = from_f<T>((w[0] * a0[c] + w[1] * a0[dv + c] + w[2] * a0[2 * dv + c] + w[3] * a0[3 * dv + c]) * f);
+}
+
+pgk_status window_attention(const void* q, const void* k, const void* v, void* out, int hq, int hkv, int q_len, int kv_len, int dk, int dv, float scale,
+                            int window, const WindowStrides& sd, const void* gate, long long gs, pgk_dtype dt, hipStream_t st) {
+    const bool flash = dt == PGK_BF16 && dk == dv && (dk == 64 || dk == 128) && scale > 0.f && sd.kh == sd.vh && sd.ks == sd.vs && aligned16(q) && aligned16(k) && aligned16(v) &&
+                       sd.qs % 8 == 0 && sd.qh % 8 == 0 && sd.ks % 8 == 0 && sd.kh % 8 == 0 && (reinterpret_cast<uintptr_t>(out) & 7u) == 0 && sd.os % 4 == 0 && sd.oh % 4 == 0;
+    if (flash) return flash_window(q, k, v, out, hq, hkv, q_len, kv_len, dk, scale, window, gate, gs, sd.qh, sd.qs, sd.kh, sd.ks, sd.oh, sd.os, st);
+    const size_t lds = ((size_t)dk + 4 * (size_t)dv + 4 * 64 + 8) * 4;
+    PGK_REQUIRE(lds <= 64 * 1024, "window_attention: head widths %d / %d do not fit LDS", dk, dv);
+    dim3 grid(q_len, hq);
+    PGK_DISPATCH_FLOAT(dt, "window_attention", (window_attn_simple_kernel<T><<<grid, 256, lds, st>>>((const T*)q, (const T*)k, (const T*)v, (T*)out, hq / hkv, q_len, kv_len, dk, dv,
+                                                                                                     scale, window, sd, (const T*)gate, gs)));
+    PGK_LAUNCH_CHECK();
+    return PGK_OK;
+}
+
+}  // namespace pgk
+
+using namespace pgk;
+
+extern "C" {
+
+pgk_status pgk_rmsnorm_f32(const float* x, const float* weight, void* out, int rows, int cols, float eps, pgk_dtype out_dt, pgk_stream s) {
+    PGK_REQUIRE(x && weight && out && rows >= 0 && cols > 0, "pgk_rmsnorm_f32: bad arguments [%d, %d]", rows, cols);
+    if (!rows) return PGK_OK;
+    PGK_DISPATCH_FLOAT(out_dt, "pgk_rmsnorm_f32", (rmsnorm_f32_kernel<T><<<rows, 256, 0, resolve_stream(s)>>>(x, weight, (T*)out, cols, eps)));
+    PGK_LAUNCH_CHECK();
+    return PGK_OK;
+}
+
+pgk_status pgk_rmsnorm_add_f32(float* x, const void* y, const float* weight, int rows, int cols, float eps, float mult, pgk_dtype y_dt, pgk_stream s) {
+    PGK_REQUIRE(x && y && weight && rows >= 0 && cols > 0, "pgk_rmsnorm_add_f32: bad arguments [%d, %d]", rows, cols);
+    if (!rows) return PGK_OK;
+    PGK_DISPATCH_FLOAT(y_dt, "pgk_rmsnorm_add_f32", (rmsnorm_add_kernel<T><<<rows, 256, 0, resolve_stream(s)>>>(x, (const T*)y, weight, cols, eps, mult)));
+    PGK_LAUNCH_CHECK();
+    return PGK_OK;
+}
+
+pgk_status pgk_window_attention(const void* q, const void* k, const void* v, void* out, int hq, int hkv, int q_len, int kv_len, int dk, int dv, float scale,
+                                int window, const void* gate, int64_t gate_stride, pgk_dtype dt, pgk_stream s) {
+    PGK_REQUIRE(q && k && v && out, "pgk_window_attention: null pointer");
+    PGK_REQUIRE(hq > 0 && hkv > 0 && hq % hkv == 0, "pgk_window_attention: n_heads mismatch (Hq=%d, Hkv=%d)", hq, hkv);
+    PGK_REQUIRE(q_len > 0 && kv_len >= q_len && dk > 0 && dv > 0 && window >= 1, "pgk_window_attention: bad shape q_len=%d kv_len=%d dk=%d dv=%d window=%d", q_len, kv_len, dk, dv, window);
+    const WindowStrides sd{dk, (long long)hq * dk, dk, (long long)hkv * dk, dv, (long long)hkv * dv, dv, (long long)hq * dv};
+    return window_attention(q, k, v, out, hq, hkv, q_len, kv_len, dk, dv, scale, window, sd, gate, gate_stride, dt, resolve_stream(s));
+}
+
+pgk_status pgk_head_gate(void* x, const void* gate, int rows, int heads, int d, int64_t gate_stride, pgk_dtype dt, pgk_stream s) {
+    PGK_REQUIRE(x && gate && rows >= 0 && heads > 0 && d > 0, "pgk_head_gate: bad arguments");
+    const size_t total = (size_t)rows * heads * d;
+    if (!total) return PGK_OK;
+    const int grid = ceil_div((long long)total, 256) > 4096 ? 4096 : ceil_div((long long)total, 256);
+    PGK_DISPATCH_FLOAT(dt, "pgk_head_gate", (head_gate_kernel<T><<<grid, 256, 0, resolve_stream(s)>>>((T*)x, (const T*)gate, total, heads, d, gate_stride)));
+    PGK_LAUNCH_CHECK();
+    return PGK_OK;
+}
+
+pgk_status pgk_pad_2d(const void* src, void* dst, int rows, int cols, int dst_rows, int dst_cols, pgk_dtype dt, pgk_stream s) {
+    PGK_REQUIRE(src && dst && rows >= 1 && cols >= 1 && dst_rows >= rows && dst_cols >= cols, "pgk_pad_2d: [%d, %d] into [%d, %d]", rows, cols, dst_rows, dst_cols);
+    const size_t total = (size_t)dst_rows * dst_cols;
+    const int grid = ceil_div((long long)total, 256) > 8192 ? 8192 : ceil_div((long long)total, 256);
+    hipStream_t st = resolve_stream(s);
+    if (dtype_size(dt) == 2) pad_2d_kernel<uint16_t><<<grid, 256, 0, st>>>((const uint16_t*)src, (uint16_t*)dst, rows, cols, dst_cols, total);
+    else if (dtype_size(dt) == 4) pad_2d_kernel<uint32_t><<<grid, 256, 0, st>>>((const uint32_t*)src, (uint32_t*)dst, rows, cols, dst_cols, total);
+    else return set_error(PGK_ERR_UNSUPPORTED, "pgk_pad_2d: dtype %d", (int)dt);
+    PGK_LAUNCH_CHECK();
+    return PGK_OK;
+}
+
+}  // extern "C"

@@ -2,8 +2,8 @@
 
 TransformerConfig carries the dimensions; ModelSpec is the data-only description of one
 architecture family (HF tensor-name patterns + architecture flags + default hyper-parameters).
-Only dense families on the hot path are described: GPT-2, Llama, Qwen2, Qwen3 (MoE families are
-out of scope)."""
+Dense families are described: GPT-2, Llama, Qwen2, Qwen3 and the layer-list family Totolorn (MoE families are
+not).  A layer-list model's config.json spells out every layer: LayerConfig."""
 
 from __future__ import annotations
 
@@ -22,8 +22,8 @@ class ModelSpec:
     attn_norm: str
     attn_norm_bias: str | None
     q_proj: str
-    k_proj: str
-    v_proj: str
+    k_proj: str | None
+    v_proj: str | None
     o_proj: str
     q_bias: str | None
     k_bias: str | None
@@ -55,6 +55,17 @@ class ModelSpec:
     default_norm_eps: float = 1e-5
     default_rope_theta: float = 10000.0
     hf_model_type: str = ""
+    # layer-list families: config.json's "architecture", and what their layers add to the fields above
+    architecture: str = ""
+    post_attn_norm: str | None = None      # norm of the sublayer's output, before the residual add
+    post_mlp_norm: str | None = None
+    kv_down_proj: str | None = None        # latent attention: hidden -> latent, its norm, latent -> keys / values
+    kv_down_norm: str | None = None
+    k_up_proj: str | None = None
+    v_up_proj: str | None = None
+    head_gate: str | None = None           # one sigmoid gate per head
+    norm_weight_offset: float = 0.0        # norms multiply by offset + weight (1: weights stored around zero)
+    residual_f32: bool = False             # the residual stream stays fp32 whatever the element type
 
 
 def _hf_decoder_spec(name: str, *, qk_norm: bool, qkv_bias: bool, eps: float, theta: float) -> ModelSpec:
@@ -95,12 +106,30 @@ GPT2_SPEC = ModelSpec(
     norm_type="layernorm", activation="gelu", use_rope=False, use_qk_norm=False, use_position_embed=True,
     qkv_combined=True, weight_transpose=True, default_norm_eps=1e-5, default_rope_theta=10000.0, hf_model_type="gpt2")
 
-MODEL_SPECS: dict[str, ModelSpec] = {"gpt2": GPT2_SPEC, "llama": LLAMA_SPEC, "qwen3": QWEN3_SPEC, "qwen2": QWEN2_SPEC}
+_T = "l{layer}."
+TOTOLORN_SPEC = ModelSpec(
+    name="totolorn", embed_tokens="embed", position_embed="pos", lm_head="head", final_norm="final.norm", final_norm_bias=None,
+    attn_norm=_T + "norm1", attn_norm_bias=None, q_proj=_T + "mix.q", k_proj=None, v_proj=None, o_proj=_T + "mix.o",
+    q_bias=None, k_bias=None, v_bias=None, o_bias=None, q_norm=None, k_norm=None, mlp_norm=_T + "norm2", mlp_norm_bias=None,
+    fc1=None, fc1_bias=None, fc2=None, fc2_bias=None, gate_proj=_T + "mlp.gate", up_proj=_T + "mlp.up", down_proj=_T + "mlp.down",
+    norm_type="rmsnorm", activation="silu", use_rope=False, use_position_embed=True, architecture="Totolorn",
+    post_attn_norm=_T + "norm1b", post_mlp_norm=_T + "norm2b", kv_down_proj=_T + "mix.dkv", kv_down_norm=_T + "mix.dkv.norm",
+    k_up_proj=_T + "mix.uk", v_up_proj=_T + "mix.uv", head_gate=_T + "mix.g", norm_weight_offset=1.0, residual_f32=True)
+
+MODEL_SPECS: dict[str, ModelSpec] = {"gpt2": GPT2_SPEC, "llama": LLAMA_SPEC, "qwen3": QWEN3_SPEC, "qwen2": QWEN2_SPEC,
+                                     "totolorn": TOTOLORN_SPEC}
 
 
-def detect_model_spec(tensor_names: list[str]) -> ModelSpec:
-    """Pick the family from checkpoint tensor names (config.py:380-431): QK-norm -> Qwen3, QKV biases ->
-    Qwen2, model.embed_tokens -> Llama, wte -> GPT-2.  MoE checkpoints are rejected (out of scope)."""
+def detect_model_spec(tensor_names: list[str], config: dict | None = None) -> ModelSpec:
+    """Pick the family: config.json's "architecture" if it names one of ours, else the checkpoint's tensor names
+    (config.py:380-431): QK-norm -> Qwen3, QKV biases -> Qwen2, model.embed_tokens -> Llama, wte -> GPT-2.  MoE checkpoints are
+    rejected."""
+    arch = (config or {}).get("architecture")
+    if arch:
+        for spec in MODEL_SPECS.values():
+            if spec.architecture == arch:
+                return spec
+        raise ValueError(f"unknown architecture {arch!r} (known: {[s.architecture for s in MODEL_SPECS.values() if s.architecture]})")
     names = set(tensor_names)
     if any("block_sparse_moe" in n or "mlp.experts" in n for n in names):
         raise ValueError("MoE checkpoints are not supported by pygpukit_amd")
@@ -111,6 +140,45 @@ def detect_model_spec(tensor_names: list[str]) -> ModelSpec:
     if "wte.weight" in names:
         return GPT2_SPEC
     raise ValueError(f"Cannot detect model type from tensor names. First 10 names: {list(tensor_names)[:10]}")
+
+
+@dataclass(frozen=True)
+class LayerConfig:
+    """One layer of a layer-list model."""
+
+    mixer: Literal["latent_attention"]
+    num_heads: int
+    head_dim: int                     # query / key width of a head
+    v_head_dim: int                   # value width of a head
+    kv_rank: int                      # latent size: what the cache holds per token
+    window: int | None                # keys a query sees, itself included (None: all before it)
+    scale: float                      # multiplies q . k
+    intermediate_size: int | None     # SwiGLU width; None: the layer has no feed-forward
+
+
+def parse_layer(i: int, entry: dict) -> LayerConfig:
+    kind = entry.get("type")
+    if kind != "latent_attention":
+        raise ValueError(f"layer {i}: unknown mixer {kind!r}")
+    m, mlp = entry["mixer"], entry.get("mlp")
+    if mlp is not None and mlp.get("kind") != "dense":
+        raise ValueError(f"layer {i}: unknown feed-forward {mlp.get('kind')!r}")
+    mask = m.get("mask")
+    return LayerConfig("latent_attention", int(m["heads"]), int(m["dim"]), int(m["vdim"]), int(m["kv_rank"]),
+                       int(mask["size"]) if mask else None, float(m["scale"]), int(mlp["ff"]) if mlp is not None else None)
+
+
+def layer_list_config(config: dict) -> "TransformerConfig":
+    """config.json of a layer-list model -> TransformerConfig.  The per-model head fields take the first layer's values."""
+    layers = tuple(parse_layer(i, e) for i, e in enumerate(config["layers"]))
+    if not layers:
+        raise ValueError("config.json lists no layers")
+    first = layers[0]
+    return TransformerConfig(vocab_size=int(config["vocab"]), hidden_size=int(config["width"]), num_layers=len(layers), num_heads=first.num_heads,
+                             num_kv_heads=first.num_heads, intermediate_size=max([l.intermediate_size or 0 for l in layers]),
+                             _head_dim=first.head_dim, norm_type="rmsnorm", activation="silu", use_rope=False,
+                             max_position_embeddings=int(config["max_positions"]), norm_eps=float(config["norm"]["eps"]), tie_word_embeddings=False,
+                             layers=layers, residual_mult=float(config["residual_mult"]))
 
 
 @dataclass
@@ -136,6 +204,8 @@ class TransformerConfig:
     norm_eps: float = 1e-5
     rope_theta: float = 10000.0
     tie_word_embeddings: bool = True
+    layers: tuple[LayerConfig, ...] | None = None    # layer-list models: every layer's own sizes
+    residual_mult: float = 1.0                       # factor of every sublayer's contribution to the residual stream
 
     def __post_init__(self):
         if self.num_kv_heads is None:

@@ -12,6 +12,11 @@ class DecodeM1(DecodeStrategy):
     def step(self, token_id: int, position: int, context_len: int, buffers):
         """-> logits [1, vocab] (buffers.logits)."""
         model = self.model
+        assert buffers.logits is not None, "logits buffer not allocated"
+        if model.config.layers is not None:      # fp32 residual stream, per-layer sizes: the block runs its own sequence of ops
+            hidden = model._decode_step_fixed_cache(token_id, position, context_len)
+            matmul_nt(hidden, model._lm_head if model._lm_head is not None else model.embed_tokens, out=buffers.logits)
+            return buffers.logits
         embedding_lookup(model.embed_tokens, buffers.hidden, token_id)
         for block in model.blocks:
             rmsnorm(buffers.hidden, block.attn_norm.weight, block.attn_norm.eps, out=buffers.norm_out)
@@ -22,7 +27,6 @@ class DecodeM1(DecodeStrategy):
             model._mlp_forward_zero_alloc(block.mlp, buffers.norm_out, buffers)
             add_inplace(buffers.hidden, buffers.residual)
         rmsnorm(buffers.hidden, model.final_norm.weight, model.final_norm.eps, out=buffers.norm_out)
-        assert buffers.logits is not None, "logits buffer not allocated"
         head = model._lm_head if model._lm_head is not None else model.embed_tokens
         matmul_nt(buffers.norm_out, head, out=buffers.logits)
         return buffers.logits

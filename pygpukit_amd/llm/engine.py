@@ -14,6 +14,8 @@ import numpy as np
 from pygpukit_amd import _hip
 from pygpukit_amd.core.array import GPUArray
 from pygpukit_amd.core.dtypes import bfloat16, float32
+from pygpukit_amd.core.factory import zeros
+from pygpukit_amd.ops.tensor import concat_axis0, pad_2d
 
 
 class Engine:
@@ -75,6 +77,30 @@ class Engine:
                   out.ctypes.data_as(C.POINTER(C.c_float)) if out is not None else None, None)
         if out is not None:
             self.last_prefill_logits = out
+        return out
+
+    def prefill_batch(self, prompts, slots=None, starts=None, *, want=None) -> np.ndarray:
+        """Several sequences in one call: prompts[i] goes to slot slots[i] (default i) from position starts[i] (default 0).  Returns the
+        fp32 logits [n, V] of every sequence's last row, or with `want` (one ascending list of row indices per sequence; layer-list
+        engines only) of exactly those rows, sequence by sequence."""
+        lens = np.asarray([len(p) for p in prompts], np.int32)
+        if lens.size == 0 or (lens < 1).any():
+            raise ValueError("prefill_batch: every prompt needs at least one token")
+        slots = np.asarray(range(len(prompts)) if slots is None else slots, np.int32)
+        starts = np.zeros(len(prompts), np.int32) if starts is None else np.asarray(starts, np.int32)
+        if len(slots) != len(prompts) or len(starts) != len(prompts) or (want is not None and len(want) != len(prompts)):
+            raise ValueError("prefill_batch: prompts, slots, starts and want must have the same length")
+        first = np.concatenate([[0], np.cumsum(lens)[:-1]])
+        rows = [[n - 1] for n in lens] if want is None else want
+        for n, r in zip(lens, rows):
+            if any(not 0 <= i < n for i in r):
+                raise ValueError("prefill_batch: wanted row outside its prompt")
+        w = np.asarray([f + i for f, r in zip(first, rows) for i in r], np.int32)
+        toks = np.ascontiguousarray(np.concatenate([np.asarray(p, np.int32) for p in prompts]))
+        out = np.empty((len(w), self.config["vocab_size"]), np.float32)
+        i32 = lambda a: a.ctypes.data_as(_hip.c_i32_p)  # noqa: E731
+        _hip.call("pgk_engine_prefill_batch", self.handle, len(prompts), i32(slots), i32(lens), i32(starts), i32(toks), len(w),
+                  i32(w) if len(w) else None, out.ctypes.data_as(C.POINTER(C.c_float)) if len(w) else None, None)
         return out
 
     # ------------------------------------------------------------------ decode
@@ -252,3 +278,130 @@ class Engine:
         self.set_sampling(0.0)
         self._captured_batch = None
         return out + toks
+
+
+def _up64(n: int) -> int:
+    return (n + 63) // 64 * 64
+
+
+class StackEngine(Engine):
+    """The native engine for layer-list models (csrc/engine_stack.hip): fp32 residual stream, norm before and after each sublayer,
+    sliding-window latent attention, every layer with its own sizes.  State, graphs, sampling and generation are Engine's.
+
+    The cache of a layer is a ring of min(window, max_seq_len) latent rows per sequence slot: a sequence goes on where it stopped
+    (or starts again at position 0); a position whose window has been overwritten is refused."""
+
+    def __init__(self, config: dict, embed: GPUArray, position_embed: GPUArray | None, head: GPUArray, final_norm: GPUArray, layers: list[dict], *,
+                 max_seq_len: int = 512, max_batch: int = 1):
+        """config: vocab_size, width, max_positions, norm_eps, residual_mult.  layers[i]: the sizes heads, dim, vdim, rank, window, scale,
+        head_pad, rank_pad, ff_pad and the packed arrays of pack_layer()."""
+        _hip.require_device()
+        dt = embed.dtype
+        if dt not in (bfloat16, float32):
+            raise NotImplementedError("the layer-list engine runs in bfloat16 or float32")
+        self.config = dict(config, num_layers=len(layers))
+        self.layers = layers
+        self.max_seq_len, self.max_batch, self.dtype = max_seq_len, max_batch, dt
+        self.weight_format = str(dt)
+        self._keep = [embed, position_embed, head, final_norm, layers]
+        wp = _up64(config["width"])
+        if head.shape != (config["vocab_size"], wp) or final_norm.shape != (1, wp) or final_norm.dtype != float32 or embed.shape != (config["vocab_size"], config["width"]):
+            raise ValueError("StackEngine: embedding / head / final norm shapes do not match the configuration")
+        if position_embed is not None and position_embed.shape != (config["max_positions"], config["width"]):
+            raise ValueError(f"StackEngine: position table {position_embed.shape}")
+        arr = (_hip.StackLayer * len(layers))()
+        for i, lw in enumerate(layers):
+            hd = lw["heads"] * lw["head_pad"]
+            ff, rp = lw["ff_pad"], lw["rank_pad"]
+            n_in = lw["w_in"].shape[0]
+            for name, shape, dtype in (("norm1", (1, wp), float32), ("norm1b", (1, wp), float32), ("norm2", (1, wp), float32), ("norm2b", (1, wp), float32),
+                                       ("c_norm", (1, rp), float32), ("w_in", (n_in, wp), dt), ("w_ukv", (2 * hd, rp), dt), ("w_o", (wp, hd), dt),
+                                       ("w_gate_up", (2 * ff, wp), dt), ("w_down", (wp, ff), dt)):
+                t = lw.get(name)
+                if t is None and not ff and name in ("norm2", "norm2b", "w_gate_up", "w_down"):
+                    continue
+                if t is None or t.shape != shape or t.dtype != dtype:
+                    raise ValueError(f"StackEngine: layer {i}: {name} must be {dtype} {shape}, got {None if t is None else (t.dtype, t.shape)}")
+                setattr(arr[i], name, t.data_ptr())
+            for name in ("heads", "dim", "vdim", "rank", "window", "head_pad", "rank_pad", "ff_pad"):
+                setattr(arr[i], name, lw[name])
+            arr[i].n_in, arr[i].scale = n_in, lw["scale"]
+        sc = _hip.StackConfig(config["vocab_size"], config["width"], len(layers), config["max_positions"], max_seq_len, max_batch, config["norm_eps"],
+                              config["residual_mult"], dt.code)
+        h = C.c_void_p()
+        _hip.call("pgk_engine_create_stack", C.byref(sc), embed._p, position_embed._p if position_embed is not None else None, head._p, final_norm._p,
+                  arr, C.byref(h))
+        self._h = h.value
+        self._captured_batch = 0
+        self.last_prefill_logits = None
+
+    @staticmethod
+    def pack_layer(q: GPUArray, kv_down: GPUArray, head_gate: GPUArray, kv_norm: GPUArray, k_up: GPUArray, v_up: GPUArray, o: GPUArray, norm1: GPUArray,
+                   norm1b: GPUArray, *, heads: int, dim: int, vdim: int, window: int, scale: float, gate_up: GPUArray | None = None,
+                   down: GPUArray | None = None, norm2: GPUArray | None = None, norm2b: GPUArray | None = None) -> dict:
+        """One layer's matrices ([out, in]; norms fp32 with offsets applied) -> the engine's padded layout: head widths to 64 / 128 / a
+        multiple of 64, every other width to a multiple of 64.  Arrays that already fit are used as they are."""
+        width, rank = q.shape[1], kv_down.shape[0]
+        wp, rp = _up64(width), _up64(rank)
+        m = max(dim, vdim)
+        hp = 64 if m <= 64 else 128 if m <= 128 else _up64(m)
+        hd = heads * hp
+
+        def head_rows(w: GPUArray, per_head: int, cols: int) -> GPUArray:      # [heads * per_head, c] -> [heads * hp, cols]
+            c = w.shape[1]
+            return pad_2d(pad_2d(w.view((heads, per_head * c)), heads, hp * c).view((hd, c)), hd, cols)
+
+        w_in = zeros((_up64(hd + rp + heads), wp), q.dtype)
+        for rows, w in ((0, head_rows(q, dim, wp)), (hd, pad_2d(kv_down, rank, wp)), (hd + rp, pad_2d(head_gate, heads, wp))):
+            _hip.call("pgk_memcpy_d2d", C.c_void_p(w_in.data_ptr() + rows * wp * w.itemsize), w._p, w.nbytes, None)
+        row = lambda w, n: pad_2d(w.view((1, w.size)), 1, n)  # noqa: E731
+        out = dict(heads=heads, dim=dim, vdim=vdim, rank=rank, window=window, scale=scale, head_pad=hp, rank_pad=rp, ff_pad=0, w_in=w_in,
+                   c_norm=row(kv_norm, rp), w_ukv=concat_axis0(head_rows(k_up, dim, rp), head_rows(v_up, vdim, rp)),
+                   w_o=pad_2d(pad_2d(o.view((width * heads, vdim)), width * heads, hp).view((width, hd)), wp, hd),
+                   norm1=row(norm1, wp), norm1b=row(norm1b, wp))
+        if gate_up is not None:
+            ff = down.shape[1]
+            fp = _up64(ff)
+            if (ff, width) != (fp, wp):
+                gate_up = concat_axis0(pad_2d(gate_up._view(0, (ff, width)), fp, wp), pad_2d(gate_up._view(ff * width, (ff, width)), fp, wp))
+            out.update(ff_pad=fp, w_gate_up=gate_up, w_down=pad_2d(down, wp, fp), norm2=row(norm2, wp), norm2b=row(norm2b, wp))
+        return out
+
+    @classmethod
+    def from_model(cls, model, *, max_seq_len: int = 512, max_batch: int = 1) -> "StackEngine":
+        c = model.config
+        width = model.embed_tokens.shape[1]
+        packed = model.__dict__.get("_stack_layers")       # packed once, shared by every engine of this model
+        if packed is None:
+            packed = []
+            for b in model.blocks:
+                a = b.attn
+                if a.head_gate is None or b.post_attn_norm is None or (b.mlp is not None and (b.post_mlp_norm is None or b.mlp.gate_up_proj is None)):
+                    raise NotImplementedError("the layer-list engine needs gated latent attention, post-norms and a fused gate / up weight")
+                if b.residual_mult != c.residual_mult or b.attn_norm.eps != c.norm_eps:
+                    raise NotImplementedError("the layer-list engine takes one residual factor and one norm epsilon for all layers")
+                mlp = {} if b.mlp is None else dict(gate_up=b.mlp.gate_up_proj.weight, down=b.mlp.down_proj.weight, norm2=b.mlp_norm.weight,
+                                                    norm2b=b.post_mlp_norm.weight)
+                packed.append(cls.pack_layer(a.q_proj.weight, a.kv_down.weight, a.head_gate.weight, a.kv_norm.weight, a.k_up.weight, a.v_up.weight,
+                                             a.o_proj.weight, b.attn_norm.weight, b.post_attn_norm.weight, heads=a.num_heads, dim=a.head_dim,
+                                             vdim=a.v_head_dim, window=a.window, scale=a.scale, **mlp))
+            head = model._lm_head if model._lm_head is not None else model.embed_tokens
+            wp = _up64(width)
+            model._stack_layers = packed
+            model._stack_head = (pad_2d(head, head.shape[0], wp), pad_2d(model.final_norm.weight.view((1, width)), 1, wp))
+        head, fnorm = model._stack_head
+        cfg = dict(vocab_size=model.embed_tokens.shape[0], width=width, hidden_size=width, max_positions=c.max_position_embeddings, norm_eps=c.norm_eps,
+                   residual_mult=c.residual_mult)
+        return cls(cfg, model.embed_tokens, model.position_embed, head, fnorm, packed, max_seq_len=max_seq_len, max_batch=max_batch)
+
+    def latent_cache(self, layer: int) -> GPUArray:
+        """[max_batch, R, rank_pad] view of layer `layer`'s latent rings: position p of a sequence is row p % R, R = min(window, max_seq_len)."""
+        p, none = C.c_void_p(), C.c_void_p()
+        _hip.call("pgk_engine_kv_ptr", self.handle, layer, C.byref(p), C.byref(none))
+        lw = self.layers[layer]
+        a = GPUArray((self.max_batch, min(lw["window"], self.max_seq_len), lw["rank_pad"]), self.dtype, p.value, owns_memory=False)
+        a._source_ref = self
+        return a
+
+    def kv_cache(self, layer: int):
+        raise NotImplementedError("a layer-list engine caches latents, not keys and values: latent_cache()")

@@ -90,6 +90,14 @@ class Attention:
         self._max_cache_len = max_seq_len
         self._confirmed_pos = self._logical_pos = 0
 
+    def fill_fixed_cache(self, present: tuple) -> None:
+        """A prompt's present_kv -> rows 0.. of the fixed cache (examples/chat/chat_cli.py:531-534)."""
+        for new, cache in zip(present, (self._k_cache, self._v_cache)):
+            kv_cache_prefill_gqa(new, cache, self.num_heads, 0)
+
+    def cache_arrays(self) -> tuple[GPUArray, ...]:
+        return self._k_cache, self._v_cache
+
     def _rope_rows(self, start: int, count: int) -> tuple[GPUArray, GPUArray]:
         """fp32 [count, D] views of the device-resident tables for positions start..start+count-1."""
         if self._cos_gpu is None:

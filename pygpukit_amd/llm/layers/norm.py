@@ -5,15 +5,28 @@ from __future__ import annotations
 from typing import Literal
 
 from pygpukit_amd.core.array import GPUArray
-from pygpukit_amd.ops.basic import layernorm, rmsnorm
+from pygpukit_amd.core.dtypes import DataType, float32
+from pygpukit_amd.ops.basic import layernorm, rmsnorm, rmsnorm_add_f32, rmsnorm_f32
 
 
 class Norm:
+    """`stream_dtype` set: the norm of an fp32 residual stream - `weight` is fp32 with any offset already added, the result leaves in
+    stream_dtype, and add_to() is the norm-then-residual-add of a sublayer's output."""
+
     def __init__(self, weight: GPUArray, bias: GPUArray | None = None,
-                 norm_type: Literal["rmsnorm", "layernorm"] = "rmsnorm", eps: float = 1e-5):
+                 norm_type: Literal["rmsnorm", "layernorm"] = "rmsnorm", eps: float = 1e-5, stream_dtype: DataType | None = None):
         self.weight, self.bias, self.norm_type, self.eps = weight, bias, norm_type, eps
+        self.stream_dtype = stream_dtype
+        if stream_dtype is not None and (norm_type != "rmsnorm" or weight.dtype != float32):
+            raise ValueError("an fp32-stream norm is an RMSNorm with a float32 weight")
+
+    def add_to(self, stream: GPUArray, y: GPUArray, mult: float = 1.0) -> GPUArray:
+        """stream += mult * norm(y), in place."""
+        return rmsnorm_add_f32(stream, y, self.weight, self.eps, mult)
 
     def __call__(self, x: GPUArray, *, out: GPUArray | None = None) -> GPUArray:
+        if self.stream_dtype is not None:
+            return rmsnorm_f32(x, self.weight, self.eps, dtype=self.stream_dtype, out=out)
         if self.norm_type == "rmsnorm":
             return rmsnorm(x, self.weight, self.eps, out=out)
         if self.bias is None:

@@ -15,8 +15,9 @@ import numpy as np
 from pygpukit_amd.core.array import GPUArray
 from pygpukit_amd.core.dtypes import bfloat16, float16, float32, uint8
 from pygpukit_amd.core.factory import from_numpy
-from pygpukit_amd.llm.config import GPT2_SPEC, LLAMA_SPEC, QWEN3_SPEC, ModelSpec, TransformerConfig, detect_model_spec
-from pygpukit_amd.llm.layers import MLP, Attention, Norm, TransformerBlock
+from pygpukit_amd.llm.config import (GPT2_SPEC, LLAMA_SPEC, QWEN3_SPEC, TOTOLORN_SPEC, ModelSpec, TransformerConfig, detect_model_spec,
+                                     layer_list_config)
+from pygpukit_amd.llm.layers import MLP, Attention, LatentAttention, Norm, TransformerBlock
 from pygpukit_amd.llm.layers.linear import LinearBF16, LinearFP8
 from pygpukit_amd.llm.models.causal import CausalTransformerModel
 from pygpukit_amd.llm.safetensors import Dtype, load_safetensors
@@ -54,7 +55,10 @@ def load_model_from_safetensors(model_path: str, dtype: str = "bfloat16", spec: 
                                 repack_weights: bool = True) -> CausalTransformerModel:
     """loader.py:132-612.  dtype: "float32" | "float16" | "bfloat16" (the reference defaults to float32; bf16 is the
     native format of the checkpoints this path serves).  `repack_weights` is accepted for signature compatibility: arrays
-    come from the device pool already."""
+    come from the device pool already.  `model_path` may be the checkpoint's folder (model.safetensors or its index)."""
+    if os.path.isdir(model_path):
+        one = os.path.join(model_path, "model.safetensors")
+        model_path = one if os.path.exists(one) else os.path.join(model_path, "model.safetensors.index.json")
     st = load_safetensors(model_path)
     names = set(st.tensor_names)
     target = {"float32": (float32, Dtype.Float32, np.float32), "float16": (float16, Dtype.Float16, np.float16),
@@ -62,9 +66,9 @@ def load_model_from_safetensors(model_path: str, dtype: str = "bfloat16", spec: 
     if target is None:
         raise ValueError(f"load_model_from_safetensors: unsupported dtype {dtype}")
     target_dt, target_id, target_np = target
-    if spec is None:
-        spec = detect_model_spec(st.tensor_names)
     hf_config = _read_config(model_path)
+    if spec is None:
+        spec = detect_model_spec(st.tensor_names, hf_config)
     fp8 = FP8QuantConfig.from_config(hf_config)
 
     def load_tensor(name: str, do_transpose: bool = False) -> GPUArray:
@@ -112,6 +116,9 @@ def load_model_from_safetensors(model_path: str, dtype: str = "bfloat16", spec: 
 
     def nm(pattern: str | None, layer: int) -> str | None:
         return None if pattern is None else pattern.format(layer=layer)
+
+    if spec.kv_down_proj is not None:
+        return _load_layer_list(st, spec, hf_config, target_dt, load_tensor, try_load)
 
     embed_info = st.tensor_info(spec.embed_tokens)
     vocab_size, hidden_size = embed_info.shape
@@ -193,6 +200,47 @@ def load_model_from_safetensors(model_path: str, dtype: str = "bfloat16", spec: 
     return CausalTransformerModel(cfg, load_tensor(spec.embed_tokens), blocks, final_norm, lm_head, position_embed, spec)
 
 
+def _load_layer_list(st, spec: ModelSpec, config: dict, dtype, load_tensor, try_load) -> CausalTransformerModel:
+    """A layer-list checkpoint: config.json gives every layer's kind and sizes, the tensors are checked against it."""
+    if not config:
+        raise ValueError(f"a {spec.name} checkpoint needs its config.json beside it")
+    cfg = layer_list_config(config)
+
+    def tensor(name: str, shape: tuple[int, ...]) -> GPUArray:
+        if name not in st:
+            raise ValueError(f"checkpoint has no tensor {name!r}")
+        got = tuple(st.tensor_info(name).shape)
+        if got != shape:
+            raise ValueError(f"{name}: shape {got}, config.json says {shape}")
+        return load_tensor(name)
+
+    def norm(name: str, width: int, offset: float) -> Norm:
+        if name not in st or tuple(st.tensor_info(name).shape) != (width,):
+            raise ValueError(f"{name}: missing or not of width {width}")
+        w = st.tensor_as_f32(name) + np.float32(offset)
+        return Norm(from_numpy(np.ascontiguousarray(w, dtype=np.float32)), None, "rmsnorm", cfg.norm_eps, stream_dtype=dtype)
+
+    H, off = cfg.hidden_size, spec.norm_weight_offset
+    blocks = []
+    for i, lc in enumerate(cfg.layers):
+        nm = lambda pattern: pattern.format(layer=i)  # noqa: E731, B023
+        attn = LatentAttention(tensor(nm(spec.q_proj), (lc.num_heads * lc.head_dim, H)), tensor(nm(spec.kv_down_proj), (lc.kv_rank, H)),
+                               norm(nm(spec.kv_down_norm), lc.kv_rank, 0.0), tensor(nm(spec.k_up_proj), (lc.num_heads * lc.head_dim, lc.kv_rank)),
+                               tensor(nm(spec.v_up_proj), (lc.num_heads * lc.v_head_dim, lc.kv_rank)),
+                               tensor(nm(spec.o_proj), (H, lc.num_heads * lc.v_head_dim)), num_heads=lc.num_heads, head_dim=lc.head_dim,
+                               v_head_dim=lc.v_head_dim, scale=lc.scale, window=lc.window, head_gate=tensor(nm(spec.head_gate), (lc.num_heads, H)))
+        mlp = mlp_norm = post_mlp = None
+        if lc.intermediate_size is not None:
+            I = lc.intermediate_size
+            mlp = MLP(cfg, gate_proj=tensor(nm(spec.gate_proj), (I, H)), up_proj=tensor(nm(spec.up_proj), (I, H)), down_proj=tensor(nm(spec.down_proj), (H, I)))
+            mlp_norm, post_mlp = norm(nm(spec.mlp_norm), H, off), norm(nm(spec.post_mlp_norm), H, off)
+        blocks.append(TransformerBlock(norm(nm(spec.attn_norm), H, off), attn, mlp_norm, mlp, norm(nm(spec.post_attn_norm), H, off), post_mlp,
+                                       cfg.residual_mult))
+    lm_head = tensor(spec.lm_head, (cfg.vocab_size, H)) if spec.lm_head in st else None
+    return CausalTransformerModel(cfg, tensor(spec.embed_tokens, (cfg.vocab_size, H)), blocks, norm(spec.final_norm, H, off), lm_head,
+                                  tensor(spec.position_embed, (cfg.max_position_embeddings, H)), spec)
+
+
 def _bf16_array(bits: np.ndarray) -> GPUArray:
     out = GPUArray(tuple(bits.shape), bfloat16)
     out.copy_from_numpy(np.ascontiguousarray(bits, dtype=np.uint16))
@@ -218,5 +266,9 @@ def load_qwen3_from_safetensors(model_path: str, dtype: str = "bfloat16") -> Cau
     return load_model_from_safetensors(model_path, dtype=dtype, spec=QWEN3_SPEC)
 
 
-__all__ = ["load_model_from_safetensors", "load_gpt2_from_safetensors", "load_llama_from_safetensors", "load_qwen3_from_safetensors",
+def load_totolorn_from_safetensors(model_path: str, dtype: str = "bfloat16") -> CausalTransformerModel:
+    return load_model_from_safetensors(model_path, dtype=dtype, spec=TOTOLORN_SPEC)
+
+
+__all__ = ["load_totolorn_from_safetensors", "load_model_from_safetensors", "load_gpt2_from_safetensors", "load_llama_from_safetensors", "load_qwen3_from_safetensors",
            "FP8QuantConfig"]

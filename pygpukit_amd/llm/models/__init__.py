@@ -1,3 +1,3 @@
-from .causal import CausalTransformerModel, GPT2Model, LlamaModel, QwenModel
+from .causal import CausalTransformerModel, GPT2Model, LlamaModel, QwenModel, TotolornModel
 
-__all__ = ["CausalTransformerModel", "GPT2Model", "LlamaModel", "QwenModel"]
+__all__ = ["CausalTransformerModel", "GPT2Model", "LlamaModel", "QwenModel", "TotolornModel"]

@@ -19,7 +19,7 @@ from pygpukit_amd.llm.buffers import DecodeBuffers
 from pygpukit_amd.llm.config import ModelSpec, TransformerConfig
 from pygpukit_amd.llm.layers import MLP, Attention, Norm, TransformerBlock
 from pygpukit_amd.llm.sampling import sample_token
-from pygpukit_amd.ops.basic import (add, add_inplace, embedding_lookup, embedding_lookup_batch, glu_packed, matmul_nt,
+from pygpukit_amd.ops.basic import (add_inplace, cast_bf16_to_f32, embedding_lookup_batch, glu_packed, matmul_nt,
                                    rmsnorm, sample_token_gpu)
 
 
@@ -51,12 +51,19 @@ class CausalTransformerModel:
         ids = np.asarray(input_ids, dtype=np.int32)
         if ids.size and (ids.min() < 0 or ids.max() >= V):
             raise ValueError(f"token id outside [0, {V})")
-        hidden = GPUArray((len(ids), self.embed_tokens.shape[1]), self.embed_tokens.dtype)
-        embedding_lookup_batch(self.embed_tokens, hidden, from_numpy(ids), len(ids))
+        stream_f32 = self.spec is not None and self.spec.residual_f32
+
+        def rows(table: GPUArray, idx: np.ndarray) -> GPUArray:
+            out = GPUArray((len(ids), table.shape[1]), table.dtype)
+            embedding_lookup_batch(table, out, from_numpy(idx), len(ids))
+            return cast_bf16_to_f32(out) if stream_f32 and table.dtype == bfloat16 else out
+
+        hidden = rows(self.embed_tokens, ids)
         if self.position_embed is not None:
-            pos = GPUArray(hidden.shape, hidden.dtype)
-            embedding_lookup_batch(self.position_embed, pos, from_numpy(np.asarray(position_ids, dtype=np.int32)), len(ids))
-            add_inplace(hidden, pos)
+            pos = np.asarray(position_ids, dtype=np.int32)
+            if pos.size and (pos.min() < 0 or pos.max() >= self.position_embed.shape[0]):
+                raise ValueError(f"position outside [0, {self.position_embed.shape[0]})")
+            add_inplace(hidden, rows(self.position_embed, pos))
         return hidden
 
     def __call__(self, input_ids: list[int], position_ids: list[int] | None = None,
@@ -150,46 +157,39 @@ class CausalTransformerModel:
 
     def _decode_step_fixed_cache(self, token_id: int, position: int, context_len: int) -> GPUArray:
         """One token through every block against the fixed caches (causal.py:799-840) -> hidden [1, H]."""
-        hidden = GPUArray((1, self.embed_tokens.shape[1]), self.embed_tokens.dtype)
-        embedding_lookup(self.embed_tokens, hidden, token_id)
-        for block in self.blocks:
-            attn_out = block.attn.forward_fixed_cache(block.attn_norm(hidden), position, context_len)
-            hidden = add(hidden, attn_out)
-            hidden = add(hidden, block.mlp(block.mlp_norm(hidden)))
-        return self.final_norm(hidden)
+        return self._decode_step_fixed_cache_batch([token_id], position, context_len)
 
     def _decode_step_fixed_cache_batch(self, token_ids: list[int], start_position: int, context_len: int) -> GPUArray:
         """M consecutive tokens of one sequence (speculative verify, causal.py:842-891) -> hidden [M, H]."""
         hidden = self._embed(token_ids, list(range(start_position, start_position + len(token_ids))))
         for block in self.blocks:
-            attn_out = block.attn.forward_fixed_cache_batch(block.attn_norm(hidden), start_position, context_len)
-            hidden = add(hidden, attn_out)
-            hidden = add(hidden, block.mlp(block.mlp_norm(hidden)))
+            hidden = block.forward_fixed_cache(hidden, start_position, context_len)
         return self.final_norm(hidden)
 
     def prefill_fixed_cache(self, input_ids: list[int]) -> GPUArray:
         """Prefill that leaves K/V in the fixed caches (the chat flow's prefill + kv_cache_prefill_gqa,
         examples/chat/chat_cli.py:531-534) -> logits [S, V]."""
-        from pygpukit_amd.ops.basic import kv_cache_prefill_gqa
-
         hidden, present = self(list(input_ids), use_cache=True)
-        for block, (k, v) in zip(self.blocks, present):
-            kv_cache_prefill_gqa(k, block.attn._k_cache, block.attn.num_heads, 0)
-            kv_cache_prefill_gqa(v, block.attn._v_cache, block.attn.num_heads, 0)
+        for block, kv in zip(self.blocks, present):
+            block.attn.fill_fixed_cache(kv)
         return self.get_logits(hidden)
 
-    def snapshot_kv_cache(self) -> list[tuple[np.ndarray, np.ndarray]]:
-        return [(b.attn._k_cache.to_numpy(), b.attn._v_cache.to_numpy()) for b in self.blocks]
+    def snapshot_kv_cache(self) -> list[tuple[np.ndarray, ...]]:
+        return [tuple(a.to_numpy() for a in b.attn.cache_arrays()) for b in self.blocks]
 
-    def restore_kv_cache(self, snapshot: list[tuple[np.ndarray, np.ndarray]]) -> None:
-        for b, (k, v) in zip(self.blocks, snapshot):
-            b.attn._k_cache.copy_from_numpy(k)
-            b.attn._v_cache.copy_from_numpy(v)
+    def restore_kv_cache(self, snapshot: list[tuple[np.ndarray, ...]]) -> None:
+        for b, saved in zip(self.blocks, snapshot):
+            for a, host in zip(b.attn.cache_arrays(), saved):
+                a.copy_from_numpy(host)
 
     # ------------------------------------------------------------------ native engine
     def build_engine(self, max_seq_len: int = 512, max_batch: int = 1):
-        """Hand this model's weights (zero copy) to the native decode/prefill engine.  Requires bf16 or fp8
-        linears, RMSNorm, SwiGLU, RoPE and no biases (Llama / Qwen3 families)."""
+        """Hand this model's weights to the native decode/prefill engine: Llama / Qwen3 families (bf16 linears, RMSNorm, SwiGLU,
+        RoPE, no biases; zero copy) and layer-list models (bf16 or fp32; copies only where a width has to be padded)."""
+        if self.config.layers is not None:
+            from pygpukit_amd.llm.engine import StackEngine
+
+            return StackEngine.from_model(self, max_seq_len=max_seq_len, max_batch=max_batch)
         from pygpukit_amd.llm.engine import Engine
         from pygpukit_amd.llm.layers.linear import LinearFP8
 
@@ -222,5 +222,6 @@ class CausalTransformerModel:
 GPT2Model = CausalTransformerModel
 LlamaModel = CausalTransformerModel
 QwenModel = CausalTransformerModel
+TotolornModel = CausalTransformerModel
 
-__all__ = ["CausalTransformerModel", "GPT2Model", "LlamaModel", "QwenModel"]
+__all__ = ["CausalTransformerModel", "GPT2Model", "LlamaModel", "QwenModel", "TotolornModel"]

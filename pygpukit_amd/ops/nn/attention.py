@@ -79,3 +79,32 @@ def sdpa_causal_fixed_cache_ptr(Q: GPUArray, K: GPUArray, V: GPUArray, out: GPUA
     ws = _workspace(hq, d, max_seq)
     call("pgk_sdpa_fixed_cache", Q._p, K._p, V._p, out._p, hq, hc, q_len, max_seq, d, float(scale), 0, context_len_buf._p,
          ws._p, Q.dtype.code, None)
+
+
+def window_attention(q: GPUArray, k: GPUArray, v: GPUArray, scale: float, window: int, *, gate: GPUArray | None = None,
+                     out: GPUArray | None = None) -> GPUArray:
+    """q [q_len, Hq, dk], k [kv_len, Hkv, dk], v [kv_len, Hkv, dv] -> [q_len, Hq, dv]: query i is position kv_len - q_len + i and sees the
+    `window` positions that end with its own.  gate [q_len, Hq]: head outputs are multiplied by its sigmoid."""
+    validate_float(q, "window_attention")
+    if q.ndim != 3 or k.ndim != 3 or v.ndim != 3 or k.dtype != q.dtype or v.dtype != q.dtype:
+        raise ValueError("window_attention expects q, k, v as [seq, heads, width] of one dtype")
+    (q_len, hq, dk), (kv_len, hkv, dk2), (kv2, hkv2, dv) = q.shape, k.shape, v.shape
+    if dk != dk2 or kv_len != kv2 or hkv != hkv2 or hq % hkv or kv_len < q_len:
+        raise ValueError(f"window_attention: shapes {q.shape}, {k.shape}, {v.shape} do not match")
+    if window < 1:
+        raise ValueError(f"window_attention: window {window}")
+    if gate is not None and (gate.shape != (q_len, hq) or gate.dtype != q.dtype):
+        raise ValueError("window_attention: gate must be [q_len, Hq] in q's dtype")
+    o = check_out(out, (q_len, hq, dv), q.dtype, "window_attention")
+    call("pgk_window_attention", q._p, k._p, v._p, o._p, hq, hkv, q_len, kv_len, dk, dv, float(scale), min(int(window), 2**30),
+         gate._p if gate is not None else None, hq, q.dtype.code, None)
+    return o
+
+
+def head_gate(x: GPUArray, gate: GPUArray) -> GPUArray:
+    """x [rows, heads, d] *= sigmoid(gate [rows, heads]) in place."""
+    validate_float(x, "head_gate")
+    if x.ndim != 3 or gate.shape != x.shape[:2] or gate.dtype != x.dtype:
+        raise ValueError(f"head_gate: x {x.shape} and gate {gate.shape} do not match")
+    call("pgk_head_gate", x._p, gate._p, x.shape[0], x.shape[1], x.shape[2], x.shape[1], x.dtype.code, None)
+    return x

@@ -3,6 +3,7 @@
 from __future__ import annotations
 
 from pygpukit_amd.core.array import GPUArray
+from pygpukit_amd.core.dtypes import float32
 from pygpukit_amd.ops._common import call, check_out, validate_float, validate_same_dtype
 
 
@@ -22,6 +23,27 @@ def rmsnorm(input: GPUArray, gamma: GPUArray, eps: float = 1e-5, *, out: GPUArra
     o = check_out(out, input.shape, input.dtype, "rmsnorm")
     call("pgk_rmsnorm", input._p, gamma._p, o._p, input.shape[0], input.shape[1], eps, input.dtype.code, None)
     return o
+
+
+def rmsnorm_f32(input: GPUArray, weight: GPUArray, eps: float = 1e-5, *, dtype=float32, out: GPUArray | None = None) -> GPUArray:
+    """RMSNorm of an fp32 stream with an fp32 weight; the result leaves in `dtype`."""
+    _check(input, weight, "rmsnorm_f32")
+    if input.dtype != float32:
+        raise ValueError("rmsnorm_f32: input and weight must be float32")
+    o = check_out(out, input.shape, dtype, "rmsnorm_f32")
+    call("pgk_rmsnorm_f32", input._p, weight._p, o._p, input.shape[0], input.shape[1], eps, o.dtype.code, None)
+    return o
+
+
+def rmsnorm_add_f32(stream: GPUArray, y: GPUArray, weight: GPUArray, eps: float = 1e-5, mult: float = 1.0) -> GPUArray:
+    """stream += mult * rmsnorm(y) * weight in place (fp32 stream and weight, y in any float type)."""
+    validate_float(y, "rmsnorm_add_f32")
+    if stream.dtype != float32 or weight.dtype != float32:
+        raise ValueError("rmsnorm_add_f32: stream and weight must be float32")
+    if stream.ndim != 2 or stream.shape != y.shape or weight.shape != (stream.shape[1],):
+        raise ValueError(f"rmsnorm_add_f32: shapes {stream.shape}, {y.shape}, {weight.shape} do not match")
+    call("pgk_rmsnorm_add_f32", stream._p, y._p, weight._p, stream.shape[0], stream.shape[1], eps, mult, y.dtype.code, None)
+    return stream
 
 
 def layernorm(input: GPUArray, gamma: GPUArray, beta: GPUArray, eps: float = 1e-5, *, out: GPUArray | None = None) -> GPUArray:

@@ -17,6 +17,17 @@ def concat_axis0(a: GPUArray, b: GPUArray) -> GPUArray:
     return out
 
 
+def pad_2d(src: GPUArray, rows: int, cols: int) -> GPUArray:
+    """[r, c] -> [rows, cols] with zeros below and to the right; the array itself when nothing is added."""
+    if src.ndim != 2 or rows < src.shape[0] or cols < src.shape[1]:
+        raise ValueError(f"pad_2d: {src.shape} into [{rows}, {cols}]")
+    if src.shape == (rows, cols):
+        return src
+    out = GPUArray((rows, cols), src.dtype)
+    call("pgk_pad_2d", src._p, out._p, src.shape[0], src.shape[1], rows, cols, src.dtype.code, None)
+    return out
+
+
 def repeat_interleave_axis1(input: GPUArray, repeats: int) -> GPUArray:
     if input.ndim != 3:
         raise ValueError(f"repeat_interleave_axis1 expects 3D input, got {input.ndim}D")
