@@ -117,6 +117,102 @@ def cpu_baseline(cfg, weights, prompt, n_decode: int) -> dict:
             "prefill_s": t_prefill}
 
 
+DESIGN_SIZES = {
+    # width, heads, head width, latent, window, ff, layers, and the dense neighbour's kv heads
+    "w1024": dict(width=1024, heads=16, dim=128, rank=256, window=1024, ff=3072, layers=8, kv_heads=8),
+    "w2048": dict(width=2048, heads=16, dim=128, rank=512, window=2048, ff=6144, layers=8, kv_heads=8),
+    "w4096": dict(width=4096, heads=32, dim=128, rank=512, window=4096, ff=14336, layers=4, kv_heads=8),
+}
+
+
+def stack_kernel_bytes(z: dict, vocab: int, ctx: int, B: int) -> dict:
+    """Algorithmic bytes per decode step and layer of each kernel class of a layer-list engine (bf16 weights and latents, fp32 rows)."""
+    W, F, hd, r, n = z["width"], z["ff"], z["heads"] * z["dim"], z["rank"], min(ctx, z["window"])
+    return {"norm_qkv": (hd + r + z["heads"]) * W * 2 + B * 4 * (2 * W + hd + r), "attn": 2 * hd * r * 2 + B * (n * r * 2 + 8 * hd + 4 * r),
+            "oproj": hd * W * 2 + B * 4 * (hd + W), "gateup": 2 * F * W * 2 + B * 4 * (2 * W + F), "down": F * W * 2 + B * 4 * (F + W),
+            "lmhead": vocab * W * 2 + B * 4 * (W + vocab)}
+
+
+def design_leg(name: str, sizes: list[str], seed: int) -> dict:
+    """--design totolorn: prefill and decode of the layer-list engine at sizes that resemble a real model's layers (random weights), beside
+    the dense QKV + RoPE engine (its closest relative here) at equal width, heads, feed-forward, depth and vocabulary."""
+    from pygpukit_amd import _hip
+    from pygpukit_amd.core.factory import from_numpy
+    from pygpukit_amd.llm import synthetic as S
+    from pygpukit_amd.llm.engine import Engine, StackEngine
+
+    if name != "totolorn":
+        raise SystemExit(f"unknown design {name}")
+    V, out = 32000, {"design": name, "vocab": V, "dtype": "bf16", "data": "synthetic", "sizes": {}}
+
+    def sync():
+        _hip.call("pgk_device_sync")
+
+    def wall(fn, reps=5):
+        fn()
+        sync()
+        best = []
+        for _ in range(reps):
+            t0 = time.perf_counter()
+            fn()
+            sync()
+            best.append((time.perf_counter() - t0) * 1e3)
+        return float(np.median(best))
+
+    for size in sizes:
+        z = DESIGN_SIZES[size]
+        W, H, D, r, F, L = z["width"], z["heads"], z["dim"], z["rank"], z["ff"], z["layers"]
+        rng = np.random.default_rng(seed)
+
+        def draw(*shape):
+            w = rng.standard_normal(shape, dtype=np.float32)
+            w *= np.float32(0.02)
+            return from_numpy(S.f32_to_bf16_bits(w).reshape(shape))
+
+        embed, head, pos = draw(V, W), draw(V, W), draw(4400, W)
+        ones = from_numpy(np.ones((1, W), np.float32))
+        stack, dense = [], []
+        b16 = S._bf16(np.ones(W, np.float32))
+        for _ in range(L):
+            gu, dn, o = draw(2 * F, W), draw(W, F), draw(W, H * D)
+            stack.append(StackEngine.pack_layer(draw(H * D, W), draw(r, W), draw(H, W), from_numpy(np.ones(r, np.float32)), draw(H * D, r), draw(H * D, r), o, ones,
+                                                ones, heads=H, dim=D, vdim=D, window=z["window"], scale=D**-0.5, gate_up=gu, down=dn, norm2=ones, norm2b=ones))
+            dense.append(dict(attn_norm=b16, mlp_norm=b16, q_norm=None, k_norm=None, w_qkv=draw((H + 2 * z["kv_heads"]) * D, W), w_o=o, w_gate_up=gu, w_down=dn))
+        scfg = dict(vocab_size=V, width=W, max_positions=4400, norm_eps=1e-5, residual_mult=0.7)
+        dcfg = dict(vocab_size=V, hidden_size=W, num_layers=L, num_heads=H, num_kv_heads=z["kv_heads"], head_dim=D, intermediate_size=F, norm_eps=1e-5, rope_theta=1e6)
+        make = {"totolorn": lambda ms, mb: StackEngine(scfg, embed, pos, head, ones, stack, max_seq_len=ms, max_batch=mb),
+                "dense": lambda ms, mb: Engine(dcfg, embed, dense, b16, head, max_seq_len=ms, max_batch=mb, use_qk_norm=False)}
+        res = {"config": z}
+        for kind, new in make.items():
+            rec = {"prefill": {}, "decode": {}}
+            e = new(4200, 1)
+            for n in (128, 512, 2048, 4096):
+                toks = [int(t) for t in np.random.default_rng(n).integers(0, V, n)]
+                ms = wall(lambda: e.prefill(toks, want_last_logits=False))
+                rec["prefill"][n] = {"ms": round(ms, 3), "tokens_per_s": round(n / ms * 1e3)}
+            for B, ctx in ((1, 512), (1, 2048), (8, 512), (32, 512), (64, 512)):
+                e = new(ctx + 96, B)
+                toks = [int(t) for t in np.random.default_rng(ctx).integers(0, V, ctx)]
+                for b in range(B):
+                    e.prefill(toks, seq=b, want_last_logits=False)
+                e.set_state([1] * B, [ctx] * B)
+                e.capture(B)
+                e.replay(4)
+                ms = wall(lambda: e.replay(8), reps=5) / 8
+                rec["decode"][f"b{B}_ctx{ctx}"] = {"ms": round(ms, 4), "tokens_per_s": round(B / ms * 1e3), "launches": e.launches_per_step()}
+                if B == 1:
+                    prof = e.profile_step(1, 8)
+                    nb = stack_kernel_bytes(z, V, ctx, 1) if kind == "totolorn" else kernel_bytes_per_launch(dcfg, ctx, 1)
+                    rec["decode"][f"b{B}_ctx{ctx}"]["kernels"] = {
+                        k: {"us_per_layer": round(us * n / (1 if k == "lmhead" else L), 2), "hbm_frac": round(nb[k] / (us * n / (1 if k == "lmhead" else L)) / 1e3 / HBM_PEAK_GBS, 3)}
+                        for k, (us, n) in prof.items() if n and k in nb and k != "argmax"}
+                del e
+            res[kind] = rec
+        out["sizes"][size] = res
+        print(size, json.dumps(res), file=sys.stderr, flush=True)
+    return out
+
+
 def main() -> None:
     ap = argparse.ArgumentParser()
     ap.add_argument("--gpus", type=int, default=1)
@@ -138,6 +234,8 @@ def main() -> None:
                     help="skip every extra leg (config 4 weak/strong; at N = 1 also context 2048 in bf16 and w8a16, config 5)")
     ap.add_argument("--config4-steps", type=int, default=32)
     ap.add_argument("--layers", type=int, default=0, help="debug only: override the layer count (result is then INVALID)")
+    ap.add_argument("--design", choices=["totolorn"], help="instead of the headline: prefill / decode of a layer-list design beside the dense engine")
+    ap.add_argument("--design-sizes", default="w1024,w2048,w4096", help="with --design: which sizes")
     args = ap.parse_args()
 
     # ONE JSON line on stdout, whatever the libraries underneath print: RCCL writes a version banner to the process's stdout
@@ -149,6 +247,10 @@ def main() -> None:
 
     def emit(obj) -> None:
         os.write(result_fd, (json.dumps(obj) + "\n").encode())
+
+    if args.design:
+        emit(design_leg(args.design, args.design_sizes.split(","), args.seed))
+        return
 
     from pygpukit_amd import _hip
     from pygpukit_amd.core.array import GPUArray
