@@ -27,6 +27,7 @@
 
 #include "engine_state.hip.h"
 #include "latent.hip.h"
+#include "pkgemm.hip.h"
 
 namespace pgk {
 
@@ -34,6 +35,10 @@ pgk_status wsgemm_nt(const bf16* a, int lda, const void* w, const bf16* wscale, 
                      int splits, int M, int N, int K, hipStream_t st);
 bool engine_gemm_swiglu_ok(int M, int I, int K, bool fp8);     // ops_gemm.hip
 pgk_status engine_gemm_swiglu_nt(const bf16* A, const void* W, const bf16* wscale, bool fp8, bf16* act, int M, int I, int K, hipStream_t st, bool packed = false);
+
+int wsgemm_pick_splits(int N, int K, bool allow_split);        // ops_wsgemm.hip
+int engine_gemm_pick_splits(int M, int N, int K);              // ops_gemm.hip: split-K slabs for prompts whose tiles do not cover the chip
+pgk_status engine_gemm_nt_slabs(const bf16* A, const void* W, float* slabs, int splits, int M, int N, int K, hipStream_t st, bool packed = false);
 
 constexpr float LOG2E = 1.4426950408889634f;
 
@@ -247,7 +252,7 @@ static pgk_status stack_gemv(const StackGemvArgs& a, hipStream_t st, int force_g
         return stack_gemv_r<WT, 2, PRO, EPI>(a, st);
     } else if constexpr (EPI == SE_LOGITS) return stack_gemv_r<WT, 4, PRO, EPI>(a, st, force_grid);
     else {
-        if (a.N >= 4096) return stack_gemv_r<WT, 4, PRO, EPI>(a, st);
+        if (a.N >= 8192) return stack_gemv_r<WT, 4, PRO, EPI>(a, st);
         if (a.N >= 2048) return stack_gemv_r<WT, 2, PRO, EPI>(a, st);
         return stack_gemv_r<WT, 1, PRO, EPI>(a, st);
     }
@@ -263,16 +268,17 @@ struct LatentArgs {
     const int32_t* positions; // [B]
     int B, H, D, dim, vdim, rank, rank_true, R, nsplit;
     float eps, scale;         // scale already times log2e
-    float* qlat;              // [B][H][rank]
+    void* qlat;               // [B][H][rank], float or bf16
     float* po;                // [B][H][nsplit][rank]
     float* pml;               // [B][H][nsplit][2]
     void* out;                // [B][ld_out] (IT): head h at h * D
     int ld_out;
 };
 
-// q_lat[b][h][r] = scale * sum_d U_k[h D + d][r] q[b][h][d]: workgroup = (head, 128 columns) x MB sequences, the four waves split d.
+// q_lat[b][h][r] = scale * sum_d U_k[h D + d][r] q[b][h][d]: workgroup = (head, 128 columns) x MB sequences, the four waves split d
+// in runs of four; 128 rows of U_k are requested before the queries are staged.  QT: element type of q_lat (bf16 for the MFMA kernel).
 // The last workgroup column normalises the MB new latent rows into the ring instead.
-template <class T, class IT, int MB>
+template <class T, class IT, class QT, int MB>
 __global__ __launch_bounds__(256) void latent_absorb_kernel(unsigned long long* tl, LatentArgs a) {
     const TLStamp tls(tl);
     const int nt = (a.rank + 127) / 128, lane = threadIdx.x & 63, wid = threadIdx.x >> 6, b0 = blockIdx.y * MB;
@@ -290,33 +296,43 @@ __global__ __launch_bounds__(256) void latent_absorb_kernel(unsigned long long* 
         tls.end();
         return;
     }
-    __shared__ float qs[MB][512], part[4][MB][128];
+    __shared__ __attribute__((aligned(16))) float qs[MB][128];
+    __shared__ float part[4][MB][128];
     const int h = blockIdx.x / nt, r0 = (blockIdx.x % nt) * 128 + 2 * lane;
     const bool live = r0 < a.rank;                                 // rank is a multiple of 64: both columns or none
     float acc[MB][2];
 #pragma unroll
     for (int m = 0; m < MB; ++m) acc[m][0] = acc[m][1] = 0.f;
-    for (int d0 = 0; d0 < a.dim; d0 += 512) {
-        const int dn = min(512, a.dim - d0);
-        __syncthreads();
-        for (int i = threadIdx.x; i < MB * dn; i += 256) {
-            const int m = i / dn, d = i % dn;
-            qs[m][d] = to_f(in[(size_t)min(b0 + m, a.B - 1) * a.ld_in + h * a.D + d0 + d]);
+    for (int d0 = 0; d0 < a.dim; d0 += 128) {
+        const int dn = min(128, a.dim - d0);
+        const T* u = reinterpret_cast<const T*>(a.w_uk) + (size_t)(h * a.D + d0) * a.rank + (live ? r0 : 0);
+        using W2 = typename std::conditional<std::is_same<T, bf16>::value, uint32_t, float2>::type;     // two columns
+        W2 wr[32];
+#pragma unroll
+        for (int i = 0; i < 32; ++i) {
+            const int d = min(4 * (4 * (i >> 2) + wid) + (i & 3), dn - 1);
+            wr[i] = *reinterpret_cast<const W2*>(u + (size_t)d * a.rank);
         }
         __syncthreads();
-        const T* u = reinterpret_cast<const T*>(a.w_uk) + (size_t)(h * a.D + d0) * a.rank + (live ? r0 : 0);
-#pragma unroll 8
-        for (int d = wid; d < dn; d += 4) {
-            float w0, w1;
-            if constexpr (std::is_same<T, bf16>::value) {
-                const uint32_t x = *reinterpret_cast<const uint32_t*>(u + (size_t)d * a.rank);
-                w0 = __uint_as_float(x << 16); w1 = __uint_as_float(x & 0xFFFF0000u);
-            } else {
-                const float2 x = *reinterpret_cast<const float2*>(u + (size_t)d * a.rank);
-                w0 = x.x; w1 = x.y;
+        for (int i = threadIdx.x; i < MB * 128; i += 256) {
+            const int m = i >> 7, d = i & 127;
+            qs[m][d] = d < dn ? to_f(in[(size_t)min(b0 + m, a.B - 1) * a.ld_in + h * a.D + d0 + d]) : 0.f;
+        }
+        __syncthreads();
+#pragma unroll
+        for (int i = 0; i < 8; ++i) {
+            float w[4][2];
+#pragma unroll
+            for (int k = 0; k < 4; ++k) {
+                if constexpr (std::is_same<T, bf16>::value) { w[k][0] = __uint_as_float(wr[4 * i + k] << 16); w[k][1] = __uint_as_float(wr[4 * i + k] & 0xFFFF0000u); }
+                else { w[k][0] = wr[4 * i + k].x; w[k][1] = wr[4 * i + k].y; }
             }
 #pragma unroll
-            for (int m = 0; m < MB; ++m) { acc[m][0] = fmaf(w0, qs[m][d], acc[m][0]); acc[m][1] = fmaf(w1, qs[m][d], acc[m][1]); }
+            for (int m = 0; m < MB; ++m) {
+                const float4 q = *reinterpret_cast<const float4*>(&qs[m][4 * (4 * i + wid)]);
+#pragma unroll
+                for (int e = 0; e < 2; ++e) acc[m][e] = fmaf(w[3][e], q.w, fmaf(w[2][e], q.z, fmaf(w[1][e], q.y, fmaf(w[0][e], q.x, acc[m][e]))));
+            }
         }
     }
 #pragma unroll
@@ -325,15 +341,15 @@ __global__ __launch_bounds__(256) void latent_absorb_kernel(unsigned long long* 
     for (int i = threadIdx.x; i < MB * 128; i += 256) {
         const int m = i >> 7, c = i & 127, r = (blockIdx.x % nt) * 128 + c;
         if (b0 + m < a.B && r < a.rank)
-            a.qlat[((size_t)(b0 + m) * a.H + h) * a.rank + r] = a.scale * (part[0][m][c] + part[1][m][c] + part[2][m][c] + part[3][m][c]);
+            reinterpret_cast<QT*>(a.qlat)[((size_t)(b0 + m) * a.H + h) * a.rank + r] = from_f<QT>(a.scale * (part[0][m][c] + part[1][m][c] + part[2][m][c] + part[3][m][c]));
     }
     tls.end();
 }
 
-// the ring rows [k0, k1) of split s out of n occupied rows
+// n occupied ring rows over nsplit splits: rows per split (a multiple of 32), the rows [k0, k1) of split s
+__device__ __forceinline__ int split_rows(int n, int nsplit) { return ((n + nsplit - 1) / nsplit + 31) / 32 * 32; }
 __device__ __forceinline__ void split_range(int n, int nsplit, int s, int& k0, int& k1) {
-    int per = (n + nsplit - 1) / nsplit;
-    per = (per + 31) / 32 * 32;
+    const int per = split_rows(n, nsplit);
     k0 = min(s * per, n);
     k1 = min(k0 + per, n);
 }
@@ -352,7 +368,7 @@ __global__ __launch_bounds__(256) void latent_attn_kernel(unsigned long long* tl
 #pragma unroll
     for (int i = 0; i < HB; ++i) {
         m[i] = -INFINITY; l[i] = 0.f;
-        const float* qp = a.qlat + ((size_t)b * a.H + min(h0 + i, a.H - 1)) * a.rank;
+        const float* qp = reinterpret_cast<const float*>(a.qlat) + ((size_t)b * a.H + min(h0 + i, a.H - 1)) * a.rank;
 #pragma unroll
         for (int j = 0; j < RC; ++j) { const int r = 64 * j + lane; q[i][j] = r < a.rank ? qp[r] : 0.f; o[i][j] = 0.f; }
     }
@@ -407,13 +423,154 @@ __global__ __launch_bounds__(256) void latent_attn_kernel(unsigned long long* tl
     tls.end();
 }
 
-// Combine the split records of (sequence, head), apply U_v (rows v of the workgroup's 32) and the head's gate.
-template <class T, class IT, int MB>
+// bf16, rank <= 64 RT <= 896: 16 heads x 64 keys per step on the matrix pipe.  Every head scores against the SAME latent rows, so one
+// LDS image of a key tile is both operands: S[head][key] = q_lat . C^T (each wave 16 keys), then O[head][r] += P . C (each wave its
+// share of the columns; C^T comes out of the row-major image through ds_read_b64_tr_b16, whose k order is 16 (j >> 2) + 4 (lane >> 4)
+// + (j & 3), and P is read back from LDS in that order).
+typedef __bf16 bf16x8_st __attribute__((ext_vector_type(8)));
+typedef float f32x4_st __attribute__((ext_vector_type(4)));
+typedef short v4s_st __attribute__((ext_vector_type(4)));
+__device__ __forceinline__ f32x4_st mfma16_st(const uint4& a, const uint4& b, f32x4_st c) {
+    return __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8_st, a), __builtin_bit_cast(bf16x8_st, b), c, 0, 0, 0);
+}
+
+constexpr int LA_PAD = 8;           // elements added to an LDS row: rows start 4 banks apart
+static size_t latent_mfma_lds(int rank) { return (size_t)(64 + 16) * (rank + LA_PAD) * 2; }
+
+template <int RT>
+__global__ __launch_bounds__(256) void latent_attn_mfma_kernel(unsigned long long* tl, LatentArgs a) {
+    const TLStamp tls(tl);
+    extern __shared__ __attribute__((aligned(16))) char la_smem[];
+    __shared__ __attribute__((aligned(16))) bf16 ps[16][72];
+    __shared__ float red[4][16];
+    const int ld = a.rank + LA_PAD, nch = a.rank / 8;
+    bf16* cs = reinterpret_cast<bf16*>(la_smem);                  // [64][ld]
+    bf16* qs = cs + 64 * ld;                                      // [16][ld]
+    const int tid = threadIdx.x, lane = tid & 63, wid = tid >> 6, l15 = lane & 15, q4 = lane >> 4;
+    const int s = blockIdx.x, h0 = blockIdx.y * 16, b = blockIdx.z;
+    const int n = min(max(a.positions[b], 0) + 1, a.R);
+    int k0, k1;
+    split_range(n, a.nsplit, s, k0, k1);
+    float m_run[4], l_run[4];
+    f32x4_st o[RT];
+#pragma unroll
+    for (int i = 0; i < 4; ++i) { m_run[i] = -INFINITY; l_run[i] = 0.f; }
+#pragma unroll
+    for (int t = 0; t < RT; ++t) o[t] = f32x4_st{0.f, 0.f, 0.f, 0.f};
+    if (k0 >= k1) {                                                // an empty split: its record says so, the sums are never read
+        if (tid < 16 && h0 + tid < a.H) {
+            float* ml = a.pml + (((size_t)b * a.H + h0 + tid) * a.nsplit + s) * 2;
+            ml[0] = -INFINITY; ml[1] = 0.f;
+        }
+        tls.end();
+        return;
+    }
+    const bf16* cb = reinterpret_cast<const bf16*>(a.cache) + (size_t)b * a.R * a.rank;
+    const bf16* qb = reinterpret_cast<const bf16*>(a.qlat) + (size_t)b * a.H * a.rank;
+    for (int c = tid; c < 16 * nch; c += 256) {
+        const int r = c / nch, k = c % nch;
+        *reinterpret_cast<uint4*>(qs + r * ld + k * 8) = *reinterpret_cast<const uint4*>(qb + (size_t)min(h0 + r, a.H - 1) * a.rank + k * 8);
+    }
+    for (int kt = k0; kt < k1; kt += 64) {
+        const int rt = k1 - kt > 32 ? 64 : 32;                    // rows of this tile that are staged
+        if (kt != k0) __syncthreads();                            // the last step's reads of cs are done
+#pragma unroll 8
+        for (int c = tid; c < rt * nch; c += 256) {
+            const int r = c / nch, k = c % nch;
+            *reinterpret_cast<uint4*>(cs + r * ld + k * 8) = *reinterpret_cast<const uint4*>(cb + (size_t)min(kt + r, k1 - 1) * a.rank + k * 8);
+        }
+        __syncthreads();
+        f32x4_st sc = {-INFINITY, -INFINITY, -INFINITY, -INFINITY};
+        const bool mine = 16 * wid < rt;                          // wave-uniform
+        if (mine) {
+            f32x4_st t = {0.f, 0.f, 0.f, 0.f};
+            const bf16* qr = qs + l15 * ld + 8 * q4;
+            const bf16* cr = cs + (16 * wid + l15) * ld + 8 * q4;
+            for (int ks = 0; ks < a.rank; ks += 32) t = mfma16_st(*reinterpret_cast<const uint4*>(qr + ks), *reinterpret_cast<const uint4*>(cr + ks), t);
+            if (kt + 16 * wid + l15 < k1) sc = t;                 // lane: heads 4 q4 + i, key 16 wid + l15
+        }
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+            const float t = group16_max(sc[i]);
+            if (l15 == 0) red[wid][4 * q4 + i] = t;
+        }
+        __syncthreads();
+        float al[4];
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+            const int hh = 4 * q4 + i;
+            const float mn = fmaxf(m_run[i], fmaxf(fmaxf(red[0][hh], red[1][hh]), fmaxf(red[2][hh], red[3][hh])));   // finite: kt < k1
+            al[i] = __builtin_amdgcn_exp2f(m_run[i] - mn);
+            m_run[i] = mn;
+            const float p = __builtin_amdgcn_exp2f(sc[i] - mn);
+            l_run[i] = l_run[i] * al[i] + p;
+            if (mine) ps[hh][16 * wid + l15] = from_f<bf16>(p);
+        }
+        __syncthreads();
+#pragma unroll
+        for (int t = 0; t < RT; ++t)
+#pragma unroll
+            for (int i = 0; i < 4; ++i) o[t][i] *= al[i];
+        for (int ks = 0; ks < rt; ks += 32) {
+            const uint2 p0 = *reinterpret_cast<const uint2*>(&ps[l15][ks + 4 * q4]), p1 = *reinterpret_cast<const uint2*>(&ps[l15][ks + 16 + 4 * q4]);
+            const uint4 pf = make_uint4(p0.x, p0.y, p1.x, p1.y);
+            const bf16* row = cs + (ks + 4 * q4 + (l15 >> 2)) * ld + 4 * (l15 & 3);
+#pragma unroll
+            for (int t = 0; t < RT; ++t) {
+                const int col = 16 * (wid + 4 * t);
+                if (col < a.rank) {                               // wave-uniform
+                    const v4s_st c0 = __builtin_amdgcn_ds_read_tr16_b64_v4i16((__attribute__((address_space(3))) v4s_st*)(row + col));
+                    const v4s_st c1 = __builtin_amdgcn_ds_read_tr16_b64_v4i16((__attribute__((address_space(3))) v4s_st*)(row + 16 * ld + col));
+                    const uint2 u0 = __builtin_bit_cast(uint2, c0), u1 = __builtin_bit_cast(uint2, c1);
+                    o[t] = mfma16_st(pf, make_uint4(u0.x, u0.y, u1.x, u1.y), o[t]);
+                }
+            }
+        }
+    }
+    // lane: heads 4 q4 + i, column l15 of each 16-column tile; the row sums are spread over the 16 lanes of a group and the waves
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+        const float t = group16_sum(l_run[i]);
+        if (l15 == 0) red[wid][4 * q4 + i] = t;
+    }
+    // (red was last read before the barrier that precedes the products)
+    __syncthreads();
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+        const int hh = h0 + 4 * q4 + i;
+        if (hh >= a.H) continue;
+        const size_t rec = ((size_t)b * a.H + hh) * a.nsplit + s;
+#pragma unroll
+        for (int t = 0; t < RT; ++t) {
+            const int col = 16 * (wid + 4 * t) + l15;
+            if (col < a.rank) a.po[rec * a.rank + col] = o[t][i];
+        }
+        if (wid == 0 && l15 == 0) {
+            a.pml[2 * rec] = m_run[i];
+            a.pml[2 * rec + 1] = red[0][4 * q4 + i] + red[1][4 * q4 + i] + red[2][4 * q4 + i] + red[3][4 * q4 + i];
+        }
+    }
+    tls.end();
+}
+
+// Combine the split records of (sequence, head), apply U_v (the workgroup's 32 rows) and the head's gate.  The waves share the splits,
+// then meet in LDS; a row of U_v is 16 lanes wide, requested before the records when the rank allows (PF 128-column pieces per row).
+template <class T, class IT, int MB, int PF>
 __global__ __launch_bounds__(256) void latent_merge_uv_kernel(unsigned long long* tl, LatentArgs a) {
     const TLStamp tls(tl);
-    extern __shared__ __attribute__((aligned(16))) float ol[];     // [MB][rank]
+    extern __shared__ __attribute__((aligned(16))) float ol[];     // [4][MB][rank]; afterwards [MB][rank]
     __shared__ float sw[MB][64];
-    const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6, h = blockIdx.x, v0 = blockIdx.y * 32, b0 = blockIdx.z * MB;
+    constexpr int NW = WTraits<T>::NW;
+    const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6, h = blockIdx.x, v0 = blockIdx.y * 32, b0 = blockIdx.z * MB, sub = lane & 15, grp = lane >> 4;
+    const T* u = reinterpret_cast<const T*>(a.w_uv) + (size_t)h * a.D * a.rank;
+    uint4 w[2][PF > 0 ? PF : 1];
+    if constexpr (PF > 0) {
+#pragma unroll
+        for (int p = 0; p < 2; ++p)
+#pragma unroll
+            for (int k = 0; k < PF; ++k)
+                w[p][k] = *reinterpret_cast<const uint4*>(u + (size_t)min(v0 + 8 * wid + 4 * p + grp, a.vdim - 1) * a.rank + min(16 * NW * k + sub * NW, a.rank - NW));
+    }
     for (int m = wid; m < MB; m += 4) {
         const size_t rec = ((size_t)min(b0 + m, a.B - 1) * a.H + h) * a.nsplit;
         const float mm = lane < a.nsplit ? a.pml[(rec + lane) * 2] : -INFINITY, ll = lane < a.nsplit ? a.pml[(rec + lane) * 2 + 1] : 0.f;
@@ -422,35 +579,61 @@ __global__ __launch_bounds__(256) void latent_merge_uv_kernel(unsigned long long
         sw[m][lane] = f / den;
     }
     __syncthreads();
-    for (int i = threadIdx.x; i < MB * a.rank; i += 256) {
-        const int m = i / a.rank, r = i % a.rank;
-        const float* p = a.po + ((size_t)min(b0 + m, a.B - 1) * a.H + h) * a.nsplit * a.rank + r;
-        float t = 0.f;
-        for (int s = 0; s < a.nsplit; ++s) {
-            const float f = sw[m][s];                              // empty splits hold zeros or nothing of this step
-            t = fmaf(f, f > 0.f ? p[(size_t)s * a.rank] : 0.f, t);
+#pragma unroll
+    for (int m = 0; m < MB; ++m) {
+        const int b = min(b0 + m, a.B - 1), n = min(max(a.positions[b], 0) + 1, a.R), per = split_rows(n, a.nsplit), nact = (n + per - 1) / per;
+        const float* rec = a.po + ((size_t)b * a.H + h) * a.nsplit * a.rank;
+        for (int r = 4 * lane; r < a.rank; r += 256) {
+            float4 t = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll 8
+            for (int s = wid; s < nact; s += 4) {
+                const float f = sw[m][s];
+                const float4 p = *reinterpret_cast<const float4*>(rec + (size_t)s * a.rank + r);
+                t.x = fmaf(f, p.x, t.x); t.y = fmaf(f, p.y, t.y); t.z = fmaf(f, p.z, t.z); t.w = fmaf(f, p.w, t.w);
+            }
+            *reinterpret_cast<float4*>(ol + ((size_t)wid * MB + m) * a.rank + r) = t;
         }
-        ol[i] = t;
     }
     __syncthreads();
-    constexpr int NW = WTraits<T>::NW;
-    const T* u = reinterpret_cast<const T*>(a.w_uv) + (size_t)h * a.D * a.rank;
-    for (int v = v0 + wid; v < min(v0 + 32, a.vdim); v += 4) {
+    const int span = MB * a.rank;
+    for (int i = 4 * threadIdx.x; i < span; i += 1024) {
+        float4 t = *reinterpret_cast<const float4*>(ol + i);
+#pragma unroll
+        for (int q = 1; q < 4; ++q) {
+            const float4 p = *reinterpret_cast<const float4*>(ol + q * span + i);
+            t.x += p.x; t.y += p.y; t.z += p.z; t.w += p.w;
+        }
+        *reinterpret_cast<float4*>(ol + i) = t;
+    }
+    __syncthreads();
+#pragma unroll
+    for (int p = 0; p < 2; ++p) {
+        const int v = v0 + 8 * wid + 4 * p + grp;
         float acc[MB];
 #pragma unroll
         for (int m = 0; m < MB; ++m) acc[m] = 0.f;
-        for (int r = lane * NW; r < a.rank; r += 64 * NW) {
-            float w[NW];
-            WTraits<T>::decode(*reinterpret_cast<const uint4*>(u + (size_t)v * a.rank + r), w);
+        auto piece = [&](const uint4& raw, int r) {
+            float f[NW];
+            WTraits<T>::decode(raw, f);
 #pragma unroll
             for (int m = 0; m < MB; ++m)
 #pragma unroll
-                for (int j = 0; j < NW; ++j) acc[m] = fmaf(w[j], ol[m * a.rank + r + j], acc[m]);
+                for (int j = 0; j < NW; j += 4) {
+                    const float4 x = *reinterpret_cast<const float4*>(ol + m * a.rank + r + j);
+                    acc[m] = fmaf(f[j + 3], x.w, fmaf(f[j + 2], x.z, fmaf(f[j + 1], x.y, fmaf(f[j], x.x, acc[m]))));
+                }
+        };
+        if constexpr (PF > 0) {
+#pragma unroll
+            for (int k = 0; k < PF; ++k) { const int r = 16 * NW * k + sub * NW; if (r < a.rank) piece(w[p][k], r); }
+        } else {
+            const T* row = u + (size_t)min(v, a.vdim - 1) * a.rank;
+            for (int r = sub * NW; r < a.rank; r += 16 * NW) piece(*reinterpret_cast<const uint4*>(row + r), r);
         }
 #pragma unroll
         for (int m = 0; m < MB; ++m) {
-            const float y = wave_sum(acc[m]);
-            if (lane == 0 && b0 + m < a.B) {
+            const float y = group16_sum(acc[m]);
+            if (sub == 0 && v < a.vdim && b0 + m < a.B) {
                 const float g = to_f(reinterpret_cast<const IT*>(a.in)[(size_t)(b0 + m) * a.ld_in + a.g_off + h]);
                 reinterpret_cast<IT*>(a.out)[(size_t)(b0 + m) * a.ld_out + h * a.D + v] = from_f<IT>(y / (1.0f + expf(-g)));
             }
@@ -535,9 +718,13 @@ struct Stack {
     std::vector<int> ring;                 // R per layer
     std::vector<int32_t> len;              // per slot: positions held (host side; advanced with every step enqueued)
     // decode buffers (rows = max_batch)
-    float *in32 = nullptr, *a32 = nullptr, *y32 = nullptr, *act32 = nullptr, *qlat = nullptr, *po = nullptr, *pml = nullptr;
-    void *x16 = nullptr, *in16 = nullptr, *a16 = nullptr, *y16 = nullptr, *gu16 = nullptr, *act16 = nullptr;
-    int max_split = 64;
+    float *in32 = nullptr, *a32 = nullptr, *y32 = nullptr, *act32 = nullptr, *po = nullptr, *pml = nullptr;
+    void *qlat = nullptr, *x16 = nullptr, *in16 = nullptr, *a16 = nullptr, *y16 = nullptr, *gu16 = nullptr, *act16 = nullptr;
+    float* slabs16 = nullptr;              // split-K slabs of a batch step's projections
+    // fragment-major copies of the layer matrices for 2..128 rows (ops_pkgemm.hip), where its shapes allow; null entries: row-major kernels
+    struct Packed { bf16 *in = nullptr, *o = nullptr, *gate_up = nullptr, *down = nullptr; };
+    std::vector<Packed> packed;
+    size_t slab_elems(int n, bool f32) const;   // fp32 elements the projections of n rows may need
     // prompt buffers, grown on demand outside capture
     void* pf = nullptr; size_t pf_bytes = 0;
     void* tab = nullptr; size_t tab_bytes = 0;
@@ -553,14 +740,36 @@ static int pick_nsplit(const Engine* e, int B, const pgk_stack_layer_t& L, int R
     return s > 64 ? 64 : (s < 1 ? 1 : s);
 }
 
-template <class T, int HB>
+constexpr int LATENT_LDS_MAX = 144 * 1024;
+#define PGK_ALLOW_LDS(kfn, lds)                                                                                                   \
+    {                                                                                                                              \
+        static bool done = false;                                                                                                  \
+        if ((lds) > 48 * 1024 && !done) {                                                                                          \
+            if (hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(kfn), hipFuncAttributeMaxDynamicSharedMemorySize, LATENT_LDS_MAX)) return e; \
+            done = true;                                                                                                           \
+        }                                                                                                                          \
+    }
+
+template <class T, int RC>
 static hipError_t launch_latent_attn(const LatentArgs& a, hipStream_t st) {
-    const dim3 grid(a.nsplit, ceil_div(a.H, HB), a.B);
-    const size_t lds = (size_t)HB * a.rank * 4;
-#define PGK_RC(N) if (a.rank <= 64 * N) return launch_k(&latent_attn_kernel<T, N, HB>, grid, dim3(256), lds, st, a);
-    PGK_RC(1) PGK_RC(2) PGK_RC(4) PGK_RC(8) PGK_RC(16)
-#undef PGK_RC
-    return launch_k(&latent_attn_kernel<T, 32, HB>, grid, dim3(256), lds, st, a);
+    return launch_k(&latent_attn_kernel<T, RC, 4>, dim3(a.nsplit, ceil_div(a.H, 4), a.B), dim3(256), (size_t)4 * a.rank * 4, st, a);
+}
+template <int RT>
+static hipError_t launch_latent_mfma(const LatentArgs& a, hipStream_t st) {
+    const size_t lds = latent_mfma_lds(a.rank);
+    PGK_ALLOW_LDS(&latent_attn_mfma_kernel<RT>, lds)
+    return launch_k(&latent_attn_mfma_kernel<RT>, dim3(a.nsplit, ceil_div(a.H, 16), a.B), dim3(256), lds, st, a);
+}
+template <class T, class IT, int MB, int PF>
+static hipError_t launch_merge_uv(const LatentArgs& a, hipStream_t st) {
+    const size_t lds = (size_t)4 * MB * a.rank * 4;
+    auto kfn = &latent_merge_uv_kernel<T, IT, MB, PF>;
+    PGK_ALLOW_LDS(kfn, lds)
+    return launch_k(kfn, dim3(a.H, ceil_div(a.vdim, 32), ceil_div(a.B, MB)), dim3(256), lds, st, a);
+}
+template <class T, class IT, class QT, int MB>
+static hipError_t launch_absorb(const LatentArgs& a, hipStream_t st) {
+    return launch_k(&latent_absorb_kernel<T, IT, QT, MB>, dim3(a.H * ceil_div(a.rank, 128) + 1, ceil_div(a.B, MB)), dim3(256), 0, st, a);
 }
 
 // absorb -> attention over the ring -> merge + U_v + gate for B sequences whose in-projection rows are in `in`
@@ -568,6 +777,7 @@ template <class T, class IT>
 static pgk_status latent_decode(Engine* e, int l, int B, const void* in, void* out, hipStream_t st, int* launches) {
     Stack* s = stack_of(e);
     const auto& L = s->layers[l];
+    constexpr bool F32 = std::is_same<T, float>::value;
     LatentArgs a{};
     a.in = in; a.ld_in = L.n_in; a.qn = L.heads * L.head_pad; a.g_off = a.qn + L.rank_pad;
     a.w_uk = L.w_ukv; a.w_uv = (const char*)L.w_ukv + (size_t)L.heads * L.head_pad * L.rank_pad * sizeof(T);
@@ -576,13 +786,31 @@ static pgk_status latent_decode(Engine* e, int l, int B, const void* in, void* o
     a.nsplit = pick_nsplit(e, B, L, a.R);
     a.eps = s->cfg.norm_eps; a.scale = L.scale * LOG2E;
     a.qlat = s->qlat; a.po = s->po; a.pml = s->pml; a.out = out; a.ld_out = L.heads * L.head_pad;
-    const int nx = L.heads * ceil_div(a.rank, 128) + 1;
-    if (B == 1) PGK_CHECK_HIP((launch_k(&latent_absorb_kernel<T, IT, 1>, dim3(nx, 1), dim3(256), 0, st, a)));
-    else PGK_CHECK_HIP((launch_k(&latent_absorb_kernel<T, IT, 4>, dim3(nx, ceil_div(B, 4)), dim3(256), 0, st, a)));
-    PGK_CHECK_HIP((launch_latent_attn<T, 4>(a, st)));
-    const int nv = ceil_div(a.vdim, 32);
-    if (B == 1) PGK_CHECK_HIP((launch_k(&latent_merge_uv_kernel<T, IT, 1>, dim3(a.H, nv, 1), dim3(256), (size_t)a.rank * 4, st, a)));
-    else PGK_CHECK_HIP((launch_k(&latent_merge_uv_kernel<T, IT, 4>, dim3(a.H, nv, ceil_div(B, 4)), dim3(256), (size_t)4 * a.rank * 4, st, a)));
+    const bool mfma = !F32 && a.rank <= 896;
+    if (!mfma) {
+        PGK_CHECK_HIP((B == 1 ? launch_absorb<T, IT, float, 1>(a, st) : launch_absorb<T, IT, float, 4>(a, st)));
+        if (a.rank <= 64) PGK_CHECK_HIP((launch_latent_attn<T, 1>(a, st)));
+        else if (a.rank <= 128) PGK_CHECK_HIP((launch_latent_attn<T, 2>(a, st)));
+        else if (a.rank <= 256) PGK_CHECK_HIP((launch_latent_attn<T, 4>(a, st)));
+        else if (a.rank <= 512) PGK_CHECK_HIP((launch_latent_attn<T, 8>(a, st)));
+        else if (a.rank <= 1024) PGK_CHECK_HIP((launch_latent_attn<T, 16>(a, st)));
+        else PGK_CHECK_HIP((launch_latent_attn<T, 32>(a, st)));
+    }
+    if constexpr (!F32) {
+        if (mfma) {
+            PGK_CHECK_HIP((B == 1 ? launch_absorb<T, IT, bf16, 1>(a, st) : launch_absorb<T, IT, bf16, 8>(a, st)));
+            if (a.rank <= 64) PGK_CHECK_HIP(launch_latent_mfma<1>(a, st));
+            else if (a.rank <= 128) PGK_CHECK_HIP(launch_latent_mfma<2>(a, st));
+            else if (a.rank <= 256) PGK_CHECK_HIP(launch_latent_mfma<4>(a, st));
+            else if (a.rank <= 512) PGK_CHECK_HIP(launch_latent_mfma<8>(a, st));
+            else PGK_CHECK_HIP(launch_latent_mfma<14>(a, st));
+        }
+    }
+    if constexpr (!F32) {
+        if (a.rank <= 256) PGK_CHECK_HIP((B == 1 ? launch_merge_uv<T, IT, 1, 2>(a, st) : launch_merge_uv<T, IT, 4, 2>(a, st)));
+        else if (a.rank <= 512) PGK_CHECK_HIP((B == 1 ? launch_merge_uv<T, IT, 1, 4>(a, st) : launch_merge_uv<T, IT, 4, 4>(a, st)));
+        else PGK_CHECK_HIP((B == 1 ? launch_merge_uv<T, IT, 1, 0>(a, st) : launch_merge_uv<T, IT, 4, 0>(a, st)));
+    } else PGK_CHECK_HIP((B == 1 ? launch_merge_uv<T, IT, 1, 0>(a, st) : launch_merge_uv<T, IT, 4, 0>(a, st)));
     *launches += 3;
     return PGK_OK;
 }
@@ -651,48 +879,119 @@ static pgk_status head_rows(Stack* s, const T* x, float* logits, int n, hipStrea
     return PGK_OK;
 }
 
-struct RowBufs { float* h; void *x, *in, *a, *y, *gu, *act; };
+struct RowBufs { float* h; void *x, *in, *a, *y, *gu, *act; float* slabs; };
 
-// feed-forward of n rows: act = silu(x W_g) * (x W_u), y = act W_d
-template <class T>
-static pgk_status rows_mlp(Stack* s, const pgk_stack_layer_t& L, const RowBufs& b, int n, hipStream_t st) {
-    constexpr pgk_dtype DT = std::is_same<T, float>::value ? PGK_F32 : PGK_BF16;
-    if (DT == PGK_BF16 && engine_gemm_swiglu_ok(n, L.ff_pad, s->Wp, false)) {
-        if (pgk_status r = engine_gemm_swiglu_nt((const bf16*)b.x, L.w_gate_up, nullptr, false, (bf16*)b.act, n, L.ff_pad, s->Wp, st)) return r;
-    } else {
-        if (pgk_status r = pgk_gemm_nt(b.x, L.w_gate_up, nullptr, b.gu, n, 2 * L.ff_pad, s->Wp, DT, st)) return r;
-        if (pgk_status r = pgk_glu_packed(b.gu, b.act, n, L.ff_pad, 0, DT, st)) return r;
+// How a [N, K] projection of n bf16 rows runs: fragment-major copy (<= 128 rows), weight-streaming kernel (<= 128 rows) or tiled
+// MFMA, and over how many split-K slabs its result is left (0: one bf16 result).
+struct ProjPlan { bool pk; int slabs; };
+static ProjPlan plan_proj(const bf16* packed, int n, int N, int K, bool split) {
+    if (n <= 128) {
+        if (packed) return {true, split ? pkgemm_pick_splits(n, N, K) : 0};
+        const int s = split && n > 1 ? wsgemm_pick_splits(N, K, true) : 1;
+        return {false, s > 1 ? s : 0};
     }
-    return pgk_gemm_nt(b.act, L.w_down, nullptr, b.y, n, s->Wp, L.ff_pad, DT, st);
+    const int s = split ? engine_gemm_pick_splits(n, N, K) : 1;
+    return {false, s > 1 ? s : 0};
+}
+size_t Stack::slab_elems(int n, bool f32) const {
+    size_t m = 64;
+    if (f32) return m;
+    for (size_t l = 0; l < layers.size(); ++l) {
+        const auto& L = layers[l];
+        const Packed P = packed.empty() ? Packed{} : packed[l];
+        const size_t need[] = {(size_t)plan_proj(P.o, n, Wp, L.heads * L.head_pad, true).slabs * n * Wp,
+                               L.ff_pad ? (size_t)plan_proj(P.down, n, Wp, L.ff_pad, true).slabs * n * Wp : 0,
+                               P.in || n > 128 ? 0 : (size_t)plan_proj(nullptr, n, L.n_in, Wp, true).slabs * n * L.n_in};
+        for (size_t z : need) m = z > m ? z : m;
+    }
+    return m;
 }
 
-// The layers on n rows of b.h; `mix(l)` turns in-projection rows b.in into attention rows b.a.  Returns the pending post-norm.
-template <class T, class Mix>
-static pgk_status rows_layers(Stack* s, const RowBufs& b, int n, hipStream_t st, const float** pend_out, Mix mix) {
+// bf16 rows = sum of fp32 slabs
+__global__ __launch_bounds__(256) void slab_rows_kernel(const float* slabs, int ns, bf16* out, size_t n4) {
+    for (size_t i = blockIdx.x * (size_t)256 + threadIdx.x; i < n4; i += (size_t)gridDim.x * 256) {
+        float4 t = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll 4
+        for (int s = 0; s < ns; ++s) {
+            const float4 q = reinterpret_cast<const float4*>(slabs)[s * n4 + i];
+            t.x += q.x; t.y += q.y; t.z += q.z; t.w += q.w;
+        }
+        store4<bf16>(out + 4 * i, t);
+    }
+}
+
+// A sublayer's last projection: y rows in the element type, or *slabs split-K slabs for the norm that follows
+template <class T>
+static pgk_status rows_out_proj(Stack* s, const RowBufs& b, const void* x, const void* w, const bf16* packed, int n, int K, int* slabs, hipStream_t st) {
+    *slabs = 0;
+    if constexpr (std::is_same<T, float>::value) return pgk_gemm_nt(x, w, nullptr, b.y, n, s->Wp, K, PGK_F32, st);
+    const ProjPlan p = plan_proj(packed, n, s->Wp, K, true);
+    *slabs = p.slabs;
+    if (p.pk) return pkgemm_nt((const bf16*)x, K, packed, b.slabs, s->Wp, PK_EPI_SLAB, p.slabs, n, s->Wp, K, nullptr, st);
+    if (!p.slabs) return pgk_gemm_nt(x, w, nullptr, b.y, n, s->Wp, K, PGK_BF16, st);
+    if (n <= 128) return wsgemm_nt((const bf16*)x, K, w, nullptr, false, b.slabs, nullptr, 1, p.slabs, n, s->Wp, K, st);
+    return engine_gemm_nt_slabs((const bf16*)x, w, b.slabs, p.slabs, n, s->Wp, K, st);
+}
+
+template <class T>
+static pgk_status rows_in_proj(Stack* s, const pgk_stack_layer_t& L, const bf16* packed, const RowBufs& b, int n, hipStream_t st) {
+    if constexpr (std::is_same<T, float>::value) return pgk_gemm_nt(b.x, L.w_in, nullptr, b.in, n, L.n_in, s->Wp, PGK_F32, st);
+    if (n <= 128 && packed) return pkgemm_nt((const bf16*)b.x, s->Wp, packed, b.in, L.n_in, PK_EPI_BF16, 1, n, L.n_in, s->Wp, nullptr, st);
+    const int slabs = n <= 128 ? plan_proj(nullptr, n, L.n_in, s->Wp, true).slabs : 0;
+    if (!slabs) return pgk_gemm_nt(b.x, L.w_in, nullptr, b.in, n, L.n_in, s->Wp, PGK_BF16, st);
+    if (pgk_status r = wsgemm_nt((const bf16*)b.x, s->Wp, L.w_in, nullptr, false, b.slabs, nullptr, 1, slabs, n, L.n_in, s->Wp, st)) return r;
+    const size_t n4 = (size_t)n * L.n_in / 4;
+    slab_rows_kernel<<<(unsigned)(n4 / 256 > 2048 ? 2048 : (n4 + 255) / 256), 256, 0, st>>>(b.slabs, slabs, (bf16*)b.in, n4);
+    PGK_LAUNCH_CHECK();
+    return PGK_OK;
+}
+
+// gate / up projection with SwiGLU of n rows: act = silu(x W_g) * (x W_u)
+template <class T>
+static pgk_status rows_gate_up(Stack* s, const pgk_stack_layer_t& L, const bf16* packed, const RowBufs& b, int n, hipStream_t st) {
     constexpr pgk_dtype DT = std::is_same<T, float>::value ? PGK_F32 : PGK_BF16;
-    const auto& c = s->cfg;
-    const float* pend = nullptr;
-    auto norm = [&](const float* gamma) -> pgk_status {
-        RowsNormArgs a{b.h, pend ? b.y : nullptr, s->Wp, pend, c.residual_mult, gamma, b.x, c.width, s->Wp, c.norm_eps, nullptr, 1};
-        return rows_norm(a, n, DT, st);
-    };
-    for (int l = 0; l < c.num_layers; ++l) {
+    if (DT == PGK_BF16 && n <= 128 && packed)
+        return pkgemm_nt((const bf16*)b.x, s->Wp, packed, b.act, L.ff_pad, PK_EPI_SWIGLU, 1, n, 2 * L.ff_pad, s->Wp, nullptr, st);
+    if (DT == PGK_BF16 && engine_gemm_swiglu_ok(n, L.ff_pad, s->Wp, false))
+        return engine_gemm_swiglu_nt((const bf16*)b.x, L.w_gate_up, nullptr, false, (bf16*)b.act, n, L.ff_pad, s->Wp, st);
+    if (pgk_status r = pgk_gemm_nt(b.x, L.w_gate_up, nullptr, b.gu, n, 2 * L.ff_pad, s->Wp, DT, st)) return r;
+    return pgk_glu_packed(b.gu, b.act, n, L.ff_pad, 0, DT, st);
+}
+
+struct Pending { const float* gain = nullptr; int slabs = 0; };     // the sublayer output whose norm and residual add are still to come
+
+static RowsNormArgs norm_args(const Stack* s, const RowBufs& b, int n, const Pending& p, const float* gamma, void* out) {
+    RowsNormArgs a{};
+    a.h = b.h; a.y = !p.gain ? nullptr : p.slabs ? (const void*)b.slabs : b.y; a.ldy = s->Wp; a.g_post = p.gain; a.mult = s->cfg.residual_mult;
+    a.gamma = gamma; a.out = out; a.W = s->cfg.width; a.ld = s->Wp; a.eps = s->cfg.norm_eps; a.store_h = 1;
+    a.nslabs = p.gain ? p.slabs : 0; a.slab_stride = (long long)n * s->Wp;
+    return a;
+}
+
+// The layers on n rows of b.h; `mix(l)` turns in-projection rows b.in into attention rows b.a.  Leaves the last sublayer pending.
+template <class T, class Mix>
+static pgk_status rows_layers(Stack* s, const RowBufs& b, int n, hipStream_t st, Pending* pend, Mix mix) {
+    constexpr pgk_dtype DT = std::is_same<T, float>::value ? PGK_F32 : PGK_BF16;
+    *pend = Pending{};
+    for (int l = 0; l < s->cfg.num_layers; ++l) {
         const auto& L = s->layers[l];
+        const Stack::Packed P = s->packed.empty() ? Stack::Packed{} : s->packed[l];
         mark(KC_NORM_QKV);
-        if (pgk_status r = norm(L.norm1)) return r;
-        if (pgk_status r = pgk_gemm_nt(b.x, L.w_in, nullptr, b.in, n, L.n_in, s->Wp, DT, st)) return r;
+        if (pgk_status r = rows_norm(norm_args(s, b, n, *pend, L.norm1, b.x), n, DT, st)) return r;
+        if (pgk_status r = rows_in_proj<T>(s, L, P.in, b, n, st)) return r;
         mark(KC_ATTN);
         if (pgk_status r = mix(l)) return r;
         mark(KC_OPROJ);
-        if (pgk_status r = pgk_gemm_nt(b.a, L.w_o, nullptr, b.y, n, s->Wp, L.heads * L.head_pad, DT, st)) return r;
-        pend = L.norm1b;
+        if (pgk_status r = rows_out_proj<T>(s, b, b.a, L.w_o, P.o, n, L.heads * L.head_pad, &pend->slabs, st)) return r;
+        pend->gain = L.norm1b;
         if (!L.ff_pad) continue;
         mark(KC_GATEUP);
-        if (pgk_status r = norm(L.norm2)) return r;
-        if (pgk_status r = rows_mlp<T>(s, L, b, n, st)) return r;
-        pend = L.norm2b;
+        if (pgk_status r = rows_norm(norm_args(s, b, n, *pend, L.norm2, b.x), n, DT, st)) return r;
+        if (pgk_status r = rows_gate_up<T>(s, L, P.gate_up, b, n, st)) return r;
+        mark(KC_DOWN);
+        if (pgk_status r = rows_out_proj<T>(s, b, b.act, L.w_down, P.down, n, L.ff_pad, &pend->slabs, st)) return r;
+        pend->gain = L.norm2b;
     }
-    *pend_out = pend;
     return PGK_OK;
 }
 
@@ -703,16 +1002,15 @@ static pgk_status step_rows(Engine* e, int B, hipStream_t st, int* launches) {
     Stack* s = stack_of(e);
     constexpr pgk_dtype DT = std::is_same<T, float>::value ? PGK_F32 : PGK_BF16;
     const auto& c = s->cfg;
-    const RowBufs b{e->h, s->x16, s->in16, s->a16, s->y16, s->gu16, s->act16};
-    const float* pend = nullptr;
+    const RowBufs b{e->h, s->x16, s->in16, s->a16, s->y16, s->gu16, s->act16, s->slabs16};
+    Pending pend;
     if (pgk_status r = rows_layers<T>(s, b, B, st, &pend, [&](int l) { return latent_decode<T, T>(e, l, B, b.in, b.a, st, launches); })) return r;
     mark(KC_LMHEAD);
-    RowsNormArgs a{b.h, pend ? b.y : nullptr, s->Wp, pend, c.residual_mult, s->final_norm, b.x, c.width, s->Wp, c.norm_eps, nullptr, 1};
-    if (pgk_status r = rows_norm(a, B, DT, st)) return r;
+    if (pgk_status r = rows_norm(norm_args(s, b, B, pend, s->final_norm, b.x), B, DT, st)) return r;
     if (pgk_status r = head_rows<T>(s, (const T*)b.x, e->logits, B, st)) return r;
     PGK_CHECK_HIP(launch_k(rows_argmax_kernel, dim3(ROWS_ARGMAX_BLOCKS, B), dim3(256), 0, st, e->logits, c.vocab_size, e->amax_val, e->amax_idx));
     *launches += 3;
-    for (const auto& L : s->layers) *launches += 3 + (L.ff_pad ? 4 : 0);
+    for (const auto& L : s->layers) *launches += 3 + (L.ff_pad ? 3 : 0);     // (one more where a projection's slabs or SwiGLU take a launch of their own)
     return PGK_OK;
 }
 
@@ -820,7 +1118,8 @@ static pgk_status stack_prefill_t(Engine* e, int n_seqs, const int32_t* slots, c
     auto up = [](size_t v) { return (v + 255) & ~(size_t)255; };
     const size_t E = sizeof(T);
     const size_t sizes[] = {(size_t)n * s->Wp * 4, (size_t)n * s->Wp * E, (size_t)n * s->max_in * E, (size_t)n * s->max_att * E, (size_t)n * s->Wp * E,
-                            (size_t)n * 2 * s->max_ff * E, (size_t)n * s->max_ff * E, c_elems * E, kv_elems * E, (size_t)wrows * s->Wp * E, (size_t)wrows * c.vocab_size * 4};
+                            (size_t)n * 2 * s->max_ff * E, (size_t)n * s->max_ff * E, c_elems * E, kv_elems * E, (size_t)wrows * s->Wp * E, (size_t)wrows * c.vocab_size * 4,
+                            s->slab_elems(n, DT == PGK_F32) * 4};
     size_t need = 0;
     for (size_t z : sizes) need += up(z);
     const size_t tab_need = up((size_t)n * 4) * 2 + up(place.size() * sizeof(RowPlace)) + up((size_t)n_want * 4);
@@ -844,6 +1143,7 @@ static pgk_status stack_prefill_t(Engine* e, int n_seqs, const int32_t* slots, c
     T* kv = (T*)take(sizes[8]);
     void* xw = take(sizes[9]);
     float* lg = (float*)take(sizes[10]);
+    b.slabs = (float*)take(sizes[11]);
     // one host image of the index tables, one copy
     std::vector<char> img(tab_need, 0);
     const size_t o_pos = up((size_t)n * 4), o_place = 2 * o_pos, o_want = o_place + up(place.size() * sizeof(RowPlace));
@@ -886,12 +1186,14 @@ static pgk_status stack_prefill_t(Engine* e, int n_seqs, const int32_t* slots, c
         }
         return PGK_OK;
     };
-    const float* pend = nullptr;
+    Pending pend;
     if (pgk_status r = rows_layers<T>(s, b, n, st, &pend, mix)) return r;
     for (int i = 0; i < n_seqs; ++i) s->len[slots[i]] = starts[i] + lens[i];
     for (int w0 = 0; w0 < n_want; w0 += 128) {
         const int m = n_want - w0 < 128 ? n_want - w0 : 128;
-        RowsNormArgs a{b.h, pend ? b.y : nullptr, s->Wp, pend, c.residual_mult, s->final_norm, xw, c.width, s->Wp, c.norm_eps, d_want + w0, 0};
+        RowsNormArgs a = norm_args(s, b, n, pend, s->final_norm, xw);
+        a.rows = d_want + w0;
+        a.store_h = 0;                        // a wanted row may be asked for twice
         if (pgk_status r = rows_norm(a, m, DT, st)) return r;
         if (pgk_status r = head_rows<T>(s, (const T*)xw, lg, m, st)) return r;
         PGK_CHECK_HIP(hipMemcpyAsync(h_logits + (size_t)w0 * c.vocab_size, lg, (size_t)m * c.vocab_size * 4, hipMemcpyDeviceToHost, st));
@@ -1006,7 +1308,7 @@ pgk_status pgk_engine_create_stack(const pgk_stack_config_t* cfg, const void* em
     A((void**)&s->a32, (size_t)s->max_att * 4, &e->ws_bytes, true);     // padding columns of a head are never written: zero
     A((void**)&s->y32, (size_t)Wp * 4, &e->ws_bytes, true);
     A((void**)&s->act32, (size_t)(s->max_ff ? s->max_ff : 64) * 4, &e->ws_bytes);
-    A((void**)&s->qlat, ql * 4, &e->ws_bytes);
+    A(&s->qlat, ql * 4, &e->ws_bytes);
     A((void**)&s->po, part * 4, &e->ws_bytes);
     A((void**)&s->pml, ml * 4, &e->ws_bytes);
     A(&s->x16, B * Wp * E, &e->ws_bytes);
@@ -1015,6 +1317,35 @@ pgk_status pgk_engine_create_stack(const pgk_stack_config_t* cfg, const void* em
     A(&s->y16, B * Wp * E, &e->ws_bytes);
     A(&s->gu16, B * 2 * (s->max_ff ? s->max_ff : 64) * E, &e->ws_bytes);
     A(&s->act16, B * (s->max_ff ? s->max_ff : 64) * E, &e->ws_bytes);
+    if (r == PGK_OK && c.dtype == PGK_BF16) {
+        // a second, fragment-major copy of the layer matrices where the skinny GEMM takes their shapes, unless that is more than a
+        // quarter of the free memory; PGK_PACKED_PREFILL=0: none
+        hipStream_t st = resolve_stream(nullptr);
+        const char* ep = getenv("PGK_PACKED_PREFILL");
+        size_t total = 0, free_b = 0, total_b = 0;
+        auto visit = [&](auto fn) {
+            for (int l = 0; l < c.num_layers; ++l) {
+                const auto& L = s->layers[l];
+                const int HD = L.heads * L.head_pad;
+                auto& P = s->packed[l];
+                if (pkgemm_shape_ok(L.n_in, Wp, false)) fn(&P.in, L.w_in, L.n_in, Wp);
+                if (pkgemm_shape_ok(Wp, HD, true)) fn(&P.o, L.w_o, Wp, HD);
+                if (!L.ff_pad) continue;
+                if (pkgemm_shape_ok(2 * L.ff_pad, Wp, false)) fn(&P.gate_up, L.w_gate_up, 2 * L.ff_pad, Wp);
+                if (pkgemm_shape_ok(Wp, L.ff_pad, true)) fn(&P.down, L.w_down, Wp, L.ff_pad);
+            }
+        };
+        s->packed.resize(c.num_layers);
+        visit([&](bf16**, const void*, int N, int K) { total += (size_t)N * K * 2; });
+        if (!(ep && atoi(ep) == 0) && hipMemGetInfo(&free_b, &total_b) == hipSuccess && total < free_b / 4)
+            visit([&](bf16** dst, const void* w, int N, int K) {
+                A((void**)dst, (size_t)N * K * 2, &e->packed_bytes);
+                if (r == PGK_OK) r = pack_weights_bf16(w, *dst, N, K, st);
+            });
+    }
+    size_t slab = 64;
+    for (int m = 2; m <= c.max_batch; ++m) { const size_t z = s->slab_elems(m, c.dtype == PGK_F32); slab = z > slab ? z : slab; }
+    A((void**)&s->slabs16, slab * 4, &e->ws_bytes);
     if (r == PGK_OK) {
         hipStream_t st = resolve_stream(nullptr);
         hipError_t he = hipSuccess;

@@ -35,6 +35,8 @@ struct RowsNormArgs {
     float eps;
     const int32_t* rows;
     int store_h;
+    int nslabs;               // > 0: y is fp32 split-K slabs, slab i at y + i * slab_stride (elements); the sublayer output is their sum
+    long long slab_stride;
 };
 pgk_status rows_norm(const RowsNormArgs& a, int n, pgk_dtype dt, hipStream_t st);
 

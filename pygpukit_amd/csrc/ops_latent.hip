@@ -26,6 +26,21 @@ __global__ __launch_bounds__(256) void rows_norm_kernel(RowsNormArgs a) {
         for (int t = 0; t < NT; ++t) {
             const int i = (threadIdx.x + 256 * t) * 4;
             y[t] = i < nt ? load4<YT>(yr + i) : make_float4(0.f, 0.f, 0.f, 0.f);
+        }
+        if constexpr (std::is_same<YT, float>::value) {
+#pragma unroll 4
+            for (int s = 1; s < a.nslabs; ++s)
+#pragma unroll
+                for (int t = 0; t < NT; ++t) {
+                    const int i = (threadIdx.x + 256 * t) * 4;
+                    if (i < nt) {
+                        const float4 q = load4<float>(reinterpret_cast<const float*>(yr) + s * a.slab_stride + i);
+                        y[t].x += q.x; y[t].y += q.y; y[t].z += q.z; y[t].w += q.w;
+                    }
+                }
+        }
+#pragma unroll
+        for (int t = 0; t < NT; ++t) {
             ss += y[t].x * y[t].x + y[t].y * y[t].y + y[t].z * y[t].z + y[t].w * y[t].w;
         }
         ss = block_sum(ss, red);
@@ -71,7 +86,7 @@ static pgk_status rows_norm_t(const RowsNormArgs& a, int n, hipStream_t st) {
 }
 
 pgk_status rows_norm(const RowsNormArgs& a, int n, pgk_dtype dt, hipStream_t st) {
-    if (dt == PGK_BF16) return rows_norm_t<bf16, bf16>(a, n, st);
+    if (dt == PGK_BF16) return a.nslabs > 0 ? rows_norm_t<bf16, float>(a, n, st) : rows_norm_t<bf16, bf16>(a, n, st);
     if (dt == PGK_F32) return rows_norm_t<float, float>(a, n, st);
     return set_error(PGK_ERR_UNSUPPORTED, "rows_norm: dtype %d", (int)dt);
 }
