@@ -266,7 +266,7 @@ struct LatentArgs {
     const float* c_norm;      // [rank]
     void* cache;              // [slots][R][rank] (T)
     const int32_t* positions; // [B]
-    int B, H, D, dim, vdim, rank, rank_true, R, nsplit;
+    int B, H, D, dim, vdim, rank, rank_true, R, nsplit, vc;
     float eps, scale;         // scale already times log2e
     void* qlat;               // [B][H][rank], float or bf16
     float* po;                // [B][H][nsplit][rank]
@@ -467,19 +467,27 @@ __global__ __launch_bounds__(256) void latent_attn_mfma_kernel(unsigned long lon
     }
     const bf16* cb = reinterpret_cast<const bf16*>(a.cache) + (size_t)b * a.R * a.rank;
     const bf16* qb = reinterpret_cast<const bf16*>(a.qlat) + (size_t)b * a.H * a.rank;
-    for (int c = tid; c < 16 * nch; c += 256) {
-        const int r = c / nch, k = c % nch;
-        *reinterpret_cast<uint4*>(qs + r * ld + k * 8) = *reinterpret_cast<const uint4*>(qb + (size_t)min(h0 + r, a.H - 1) * a.rank + k * 8);
-    }
+    // 16-byte pieces of the query block and of a key tile, all requested before the first is stored.  LPR lanes per row (a power of
+    // two: no division), lanes past a row's end repeat its last piece.
+    constexpr int LPR = RT >= 8 ? 64 : 8 * RT, HALF = RT > 8 ? 2 : 1, RPP = 256 / LPR, QN = (RPP >= 16 ? 1 : 16 / RPP) * HALF, CN = 64 / RPP * HALF;
+    const int r_in = tid / LPR, k_in = tid % LPR;
+    auto q_row = [&](int i) { return min(i / HALF * RPP + r_in, 15); };
+    auto col = [&](int i) { return min(k_in + (i % HALF) * LPR, nch - 1) * 8; };
+    u32x4 qv[QN], cv[CN];                                         // (vector type: a uint4 array carried around the loop is left in scratch memory)
+#pragma unroll
+    for (int i = 0; i < QN; ++i) qv[i] = *reinterpret_cast<const u32x4*>(qb + (size_t)(min(h0 + q_row(i), a.H - 1) * a.rank + col(i)));
+#pragma unroll
+    for (int i = 0; i < CN; ++i) cv[i] = *reinterpret_cast<const u32x4*>(cb + (size_t)(min(k0 + i / HALF * RPP + r_in, k1 - 1) * a.rank + col(i)));
+#pragma unroll
+    for (int i = 0; i < QN; ++i) *reinterpret_cast<u32x4*>(qs + q_row(i) * ld + col(i)) = qv[i];
     for (int kt = k0; kt < k1; kt += 64) {
-        const int rt = k1 - kt > 32 ? 64 : 32;                    // rows of this tile that are staged
+        const int rt = k1 - kt > 32 ? 64 : 32;                    // rows of this tile that take part (the rest repeat the last key)
         if (kt != k0) __syncthreads();                            // the last step's reads of cs are done
-#pragma unroll 8
-        for (int c = tid; c < rt * nch; c += 256) {
-            const int r = c / nch, k = c % nch;
-            *reinterpret_cast<uint4*>(cs + r * ld + k * 8) = *reinterpret_cast<const uint4*>(cb + (size_t)min(kt + r, k1 - 1) * a.rank + k * 8);
-        }
+#pragma unroll
+        for (int i = 0; i < CN; ++i) *reinterpret_cast<u32x4*>(cs + (i / HALF * RPP + r_in) * ld + col(i)) = cv[i];
         __syncthreads();
+#pragma unroll
+        for (int i = 0; i < CN; ++i) cv[i] = *reinterpret_cast<const u32x4*>(cb + (size_t)(min(kt + 64 + i / HALF * RPP + r_in, k1 - 1) * a.rank + col(i)));     // the next tile travels under this one's products
         f32x4_st sc = {-INFINITY, -INFINITY, -INFINITY, -INFINITY};
         const bool mine = 16 * wid < rt;                          // wave-uniform
         if (mine) {
@@ -553,7 +561,7 @@ __global__ __launch_bounds__(256) void latent_attn_mfma_kernel(unsigned long lon
     tls.end();
 }
 
-// Combine the split records of (sequence, head), apply U_v (the workgroup's 32 rows) and the head's gate.  The waves share the splits,
+// Combine the split records of (sequence, head), apply U_v (the workgroup's vc runs of 32 rows) and the head's gate.  The waves share the splits,
 // then meet in LDS; a row of U_v is 16 lanes wide, requested before the records when the rank allows (PF 128-column pieces per row).
 template <class T, class IT, int MB, int PF>
 __global__ __launch_bounds__(256) void latent_merge_uv_kernel(unsigned long long* tl, LatentArgs a) {
@@ -561,7 +569,8 @@ __global__ __launch_bounds__(256) void latent_merge_uv_kernel(unsigned long long
     extern __shared__ __attribute__((aligned(16))) float ol[];     // [4][MB][rank]; afterwards [MB][rank]
     __shared__ float sw[MB][64];
     constexpr int NW = WTraits<T>::NW;
-    const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6, h = blockIdx.x, v0 = blockIdx.y * 32, b0 = blockIdx.z * MB, sub = lane & 15, grp = lane >> 4;
+    const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6, h = blockIdx.x, b0 = blockIdx.z * MB, sub = lane & 15, grp = lane >> 4;
+    int v0 = blockIdx.y * 32 * a.vc;
     const T* u = reinterpret_cast<const T*>(a.w_uv) + (size_t)h * a.D * a.rank;
     uint4 w[2][PF > 0 ? PF : 1];
     if constexpr (PF > 0) {
@@ -579,19 +588,37 @@ __global__ __launch_bounds__(256) void latent_merge_uv_kernel(unsigned long long
         sw[m][lane] = f / den;
     }
     __syncthreads();
+    int nact[MB];
 #pragma unroll
     for (int m = 0; m < MB; ++m) {
-        const int b = min(b0 + m, a.B - 1), n = min(max(a.positions[b], 0) + 1, a.R), per = split_rows(n, a.nsplit), nact = (n + per - 1) / per;
-        const float* rec = a.po + ((size_t)b * a.H + h) * a.nsplit * a.rank;
-        for (int r = 4 * lane; r < a.rank; r += 256) {
-            float4 t = {0.f, 0.f, 0.f, 0.f};
-#pragma unroll 8
-            for (int s = wid; s < nact; s += 4) {
-                const float f = sw[m][s];
-                const float4 p = *reinterpret_cast<const float4*>(rec + (size_t)s * a.rank + r);
-                t.x = fmaf(f, p.x, t.x); t.y = fmaf(f, p.y, t.y); t.z = fmaf(f, p.z, t.z); t.w = fmaf(f, p.w, t.w);
-            }
-            *reinterpret_cast<float4*>(ol + ((size_t)wid * MB + m) * a.rank + r) = t;
+        const int n = min(max(a.positions[min(b0 + m, a.B - 1)], 0) + 1, a.R), per = split_rows(n, a.nsplit);
+        nact[m] = (n + per - 1) / per;
+    }
+    for (int r0 = 0; r0 < a.rank; r0 += 256) {
+        const int r = r0 + 4 * lane, rc = min(r, a.rank - 4);
+        float4 t[MB];
+        constexpr int SU = MB == 1 ? 8 : 4;                        // records in flight per sequence: clamped loads, weight 0 beyond the last
+        int most = 0;
+#pragma unroll
+        for (int m = 0; m < MB; ++m) { t[m] = make_float4(0.f, 0.f, 0.f, 0.f); most = max(most, nact[m]); }
+        for (int s0 = wid; s0 < most; s0 += 4 * SU) {
+            float4 p[MB][SU];
+#pragma unroll
+            for (int m = 0; m < MB; ++m)
+#pragma unroll
+                for (int k = 0; k < SU; ++k)
+                    p[m][k] = *reinterpret_cast<const float4*>(a.po + (((size_t)min(b0 + m, a.B - 1) * a.H + h) * a.nsplit + min(s0 + 4 * k, nact[m] - 1)) * a.rank + rc);
+#pragma unroll
+            for (int m = 0; m < MB; ++m)
+#pragma unroll
+                for (int k = 0; k < SU; ++k) {
+                    const float f = s0 + 4 * k < nact[m] ? sw[m][s0 + 4 * k] : 0.f;
+                    t[m].x = fmaf(f, p[m][k].x, t[m].x); t[m].y = fmaf(f, p[m][k].y, t[m].y); t[m].z = fmaf(f, p[m][k].z, t[m].z); t[m].w = fmaf(f, p[m][k].w, t[m].w);
+                }
+        }
+        if (r < a.rank) {
+#pragma unroll
+            for (int m = 0; m < MB; ++m) *reinterpret_cast<float4*>(ol + ((size_t)wid * MB + m) * a.rank + r) = t[m];
         }
     }
     __syncthreads();
@@ -606,36 +633,48 @@ __global__ __launch_bounds__(256) void latent_merge_uv_kernel(unsigned long long
         *reinterpret_cast<float4*>(ol + i) = t;
     }
     __syncthreads();
-#pragma unroll
-    for (int p = 0; p < 2; ++p) {
-        const int v = v0 + 8 * wid + 4 * p + grp;
-        float acc[MB];
-#pragma unroll
-        for (int m = 0; m < MB; ++m) acc[m] = 0.f;
-        auto piece = [&](const uint4& raw, int r) {
-            float f[NW];
-            WTraits<T>::decode(raw, f);
-#pragma unroll
-            for (int m = 0; m < MB; ++m)
-#pragma unroll
-                for (int j = 0; j < NW; j += 4) {
-                    const float4 x = *reinterpret_cast<const float4*>(ol + m * a.rank + r + j);
-                    acc[m] = fmaf(f[j + 3], x.w, fmaf(f[j + 2], x.z, fmaf(f[j + 1], x.y, fmaf(f[j], x.x, acc[m]))));
-                }
-        };
+    for (int c = 0; c < a.vc; ++c, v0 += 32) {
+        if (v0 >= a.vdim) break;                                   // block-uniform
         if constexpr (PF > 0) {
+            if (c > 0) {
 #pragma unroll
-            for (int k = 0; k < PF; ++k) { const int r = 16 * NW * k + sub * NW; if (r < a.rank) piece(w[p][k], r); }
-        } else {
-            const T* row = u + (size_t)min(v, a.vdim - 1) * a.rank;
-            for (int r = sub * NW; r < a.rank; r += 16 * NW) piece(*reinterpret_cast<const uint4*>(row + r), r);
+                for (int p = 0; p < 2; ++p)
+#pragma unroll
+                    for (int k = 0; k < PF; ++k)
+                        w[p][k] = *reinterpret_cast<const uint4*>(u + (size_t)min(v0 + 8 * wid + 4 * p + grp, a.vdim - 1) * a.rank + min(16 * NW * k + sub * NW, a.rank - NW));
+            }
         }
 #pragma unroll
-        for (int m = 0; m < MB; ++m) {
-            const float y = group16_sum(acc[m]);
-            if (sub == 0 && v < a.vdim && b0 + m < a.B) {
-                const float g = to_f(reinterpret_cast<const IT*>(a.in)[(size_t)(b0 + m) * a.ld_in + a.g_off + h]);
-                reinterpret_cast<IT*>(a.out)[(size_t)(b0 + m) * a.ld_out + h * a.D + v] = from_f<IT>(y / (1.0f + expf(-g)));
+        for (int p = 0; p < 2; ++p) {
+            const int v = v0 + 8 * wid + 4 * p + grp;
+            float acc[MB];
+#pragma unroll
+            for (int m = 0; m < MB; ++m) acc[m] = 0.f;
+            auto piece = [&](const uint4& raw, int r) {
+                float f[NW];
+                WTraits<T>::decode(raw, f);
+#pragma unroll
+                for (int m = 0; m < MB; ++m)
+#pragma unroll
+                    for (int j = 0; j < NW; j += 4) {
+                        const float4 x = *reinterpret_cast<const float4*>(ol + m * a.rank + r + j);
+                        acc[m] = fmaf(f[j + 3], x.w, fmaf(f[j + 2], x.z, fmaf(f[j + 1], x.y, fmaf(f[j], x.x, acc[m]))));
+                    }
+            };
+            if constexpr (PF > 0) {
+#pragma unroll
+                for (int k = 0; k < PF; ++k) { const int r = 16 * NW * k + sub * NW; if (r < a.rank) piece(w[p][k], r); }
+            } else {
+                const T* row = u + (size_t)min(v, a.vdim - 1) * a.rank;
+                for (int r = sub * NW; r < a.rank; r += 16 * NW) piece(*reinterpret_cast<const uint4*>(row + r), r);
+            }
+#pragma unroll
+            for (int m = 0; m < MB; ++m) {
+                const float y = group16_sum(acc[m]);
+                if (sub == 0 && v < a.vdim && b0 + m < a.B) {
+                    const float g = to_f(reinterpret_cast<const IT*>(a.in)[(size_t)(b0 + m) * a.ld_in + a.g_off + h]);
+                    reinterpret_cast<IT*>(a.out)[(size_t)(b0 + m) * a.ld_out + h * a.D + v] = from_f<IT>(y / (1.0f + expf(-g)));
+                }
             }
         }
     }
@@ -734,8 +773,8 @@ static Stack* stack_of(const Engine* e) { return (Stack*)e->kind_state; }
 
 static int pick_nsplit(const Engine* e, int B, const pgk_stack_layer_t& L, int R) {
     const int htiles = ceil_div(L.heads, 16);
-    int s = ceil_div(R, 32);
-    const int want = 2 * e->cu_count / (B * htiles) > 0 ? 2 * e->cu_count / (B * htiles) : 1;
+    int s = ceil_div(R, 64);
+    const int want = e->cu_count / (B * htiles) > 0 ? e->cu_count / (B * htiles) : 1;      // one workgroup per CU (its LDS)
     if (s > want) s = want;
     return s > 64 ? 64 : (s < 1 ? 1 : s);
 }
@@ -765,7 +804,7 @@ static hipError_t launch_merge_uv(const LatentArgs& a, hipStream_t st) {
     const size_t lds = (size_t)4 * MB * a.rank * 4;
     auto kfn = &latent_merge_uv_kernel<T, IT, MB, PF>;
     PGK_ALLOW_LDS(kfn, lds)
-    return launch_k(kfn, dim3(a.H, ceil_div(a.vdim, 32), ceil_div(a.B, MB)), dim3(256), lds, st, a);
+    return launch_k(kfn, dim3(a.H, ceil_div(a.vdim, 32 * a.vc), ceil_div(a.B, MB)), dim3(256), lds, st, a);
 }
 template <class T, class IT, class QT, int MB>
 static hipError_t launch_absorb(const LatentArgs& a, hipStream_t st) {
@@ -784,6 +823,7 @@ static pgk_status latent_decode(Engine* e, int l, int B, const void* in, void* o
     a.c_norm = L.c_norm; a.cache = s->cache[l]; a.positions = e->positions;
     a.B = B; a.H = L.heads; a.D = L.head_pad; a.dim = L.dim; a.vdim = L.vdim; a.rank = L.rank_pad; a.rank_true = L.rank; a.R = s->ring[l];
     a.nsplit = pick_nsplit(e, B, L, a.R);
+    a.vc = B >= 16 ? 4 : 1;      // many sequences: fewer workgroups, each combines its records once for all its rows
     a.eps = s->cfg.norm_eps; a.scale = L.scale * LOG2E;
     a.qlat = s->qlat; a.po = s->po; a.pml = s->pml; a.out = out; a.ld_out = L.heads * L.head_pad;
     const bool mfma = !F32 && a.rank <= 896;
@@ -798,7 +838,7 @@ static pgk_status latent_decode(Engine* e, int l, int B, const void* in, void* o
     }
     if constexpr (!F32) {
         if (mfma) {
-            PGK_CHECK_HIP((B == 1 ? launch_absorb<T, IT, bf16, 1>(a, st) : launch_absorb<T, IT, bf16, 8>(a, st)));
+            PGK_CHECK_HIP((B == 1 ? launch_absorb<T, IT, bf16, 1>(a, st) : B < 32 ? launch_absorb<T, IT, bf16, 4>(a, st) : launch_absorb<T, IT, bf16, 8>(a, st)));
             if (a.rank <= 64) PGK_CHECK_HIP(launch_latent_mfma<1>(a, st));
             else if (a.rank <= 128) PGK_CHECK_HIP(launch_latent_mfma<2>(a, st));
             else if (a.rank <= 256) PGK_CHECK_HIP(launch_latent_mfma<4>(a, st));
@@ -807,10 +847,10 @@ static pgk_status latent_decode(Engine* e, int l, int B, const void* in, void* o
         }
     }
     if constexpr (!F32) {
-        if (a.rank <= 256) PGK_CHECK_HIP((B == 1 ? launch_merge_uv<T, IT, 1, 2>(a, st) : launch_merge_uv<T, IT, 4, 2>(a, st)));
-        else if (a.rank <= 512) PGK_CHECK_HIP((B == 1 ? launch_merge_uv<T, IT, 1, 4>(a, st) : launch_merge_uv<T, IT, 4, 4>(a, st)));
-        else PGK_CHECK_HIP((B == 1 ? launch_merge_uv<T, IT, 1, 0>(a, st) : launch_merge_uv<T, IT, 4, 0>(a, st)));
-    } else PGK_CHECK_HIP((B == 1 ? launch_merge_uv<T, IT, 1, 0>(a, st) : launch_merge_uv<T, IT, 4, 0>(a, st)));
+        if (a.rank <= 256) PGK_CHECK_HIP((B < 16 ? launch_merge_uv<T, IT, 1, 2>(a, st) : launch_merge_uv<T, IT, 4, 2>(a, st)));
+        else if (a.rank <= 512) PGK_CHECK_HIP((B < 16 ? launch_merge_uv<T, IT, 1, 4>(a, st) : launch_merge_uv<T, IT, 4, 4>(a, st)));
+        else PGK_CHECK_HIP((B < 16 ? launch_merge_uv<T, IT, 1, 0>(a, st) : launch_merge_uv<T, IT, 4, 0>(a, st)));
+    } else PGK_CHECK_HIP((B < 16 ? launch_merge_uv<T, IT, 1, 0>(a, st) : launch_merge_uv<T, IT, 4, 0>(a, st)));
     *launches += 3;
     return PGK_OK;
 }

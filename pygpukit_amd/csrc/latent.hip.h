@@ -48,4 +48,8 @@ pgk_status flash_window(const void* q, const void* k, const void* v, void* out, 
                         int window, const void* gate, long long gs, long long qh, long long qs, long long kh, long long ks, long long oh,
                         long long os, hipStream_t st);   // ops_flash.hip
 
+// ops_attention.hip: kv_len <= 128, head width 128, plain causal mask, bf16
+pgk_status attn_short_gated(const void* q, const void* k, const void* v, void* out, int hq, int hkv, int q_len, int kv_len, float scale, const WindowStrides& sd,
+                            const void* gate, long long gs, hipStream_t st);
+
 }  // namespace pgk

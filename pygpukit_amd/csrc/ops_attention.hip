@@ -13,6 +13,7 @@
 #include <cstring>
 
 #include "attn_core.hip.h"
+#include "latent.hip.h"
 #include "pgk_internal.h"
 
 namespace pgk {
@@ -194,7 +195,8 @@ __device__ __forceinline__ int sa_voff(int row, int ch) { return row * 256 + ((c
 
 template <int NW>
 __global__ __launch_bounds__(64 * NW) void attn_short_kernel(const bf16* q, const bf16* k, const bf16* v, bf16* out, int hq, int hkv,
-                                                             int q_len, int kv_len, float scale, AttnStrides sd) {
+                                                             int q_len, int kv_len, float scale, AttnStrides sd, const bf16* gate = nullptr,
+                                                             long long gs = 0) {      // gate: see attn_short_gated
     constexpr int D = 128, NT = 8;
     __shared__ __attribute__((aligned(16))) char k_lds[128 * 256];
     __shared__ __attribute__((aligned(16))) char v_lds[128 * 256];
@@ -302,7 +304,8 @@ __global__ __launch_bounds__(64 * NW) void attn_short_kernel(const bf16* q, cons
         }
     }
     if (qrow < q_len) {
-        const float inv = ls > 0.f ? 1.f / ls : 0.f;
+        float inv = ls > 0.f ? 1.f / ls : 0.f;
+        if (gate) inv /= 1.0f + __expf(-to_f(gate[(long long)qrow * gs + head]));
         bf16* op = out + (size_t)head * sd.oh + (size_t)qrow * sd.os + 4 * q4;
 #pragma unroll
         for (int i = 0; i < D / 16; ++i) {
@@ -402,6 +405,17 @@ static pgk_status launch_prefill(const T* q, const T* k, const T* v, T* out, int
                                  float scale, const AttnStrides& sd, hipStream_t st) {
     dim3 grid(ceil_div(q_len, FA_BQ), hq);
     flash_prefill_kernel<T, D><<<grid, 256, 0, st>>>(q, k, v, out, hq, hkv, q_len, kv_len, scale, sd);
+    PGK_CHECK_HIP(hipGetLastError());
+    return PGK_OK;
+}
+
+// attn_short_kernel with a gate per (query row, head): the head's output row times sigmoid(gate[row * gs + head]) (null: none)
+pgk_status attn_short_gated(const void* q, const void* k, const void* v, void* out, int hq, int hkv, int q_len, int kv_len, float scale, const WindowStrides& w,
+                            const void* gate, long long gs, hipStream_t st) {
+    PGK_REQUIRE(kv_len <= 128 && kv_len >= q_len && w.kh == w.vh && w.ks == w.vs, "attn_short_gated: q_len=%d kv_len=%d", q_len, kv_len);
+    const AttnStrides sd{w.qh, w.qs, w.kh, w.ks, w.oh, w.os};
+    attn_short_kernel<2><<<dim3(ceil_div(q_len, 32), hq), 128, 0, st>>>((const bf16*)q, (const bf16*)k, (const bf16*)v, (bf16*)out, hq, hkv, q_len, kv_len, scale, sd,
+                                                                      (const bf16*)gate, gs);
     PGK_CHECK_HIP(hipGetLastError());
     return PGK_OK;
 }

@@ -28,16 +28,25 @@ __global__ __launch_bounds__(256) void rows_norm_kernel(RowsNormArgs a) {
             y[t] = i < nt ? load4<YT>(yr + i) : make_float4(0.f, 0.f, 0.f, 0.f);
         }
         if constexpr (std::is_same<YT, float>::value) {
-#pragma unroll 4
-            for (int s = 1; s < a.nslabs; ++s)
+            constexpr int SU = NT <= 4 ? 16 / NT : 2;      // slabs in flight: unconditional loads (clamped), masked adds
+            for (int s0 = 1; s0 < a.nslabs; s0 += SU) {
+                float4 q[SU][NT];
 #pragma unroll
-                for (int t = 0; t < NT; ++t) {
-                    const int i = (threadIdx.x + 256 * t) * 4;
-                    if (i < nt) {
-                        const float4 q = load4<float>(reinterpret_cast<const float*>(yr) + s * a.slab_stride + i);
-                        y[t].x += q.x; y[t].y += q.y; y[t].z += q.z; y[t].w += q.w;
+                for (int s = 0; s < SU; ++s)
+#pragma unroll
+                    for (int t = 0; t < NT; ++t)
+                        q[s][t] = load4<float>(reinterpret_cast<const float*>(yr) + min(s0 + s, a.nslabs - 1) * a.slab_stride + min((int)(threadIdx.x + 256 * t) * 4, nt - 4));
+#pragma unroll
+                for (int s = 0; s < SU; ++s) {
+                    const float w = s0 + s < a.nslabs ? 1.f : 0.f;
+#pragma unroll
+                    for (int t = 0; t < NT; ++t) {
+                        const float m = (int)(threadIdx.x + 256 * t) * 4 < nt ? w : 0.f;
+                        y[t].x = fmaf(m, q[s][t].x, y[t].x); y[t].y = fmaf(m, q[s][t].y, y[t].y);
+                        y[t].z = fmaf(m, q[s][t].z, y[t].z); y[t].w = fmaf(m, q[s][t].w, y[t].w);
                     }
                 }
+            }
         }
 #pragma unroll
         for (int t = 0; t < NT; ++t) {
@@ -185,6 +194,8 @@ pgk_status window_attention(const void* q, const void* k, const void* v, void* o
                             int window, const WindowStrides& sd, const void* gate, long long gs, pgk_dtype dt, hipStream_t st) {
     const bool flash = dt == PGK_BF16 && dk == dv && (dk == 64 || dk == 128) && scale > 0.f && sd.kh == sd.vh && sd.ks == sd.vs && aligned16(q) && aligned16(k) && aligned16(v) &&
                        sd.qs % 8 == 0 && sd.qh % 8 == 0 && sd.ks % 8 == 0 && sd.kh % 8 == 0 && (reinterpret_cast<uintptr_t>(out) & 7u) == 0 && sd.os % 4 == 0 && sd.oh % 4 == 0;
+    // the whole context in one tile and inside every query's window
+    if (flash && dk == 128 && kv_len <= 128 && window >= kv_len) return attn_short_gated(q, k, v, out, hq, hkv, q_len, kv_len, scale, sd, gate, gs, st);
     if (flash) return flash_window(q, k, v, out, hq, hkv, q_len, kv_len, dk, scale, window, gate, gs, sd.qh, sd.qs, sd.kh, sd.ks, sd.oh, sd.os, st);
     const size_t lds = ((size_t)dk + 4 * (size_t)dv + 4 * 64 + 8) * 4;
     PGK_REQUIRE(lds <= 64 * 1024, "window_attention: head widths %d / %d do not fit LDS", dk, dv);
