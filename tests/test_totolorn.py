@@ -39,6 +39,12 @@ CONFIGS = {
     # head width above 128 (no MFMA prompt kernel) and a latent above 512
     "wide": config(192, 130, [(mixer(3, 144, 72, 520, 20, 0.15), 128), (mixer(2, 136, 160, 64, 70, 0.12), None)], 160, 1e-5, 0.8),
     # widths the engine takes without padding, 16 and 20 heads, windows around the 64-key tiles of the prompt kernel
+    # long rows (every preload depth of the one-row projection, split-K slabs) and latents past each width class of the decode kernels
+    "long": config(1100, 120, [(mixer(2, 30, 30, 30, 50, 0.3), 4200), (mixer(2, 20, 64, 1000, 9, 0.4), 2100)], 320, 1e-5, 0.9),
+    "widest": config(4200, 50, [(mixer(3, 64, 64, 2000, 30, 0.2), 70)], 170),
+    "middle": config(2100, 50, [(mixer(2, 64, 64, 300, 30, 0.2), None)], 170),
+    # many heads and a window of several hundred: several key tiles per split
+    "deep": config(64, 90, [(mixer(17, 32, 128, 256, 600, 0.3), 64), (mixer(33, 16, 48, 70, 1000, 0.4), None)], 720),
     "tiles": config(128, 256, [(mixer(16, 64, 64, 128, 65, 0.3), 256), (mixer(20, 128, 128, 192, 64, 0.2), 192), (mixer(4, 64, 48, 64, 127, 0.3), 64)], 700),
 }
 
@@ -252,7 +258,8 @@ def test_head_gate_and_pad(dtype):
 @gpu
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
 @pytest.mark.parametrize("heads,dk,dv", [(2, 64, 64), (3, 128, 128), (2, 20, 36), (1, 200, 64)])
-@pytest.mark.parametrize("q_len,kv_len,window", [(1, 1, 1), (5, 5, 2), (130, 130, 1), (200, 333, 64), (70, 300, 65), (129, 257, 63), (300, 300, 1000), (2, 400, 129)])
+@pytest.mark.parametrize("q_len,kv_len,window", [(1, 1, 1), (5, 5, 2), (130, 130, 1), (200, 333, 64), (70, 300, 65), (129, 257, 63), (300, 300, 1000), (2, 400, 129),
+                                                 (100, 128, 500), (128, 128, 128), (30, 90, 90)])
 def test_window_attention(heads, dk, dv, q_len, kv_len, window, dtype):
     from pygpukit_amd.ops.basic import window_attention
 
@@ -446,6 +453,43 @@ def test_unequal_batch_and_slots_used_again(models, name, dtype):
         for i in live:
             s.release((round_, i))
     assert s.live == ()
+
+
+@gpu
+@both
+@pytest.mark.parametrize("batch", [1, 2, 17, 40])
+def test_deep_windows_in_batches(models, dtype, batch):
+    """Sequences around and beyond a 600-key window, in batch sizes that give a split one key tile and several."""
+    cfg, W, model = models("deep", dtype)
+    n = 700
+    t, want = reference("deep", n)
+    e = model.build_engine(max_seq_len=720, max_batch=batch)
+    at = [(590 + 13 * b) % 690 + 1 if b < 8 else 1 + (37 * b) % 680 for b in range(batch)]
+    e.prefill_batch([t[:p] for p in at], want=[[]] * batch)
+    worst = 0.0
+    for i in range(6):
+        e.set_state([t[p + i] for p in at], [p + i for p in at])
+        e.decode_step(batch)
+        worst = max(worst, logit_err(e.logits(batch).to_numpy(), want[[p + i for p in at]]))
+    assert worst < TOL[dtype]
+
+
+@gpu
+@pytest.mark.parametrize("packed", ["0", "1"])
+@pytest.mark.parametrize("name", ["long", "tiles"])
+def test_projection_routes_agree(models, name, packed, monkeypatch):
+    """Fragment-major copies on and off: prompts of 2..300 rows and batches take other kernels, the logits stay the same."""
+    monkeypatch.setenv("PGK_PACKED_PREFILL", packed)
+    cfg, W, model = models(name, "bfloat16")
+    t, want = reference(name, 300)
+    e = model.build_engine(max_seq_len=310, max_batch=12)
+    for n in (2, 20, 100, 128, 129, 300):
+        assert logit_err(e.prefill_batch([t[:n]], want=[[0, n // 2, n - 1]]), want[[0, n // 2, n - 1]]) < TOL["bfloat16"]
+    at = [3 * b + 1 for b in range(12)]
+    e.prefill_batch([t[:p] for p in at], want=[[]] * 12)
+    e.set_state([t[p] for p in at], at)
+    e.decode_step(12)
+    assert logit_err(e.logits(12).to_numpy(), want[at]) < TOL["bfloat16"]
 
 
 @gpu
