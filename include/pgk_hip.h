@@ -101,7 +101,7 @@ pgk_status pgk_memset(void* dst, int value, size_t nbytes, pgk_stream stream);
 pgk_status pgk_fill(void* dst, double value, size_t n, pgk_dtype dt, pgk_stream stream); /* ones() */
 
 /* ------------------------------------------------------- streams / events / graphs -- */
-/* Stream(priority) native/core/stream.hpp:21-35 */
+/* Stream(priority) native/core/stream.hpp:21-35; every stream is created at the default priority, `high_priority` is ignored */
 pgk_status pgk_stream_create(pgk_stream* out, int high_priority);
 pgk_status pgk_stream_destroy(pgk_stream s);
 pgk_status pgk_stream_sync(pgk_stream s);
