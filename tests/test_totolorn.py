@@ -114,7 +114,7 @@ def test_config_is_read_layer_by_layer():
 
 def test_oracle_mechanisms_on_hand_made_numbers():
     x = np.array([[3.0, 4.0]])
-    np.testing.assert_allclose(R.norm_aturnzero(x, np.array([0.0, 1.0]), 0.0), x / np.sqrt(12.5) * [1.0, 2.0])
+    np.testing.assert_allclose(R.norm_around_zero(x, np.array([0.0, 1.0]), 0.0), x / np.sqrt(12.5) * [1.0, 2.0])
     np.testing.assert_array_equal(R.window_mask(4, 2), [[1, 0, 0, 0], [1, 1, 0, 0], [0, 1, 1, 0], [0, 0, 1, 1]])
     v = np.arange(5.0)[:, None, None]
     assert R.attend(np.zeros((5, 1, 2)), np.zeros((5, 1, 2)), v, 1.0, 3)[4, 0, 0] == 3.0           # mean of the last three values
@@ -230,11 +230,11 @@ def test_stream_norms(rows, cols, dtype):
     x, y, w = rng.standard_normal((rows, cols)), rounded(rng.standard_normal((rows, cols)) * 3, dtype), rng.standard_normal(cols)
     x, w = x.astype(np.float32), w.astype(np.float32)
     got = host(rmsnorm_f32(dev(x, "float32"), dev(w, "float32"), 1e-3, dtype=DataType.from_string(dtype)))
-    want = R.norm_aturnzero(x.astype(np.float64), w - 1.0, 1e-3)
+    want = R.norm_around_zero(x.astype(np.float64), w - 1.0, 1e-3)
     assert np.max(np.abs(got - want)) <= OP_TOL[dtype] * np.max(np.abs(want))
     s = dev(x, "float32")
     got = host(rmsnorm_add_f32(s, dev(y, dtype), dev(w, "float32"), 1e-3, 0.3))
-    want = x + 0.3 * R.norm_aturnzero(y.astype(np.float64), w.astype(np.float64) - 1.0, 1e-3)
+    want = x + 0.3 * R.norm_around_zero(y.astype(np.float64), w.astype(np.float64) - 1.0, 1e-3)
     assert np.max(np.abs(got - want)) <= 2e-6 * np.max(np.abs(want))
 
 
@@ -436,22 +436,22 @@ def test_unequal_batch_and_slots_used_again(models, name, dtype):
     lens = [1, 40, 7, 90]
     ref = [reference(name, n + 12, seed=20 + i) for i, n in enumerate(lens)]
     s = BatchScheduler(model.build_engine(max_seq_len=128, max_batch=4))
-    for turn in range(2):                                    # the second time every slot holds another request's leftovers
-        order = [3, 1, 0, 2] if turn else [0, 1, 2, 3]
-        out = s.step([((turn, i), ref[i][0][:lens[i]], [lens[i] - 1, 0]) for i in order])
+    for again in range(2):                                    # the second time every slot holds another request's leftovers
+        order = [3, 1, 0, 2] if again else [0, 1, 2, 3]
+        out = s.step([((again, i), ref[i][0][:lens[i]], [lens[i] - 1, 0]) for i in order])
         for i, o in zip(order, out):
             assert logit_err(o, ref[i][1][[lens[i] - 1, 0]]) < TOL[dtype]
         live = list(order)
         for k in range(12):
-            out = s.step([((turn, i), [ref[i][0][lens[i] + k]], [0]) for i in live])
+            out = s.step([((again, i), [ref[i][0][lens[i] + k]], [0]) for i in live])
             for i, o in zip(live, out):
                 assert logit_err(o, ref[i][1][[lens[i] + k]]) < TOL[dtype]
             if k == 4:                                         # shorter ones end earlier
                 for i in (1, 0):
-                    s.release((turn, i))
+                    s.release((again, i))
                     live.remove(i)
         for i in live:
-            s.release((turn, i))
+            s.release((again, i))
     assert s.live == ()
 
 
