@@ -23,7 +23,7 @@ Extra objects on the JSON line:
                    launch / its average dispatch duration (start/stop events on every launch of eager steps on the
                    launch stream: the begin -> end interval rocprofv3 --kernel-trace reports), vs 8 TB/s HBM;
                    `traffic` = HBM bytes per launch, only when THIS run is itself a rocprofv3 --pmc pass whose counters a
-                   later reduction fills in (null otherwise; the round's measured values are in profiles/README.md).
+                   later reduction fills in (null otherwise).
   roofline_kernels the same row for every kernel of the step (per-launch us, bytes, frac, share of the step).
   step_roofline    whole decode step: algorithmic bytes per token / measured step time.
   prefill          ms, TFLOP/s and fraction of the 2.5 PFLOP/s dense bf16 MFMA peak for the 128-token prompt.
@@ -43,12 +43,12 @@ import numpy as np
 ROOT = os.path.dirname(os.path.abspath(__file__))
 sys.path.insert(0, ROOT)
 
-HBM_PEAK_GBS = 8000.0          # MI355X_MICROARCH.md: HBM3E 8 TB/s spec (6.3 TB/s measured copy)
+HBM_PEAK_GBS = 8000.0          # HBM3E 8 TB/s spec (6.3 TB/s measured copy)
 MFMA_BF16_PEAK_TFLOPS = 2500.0  # dense bf16
 
 
 def algorithmic_bytes_per_token(cfg: dict, ctx: int, weight_format: str) -> dict:
-    """weights read once per step + un-expanded bf16 KV rows + KV write + logits."""
+    """Weights read once per step + un-expanded bf16 KV rows + KV write + logits."""
     H, I, V, L = cfg["hidden_size"], cfg["intermediate_size"], cfg["vocab_size"], cfg["num_layers"]
     D, Hq, Hkv = cfg["head_dim"], cfg["num_heads"], cfg["num_kv_heads"]
     lin = L * ((Hq + 2 * Hkv) * D * H + H * Hq * D + 2 * I * H + H * I)
@@ -63,8 +63,7 @@ def algorithmic_bytes_per_token(cfg: dict, ctx: int, weight_format: str) -> dict
 
 def kernel_bytes_per_launch(cfg: dict, ctx: int, B: int) -> dict:
     """Algorithmic bytes ONE launch of each decode-step kernel class moves (bf16 weights, batch B, context ctx):
-    the weight matrix once, the fp32 activation vectors in and out once per sequence, K/V rows once per sequence.
-    DESIGN.md 4.1 lists the same terms."""
+    the weight matrix once, the fp32 activation vectors in and out once per sequence, K/V rows once per sequence."""
     H, I, V = cfg["hidden_size"], cfg["intermediate_size"], cfg["vocab_size"]
     D, Hq, Hkv = cfg["head_dim"], cfg["num_heads"], cfg["num_kv_heads"]
     nqkv, qd = (Hq + 2 * Hkv) * D, Hq * D
@@ -476,7 +475,7 @@ def main() -> None:
             toks = [int(t) for t in np.random.default_rng(4000 + args.seed).integers(0, V5, S_tok)]
             out = {"tokens": S_tok, "layers": L5, "flops": flops,
                    "parity": "BASELINE's 5e-2 end-to-end bar (fp8 vs bf16 logits) is NOT met on random-init weights at 32 layers "
-                             "(e4m3 quantisation itself, oracle included); it is met per GEMM: DESIGN.md 4.3, profiles/r02_config5_depth_error.json"}
+                             "(e4m3 quantisation itself, oracle included); it is met per GEMM: profiles/r02_config5_depth_error.json"}
             for fmt, peak in (("fp8a8", 2 * MFMA_BF16_PEAK_TFLOPS), ("bf16", MFMA_BF16_PEAK_TFLOPS)):
                 e5 = Engine(c5, w5["embed"], w5["bf16"] if fmt == "bf16" else w5["fp8"], w5["final_norm"], None, max_seq_len=S_tok + 8,
                             max_batch=1, weight_format=fmt, use_qk_norm=False)

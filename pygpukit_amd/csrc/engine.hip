@@ -1623,7 +1623,7 @@ static pgk_status decode_chunk(Engine* e, int b0, bool last, hipStream_t st, int
     float* h2 = e->h2 + (size_t)b0 * H;
     // fused attention+o_proj recomputes a KV head's attention in every row-slice workgroup: right for one
     // sequence at short context, wasteful for a batch.
-    // (two sequences ran the fused kernel too until round 3: its 96-KB workgroups are one per CU, so 2 x 256 of them took two
+    // (two sequences used to run the fused kernel too: its 96-KB workgroups are one per CU, so 2 x 256 of them took two
     // rounds - 9.4 us per layer against 3.7 + 2.4 for whole-context attention + an o_proj GEMV: 0.80 -> 0.66 ms per step)
     const bool fused = e->fused_attn && short_ctx && M == 1;
     const bool direct = !fused && short_ctx && M >= 2;
@@ -1933,7 +1933,7 @@ static pgk_status dense_prefill(Engine* e, int seq, const int32_t* h_tokens, int
     PGK_REQUIRE(n >= 1 && start_pos >= 0 && start_pos + n <= c.max_seq_len, "pgk_engine_prefill: positions %d..%d outside cache of %d",
                 start_pos, start_pos + n, c.max_seq_len);
     // (prompts of 129..256 tokens used to run as two chunks of <= 128 through the packed-weight kernels; since the staged 128-tile
-    // GEMM and the epilogue fusions of round 3 the long-prompt path is faster at every such length: 144 tokens 1.94 vs 2.38 ms,
+    // GEMM and the epilogue fusions the long-prompt path is faster at every such length: 144 tokens 1.94 vs 2.38 ms,
     // 256 tokens 2.27 vs 2.62)
     const int H = c.hidden_size, I = c.intermediate_size, D = c.head_dim, QD = c.num_heads * D, NQKV = e->qkv_dim();
     // workspace: h32 [n,H] f32 | x [n,H] | qkv [n,NQKV] | attn [n,QD] | gu [n,2I] | act [n,I]  (bf16)

@@ -7,7 +7,7 @@ Two things are called "batch" on this path:
     reference has no implementation of: `init_graph` / `step_graph_independent` / `run_greedy` drive the
     native engine with batch B; each sequence follows exactly the single-sequence semantics.
 The reference's captured batch graph replays baked scalars for the KV write / attention
-(batch.py:207-209; SURVEY.md 3.4) - not reproduced: positions are read from device memory."""
+(batch.py:207-209) - not reproduced: positions are read from device memory."""
 
 from __future__ import annotations
 
@@ -38,7 +38,7 @@ class DecodeBatch(DecodeStrategy):
     def step_graph(self, token_ids: list[int], start_position: int, context_len: int):
         """batch.py:308-363: the verify step for exactly `batch_size` tokens after init_graph() -> logits
         [batch_size, vocab].  Same result as step_batch; nothing is replayed from baked scalars (the reference's
-        captured graph freezes the KV-write position, SURVEY.md 3.4): positions are read from device memory."""
+        captured graph freezes the KV-write position): positions are read from device memory."""
         assert self._graph_ready, "Call init_graph() first"
         if len(token_ids) != self.batch_size:
             raise ValueError(f"token_ids length ({len(token_ids)}) must match batch_size ({self.batch_size})")

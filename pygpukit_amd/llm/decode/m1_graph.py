@@ -46,7 +46,7 @@ class DecodeM1Graph(DecodeStrategy):
         the object exists for code that addresses buffers by name: `logits`, `token_id_buf` and `position_buf` ARE the
         engine's live device state (the step's fp32 logits; the token / position the next replay consumes, updated
         by every replay); the per-layer activation fields have the reference's names and shapes but no step writes
-        them (INTEGRATION.md)."""
+        them."""
         if not self._graph_ready:
             return None
         if self._decode_buffers is None:

@@ -75,7 +75,7 @@ def build_gpt2_from_weights(cfg: dict, weights: dict, *, dtype: str = "float32",
     """CausalTransformerModel (GPT-2 style: learned positions, LayerNorm, GELU MLP, no RoPE) on the GPU from the
     weight dict of BASELINE config 1 ({"wte", "wpe", "layers": [{q,k,v,o,fc1,fc2}]}); LayerNorm gamma=1, beta=0.
     `biases` (optional, {"q","k","v","o","fc1","fc2"} -> per-layer list of vectors) adds Linear biases, which the
-    reference's CPU path cannot run (SURVEY 8c) but real GPT-2 checkpoints carry."""
+    reference's CPU path cannot run but real GPT-2 checkpoints carry."""
     from pygpukit_amd.llm.config import GPT2_SPEC, TransformerConfig
     from pygpukit_amd.llm.layers import MLP, Attention, Norm, TransformerBlock
     from pygpukit_amd.llm.models.causal import CausalTransformerModel
