@@ -354,11 +354,27 @@ pgk_status pgk_rmsnorm_f32(const float* x, const float* weight, void* out, int r
 pgk_status pgk_rmsnorm_add_f32(float* x, const void* y, const float* weight, int rows, int cols, float eps, float mult,
                                pgk_dtype y_dt, pgk_stream s);
 /* Sliding-window causal attention: q [q_len, hq, dk], k [kv_len, hkv, dk], v [kv_len, hkv, dv] -> out [q_len, hq, dv]; query i is
- * position kv_len - q_len + i and sees the `window` positions that end with its own.  gate (or NULL): [q_len rows of gate_stride
- * elements][hq], the head's output is multiplied by sigmoid(gate). */
+ * position kv_len - q_len + i and sees the `window` positions that end with its own.  gate (or NULL): rows of gate_stride elements,
+ * [hq] (one value per head) or, gate_elementwise, [hq, dv]; the output is multiplied by sigmoid(gate).  slopes (or NULL): fp32 [hq],
+ * slopes[head] * distance is taken off the scaled score. */
 pgk_status pgk_window_attention(const void* q, const void* k, const void* v, void* out, int hq, int hkv, int q_len, int kv_len,
-                                int dk, int dv, float scale, int window, const void* gate, int64_t gate_stride, pgk_dtype dt,
-                                pgk_stream s);
+                                int dk, int dv, float scale, int window, const void* gate, int64_t gate_stride,
+                                int gate_elementwise, const float* slopes, pgk_dtype dt, pgk_stream s);
+/* y_t = sum_j w[:, j] * u_(t - taps + 1 + j) per channel: u [n, channels], w [channels, taps], past [taps - 1, channels] = the rows
+ * before u (NULL: zeros) */
+pgk_status pgk_short_conv(const void* u, const void* past, const void* w, void* out, int n, int channels, int taps, pgk_dtype dt,
+                          pgk_stream s);
+/* x *= sigmoid(gate), n elements, in place */
+pgk_status pgk_sigmoid_mul(void* x, const void* gate, size_t n, pgk_dtype dt, pgk_stream s);
+/* xIELU: z > 0: a z^2 + z / 2;  z <= 0: b (exp(z) - 1 - z) + z / 2 */
+pgk_status pgk_xielu(const void* x, void* y, size_t n, float a, float b, pgk_dtype dt, pgk_stream s);
+/* Gated linear recurrence over n rows of one sequence: q, f [n, heads * dim] (before their activations), v [n, heads * vdim], f_bias
+ * (or NULL) and lower fp32 [heads * dim]; gate g = lower + (1 - lower) sigmoid(f + f_bias), S <- diag(g) S + (1 - g) v^T,
+ * o = S^T silu(q), with norm (or NULL; fp32 [vdim]) o / rms(o) * norm.  state: fp32 [heads, dim, vdim], read unless `fresh`, updated.
+ * dt: PGK_BF16 or PGK_F32 */
+pgk_status pgk_gated_recurrence(const void* q, const void* f, const void* v, const float* f_bias, const float* lower,
+                                const float* norm, float* state, void* out, int n, int fresh, int heads, int dim, int vdim,
+                                float eps, pgk_dtype dt, pgk_stream s);
 /* x[row][head][:] *= sigmoid(gate[row][head]) in place */
 pgk_status pgk_head_gate(void* x, const void* gate, int rows, int heads, int d, int64_t gate_stride, pgk_dtype dt, pgk_stream s);
 /* dst [dst_rows, dst_cols] = src [rows, cols] with zeros around it */
@@ -394,26 +410,42 @@ typedef struct {
 
 pgk_status pgk_engine_create(const pgk_model_config_t* cfg, const void* embed, const void* lm_head,
                              const void* final_norm, const pgk_layer_weights_t* layers, pgk_engine* out);
-/* Layer-list decoders (csrc/engine_stack.hip): fp32 residual stream, norm before and after each sublayer, sliding-window latent
- * attention with a per-head output gate, dense SwiGLU or no feed-forward; every layer has its own sizes.  dtype PGK_BF16 or PGK_F32
- * is the element type of the tables, matrices, activations and the latent cache; norm weights are fp32 with any offset applied.
- * Caller pads with zeros: Wp = width up to a multiple of 64, head_pad >= dim and vdim (64, 128 or a larger multiple of 64),
- * rank_pad and ff_pad multiples of 64 (ff_pad 0: the layer has no feed-forward), n_in a multiple of 64. */
+/* Layer-list decoders (csrc/engine_stack.hip): fp32 residual stream, a norm after each sublayer and optionally before it, one of
+ * several mixers per layer, dense SwiGLU / xIELU or no feed-forward; every layer has its own sizes.  dtype PGK_BF16 or PGK_F32 is the
+ * element type of the tables, matrices, activations and caches; norm weights, biases, taps and gates' constants are fp32 with any
+ * offset applied.  Caller pads with zeros: Wp = width up to a multiple of 64; n_in, n_att and ff_pad multiples of 64 (ff_pad 0: the
+ * layer has no feed-forward).
+ * PGK_MIX_LATENT     latent attention over a sliding window with a per-head output gate.  head_pad >= dim and vdim: 64, 128 or a
+ *                    larger multiple of 64; rank_pad a multiple of 64.  w_in rows: heads x head_pad queries | rank_pad latents |
+ *                    heads gates.
+ * PGK_MIX_ATTENTION  grouped heads over a K/V ring: q, k, v = taps over time of (w_in x + b_in), RMS norm over the whole q and k
+ *                    rows, distance bias, elementwise output gate.  head_pad as above (at most 1024).  w_in rows: heads x head_pad q |
+ *                    kv_heads x head_pad k | the same v | heads x head_pad gates; with kv_from >= 0 (that layer's keys and values)
+ *                    q | gates.  conv [taps][q, k, v rows] or NULL, slopes [heads] or NULL.
+ * PGK_MIX_HGRN2      gated linear recurrence (pgk_gated_recurrence).  head_pad, vhead_pad: dim, vdim up to multiples of 16.  w_in
+ *                    rows: heads x head_pad q | the same f | heads x vhead_pad v. */
+typedef enum { PGK_MIX_LATENT = 0, PGK_MIX_ATTENTION = 1, PGK_MIX_HGRN2 = 2 } pgk_mixer;
+typedef enum { PGK_FF_SWIGLU = 0, PGK_FF_XIELU = 1 } pgk_ff;
 typedef struct {
     int vocab_size, width, num_layers, max_positions, max_seq_len, max_batch;
     float norm_eps, residual_mult;
     pgk_dtype dtype;
 } pgk_stack_config_t;
 typedef struct {
-    int heads, dim, vdim, rank, window;            /* true sizes; window: keys a query sees, itself included */
-    int head_pad, rank_pad, n_in, ff_pad;
-    float scale;
-    const float *norm1, *norm1b, *norm2, *norm2b;  /* [Wp] */
-    const void* w_in;                              /* [n_in, Wp]: heads x head_pad query rows, rank_pad latent rows, heads gate rows */
-    const float* c_norm;                           /* [rank_pad] */
-    const void* w_ukv;                             /* [2 heads head_pad, rank_pad]: key rows, then value rows */
-    const void* w_o;                               /* [Wp, heads head_pad] */
-    const void* w_gate_up;                         /* [2 ff_pad, Wp] */
+    int mixer, ff;                                 /* pgk_mixer, pgk_ff */
+    int heads, kv_heads, dim, vdim, rank;          /* true sizes */
+    int window, taps, kv_from;                     /* window: keys a query sees, itself included; kv_from: -1 or an earlier layer */
+    int head_pad, vhead_pad, rank_pad, n_in, n_att, ff_pad;
+    float scale, act_pos, act_neg;                 /* act_*: pgk_xielu's a and b */
+    const float *norm1, *norm1b, *norm2, *norm2b;  /* [Wp]; norm1 / norm2 NULL: the sublayer reads the stream itself */
+    const void* w_in;                              /* [n_in, Wp] */
+    const float* b_in;                             /* [n_in] or NULL */
+    const float *conv, *q_norm, *k_norm, *slopes;  /* attention */
+    const float *lower, *o_norm;                   /* hgrn2: [heads * head_pad], [vhead_pad] */
+    const float* c_norm;                           /* latent: [rank_pad] */
+    const void* w_ukv;                             /* latent: [2 heads head_pad, rank_pad]: key rows, then value rows */
+    const void* w_o;                               /* [Wp, n_att] */
+    const void* w_gate_up;                         /* [2 ff_pad, Wp]; xIELU: [ff_pad, Wp] */
     const void* w_down;                            /* [Wp, ff_pad] */
 } pgk_stack_layer_t;
 /* embed [vocab, width], pos_embed [max_positions, width] or NULL, head [vocab, Wp], final_norm [Wp] */

@@ -52,8 +52,15 @@ class StackConfig(C.Structure):
 
 
 class StackLayer(C.Structure):
-    _fields_ = [(n, C.c_int) for n in ("heads", "dim", "vdim", "rank", "window", "head_pad", "rank_pad", "n_in", "ff_pad")] + [("scale", C.c_float)] + \
-               [(n, C.c_void_p) for n in ("norm1", "norm1b", "norm2", "norm2b", "w_in", "c_norm", "w_ukv", "w_o", "w_gate_up", "w_down")]
+    _fields_ = [(n, C.c_int) for n in ("mixer", "ff", "heads", "kv_heads", "dim", "vdim", "rank", "window", "taps", "kv_from", "head_pad", "vhead_pad", "rank_pad",
+                                       "n_in", "n_att", "ff_pad")] + \
+               [(n, C.c_float) for n in ("scale", "act_pos", "act_neg")] + \
+               [(n, C.c_void_p) for n in ("norm1", "norm1b", "norm2", "norm2b", "w_in", "b_in", "conv", "q_norm", "k_norm", "slopes", "lower", "o_norm", "c_norm",
+                                          "w_ukv", "w_o", "w_gate_up", "w_down")]
+
+
+MIX_LATENT, MIX_ATTENTION, MIX_HGRN2 = 0, 1, 2      # pgk_mixer
+FF_SWIGLU, FF_XIELU = 0, 1                          # pgk_ff
 
 
 # name -> (argtypes); every function returns pgk_status (int) unless listed in _NON_STATUS
@@ -114,7 +121,9 @@ _PROTOS = {
     "pgk_engine_prefill_batch": [_V, _I, c_i32_p, c_i32_p, c_i32_p, c_i32_p, _I, c_i32_p, C.POINTER(_F), _V],
     "pgk_engine_create_stack": [C.POINTER(StackConfig), _V, _V, _V, _V, C.POINTER(StackLayer), c_void_pp],
     "pgk_rmsnorm_f32": [_V, _V, _V, _I, _I, _F, _I, _V], "pgk_rmsnorm_add_f32": [_V, _V, _V, _I, _I, _F, _F, _I, _V],
-    "pgk_window_attention": [_V, _V, _V, _V, _I, _I, _I, _I, _I, _I, _F, _I, _V, _I64, _I, _V],
+    "pgk_window_attention": [_V, _V, _V, _V, _I, _I, _I, _I, _I, _I, _F, _I, _V, _I64, _I, _V, _I, _V],
+    "pgk_short_conv": [_V, _V, _V, _V, _I, _I, _I, _I, _V], "pgk_sigmoid_mul": [_V, _V, _Z, _I, _V], "pgk_xielu": [_V, _V, _Z, _F, _F, _I, _V],
+    "pgk_gated_recurrence": [_V, _V, _V, _V, _V, _V, _V, _V, _I, _I, _I, _I, _I, _F, _I, _V],
     "pgk_head_gate": [_V, _V, _I, _I, _I, _I64, _I, _V], "pgk_pad_2d": [_V, _V, _I, _I, _I, _I, _I, _V],
     "pgk_engine_set_state": [_V, c_i32_p, c_i32_p, _I, _V], "pgk_engine_decode_step": [_V, _I, _V],
     "pgk_engine_profile_step": [_V, _I, _I, C.POINTER(_F), C.POINTER(_I), _V],

@@ -1,15 +1,23 @@
-// Native engine for layer-list decoders: an fp32 residual stream, RMSNorm before AND after each sublayer, latent attention over a
-// sliding window (the cache holds one normalised latent row per token, not keys and values), dense SwiGLU or no feed-forward.
-// Every layer has its own sizes.  Elements are bf16 (fp32 stream, norms, scores and softmax) or fp32 throughout.
+// Native engine for layer-list decoders: an fp32 residual stream, RMSNorm after each sublayer and, where a layer has one, before it;
+// a dense feed-forward (SwiGLU or xIELU) or none.  Every layer has its own mixer and its own sizes.  Elements are bf16 (fp32 stream, norms,
+// scores, softmax, recurrent states) or fp32 throughout.
 //
-//   x   <- x + m * rho(O (sigmoid(G h) * attention(Q h, c)); n1b),  h = rho(x; n1),  c = rms(D h) * w_c,  k = U_k c,  v = U_v c
-//   x   <- x + m * rho(W_d (silu(W_g h) * W_u h); n2b),             h = rho(x; n2)
+//   x   <- x + m * rho(O mixer(h); n1b),            h = rho(x; n1) or x
+//   x   <- x + m * rho(W_d act(W_u h); n2b),        h = rho(x; n2) or x
 //
-// Cache: per layer [slot][R][rank] latents, R = min(window, max_seq_len); position p lives in row p mod R, so a full ring IS the
+// Mixers (pgk_mixer):
+//   latent attention  sigmoid(G h) * attention(Q h, c),  c = rms(D h) * w_c,  k = U_k c,  v = U_v c: over a sliding window; the cache holds
+//                     one normalised latent row per token, not keys and values.  The kernels are in this file.
+//   attention         taps over time and norms on q, k, v, a K/V ring (which another layer may own), distance bias, elementwise gate:
+//                     ops_gated_attn.hip
+//   hgrn2             gated linear recurrence with an fp32 state per sequence and head: ops_recurrence.hip
+// In a step a mixer takes the in-projection row(s) and leaves the rows that the out-projection multiplies.
+//
+// Latent cache: per layer [slot][R][rank] latents, R = min(window, max_seq_len); position p lives in row p mod R, so a full ring IS the
 // window and a decode step needs no mask.  Keys and values are never stored: decode folds U_k into the query (q_lat = U_k^T q, scores
 // q_lat . c) and applies U_v to the probability-weighted latent sum, prefill expands the latents it needs into a scratch K | V.
 //
-// Decode, one sequence (fp32 between kernels):
+// Decode of a latent layer, one sequence (fp32 between kernels):
 //   in_proj    [pending: x += m rho(y; n2b)] q | latent | gate = W_in . rho(x; n1)
 //   absorb     q_lat = scale log2e U_k^T q per head;  the new latent row -> ring
 //   attn       split over the ring: scores, softmax, sum p c  -> partial records
@@ -27,6 +35,7 @@
 
 #include "engine_state.hip.h"
 #include "latent.hip.h"
+#include "mixers.hip.h"
 #include "pkgemm.hip.h"
 
 namespace pgk {
@@ -44,7 +53,7 @@ constexpr float LOG2E = 1.4426950408889634f;
 
 // -------------------------------------------------------------------------------------------- one-row projection
 enum { SP_NORM = 0, SP_PLAIN = 1 };
-enum { SE_STORE = 0, SE_SWIGLU = 1, SE_LOGITS = 2 };
+enum { SE_STORE = 0, SE_SWIGLU = 1, SE_LOGITS = 2, SE_XIELU = 3 };
 
 struct StackGemvArgs {
     const void* w;            // [N][K] (SE_SWIGLU: [2 N][K], gate rows then up rows)
@@ -53,10 +62,11 @@ struct StackGemvArgs {
     const float* y;           // SP_NORM: pending sublayer output (null: none)
     const float* g_post;      // its post-norm weight
     float* x_out;             // where workgroup 0 writes the updated residual row (another buffer than x; null: nowhere)
-    const float* gamma;
+    const float* gamma;       // null: the row is taken as it is
     float eps, mult;
     float* out;               // [N]
     float* amax_val; int* amax_idx;
+    float act_pos, act_neg;   // SE_XIELU
 };
 
 // 256 threads; a wave owns R weight rows per trip.  C > 0: the first trip's C chunks of every row are requested before the prologue
@@ -88,10 +98,11 @@ __global__ __launch_bounds__(256) void stack_gemv_kernel(unsigned long long* tl,
             v[t] = *reinterpret_cast<const float4*>(a.x + i);
             if constexpr (PRO == SP_NORM) {
                 const float* yp = a.y ? a.y : a.x;                // unconditional loads; masked below
-                const float* pp = a.y ? a.g_post : a.gamma;
+                const float* gm_p = a.gamma ? a.gamma : a.x;
+                const float* pp = a.y ? a.g_post : gm_p;
                 y[t] = *reinterpret_cast<const float4*>(yp + i);
                 gp[t] = *reinterpret_cast<const float4*>(pp + i);
-                gm[t] = *reinterpret_cast<const float4*>(a.gamma + i);
+                gm[t] = *reinterpret_cast<const float4*>(gm_p + i);
             }
         }
         __builtin_amdgcn_sched_barrier(0);
@@ -117,15 +128,17 @@ __global__ __launch_bounds__(256) void stack_gemv_kernel(unsigned long long* tl,
                     if (a.x_out && blockIdx.x == 0 && i < K) *reinterpret_cast<float4*>(a.x_out + i) = v[t];
                 }
             }
-            ss = 0.f;
+            if (a.gamma) {
+                ss = 0.f;
 #pragma unroll
-            for (int t = 0; t < NT; ++t)
-                if ((int)(threadIdx.x + 256 * t) * 4 < K) ss += v[t].x * v[t].x + v[t].y * v[t].y + v[t].z * v[t].z + v[t].w * v[t].w;
-            ss = block_sum(ss, red);
-            const float inv = 1.0f / sqrtf(ss / a.W + a.eps);
+                for (int t = 0; t < NT; ++t)
+                    if ((int)(threadIdx.x + 256 * t) * 4 < K) ss += v[t].x * v[t].x + v[t].y * v[t].y + v[t].z * v[t].z + v[t].w * v[t].w;
+                ss = block_sum(ss, red);
+                const float inv = 1.0f / sqrtf(ss / a.W + a.eps);
 #pragma unroll
-            for (int t = 0; t < NT; ++t) {
-                v[t].x *= inv * gm[t].x; v[t].y *= inv * gm[t].y; v[t].z *= inv * gm[t].z; v[t].w *= inv * gm[t].w;
+                for (int t = 0; t < NT; ++t) {
+                    v[t].x *= inv * gm[t].x; v[t].y *= inv * gm[t].y; v[t].z *= inv * gm[t].z; v[t].w *= inv * gm[t].w;
+                }
             }
         }
 #pragma unroll
@@ -148,8 +161,8 @@ __global__ __launch_bounds__(256) void stack_gemv_kernel(unsigned long long* tl,
                 if (a.y && a.x_out && blockIdx.x == 0) a.x_out[i] = v;
                 ss = fmaf(v, v, ss);
             }
-            const float inv = 1.0f / sqrtf(block_sum(ss, red) / a.W + a.eps);
-            for (int i = threadIdx.x; i < K; i += 256) xs[i] = from_f<WT>(xin(i) * inv * a.gamma[i]);
+            const float inv = a.gamma ? 1.0f / sqrtf(block_sum(ss, red) / a.W + a.eps) : 1.0f;
+            for (int i = threadIdx.x; i < K; i += 256) xs[i] = from_f<WT>(a.gamma ? xin(i) * inv * a.gamma[i] : xin(i));
         } else {
             for (int i = threadIdx.x; i < K; i += 256) xs[i] = from_f<WT>(a.x[i]);
         }
@@ -195,6 +208,7 @@ __global__ __launch_bounds__(256) void stack_gemv_kernel(unsigned long long* tl,
                 if (n0 + r < N) {
                     float o = acc[r][0];
                     if constexpr (EPI == SE_SWIGLU) o = o / (1.0f + (std::is_same<WT, float>::value ? expf(-o) : __expf(-o))) * acc[r + R / 2][0];
+                    if constexpr (EPI == SE_XIELU) o = xielu<std::is_same<WT, float>::value>(o, a.act_pos, a.act_neg);
                     a.out[n0 + r] = o;
                     if constexpr (EPI == SE_LOGITS) { if (o > best_v) { best_v = o; best_i = n0 + r; } }
                 }
@@ -246,7 +260,7 @@ static pgk_status stack_gemv_r(const StackGemvArgs& a, hipStream_t st, int force
 
 template <class WT, int PRO, int EPI>
 static pgk_status stack_gemv(const StackGemvArgs& a, hipStream_t st, int force_grid = 0) {
-    if constexpr (std::is_same<WT, float>::value) return stack_gemv_r<WT, EPI == SE_STORE ? 1 : 2, PRO, EPI>(a, st, force_grid);
+    if constexpr (std::is_same<WT, float>::value) return stack_gemv_r<WT, EPI == SE_STORE || EPI == SE_XIELU ? 1 : 2, PRO, EPI>(a, st, force_grid);
     else if constexpr (EPI == SE_SWIGLU) {
         if (a.N >= 4096) return stack_gemv_r<WT, 4, PRO, EPI>(a, st);
         return stack_gemv_r<WT, 2, PRO, EPI>(a, st);
@@ -344,14 +358,6 @@ __global__ __launch_bounds__(256) void latent_absorb_kernel(unsigned long long* 
             reinterpret_cast<QT*>(a.qlat)[((size_t)(b0 + m) * a.H + h) * a.rank + r] = from_f<QT>(a.scale * (part[0][m][c] + part[1][m][c] + part[2][m][c] + part[3][m][c]));
     }
     tls.end();
-}
-
-// n occupied ring rows over nsplit splits: rows per split (a multiple of 32), the rows [k0, k1) of split s
-__device__ __forceinline__ int split_rows(int n, int nsplit) { return ((n + nsplit - 1) / nsplit + 31) / 32 * 32; }
-__device__ __forceinline__ void split_range(int n, int nsplit, int s, int& k0, int& k1) {
-    const int per = split_rows(n, nsplit);
-    k0 = min(s * per, n);
-    k1 = min(k0 + per, n);
 }
 
 // Any rank up to 2048, any element type: a wave walks every fourth key, one strided element per lane and 64 columns.
@@ -690,9 +696,6 @@ __global__ void stack_embed_kernel(const T* embed, const T* pos, const int32_t* 
     for (int i = threadIdx.x; i < ld; i += blockDim.x) h[row * ld + i] = i < W ? to_f(e[i]) + (p ? to_f(p[i]) : 0.f) : 0.f;
 }
 
-// A prompt row's place: position, cache slot, row in the latent scratch, and whether it is one of the last R of its sequence (the ones the ring keeps)
-struct RowPlace { int32_t pos, slot, kv, store; };
-
 // latents of positions already in the ring -> scratch rows (a portion that continues a sequence)
 template <class T>
 __global__ void latent_gather_kernel(const RowPlace* pl, const T* cache, T* c_all, int R, int rank) {
@@ -752,13 +755,16 @@ struct Stack {
     std::vector<pgk_stack_layer_t> layers;
     const void *embed = nullptr, *pos = nullptr, *head = nullptr;
     const float* final_norm = nullptr;
-    int Wp = 0, max_in = 0, max_att = 0, max_ff = 0, max_heads_rank = 0, max_heads = 0;
-    std::vector<void*> cache;              // per layer [max_batch][R][rank]
-    std::vector<int> ring;                 // R per layer
+    int Wp = 0, max_in = 0, max_att = 0, max_ff = 0, max_q = 0;
+    // per layer: latent rows [max_batch][R][rank] or K/V rows [max_batch][k, v][kv heads][R][head width] (a layer that takes another
+    // one's: that one's pointer) or recurrent states [max_batch][heads][dim][vdim] in fp32
+    std::vector<void*> cache;
+    std::vector<int> ring, reach;          // R; keys the cache has to keep (the largest window of the layers that read it).  0: no ring
+    std::vector<void*> taps;               // rings of projected values [max_batch][taps][channels], or null
     std::vector<int32_t> len;              // per slot: positions held (host side; advanced with every step enqueued)
     // decode buffers (rows = max_batch)
     float *in32 = nullptr, *a32 = nullptr, *y32 = nullptr, *act32 = nullptr, *po = nullptr, *pml = nullptr;
-    void *qlat = nullptr, *x16 = nullptr, *in16 = nullptr, *a16 = nullptr, *y16 = nullptr, *gu16 = nullptr, *act16 = nullptr;
+    void *qlat = nullptr, *qx = nullptr, *x16 = nullptr, *in16 = nullptr, *a16 = nullptr, *y16 = nullptr, *gu16 = nullptr, *act16 = nullptr;
     float* slabs16 = nullptr;              // split-K slabs of a batch step's projections
     // fragment-major copies of the layer matrices for 2..128 rows (ops_pkgemm.hip), where its shapes allow; null entries: row-major kernels
     struct Packed { bf16 *in = nullptr, *o = nullptr, *gate_up = nullptr, *down = nullptr; };
@@ -770,6 +776,8 @@ struct Stack {
     size_t esize() const { return cfg.dtype == PGK_F32 ? 4 : 2; }
 };
 static Stack* stack_of(const Engine* e) { return (Stack*)e->kind_state; }
+static int kv_source(const pgk_stack_layer_t& L, int l) { return L.kv_from >= 0 ? L.kv_from : l; }
+static int up_rows(const pgk_stack_layer_t& L) { return (L.ff == PGK_FF_SWIGLU ? 2 : 1) * L.ff_pad; }     // rows of the first feed-forward matrix
 
 static int pick_nsplit(const Engine* e, int B, const pgk_stack_layer_t& L, int R) {
     const int htiles = ceil_div(L.heads, 16);
@@ -855,6 +863,54 @@ static pgk_status latent_decode(Engine* e, int l, int B, const void* in, void* o
     return PGK_OK;
 }
 
+// taps and norms -> attention over the ring (split) -> combine and gate
+template <class T, class IT>
+static pgk_status attention_decode(Engine* e, int l, int B, const void* in, void* out, hipStream_t st, int* launches) {
+    Stack* s = stack_of(e);
+    const auto& L = s->layers[l];
+    const int src = kv_source(L, l), HD = L.heads * L.head_pad, GD = L.kv_from >= 0 ? 0 : L.kv_heads * L.head_pad;
+    constexpr pgk_dtype DT = std::is_same<T, float>::value ? PGK_F32 : PGK_BF16;
+    constexpr bool IO32 = std::is_same<IT, float>::value;
+    ConvArgs c{};
+    c.in = in; c.ld_in = L.n_in; c.bias = L.b_in; c.conv = L.conv; c.taps = L.taps; c.n_q = HD; c.n_kv = GD; c.D = L.head_pad; c.n = B; c.R = s->ring[src];
+    c.q_norm = L.q_norm; c.k_norm = L.k_norm; c.q_true = L.heads * L.dim; c.k_true = L.kv_heads * L.dim; c.eps = s->cfg.norm_eps; c.q_mult = L.scale * LOG2E;
+    c.tap_ring = s->taps[l]; c.positions = e->positions; c.q_out = s->qx; c.ld_q = HD; c.cache = s->cache[src];
+    if (pgk_status r = conv_rows(c, DT, IO32, kv_attn_q32(L.head_pad, DT), st)) return r;
+    KvAttnArgs a{};
+    a.q = s->qx; a.cache = s->cache[src]; a.slopes = L.slopes; a.positions = e->positions;
+    a.B = B; a.H = L.heads; a.G = L.kv_heads; a.D = L.head_pad; a.R = s->ring[src]; a.window = L.window;
+    a.nsplit = kv_attn_splits(B, L.heads, L.kv_heads, L.window < a.R ? L.window : a.R, e->cu_count);
+    a.po = s->po; a.pml = s->pml; a.gate = (const IT*)in + HD + 2 * GD; a.ld_gate = L.n_in; a.out = out; a.ld_out = HD;
+    *launches += 1;
+    return kv_attn_decode(a, DT, IO32, st, launches);
+}
+
+static RecurArgs recur_args(const Stack* s, int l, const void* in, void* out, int n) {
+    const auto& L = s->layers[l];
+    RecurArgs a{};
+    a.in = in; a.ld_in = L.n_in; a.f_off = L.heads * L.head_pad; a.v_off = 2 * a.f_off;
+    a.bias = L.b_in ? L.b_in + a.f_off : nullptr; a.lower = L.lower; a.norm = L.o_norm;
+    a.H = L.heads; a.dim = L.head_pad; a.vdim = L.vhead_pad; a.vdim_true = L.vdim; a.n = n; a.eps = s->cfg.norm_eps;
+    a.state = (float*)s->cache[l]; a.out = out; a.ld_out = L.n_att;
+    return a;
+}
+
+// The mixer of layer l for the next token of B sequences: in-projection rows `in` -> out-projection rows `out`
+template <class T, class IT>
+static pgk_status mix_decode(Engine* e, int l, int B, const void* in, void* out, hipStream_t st, int* launches) {
+    Stack* s = stack_of(e);
+    switch (s->layers[l].mixer) {
+        case PGK_MIX_LATENT: return latent_decode<T, IT>(e, l, B, in, out, st, launches);
+        case PGK_MIX_ATTENTION: return attention_decode<T, IT>(e, l, B, in, out, st, launches);
+        default: {
+            RecurArgs a = recur_args(s, l, in, out, B);
+            a.positions = e->positions;
+            *launches += 1;
+            return recur_rows(a, std::is_same<T, float>::value ? PGK_F32 : PGK_BF16, std::is_same<IT, float>::value, st);
+        }
+    }
+}
+
 // ---- one sequence: fused steps, fp32 between kernels ----
 template <class T>
 static pgk_status step_one(Engine* e, hipStream_t st, int* launches) {
@@ -876,10 +932,10 @@ static pgk_status step_one(Engine* e, hipStream_t st, int* launches) {
         if (pgk_status r = stack_gemv<T, SP_NORM, SE_STORE>(a, st)) return r;
         settle();
         mark(KC_ATTN);
-        if (pgk_status r = latent_decode<T, float>(e, l, 1, s->in32, s->a32, st, launches)) return r;
+        if (pgk_status r = mix_decode<T, float>(e, l, 1, s->in32, s->a32, st, launches)) return r;
         mark(KC_OPROJ);
         a = StackGemvArgs{};
-        a.w = L.w_o; a.N = s->Wp; a.K = L.heads * L.head_pad; a.x = s->a32; a.out = s->y32;
+        a.w = L.w_o; a.N = s->Wp; a.K = L.n_att; a.x = s->a32; a.out = s->y32;
         if (pgk_status r = stack_gemv<T, SP_PLAIN, SE_STORE>(a, st)) return r;
         pend = L.norm1b;
         *launches += 2;
@@ -888,7 +944,8 @@ static pgk_status step_one(Engine* e, hipStream_t st, int* launches) {
         a = StackGemvArgs{};
         norm_in(a, L.norm2);
         a.w = L.w_gate_up; a.N = L.ff_pad; a.out = s->act32;
-        if (pgk_status r = stack_gemv<T, SP_NORM, SE_SWIGLU>(a, st)) return r;
+        a.act_pos = L.act_pos; a.act_neg = L.act_neg;
+        if (pgk_status r = L.ff == PGK_FF_SWIGLU ? stack_gemv<T, SP_NORM, SE_SWIGLU>(a, st) : stack_gemv<T, SP_NORM, SE_XIELU>(a, st)) return r;
         settle();
         mark(KC_DOWN);
         a = StackGemvArgs{};
@@ -919,7 +976,7 @@ static pgk_status head_rows(Stack* s, const T* x, float* logits, int n, hipStrea
     return PGK_OK;
 }
 
-struct RowBufs { float* h; void *x, *in, *a, *y, *gu, *act; float* slabs; };
+struct RowBufs { float* h; void *x, *in, *a, *y, *gu, *act; float* slabs; void* q; };
 
 // How a [N, K] projection of n bf16 rows runs: fragment-major copy (<= 128 rows), weight-streaming kernel (<= 128 rows) or tiled
 // MFMA, and over how many split-K slabs its result is left (0: one bf16 result).
@@ -939,7 +996,7 @@ size_t Stack::slab_elems(int n, bool f32) const {
     for (size_t l = 0; l < layers.size(); ++l) {
         const auto& L = layers[l];
         const Packed P = packed.empty() ? Packed{} : packed[l];
-        const size_t need[] = {(size_t)plan_proj(P.o, n, Wp, L.heads * L.head_pad, true).slabs * n * Wp,
+        const size_t need[] = {(size_t)plan_proj(P.o, n, Wp, L.n_att, true).slabs * n * Wp,
                                L.ff_pad ? (size_t)plan_proj(P.down, n, Wp, L.ff_pad, true).slabs * n * Wp : 0,
                                P.in || n > 128 ? 0 : (size_t)plan_proj(nullptr, n, L.n_in, Wp, true).slabs * n * L.n_in};
         for (size_t z : need) m = z > m ? z : m;
@@ -986,10 +1043,16 @@ static pgk_status rows_in_proj(Stack* s, const pgk_stack_layer_t& L, const bf16*
     return PGK_OK;
 }
 
-// gate / up projection with SwiGLU of n rows: act = silu(x W_g) * (x W_u)
+// first feed-forward projection of n rows: act = silu(x W_g) * (x W_u), or xIELU(x W_u)
 template <class T>
 static pgk_status rows_gate_up(Stack* s, const pgk_stack_layer_t& L, const bf16* packed, const RowBufs& b, int n, hipStream_t st) {
     constexpr pgk_dtype DT = std::is_same<T, float>::value ? PGK_F32 : PGK_BF16;
+    if (L.ff == PGK_FF_XIELU) {
+        if (DT == PGK_BF16 && n <= 128 && packed) {
+            if (pgk_status r = pkgemm_nt((const bf16*)b.x, s->Wp, packed, b.act, L.ff_pad, PK_EPI_BF16, 1, n, L.ff_pad, s->Wp, nullptr, st)) return r;
+        } else if (pgk_status r = pgk_gemm_nt(b.x, L.w_gate_up, nullptr, b.act, n, L.ff_pad, s->Wp, DT, st)) return r;
+        return pgk_xielu(b.act, b.act, (size_t)n * L.ff_pad, L.act_pos, L.act_neg, DT, st);
+    }
     if (DT == PGK_BF16 && n <= 128 && packed)
         return pkgemm_nt((const bf16*)b.x, s->Wp, packed, b.act, L.ff_pad, PK_EPI_SWIGLU, 1, n, 2 * L.ff_pad, s->Wp, nullptr, st);
     if (DT == PGK_BF16 && engine_gemm_swiglu_ok(n, L.ff_pad, s->Wp, false))
@@ -1022,7 +1085,7 @@ static pgk_status rows_layers(Stack* s, const RowBufs& b, int n, hipStream_t st,
         mark(KC_ATTN);
         if (pgk_status r = mix(l)) return r;
         mark(KC_OPROJ);
-        if (pgk_status r = rows_out_proj<T>(s, b, b.a, L.w_o, P.o, n, L.heads * L.head_pad, &pend->slabs, st)) return r;
+        if (pgk_status r = rows_out_proj<T>(s, b, b.a, L.w_o, P.o, n, L.n_att, &pend->slabs, st)) return r;
         pend->gain = L.norm1b;
         if (!L.ff_pad) continue;
         mark(KC_GATEUP);
@@ -1042,9 +1105,9 @@ static pgk_status step_rows(Engine* e, int B, hipStream_t st, int* launches) {
     Stack* s = stack_of(e);
     constexpr pgk_dtype DT = std::is_same<T, float>::value ? PGK_F32 : PGK_BF16;
     const auto& c = s->cfg;
-    const RowBufs b{e->h, s->x16, s->in16, s->a16, s->y16, s->gu16, s->act16, s->slabs16};
+    const RowBufs b{e->h, s->x16, s->in16, s->a16, s->y16, s->gu16, s->act16, s->slabs16, nullptr};
     Pending pend;
-    if (pgk_status r = rows_layers<T>(s, b, B, st, &pend, [&](int l) { return latent_decode<T, T>(e, l, B, b.in, b.a, st, launches); })) return r;
+    if (pgk_status r = rows_layers<T>(s, b, B, st, &pend, [&](int l) { return mix_decode<T, T>(e, l, B, b.in, b.a, st, launches); })) return r;
     mark(KC_LMHEAD);
     if (pgk_status r = rows_norm(norm_args(s, b, B, pend, s->final_norm, b.x), B, DT, st)) return r;
     if (pgk_status r = head_rows<T>(s, (const T*)b.x, e->logits, B, st)) return r;
@@ -1089,16 +1152,19 @@ static pgk_status stack_embed_state(Engine* e, int batch, hipStream_t st) {
     return PGK_OK;
 }
 
-// May slot `slot` go on at `pos`?  Position 0 starts a new sequence; otherwise the rows its windows reach must still be in the rings
-// (a ring row is overwritten by the position `R` later).
+// May slot `slot` go on at `pos`?  Position 0 starts a new sequence; otherwise the rows its windows and taps reach must still be in the
+// rings (a ring row is overwritten by the position `R` later), and a recurrent state only goes on where it stands.
 static pgk_status check_position(const Engine* e, int slot, int pos) {
     const Stack* s = stack_of(e);
     const int len = s->len[slot];
     PGK_REQUIRE(pos <= len, "engine: slot %d holds %d positions, cannot go on at position %d", slot, len, pos);
     if (pos == 0 || pos == len) return PGK_OK;
     for (int l = 0; l < s->cfg.num_layers; ++l) {
-        const int R = s->ring[l], first = pos - s->layers[l].window + 1 > 0 ? pos - s->layers[l].window + 1 : 0;
-        PGK_REQUIRE(first + R >= len, "engine: slot %d has moved on to position %d; the window of position %d is no longer in its ring", slot, len, pos);
+        const auto& L = s->layers[l];
+        PGK_REQUIRE(L.mixer != PGK_MIX_HGRN2, "engine: slot %d has moved on to position %d; its recurrent state cannot go back to position %d", slot, len, pos);
+        auto kept = [&](int back, int R) { return (pos - back > 0 ? pos - back : 0) + R >= len; };
+        PGK_REQUIRE(kept(L.window - 1, s->ring[kv_source(L, l)]) && (L.mixer != PGK_MIX_ATTENTION || !L.conv || kept(L.taps - 1, L.taps)),
+                    "engine: slot %d has moved on to position %d; the window of position %d is no longer in its ring", slot, len, pos);
     }
     return PGK_OK;
 }
@@ -1124,21 +1190,23 @@ static pgk_status stack_prefill_t(Engine* e, int n_seqs, const int32_t* slots, c
         if (pgk_status r = check_position(e, slots[i], starts[i])) return r;
     int n = 0;
     for (int i = 0; i < n_seqs; ++i) n += lens[i];
-    // per layer: which latent rows a sequence's queries reach (its own rows and up to window - 1 before them)
+    // per layer with a ring: which cached rows a sequence's queries reach (its own and up to reach - 1 before them)
     struct LayerRows { size_t past0 = 0; int n_past = 0, n_kv = 0; };
     std::vector<LayerRows> lr(c.num_layers);
     std::vector<RowPlace> place;                        // per layer: n_past gathered rows, then n new rows (equal layers share them)
     std::vector<int> share(c.num_layers, -1);
     int max_kv = 0;
+    auto past_of = [&](int l, int i) { return starts[i] < s->reach[l] - 1 ? starts[i] : s->reach[l] - 1; };
     for (int l = 0; l < c.num_layers; ++l) {
+        if (!s->reach[l]) continue;
         for (int k = 0; k < l && share[l] < 0; ++k)
-            if (share[k] < 0 && s->ring[k] == s->ring[l] && s->layers[k].window == s->layers[l].window) share[l] = k;
+            if (share[k] < 0 && s->ring[k] == s->ring[l] && s->reach[k] == s->reach[l]) share[l] = k;
         if (share[l] >= 0) { lr[l] = lr[share[l]]; continue; }
         lr[l].past0 = place.size();
         int kv = 0;
         std::vector<RowPlace> fresh;
         for (int i = 0; i < n_seqs; ++i) {
-            const int past = starts[i] < s->layers[l].window - 1 ? starts[i] : s->layers[l].window - 1, end = starts[i] + lens[i];
+            const int past = past_of(l, i), end = starts[i] + lens[i];
             for (int p = starts[i] - past; p < starts[i]; ++p) place.push_back(RowPlace{p, slots[i], kv++, 0});
             for (int p = starts[i]; p < end; ++p) fresh.push_back(RowPlace{p, slots[i], kv++, p >= end - s->ring[l] ? 1 : 0});
             lr[l].n_past += past;
@@ -1147,11 +1215,17 @@ static pgk_status stack_prefill_t(Engine* e, int n_seqs, const int32_t* slots, c
         if (kv > max_kv) max_kv = kv;
         place.insert(place.end(), fresh.begin(), fresh.end());
     }
-    size_t kv_elems = 0, c_elems = 0;
+    // K/V scratch: one region that the layers use in turn, and one of its own for every layer whose keys others take
+    size_t kv_elems = 0, c_elems = 0, own_elems = 0;
+    std::vector<size_t> own(c.num_layers, 0);           // 1 + offset
+    for (int l = 0; l < c.num_layers; ++l)
+        if (s->layers[l].kv_from >= 0) own[s->layers[l].kv_from] = 1;
     for (int l = 0; l < c.num_layers; ++l) {
         const auto& L = s->layers[l];
-        const size_t ke = (size_t)lr[l].n_kv * 2 * L.heads * L.head_pad, ce = (size_t)lr[l].n_kv * L.rank_pad;
-        if (ke > kv_elems) kv_elems = ke;
+        if (!s->reach[l]) continue;
+        const size_t ke = (size_t)lr[l].n_kv * 2 * L.kv_heads * L.head_pad, ce = (size_t)lr[l].n_kv * L.rank_pad;
+        if (own[l]) { own[l] = 1 + own_elems; own_elems += (ke + 127) & ~(size_t)127; }
+        else if (ke > kv_elems) kv_elems = ke;
         if (ce > c_elems) c_elems = ce;
     }
     const int wrows = n_want < 128 ? n_want : 128;
@@ -1159,10 +1233,10 @@ static pgk_status stack_prefill_t(Engine* e, int n_seqs, const int32_t* slots, c
     const size_t E = sizeof(T);
     const size_t sizes[] = {(size_t)n * s->Wp * 4, (size_t)n * s->Wp * E, (size_t)n * s->max_in * E, (size_t)n * s->max_att * E, (size_t)n * s->Wp * E,
                             (size_t)n * 2 * s->max_ff * E, (size_t)n * s->max_ff * E, c_elems * E, kv_elems * E, (size_t)wrows * s->Wp * E, (size_t)wrows * c.vocab_size * 4,
-                            s->slab_elems(n, DT == PGK_F32) * 4};
+                            s->slab_elems(n, DT == PGK_F32) * 4, (size_t)n * s->max_q * E, own_elems * E};
     size_t need = 0;
     for (size_t z : sizes) need += up(z);
-    const size_t tab_need = up((size_t)n * 4) * 2 + up(place.size() * sizeof(RowPlace)) + up((size_t)n_want * 4);
+    const size_t tab_need = up((size_t)n * 4) * 2 + up(place.size() * sizeof(RowPlace)) + up((size_t)n_want * 4) + up((size_t)n * sizeof(RowSrc)) + up(n_seqs * sizeof(SeqSpan));
     auto grow = [&](void** p, size_t* have, size_t want_bytes) -> pgk_status {
         if (want_bytes <= *have) return PGK_OK;
         if (*p) { PGK_CHECK_HIP(hipStreamSynchronize(st)); pgk_free(*p); }
@@ -1184,12 +1258,20 @@ static pgk_status stack_prefill_t(Engine* e, int n_seqs, const int32_t* slots, c
     void* xw = take(sizes[9]);
     float* lg = (float*)take(sizes[10]);
     b.slabs = (float*)take(sizes[11]);
+    b.q = take(sizes[12]);
+    T* kv_own = (T*)take(sizes[13]);
     // one host image of the index tables, one copy
     std::vector<char> img(tab_need, 0);
-    const size_t o_pos = up((size_t)n * 4), o_place = 2 * o_pos, o_want = o_place + up(place.size() * sizeof(RowPlace));
+    const size_t o_pos = up((size_t)n * 4), o_place = 2 * o_pos, o_want = o_place + up(place.size() * sizeof(RowPlace)),
+                 o_rows = o_want + up((size_t)n_want * 4), o_seqs = o_rows + up((size_t)n * sizeof(RowSrc));
     memcpy(img.data(), tokens, (size_t)n * 4);
-    for (int i = 0, row = 0; i < n_seqs; ++i)
-        for (int j = 0; j < lens[i]; ++j, ++row) ((int32_t*)(img.data() + o_pos))[row] = starts[i] + j;
+    for (int i = 0, row = 0; i < n_seqs; ++i) {
+        ((SeqSpan*)(img.data() + o_seqs))[i] = SeqSpan{row, lens[i], starts[i], slots[i]};
+        for (int j = 0, first = row; j < lens[i]; ++j, ++row) {
+            ((int32_t*)(img.data() + o_pos))[row] = starts[i] + j;
+            ((RowSrc*)(img.data() + o_rows))[row] = RowSrc{starts[i] + j, slots[i], first};
+        }
+    }
     if (!place.empty()) memcpy(img.data() + o_place, place.data(), place.size() * sizeof(RowPlace));
     if (n_want) memcpy(img.data() + o_want, want, (size_t)n_want * 4);
     PGK_CHECK_HIP(hipMemcpyAsync(s->tab, img.data(), tab_need, hipMemcpyHostToDevice, st));
@@ -1198,9 +1280,11 @@ static pgk_status stack_prefill_t(Engine* e, int n_seqs, const int32_t* slots, c
     const int32_t* d_pos = (const int32_t*)((char*)s->tab + o_pos);
     const RowPlace* d_place = (const RowPlace*)((char*)s->tab + o_place);
     const int32_t* d_want = (const int32_t*)((char*)s->tab + o_want);
+    const RowSrc* d_rows = (const RowSrc*)((char*)s->tab + o_rows);
+    const SeqSpan* d_seqs = (const SeqSpan*)((char*)s->tab + o_seqs);
     stack_embed_kernel<T><<<n, 256, 0, st>>>((const T*)s->embed, (const T*)s->pos, d_tok, d_pos, b.h, c.width, s->Wp, c.max_positions);
     PGK_LAUNCH_CHECK();
-    auto mix = [&](int l) -> pgk_status {
+    auto latent = [&](int l) -> pgk_status {
         const auto& L = s->layers[l];
         const LayerRows& w = lr[l];
         const int HD = L.heads * L.head_pad, R = s->ring[l];
@@ -1215,16 +1299,58 @@ static pgk_status stack_prefill_t(Engine* e, int n_seqs, const int32_t* slots, c
         int row = 0, kv0 = 0;
         const WindowStrides sd{L.head_pad, L.n_in, L.head_pad, 2 * HD, L.head_pad, 2 * HD, L.head_pad, HD};
         for (int i = 0; i < n_seqs; ++i) {
-            const int past = starts[i] < L.window - 1 ? starts[i] : L.window - 1, klen = past + lens[i];
+            const int klen = past_of(l, i) + lens[i];
             const T* q = (const T*)b.in + (size_t)row * L.n_in;
             const T* k = kv + (size_t)kv0 * 2 * HD;
             if (pgk_status r = window_attention(q, k, k + HD, (T*)b.a + (size_t)row * HD, L.heads, L.heads, lens[i], klen, L.head_pad, L.head_pad, L.scale, L.window, sd,
-                                                q + HD + L.rank_pad, L.n_in, DT, st))
+                                                OutGate{q + HD + L.rank_pad, L.n_in, 1, 0}, nullptr, DT, st))
                 return r;
             row += lens[i];
             kv0 += klen;
         }
         return PGK_OK;
+    };
+    auto attention = [&](int l) -> pgk_status {
+        const auto& L = s->layers[l];
+        const int src = kv_source(L, l), HD = L.heads * L.head_pad, GD = L.kv_heads * L.head_pad, R = s->ring[src];
+        const bool mine = src == l;
+        const LayerRows& w = lr[src];
+        T* rows = own[src] ? kv_own + (own[src] - 1) : kv;
+        if (mine)
+            if (pgk_status r = kv_gather(d_place + w.past0, w.n_past, s->cache[l], rows, 2 * GD, GD, L.head_pad, R, DT, st)) return r;
+        ConvArgs a{};
+        a.in = b.in; a.ld_in = L.n_in; a.bias = L.b_in; a.conv = L.conv; a.taps = L.taps; a.n_q = HD; a.n_kv = mine ? GD : 0; a.D = L.head_pad; a.n = n; a.R = R;
+        a.q_norm = L.q_norm; a.k_norm = L.k_norm; a.q_true = L.heads * L.dim; a.k_true = L.kv_heads * L.dim; a.eps = c.norm_eps; a.q_mult = 1.f;
+        a.tap_ring = s->taps[l]; a.rows = d_rows; a.place = d_place + w.past0 + w.n_past; a.q_out = b.q; a.ld_q = HD; a.kv_rows = rows; a.ld_kv = 2 * GD; a.cache = s->cache[src];
+        if (pgk_status r = conv_rows(a, DT, DT == PGK_F32, DT == PGK_F32, st)) return r;
+        const int channels = HD + 2 * a.n_kv;
+        if (L.conv)
+            if (pgk_status r = conv_save(b.in, L.n_in, d_seqs, n_seqs, s->taps[l], L.taps, channels, DT, st)) return r;
+        int row = 0, kv0 = 0;
+        const WindowStrides sd{L.head_pad, HD, L.head_pad, 2 * GD, L.head_pad, 2 * GD, L.head_pad, HD};
+        for (int i = 0; i < n_seqs; ++i) {
+            const int klen = past_of(src, i) + lens[i];
+            const T* k = rows + (size_t)kv0 * 2 * GD;
+            const OutGate gate{(const T*)b.in + (size_t)row * L.n_in + channels, L.n_in, L.head_pad, 1};
+            if (pgk_status r = window_attention((const T*)b.q + (size_t)row * HD, k, k + GD, (T*)b.a + (size_t)row * HD, L.heads, L.kv_heads, lens[i], klen, L.head_pad, L.head_pad,
+                                                L.scale, L.window, sd, gate, L.slopes, DT, st))
+                return r;
+            row += lens[i];
+            kv0 += klen;
+        }
+        return PGK_OK;
+    };
+    auto recurrence = [&](int l) -> pgk_status {
+        RecurArgs a = recur_args(s, l, b.in, b.a, n);
+        a.seqs = d_seqs; a.n_seqs = n_seqs;
+        return recur_rows(a, DT, DT == PGK_F32, st);
+    };
+    auto mix = [&](int l) -> pgk_status {
+        switch (s->layers[l].mixer) {
+            case PGK_MIX_LATENT: return latent(l);
+            case PGK_MIX_ATTENTION: return attention(l);
+            default: return recurrence(l);
+        }
     };
     Pending pend;
     if (pgk_status r = rows_layers<T>(s, b, n, st, &pend, mix)) return r;
@@ -1248,10 +1374,12 @@ static pgk_status stack_prefill(Engine* e, int n_seqs, const int32_t* slots, con
     return stack_prefill_t<bf16>(e, n_seqs, slots, lens, starts, tokens, n_want, want, h_logits, st);
 }
 
-// layer l's latent ring [max_batch][R][rank_pad]; there is no value cache
+// layer l's latent ring, K/V ring (values after the keys of a slot: v points at the first slot's) or recurrent states
 static pgk_status stack_kv_ptr(Engine* e, int layer, void** k, void** v) {
-    *k = stack_of(e)->cache[layer];
-    *v = nullptr;
+    const Stack* s = stack_of(e);
+    const auto& L = s->layers[layer];
+    *k = s->cache[layer];
+    *v = L.mixer == PGK_MIX_ATTENTION ? (char*)s->cache[layer] + (size_t)L.kv_heads * s->ring[kv_source(L, layer)] * L.head_pad * s->esize() : nullptr;
     return PGK_OK;
 }
 
@@ -1281,13 +1409,31 @@ pgk_status pgk_engine_create_stack(const pgk_stack_config_t* cfg, const void* em
     const int Wp = ceil_div(c.width, 64) * 64;
     for (int l = 0; l < c.num_layers; ++l) {
         const auto& L = layers[l];
-        PGK_REQUIRE(L.heads >= 1 && L.dim >= 1 && L.vdim >= 1 && L.rank >= 1 && L.window >= 1, "pgk_engine_create_stack: layer %d: bad mixer sizes", l);
-        PGK_REQUIRE(L.head_pad % 64 == 0 && L.head_pad >= L.dim && L.head_pad >= L.vdim, "pgk_engine_create_stack: layer %d: head pad %d for widths %d / %d", l, L.head_pad, L.dim, L.vdim);
-        PGK_REQUIRE(L.rank_pad % 64 == 0 && L.rank_pad >= L.rank && L.rank_pad <= 2048, "pgk_engine_create_stack: layer %d: latent size %d padded to %d (at most 2048)", l, L.rank, L.rank_pad);
-        PGK_REQUIRE(L.n_in % 64 == 0 && L.n_in >= L.heads * L.head_pad + L.rank_pad + L.heads, "pgk_engine_create_stack: layer %d: in-projection rows %d", l, L.n_in);
+        PGK_REQUIRE(L.mixer >= PGK_MIX_LATENT && L.mixer <= PGK_MIX_HGRN2 && (L.ff == PGK_FF_SWIGLU || L.ff == PGK_FF_XIELU), "pgk_engine_create_stack: layer %d: mixer %d, feed-forward %d", l, L.mixer, L.ff);
+        PGK_REQUIRE(L.heads >= 1 && L.dim >= 1 && L.vdim >= 1, "pgk_engine_create_stack: layer %d: bad mixer sizes", l);
         PGK_REQUIRE(L.ff_pad % 64 == 0 && L.ff_pad >= 0, "pgk_engine_create_stack: layer %d: feed-forward pad %d", l, L.ff_pad);
-        PGK_REQUIRE(L.norm1 && L.norm1b && L.w_in && L.c_norm && L.w_ukv && L.w_o && (!L.ff_pad || (L.norm2 && L.norm2b && L.w_gate_up && L.w_down)),
-                    "pgk_engine_create_stack: layer %d: missing weights", l);
+        PGK_REQUIRE(L.n_in % 64 == 0 && L.n_att % 64 == 0, "pgk_engine_create_stack: layer %d: %d in-projection rows, %d out-projection columns", l, L.n_in, L.n_att);
+        PGK_REQUIRE(L.norm1b && L.w_in && L.w_o && (!L.ff_pad || (L.norm2b && L.w_gate_up && L.w_down)), "pgk_engine_create_stack: layer %d: missing weights", l);
+        const int HD = L.heads * L.head_pad;
+        if (L.mixer == PGK_MIX_HGRN2) {
+            PGK_REQUIRE(L.head_pad % 16 == 0 && L.vhead_pad % 16 == 0 && L.head_pad >= L.dim && L.vhead_pad >= L.vdim && L.n_in >= 2 * HD + L.heads * L.vhead_pad && L.n_att >= L.heads * L.vhead_pad,
+                        "pgk_engine_create_stack: layer %d: head widths %d / %d padded to %d / %d", l, L.dim, L.vdim, L.head_pad, L.vhead_pad);
+            PGK_REQUIRE(L.lower && L.o_norm, "pgk_engine_create_stack: layer %d: missing weights", l);
+            continue;
+        }
+        PGK_REQUIRE(L.window >= 1 && L.head_pad % 64 == 0 && L.head_pad >= L.dim && L.head_pad >= L.vdim && L.n_att == HD, "pgk_engine_create_stack: layer %d: window %d, head pad %d for widths %d / %d", l, L.window, L.head_pad, L.dim, L.vdim);
+        if (L.mixer == PGK_MIX_LATENT) {
+            PGK_REQUIRE(L.rank >= 1 && L.rank_pad % 64 == 0 && L.rank_pad >= L.rank && L.rank_pad <= 2048, "pgk_engine_create_stack: layer %d: latent size %d padded to %d (at most 2048)", l, L.rank, L.rank_pad);
+            PGK_REQUIRE(L.n_in >= HD + L.rank_pad + L.heads && L.kv_heads == L.heads && L.kv_from < 0, "pgk_engine_create_stack: layer %d: in-projection rows %d", l, L.n_in);
+            PGK_REQUIRE(L.norm1 && L.c_norm && L.w_ukv, "pgk_engine_create_stack: layer %d: missing weights", l);
+        } else {
+            PGK_REQUIRE(L.kv_heads >= 1 && L.heads % L.kv_heads == 0 && L.head_pad <= 1024 && L.taps >= 1, "pgk_engine_create_stack: layer %d: %d / %d heads of %d, %d taps", l, L.heads, L.kv_heads, L.head_pad, L.taps);
+            PGK_REQUIRE(L.n_in >= 2 * HD + (L.kv_from < 0 ? 2 * L.kv_heads * L.head_pad : 0), "pgk_engine_create_stack: layer %d: in-projection rows %d", l, L.n_in);
+            if (L.kv_from >= 0) {
+                PGK_REQUIRE(L.kv_from < l && layers[L.kv_from].mixer == PGK_MIX_ATTENTION && layers[L.kv_from].kv_from < 0 && layers[L.kv_from].kv_heads == L.kv_heads && layers[L.kv_from].head_pad == L.head_pad,
+                            "pgk_engine_create_stack: layer %d cannot take the keys and values of layer %d", l, L.kv_from);
+            }
+        }
     }
     Engine* e = new Engine();
     Stack* s = new Stack();
@@ -1317,22 +1463,36 @@ pgk_status pgk_engine_create_stack(const pgk_stack_config_t* cfg, const void* em
     };
     const size_t B = c.max_batch, E = s->esize();
     size_t part = 0, ml = 0, ql = 0;
+    auto most = [](auto& m, auto v) { if (v > m) m = v; };
+    s->reach.assign(c.num_layers, 0);
+    for (int l = 0; l < c.num_layers; ++l)
+        if (s->layers[l].mixer != PGK_MIX_HGRN2) most(s->reach[kv_source(s->layers[l], l)], s->layers[l].window);
     for (int l = 0; l < c.num_layers; ++l) {
         const auto& L = s->layers[l];
-        const int R = L.window < c.max_seq_len ? L.window : c.max_seq_len;
+        const int R = s->reach[l] < c.max_seq_len ? s->reach[l] : c.max_seq_len, HD = L.heads * L.head_pad;
         s->ring.push_back(R);
-        void* p = nullptr;
-        A(&p, B * R * L.rank_pad * E, &e->kv_bytes, true);
-        s->cache.push_back(p);
-        if (L.n_in > s->max_in) s->max_in = L.n_in;
-        if (L.heads * L.head_pad > s->max_att) s->max_att = L.heads * L.head_pad;
-        if (L.ff_pad > s->max_ff) s->max_ff = L.ff_pad;
-        for (int m = 1; m <= c.max_batch; ++m) {
-            const size_t ns = (size_t)pick_nsplit(e, m, L, R) * m * L.heads;
-            if (ns * L.rank_pad > part) part = ns * L.rank_pad;
-            if (ns * 2 > ml) ml = ns * 2;
+        void *p = nullptr, *t = nullptr;
+        if (L.mixer == PGK_MIX_LATENT) A(&p, B * R * L.rank_pad * E, &e->kv_bytes, true);
+        else if (L.mixer == PGK_MIX_HGRN2) A(&p, B * HD * L.vhead_pad * 4, &e->kv_bytes, true);
+        else {
+            const int GD = L.kv_heads * L.head_pad;
+            if (L.kv_from < 0) A(&p, B * 2 * R * GD * E, &e->kv_bytes, true);
+            else p = s->cache[L.kv_from];
+            if (L.conv) A(&t, B * L.taps * (HD + (L.kv_from < 0 ? 2 * GD : 0)) * E, &e->kv_bytes, true);
+            most(s->max_q, HD);
         }
-        if (B * L.heads * L.rank_pad > ql) ql = B * L.heads * L.rank_pad;
+        s->cache.push_back(p);
+        s->taps.push_back(t);
+        most(s->max_in, L.n_in);
+        most(s->max_att, L.n_att);
+        most(s->max_ff, L.ff_pad);
+        for (int m = 1; m <= c.max_batch && L.mixer != PGK_MIX_HGRN2; ++m) {
+            const int src = kv_source(L, l), keys = L.window < s->ring[src] ? L.window : s->ring[src];
+            const size_t ns = (size_t)(L.mixer == PGK_MIX_LATENT ? pick_nsplit(e, m, L, R) : kv_attn_splits(m, L.heads, L.kv_heads, keys, e->cu_count)) * m * L.heads;
+            most(part, ns * (L.mixer == PGK_MIX_LATENT ? L.rank_pad : L.head_pad));
+            most(ml, ns * 2);
+        }
+        if (L.mixer == PGK_MIX_LATENT) most(ql, B * L.heads * L.rank_pad);
     }
     A((void**)&e->tokens, B * 4, &e->ws_bytes, true);
     A((void**)&e->positions, B * 4, &e->ws_bytes, true);
@@ -1348,9 +1508,11 @@ pgk_status pgk_engine_create_stack(const pgk_stack_config_t* cfg, const void* em
     A((void**)&s->a32, (size_t)s->max_att * 4, &e->ws_bytes, true);     // padding columns of a head are never written: zero
     A((void**)&s->y32, (size_t)Wp * 4, &e->ws_bytes, true);
     A((void**)&s->act32, (size_t)(s->max_ff ? s->max_ff : 64) * 4, &e->ws_bytes);
-    A(&s->qlat, ql * 4, &e->ws_bytes);
-    A((void**)&s->po, part * 4, &e->ws_bytes);
-    A((void**)&s->pml, ml * 4, &e->ws_bytes);
+    auto some = [](size_t v) { return v ? v : (size_t)64; };
+    A(&s->qlat, some(ql) * 4, &e->ws_bytes);
+    A(&s->qx, some(B * s->max_q) * 4, &e->ws_bytes);
+    A((void**)&s->po, some(part) * 4, &e->ws_bytes);
+    A((void**)&s->pml, some(ml) * 4, &e->ws_bytes);
     A(&s->x16, B * Wp * E, &e->ws_bytes);
     A(&s->in16, B * s->max_in * E, &e->ws_bytes);
     A(&s->a16, B * s->max_att * E, &e->ws_bytes, true);
@@ -1366,12 +1528,11 @@ pgk_status pgk_engine_create_stack(const pgk_stack_config_t* cfg, const void* em
         auto visit = [&](auto fn) {
             for (int l = 0; l < c.num_layers; ++l) {
                 const auto& L = s->layers[l];
-                const int HD = L.heads * L.head_pad;
                 auto& P = s->packed[l];
                 if (pkgemm_shape_ok(L.n_in, Wp, false)) fn(&P.in, L.w_in, L.n_in, Wp);
-                if (pkgemm_shape_ok(Wp, HD, true)) fn(&P.o, L.w_o, Wp, HD);
+                if (pkgemm_shape_ok(Wp, L.n_att, true)) fn(&P.o, L.w_o, Wp, L.n_att);
                 if (!L.ff_pad) continue;
-                if (pkgemm_shape_ok(2 * L.ff_pad, Wp, false)) fn(&P.gate_up, L.w_gate_up, 2 * L.ff_pad, Wp);
+                if (pkgemm_shape_ok(up_rows(L), Wp, false)) fn(&P.gate_up, L.w_gate_up, up_rows(L), Wp);
                 if (pkgemm_shape_ok(Wp, L.ff_pad, true)) fn(&P.down, L.w_down, Wp, L.ff_pad);
             }
         };

@@ -19,9 +19,15 @@ template <> __device__ __forceinline__ void store4<bf16>(bf16* p, const float4& 
     *reinterpret_cast<uint2*>(p) = make_uint2(pack_bf16x2(v.x, v.y), pack_bf16x2(v.z, v.w));
 }
 
+// xIELU with its two softplus'ed factors: z > 0: a z^2 + z / 2,  z <= 0: b (exp(z) - 1 - z) + z / 2  (EXACT: the fp32 engines' form)
+template <bool EXACT> __device__ __forceinline__ float xielu(float z, float a, float b) {
+    const float n = fminf(z, 0.f), e = EXACT ? expm1f(n) : __expf(n) - 1.0f;
+    return fmaf(0.5f, z, z > 0.f ? a * z * z : b * (e - n));
+}
+
 // One sandwich step on rows of the fp32 stream h [*][ld] (columns W..ld are zero padding):
 //   y given:    h += mult * y / rms(y) * g_post       (y rows in the engine's element type, row stride ldy; store_h: write h back)
-//   out given:  out[i] = h / rms(h) * gamma           (rows of stride ld in the engine's element type)
+//   out given:  out[i] = h / rms(h) * gamma           (rows of stride ld in the engine's element type; gamma null: out[i] = h)
 // Workgroup i works on row rows[i] (null: row i) and writes out row i.  The norm weights are fp32, offsets already applied.
 struct RowsNormArgs {
     float* h;
@@ -41,11 +47,15 @@ struct RowsNormArgs {
 pgk_status rows_norm(const RowsNormArgs& a, int n, pgk_dtype dt, hipStream_t st);
 
 struct WindowStrides { long long qh, qs, kh, ks, vh, vs, oh, os; };   // elements: per head, per row
-// out[i] = sigmoid(gate[i][head]) * softmax over keys i' with 0 <= i - i' < window (queries are the last q_len of kv_len positions)
+// Output gate: the result is multiplied by sigmoid(p[row * gs + head * gh + column * gc]).  One value per head: gh 1, gc 0; one per
+// element: gh the head stride, gc 1.  p null: none.
+struct OutGate { const void* p; long long gs; int gh, gc; };
+// out[i] = gate * softmax over keys i' with 0 <= i - i' < window (queries are the last q_len of kv_len positions) of
+// scale * q . k - slopes[head] * (i - i')   (slopes fp32, or null)
 pgk_status window_attention(const void* q, const void* k, const void* v, void* out, int hq, int hkv, int q_len, int kv_len, int dk, int dv, float scale,
-                            int window, const WindowStrides& sd, const void* gate, long long gs, pgk_dtype dt, hipStream_t st);
+                            int window, const WindowStrides& sd, const OutGate& gate, const float* slopes, pgk_dtype dt, hipStream_t st);
 pgk_status flash_window(const void* q, const void* k, const void* v, void* out, int hq, int hkv, int q_len, int kv_len, int d, float scale,
-                        int window, const void* gate, long long gs, long long qh, long long qs, long long kh, long long ks, long long oh,
+                        int window, const OutGate& gate, const float* slopes, long long qh, long long qs, long long kh, long long ks, long long oh,
                         long long os, hipStream_t st);   // ops_flash.hip
 
 // ops_attention.hip: kv_len <= 128, head width 128, plain causal mask, bf16

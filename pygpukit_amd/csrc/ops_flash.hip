@@ -20,6 +20,7 @@
 
 #include <type_traits>
 
+#include "latent.hip.h"
 #include "pgk_device.hip.h"
 #include "pgk_internal.h"
 
@@ -70,19 +71,35 @@ struct FlashSplit {
 };
 
 // Sliding window (WIN instantiations): query i sees keys i - window + 1 .. i, tiles left of a workgroup's first window are never
-// loaded.  `gate` (may be null): one value per (query row, head) at gate[row * gs + head]; the head's output row is multiplied by
-// its sigmoid.  The scores are scaled in fp32 after the product (scale > 0: the running maximum is kept on unscaled scores).
+// loaded.  `gate`: OutGate, one value per (query row, head) or per element.  The scores are scaled in fp32 after the product
+// (scale > 0: the running maximum is kept on unscaled scores).
+// BIAS instantiations: slopes[head] * (query - key) is taken off the scaled score - the accumulators of S = K . Q^T start at
+// -slope / scale * (query - key) instead of zero.
 struct FlashWindow {
     int window;
-    const void* gate;
-    long long gs;
+    OutGate gate;
+    const float* slopes;
+    float inv_scale;
 };
 template <class T> __device__ __forceinline__ float flash_gate(const FlashWindow& w, int qrow, int head) {
-    if (!w.gate) return 1.f;
-    return 1.0f / (1.0f + __expf(-to_f(reinterpret_cast<const T*>(w.gate)[(long long)qrow * w.gs + head])));
+    if (!w.gate.p || w.gate.gc) return 1.f;
+    return 1.0f / (1.0f + __expf(-to_f(reinterpret_cast<const T*>(w.gate.p)[(long long)qrow * w.gate.gs + head * w.gate.gh])));
+}
+// the elementwise form: N consecutive columns (aligned to N elements) from column c on
+template <class T, int N> __device__ __forceinline__ void flash_gate_cols(const FlashWindow& w, int qrow, int head, int c, float (&y)[N]) {
+    const T* g = reinterpret_cast<const T*>(w.gate.p) + (long long)qrow * w.gate.gs + head * w.gate.gh + c;
+    uint2 raw[N / 4];
+#pragma unroll
+    for (int j = 0; j < N / 4; ++j) raw[j] = *reinterpret_cast<const uint2*>(g + 4 * j);
+#pragma unroll
+    for (int j = 0; j < N; ++j) {
+        const uint32_t word = j & 2 ? raw[j / 4].y : raw[j / 4].x;
+        const uint16_t half = (uint16_t)(j & 1 ? word >> 16 : word);
+        y[j] /= 1.0f + __expf(-to_f(__builtin_bit_cast(T, half)));
+    }
 }
 
-template <class T, int D, bool WIN = false>
+template <class T, int D, bool WIN = false, bool BIAS = false>
 __global__ __launch_bounds__(FL_THREADS, 2) void flash_fwd_kernel(const T* q, const T* k, const T* vt, T* out, int hq, int hkv,
                                                               int q_len, int kv_len, int kv_pad, float scale_log2e, FlashStrides sd,
                                                               FlashSplit sp, FlashWindow win) {
@@ -215,9 +232,19 @@ __global__ __launch_bounds__(FL_THREADS, 2) void flash_fwd_kernel(const T* q, co
         }
     };
     // S^T = K . Q^T of one tile: two 32-kv sub-tiles (rows = positions, column = this lane's query)
-    auto qk = [&](int buf, f32x16_fl& s0, f32x16_fl& s1) {
+    const float slope = BIAS ? win.slopes[head] * win.inv_scale : 0.f;
+    auto qk = [&](int buf, int t, f32x16_fl& s0, f32x16_fl& s1) {
+        if constexpr (BIAS) {            // rows are keys kv0 + (r & 3) + 8 (r >> 2) + 4 h (+ 32), this lane's query is position qpos
+            const float b0 = slope * (float)(t * FL_BKV + 4 * h - (causal_off + qw0 + ql));
 #pragma unroll
-        for (int r = 0; r < 16; ++r) { s0[r] = 0.f; s1[r] = 0.f; }
+            for (int r = 0; r < 16; ++r) {
+                s0[r] = fmaf(slope, (float)((r & 3) + 8 * (r >> 2)), b0);
+                s1[r] = fmaf(slope, (float)(32 + (r & 3) + 8 * (r >> 2)), b0);
+            }
+        } else {
+#pragma unroll
+            for (int r = 0; r < 16; ++r) { s0[r] = 0.f; s1[r] = 0.f; }
+        }
 #pragma unroll
         for (int ks = 0; ks < KS; ++ks) {
             const uint4 a0 = *reinterpret_cast<const uint4*>(Ks(buf) + fl_k_off<D>(ql, 2 * ks + h));
@@ -254,7 +281,7 @@ __global__ __launch_bounds__(FL_THREADS, 2) void flash_fwd_kernel(const T* q, co
         const int buf = t & 1, kv0 = t * FL_BKV;
         if (t + 1 < t1) { load_k(t + 1); load_v(t + 1); }
         const bool cur = live(t);
-        if (cur) qk(buf, sc0, sc1);
+        if (cur) qk(buf, t, sc0, sc1);
         if (cur) {
             // ---- mask, online softmax (this lane: query qw0 + ql, kv rows (r&3) + 8(r>>2) + 4h of each sub-tile) ----
             const bool need_mask = kv0 + FL_BKV - 1 > causal_off + qw0 || kv0 + FL_BKV > kv_len ||
@@ -373,10 +400,9 @@ __global__ __launch_bounds__(FL_THREADS, 2) void flash_fwd_kernel(const T* q, co
         for (int i = 0; i < DT; ++i)
 #pragma unroll
             for (int g = 0; g < 4; ++g) {
-                uint2 w;
-                w.x = pack16x2<T>(o[i][4 * g] * inv, o[i][4 * g + 1] * inv);
-                w.y = pack16x2<T>(o[i][4 * g + 2] * inv, o[i][4 * g + 3] * inv);
-                *reinterpret_cast<uint2*>(orow + i * 32 + 8 * g + 4 * h) = w;
+                float y[4] = {o[i][4 * g] * inv, o[i][4 * g + 1] * inv, o[i][4 * g + 2] * inv, o[i][4 * g + 3] * inv};
+                if constexpr (WIN) { if (win.gate.gc && sp.nsplit == 1) flash_gate_cols<T, 4>(win, qrow, head, i * 32 + 8 * g + 4 * h, y); }
+                *reinterpret_cast<uint2*>(orow + i * 32 + 8 * g + 4 * h) = make_uint2(pack16x2<T>(y[0], y[1]), pack16x2<T>(y[2], y[3]));
             }
         if (sp.nsplit > 1 && h == 0) {
             float* ml = sp.ml + (((size_t)split * hq + head) * q_len + qrow) * 2;
@@ -415,6 +441,7 @@ __global__ __launch_bounds__(256) void flash_merge_kernel(const float* ml, const
     const float inv = (den > 0.f ? 1.f / den : 0.f) * flash_gate<T>(win, qrow, head);
 #pragma unroll
     for (int j = 0; j < 8; ++j) acc[j] *= inv;
+    if (win.gate.gc) flash_gate_cols<T, 8>(win, qrow, head, c * 8, acc);
     Vec<T> v;
     v.from_float(acc);
     if constexpr (std::is_same<T, bf16>::value && D == 128) {
@@ -466,7 +493,7 @@ __global__ __launch_bounds__(256) void transpose_v_kernel(const T* v, T* vt, int
     }
 }
 
-template <class T, int D, bool WIN = false>
+template <class T, int D, bool WIN = false, bool BIAS = false>
 static pgk_status flash_launch(const T* q, const T* k, const T* v, T* out, int hq, int hkv, int q_len, int kv_len, float scale,
                                const FlashStrides& sd, hipStream_t st, uint8_t* q8 = nullptr, float* q8s = nullptr, const FlashWindow& win = FlashWindow{}) {
     const int kv_pad = ceil_div(kv_len, 64) * 64;
@@ -498,11 +525,11 @@ static pgk_status flash_launch(const T* q, const T* k, const T* v, T* out, int h
     constexpr size_t LDS = 2 * (size_t)(64 * D * 2) + 2 * (size_t)(D * 128);
     static bool attr_done = false;
     if (LDS > 48 * 1024 && !attr_done) {
-        PGK_CHECK_HIP(hipFuncSetAttribute(reinterpret_cast<const void*>(&flash_fwd_kernel<T, D, WIN>),
+        PGK_CHECK_HIP(hipFuncSetAttribute(reinterpret_cast<const void*>(&flash_fwd_kernel<T, D, WIN, BIAS>),
                                           hipFuncAttributeMaxDynamicSharedMemorySize, (int)LDS));
         attr_done = true;
     }
-    flash_fwd_kernel<T, D, WIN><<<nqt * hq * nsplit, FL_THREADS, LDS, st>>>(q, k, (const T*)vt, out, hq, hkv, q_len, kv_len, kv_pad,
+    flash_fwd_kernel<T, D, WIN, BIAS><<<nqt * hq * nsplit, FL_THREADS, LDS, st>>>(q, k, (const T*)vt, out, hq, hkv, q_len, kv_len, kv_pad,
                                                                       scale * 1.4426950408889634f, sd, sp, win);
     hipError_t e = hipGetLastError();
     if (e == hipSuccess && nsplit > 1) {
@@ -528,14 +555,16 @@ pgk_status flash_prefill(const void* q, const void* k, const void* v, void* out,
     return flash_launch<f16, 64>((const f16*)q, (const f16*)k, (const f16*)v, (f16*)out, hq, hkv, q_len, kv_len, scale, sd, st);
 }
 
-// sliding-window causal attention with an optional per-head output gate (bf16, head_dim 64 / 128, one key head per query head or
+// sliding-window causal attention with an optional output gate and distance bias (bf16, head_dim 64 / 128, one key head per query head or
 // a divisor, scale > 0): ops_latent.hip, engine_stack.hip
 pgk_status flash_window(const void* q, const void* k, const void* v, void* out, int hq, int hkv, int q_len, int kv_len, int d, float scale,
-                        int window, const void* gate, long long gs, long long qh, long long qs, long long kh, long long ks, long long oh,
+                        int window, const OutGate& gate, const float* slopes, long long qh, long long qs, long long kh, long long ks, long long oh,
                         long long os, hipStream_t st) {
     PGK_REQUIRE((d == 64 || d == 128) && window >= 1 && scale > 0.f && kv_len >= q_len, "flash_window: d=%d window=%d q_len=%d kv_len=%d", d, window, q_len, kv_len);
     const FlashStrides sd{qh, qs, kh, ks, oh, os};
-    const FlashWindow win{window, gate, gs};
+    const FlashWindow win{window, gate, slopes, 1.0f / scale};
+    if (slopes && d == 128) return flash_launch<bf16, 128, true, true>((const bf16*)q, (const bf16*)k, (const bf16*)v, (bf16*)out, hq, hkv, q_len, kv_len, scale, sd, st, nullptr, nullptr, win);
+    if (slopes) return flash_launch<bf16, 64, true, true>((const bf16*)q, (const bf16*)k, (const bf16*)v, (bf16*)out, hq, hkv, q_len, kv_len, scale, sd, st, nullptr, nullptr, win);
     if (d == 128) return flash_launch<bf16, 128, true>((const bf16*)q, (const bf16*)k, (const bf16*)v, (bf16*)out, hq, hkv, q_len, kv_len, scale, sd, st, nullptr, nullptr, win);
     return flash_launch<bf16, 64, true>((const bf16*)q, (const bf16*)k, (const bf16*)v, (bf16*)out, hq, hkv, q_len, kv_len, scale, sd, st, nullptr, nullptr, win);
 }

@@ -66,6 +66,15 @@ __global__ __launch_bounds__(256) void rows_norm_kernel(RowsNormArgs a) {
         }
     }
     if (!a.out) return;
+    if (!a.gamma) {                                     // the sublayer reads the stream itself
+        T* o = reinterpret_cast<T*>(a.out) + (size_t)blockIdx.x * a.ld;
+#pragma unroll
+        for (int t = 0; t < NT; ++t) {
+            const int i = (threadIdx.x + 256 * t) * 4;
+            if (i < nt) store4<T>(o + i, v[t]);
+        }
+        return;
+    }
     float ss = 0.f;
 #pragma unroll
     for (int t = 0; t < NT; ++t) ss += v[t].x * v[t].x + v[t].y * v[t].y + v[t].z * v[t].z + v[t].w * v[t].w;
@@ -132,6 +141,23 @@ __global__ __launch_bounds__(256) void head_gate_kernel(T* x, const T* gate, siz
     }
 }
 
+template <class T>
+__global__ __launch_bounds__(256) void xielu_kernel(const T* x, T* y, size_t n, float a, float b) {
+    constexpr int N = Vec<T>::N;
+    const size_t stride = (size_t)gridDim.x * 256, i0 = blockIdx.x * (size_t)256 + threadIdx.x;
+    for (size_t i = i0; i < n / N; i += stride) {
+        Vec<T> v;
+        v.load(x + i * N);
+        float f[N];
+        v.to_float(f);
+#pragma unroll
+        for (int j = 0; j < N; ++j) f[j] = xielu<std::is_same<T, float>::value>(f[j], a, b);
+        v.from_float(f);
+        v.store(y + i * N);
+    }
+    for (size_t i = n / N * N + i0; i < n; i += stride) y[i] = from_f<T>(xielu<std::is_same<T, float>::value>(to_f(x[i]), a, b));
+}
+
 template <class E>
 __global__ __launch_bounds__(256) void pad_2d_kernel(const E* src, E* dst, int rows, int cols, int dcols, size_t total) {
     for (size_t i = blockIdx.x * (size_t)256 + threadIdx.x; i < total; i += (size_t)gridDim.x * 256) {
@@ -144,7 +170,7 @@ __global__ __launch_bounds__(256) void pad_2d_kernel(const E* src, E* dst, int r
 // 64 keys (a lane per key for the scores, a lane per value column for the sum), the four partial softmaxes meet in LDS.
 template <class T>
 __global__ __launch_bounds__(256) void window_attn_simple_kernel(const T* q, const T* k, const T* v, T* out, int rep, int q_len, int kv_len, int dk, int dv,
-                                                                 float scale, int window, WindowStrides sd, const T* gate, long long gs) {
+                                                                 float scale, int window, WindowStrides sd, OutGate gate, const float* slopes) {
     extern __shared__ float wsm[];
     const int row = blockIdx.x, head = blockIdx.y, kvh = head / rep, lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
     float* qs = wsm;                          // [dk]
@@ -159,12 +185,13 @@ __global__ __launch_bounds__(256) void window_attn_simple_kernel(const T* q, con
     const T* kh = k + kvh * sd.kh;
     const T* vh = v + kvh * sd.vh;
     float m = -INFINITY, l = 0.f;
+    const float slope = slopes ? slopes[head] : 0.f;
     for (int k0 = lo + 64 * wid; k0 <= qpos; k0 += 256) {          // wave-uniform
         const int key = k0 + lane, kn = min(64, qpos + 1 - k0);
         float s = 0.f;
         const T* kr = kh + (long long)min(key, qpos) * sd.ks;
         for (int d = 0; d < dk; ++d) s = fmaf(qs[d], to_f(kr[d]), s);
-        s = lane < kn ? s * scale : -INFINITY;
+        s = lane < kn ? fmaf(s, scale, -slope * (float)(qpos - key)) : -INFINITY;
         const float mn = fmaxf(m, wave_max(s)), alpha = expf(m - mn), p = expf(s - mn);      // mn is finite: kn >= 1
         m = mn;
         l = l * alpha + wave_sum(p);
@@ -183,25 +210,29 @@ __global__ __launch_bounds__(256) void window_attn_simple_kernel(const T* q, con
     float mm = -INFINITY, den = 0.f, w[4];
     for (int i = 0; i < 4; ++i) mm = fmaxf(mm, ml[2 * i]);
     for (int i = 0; i < 4; ++i) { w[i] = ml[2 * i + 1] > 0.f ? expf(ml[2 * i] - mm) : 0.f; den += w[i] * ml[2 * i + 1]; }
-    float f = 1.f / den;
-    if (gate) f /= 1.0f + expf(-to_f(gate[(long long)row * gs + head]));
+    const float f = 1.f / den;
     const float* a0 = wsm + dk;
     T* o = out + head * sd.oh + row * sd.os;
-    for (int c = threadIdx.x; c < dv; c += 256) o[c] = from_f<T>((w[0] * a0[c] + w[1] * a0[dv + c] + w[2] * a0[2 * dv + c] + w[3] * a0[3 * dv + c]) * f);
+    const T* g = reinterpret_cast<const T*>(gate.p);
+    for (int c = threadIdx.x; c < dv; c += 256) {
+        const float y = (w[0] * a0[c] + w[1] * a0[dv + c] + w[2] * a0[2 * dv + c] + w[3] * a0[3 * dv + c]) * f;
+        o[c] = from_f<T>(g ? y / (1.0f + expf(-to_f(g[(long long)row * gate.gs + head * gate.gh + c * gate.gc]))) : y);
+    }
 }
 
 pgk_status window_attention(const void* q, const void* k, const void* v, void* out, int hq, int hkv, int q_len, int kv_len, int dk, int dv, float scale,
-                            int window, const WindowStrides& sd, const void* gate, long long gs, pgk_dtype dt, hipStream_t st) {
+                            int window, const WindowStrides& sd, const OutGate& gate, const float* slopes, pgk_dtype dt, hipStream_t st) {
     const bool flash = dt == PGK_BF16 && dk == dv && (dk == 64 || dk == 128) && scale > 0.f && sd.kh == sd.vh && sd.ks == sd.vs && aligned16(q) && aligned16(k) && aligned16(v) &&
-                       sd.qs % 8 == 0 && sd.qh % 8 == 0 && sd.ks % 8 == 0 && sd.kh % 8 == 0 && (reinterpret_cast<uintptr_t>(out) & 7u) == 0 && sd.os % 4 == 0 && sd.oh % 4 == 0;
+                       sd.qs % 8 == 0 && sd.qh % 8 == 0 && sd.ks % 8 == 0 && sd.kh % 8 == 0 && (reinterpret_cast<uintptr_t>(out) & 7u) == 0 && sd.os % 4 == 0 && sd.oh % 4 == 0 &&
+                       (!gate.gc || (gate.gc == 1 && gate.gs % 4 == 0 && gate.gh % 4 == 0 && (reinterpret_cast<uintptr_t>(gate.p) & 7u) == 0));
     // the whole context in one tile and inside every query's window
-    if (flash && dk == 128 && kv_len <= 128 && window >= kv_len) return attn_short_gated(q, k, v, out, hq, hkv, q_len, kv_len, scale, sd, gate, gs, st);
-    if (flash) return flash_window(q, k, v, out, hq, hkv, q_len, kv_len, dk, scale, window, gate, gs, sd.qh, sd.qs, sd.kh, sd.ks, sd.oh, sd.os, st);
+    if (flash && dk == 128 && kv_len <= 128 && window >= kv_len && !slopes && !gate.gc && (!gate.p || gate.gh == 1)) return attn_short_gated(q, k, v, out, hq, hkv, q_len, kv_len, scale, sd, gate.p, gate.gs, st);
+    if (flash) return flash_window(q, k, v, out, hq, hkv, q_len, kv_len, dk, scale, window, gate, slopes, sd.qh, sd.qs, sd.kh, sd.ks, sd.oh, sd.os, st);
     const size_t lds = ((size_t)dk + 4 * (size_t)dv + 4 * 64 + 8) * 4;
     PGK_REQUIRE(lds <= 64 * 1024, "window_attention: head widths %d / %d do not fit LDS", dk, dv);
     dim3 grid(q_len, hq);
     PGK_DISPATCH_FLOAT(dt, "window_attention", (window_attn_simple_kernel<T><<<grid, 256, lds, st>>>((const T*)q, (const T*)k, (const T*)v, (T*)out, hq / hkv, q_len, kv_len, dk, dv,
-                                                                                                     scale, window, sd, (const T*)gate, gs)));
+                                                                                                     scale, window, sd, gate, slopes)));
     PGK_LAUNCH_CHECK();
     return PGK_OK;
 }
@@ -229,12 +260,22 @@ pgk_status pgk_rmsnorm_add_f32(float* x, const void* y, const float* weight, int
 }
 
 pgk_status pgk_window_attention(const void* q, const void* k, const void* v, void* out, int hq, int hkv, int q_len, int kv_len, int dk, int dv, float scale,
-                                int window, const void* gate, int64_t gate_stride, pgk_dtype dt, pgk_stream s) {
+                                int window, const void* gate, int64_t gate_stride, int gate_elementwise, const float* slopes, pgk_dtype dt, pgk_stream s) {
     PGK_REQUIRE(q && k && v && out, "pgk_window_attention: null pointer");
     PGK_REQUIRE(hq > 0 && hkv > 0 && hq % hkv == 0, "pgk_window_attention: n_heads mismatch (Hq=%d, Hkv=%d)", hq, hkv);
     PGK_REQUIRE(q_len > 0 && kv_len >= q_len && dk > 0 && dv > 0 && window >= 1, "pgk_window_attention: bad shape q_len=%d kv_len=%d dk=%d dv=%d window=%d", q_len, kv_len, dk, dv, window);
     const WindowStrides sd{dk, (long long)hq * dk, dk, (long long)hkv * dk, dv, (long long)hkv * dv, dv, (long long)hq * dv};
-    return window_attention(q, k, v, out, hq, hkv, q_len, kv_len, dk, dv, scale, window, sd, gate, gate_stride, dt, resolve_stream(s));
+    const OutGate og{gate, gate_stride, gate_elementwise ? dv : 1, gate_elementwise ? 1 : 0};
+    return window_attention(q, k, v, out, hq, hkv, q_len, kv_len, dk, dv, scale, window, sd, og, slopes, dt, resolve_stream(s));
+}
+
+pgk_status pgk_xielu(const void* x, void* y, size_t n, float a, float b, pgk_dtype dt, pgk_stream s) {
+    PGK_REQUIRE(x && y && aligned16(x) && aligned16(y), "pgk_xielu: null or unaligned pointer");
+    if (!n) return PGK_OK;
+    const size_t blocks = (n / 4 + 255) / 256 + 1;
+    PGK_DISPATCH_FLOAT(dt, "pgk_xielu", (xielu_kernel<T><<<(int)(blocks > 8192 ? 8192 : blocks), 256, 0, resolve_stream(s)>>>((const T*)x, (T*)y, n, a, b)));
+    PGK_LAUNCH_CHECK();
+    return PGK_OK;
 }
 
 pgk_status pgk_head_gate(void* x, const void* gate, int rows, int heads, int d, int64_t gate_stride, pgk_dtype dt, pgk_stream s) {

@@ -2,7 +2,7 @@
 
 TransformerConfig carries the dimensions; ModelSpec is the data-only description of one
 architecture family (HF tensor-name patterns + architecture flags + default hyper-parameters).
-Dense families are described: GPT-2, Llama, Qwen2, Qwen3 and the layer-list family Totolorn (MoE families are
+Dense families are described: GPT-2, Llama, Qwen2, Qwen3 and the layer-list families Totolorn and Malasun (MoE families are
 not).  A layer-list model's config.json spells out every layer: LayerConfig."""
 
 from __future__ import annotations
@@ -19,7 +19,7 @@ class ModelSpec:
     lm_head: str | None
     final_norm: str
     final_norm_bias: str | None
-    attn_norm: str
+    attn_norm: str | None
     attn_norm_bias: str | None
     q_proj: str
     k_proj: str | None
@@ -31,7 +31,7 @@ class ModelSpec:
     o_bias: str | None
     q_norm: str | None
     k_norm: str | None
-    mlp_norm: str
+    mlp_norm: str | None
     mlp_norm_bias: str | None
     fc1: str | None
     fc1_bias: str | None
@@ -45,7 +45,7 @@ class ModelSpec:
     expert_up_proj: str | None = None
     expert_down_proj: str | None = None
     norm_type: Literal["rmsnorm", "layernorm"] = "rmsnorm"
-    activation: Literal["gelu", "silu"] = "silu"
+    activation: Literal["gelu", "silu", "xielu"] = "silu"
     use_rope: bool = True
     use_qk_norm: bool = False
     use_position_embed: bool = False
@@ -64,6 +64,16 @@ class ModelSpec:
     k_up_proj: str | None = None
     v_up_proj: str | None = None
     head_gate: str | None = None           # one sigmoid gate per head
+    q_conv: str | None = None              # taps over time on the channels of q, k, v
+    k_conv: str | None = None
+    v_conv: str | None = None
+    out_gate: str | None = None            # one sigmoid gate per element of the mixer's output
+    forget_proj: str | None = None         # gated recurrence: forget gate, its bias and lower bound, norm of a head's output
+    forget_bias: str | None = None
+    forget_lower: str | None = None
+    head_norm: str | None = None
+    act_params: str | None = None          # numbers of the activation
+    norm_scalar: bool = False              # a norm's weight is one number
     norm_weight_offset: float = 0.0        # norms multiply by offset + weight (1: weights stored around zero)
     residual_f32: bool = False             # the residual stream stays fp32 whatever the element type
 
@@ -116,8 +126,18 @@ TOTOLORN_SPEC = ModelSpec(
     post_attn_norm=_T + "norm1b", post_mlp_norm=_T + "norm2b", kv_down_proj=_T + "mix.dkv", kv_down_norm=_T + "mix.dkv.norm",
     k_up_proj=_T + "mix.uk", v_up_proj=_T + "mix.uv", head_gate=_T + "mix.g", norm_weight_offset=1.0, residual_f32=True)
 
+MALASUN_SPEC = ModelSpec(
+    name="malasun", embed_tokens="embed", position_embed=None, lm_head="head", final_norm="final.norm", final_norm_bias=None,
+    attn_norm=None, attn_norm_bias=None, q_proj=_T + "mix.q", k_proj=_T + "mix.k", v_proj=_T + "mix.v", o_proj=_T + "mix.o",
+    q_bias=_T + "mix.q.b", k_bias=_T + "mix.k.b", v_bias=_T + "mix.v.b", o_bias=None, q_norm=_T + "mix.q.norm", k_norm=_T + "mix.k.norm",
+    mlp_norm=None, mlp_norm_bias=None, fc1=_T + "mlp.up", fc1_bias=None, fc2=_T + "mlp.down", fc2_bias=None,
+    gate_proj=None, up_proj=None, down_proj=None, norm_type="rmsnorm", activation="xielu", use_rope=False, use_qk_norm=True,
+    architecture="Malasun", post_attn_norm=_T + "norm1", post_mlp_norm=_T + "norm2", q_conv=_T + "mix.q.conv", k_conv=_T + "mix.k.conv",
+    v_conv=_T + "mix.v.conv", out_gate=_T + "mix.g", forget_proj=_T + "mix.f", forget_bias=_T + "mix.f.b", forget_lower=_T + "mix.lower",
+    head_norm=_T + "mix.norm", act_params=_T + "mlp.act", norm_scalar=True, residual_f32=True)
+
 MODEL_SPECS: dict[str, ModelSpec] = {"gpt2": GPT2_SPEC, "llama": LLAMA_SPEC, "qwen3": QWEN3_SPEC, "qwen2": QWEN2_SPEC,
-                                     "totolorn": TOTOLORN_SPEC}
+                                     "totolorn": TOTOLORN_SPEC, "malasun": MALASUN_SPEC}
 
 
 def detect_model_spec(tensor_names: list[str], config: dict | None = None) -> ModelSpec:
@@ -146,26 +166,45 @@ def detect_model_spec(tensor_names: list[str], config: dict | None = None) -> Mo
 class LayerConfig:
     """One layer of a layer-list model."""
 
-    mixer: Literal["latent_attention"]
+    mixer: Literal["latent_attention", "attention", "hgrn2"]
     num_heads: int
     head_dim: int                     # query / key width of a head
     v_head_dim: int                   # value width of a head
-    kv_rank: int                      # latent size: what the cache holds per token
+    kv_rank: int                      # latent attention: latent size, what the cache holds per token
     window: int | None                # keys a query sees, itself included (None: all before it)
     scale: float                      # multiplies q . k
-    intermediate_size: int | None     # SwiGLU width; None: the layer has no feed-forward
+    intermediate_size: int | None     # feed-forward width; None: the layer has no feed-forward
+    num_kv_heads: int = 0             # attention: key / value heads
+    conv_taps: int | None = None      # attention: taps over time on q, k, v (None: no convolution)
+    kv_from: int | None = None        # attention: the layer whose keys and values this one uses (None: its own)
 
 
 def parse_layer(i: int, entry: dict) -> LayerConfig:
-    kind = entry.get("type")
-    if kind != "latent_attention":
+    kind, mlp = entry.get("type"), entry.get("mlp")
+    if kind not in ("latent_attention", "attention", "hgrn2"):
         raise ValueError(f"layer {i}: unknown mixer {kind!r}")
-    m, mlp = entry["mixer"], entry.get("mlp")
+    m = entry["mixer"]
     if mlp is not None and mlp.get("kind") != "dense":
         raise ValueError(f"layer {i}: unknown feed-forward {mlp.get('kind')!r}")
+    ff = int(mlp["ff"]) if mlp is not None else None
+    heads, dim, vdim = int(m["heads"]), int(m["dim"]), int(m["vdim"])
+    if kind == "hgrn2":
+        return LayerConfig(kind, heads, dim, vdim, 0, None, 1.0, ff)
     mask = m.get("mask")
-    return LayerConfig("latent_attention", int(m["heads"]), int(m["dim"]), int(m["vdim"]), int(m["kv_rank"]),
-                       int(mask["size"]) if mask else None, float(m["scale"]), int(mlp["ff"]) if mlp is not None else None)
+    window = int(mask["size"]) if mask else None
+    if kind == "latent_attention":
+        return LayerConfig(kind, heads, dim, vdim, int(m["kv_rank"]), window, float(m["scale"]), ff)
+    taps, src = m.get("conv"), m.get("kv_from")
+    return LayerConfig(kind, heads, dim, vdim, 0, window, float(m["scale"]), ff, int(m["kv_heads"]), int(taps) if taps is not None else None,
+                       int(src) if src is not None else None)
+
+
+def distance_slopes(heads: int) -> list[float]:
+    """Slopes of the distance bias: 2^(-8 (h + 1) / heads) for head h."""
+    return [2.0 ** (-8.0 * (h + 1) / heads) for h in range(heads)]
+
+
+NO_POSITION_LIMIT = 2**30       # models without learned positions
 
 
 def layer_list_config(config: dict) -> "TransformerConfig":
@@ -173,12 +212,20 @@ def layer_list_config(config: dict) -> "TransformerConfig":
     layers = tuple(parse_layer(i, e) for i, e in enumerate(config["layers"]))
     if not layers:
         raise ValueError("config.json lists no layers")
+    for i, l in enumerate(layers):
+        if l.mixer == "attention" and (l.num_kv_heads < 1 or l.num_heads % l.num_kv_heads):
+            raise ValueError(f"layer {i}: {l.num_heads} query heads over {l.num_kv_heads} key heads")
+        if l.kv_from is not None:
+            s = layers[l.kv_from] if 0 <= l.kv_from < i else None
+            if s is None or s.mixer != "attention" or s.kv_from is not None or (s.num_kv_heads, s.head_dim, s.v_head_dim) != (l.num_kv_heads, l.head_dim, l.v_head_dim):
+                raise ValueError(f"layer {i}: cannot take the keys and values of layer {l.kv_from}")
     first = layers[0]
+    spec = next((s for s in MODEL_SPECS.values() if s.architecture == config.get("architecture")), TOTOLORN_SPEC)
     return TransformerConfig(vocab_size=int(config["vocab"]), hidden_size=int(config["width"]), num_layers=len(layers), num_heads=first.num_heads,
-                             num_kv_heads=first.num_heads, intermediate_size=max([l.intermediate_size or 0 for l in layers]),
-                             _head_dim=first.head_dim, norm_type="rmsnorm", activation="silu", use_rope=False,
-                             max_position_embeddings=int(config["max_positions"]), norm_eps=float(config["norm"]["eps"]), tie_word_embeddings=False,
-                             layers=layers, residual_mult=float(config["residual_mult"]))
+                             num_kv_heads=first.num_kv_heads or first.num_heads, intermediate_size=max([l.intermediate_size or 0 for l in layers]),
+                             _head_dim=first.head_dim, norm_type="rmsnorm", activation=spec.activation, use_rope=False,
+                             max_position_embeddings=int(config["max_positions"]) if spec.use_position_embed else NO_POSITION_LIMIT,
+                             norm_eps=float(config["norm"]["eps"]), tie_word_embeddings=False, layers=layers, residual_mult=float(config.get("residual_mult", 1.0)))
 
 
 @dataclass
@@ -197,7 +244,7 @@ class TransformerConfig:
     num_experts_per_tok: int = 2
     moe_intermediate_size: int | None = None
     norm_type: Literal["rmsnorm", "layernorm"] = "rmsnorm"
-    activation: Literal["gelu", "silu"] = "silu"
+    activation: Literal["gelu", "silu", "xielu"] = "silu"
     use_rope: bool = True
     causal: bool = True
     max_position_embeddings: int = 2048

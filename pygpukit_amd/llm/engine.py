@@ -14,7 +14,7 @@ import numpy as np
 from pygpukit_amd import _hip
 from pygpukit_amd.core.array import GPUArray
 from pygpukit_amd.core.dtypes import bfloat16, float32
-from pygpukit_amd.core.factory import zeros
+from pygpukit_amd.core.factory import from_numpy, zeros
 from pygpukit_amd.ops.tensor import concat_axis0, pad_2d
 
 
@@ -280,21 +280,77 @@ class Engine:
         return out + toks
 
 
+NO_WINDOW = 2**30
+
+
+def _up(n: int, m: int) -> int:
+    return (n + m - 1) // m * m
+
+
 def _up64(n: int) -> int:
-    return (n + 63) // 64 * 64
+    return _up(n, 64)
+
+
+def _attention_pad(dim: int, vdim: int) -> int:
+    """Head width the attention kernels run at: 64, 128 or a larger multiple of 64."""
+    m = max(dim, vdim)
+    return 64 if m <= 64 else 128 if m <= 128 else _up64(m)
+
+
+def _head_rows(w: GPUArray, heads: int, per_head: int, pad: int, cols: int) -> GPUArray:
+    """[heads * per_head, c] -> [heads * pad, cols]"""
+    c = w.shape[1]
+    return pad_2d(pad_2d(w.view((heads, per_head * c)), heads, pad * c).view((heads * pad, c)), heads * pad, cols)
+
+
+def _head_cols(w: GPUArray, heads: int, per_head: int, pad: int, rows: int, cols: int) -> GPUArray:
+    """[r, heads * per_head] -> [rows, cols], heads pad columns apart"""
+    r = w.shape[0]
+    return pad_2d(pad_2d(w.view((r * heads, per_head)), r * heads, pad).view((r, heads * pad)), rows, cols)
+
+
+def _stack_rows(parts: list[GPUArray]) -> GPUArray:
+    """Matrices of one width below each other, zero rows up to a multiple of 64."""
+    cols = parts[0].shape[1]
+    out = zeros((_up64(sum(w.shape[0] for w in parts)), cols), parts[0].dtype)
+    at = 0
+    for w in parts:
+        _hip.call("pgk_memcpy_d2d", C.c_void_p(out.data_ptr() + at * cols * w.itemsize), w._p, w.nbytes, None)
+        at += w.shape[0]
+    return out
+
+
+def _row(w: GPUArray, n: int) -> GPUArray:
+    return pad_2d(w.view((1, w.size)), 1, n)
+
+
+def _host_f32(a: GPUArray) -> np.ndarray:
+    h = a.to_numpy()
+    return (h.astype(np.uint32) << 16).view(np.float32) if a.dtype == bfloat16 else h.astype(np.float32)
+
+
+def _pad_heads(v: np.ndarray, heads: int, pad: int, fill: float = 0.0) -> np.ndarray:
+    """[..., heads * d] -> [..., heads * pad]"""
+    d = v.shape[-1] // heads
+    out = np.full((*v.shape[:-1], heads, pad), fill, np.float32)
+    out[..., :d] = v.reshape(*v.shape[:-1], heads, d)
+    return out.reshape(*v.shape[:-1], heads * pad)
 
 
 class StackEngine(Engine):
-    """The native engine for layer-list models (csrc/engine_stack.hip): fp32 residual stream, norm before and after each sublayer,
-    sliding-window latent attention, every layer with its own sizes.  State, graphs, sampling and generation are Engine's.
+    """The native engine for layer-list models (csrc/engine_stack.hip): fp32 residual stream, a norm after each sublayer and optionally
+    before it, a mixer per layer (latent attention, attention over a K/V ring, gated linear recurrence), every layer with its own
+    sizes.  State, graphs, sampling and generation are Engine's.
 
-    The cache of a layer is a ring of min(window, max_seq_len) latent rows per sequence slot: a sequence goes on where it stopped
-    (or starts again at position 0); a position whose window has been overwritten is refused."""
+    The cache of an attention layer is a ring of min(window, max_seq_len) rows per sequence slot, that of a recurrent one a state: a
+    sequence goes on where it stopped (or starts again at position 0); a position whose window or state has been overwritten is refused."""
+
+    _SIZES = ("mixer", "ff", "heads", "kv_heads", "dim", "vdim", "rank", "window", "taps", "kv_from", "head_pad", "vhead_pad", "rank_pad", "n_att", "ff_pad")
 
     def __init__(self, config: dict, embed: GPUArray, position_embed: GPUArray | None, head: GPUArray, final_norm: GPUArray, layers: list[dict], *,
                  max_seq_len: int = 512, max_batch: int = 1):
-        """config: vocab_size, width, max_positions, norm_eps, residual_mult.  layers[i]: the sizes heads, dim, vdim, rank, window, scale,
-        head_pad, rank_pad, ff_pad and the packed arrays of pack_layer()."""
+        """config: vocab_size, width, max_positions, norm_eps, residual_mult.  layers[i]: the sizes and packed arrays of pack_layer(),
+        pack_attention() or pack_recurrence()."""
         _hip.require_device()
         dt = embed.dtype
         if dt not in (bfloat16, float32):
@@ -311,21 +367,32 @@ class StackEngine(Engine):
             raise ValueError(f"StackEngine: position table {position_embed.shape}")
         arr = (_hip.StackLayer * len(layers))()
         for i, lw in enumerate(layers):
-            hd = lw["heads"] * lw["head_pad"]
-            ff, rp = lw["ff_pad"], lw["rank_pad"]
-            n_in = lw["w_in"].shape[0]
-            for name, shape, dtype in (("norm1", (1, wp), float32), ("norm1b", (1, wp), float32), ("norm2", (1, wp), float32), ("norm2b", (1, wp), float32),
-                                       ("c_norm", (1, rp), float32), ("w_in", (n_in, wp), dt), ("w_ukv", (2 * hd, rp), dt), ("w_o", (wp, hd), dt),
-                                       ("w_gate_up", (2 * ff, wp), dt), ("w_down", (wp, ff), dt)):
+            hd, gd = lw["heads"] * lw["head_pad"], 0 if lw["kv_from"] >= 0 else lw["kv_heads"] * lw["head_pad"]
+            ff, rp, n_in, n_att = lw["ff_pad"], lw["rank_pad"], lw["w_in"].shape[0], lw["n_att"]
+            up = 2 * ff if lw["ff"] == _hip.FF_SWIGLU else ff
+            # name -> (shape, dtype, may be absent)
+            want = {"norm1": ((1, wp), float32, True), "norm1b": ((1, wp), float32, False), "w_in": ((n_in, wp), dt, False), "w_o": ((wp, n_att), dt, False),
+                    "b_in": ((1, n_in), float32, True)}
+            if ff:
+                want.update(norm2=((1, wp), float32, True), norm2b=((1, wp), float32, False), w_gate_up=((up, wp), dt, False), w_down=((wp, ff), dt, False))
+            if lw["mixer"] == _hip.MIX_LATENT:
+                want.update(c_norm=((1, rp), float32, False), w_ukv=((2 * hd, rp), dt, False))
+            elif lw["mixer"] == _hip.MIX_ATTENTION:
+                want.update(conv=((lw["taps"], hd + 2 * gd), float32, True), q_norm=((1, hd), float32, True), k_norm=((1, gd), float32, True),
+                            slopes=((1, lw["heads"]), float32, True))
+            else:
+                want.update(lower=((1, hd), float32, False), o_norm=((1, lw["vhead_pad"]), float32, False))
+            for name, (shape, dtype, optional) in want.items():
                 t = lw.get(name)
-                if t is None and not ff and name in ("norm2", "norm2b", "w_gate_up", "w_down"):
+                if t is None and optional:
                     continue
                 if t is None or t.shape != shape or t.dtype != dtype:
                     raise ValueError(f"StackEngine: layer {i}: {name} must be {dtype} {shape}, got {None if t is None else (t.dtype, t.shape)}")
                 setattr(arr[i], name, t.data_ptr())
-            for name in ("heads", "dim", "vdim", "rank", "window", "head_pad", "rank_pad", "ff_pad"):
+            for name in self._SIZES:
                 setattr(arr[i], name, lw[name])
             arr[i].n_in, arr[i].scale = n_in, lw["scale"]
+            arr[i].act_pos, arr[i].act_neg = lw.get("act_params", (0.0, 0.0))
         sc = _hip.StackConfig(config["vocab_size"], config["width"], len(layers), config["max_positions"], max_seq_len, max_batch, config["norm_eps"],
                               config["residual_mult"], dt.code)
         h = C.c_void_p()
@@ -336,36 +403,126 @@ class StackEngine(Engine):
         self.last_prefill_logits = None
 
     @staticmethod
-    def pack_layer(q: GPUArray, kv_down: GPUArray, head_gate: GPUArray, kv_norm: GPUArray, k_up: GPUArray, v_up: GPUArray, o: GPUArray, norm1: GPUArray,
-                   norm1b: GPUArray, *, heads: int, dim: int, vdim: int, window: int, scale: float, gate_up: GPUArray | None = None,
-                   down: GPUArray | None = None, norm2: GPUArray | None = None, norm2b: GPUArray | None = None) -> dict:
-        """One layer's matrices ([out, in]; norms fp32 with offsets applied) -> the engine's padded layout: head widths to 64 / 128 / a
-        multiple of 64, every other width to a multiple of 64.  Arrays that already fit are used as they are."""
-        width, rank = q.shape[1], kv_down.shape[0]
-        wp, rp = _up64(width), _up64(rank)
-        m = max(dim, vdim)
-        hp = 64 if m <= 64 else 128 if m <= 128 else _up64(m)
-        hd = heads * hp
-
-        def head_rows(w: GPUArray, per_head: int, cols: int) -> GPUArray:      # [heads * per_head, c] -> [heads * hp, cols]
-            c = w.shape[1]
-            return pad_2d(pad_2d(w.view((heads, per_head * c)), heads, hp * c).view((hd, c)), hd, cols)
-
-        w_in = zeros((_up64(hd + rp + heads), wp), q.dtype)
-        for rows, w in ((0, head_rows(q, dim, wp)), (hd, pad_2d(kv_down, rank, wp)), (hd + rp, pad_2d(head_gate, heads, wp))):
-            _hip.call("pgk_memcpy_d2d", C.c_void_p(w_in.data_ptr() + rows * wp * w.itemsize), w._p, w.nbytes, None)
-        row = lambda w, n: pad_2d(w.view((1, w.size)), 1, n)  # noqa: E731
-        out = dict(heads=heads, dim=dim, vdim=vdim, rank=rank, window=window, scale=scale, head_pad=hp, rank_pad=rp, ff_pad=0, w_in=w_in,
-                   c_norm=row(kv_norm, rp), w_ukv=concat_axis0(head_rows(k_up, dim, rp), head_rows(v_up, vdim, rp)),
-                   w_o=pad_2d(pad_2d(o.view((width * heads, vdim)), width * heads, hp).view((width, hd)), wp, hd),
-                   norm1=row(norm1, wp), norm1b=row(norm1b, wp))
+    def _pack_common(width: int, norm1: GPUArray | None, norm1b: GPUArray, gate_up: GPUArray | None, down: GPUArray | None, norm2: GPUArray | None,
+                     norm2b: GPUArray | None, act_params: tuple[float, float] | None) -> dict:
+        """Norms and feed-forward of a layer.  gate_up: the SwiGLU matrix [2 ff, width], or with act_params (xIELU's two factors)
+        the up-projection [ff, width]."""
+        wp = _up64(width)
+        out = dict(norm1=None if norm1 is None else _row(norm1, wp), norm1b=_row(norm1b, wp), ff_pad=0, ff=_hip.FF_SWIGLU if act_params is None else _hip.FF_XIELU,
+                   rank=0, rank_pad=0, kv_from=-1, taps=1, window=NO_WINDOW, scale=1.0)
+        if act_params is not None:
+            out["act_params"] = act_params
         if gate_up is not None:
             ff = down.shape[1]
             fp = _up64(ff)
-            if (ff, width) != (fp, wp):
+            if act_params is not None:
+                gate_up = pad_2d(gate_up, fp, wp)
+            elif (ff, width) != (fp, wp):
                 gate_up = concat_axis0(pad_2d(gate_up._view(0, (ff, width)), fp, wp), pad_2d(gate_up._view(ff * width, (ff, width)), fp, wp))
-            out.update(ff_pad=fp, w_gate_up=gate_up, w_down=pad_2d(down, wp, fp), norm2=row(norm2, wp), norm2b=row(norm2b, wp))
+            out.update(ff_pad=fp, w_gate_up=gate_up, w_down=pad_2d(down, wp, fp), norm2=None if norm2 is None else _row(norm2, wp), norm2b=_row(norm2b, wp))
         return out
+
+    @classmethod
+    def pack_layer(cls, q: GPUArray, kv_down: GPUArray, head_gate: GPUArray, kv_norm: GPUArray, k_up: GPUArray, v_up: GPUArray, o: GPUArray, norm1: GPUArray,
+                   norm1b: GPUArray, *, heads: int, dim: int, vdim: int, window: int, scale: float, gate_up: GPUArray | None = None,
+                   down: GPUArray | None = None, norm2: GPUArray | None = None, norm2b: GPUArray | None = None,
+                   act_params: tuple[float, float] | None = None) -> dict:
+        """One latent-attention layer's matrices ([out, in]; norms fp32 with offsets applied) -> the engine's padded layout: head widths to
+        64 / 128 / a multiple of 64, every other width to a multiple of 64.  Arrays that already fit are used as they are."""
+        width, rank = q.shape[1], kv_down.shape[0]
+        wp, rp, hp = _up64(width), _up64(rank), _attention_pad(dim, vdim)
+        hd = heads * hp
+        out = cls._pack_common(width, norm1, norm1b, gate_up, down, norm2, norm2b, act_params)
+        out.update(mixer=_hip.MIX_LATENT, heads=heads, kv_heads=heads, dim=dim, vdim=vdim, rank=rank, window=window, scale=scale, head_pad=hp, vhead_pad=hp, rank_pad=rp,
+                   n_att=hd, w_in=_stack_rows([_head_rows(q, heads, dim, hp, wp), pad_2d(kv_down, rp, wp), pad_2d(head_gate, heads, wp)]), c_norm=_row(kv_norm, rp),
+                   w_ukv=concat_axis0(_head_rows(k_up, heads, dim, hp, rp), _head_rows(v_up, heads, vdim, hp, rp)), w_o=_head_cols(o, heads, vdim, hp, wp, hd))
+        return out
+
+    @classmethod
+    def pack_attention(cls, q: GPUArray, k: GPUArray | None, v: GPUArray | None, gate: GPUArray, o: GPUArray, norm1: GPUArray | None, norm1b: GPUArray, *, heads: int,
+                       kv_heads: int, dim: int, vdim: int, window: int, scale: float, biases: tuple = (None, None, None), convs: tuple = (None, None, None),
+                       q_norm: GPUArray | None = None, k_norm: GPUArray | None = None, slopes: GPUArray | None = None, kv_from: int | None = None,
+                       gate_up: GPUArray | None = None, down: GPUArray | None = None, norm2: GPUArray | None = None, norm2b: GPUArray | None = None,
+                       act_params: tuple[float, float] | None = None) -> dict:
+        """One layer of attention over a K/V ring: q, k, v, gate, o [out, in]; biases and convs ([channels, taps]) of q, k, v; norms of the
+        whole q and k rows; slopes [heads]; kv_from: the layer whose keys and values it takes (k, v are None then)."""
+        width = q.shape[1]
+        wp, hp = _up64(width), _attention_pad(dim, vdim)
+        parts = [(q, heads, dim)] + ([] if kv_from is not None else [(k, kv_heads, dim), (v, kv_heads, vdim)])
+        mats = [_head_rows(w, n, d, hp, wp) for w, n, d in parts] + [_head_rows(gate, heads, vdim, hp, wp)]
+        w_in = _stack_rows(mats)
+        out = cls._pack_common(width, norm1, norm1b, gate_up, down, norm2, norm2b, act_params)
+        rows = sum(m.shape[0] for m in mats[:-1])
+
+        def channels(arrays: tuple) -> np.ndarray:        # [..., channels] of q (, k, v) -> padded heads side by side
+            return np.concatenate([_pad_heads(_host_f32(a).T, n, hp) for a, (_, n, _) in zip(arrays, parts)], axis=-1)
+
+        b_in = conv = None
+        if biases[0] is not None:
+            b = np.zeros((1, w_in.shape[0]), np.float32)
+            b[0, :rows] = channels(biases)
+            b_in = from_numpy(b)
+        if convs[0] is not None:
+            conv = from_numpy(np.ascontiguousarray(channels(convs)))
+        vec = lambda a, n: None if a is None else from_numpy(_pad_heads(_host_f32(a).reshape(1, -1), n, hp))  # noqa: E731
+        out.update(mixer=_hip.MIX_ATTENTION, heads=heads, kv_heads=kv_heads, dim=dim, vdim=vdim, window=window, scale=scale, head_pad=hp, vhead_pad=hp, n_att=heads * hp,
+                   kv_from=-1 if kv_from is None else kv_from, taps=1 if conv is None else conv.shape[0], w_in=w_in, b_in=b_in, conv=conv, q_norm=vec(q_norm, heads),
+                   k_norm=None if kv_from is not None else vec(k_norm, kv_heads), slopes=None if slopes is None else slopes.view((1, heads)),
+                   w_o=_head_cols(o, heads, vdim, hp, wp, heads * hp))
+        return out
+
+    @classmethod
+    def pack_recurrence(cls, q: GPUArray, forget: GPUArray, v: GPUArray, o: GPUArray, forget_bias: GPUArray, lower: GPUArray, head_norm: GPUArray,
+                        norm1: GPUArray | None, norm1b: GPUArray, *, heads: int, dim: int, vdim: int, gate_up: GPUArray | None = None, down: GPUArray | None = None,
+                        norm2: GPUArray | None = None, norm2b: GPUArray | None = None, act_params: tuple[float, float] | None = None) -> dict:
+        """One gated-recurrence layer: q, forget, v, o [out, in]; forget_bias, lower and head_norm fp32.  Padding channels keep an empty
+        state: their lower bound is 1, so nothing is written."""
+        width = q.shape[1]
+        wp, dp, vp = _up64(width), _up(dim, 16), _up(vdim, 16)
+        w_in = _stack_rows([_head_rows(q, heads, dim, dp, wp), _head_rows(forget, heads, dim, dp, wp), _head_rows(v, heads, vdim, vp, wp)])
+        n_att = _up64(heads * vp)
+        b = np.zeros((1, w_in.shape[0]), np.float32)
+        b[0, heads * dp:2 * heads * dp] = _pad_heads(_host_f32(forget_bias).reshape(1, -1), heads, dp)
+        out = cls._pack_common(width, norm1, norm1b, gate_up, down, norm2, norm2b, act_params)
+        out.update(mixer=_hip.MIX_HGRN2, heads=heads, kv_heads=heads, dim=dim, vdim=vdim, head_pad=dp, vhead_pad=vp, n_att=n_att, w_in=w_in, b_in=from_numpy(b),
+                   lower=from_numpy(_pad_heads(_host_f32(lower).reshape(1, -1), heads, dp, 1.0)), o_norm=_row(head_norm, vp),
+                   w_o=_head_cols(o, heads, vdim, vp, wp, n_att))
+        return out
+
+    @classmethod
+    def _pack_block(cls, b, c) -> dict:
+        from pygpukit_amd.llm.layers import GatedRecurrence, GatedWindowAttention, LatentAttention
+
+        a = b.attn
+        if b.post_attn_norm is None or (b.mlp is not None and b.post_mlp_norm is None):
+            raise NotImplementedError("the layer-list engine needs a norm after each sublayer")
+        if b.residual_mult != c.residual_mult or b.post_attn_norm.eps != c.norm_eps:
+            raise NotImplementedError("the layer-list engine takes one residual factor and one norm epsilon for all layers")
+        weight = lambda n: None if n is None else n.weight  # noqa: E731
+        common = {}
+        if b.mlp is not None:
+            xielu = b.mlp.activation == "xielu"
+            if not xielu and b.mlp.gate_up_proj is None:
+                raise NotImplementedError("the layer-list engine needs a fused gate / up weight")
+            common = dict(gate_up=b.mlp.fc1.weight if xielu else b.mlp.gate_up_proj.weight, down=b.mlp.fc2.weight if xielu else b.mlp.down_proj.weight,
+                          norm2=weight(b.mlp_norm), norm2b=b.post_mlp_norm.weight, act_params=b.mlp.act_params if xielu else None)
+        norms = (weight(b.attn_norm), b.post_attn_norm.weight)
+        if isinstance(a, LatentAttention):
+            if a.head_gate is None or b.attn_norm is None:
+                raise NotImplementedError("the layer-list engine needs a norm before gated latent attention")
+            return cls.pack_layer(a.q_proj.weight, a.kv_down.weight, a.head_gate.weight, a.kv_norm.weight, a.k_up.weight, a.v_up.weight, a.o_proj.weight, *norms,
+                                  heads=a.num_heads, dim=a.head_dim, vdim=a.v_head_dim, window=a.window, scale=a.scale, **common)
+        if isinstance(a, GatedWindowAttention):
+            own = a.source is None
+            return cls.pack_attention(a.q_proj.weight, a.k_proj.weight if own else None, a.v_proj.weight if own else None, a.out_gate.weight, a.o_proj.weight, *norms,
+                                      heads=a.num_heads, kv_heads=a.num_kv_heads, dim=a.head_dim, vdim=a.v_head_dim, window=a.window, scale=a.scale,
+                                      biases=(a.q_proj.bias, a.k_proj.bias, a.v_proj.bias) if own else (a.q_proj.bias,),
+                                      convs=(a.q_conv, a.k_conv, a.v_conv) if own else (a.q_conv,), q_norm=weight(a.q_norm), k_norm=weight(a.k_norm), slopes=a.slopes,
+                                      kv_from=a.kv_from, **common)
+        if isinstance(a, GatedRecurrence):
+            return cls.pack_recurrence(a.q_proj.weight, a.forget_proj.weight, a.v_proj.weight, a.o_proj.weight, a.forget_bias, a.lower, a.head_norm, *norms,
+                                       heads=a.num_heads, dim=a.head_dim, vdim=a.v_head_dim, **common)
+        raise NotImplementedError(f"the layer-list engine has no {type(a).__name__}")
 
     @classmethod
     def from_model(cls, model, *, max_seq_len: int = 512, max_batch: int = 1) -> "StackEngine":
@@ -373,35 +530,36 @@ class StackEngine(Engine):
         width = model.embed_tokens.shape[1]
         packed = model.__dict__.get("_stack_layers")       # packed once, shared by every engine of this model
         if packed is None:
-            packed = []
-            for b in model.blocks:
-                a = b.attn
-                if a.head_gate is None or b.post_attn_norm is None or (b.mlp is not None and (b.post_mlp_norm is None or b.mlp.gate_up_proj is None)):
-                    raise NotImplementedError("the layer-list engine needs gated latent attention, post-norms and a fused gate / up weight")
-                if b.residual_mult != c.residual_mult or b.attn_norm.eps != c.norm_eps:
-                    raise NotImplementedError("the layer-list engine takes one residual factor and one norm epsilon for all layers")
-                mlp = {} if b.mlp is None else dict(gate_up=b.mlp.gate_up_proj.weight, down=b.mlp.down_proj.weight, norm2=b.mlp_norm.weight,
-                                                    norm2b=b.post_mlp_norm.weight)
-                packed.append(cls.pack_layer(a.q_proj.weight, a.kv_down.weight, a.head_gate.weight, a.kv_norm.weight, a.k_up.weight, a.v_up.weight,
-                                             a.o_proj.weight, b.attn_norm.weight, b.post_attn_norm.weight, heads=a.num_heads, dim=a.head_dim,
-                                             vdim=a.v_head_dim, window=a.window, scale=a.scale, **mlp))
+            packed = [cls._pack_block(b, c) for b in model.blocks]
             head = model._lm_head if model._lm_head is not None else model.embed_tokens
             wp = _up64(width)
             model._stack_layers = packed
-            model._stack_head = (pad_2d(head, head.shape[0], wp), pad_2d(model.final_norm.weight.view((1, width)), 1, wp))
+            model._stack_head = (pad_2d(head, head.shape[0], wp), _row(model.final_norm.weight, wp))
         head, fnorm = model._stack_head
         cfg = dict(vocab_size=model.embed_tokens.shape[0], width=width, hidden_size=width, max_positions=c.max_position_embeddings, norm_eps=c.norm_eps,
                    residual_mult=c.residual_mult)
         return cls(cfg, model.embed_tokens, model.position_embed, head, fnorm, packed, max_seq_len=max_seq_len, max_batch=max_batch)
 
-    def latent_cache(self, layer: int) -> GPUArray:
-        """[max_batch, R, rank_pad] view of layer `layer`'s latent rings: position p of a sequence is row p % R, R = min(window, max_seq_len)."""
+    def _layer_memory(self, layer: int, shape: tuple[int, ...], dtype) -> GPUArray:
         p, none = C.c_void_p(), C.c_void_p()
         _hip.call("pgk_engine_kv_ptr", self.handle, layer, C.byref(p), C.byref(none))
-        lw = self.layers[layer]
-        a = GPUArray((self.max_batch, min(lw["window"], self.max_seq_len), lw["rank_pad"]), self.dtype, p.value, owns_memory=False)
+        a = GPUArray(shape, dtype, p.value, owns_memory=False)
         a._source_ref = self
         return a
 
+    def latent_cache(self, layer: int) -> GPUArray:
+        """[max_batch, R, rank_pad] view of layer `layer`'s latent rings: position p of a sequence is row p % R, R = min(window, max_seq_len)."""
+        lw = self.layers[layer]
+        if lw["mixer"] != _hip.MIX_LATENT:
+            raise ValueError(f"layer {layer} caches no latents")
+        return self._layer_memory(layer, (self.max_batch, min(lw["window"], self.max_seq_len), lw["rank_pad"]), self.dtype)
+
+    def recurrent_state(self, layer: int) -> GPUArray:
+        """float32 [max_batch, heads, dim, vdim] (widths padded) view of layer `layer`'s states."""
+        lw = self.layers[layer]
+        if lw["mixer"] != _hip.MIX_HGRN2:
+            raise ValueError(f"layer {layer} has no recurrent state")
+        return self._layer_memory(layer, (self.max_batch, lw["heads"], lw["head_pad"], lw["vhead_pad"]), float32)
+
     def kv_cache(self, layer: int):
-        raise NotImplementedError("a layer-list engine caches latents, not keys and values: latent_cache()")
+        raise NotImplementedError("a layer-list engine's caches are rings and states: latent_cache(), recurrent_state()")

@@ -1,4 +1,4 @@
-"""MLP layer (reference: src/pygpukit/llm/layers/mlp.py:25-98): GELU (fc1 -> gelu -> fc2) or SwiGLU
+"""MLP layer (reference: src/pygpukit/llm/layers/mlp.py:25-98): GELU (fc1 -> gelu -> fc2), xIELU in its place, or SwiGLU
 (silu(gate) * up -> down).  With raw bf16 weights gate and up are fused into ONE [2I, H] weight
 (mlp.py:84-86); here gate_proj / up_proj are zero-copy row views of that fused weight, so the bytes exist
 once, and the forward is one projection + one packed GLU kernel + the down projection."""
@@ -8,7 +8,7 @@ from __future__ import annotations
 from typing import TYPE_CHECKING
 
 from pygpukit_amd.core.array import GPUArray
-from pygpukit_amd.ops.basic import concat_axis0, gelu, glu_packed, swiglu
+from pygpukit_amd.ops.basic import concat_axis0, gelu, glu_packed, swiglu, xielu
 
 from .linear import LinearBF16, LinearFP8
 
@@ -24,12 +24,18 @@ def _wrap(proj, bias=None):
 
 class MLP:
     def __init__(self, config: "TransformerConfig", fc1_weight=None, fc1_bias: GPUArray | None = None, fc2_weight=None,
-                 fc2_bias: GPUArray | None = None, gate_proj=None, up_proj=None, down_proj=None):
+                 fc2_bias: GPUArray | None = None, gate_proj=None, up_proj=None, down_proj=None,
+                 act_params: tuple[float, float] | None = None):
+        """act_params: xIELU's two factors (of z^2 and of exp(z) - 1 - z)."""
         self.config = config
         self.activation = config.activation
-        if config.activation == "gelu":
+        self.gate_up_proj: LinearBF16 | None = None
+        if config.activation in ("gelu", "xielu"):
             if fc1_weight is None or fc2_weight is None:
-                raise ValueError("GELU MLP requires fc1_weight and fc2_weight")
+                raise ValueError(f"{config.activation} MLP requires fc1_weight and fc2_weight")
+            if (act_params is not None) != (config.activation == "xielu"):
+                raise ValueError("act_params are xIELU's")
+            self.act_params = act_params
             self.fc1, self.fc2 = _wrap(fc1_weight, fc1_bias), _wrap(fc2_weight, fc2_bias)
             return
         if gate_proj is None or up_proj is None or down_proj is None:
@@ -38,12 +44,11 @@ class MLP:
         if isinstance(gate_proj, GPUArray) and isinstance(up_proj, GPUArray):
             inter, hidden = gate_proj.shape
             fused = concat_axis0(gate_proj, up_proj)
-            self.gate_up_proj: LinearBF16 | None = LinearBF16(fused, None)
+            self.gate_up_proj = LinearBF16(fused, None)
             self.gate_proj = LinearBF16(fused._view(0, (inter, hidden)))
             self.up_proj = LinearBF16(fused._view(inter * hidden, (inter, hidden)))
             self.intermediate_size = inter
         else:
-            self.gate_up_proj = None
             self.gate_proj, self.up_proj = _wrap(gate_proj), _wrap(up_proj)
             self.intermediate_size = self.gate_proj.out_features
 
@@ -51,6 +56,9 @@ class MLP:
         if self.activation == "gelu":
             h = self.fc1(x)
             return self.fc2(gelu(h, out=h))
+        if self.activation == "xielu":
+            h = self.fc1(x)
+            return self.fc2(xielu(h, *self.act_params, out=h))
         if self.gate_up_proj is not None:
             act = glu_packed(self.gate_up_proj(x), self.intermediate_size)
         else:

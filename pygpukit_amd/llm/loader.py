@@ -15,9 +15,9 @@ import numpy as np
 from pygpukit_amd.core.array import GPUArray
 from pygpukit_amd.core.dtypes import bfloat16, float16, float32, uint8
 from pygpukit_amd.core.factory import from_numpy
-from pygpukit_amd.llm.config import (GPT2_SPEC, LLAMA_SPEC, QWEN3_SPEC, TOTOLORN_SPEC, ModelSpec, TransformerConfig, detect_model_spec,
-                                     layer_list_config)
-from pygpukit_amd.llm.layers import MLP, Attention, LatentAttention, Norm, TransformerBlock
+from pygpukit_amd.llm.config import (GPT2_SPEC, LLAMA_SPEC, MALASUN_SPEC, QWEN3_SPEC, TOTOLORN_SPEC, LayerConfig, ModelSpec, TransformerConfig,
+                                     detect_model_spec, distance_slopes, layer_list_config)
+from pygpukit_amd.llm.layers import MLP, Attention, GatedRecurrence, GatedWindowAttention, LatentAttention, Norm, TransformerBlock
 from pygpukit_amd.llm.layers.linear import LinearBF16, LinearFP8
 from pygpukit_amd.llm.models.causal import CausalTransformerModel
 from pygpukit_amd.llm.safetensors import Dtype, load_safetensors
@@ -117,7 +117,7 @@ def load_model_from_safetensors(model_path: str, dtype: str = "bfloat16", spec: 
     def nm(pattern: str | None, layer: int) -> str | None:
         return None if pattern is None else pattern.format(layer=layer)
 
-    if spec.kv_down_proj is not None:
+    if spec.architecture:
         return _load_layer_list(st, spec, hf_config, target_dt, load_tensor, try_load)
 
     embed_info = st.tensor_info(spec.embed_tokens)
@@ -214,31 +214,71 @@ def _load_layer_list(st, spec: ModelSpec, config: dict, dtype, load_tensor, try_
             raise ValueError(f"{name}: shape {got}, config.json says {shape}")
         return load_tensor(name)
 
-    def norm(name: str, width: int, offset: float) -> Norm:
-        if name not in st or tuple(st.tensor_info(name).shape) != (width,):
-            raise ValueError(f"{name}: missing or not of width {width}")
-        w = st.tensor_as_f32(name) + np.float32(offset)
-        return Norm(from_numpy(np.ascontiguousarray(w, dtype=np.float32)), None, "rmsnorm", cfg.norm_eps, stream_dtype=dtype)
+    def fp32(name: str, size: int) -> np.ndarray:
+        if name not in st or int(np.prod(st.tensor_info(name).shape)) != size:
+            raise ValueError(f"{name}: missing or not of {size} elements")
+        return np.ascontiguousarray(st.tensor_as_f32(name), dtype=np.float32).reshape(size)
 
-    H, off = cfg.hidden_size, spec.norm_weight_offset
-    blocks = []
-    for i, lc in enumerate(cfg.layers):
-        nm = lambda pattern: pattern.format(layer=i)  # noqa: E731, B023
-        attn = LatentAttention(tensor(nm(spec.q_proj), (lc.num_heads * lc.head_dim, H)), tensor(nm(spec.kv_down_proj), (lc.kv_rank, H)),
+    def norm(name: str, width: int, offset: float, scalar: bool = False) -> Norm:
+        w = np.repeat(fp32(name, 1), width) if scalar else fp32(name, width)
+        return Norm(from_numpy(w + np.float32(offset)), None, "rmsnorm", cfg.norm_eps, stream_dtype=dtype)
+
+    H, off, one = cfg.hidden_size, spec.norm_weight_offset, spec.norm_scalar
+    blocks: list[TransformerBlock] = []
+
+    def latent_mixer(lc: LayerConfig, nm) -> LatentAttention:
+        return LatentAttention(tensor(nm(spec.q_proj), (lc.num_heads * lc.head_dim, H)), tensor(nm(spec.kv_down_proj), (lc.kv_rank, H)),
                                norm(nm(spec.kv_down_norm), lc.kv_rank, 0.0), tensor(nm(spec.k_up_proj), (lc.num_heads * lc.head_dim, lc.kv_rank)),
                                tensor(nm(spec.v_up_proj), (lc.num_heads * lc.v_head_dim, lc.kv_rank)),
                                tensor(nm(spec.o_proj), (H, lc.num_heads * lc.v_head_dim)), num_heads=lc.num_heads, head_dim=lc.head_dim,
                                v_head_dim=lc.v_head_dim, scale=lc.scale, window=lc.window, head_gate=tensor(nm(spec.head_gate), (lc.num_heads, H)))
+
+    def attention_mixer(lc: LayerConfig, nm) -> GatedWindowAttention:
+        q, k, v = lc.num_heads * lc.head_dim, lc.num_kv_heads * lc.head_dim, lc.num_kv_heads * lc.v_head_dim
+        own = lc.kv_from is None
+
+        def proj(weight: str, bias: str, rows: int) -> LinearBF16:
+            return LinearBF16(tensor(nm(weight), (rows, H)), tensor(nm(bias), (rows,)))
+
+        def conv(name: str, rows: int) -> GPUArray | None:
+            return None if lc.conv_taps is None else tensor(nm(name), (rows, lc.conv_taps))
+
+        return GatedWindowAttention(
+            proj(spec.q_proj, spec.q_bias, q), proj(spec.k_proj, spec.k_bias, k) if own else None, proj(spec.v_proj, spec.v_bias, v) if own else None,
+            tensor(nm(spec.o_proj), (H, lc.num_heads * lc.v_head_dim)), tensor(nm(spec.out_gate), (lc.num_heads * lc.v_head_dim, H)), num_heads=lc.num_heads,
+            num_kv_heads=lc.num_kv_heads, head_dim=lc.head_dim, v_head_dim=lc.v_head_dim, scale=lc.scale, window=lc.window, q_norm=norm(nm(spec.q_norm), q, 0.0),
+            k_norm=norm(nm(spec.k_norm), k, 0.0) if own else None, q_conv=conv(spec.q_conv, q), k_conv=conv(spec.k_conv, k) if own else None,
+            v_conv=conv(spec.v_conv, v) if own else None, slopes=from_numpy(np.asarray(distance_slopes(lc.num_heads), np.float32)),
+            source=None if own else blocks[lc.kv_from].attn, kv_from=lc.kv_from)
+
+    def recurrent_mixer(lc: LayerConfig, nm) -> GatedRecurrence:
+        qk, v = lc.num_heads * lc.head_dim, lc.num_heads * lc.v_head_dim
+        return GatedRecurrence(tensor(nm(spec.q_proj), (qk, H)), tensor(nm(spec.forget_proj), (qk, H)), tensor(nm(spec.v_proj), (v, H)), tensor(nm(spec.o_proj), (H, v)),
+                               from_numpy(fp32(nm(spec.forget_bias), qk)), from_numpy(fp32(nm(spec.forget_lower), qk)), from_numpy(fp32(nm(spec.head_norm), lc.v_head_dim)),
+                               num_heads=lc.num_heads, head_dim=lc.head_dim, v_head_dim=lc.v_head_dim, eps=cfg.norm_eps)
+
+    mixers = {"latent_attention": (latent_mixer, spec.kv_down_proj), "attention": (attention_mixer, spec.out_gate), "hgrn2": (recurrent_mixer, spec.forget_proj)}
+    for i, lc in enumerate(cfg.layers):
+        nm = lambda pattern: pattern.format(layer=i)  # noqa: E731, B023
+        make, known = mixers[lc.mixer]
+        if known is None:
+            raise ValueError(f"layer {i}: {spec.name} models have no {lc.mixer} layers")
         mlp = mlp_norm = post_mlp = None
+        attn = make(lc, nm)
         if lc.intermediate_size is not None:
             I = lc.intermediate_size
-            mlp = MLP(cfg, gate_proj=tensor(nm(spec.gate_proj), (I, H)), up_proj=tensor(nm(spec.up_proj), (I, H)), down_proj=tensor(nm(spec.down_proj), (H, I)))
-            mlp_norm, post_mlp = norm(nm(spec.mlp_norm), H, off), norm(nm(spec.post_mlp_norm), H, off)
-        blocks.append(TransformerBlock(norm(nm(spec.attn_norm), H, off), attn, mlp_norm, mlp, norm(nm(spec.post_attn_norm), H, off), post_mlp,
-                                       cfg.residual_mult))
+            if spec.activation == "xielu":
+                p, q = (float(x) for x in np.logaddexp(0.0, fp32(nm(spec.act_params), 2).astype(np.float64)))
+                mlp = MLP(cfg, fc1_weight=tensor(nm(spec.fc1), (I, H)), fc2_weight=tensor(nm(spec.fc2), (H, I)), act_params=(p, 0.5 + q))
+            else:
+                mlp = MLP(cfg, gate_proj=tensor(nm(spec.gate_proj), (I, H)), up_proj=tensor(nm(spec.up_proj), (I, H)), down_proj=tensor(nm(spec.down_proj), (H, I)))
+            mlp_norm = norm(nm(spec.mlp_norm), H, off, one) if spec.mlp_norm else None
+            post_mlp = norm(nm(spec.post_mlp_norm), H, off, one)
+        blocks.append(TransformerBlock(norm(nm(spec.attn_norm), H, off, one) if spec.attn_norm else None, attn, mlp_norm, mlp,
+                                       norm(nm(spec.post_attn_norm), H, off, one), post_mlp, cfg.residual_mult))
     lm_head = tensor(spec.lm_head, (cfg.vocab_size, H)) if spec.lm_head in st else None
-    return CausalTransformerModel(cfg, tensor(spec.embed_tokens, (cfg.vocab_size, H)), blocks, norm(spec.final_norm, H, off), lm_head,
-                                  tensor(spec.position_embed, (cfg.max_position_embeddings, H)), spec)
+    pos = tensor(spec.position_embed, (cfg.max_position_embeddings, H)) if spec.use_position_embed else None
+    return CausalTransformerModel(cfg, tensor(spec.embed_tokens, (cfg.vocab_size, H)), blocks, norm(spec.final_norm, H, off, one), lm_head, pos, spec)
 
 
 def _bf16_array(bits: np.ndarray) -> GPUArray:
@@ -270,5 +310,9 @@ def load_totolorn_from_safetensors(model_path: str, dtype: str = "bfloat16") -> 
     return load_model_from_safetensors(model_path, dtype=dtype, spec=TOTOLORN_SPEC)
 
 
-__all__ = ["load_totolorn_from_safetensors", "load_model_from_safetensors", "load_gpt2_from_safetensors", "load_llama_from_safetensors", "load_qwen3_from_safetensors",
+def load_malasun_from_safetensors(model_path: str, dtype: str = "bfloat16") -> CausalTransformerModel:
+    return load_model_from_safetensors(model_path, dtype=dtype, spec=MALASUN_SPEC)
+
+
+__all__ = ["load_malasun_from_safetensors", "load_totolorn_from_safetensors", "load_model_from_safetensors", "load_gpt2_from_safetensors", "load_llama_from_safetensors", "load_qwen3_from_safetensors",
            "FP8QuantConfig"]

@@ -71,14 +71,16 @@ class CausalTransformerModel:
         seq_len = len(input_ids)
         if position_ids is None:
             past_len = 0
-            if past_key_values is not None and past_key_values[0] is not None:
-                past_len = past_key_values[0][0].shape[0]
+            if past_key_values is not None:
+                past_len = next((p[0].shape[0] for b, p in zip(self.blocks, past_key_values) if p is not None and getattr(b.attn, "cache_rows", True)), 0)
             position_ids = list(range(past_len, past_len + seq_len))
         hidden = self._embed(input_ids, position_ids)
         present = []
+        sources = {getattr(b.attn, "kv_from", None) for b in self.blocks}
         for i, block in enumerate(self.blocks):
             past_kv = past_key_values[i] if past_key_values else None
-            hidden, kv = block(hidden, position_ids, past_kv, use_cache)
+            src = getattr(block.attn, "kv_from", None)
+            hidden, kv = block(hidden, position_ids, past_kv, use_cache or i in sources, None if src is None else present[src])
             present.append(kv)
         hidden = self.final_norm(hidden)
         return (hidden, present) if use_cache else (hidden, None)
@@ -223,5 +225,6 @@ GPT2Model = CausalTransformerModel
 LlamaModel = CausalTransformerModel
 QwenModel = CausalTransformerModel
 TotolornModel = CausalTransformerModel
+MalasunModel = CausalTransformerModel
 
-__all__ = ["CausalTransformerModel", "GPT2Model", "LlamaModel", "QwenModel", "TotolornModel"]
+__all__ = ["CausalTransformerModel", "GPT2Model", "LlamaModel", "QwenModel", "TotolornModel", "MalasunModel"]

@@ -35,3 +35,11 @@ def tanh(a: GPUArray, *, out: GPUArray | None = None) -> GPUArray:
 
 def relu2(a: GPUArray, *, out: GPUArray | None = None) -> GPUArray:
     return _act(a, "relu2", out)
+
+
+def xielu(a: GPUArray, pos: float, neg: float, *, out: GPUArray | None = None) -> GPUArray:
+    """z > 0: pos * z^2 + z / 2;  z <= 0: neg * (exp(z) - 1 - z) + z / 2.  `out` may alias the input."""
+    validate_float(a, "xielu")
+    o = check_out(out, a.shape, a.dtype, "xielu")
+    call("pgk_xielu", a._p, o._p, a.size, float(pos), float(neg), a.dtype.code, None)
+    return o

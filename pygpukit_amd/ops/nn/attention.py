@@ -82,9 +82,10 @@ def sdpa_causal_fixed_cache_ptr(Q: GPUArray, K: GPUArray, V: GPUArray, out: GPUA
 
 
 def window_attention(q: GPUArray, k: GPUArray, v: GPUArray, scale: float, window: int, *, gate: GPUArray | None = None,
-                     out: GPUArray | None = None) -> GPUArray:
+                     slopes: GPUArray | None = None, out: GPUArray | None = None) -> GPUArray:
     """q [q_len, Hq, dk], k [kv_len, Hkv, dk], v [kv_len, Hkv, dv] -> [q_len, Hq, dv]: query i is position kv_len - q_len + i and sees the
-    `window` positions that end with its own.  gate [q_len, Hq]: head outputs are multiplied by its sigmoid."""
+    `window` positions that end with its own.  gate [q_len, Hq] or [q_len, Hq, dv]: head outputs (or their elements) are multiplied by
+    its sigmoid.  slopes float32 [Hq]: slope * distance is taken off the scaled score."""
     validate_float(q, "window_attention")
     if q.ndim != 3 or k.ndim != 3 or v.ndim != 3 or k.dtype != q.dtype or v.dtype != q.dtype:
         raise ValueError("window_attention expects q, k, v as [seq, heads, width] of one dtype")
@@ -93,11 +94,14 @@ def window_attention(q: GPUArray, k: GPUArray, v: GPUArray, scale: float, window
         raise ValueError(f"window_attention: shapes {q.shape}, {k.shape}, {v.shape} do not match")
     if window < 1:
         raise ValueError(f"window_attention: window {window}")
-    if gate is not None and (gate.shape != (q_len, hq) or gate.dtype != q.dtype):
-        raise ValueError("window_attention: gate must be [q_len, Hq] in q's dtype")
+    if gate is not None and (gate.shape not in ((q_len, hq), (q_len, hq, dv)) or gate.dtype != q.dtype):
+        raise ValueError("window_attention: gate must be [q_len, Hq] or [q_len, Hq, dv] in q's dtype")
+    if slopes is not None and (slopes.shape != (hq,) or slopes.dtype != float32):
+        raise ValueError("window_attention: slopes must be float32 [Hq]")
+    each = gate is not None and gate.ndim == 3
     o = check_out(out, (q_len, hq, dv), q.dtype, "window_attention")
     call("pgk_window_attention", q._p, k._p, v._p, o._p, hq, hkv, q_len, kv_len, dk, dv, float(scale), min(int(window), 2**30),
-         gate._p if gate is not None else None, hq, q.dtype.code, None)
+         gate._p if gate is not None else None, hq * dv if each else hq, int(each), slopes._p if slopes is not None else None, q.dtype.code, None)
     return o
 
 
@@ -107,4 +111,13 @@ def head_gate(x: GPUArray, gate: GPUArray) -> GPUArray:
     if x.ndim != 3 or gate.shape != x.shape[:2] or gate.dtype != x.dtype:
         raise ValueError(f"head_gate: x {x.shape} and gate {gate.shape} do not match")
     call("pgk_head_gate", x._p, gate._p, x.shape[0], x.shape[1], x.shape[2], x.shape[1], x.dtype.code, None)
+    return x
+
+
+def sigmoid_mul(x: GPUArray, gate: GPUArray) -> GPUArray:
+    """x *= sigmoid(gate), element by element, in place."""
+    validate_float(x, "sigmoid_mul")
+    if gate.shape != x.shape or gate.dtype != x.dtype:
+        raise ValueError(f"sigmoid_mul: x {x.shape} and gate {gate.shape} do not match")
+    call("pgk_sigmoid_mul", x._p, gate._p, x.size, x.dtype.code, None)
     return x
