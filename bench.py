@@ -117,31 +117,39 @@ def cpu_baseline(cfg, weights, prompt, n_decode: int) -> dict:
 
 
 DESIGN_SIZES = {
-    # width, heads, head width, latent, window, ff, layers, and the dense neighbour's kv heads
+    # width, heads, head width, latent (Totolorn), window, ff, layers, and the kv heads of Malasun and the dense engine
     "w1024": dict(width=1024, heads=16, dim=128, rank=256, window=1024, ff=3072, layers=8, kv_heads=8),
     "w2048": dict(width=2048, heads=16, dim=128, rank=512, window=2048, ff=6144, layers=8, kv_heads=8),
     "w4096": dict(width=4096, heads=32, dim=128, rank=512, window=4096, ff=14336, layers=4, kv_heads=8),
 }
 
 
-def stack_kernel_bytes(z: dict, vocab: int, ctx: int, B: int) -> dict:
-    """Algorithmic bytes per decode step and layer of each kernel class of a layer-list engine (bf16 weights and latents, fp32 rows)."""
-    W, F, hd, r, n = z["width"], z["ff"], z["heads"] * z["dim"], z["rank"], min(ctx, z["window"])
-    return {"norm_qkv": (hd + r + z["heads"]) * W * 2 + B * 4 * (2 * W + hd + r), "attn": 2 * hd * r * 2 + B * (n * r * 2 + 8 * hd + 4 * r),
-            "oproj": hd * W * 2 + B * 4 * (hd + W), "gateup": 2 * F * W * 2 + B * 4 * (2 * W + F), "down": F * W * 2 + B * 4 * (F + W),
-            "lmhead": vocab * W * 2 + B * 4 * (W + vocab)}
+def stack_kernel_bytes(kind: str, z: dict, vocab: int, ctx: int, B: int) -> dict:
+    """Algorithmic bytes of ONE decode step of a layer-list engine by kernel class (bf16 weights and caches, fp32 rows and states)."""
+    W, F, H, D, L, n = z["width"], z["ff"], z["heads"], z["dim"], z["layers"], min(ctx, z["window"])
+    hd, gd, r = H * D, z["kv_heads"] * D, z["rank"]
+    out = {"oproj": L * (hd * W * 2 + B * 4 * (hd + W)), "down": L * (F * W * 2 + B * 4 * (F + W)), "lmhead": vocab * W * 2 + B * 4 * (W + vocab)}
+    if kind == "totolorn":
+        out.update(norm_qkv=L * ((hd + r + H) * W * 2 + B * 4 * (2 * W + hd + r)), attn=L * (2 * hd * r * 2 + B * (n * r * 2 + 8 * hd + 4 * r)),
+                   gateup=L * (2 * F * W * 2 + B * 4 * (2 * W + F)))
+        return out
+    A = L // 2                      # attention layers; as many recurrent ones
+    n_in = {"attention": 2 * hd + 2 * gd, "hgrn2": 3 * hd}
+    out.update(norm_qkv=A * sum(w * W * 2 + B * 4 * (2 * W + w) for w in n_in.values()), gateup=L * (F * W * 2 + B * 4 * (2 * W + F)),
+               attn=A * (4 * 4 * (hd + 2 * gd) + B * (n * gd * 2 * 2 + 4 * (2 * n_in["attention"] + hd))), recur=A * B * (2 * hd * D * 4 + 4 * 4 * hd))
+    return out
 
 
 def design_leg(name: str, sizes: list[str], seed: int) -> dict:
-    """--design totolorn: prefill and decode of the layer-list engine at sizes that resemble a real model's layers (random weights), beside
-    the dense QKV + RoPE engine (its closest relative here) at equal width, heads, feed-forward, depth and vocabulary."""
+    """--design totolorn | malasun: prefill and decode of the layer-list engine at sizes that resemble a real model's layers (random
+    weights), beside its closest relatives here at equal width, heads, feed-forward width, depth and vocabulary: the dense QKV + RoPE
+    engine, and for Malasun (every other layer attention, the others recurrent) Totolorn too."""
     from pygpukit_amd import _hip
     from pygpukit_amd.core.factory import from_numpy
     from pygpukit_amd.llm import synthetic as S
+    from pygpukit_amd.llm.config import distance_slopes
     from pygpukit_amd.llm.engine import Engine, StackEngine
 
-    if name != "totolorn":
-        raise SystemExit(f"unknown design {name}")
     V = 32000
     out = {"design": name, "vocab": V, "dtype": "bf16", "data": "synthetic", "sizes": {}}
 
@@ -161,7 +169,7 @@ def design_leg(name: str, sizes: list[str], seed: int) -> dict:
 
     for size in sizes:
         z = DESIGN_SIZES[size]
-        W, H, D, r, F, L = z["width"], z["heads"], z["dim"], z["rank"], z["ff"], z["layers"]
+        W, H, G, D, r, F, L = z["width"], z["heads"], z["kv_heads"], z["dim"], z["rank"], z["ff"], z["layers"]
         rng = np.random.default_rng(seed)
 
         def draw(*shape):
@@ -169,19 +177,36 @@ def design_leg(name: str, sizes: list[str], seed: int) -> dict:
             w *= np.float32(0.02)
             return from_numpy(S.f32_to_bf16_bits(w).reshape(shape))
 
+        def ones(*shape):
+            return from_numpy(np.ones(shape, np.float32))
+
         embed, head, pos = draw(V, W), draw(V, W), draw(4400, W)
-        ones = from_numpy(np.ones((1, W), np.float32))
-        stack, dense = [], []
+        one = ones(1, W)
         b16 = S._bf16(np.ones(W, np.float32))
-        for _ in range(L):
+        totolorn, malasun, dense = [], [], []
+        for l in range(L):
             gu, dn, o = draw(2 * F, W), draw(W, F), draw(W, H * D)
-            stack.append(StackEngine.pack_layer(draw(H * D, W), draw(r, W), draw(H, W), from_numpy(np.ones(r, np.float32)), draw(H * D, r), draw(H * D, r), o, ones,
-                                                ones, heads=H, dim=D, vdim=D, window=z["window"], scale=D**-0.5, gate_up=gu, down=dn, norm2=ones, norm2b=ones))
-            dense.append(dict(attn_norm=b16, mlp_norm=b16, q_norm=None, k_norm=None, w_qkv=draw((H + 2 * z["kv_heads"]) * D, W), w_o=o, w_gate_up=gu, w_down=dn))
+            dense.append(dict(attn_norm=b16, mlp_norm=b16, q_norm=None, k_norm=None, w_qkv=draw((H + 2 * G) * D, W), w_o=o, w_gate_up=gu, w_down=dn))
+            totolorn.append(StackEngine.pack_layer(draw(H * D, W), draw(r, W), draw(H, W), ones(r), draw(H * D, r), draw(H * D, r), o, one, one, heads=H, dim=D, vdim=D,
+                                                   window=z["window"], scale=D**-0.5, gate_up=gu, down=dn, norm2=one, norm2b=one))
+            if name != "malasun":
+                continue
+            ff = dict(gate_up=gu._view(0, (F, W)), down=dn, norm2b=one, act_params=(0.8, 1.2))
+            if l % 2 == 0:
+                widths = (H * D, G * D, G * D)
+                malasun.append(StackEngine.pack_attention(*(draw(w, W) for w in widths), draw(H * D, W), o, None, one, heads=H, kv_heads=G, dim=D, vdim=D,
+                                                          window=z["window"], scale=D**-0.5, biases=tuple(draw(w) for w in widths), convs=tuple(draw(w, 4) for w in widths),
+                                                          q_norm=ones(H * D), k_norm=ones(G * D), slopes=from_numpy(np.asarray(distance_slopes(H), np.float32)), **ff))
+            else:
+                malasun.append(StackEngine.pack_recurrence(*(draw(H * D, W) for _ in range(3)), o, from_numpy(np.full(H * D, 3.0, np.float32)),
+                                                           from_numpy(np.full(H * D, 0.2, np.float32)), ones(D), None, one, heads=H, dim=D, vdim=D, **ff))
         scfg = dict(vocab_size=V, width=W, max_positions=4400, norm_eps=1e-5, residual_mult=0.7)
-        dcfg = dict(vocab_size=V, hidden_size=W, num_layers=L, num_heads=H, num_kv_heads=z["kv_heads"], head_dim=D, intermediate_size=F, norm_eps=1e-5, rope_theta=1e6)
-        make = {"totolorn": lambda ms, mb: StackEngine(scfg, embed, pos, head, ones, stack, max_seq_len=ms, max_batch=mb),
+        dcfg = dict(vocab_size=V, hidden_size=W, num_layers=L, num_heads=H, num_kv_heads=G, head_dim=D, intermediate_size=F, norm_eps=1e-5, rope_theta=1e6)
+        make = {"malasun": lambda ms, mb: StackEngine(dict(scfg, residual_mult=1.0), embed, None, head, one, malasun, max_seq_len=ms, max_batch=mb),
+                "totolorn": lambda ms, mb: StackEngine(scfg, embed, pos, head, one, totolorn, max_seq_len=ms, max_batch=mb),
                 "dense": lambda ms, mb: Engine(dcfg, embed, dense, b16, head, max_seq_len=ms, max_batch=mb, use_qk_norm=False)}
+        if name != "malasun":
+            del make["malasun"]
         res = {"config": z}
         for kind, new in make.items():
             rec = {"prefill": {}, "decode": {}}
@@ -204,11 +229,12 @@ def design_leg(name: str, sizes: list[str], seed: int) -> dict:
                 e.replay(4)
                 ms = wall(lambda: e.replay(8), reps=5) / 8
                 rec["decode"][f"b{B}_ctx{ctx}"] = {"ms": round(ms, 4), "tokens_per_s": round(B / ms * 1e3), "launches": e.launches_per_step()}
-                if B == 1:
-                    prof = e.profile_step(1, 8)
-                    nb = stack_kernel_bytes(z, V, ctx, 1) if kind == "totolorn" else kernel_bytes_per_launch(dcfg, ctx, 1)
+                if B == 1 or kind != "dense":
+                    prof = e.profile_step(B, 8)
+                    nb = stack_kernel_bytes(kind, z, V, ctx, B) if kind != "dense" else {k: v * (1 if k == "lmhead" else L) for k, v in kernel_bytes_per_launch(dcfg, ctx, B).items()}
+                    per = {"lmhead": 1, "attn": L // 2 if kind == "malasun" else L, "recur": L // 2}      # layers that have the class
                     rec["decode"][f"b{B}_ctx{ctx}"]["kernels"] = {
-                        k: {"us_per_layer": round(us * n / (1 if k == "lmhead" else L), 2), "hbm_frac": round(nb[k] / (us * n / (1 if k == "lmhead" else L)) / 1e3 / HBM_PEAK_GBS, 3)}
+                        k: {"us_per_layer": round(us * n / per.get(k, L), 2), "hbm_frac": round(nb[k] / (us * n) / 1e3 / HBM_PEAK_GBS, 3)}
                         for k, (us, n) in prof.items() if n and k in nb and k != "argmax"}
                 del e
             res[kind] = rec
@@ -238,7 +264,7 @@ def main() -> None:
                     help="skip every extra leg (config 4 weak/strong; at N = 1 also context 2048 in bf16 and w8a16, config 5)")
     ap.add_argument("--config4-steps", type=int, default=32)
     ap.add_argument("--layers", type=int, default=0, help="debug only: override the layer count (result is then INVALID)")
-    ap.add_argument("--design", choices=["totolorn"], help="instead of the headline: prefill / decode of a layer-list design beside the dense engine")
+    ap.add_argument("--design", choices=["totolorn", "malasun"], help="instead of the headline: prefill / decode of a layer-list design beside its relatives")
     ap.add_argument("--design-sizes", default="w1024,w2048,w4096", help="with --design: which sizes")
     args = ap.parse_args()
 

@@ -24,7 +24,7 @@ namespace pgk {
 //     when set, each workgroup stores the 100 MHz s_memrealtime value at its first instruction and after its last
 //     barrier into its own 16-byte slot - plain stores to distinct addresses, no atomics, nothing another kernel reads.
 //     pgk_engine_timeline reduces them per launch to first start / last start / first end / last end.
-enum { KC_EMBED = 0, KC_NORM_QKV, KC_ATTN, KC_OPROJ, KC_GATEUP, KC_DOWN, KC_LMHEAD, KC_ARGMAX, KC_COUNT };
+enum { KC_EMBED = 0, KC_NORM_QKV, KC_ATTN, KC_OPROJ, KC_GATEUP, KC_DOWN, KC_LMHEAD, KC_ARGMAX, KC_RECUR, KC_COUNT };
 constexpr int TL_MAXWG = 2048;        // workgroup slots per launch (larger grids stamp their first 2048 workgroups)
 
 struct TLInfo { int cls, nwg; };

@@ -931,7 +931,7 @@ static pgk_status step_one(Engine* e, hipStream_t st, int* launches) {
         a.w = L.w_in; a.N = L.n_in; a.out = s->in32;
         if (pgk_status r = stack_gemv<T, SP_NORM, SE_STORE>(a, st)) return r;
         settle();
-        mark(KC_ATTN);
+        mark(L.mixer == PGK_MIX_HGRN2 ? KC_RECUR : KC_ATTN);
         if (pgk_status r = mix_decode<T, float>(e, l, 1, s->in32, s->a32, st, launches)) return r;
         mark(KC_OPROJ);
         a = StackGemvArgs{};
@@ -1082,7 +1082,7 @@ static pgk_status rows_layers(Stack* s, const RowBufs& b, int n, hipStream_t st,
         mark(KC_NORM_QKV);
         if (pgk_status r = rows_norm(norm_args(s, b, n, *pend, L.norm1, b.x), n, DT, st)) return r;
         if (pgk_status r = rows_in_proj<T>(s, L, P.in, b, n, st)) return r;
-        mark(KC_ATTN);
+        mark(L.mixer == PGK_MIX_HGRN2 ? KC_RECUR : KC_ATTN);
         if (pgk_status r = mix(l)) return r;
         mark(KC_OPROJ);
         if (pgk_status r = rows_out_proj<T>(s, b, b.a, L.w_o, P.o, n, L.n_att, &pend->slabs, st)) return r;
@@ -1228,15 +1228,46 @@ static pgk_status stack_prefill_t(Engine* e, int n_seqs, const int32_t* slots, c
         else if (ke > kv_elems) kv_elems = ke;
         if (ce > c_elems) c_elems = ce;
     }
+    // chunk tables of the recurrent layers, one per chunk length
+    int longest = 0;
+    for (int i = 0; i < n_seqs; ++i) longest = lens[i] > longest ? lens[i] : longest;
+    struct Chunks { int rows = 0; std::vector<RecurChunk> list; std::vector<int32_t> of_seq; size_t o_list = 0, o_seq = 0; };
+    std::vector<Chunks> chunkings;
+    std::vector<int> chunking(c.num_layers, -1);
+    size_t chunk_ws = 0, chunk_tab = 0;
+    for (int l = 0; l < c.num_layers; ++l) {
+        const auto& L = s->layers[l];
+        const int C = L.mixer == PGK_MIX_HGRN2 && longest >= RECUR_CHUNKED_FROM ? recur_chunk_rows(L.head_pad, L.vhead_pad) : 0;
+        if (!C) continue;
+        for (size_t k = 0; k < chunkings.size(); ++k) if (chunkings[k].rows == C) chunking[l] = (int)k;
+        if (chunking[l] < 0) {
+            Chunks t;
+            t.rows = C;
+            for (int i = 0, row = 0; i < n_seqs; row += lens[i++]) {
+                t.of_seq.push_back((int32_t)t.list.size());
+                for (int r = 0; r < lens[i]; r += C) t.list.push_back(RecurChunk{row + r, lens[i] - r < C ? lens[i] - r : C});
+            }
+            t.of_seq.push_back((int32_t)t.list.size());
+            chunking[l] = (int)chunkings.size();
+            chunkings.push_back(t);
+        }
+        const size_t need = recur_chunk_bytes(recur_args(s, l, nullptr, nullptr, n), (int)chunkings[chunking[l]].list.size());
+        if (need > chunk_ws) chunk_ws = need;
+    }
     const int wrows = n_want < 128 ? n_want : 128;
     auto up = [](size_t v) { return (v + 255) & ~(size_t)255; };
     const size_t E = sizeof(T);
     const size_t sizes[] = {(size_t)n * s->Wp * 4, (size_t)n * s->Wp * E, (size_t)n * s->max_in * E, (size_t)n * s->max_att * E, (size_t)n * s->Wp * E,
                             (size_t)n * 2 * s->max_ff * E, (size_t)n * s->max_ff * E, c_elems * E, kv_elems * E, (size_t)wrows * s->Wp * E, (size_t)wrows * c.vocab_size * 4,
-                            s->slab_elems(n, DT == PGK_F32) * 4, (size_t)n * s->max_q * E, own_elems * E};
+                            s->slab_elems(n, DT == PGK_F32) * 4, (size_t)n * s->max_q * E, own_elems * E, chunk_ws};
+    for (auto& t : chunkings) {
+        t.o_list = chunk_tab;
+        t.o_seq = t.o_list + up(t.list.size() * sizeof(RecurChunk));
+        chunk_tab = t.o_seq + up(t.of_seq.size() * 4);
+    }
     size_t need = 0;
     for (size_t z : sizes) need += up(z);
-    const size_t tab_need = up((size_t)n * 4) * 2 + up(place.size() * sizeof(RowPlace)) + up((size_t)n_want * 4) + up((size_t)n * sizeof(RowSrc)) + up(n_seqs * sizeof(SeqSpan));
+    const size_t tab_need = up((size_t)n * 4) * 2 + up(place.size() * sizeof(RowPlace)) + up((size_t)n_want * 4) + up((size_t)n * sizeof(RowSrc)) + up(n_seqs * sizeof(SeqSpan)) + chunk_tab;
     auto grow = [&](void** p, size_t* have, size_t want_bytes) -> pgk_status {
         if (want_bytes <= *have) return PGK_OK;
         if (*p) { PGK_CHECK_HIP(hipStreamSynchronize(st)); pgk_free(*p); }
@@ -1260,10 +1291,11 @@ static pgk_status stack_prefill_t(Engine* e, int n_seqs, const int32_t* slots, c
     b.slabs = (float*)take(sizes[11]);
     b.q = take(sizes[12]);
     T* kv_own = (T*)take(sizes[13]);
+    void* ws_chunk = take(sizes[14]);
     // one host image of the index tables, one copy
     std::vector<char> img(tab_need, 0);
     const size_t o_pos = up((size_t)n * 4), o_place = 2 * o_pos, o_want = o_place + up(place.size() * sizeof(RowPlace)),
-                 o_rows = o_want + up((size_t)n_want * 4), o_seqs = o_rows + up((size_t)n * sizeof(RowSrc));
+                 o_rows = o_want + up((size_t)n_want * 4), o_seqs = o_rows + up((size_t)n * sizeof(RowSrc)), o_chunk = o_seqs + up(n_seqs * sizeof(SeqSpan));
     memcpy(img.data(), tokens, (size_t)n * 4);
     for (int i = 0, row = 0; i < n_seqs; ++i) {
         ((SeqSpan*)(img.data() + o_seqs))[i] = SeqSpan{row, lens[i], starts[i], slots[i]};
@@ -1274,6 +1306,10 @@ static pgk_status stack_prefill_t(Engine* e, int n_seqs, const int32_t* slots, c
     }
     if (!place.empty()) memcpy(img.data() + o_place, place.data(), place.size() * sizeof(RowPlace));
     if (n_want) memcpy(img.data() + o_want, want, (size_t)n_want * 4);
+    for (const auto& t : chunkings) {
+        memcpy(img.data() + o_chunk + t.o_list, t.list.data(), t.list.size() * sizeof(RecurChunk));
+        memcpy(img.data() + o_chunk + t.o_seq, t.of_seq.data(), t.of_seq.size() * 4);
+    }
     PGK_CHECK_HIP(hipMemcpyAsync(s->tab, img.data(), tab_need, hipMemcpyHostToDevice, st));
     PGK_CHECK_HIP(hipStreamSynchronize(st));      // the image is pageable host memory
     const int32_t* d_tok = (const int32_t*)s->tab;
@@ -1343,6 +1379,11 @@ static pgk_status stack_prefill_t(Engine* e, int n_seqs, const int32_t* slots, c
     auto recurrence = [&](int l) -> pgk_status {
         RecurArgs a = recur_args(s, l, b.in, b.a, n);
         a.seqs = d_seqs; a.n_seqs = n_seqs;
+        if (chunking[l] >= 0) {
+            const Chunks& t = chunkings[chunking[l]];
+            const char* tab = (const char*)s->tab + o_chunk;
+            return recur_chunked(a, (const RecurChunk*)(tab + t.o_list), (int)t.list.size(), (const int32_t*)(tab + t.o_seq), ws_chunk, DT, st);
+        }
         return recur_rows(a, DT, DT == PGK_F32, st);
     };
     auto mix = [&](int l) -> pgk_status {

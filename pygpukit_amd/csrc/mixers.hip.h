@@ -88,7 +88,8 @@ struct RecurArgs {
 };
 pgk_status recur_rows(const RecurArgs& a, pgk_dtype dt, bool io32, hipStream_t st);
 size_t recur_chunk_bytes(const RecurArgs& a, int n_chunks);                                     // workspace of the chunked form
-struct RecurChunk { int32_t row0, len, seq, first; };                                           // first: index of its sequence's first chunk
+struct RecurChunk { int32_t row0, len; };
+constexpr int RECUR_CHUNKED_FROM = 16;                                                          // rows of the longest portion from which the chunked form pays
 int recur_chunk_rows(int dim, int vdim);                                                        // rows per chunk; 0: sizes the chunked form does not take
 // the chunked form: chunks in order, sequence by sequence (chunk_of_seq[i] .. chunk_of_seq[i + 1] are sequence i's)
 pgk_status recur_chunked(const RecurArgs& a, const RecurChunk* chunks, int n_chunks, const int32_t* chunk_of_seq, void* ws, pgk_dtype dt, hipStream_t st);

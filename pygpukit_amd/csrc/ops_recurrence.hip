@@ -1,7 +1,17 @@
 // Gated linear recurrence (mixers.hip.h): per head a state S [dim][vdim] in fp32, S <- diag(f) S + (1 - f) v^T, o = S^T q.
 // Gates, state and the head norm are fp32 whatever the element type.
+//
+// Two forms.  Token by token (decode, short portions): one workgroup per sequence and head walks its rows.  Chunked (prompts): rows in
+// chunks of C, all chunks at once -
+//   1. every chunk on its own:  U = sum_j (k_j prod_{t > j} f_t) v_j^T and D = prod_t f_t over its rows         (k = 1 - f)
+//   2. along the chunks of a sequence:  S_c = S before chunk c,  S <- diag(D) S + U
+//   3. every chunk:  o_i = S_c^T (q_i prod_{t <= i} f_t) + sum_{j <= i} A_ij v_j,  A_ij = sum_d q_i k_j prod_{j < t <= i} f_t
+// Decays are products of f over rows, never quotients or differences of logarithms, so a gate near zero costs no accuracy and nothing
+// overflows.  A is built in blocks of 16 rows: off the diagonal from factors that reach to a block's edge (q from the block's start, k to
+// its block's end, whole blocks between), on the diagonal pair by pair.  All products are fp32 (v_mfma_f32_16x16x4_f32).
 
 #include <type_traits>
+#include <vector>
 
 #include "mixers.hip.h"
 
@@ -113,6 +123,373 @@ pgk_status recur_rows(const RecurArgs& a, pgk_dtype dt, bool io32, hipStream_t s
     return dt == PGK_F32 || io32 ? recur_scan<float>(a, st) : recur_scan<bf16>(a, st);
 }
 
+// -------------------------------------------------------------------------------------------- chunks
+typedef float f32x4_rc __attribute__((ext_vector_type(4)));
+__device__ __forceinline__ f32x4_rc mfma4(float a, float b, f32x4_rc c) { return __builtin_amdgcn_mfma_f32_16x16x4f32(a, b, c, 0, 0, 0); }
+
+// LDS row strides (floats; widths are multiples of 16).  Operands whose k index runs over rows want 16 x odd, those whose k index runs
+// along a row want 4 x odd: the 64 lanes of a load then fall on 64 banks.
+__host__ __device__ constexpr int rc_col_stride(int w) { return (w / 16) % 2 ? w : w + 16; }
+__host__ __device__ constexpr int rc_row_stride(int w) { return w + 4; }
+
+static size_t rc_state_lds(int C, int dim, int vdim) { return ((size_t)C * (rc_col_stride(dim) + rc_col_stride(vdim)) + (C / 16) * dim) * 4; }
+static size_t rc_out_lds(int C, int dim) { return ((size_t)3 * C * rc_row_stride(dim) + C * rc_row_stride(C) + (C / 16) * dim + 8 * C) * 4; }
+constexpr size_t RC_LDS_MAX = 156 * 1024;
+
+int recur_chunk_rows(int dim, int vdim) {
+    if (dim % 16 || vdim % 16 || vdim > 512) return 0;
+    for (int C = 64; C >= 32; C /= 2)
+        if (rc_state_lds(C, dim, vdim) <= RC_LDS_MAX && rc_out_lds(C, dim) <= RC_LDS_MAX) return C;
+    return 0;
+}
+size_t recur_chunk_bytes(const RecurArgs& a, int n_chunks) { return (size_t)n_chunks * a.H * ((size_t)a.dim * a.vdim + a.dim) * 4; }
+
+// 1: U [chunk][head][dim][vdim], D [chunk][head][dim]
+template <class T, int C>
+__global__ __launch_bounds__(256) void recur_chunk_state_kernel(RecurArgs a, const RecurChunk* chunks, float* U, float* D) {
+    extern __shared__ __attribute__((aligned(16))) float sm[];
+    constexpr int NS = C / 16;
+    const int dim = a.dim, vdim = a.vdim, ks = rc_col_stride(dim), vs = rc_col_stride(vdim), h = blockIdx.x;
+    float *kr = sm, *v = kr + C * ks, *F = v + C * vs;
+    const RecurChunk ch = chunks[blockIdx.y];
+    const int tid = threadIdx.x, lane = tid & 63, wid = tid >> 6, l15 = lane & 15, q4 = lane >> 4;
+    const T* in = reinterpret_cast<const T*>(a.in) + (size_t)ch.row0 * a.ld_in;
+    // k times the decay to the end of its block of 16 rows, and the blocks' decays
+    for (int t = tid; t < NS * dim; t += 256) {
+        const int b = t / dim, d = t % dim;
+        const T* z = in + a.f_off + h * dim + d;
+        const float bias = a.bias ? a.bias[h * dim + d] : 0.f, low = a.lower[h * dim + d];
+        float zf[16];
+#pragma unroll
+        for (int r = 0; r < 16; ++r) zf[r] = to_f(z[(size_t)min(16 * b + r, ch.len - 1) * a.ld_in]);
+        float run = 1.f;
+#pragma unroll
+        for (int r = 15; r >= 0; --r) {
+            float f, k;
+            rc_gate(zf[r] + bias, low, f, k);
+            const bool live = 16 * b + r < ch.len;
+            kr[(16 * b + r) * ks + d] = live ? k * run : 0.f;
+            run *= live ? f : 1.f;
+        }
+        F[b * dim + d] = run;
+    }
+    for (int t = tid; t < C * vdim / 4; t += 256) {
+        const int r = t / (vdim / 4), c = t % (vdim / 4) * 4;
+        *reinterpret_cast<float4*>(v + r * vs + c) = load4<T>(in + (size_t)min(r, ch.len - 1) * a.ld_in + a.v_off + h * vdim + c);
+    }
+    __syncthreads();
+    const size_t rec = (size_t)blockIdx.y * a.H + h;
+    for (int d = tid; d < dim; d += 256) {
+        float run = 1.f;
+#pragma unroll
+        for (int b = 0; b < NS; ++b) run *= F[b * dim + d];
+        D[rec * dim + d] = run;
+    }
+    float* u = U + rec * dim * vdim;
+    for (int dt = wid; dt < dim / 16; dt += 4) {
+        float m[NS];                                               // decay from a block's end to the chunk's
+        m[NS - 1] = 1.f;
+#pragma unroll
+        for (int b = NS - 2; b >= 0; --b) m[b] = m[b + 1] * F[(b + 1) * dim + 16 * dt + l15];
+        for (int v0 = 0; v0 < vdim; v0 += 128) {
+            f32x4_rc acc[8];
+#pragma unroll
+            for (int t = 0; t < 8; ++t) acc[t] = f32x4_rc{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+            for (int b = 0; b < NS; ++b)
+#pragma unroll
+                for (int s = 0; s < 4; ++s) {
+                    const int j = 16 * b + 4 * s + q4;
+                    const float x = kr[j * ks + 16 * dt + l15] * m[b];
+#pragma unroll
+                    for (int t = 0; t < 8; ++t)
+                        if (v0 + 16 * t < vdim) acc[t] = mfma4(x, v[j * vs + v0 + 16 * t + l15], acc[t]);       // wave-uniform
+                }
+#pragma unroll
+            for (int t = 0; t < 8; ++t)
+                if (v0 + 16 * t < vdim) {
+#pragma unroll
+                    for (int r = 0; r < 4; ++r) u[(size_t)(16 * dt + 4 * q4 + r) * vdim + v0 + 16 * t + l15] = acc[t][r];
+                }
+        }
+    }
+}
+
+// 2: U becomes the state before each chunk, the slot's state moves on
+__global__ __launch_bounds__(256) void recur_chunk_scan_kernel(RecurArgs a, const int32_t* chunk_of_seq, float* U, const float* D) {
+    const int h = blockIdx.y, n4 = a.dim * a.vdim / 4, i = blockIdx.x * 256 + threadIdx.x;
+    if (i >= n4) return;
+    const SeqSpan s = a.seqs[blockIdx.z];
+    const int c0 = chunk_of_seq[blockIdx.z], c1 = chunk_of_seq[blockIdx.z + 1], d = 4 * i / a.vdim;
+    float4* st = reinterpret_cast<float4*>(a.state + ((size_t)s.slot * a.H + h) * a.dim * a.vdim) + i;
+    float4 S = s.start > 0 ? *st : make_float4(0.f, 0.f, 0.f, 0.f);
+    auto at = [&](int c) { return reinterpret_cast<float4*>(U + ((size_t)c * a.H + h) * a.dim * a.vdim) + i; };
+    constexpr int P = 8;                                           // chunks in flight
+    for (int c = c0; c < c1; c += P) {
+        float4 u[P];
+        float w[P];
+#pragma unroll
+        for (int k = 0; k < P; ++k) {
+            const int cc = min(c + k, c1 - 1);
+            u[k] = *at(cc);
+            w[k] = D[((size_t)cc * a.H + h) * a.dim + d];
+        }
+#pragma unroll
+        for (int k = 0; k < P; ++k) {
+            if (c + k >= c1) break;
+            *at(c + k) = S;
+            S.x = fmaf(w[k], S.x, u[k].x); S.y = fmaf(w[k], S.y, u[k].y); S.z = fmaf(w[k], S.z, u[k].z); S.w = fmaf(w[k], S.w, u[k].w);
+        }
+    }
+    *st = S;
+}
+
+// 3: output rows.  Eight waves; NVT column tiles of 16 per wave.
+template <class T, int C, int NVT>
+__global__ __launch_bounds__(512) void recur_chunk_out_kernel(RecurArgs a, const RecurChunk* chunks, const float* U) {
+    extern __shared__ __attribute__((aligned(16))) float sm[];
+    constexpr int NS = C / 16, AS = rc_row_stride(C);
+    const int dim = a.dim, vdim = a.vdim, S = rc_row_stride(dim), h = blockIdx.x;
+    float *q = sm, *f = q + C * S, *k = f + C * S, *A = k + C * S, *F = A + C * AS, *red = F + NS * dim;
+    const RecurChunk ch = chunks[blockIdx.y];
+    const int tid = threadIdx.x, lane = tid & 63, wid = tid >> 6, l15 = lane & 15, q4 = lane >> 4;
+    const T* in = reinterpret_cast<const T*>(a.in) + (size_t)ch.row0 * a.ld_in;
+    for (int t = tid; t < C * dim / 4; t += 512) {
+        const int r = t / (dim / 4), c = t % (dim / 4) * 4, rr = min(r, ch.len - 1);
+        const float4 zq = load4<T>(in + (size_t)rr * a.ld_in + a.q_off + h * dim + c), zf = load4<T>(in + (size_t)rr * a.ld_in + a.f_off + h * dim + c);
+        const float4 b = a.bias ? *reinterpret_cast<const float4*>(a.bias + h * dim + c) : make_float4(0.f, 0.f, 0.f, 0.f);
+        const float4 low = *reinterpret_cast<const float4*>(a.lower + h * dim + c);
+        float4 qq = {zq.x * rc_sigmoid(zq.x), zq.y * rc_sigmoid(zq.y), zq.z * rc_sigmoid(zq.z), zq.w * rc_sigmoid(zq.w)}, ff, kk;
+        rc_gate(zf.x + b.x, low.x, ff.x, kk.x); rc_gate(zf.y + b.y, low.y, ff.y, kk.y);
+        rc_gate(zf.z + b.z, low.z, ff.z, kk.z); rc_gate(zf.w + b.w, low.w, ff.w, kk.w);
+        if (r >= ch.len) { qq = kk = make_float4(0.f, 0.f, 0.f, 0.f); ff = make_float4(1.f, 1.f, 1.f, 1.f); }
+        *reinterpret_cast<float4*>(q + r * S + c) = qq;
+        *reinterpret_cast<float4*>(f + r * S + c) = ff;
+        *reinterpret_cast<float4*>(k + r * S + c) = kk;
+    }
+    __syncthreads();
+    // diagonal blocks, pair by pair: two waves per block, rows 0..7 and 8..15.  Lane: column j = lane & 7 (and j + 8), every eighth
+    // group of 8 channels; w = k_j times the decay from j to the row at hand.
+    if ((wid >> 1) < NS) {
+        const int r0 = 16 * (wid >> 1), half = wid & 1, jl = lane & 7, dg = lane >> 3;
+        float lo[8], hi[8];
+#pragma unroll
+        for (int i = 0; i < 8; ++i) lo[i] = hi[i] = 0.f;
+        for (int c = 8 * dg; c < dim; c += 64) {
+            float wl[8], wh[8];
+            auto row8 = [&](const float* p, float (&x)[8]) {
+                const float4 u = *reinterpret_cast<const float4*>(p), v = *reinterpret_cast<const float4*>(p + 4);
+                x[0] = u.x; x[1] = u.y; x[2] = u.z; x[3] = u.w; x[4] = v.x; x[5] = v.y; x[6] = v.z; x[7] = v.w;
+            };
+            row8(k + (r0 + jl) * S + c, wl);
+            if (half) {
+                row8(k + (r0 + 8 + jl) * S + c, wh);
+#pragma unroll
+                for (int i = 1; i < 8; ++i) {
+                    float g[8];
+                    row8(f + (r0 + i) * S + c, g);
+#pragma unroll
+                    for (int e = 0; e < 8; ++e) wl[e] *= i > jl ? g[e] : 1.f;
+                }
+            }
+#pragma unroll
+            for (int i = 0; i < 8; ++i) {
+                float g[8], x[8];
+                const int row = r0 + 8 * half + i;
+                row8(f + row * S + c, g);
+                row8(q + row * S + c, x);
+                if (half) {
+#pragma unroll
+                    for (int e = 0; e < 8; ++e) {
+                        wl[e] *= g[e];
+                        lo[i] = fmaf(x[e], wl[e], lo[i]);
+                        wh[e] *= i > jl ? g[e] : 1.f;
+                        hi[i] = fmaf(x[e], wh[e], hi[i]);
+                    }
+                } else {
+#pragma unroll
+                    for (int e = 0; e < 8; ++e) {
+                        wl[e] *= i > jl ? g[e] : 1.f;
+                        lo[i] = fmaf(x[e], wl[e], lo[i]);
+                    }
+                }
+            }
+        }
+#pragma unroll
+        for (int i = 0; i < 8; ++i) {
+            float x = lo[i], y = hi[i];
+            x += dpp_f<DPP_ROR8>(x); x += __shfl_xor(x, 16, 64); x += __shfl_xor(x, 32, 64);
+            y += dpp_f<DPP_ROR8>(y); y += __shfl_xor(y, 16, 64); y += __shfl_xor(y, 32, 64);
+            float* row = A + (r0 + 8 * half + i) * AS + r0;
+            if (dg == 0) {
+                row[jl] = half || i >= jl ? x : 0.f;
+                row[8 + jl] = half && i >= jl ? y : 0.f;
+            }
+        }
+    }
+    __syncthreads();
+    // q times the decay from its block's start (its own row included), k times the decay to its block's end
+    for (int t = tid; t < NS * dim; t += 512) {
+        const int b = t / dim, d = t % dim;
+        float g[16], run = 1.f;
+#pragma unroll
+        for (int r = 0; r < 16; ++r) {
+            g[r] = f[(16 * b + r) * S + d];
+            run *= g[r];
+            q[(16 * b + r) * S + d] *= run;
+        }
+        F[b * dim + d] = run;
+        run = 1.f;
+#pragma unroll
+        for (int r = 15; r >= 0; --r) {
+            k[(16 * b + r) * S + d] *= run;
+            run *= g[r];
+        }
+    }
+    __syncthreads();
+    // blocks below the diagonal
+    for (int p = wid; p < NS * (NS - 1) / 2; p += 8) {
+        int bi = 1, bj = p;
+        while (bj >= bi) { bj -= bi; ++bi; }
+        f32x4_rc acc = {0.f, 0.f, 0.f, 0.f};
+        for (int d0 = 0; d0 < dim; d0 += 4) {
+            const int d = d0 + q4;
+            float x = q[(16 * bi + l15) * S + d];
+            for (int b = bj + 1; b < bi; ++b) x *= F[b * dim + d];
+            acc = mfma4(x, k[(16 * bj + l15) * S + d], acc);
+        }
+#pragma unroll
+        for (int r = 0; r < 4; ++r) A[(16 * bi + 4 * q4 + r) * AS + 16 * bj + l15] = acc[r];
+    }
+    __syncthreads();
+    // o = q S + A v: a wave has every row of its column tiles
+    const float* st = U + ((size_t)blockIdx.y * a.H + h) * dim * vdim;
+    f32x4_rc o[NVT][NS];
+#pragma unroll
+    for (int t = 0; t < NVT; ++t)
+#pragma unroll
+        for (int b = 0; b < NS; ++b) o[t][b] = f32x4_rc{0.f, 0.f, 0.f, 0.f};
+    constexpr int SU = 4;                                          // k-steps whose state rows are requested together
+    for (int d0 = 0; d0 < dim; d0 += 4 * SU) {
+        float x[NVT][SU];
+#pragma unroll
+        for (int t = 0; t < NVT; ++t)
+#pragma unroll
+            for (int u = 0; u < SU; ++u) x[t][u] = st[(size_t)(d0 + 4 * u + q4) * vdim + min(16 * (wid + 8 * t), vdim - 16) + l15];
+#pragma unroll
+        for (int u = 0; u < SU; ++u) {
+            const int d = d0 + 4 * u + q4;
+            float m = 1.f;
+#pragma unroll
+            for (int b = 0; b < NS; ++b) {
+                const float y = q[(16 * b + l15) * S + d] * m;
+#pragma unroll
+                for (int t = 0; t < NVT; ++t) o[t][b] = mfma4(y, x[t][u], o[t][b]);
+                m *= F[b * dim + d];
+            }
+        }
+    }
+    const T* v = in + a.v_off + h * vdim;
+#pragma unroll
+    for (int bj = 0; bj < NS; ++bj) {
+        float x[NVT][4];
+#pragma unroll
+        for (int t = 0; t < NVT; ++t)
+#pragma unroll
+            for (int u = 0; u < 4; ++u) x[t][u] = to_f(v[(size_t)min(16 * bj + 4 * u + q4, ch.len - 1) * a.ld_in + min(16 * (wid + 8 * t), vdim - 16) + l15]);
+#pragma unroll
+        for (int b = 0; b < NS; ++b) {
+            if (b < bj) continue;
+#pragma unroll
+            for (int u = 0; u < 4; ++u) {
+                const float y = A[(16 * b + l15) * AS + 16 * bj + 4 * u + q4];
+#pragma unroll
+                for (int t = 0; t < NVT; ++t) o[t][b] = mfma4(y, x[t][u], o[t][b]);
+            }
+        }
+    }
+    // lane: rows 16 b + 4 q4 + r, column l15 of each tile
+    float inv[NS][4];
+#pragma unroll
+    for (int b = 0; b < NS; ++b)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+            float ss = 0.f;
+#pragma unroll
+            for (int t = 0; t < NVT; ++t) ss += 16 * (wid + 8 * t) < vdim ? o[t][b][r] * o[t][b][r] : 0.f;
+            ss = group16_sum(ss);
+            if (l15 == 0) red[wid * C + 16 * b + 4 * q4 + r] = ss;
+        }
+    __syncthreads();
+#pragma unroll
+    for (int b = 0; b < NS; ++b)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+            float ss = 0.f;
+#pragma unroll
+            for (int w = 0; w < 8; ++w) ss += red[w * C + 16 * b + 4 * q4 + r];
+            inv[b][r] = a.norm ? 1.0f / sqrtf(ss / a.vdim_true + a.eps) : 1.0f;
+        }
+    T* out = reinterpret_cast<T*>(a.out) + (size_t)ch.row0 * a.ld_out;
+#pragma unroll
+    for (int t = 0; t < NVT; ++t) {
+        const int c = 16 * (wid + 8 * t) + l15;
+        if (16 * (wid + 8 * t) >= vdim) break;                     // wave-uniform
+        const float g = a.norm ? a.norm[c] : 1.f;
+#pragma unroll
+        for (int b = 0; b < NS; ++b)
+#pragma unroll
+            for (int r = 0; r < 4; ++r) {
+                const int row = 16 * b + 4 * q4 + r;
+                if (row < ch.len) out[(size_t)row * a.ld_out + h * vdim + c] = from_f<T>(o[t][b][r] * inv[b][r] * g);
+            }
+    }
+    if (h == a.H - 1 && a.ld_out > a.H * vdim) {
+        const int tail = a.ld_out - a.H * vdim;
+        for (int t = tid; t < ch.len * tail; t += 512) out[(size_t)(t / tail) * a.ld_out + a.H * vdim + t % tail] = from_f<T>(0.f);
+    }
+}
+
+template <class K>
+static hipError_t rc_allow_lds(K kfn, size_t lds, bool& done) {
+    if (lds <= 48 * 1024 || done) return hipSuccess;
+    done = true;
+    return hipFuncSetAttribute(reinterpret_cast<const void*>(kfn), hipFuncAttributeMaxDynamicSharedMemorySize, (int)RC_LDS_MAX);
+}
+
+template <class T, int C, int NVT>
+static hipError_t launch_chunk_out(const RecurArgs& a, const RecurChunk* chunks, int n_chunks, const float* U, hipStream_t st) {
+    static bool done = false;
+    const size_t lds = rc_out_lds(C, a.dim);
+    if (hipError_t e = rc_allow_lds(&recur_chunk_out_kernel<T, C, NVT>, lds, done)) return e;
+    recur_chunk_out_kernel<T, C, NVT><<<dim3(a.H, n_chunks), 512, lds, st>>>(a, chunks, U);
+    return hipGetLastError();
+}
+
+template <class T, int C>
+static pgk_status recur_chunked_t(const RecurArgs& a, const RecurChunk* chunks, int n_chunks, const int32_t* chunk_of_seq, void* ws, hipStream_t st) {
+    float *U = (float*)ws, *D = U + (size_t)n_chunks * a.H * a.dim * a.vdim;
+    static bool done = false;
+    const size_t lds = rc_state_lds(C, a.dim, a.vdim);
+    PGK_CHECK_HIP(rc_allow_lds(&recur_chunk_state_kernel<T, C>, lds, done));
+    recur_chunk_state_kernel<T, C><<<dim3(a.H, n_chunks), 256, lds, st>>>(a, chunks, U, D);
+    PGK_LAUNCH_CHECK();
+    recur_chunk_scan_kernel<<<dim3(ceil_div(a.dim * a.vdim / 4, 256), a.H, a.n_seqs), 256, 0, st>>>(a, chunk_of_seq, U, D);
+    PGK_LAUNCH_CHECK();
+    if (a.vdim <= 128) PGK_CHECK_HIP((launch_chunk_out<T, C, 1>(a, chunks, n_chunks, U, st)));
+    else if (a.vdim <= 256) PGK_CHECK_HIP((launch_chunk_out<T, C, 2>(a, chunks, n_chunks, U, st)));
+    else PGK_CHECK_HIP((launch_chunk_out<T, C, 4>(a, chunks, n_chunks, U, st)));
+    return PGK_OK;
+}
+
+pgk_status recur_chunked(const RecurArgs& a, const RecurChunk* chunks, int n_chunks, const int32_t* chunk_of_seq, void* ws, pgk_dtype dt, hipStream_t st) {
+    const int C = recur_chunk_rows(a.dim, a.vdim);
+    PGK_REQUIRE(C && a.seqs && chunks && n_chunks >= 1 && n_chunks <= 65535 && a.H * a.vdim <= a.ld_out && a.ld_in % 4 == 0 && a.q_off % 4 == 0 && a.f_off % 4 == 0 && a.v_off % 4 == 0,
+                "recurrence: %d chunks of head widths %d / %d", n_chunks, a.dim, a.vdim);
+    if (dt == PGK_F32) return C == 64 ? recur_chunked_t<float, 64>(a, chunks, n_chunks, chunk_of_seq, ws, st) : recur_chunked_t<float, 32>(a, chunks, n_chunks, chunk_of_seq, ws, st);
+    return C == 64 ? recur_chunked_t<bf16, 64>(a, chunks, n_chunks, chunk_of_seq, ws, st) : recur_chunked_t<bf16, 32>(a, chunks, n_chunks, chunk_of_seq, ws, st);
+}
+
 }  // namespace pgk
 
 using namespace pgk;
@@ -125,22 +502,34 @@ pgk_status pgk_gated_recurrence(const void* q, const void* f, const void* v, con
     PGK_REQUIRE(n >= 1 && heads >= 1 && dim >= 1 && vdim >= 1, "pgk_gated_recurrence: bad shape %d x %d x %d, %d rows", heads, dim, vdim, n);
     PGK_REQUIRE(dt == PGK_BF16 || dt == PGK_F32, "pgk_gated_recurrence: dtype %d (bf16 or f32)", (int)dt);
     hipStream_t st = resolve_stream(s);
-    // one row buffer q | f | v, and the portion table behind it
-    const size_t E = dtype_size(dt), row = (size_t)heads * (2 * dim + vdim), bytes = ((size_t)n * row * E + 255) & ~(size_t)255;
-    char* ws = nullptr;
-    if (pgk_status r = pgk_malloc((void**)&ws, bytes + sizeof(SeqSpan))) return r;
-    const size_t wq = (size_t)heads * dim * E, wv = (size_t)heads * vdim * E;
+    // one row buffer q | f | v, the tables and the chunked form's workspace behind it
+    const size_t E = dtype_size(dt), row = (size_t)heads * (2 * dim + vdim);
+    auto up = [](size_t b) { return (b + 255) & ~(size_t)255; };
+    RecurArgs a{};
+    a.ld_in = (int)row; a.f_off = heads * dim; a.v_off = 2 * heads * dim;
+    a.bias = f_bias; a.lower = lower; a.norm = norm; a.H = heads; a.dim = dim; a.vdim = a.vdim_true = vdim; a.n = n; a.eps = eps;
+    a.state = state; a.n_seqs = 1; a.out = out; a.ld_out = heads * vdim;
+    const int C = n >= RECUR_CHUNKED_FROM ? recur_chunk_rows(dim, vdim) : 0, nch = C ? ceil_div(n, C) : 0;
+    std::vector<RecurChunk> chunks;
+    for (int c = 0; c < nch; ++c) chunks.push_back(RecurChunk{c * C, n - c * C < C ? n - c * C : C});
+    const int32_t of_seq[2] = {0, nch};
     const SeqSpan span{0, n, fresh ? 0 : 1, 0};
+    const size_t o_span = up((size_t)n * row * E), o_of = o_span + up(sizeof(span)), o_ch = o_of + up(sizeof(of_seq)), o_ws = o_ch + up(nch * sizeof(RecurChunk));
+    char* ws = nullptr;
+    if (pgk_status r = pgk_malloc((void**)&ws, o_ws + (nch ? recur_chunk_bytes(a, nch) : 0) + 256)) return r;
+    const size_t wq = (size_t)heads * dim * E, wv = (size_t)heads * vdim * E;
     hipError_t e = hipMemcpy2DAsync(ws, row * E, q, wq, wq, n, hipMemcpyDeviceToDevice, st);
     if (e == hipSuccess) e = hipMemcpy2DAsync(ws + wq, row * E, f, wq, wq, n, hipMemcpyDeviceToDevice, st);
     if (e == hipSuccess) e = hipMemcpy2DAsync(ws + 2 * wq, row * E, v, wv, wv, n, hipMemcpyDeviceToDevice, st);
-    if (e == hipSuccess) e = hipMemcpyAsync(ws + bytes, &span, sizeof(span), hipMemcpyHostToDevice, st);
+    if (e == hipSuccess) e = hipMemcpyAsync(ws + o_span, &span, sizeof(span), hipMemcpyHostToDevice, st);
+    if (e == hipSuccess) e = hipMemcpyAsync(ws + o_of, of_seq, sizeof(of_seq), hipMemcpyHostToDevice, st);
+    if (e == hipSuccess && nch) e = hipMemcpyAsync(ws + o_ch, chunks.data(), nch * sizeof(RecurChunk), hipMemcpyHostToDevice, st);
     if (e == hipSuccess) e = hipStreamSynchronize(st);
-    RecurArgs a{};
-    a.in = ws; a.ld_in = (int)row; a.f_off = heads * dim; a.v_off = 2 * heads * dim;
-    a.bias = f_bias; a.lower = lower; a.norm = norm; a.H = heads; a.dim = dim; a.vdim = a.vdim_true = vdim; a.n = n; a.eps = eps;
-    a.state = state; a.seqs = (const SeqSpan*)(ws + bytes); a.n_seqs = 1; a.out = out; a.ld_out = heads * vdim;
-    pgk_status r = e == hipSuccess ? recur_rows(a, dt, false, st) : set_error(PGK_ERR_HIP, "pgk_gated_recurrence: %s", hipGetErrorString(e));
+    a.in = ws; a.seqs = (const SeqSpan*)(ws + o_span);
+    pgk_status r;
+    if (e != hipSuccess) r = set_error(PGK_ERR_HIP, "pgk_gated_recurrence: %s", hipGetErrorString(e));
+    else if (nch) r = recur_chunked(a, (const RecurChunk*)(ws + o_ch), nch, (const int32_t*)(ws + o_of), ws + o_ws, dt, st);
+    else r = recur_rows(a, dt, false, st);
     pgk_free(ws);       // stream-ordered reuse: later work on this stream runs after the kernel above
     return r;
 }

@@ -140,13 +140,13 @@ class Engine:
         """Enqueue one eager (un-captured) step."""
         _hip.call("pgk_engine_decode_step", self.handle, batch, None)
 
-    KERNEL_CLASSES = ("embed", "norm_qkv", "attn", "oproj", "gateup", "down", "lmhead", "argmax")
+    KERNEL_CLASSES = ("embed", "norm_qkv", "attn", "oproj", "gateup", "down", "lmhead", "argmax", "recur")
 
     def profile_step(self, batch: int = 1, n_iters: int = 8) -> dict:
         """Eager steps, every launch bracketed by its own start/stop event (the dispatch's begin -> end interval, what
         rocprofv3 --kernel-trace reports) -> {class: (avg_us_per_launch, launches_per_step)}."""
-        ms = (C.c_float * 8)()
-        cnt = (C.c_int * 8)()
+        ms = (C.c_float * len(self.KERNEL_CLASSES))()
+        cnt = (C.c_int * len(self.KERNEL_CLASSES))()
         _hip.call("pgk_engine_profile_step", self.handle, batch, n_iters, ms, cnt, None)
         return {name: ((ms[i] * 1e3 / cnt[i]) if cnt[i] else 0.0, cnt[i] // n_iters) for i, name in enumerate(self.KERNEL_CLASSES)}
 

@@ -14,6 +14,7 @@ import sys
 import numpy as np
 import pytest
 
+from tests.layer_list import FakeEngine, dev, host, logit_err, rounded, save, tokens
 from oracle import cpu_ref as O
 from oracle import totolorn_ref as R
 
@@ -74,24 +75,6 @@ def weights(cfg, seed=0, sharp=2.5):
     return {k: O.bf16_bits_to_f32(O.f32_to_bf16_bits(v)).reshape(v.shape) for k, v in W.items()}
 
 
-def save(folder, cfg, W):
-    from pygpukit_amd.llm.safetensors import save_safetensors
-
-    with open(os.path.join(folder, "config.json"), "w", encoding="utf-8") as f:
-        json.dump(cfg, f)
-    save_safetensors(os.path.join(folder, "model.safetensors"), {k: (O.f32_to_bf16_bits(v).reshape(v.shape), "BF16") for k, v in W.items()})
-    return str(folder)
-
-
-def logit_err(got, want):
-    d = np.asarray(got, np.float64) - want
-    return float(np.max(np.sqrt(np.mean(d * d, axis=-1)) / np.sqrt(np.mean(want * want))))
-
-
-def tokens(cfg, n, seed):
-    return [int(t) for t in np.random.default_rng(seed).integers(0, cfg["vocab"], n)]
-
-
 # ------------------------------------------------------------------------------------------------ CPU: configuration, oracle, scheduler
 def test_config_is_read_layer_by_layer():
     from pygpukit_amd.llm import TOTOLORN_SPEC, detect_model_spec, layer_list_config
@@ -137,32 +120,6 @@ def test_weights_tell_windows_apart(name):
             assert logit_err(R.forward(t, other, W), want) > 500 * TOL["float32"]
 
 
-class FakeEngine:
-    """Records what the scheduler asks for; the `logits` of a row are (slot, position, token)."""
-
-    def __init__(self, max_batch=3, max_seq_len=20):
-        self.max_batch, self.max_seq_len, self.config, self.calls = max_batch, max_seq_len, {"vocab_size": 3}, []
-
-    def prefill_batch(self, prompts, slots, starts, want):
-        self.calls.append(("prefill", list(slots), list(starts), [len(p) for p in prompts]))
-        return np.array([(s, st + i, p[i]) for p, s, st, w in zip(prompts, slots, starts, want) for i in w], np.float32).reshape(-1, 3)
-
-    def set_state(self, tok, pos):
-        self.state = [(i, p, t) for i, (t, p) in enumerate(zip(tok, pos))]
-
-    def decode_step(self, rows):
-        self.calls.append(("decode", rows))
-
-    def logits(self, rows):
-        state = self.state
-
-        class A:
-            @staticmethod
-            def to_numpy():
-                return np.array(state, np.float32)
-        return A()
-
-
 def test_scheduler_slots_batches_and_order():
     from pygpukit_amd.llm.scheduler import BatchScheduler
 
@@ -195,27 +152,6 @@ def test_scheduler_slots_batches_and_order():
 
 
 # ------------------------------------------------------------------------------------------------ GPU: operators
-def dev(x, dtype):
-    from pygpukit_amd.core.factory import from_numpy
-
-    x = np.ascontiguousarray(x, np.float32)
-    if dtype == "float32":
-        return from_numpy(x)
-    return from_numpy(x.astype(np.float16) if dtype == "float16" else O.f32_to_bf16_bits(x).reshape(x.shape))
-
-
-def host(a):
-    h = a.to_numpy()
-    return O.bf16_bits_to_f32(h).reshape(h.shape) if h.dtype == np.uint16 else h.astype(np.float32)
-
-
-def rounded(x, dtype):
-    x = np.asarray(x, np.float32)
-    if dtype == "bfloat16":
-        return O.bf16_bits_to_f32(O.f32_to_bf16_bits(x)).reshape(x.shape)
-    return x.astype(np.float16).astype(np.float32) if dtype == "float16" else x
-
-
 OP_TOL = {"float32": 2e-6, "float16": 2e-3, "bfloat16": 1.2e-2}
 
 
