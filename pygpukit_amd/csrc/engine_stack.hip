@@ -45,6 +45,9 @@ pgk_status wsgemm_nt(const bf16* a, int lda, const void* w, const bf16* wscale, 
 bool engine_gemm_swiglu_ok(int M, int I, int K, bool fp8);     // ops_gemm.hip
 pgk_status engine_gemm_swiglu_nt(const bf16* A, const void* W, const bf16* wscale, bool fp8, bf16* act, int M, int I, int K, hipStream_t st, bool packed = false);
 
+bool engine_gemm_xielu_ok(int M, int N, int K);                // ops_gemm.hip
+pgk_status engine_gemm_xielu_nt(const bf16* A, const bf16* W, bf16* act, int M, int N, int K, float pos, float neg, hipStream_t st);
+
 int wsgemm_pick_splits(int N, int K, bool allow_split);        // ops_wsgemm.hip
 int engine_gemm_pick_splits(int M, int N, int K);              // ops_gemm.hip: split-K slabs for prompts whose tiles do not cover the chip
 pgk_status engine_gemm_nt_slabs(const bf16* A, const void* W, float* slabs, int splits, int M, int N, int K, hipStream_t st, bool packed = false);
@@ -693,6 +696,14 @@ __global__ void stack_embed_kernel(const T* embed, const T* pos, const int32_t* 
     const size_t row = blockIdx.x;
     const T* e = embed + (size_t)tok[row] * W;
     const T* p = pos ? pos + (size_t)min(max(position[row], 0), npos - 1) * W : nullptr;
+    if (W == ld) {                                                 // (a multiple of 64)
+        for (int i = 4 * threadIdx.x; i < ld; i += 4 * blockDim.x) {
+            float4 v = load4<T>(e + i);
+            if (p) { const float4 q = load4<T>(p + i); v.x += q.x; v.y += q.y; v.z += q.z; v.w += q.w; }
+            *reinterpret_cast<float4*>(h + row * ld + i) = v;
+        }
+        return;
+    }
     for (int i = threadIdx.x; i < ld; i += blockDim.x) h[row * ld + i] = i < W ? to_f(e[i]) + (p ? to_f(p[i]) : 0.f) : 0.f;
 }
 
@@ -1049,8 +1060,13 @@ static pgk_status rows_gate_up(Stack* s, const pgk_stack_layer_t& L, const bf16*
     constexpr pgk_dtype DT = std::is_same<T, float>::value ? PGK_F32 : PGK_BF16;
     if (L.ff == PGK_FF_XIELU) {
         if (DT == PGK_BF16 && n <= 128 && packed) {
-            if (pgk_status r = pkgemm_nt((const bf16*)b.x, s->Wp, packed, b.act, L.ff_pad, PK_EPI_BF16, 1, n, L.ff_pad, s->Wp, nullptr, st)) return r;
-        } else if (pgk_status r = pgk_gemm_nt(b.x, L.w_gate_up, nullptr, b.act, n, L.ff_pad, s->Wp, DT, st)) return r;
+            PkArgs g{};
+            g.act_pos = L.act_pos; g.act_neg = L.act_neg;
+            return pkgemm_nt((const bf16*)b.x, s->Wp, packed, b.act, L.ff_pad, PK_EPI_XIELU, 1, n, L.ff_pad, s->Wp, &g, st);
+        }
+        if (DT == PGK_BF16 && engine_gemm_xielu_ok(n, L.ff_pad, s->Wp))
+            return engine_gemm_xielu_nt((const bf16*)b.x, (const bf16*)L.w_gate_up, (bf16*)b.act, n, L.ff_pad, s->Wp, L.act_pos, L.act_neg, st);
+        if (pgk_status r = pgk_gemm_nt(b.x, L.w_gate_up, nullptr, b.act, n, L.ff_pad, s->Wp, DT, st)) return r;
         return pgk_xielu(b.act, b.act, (size_t)n * L.ff_pad, L.act_pos, L.act_neg, DT, st);
     }
     if (DT == PGK_BF16 && n <= 128 && packed)

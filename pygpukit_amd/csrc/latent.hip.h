@@ -19,12 +19,6 @@ template <> __device__ __forceinline__ void store4<bf16>(bf16* p, const float4& 
     *reinterpret_cast<uint2*>(p) = make_uint2(pack_bf16x2(v.x, v.y), pack_bf16x2(v.z, v.w));
 }
 
-// xIELU with its two softplus'ed factors: z > 0: a z^2 + z / 2,  z <= 0: b (exp(z) - 1 - z) + z / 2  (EXACT: the fp32 engines' form)
-template <bool EXACT> __device__ __forceinline__ float xielu(float z, float a, float b) {
-    const float n = fminf(z, 0.f), e = EXACT ? expm1f(n) : __expf(n) - 1.0f;
-    return fmaf(0.5f, z, z > 0.f ? a * z * z : b * (e - n));
-}
-
 // One sandwich step on rows of the fp32 stream h [*][ld] (columns W..ld are zero padding):
 //   y given:    h += mult * y / rms(y) * g_post       (y rows in the engine's element type, row stride ldy; store_h: write h back)
 //   out given:  out[i] = h / rms(h) * gamma           (rows of stride ld in the engine's element type; gamma null: out[i] = h)

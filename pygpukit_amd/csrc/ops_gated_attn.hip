@@ -10,126 +10,206 @@ namespace pgk {
 constexpr float GA_LOG2E = 1.4426950408889634f;
 
 // -------------------------------------------------------------------------------------------- short convolution, norms
-// RB rows per workgroup, four channels per thread and trip; the taps are computed twice (sums of squares, then results): the second
-// time they come from the L1.  TAPS 0: any number.
-template <class T, class IT, class QT, int TAPS, int RB>
-__global__ __launch_bounds__(1024) void conv_rows_kernel(unsigned long long* tl, ConvArgs a) {
-    const TLStamp tls(tl);
-    __shared__ float red[16][2 * RB];
-    const int taps = TAPS ? TAPS : a.taps, nc = a.n_q + 2 * a.n_kv, tid = threadIdx.x, nt = blockDim.x, r0 = blockIdx.x * RB;
-    const IT* in = reinterpret_cast<const IT*>(a.in);
-    T* ring = reinterpret_cast<T*>(a.tap_ring);
-    int pos[RB], slot[RB], first[RB];
-#pragma unroll
-    for (int m = 0; m < RB; ++m) {
-        const int r = min(r0 + m, a.n - 1);
-        if (a.rows) { const RowSrc s = a.rows[r]; pos[m] = s.pos; slot[m] = s.slot; first[m] = s.first; }
-        else { pos[m] = max(a.positions[r], 0); slot[m] = r; first[m] = r; }
+// Where the channels c .. c + 3 (all of q, of k or of v) of one row go: normalised values to q_out, or to the scratch row and the cache.
+template <class T, class QT>
+__device__ __forceinline__ void conv_store(const ConvArgs& a, int row, int pos, int slot, int c, float4 y, float inv_q, float inv_k) {
+    if (c < a.n_q) {
+        const float s = a.q_norm ? inv_q * a.q_mult : a.q_mult;
+        const float4 g = a.q_norm ? *reinterpret_cast<const float4*>(a.q_norm + c) : make_float4(1.f, 1.f, 1.f, 1.f);
+        y.x *= s * g.x; y.y *= s * g.y; y.z *= s * g.z; y.w *= s * g.w;
+        store4<QT>(reinterpret_cast<QT*>(a.q_out) + (size_t)row * a.ld_q + c, y);
+        return;
     }
-    auto conv4 = [&](int m, int c) -> float4 {
-        const int r = min(r0 + m, a.n - 1);
-        const float4 b = a.bias ? *reinterpret_cast<const float4*>(a.bias + c) : make_float4(0.f, 0.f, 0.f, 0.f);
-        float4 y = load4<IT>(in + (size_t)r * a.ld_in + c);
-        y.x += b.x; y.y += b.y; y.z += b.z; y.w += b.w;
-        if (!a.conv) return y;
-        const float4 w0 = *reinterpret_cast<const float4*>(a.conv + (size_t)(taps - 1) * nc + c);
-        y.x *= w0.x; y.y *= w0.y; y.z *= w0.z; y.w *= w0.w;
-        auto tap = [&](int back) {
-            const int p = pos[m] - back;
-            if (p < 0) return;                                     // before the sequence's start: zero, bias included
-            const float4 w = *reinterpret_cast<const float4*>(a.conv + (size_t)(taps - 1 - back) * nc + c);
-            const float4 u = r - back >= first[m] ? load4<IT>(in + (size_t)(r - back) * a.ld_in + c)
-                                                  : load4<T>(ring + ((size_t)slot[m] * taps + p % taps) * nc + c);
-            y.x = fmaf(w.x, u.x + b.x, y.x); y.y = fmaf(w.y, u.y + b.y, y.y); y.z = fmaf(w.z, u.z + b.z, y.z); y.w = fmaf(w.w, u.w + b.w, y.w);
-        };
-        if constexpr (TAPS > 0) {
-#pragma unroll
-            for (int back = 1; back < TAPS; ++back) tap(back);
-        } else {
-            for (int back = 1; back < taps; ++back) tap(back);
-        }
-        return y;
-    };
-    float ss[2 * RB];
-#pragma unroll
-    for (int i = 0; i < 2 * RB; ++i) ss[i] = 0.f;
-    for (int c = 4 * tid; c < a.n_q + a.n_kv; c += 4 * nt) {
-#pragma unroll
-        for (int m = 0; m < RB; ++m) {
-            const float4 y = conv4(m, c);
-            const float t = y.x * y.x + y.y * y.y + y.z * y.z + y.w * y.w;
-            ss[2 * m] += c < a.n_q ? t : 0.f;
-            ss[2 * m + 1] += c < a.n_q ? 0.f : t;
-        }
+    const bool is_k = c < a.n_q + a.n_kv;
+    const int kc = c - a.n_q - (is_k ? 0 : a.n_kv);
+    if (is_k && a.k_norm) {
+        const float4 g = *reinterpret_cast<const float4*>(a.k_norm + kc);
+        y.x *= inv_k * g.x; y.y *= inv_k * g.y; y.z *= inv_k * g.z; y.w *= inv_k * g.w;
     }
+    if (a.place) {
+        const RowPlace p = a.place[row];
+        store4<T>(reinterpret_cast<T*>(a.kv_rows) + (size_t)p.kv * a.ld_kv + (is_k ? 0 : a.n_kv) + kc, y);
+        if (!p.store) return;
+    }
+    store4<T>(reinterpret_cast<T*>(a.cache) + ((((size_t)slot * 2 + (is_k ? 0 : 1)) * (a.n_kv / a.D) + kc / a.D) * a.R + pos % a.R) * a.D + kc % a.D, y);
+}
+
+// Per-row scales of q and k from per-thread sums of squares (q, k of every row in turn)
+template <int RB>
+__device__ __forceinline__ void conv_scales(const ConvArgs& a, float (&ss)[2 * RB], float (&red)[16][2 * RB], float (&inv)[2 * RB]) {
 #pragma unroll
     for (int i = 0; i < 2 * RB; ++i) {
         const float t = wave_sum(ss[i]);
-        if ((tid & 63) == 0) red[tid >> 6][i] = t;
+        if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6][i] = t;
     }
     __syncthreads();
-    float inv[2 * RB];
 #pragma unroll
     for (int i = 0; i < 2 * RB; ++i) {
         float t = 0.f;
-        for (int w = 0; w < (nt >> 6); ++w) t += red[w][i];
+        for (int w = 0; w < (int)(blockDim.x >> 6); ++w) t += red[w][i];
         inv[i] = 1.0f / sqrtf(t / ((i & 1) ? max(a.k_true, 1) : a.q_true) + a.eps);
     }
-    for (int c = 4 * tid; c < nc; c += 4 * nt) {
+}
+
+__device__ __forceinline__ RowSrc conv_row(const ConvArgs& a, int r) {
+    return a.rows ? a.rows[r] : RowSrc{max(a.positions[r], 0), r, r};
+}
+
+// Up to four taps: RB rows and QPT groups of four channels per thread, everything requested up front and kept in registers.  Rows of one
+// portion share the rows above them (a window of RB + 3 loads); a workgroup that spans two portions loads each row's taps by itself.
+constexpr int CONV_MT = 4;
+template <class T, class IT, class QT, int RB, int QPT>
+__global__ __launch_bounds__(1024, RB * QPT <= 2 ? 8 : 4) void conv_rows_kernel(unsigned long long* tl, ConvArgs a) {
+    const TLStamp tls(tl);
+    __shared__ float red[16][2 * RB];
+    constexpr int NW = RB + CONV_MT - 1;
+    const int taps = a.taps, nc = a.n_q + 2 * a.n_kv, nt = blockDim.x, r0 = blockIdx.x * RB, last = a.n - 1;
+    const IT* in = reinterpret_cast<const IT*>(a.in);
+    T* ring = reinterpret_cast<T*>(a.tap_ring);
+    RowSrc src[RB];
+#pragma unroll
+    for (int m = 0; m < RB; ++m) src[m] = conv_row(a, min(r0 + m, last));
+    int c[QPT];
+    float4 b[QPT], w[QPT][CONV_MT], y[QPT][RB];
+    const float4 zero = {0.f, 0.f, 0.f, 0.f};
+    // the projected values of position pos - back for the row `r` of portion s (zero before the sequence's start, bias included)
+    auto fetch = [&](const RowSrc& s, int r, int back, int cc) -> float4 {
+        const int p = s.pos - back;
+        if (p < 0 || back >= taps) return zero;
+        return r - back >= s.first ? load4<IT>(in + (size_t)(r - back) * a.ld_in + cc) : load4<T>(ring + ((size_t)s.slot * taps + p % taps) * nc + cc);
+    };
+    auto add = [](float4 u, const float4& v) { u.x += v.x; u.y += v.y; u.z += v.z; u.w += v.w; return u; };
+    auto fma4 = [](const float4& x, const float4& u, float4 acc) {
+        acc.x = fmaf(x.x, u.x, acc.x); acc.y = fmaf(x.y, u.y, acc.y); acc.z = fmaf(x.z, u.z, acc.z); acc.w = fmaf(x.w, u.w, acc.w);
+        return acc;
+    };
+    const bool whole = src[RB - 1].first == src[0].first;          // workgroup-uniform
+    if (whole) {
+        float4 u[QPT][NW];
+#pragma unroll
+        for (int q = 0; q < QPT; ++q) {
+            c[q] = 4 * (threadIdx.x + q * nt);
+            const int cc = min(c[q], nc - 4);
+#pragma unroll
+            for (int i = 0; i < NW; ++i) {
+                const int back = CONV_MT - 1 - i;                  // of row r0: negative for the rows below it
+                u[q][i] = back > 0 ? fetch(src[0], r0, back, cc) : load4<IT>(in + (size_t)min(r0 - back, last) * a.ld_in + cc);
+            }
+            b[q] = a.bias ? *reinterpret_cast<const float4*>(a.bias + cc) : zero;
+#pragma unroll
+            for (int k = 0; k < CONV_MT; ++k)
+                w[q][k] = k >= taps ? zero : a.conv ? *reinterpret_cast<const float4*>(a.conv + (size_t)(taps - 1 - k) * nc + cc) : make_float4(1.f, 1.f, 1.f, 1.f);
+        }
+#pragma unroll
+        for (int q = 0; q < QPT; ++q)
+#pragma unroll
+            for (int i = 0; i < NW; ++i)
+                if (src[0].pos - (CONV_MT - 1 - i) >= 0) u[q][i] = add(u[q][i], b[q]);
+#pragma unroll
+        for (int q = 0; q < QPT; ++q)
+#pragma unroll
+            for (int m = 0; m < RB; ++m) {
+                y[q][m] = zero;
+#pragma unroll
+                for (int k = 0; k < CONV_MT; ++k) y[q][m] = fma4(w[q][k], u[q][m + CONV_MT - 1 - k], y[q][m]);
+            }
+    } else {
+#pragma unroll
+        for (int q = 0; q < QPT; ++q) {
+            c[q] = 4 * (threadIdx.x + q * nt);
+            const int cc = min(c[q], nc - 4);
+            b[q] = a.bias ? *reinterpret_cast<const float4*>(a.bias + cc) : zero;
+#pragma unroll
+            for (int m = 0; m < RB; ++m) {
+                const int r = min(r0 + m, last);
+                y[q][m] = zero;
+                for (int k = 0; k < taps; ++k) {
+                    if (src[m].pos - k < 0) break;
+                    const float4 x = a.conv ? *reinterpret_cast<const float4*>(a.conv + (size_t)(taps - 1 - k) * nc + cc) : make_float4(1.f, 1.f, 1.f, 1.f);
+                    y[q][m] = fma4(x, add(fetch(src[m], r, k, cc), b[q]), y[q][m]);
+                }
+            }
+        }
+    }
+    float ss[2 * RB], inv[2 * RB];
+#pragma unroll
+    for (int i = 0; i < 2 * RB; ++i) ss[i] = 0.f;
+#pragma unroll
+    for (int q = 0; q < QPT; ++q)
 #pragma unroll
         for (int m = 0; m < RB; ++m) {
-            if (r0 + m >= a.n) break;
-            float4 y = conv4(m, c);
-            if (c < a.n_q) {
-                if (a.q_norm) {
-                    const float4 g = *reinterpret_cast<const float4*>(a.q_norm + c);
-                    const float s = inv[2 * m] * a.q_mult;
-                    y.x *= s * g.x; y.y *= s * g.y; y.z *= s * g.z; y.w *= s * g.w;
-                } else { y.x *= a.q_mult; y.y *= a.q_mult; y.z *= a.q_mult; y.w *= a.q_mult; }
-                store4<QT>(reinterpret_cast<QT*>(a.q_out) + (size_t)(r0 + m) * a.ld_q + c, y);
-            } else {
-                const bool is_k = c < a.n_q + a.n_kv;
-                const int kc = c - a.n_q - (is_k ? 0 : a.n_kv);
-                if (is_k && a.k_norm) {
-                    const float4 g = *reinterpret_cast<const float4*>(a.k_norm + kc);
-                    const float s = inv[2 * m + 1];
-                    y.x *= s * g.x; y.y *= s * g.y; y.z *= s * g.z; y.w *= s * g.w;
-                }
-                bool keep = true;
-                if (a.place) {
-                    const RowPlace p = a.place[r0 + m];
-                    store4<T>(reinterpret_cast<T*>(a.kv_rows) + (size_t)p.kv * a.ld_kv + (is_k ? 0 : a.n_kv) + kc, y);
-                    keep = p.store != 0;
-                }
-                if (keep)
-                    store4<T>(reinterpret_cast<T*>(a.cache) + ((((size_t)slot[m] * 2 + (is_k ? 0 : 1)) * (a.n_kv / a.D) + kc / a.D) * a.R + pos[m] % a.R) * a.D + kc % a.D, y);
-            }
-            if (!a.rows && a.conv) store4<T>(ring + ((size_t)slot[m] * taps + pos[m] % taps) * nc + c, load4<IT>(in + (size_t)(r0 + m) * a.ld_in + c));
+            const float t = y[q][m].x * y[q][m].x + y[q][m].y * y[q][m].y + y[q][m].z * y[q][m].z + y[q][m].w * y[q][m].w;
+            ss[2 * m] += c[q] < a.n_q ? t : 0.f;
+            ss[2 * m + 1] += c[q] >= a.n_q && c[q] < a.n_q + a.n_kv ? t : 0.f;
+        }
+    conv_scales<RB>(a, ss, red, inv);
+#pragma unroll
+    for (int q = 0; q < QPT; ++q) {
+        if (c[q] >= nc) break;
+#pragma unroll
+        for (int m = 0; m < RB; ++m) {
+            if (r0 + m > last) break;
+            conv_store<T, QT>(a, r0 + m, src[m].pos, src[m].slot, c[q], y[q][m], inv[2 * m], inv[2 * m + 1]);
+            if (!a.rows && a.conv) store4<T>(ring + ((size_t)src[m].slot * taps + src[m].pos % taps) * nc + c[q], load4<IT>(in + (size_t)(r0 + m) * a.ld_in + c[q]));
         }
     }
     tls.end();
 }
 
+// Any number of taps and channels, one row per workgroup: the taps are computed twice (sums of squares, then results)
+template <class T, class IT, class QT>
+__global__ __launch_bounds__(256) void conv_rows_any_kernel(unsigned long long* tl, ConvArgs a) {
+    const TLStamp tls(tl);
+    __shared__ float red[16][2];
+    const int taps = a.taps, nc = a.n_q + 2 * a.n_kv, r = blockIdx.x;
+    const IT* in = reinterpret_cast<const IT*>(a.in);
+    T* ring = reinterpret_cast<T*>(a.tap_ring);
+    const RowSrc s = conv_row(a, r);
+    auto conv4 = [&](int c) -> float4 {
+        const float4 b = a.bias ? *reinterpret_cast<const float4*>(a.bias + c) : make_float4(0.f, 0.f, 0.f, 0.f);
+        float4 y = {0.f, 0.f, 0.f, 0.f};
+        for (int back = 0; back < taps && s.pos - back >= 0; ++back) {
+            const float4 w = a.conv ? *reinterpret_cast<const float4*>(a.conv + (size_t)(taps - 1 - back) * nc + c) : make_float4(1.f, 1.f, 1.f, 1.f);
+            const float4 u = r - back >= s.first ? load4<IT>(in + (size_t)(r - back) * a.ld_in + c) : load4<T>(ring + ((size_t)s.slot * taps + (s.pos - back) % taps) * nc + c);
+            y.x = fmaf(w.x, u.x + b.x, y.x); y.y = fmaf(w.y, u.y + b.y, y.y); y.z = fmaf(w.z, u.z + b.z, y.z); y.w = fmaf(w.w, u.w + b.w, y.w);
+        }
+        return y;
+    };
+    float ss[2] = {0.f, 0.f}, inv[2];
+    for (int c = 4 * threadIdx.x; c < a.n_q + a.n_kv; c += 1024) {
+        const float4 y = conv4(c);
+        ss[c < a.n_q ? 0 : 1] += y.x * y.x + y.y * y.y + y.z * y.z + y.w * y.w;
+    }
+    conv_scales<1>(a, ss, red, inv);
+    for (int c = 4 * threadIdx.x; c < nc; c += 1024) {
+        conv_store<T, QT>(a, r, s.pos, s.slot, c, conv4(c), inv[0], inv[1]);
+        // (the row written is read by no tap of this step, and its channels by this thread only)
+        if (!a.rows && a.conv) store4<T>(ring + ((size_t)s.slot * taps + s.pos % taps) * nc + c, load4<IT>(in + (size_t)r * a.ld_in + c));
+    }
+    tls.end();
+}
+
 template <class T, class IT, class QT, int RB>
-static hipError_t conv_rows_launch(const ConvArgs& a, int threads, hipStream_t st) {
-    const dim3 grid(ceil_div(a.n, RB)), block(threads);
-    if (a.taps == 4) return launch_k(&conv_rows_kernel<T, IT, QT, 4, RB>, grid, block, 0, st, a);
-    return launch_k(&conv_rows_kernel<T, IT, QT, 0, RB>, grid, block, 0, st, a);
+static hipError_t conv_rows_launch(const ConvArgs& a, hipStream_t st) {
+    const int quads = (a.n_q + 2 * a.n_kv) / 4;
+    auto waves = [](int t) { return (t + 63) / 64 * 64; };
+    if (a.taps > CONV_MT || quads > 4096 || (RB > 1 && quads > 2048)) return launch_k(&conv_rows_any_kernel<T, IT, QT>, dim3(a.n), dim3(256), 0, st, a);
+    if (quads <= 1024) return launch_k(&conv_rows_kernel<T, IT, QT, RB, 1>, dim3(ceil_div(a.n, RB)), dim3(waves(quads)), 0, st, a);
+    if (quads <= 2048) return launch_k(&conv_rows_kernel<T, IT, QT, RB, 2>, dim3(ceil_div(a.n, RB)), dim3(waves((quads + 1) / 2)), 0, st, a);
+    return launch_k(&conv_rows_kernel<T, IT, QT, 1, 4>, dim3(a.n), dim3(waves((quads + 3) / 4)), 0, st, a);
 }
 
 pgk_status conv_rows(const ConvArgs& a, pgk_dtype dt, bool in32, bool q32, hipStream_t st) {
     PGK_REQUIRE(a.n >= 1 && a.n_q % 4 == 0 && a.n_kv % 4 == 0 && a.D % 4 == 0 && (a.n_kv == 0 || a.n_kv % a.D == 0) && a.ld_in % 4 == 0 && a.ld_q % 4 == 0 && a.taps >= 1,
                 "conv_rows: %d rows of %d + 2 x %d channels, heads of %d, %d taps", a.n, a.n_q, a.n_kv, a.D, a.taps);
-    const int quads = (a.n_q + 2 * a.n_kv) / 4;
     if (a.rows) {                                                  // prompt: rows and q in the element type
-        if (dt == PGK_F32) PGK_CHECK_HIP((conv_rows_launch<float, float, float, 4>(a, 256, st)));
-        else PGK_CHECK_HIP((conv_rows_launch<bf16, bf16, bf16, 4>(a, 256, st)));
+        if (dt == PGK_F32) PGK_CHECK_HIP((a.n > 512 ? conv_rows_launch<float, float, float, 2>(a, st) : conv_rows_launch<float, float, float, 1>(a, st)));
+        else PGK_CHECK_HIP((a.n > 512 ? conv_rows_launch<bf16, bf16, bf16, 2>(a, st) : conv_rows_launch<bf16, bf16, bf16, 1>(a, st)));
         return PGK_OK;
     }
-    const int threads = quads > 512 ? 1024 : quads > 256 ? 512 : 256;
-    if (dt == PGK_F32) PGK_CHECK_HIP((conv_rows_launch<float, float, float, 1>(a, threads, st)));
-    else if (in32) PGK_CHECK_HIP((q32 ? conv_rows_launch<bf16, float, float, 1>(a, threads, st) : conv_rows_launch<bf16, float, bf16, 1>(a, threads, st)));
-    else PGK_CHECK_HIP((q32 ? conv_rows_launch<bf16, bf16, float, 1>(a, threads, st) : conv_rows_launch<bf16, bf16, bf16, 1>(a, threads, st)));
+    if (dt == PGK_F32) PGK_CHECK_HIP((conv_rows_launch<float, float, float, 1>(a, st)));
+    else if (in32) PGK_CHECK_HIP((q32 ? conv_rows_launch<bf16, float, float, 1>(a, st) : conv_rows_launch<bf16, float, bf16, 1>(a, st)));
+    else PGK_CHECK_HIP((q32 ? conv_rows_launch<bf16, bf16, float, 1>(a, st) : conv_rows_launch<bf16, bf16, bf16, 1>(a, st)));
     return PGK_OK;
 }
 

@@ -17,11 +17,14 @@
 
 namespace pgk {
 
-__device__ __forceinline__ float rc_sigmoid(float z) { return 1.0f / (1.0f + expf(-z)); }
+// EXACT: the fp32 engines' form; otherwise the hardware's exponential and reciprocal (fp32, a few units in the last place)
+template <bool EXACT> __device__ __forceinline__ float rc_exp(float z) { return EXACT ? expf(z) : __expf(z); }
+template <bool EXACT> __device__ __forceinline__ float rc_recip(float z) { return EXACT ? 1.0f / z : __builtin_amdgcn_rcpf(z); }
+template <bool EXACT> __device__ __forceinline__ float rc_silu(float z) { return z * rc_recip<EXACT>(1.0f + rc_exp<EXACT>(-z)); }
 
 // forget gate and write strength: f = l + (1 - l) sigmoid(z), 1 - f = (1 - l) sigmoid(-z) (no cancellation near f = 1)
-__device__ __forceinline__ void rc_gate(float z, float lower, float& f, float& k) {
-    const float e = expf(-fabsf(z)), big = 1.0f / (1.0f + e), small = e * big;
+template <bool EXACT> __device__ __forceinline__ void rc_gate(float z, float lower, float& f, float& k) {
+    const float e = rc_exp<EXACT>(-fabsf(z)), big = rc_recip<EXACT>(1.0f + e), small = e * big;
     f = fmaf(1.0f - lower, z >= 0.f ? big : small, lower);
     k = (1.0f - lower) * (z >= 0.f ? small : big);
 }
@@ -29,7 +32,7 @@ __device__ __forceinline__ void rc_gate(float z, float lower, float& f, float& k
 // -------------------------------------------------------------------------------------------- token by token
 // One workgroup per (sequence, head).  A thread owns VEC columns of every NG-th state row (VEC = 4: one 16-byte access each); a
 // sequence that starts (position 0) begins with a zero state without reading the slot.
-template <class IT, int VEC>
+template <class IT, bool EXACT, int VEC>
 __global__ __launch_bounds__(512) void recur_scan_kernel(unsigned long long* tl, RecurArgs a) {
     const TLStamp tls(tl);
     extern __shared__ float sm[];
@@ -46,8 +49,8 @@ __global__ __launch_bounds__(512) void recur_scan_kernel(unsigned long long* tl,
         const bool fresh = s.start + t == 0;
         for (int d = tid; d < dim; d += NT) {
             const float zq = to_f(in[a.q_off + h * dim + d]), zf = to_f(in[a.f_off + h * dim + d]) + (a.bias ? a.bias[h * dim + d] : 0.f);
-            q[d] = zq * rc_sigmoid(zq);
-            rc_gate(zf, a.lower[h * dim + d], f[d], k[d]);
+            q[d] = rc_silu<EXACT>(zq);
+            rc_gate<EXACT>(zf, a.lower[h * dim + d], f[d], k[d]);
         }
         for (int i = tid; i < vdim; i += NT) v[i] = to_f(in[a.v_off + h * vdim + i]);
         __syncthreads();
@@ -106,26 +109,31 @@ __global__ __launch_bounds__(512) void recur_scan_kernel(unsigned long long* tl,
     tls.end();
 }
 
-template <class IT>
+template <class IT, bool EXACT>
 static pgk_status recur_scan(const RecurArgs& a, hipStream_t st) {
     const int B = a.seqs ? a.n_seqs : a.n, threads = a.dim * a.vdim >= 8192 ? 512 : 256;
     const bool vec = a.vdim % 4 == 0;
     const int cols = vec ? a.vdim / 4 : a.vdim, groups = threads / cols > 0 ? threads / cols : 1;
     const size_t lds = (size_t)(3 * a.dim + a.vdim + groups * a.vdim) * 4;
     PGK_REQUIRE(lds <= 64 * 1024, "recurrence: head widths %d / %d do not fit LDS", a.dim, a.vdim);
-    if (vec) PGK_CHECK_HIP(launch_k(&recur_scan_kernel<IT, 4>, dim3(a.H, B), dim3(threads), lds, st, a));
-    else PGK_CHECK_HIP(launch_k(&recur_scan_kernel<IT, 1>, dim3(a.H, B), dim3(threads), lds, st, a));
+    if (vec) PGK_CHECK_HIP(launch_k(&recur_scan_kernel<IT, EXACT, 4>, dim3(a.H, B), dim3(threads), lds, st, a));
+    else PGK_CHECK_HIP(launch_k(&recur_scan_kernel<IT, EXACT, 1>, dim3(a.H, B), dim3(threads), lds, st, a));
     return PGK_OK;
 }
 
 pgk_status recur_rows(const RecurArgs& a, pgk_dtype dt, bool io32, hipStream_t st) {
     PGK_REQUIRE(a.H >= 1 && a.dim >= 1 && a.vdim >= 1 && a.ld_out >= a.H * a.vdim && (a.seqs || a.positions), "recurrence: bad sizes");
-    return dt == PGK_F32 || io32 ? recur_scan<float>(a, st) : recur_scan<bf16>(a, st);
+    if (dt == PGK_F32) return recur_scan<float, true>(a, st);
+    return io32 ? recur_scan<float, false>(a, st) : recur_scan<bf16, false>(a, st);
 }
 
 // -------------------------------------------------------------------------------------------- chunks
 typedef float f32x4_rc __attribute__((ext_vector_type(4)));
 __device__ __forceinline__ f32x4_rc mfma4(float a, float b, f32x4_rc c) { return __builtin_amdgcn_mfma_f32_16x16x4f32(a, b, c, 0, 0, 0); }
+// Four products in a row take k in the order 4 (lane >> 4) + step instead of 4 step + (lane >> 4), where both operands can: a lane's four
+// values of a row are then neighbours, one 16-byte access.
+__device__ __forceinline__ float4 ld4(const float* p) { return *reinterpret_cast<const float4*>(p); }
+__device__ __forceinline__ float4 mul4(const float4& a, const float4& b) { return make_float4(a.x * b.x, a.y * b.y, a.z * b.z, a.w * b.w); }
 
 // LDS row strides (floats; widths are multiples of 16).  Operands whose k index runs over rows want 16 x odd, those whose k index runs
 // along a row want 4 x odd: the 64 lanes of a load then fall on 64 banks.
@@ -144,73 +152,79 @@ int recur_chunk_rows(int dim, int vdim) {
 }
 size_t recur_chunk_bytes(const RecurArgs& a, int n_chunks) { return (size_t)n_chunks * a.H * ((size_t)a.dim * a.vdim + a.dim) * 4; }
 
-// 1: U [chunk][head][dim][vdim], D [chunk][head][dim]
-template <class T, int C>
-__global__ __launch_bounds__(256) void recur_chunk_state_kernel(RecurArgs a, const RecurChunk* chunks, float* U, float* D) {
+// 1: U [chunk][head][dim][vdim], D [chunk][head][dim].  Eight waves; VT column tiles of 16 at a time (vdim is a multiple of 16 VT).
+template <class T, int C, int VT>
+__global__ __launch_bounds__(512) void recur_chunk_state_kernel(RecurArgs a, const RecurChunk* chunks, float* U, float* D) {
     extern __shared__ __attribute__((aligned(16))) float sm[];
-    constexpr int NS = C / 16;
+    constexpr int NS = C / 16, VB = 4;
+    constexpr bool EXACT = std::is_same<T, float>::value;
     const int dim = a.dim, vdim = a.vdim, ks = rc_col_stride(dim), vs = rc_col_stride(vdim), h = blockIdx.x;
     float *kr = sm, *v = kr + C * ks, *F = v + C * vs;
     const RecurChunk ch = chunks[blockIdx.y];
-    const int tid = threadIdx.x, lane = tid & 63, wid = tid >> 6, l15 = lane & 15, q4 = lane >> 4;
+    const int tid = threadIdx.x, lane = tid & 63, wid = tid >> 6, l15 = lane & 15, q4 = lane >> 4, last = ch.len - 1;
     const T* in = reinterpret_cast<const T*>(a.in) + (size_t)ch.row0 * a.ld_in;
-    // k times the decay to the end of its block of 16 rows, and the blocks' decays
-    for (int t = tid; t < NS * dim; t += 256) {
-        const int b = t / dim, d = t % dim;
+    const T* vin = in + a.v_off + h * vdim;
+    const int nv = C * vdim / 4, v4 = vdim / 4;
+    // k times the decay to the end of its block of 16 rows, and the blocks' decays; the first values travel with the first gates
+    float4 vv[VB];
+    for (int t = tid, t0 = 0; t < NS * dim || t0 == 0; t += 512, t0 = 1) {
+        const int b = min(t / dim, NS - 1), d = t % dim;
         const T* z = in + a.f_off + h * dim + d;
-        const float bias = a.bias ? a.bias[h * dim + d] : 0.f, low = a.lower[h * dim + d];
         float zf[16];
 #pragma unroll
-        for (int r = 0; r < 16; ++r) zf[r] = to_f(z[(size_t)min(16 * b + r, ch.len - 1) * a.ld_in]);
+        for (int r = 0; r < 16; ++r) zf[r] = to_f(z[(size_t)min(16 * b + r, last) * a.ld_in]);
+        const float bias = a.bias ? a.bias[h * dim + d] : 0.f, low = a.lower[h * dim + d];
+        if (t0 == 0) {
+#pragma unroll
+            for (int i = 0; i < VB; ++i) { const int e = min(tid + 512 * i, nv - 1); vv[i] = load4<T>(vin + (size_t)min(e / v4, last) * a.ld_in + e % v4 * 4); }
+        }
         float run = 1.f;
 #pragma unroll
         for (int r = 15; r >= 0; --r) {
             float f, k;
-            rc_gate(zf[r] + bias, low, f, k);
-            const bool live = 16 * b + r < ch.len;
-            kr[(16 * b + r) * ks + d] = live ? k * run : 0.f;
+            rc_gate<EXACT>(zf[r] + bias, low, f, k);
+            const bool live = 16 * b + r <= last;
+            if (t < NS * dim) kr[(16 * b + r) * ks + d] = live ? k * run : 0.f;
             run *= live ? f : 1.f;
         }
-        F[b * dim + d] = run;
+        if (t < NS * dim) F[b * dim + d] = run;
     }
-    for (int t = tid; t < C * vdim / 4; t += 256) {
-        const int r = t / (vdim / 4), c = t % (vdim / 4) * 4;
-        *reinterpret_cast<float4*>(v + r * vs + c) = load4<T>(in + (size_t)min(r, ch.len - 1) * a.ld_in + a.v_off + h * vdim + c);
-    }
+#pragma unroll
+    for (int i = 0; i < VB; ++i) { const int e = tid + 512 * i; if (e < nv) *reinterpret_cast<float4*>(v + e / v4 * vs + e % v4 * 4) = vv[i]; }
+    for (int e = tid + 512 * VB; e < nv; e += 512) *reinterpret_cast<float4*>(v + e / v4 * vs + e % v4 * 4) = load4<T>(vin + (size_t)min(e / v4, last) * a.ld_in + e % v4 * 4);
     __syncthreads();
     const size_t rec = (size_t)blockIdx.y * a.H + h;
-    for (int d = tid; d < dim; d += 256) {
+    for (int d = tid; d < dim; d += 512) {
         float run = 1.f;
 #pragma unroll
         for (int b = 0; b < NS; ++b) run *= F[b * dim + d];
         D[rec * dim + d] = run;
     }
     float* u = U + rec * dim * vdim;
-    for (int dt = wid; dt < dim / 16; dt += 4) {
-        float m[NS];                                               // decay from a block's end to the chunk's
-        m[NS - 1] = 1.f;
+    for (int dt = wid; dt < dim / 16; dt += 8) {
+        float x[NS][4], m = 1.f;                                   // k times the decay to the chunk's end
 #pragma unroll
-        for (int b = NS - 2; b >= 0; --b) m[b] = m[b + 1] * F[(b + 1) * dim + 16 * dt + l15];
-        for (int v0 = 0; v0 < vdim; v0 += 128) {
-            f32x4_rc acc[8];
+        for (int b = NS - 1; b >= 0; --b) {
 #pragma unroll
-            for (int t = 0; t < 8; ++t) acc[t] = f32x4_rc{0.f, 0.f, 0.f, 0.f};
+            for (int s = 0; s < 4; ++s) x[b][s] = kr[(16 * b + 4 * s + q4) * ks + 16 * dt + l15] * m;
+            m *= F[b * dim + 16 * dt + l15];
+        }
+        for (int v0 = 0; v0 < vdim; v0 += 16 * VT) {
+            f32x4_rc acc[VT];
+#pragma unroll
+            for (int t = 0; t < VT; ++t) acc[t] = f32x4_rc{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
             for (int b = 0; b < NS; ++b)
 #pragma unroll
                 for (int s = 0; s < 4; ++s) {
-                    const int j = 16 * b + 4 * s + q4;
-                    const float x = kr[j * ks + 16 * dt + l15] * m[b];
+                    const float* vr = v + (16 * b + 4 * s + q4) * vs + v0 + l15;
 #pragma unroll
-                    for (int t = 0; t < 8; ++t)
-                        if (v0 + 16 * t < vdim) acc[t] = mfma4(x, v[j * vs + v0 + 16 * t + l15], acc[t]);       // wave-uniform
+                    for (int t = 0; t < VT; ++t) acc[t] = mfma4(x[b][s], vr[16 * t], acc[t]);
                 }
 #pragma unroll
-            for (int t = 0; t < 8; ++t)
-                if (v0 + 16 * t < vdim) {
+            for (int t = 0; t < VT; ++t)
 #pragma unroll
-                    for (int r = 0; r < 4; ++r) u[(size_t)(16 * dt + 4 * q4 + r) * vdim + v0 + 16 * t + l15] = acc[t][r];
-                }
+                for (int r = 0; r < 4; ++r) u[(size_t)(16 * dt + 4 * q4 + r) * vdim + v0 + 16 * t + l15] = acc[t][r];
         }
     }
 }
@@ -244,34 +258,69 @@ __global__ __launch_bounds__(256) void recur_chunk_scan_kernel(RecurArgs a, cons
     *st = S;
 }
 
-// 3: output rows.  Eight waves; NVT column tiles of 16 per wave.
+// 3: output rows.  Eight waves; NVT column tiles of 16 per wave.  The values and the first rows of the state travel while the gates and
+// the decays are worked out.
 template <class T, int C, int NVT>
 __global__ __launch_bounds__(512) void recur_chunk_out_kernel(RecurArgs a, const RecurChunk* chunks, const float* U) {
     extern __shared__ __attribute__((aligned(16))) float sm[];
     constexpr int NS = C / 16, AS = rc_row_stride(C);
+    constexpr bool EXACT = std::is_same<T, float>::value;
     const int dim = a.dim, vdim = a.vdim, S = rc_row_stride(dim), h = blockIdx.x;
     float *q = sm, *f = q + C * S, *k = f + C * S, *A = k + C * S, *F = A + C * AS, *red = F + NS * dim;
     const RecurChunk ch = chunks[blockIdx.y];
     const int tid = threadIdx.x, lane = tid & 63, wid = tid >> 6, l15 = lane & 15, q4 = lane >> 4;
     const T* in = reinterpret_cast<const T*>(a.in) + (size_t)ch.row0 * a.ld_in;
-    for (int t = tid; t < C * dim / 4; t += 512) {
-        const int r = t / (dim / 4), c = t % (dim / 4) * 4, rr = min(r, ch.len - 1);
-        const float4 zq = load4<T>(in + (size_t)rr * a.ld_in + a.q_off + h * dim + c), zf = load4<T>(in + (size_t)rr * a.ld_in + a.f_off + h * dim + c);
+    const int nz = C * dim / 4, d4 = dim / 4, last = ch.len - 1;
+    const float* st = U + ((size_t)blockIdx.y * a.H + h) * dim * vdim;
+    constexpr int ZB = 4, PRE = 8 / NVT;                           // pieces of the rows requested first; blocks of 16 state rows requested ahead
+    float4 pq[ZB], pf[ZB];
+#pragma unroll
+    for (int i = 0; i < ZB; ++i) {
+        const int t = min(tid + 512 * i, nz - 1);
+        const T* row = in + (size_t)min(t / d4, last) * a.ld_in + h * dim + t % d4 * 4;
+        pq[i] = load4<T>(row + a.q_off);
+        pf[i] = load4<T>(row + a.f_off);
+    }
+    int col[NVT];                                                  // this lane's column of each tile (tiles beyond the last repeat it)
+#pragma unroll
+    for (int t = 0; t < NVT; ++t) col[t] = min(16 * (wid + 8 * t), vdim - 16) + l15;
+    float pv[NVT][NS][4], ps[NVT][PRE][4];
+    const T* v = in + a.v_off + h * vdim;
+#pragma unroll
+    for (int t = 0; t < NVT; ++t) {
+#pragma unroll
+        for (int b = 0; b < NS; ++b)
+#pragma unroll
+            for (int u = 0; u < 4; ++u) pv[t][b][u] = to_f(v[(size_t)min(16 * b + 4 * q4 + u, last) * a.ld_in + col[t]]);
+#pragma unroll
+        for (int b = 0; b < PRE; ++b)
+#pragma unroll
+            for (int u = 0; u < 4; ++u) ps[t][b][u] = st[(size_t)min(16 * b + 4 * q4 + u, dim - 1) * vdim + col[t]];
+    }
+    auto gates = [&](int t, const float4& zq, const float4& zf) {
+        const int r = t / d4, c = t % d4 * 4;
         const float4 b = a.bias ? *reinterpret_cast<const float4*>(a.bias + h * dim + c) : make_float4(0.f, 0.f, 0.f, 0.f);
         const float4 low = *reinterpret_cast<const float4*>(a.lower + h * dim + c);
-        float4 qq = {zq.x * rc_sigmoid(zq.x), zq.y * rc_sigmoid(zq.y), zq.z * rc_sigmoid(zq.z), zq.w * rc_sigmoid(zq.w)}, ff, kk;
-        rc_gate(zf.x + b.x, low.x, ff.x, kk.x); rc_gate(zf.y + b.y, low.y, ff.y, kk.y);
-        rc_gate(zf.z + b.z, low.z, ff.z, kk.z); rc_gate(zf.w + b.w, low.w, ff.w, kk.w);
+        float4 qq = {rc_silu<EXACT>(zq.x), rc_silu<EXACT>(zq.y), rc_silu<EXACT>(zq.z), rc_silu<EXACT>(zq.w)}, ff, kk;
+        rc_gate<EXACT>(zf.x + b.x, low.x, ff.x, kk.x); rc_gate<EXACT>(zf.y + b.y, low.y, ff.y, kk.y);
+        rc_gate<EXACT>(zf.z + b.z, low.z, ff.z, kk.z); rc_gate<EXACT>(zf.w + b.w, low.w, ff.w, kk.w);
         if (r >= ch.len) { qq = kk = make_float4(0.f, 0.f, 0.f, 0.f); ff = make_float4(1.f, 1.f, 1.f, 1.f); }
         *reinterpret_cast<float4*>(q + r * S + c) = qq;
         *reinterpret_cast<float4*>(f + r * S + c) = ff;
         *reinterpret_cast<float4*>(k + r * S + c) = kk;
+    };
+#pragma unroll
+    for (int i = 0; i < ZB; ++i) if (tid + 512 * i < nz) gates(tid + 512 * i, pq[i], pf[i]);
+    for (int t = tid + 512 * ZB; t < nz; t += 512) {
+        const T* row = in + (size_t)min(t / d4, last) * a.ld_in + h * dim + t % d4 * 4;
+        gates(t, load4<T>(row + a.q_off), load4<T>(row + a.f_off));
     }
     __syncthreads();
     // diagonal blocks, pair by pair: two waves per block, rows 0..7 and 8..15.  Lane: column j = lane & 7 (and j + 8), every eighth
     // group of 8 channels; w = k_j times the decay from j to the row at hand.
     if ((wid >> 1) < NS) {
-        const int r0 = 16 * (wid >> 1), half = wid & 1, jl = lane & 7, dg = lane >> 3;
+        // (waves w and w + 4 share a SIMD: one of them takes the shorter half)
+        const int r0 = 16 * (wid >> 1), half = (wid ^ (wid >> 2)) & 1, jl = lane & 7, dg = lane >> 3;
         float lo[8], hi[8];
 #pragma unroll
         for (int i = 0; i < 8; ++i) lo[i] = hi[i] = 0.f;
@@ -351,63 +400,73 @@ __global__ __launch_bounds__(512) void recur_chunk_out_kernel(RecurArgs a, const
     for (int p = wid; p < NS * (NS - 1) / 2; p += 8) {
         int bi = 1, bj = p;
         while (bj >= bi) { bj -= bi; ++bi; }
-        f32x4_rc acc = {0.f, 0.f, 0.f, 0.f};
-        for (int d0 = 0; d0 < dim; d0 += 4) {
-            const int d = d0 + q4;
-            float x = q[(16 * bi + l15) * S + d];
-            for (int b = bj + 1; b < bi; ++b) x *= F[b * dim + d];
-            acc = mfma4(x, k[(16 * bj + l15) * S + d], acc);
+        f32x4_rc acc[4];
+#pragma unroll
+        for (int u = 0; u < 4; ++u) acc[u] = f32x4_rc{0.f, 0.f, 0.f, 0.f};
+#pragma unroll 2
+        for (int d0 = 0; d0 < dim; d0 += 16) {
+            const int d = d0 + 4 * q4;
+            float4 x = ld4(q + (16 * bi + l15) * S + d);
+            const float4 y = ld4(k + (16 * bj + l15) * S + d);
+            if (bj + 1 < bi) x = mul4(x, ld4(F + (bj + 1) * dim + d));
+            if (bj + 2 < bi) x = mul4(x, ld4(F + (bj + 2) * dim + d));        // (NS <= 4: at most two blocks between)
+            acc[0] = mfma4(x.x, y.x, acc[0]); acc[1] = mfma4(x.y, y.y, acc[1]);
+            acc[2] = mfma4(x.z, y.z, acc[2]); acc[3] = mfma4(x.w, y.w, acc[3]);
         }
 #pragma unroll
-        for (int r = 0; r < 4; ++r) A[(16 * bi + 4 * q4 + r) * AS + 16 * bj + l15] = acc[r];
+        for (int r = 0; r < 4; ++r) A[(16 * bi + 4 * q4 + r) * AS + 16 * bj + l15] = (acc[0][r] + acc[1][r]) + (acc[2][r] + acc[3][r]);
     }
     __syncthreads();
     // o = q S + A v: a wave has every row of its column tiles
-    const float* st = U + ((size_t)blockIdx.y * a.H + h) * dim * vdim;
     f32x4_rc o[NVT][NS];
 #pragma unroll
     for (int t = 0; t < NVT; ++t)
 #pragma unroll
         for (int b = 0; b < NS; ++b) o[t][b] = f32x4_rc{0.f, 0.f, 0.f, 0.f};
-    constexpr int SU = 4;                                          // k-steps whose state rows are requested together
-    for (int d0 = 0; d0 < dim; d0 += 4 * SU) {
-        float x[NVT][SU];
+    auto rows16 = [&](int d0, const float (&x)[NVT][4]) {          // 16 state rows
+        const int d = d0 + 4 * q4;
+        float4 y[NS], m = ld4(F + d);
 #pragma unroll
-        for (int t = 0; t < NVT; ++t)
-#pragma unroll
-            for (int u = 0; u < SU; ++u) x[t][u] = st[(size_t)(d0 + 4 * u + q4) * vdim + min(16 * (wid + 8 * t), vdim - 16) + l15];
-#pragma unroll
-        for (int u = 0; u < SU; ++u) {
-            const int d = d0 + 4 * u + q4;
-            float m = 1.f;
-#pragma unroll
-            for (int b = 0; b < NS; ++b) {
-                const float y = q[(16 * b + l15) * S + d] * m;
-#pragma unroll
-                for (int t = 0; t < NVT; ++t) o[t][b] = mfma4(y, x[t][u], o[t][b]);
-                m *= F[b * dim + d];
-            }
+        for (int b = 0; b < NS; ++b) {
+            y[b] = ld4(q + (16 * b + l15) * S + d);
+            if (b > 0) y[b] = mul4(y[b], m);
+            if (b > 0 && b + 1 < NS) m = mul4(m, ld4(F + b * dim + d));
         }
-    }
-    const T* v = in + a.v_off + h * vdim;
 #pragma unroll
-    for (int bj = 0; bj < NS; ++bj) {
+        for (int u = 0; u < 4; ++u)
+#pragma unroll
+            for (int b = 0; b < NS; ++b)
+#pragma unroll
+                for (int t = 0; t < NVT; ++t) o[t][b] = mfma4(u == 0 ? y[b].x : u == 1 ? y[b].y : u == 2 ? y[b].z : y[b].w, x[t][u], o[t][b]);
+    };
+#pragma unroll
+    for (int i = 0; i < PRE; ++i)
+        if (16 * i < dim) {                                        // uniform
+            float x[NVT][4];
+#pragma unroll
+            for (int t = 0; t < NVT; ++t)
+#pragma unroll
+                for (int u = 0; u < 4; ++u) x[t][u] = ps[t][i][u];
+            rows16(16 * i, x);
+        }
+    for (int d0 = 16 * PRE; d0 < dim; d0 += 16) {
         float x[NVT][4];
 #pragma unroll
         for (int t = 0; t < NVT; ++t)
 #pragma unroll
-            for (int u = 0; u < 4; ++u) x[t][u] = to_f(v[(size_t)min(16 * bj + 4 * u + q4, ch.len - 1) * a.ld_in + min(16 * (wid + 8 * t), vdim - 16) + l15]);
-#pragma unroll
-        for (int b = 0; b < NS; ++b) {
-            if (b < bj) continue;
-#pragma unroll
-            for (int u = 0; u < 4; ++u) {
-                const float y = A[(16 * b + l15) * AS + 16 * bj + 4 * u + q4];
-#pragma unroll
-                for (int t = 0; t < NVT; ++t) o[t][b] = mfma4(y, x[t][u], o[t][b]);
-            }
-        }
+            for (int u = 0; u < 4; ++u) x[t][u] = st[(size_t)(d0 + 4 * q4 + u) * vdim + col[t]];
+        rows16(d0, x);
     }
+#pragma unroll
+    for (int bj = 0; bj < NS; ++bj)
+#pragma unroll
+        for (int b = bj; b < NS; ++b) {
+            const float4 y = ld4(A + (16 * b + l15) * AS + 16 * bj + 4 * q4);
+#pragma unroll
+            for (int u = 0; u < 4; ++u)
+#pragma unroll
+                for (int t = 0; t < NVT; ++t) o[t][b] = mfma4(u == 0 ? y.x : u == 1 ? y.y : u == 2 ? y.z : y.w, pv[t][bj][u], o[t][b]);
+        }
     // lane: rows 16 b + 4 q4 + r, column l15 of each tile
     float inv[NS][4];
 #pragma unroll
@@ -421,16 +480,21 @@ __global__ __launch_bounds__(512) void recur_chunk_out_kernel(RecurArgs a, const
             if (l15 == 0) red[wid * C + 16 * b + 4 * q4 + r] = ss;
         }
     __syncthreads();
+    if (tid < C) {
+        float ss = 0.f;
 #pragma unroll
-    for (int b = 0; b < NS; ++b)
+        for (int w = 0; w < 8; ++w) ss += red[w * C + tid];
+        A[tid] = a.norm ? 1.0f / sqrtf(ss / a.vdim_true + a.eps) : 1.0f;      // (A has been read)
+    }
+    __syncthreads();
 #pragma unroll
-        for (int r = 0; r < 4; ++r) {
-            float ss = 0.f;
-#pragma unroll
-            for (int w = 0; w < 8; ++w) ss += red[w * C + 16 * b + 4 * q4 + r];
-            inv[b][r] = a.norm ? 1.0f / sqrtf(ss / a.vdim_true + a.eps) : 1.0f;
-        }
+    for (int b = 0; b < NS; ++b) {
+        const float4 t = ld4(A + 16 * b + 4 * q4);
+        inv[b][0] = t.x; inv[b][1] = t.y; inv[b][2] = t.z; inv[b][3] = t.w;
+    }
     T* out = reinterpret_cast<T*>(a.out) + (size_t)ch.row0 * a.ld_out;
+    const int ys = rc_row_stride(vdim);
+    const bool staged = ys <= 3 * S;                               // the rows leave through the space of q, f and k (no longer read), whole pieces at a time
 #pragma unroll
     for (int t = 0; t < NVT; ++t) {
         const int c = 16 * (wid + 8 * t) + l15;
@@ -441,8 +505,17 @@ __global__ __launch_bounds__(512) void recur_chunk_out_kernel(RecurArgs a, const
 #pragma unroll
             for (int r = 0; r < 4; ++r) {
                 const int row = 16 * b + 4 * q4 + r;
-                if (row < ch.len) out[(size_t)row * a.ld_out + h * vdim + c] = from_f<T>(o[t][b][r] * inv[b][r] * g);
+                const float y = o[t][b][r] * inv[b][r] * g;
+                if (staged) q[row * ys + c] = y;
+                else if (row < ch.len) out[(size_t)row * a.ld_out + h * vdim + c] = from_f<T>(y);
             }
+    }
+    if (staged) {
+        __syncthreads();
+        for (int t = tid; t < ch.len * (vdim / 4); t += 512) {
+            const int r = t / (vdim / 4), c = t % (vdim / 4) * 4;
+            store4<T>(out + (size_t)r * a.ld_out + h * vdim + c, ld4(q + r * ys + c));
+        }
     }
     if (h == a.H - 1 && a.ld_out > a.H * vdim) {
         const int tail = a.ld_out - a.H * vdim;
@@ -466,14 +539,21 @@ static hipError_t launch_chunk_out(const RecurArgs& a, const RecurChunk* chunks,
     return hipGetLastError();
 }
 
+template <class T, int C, int VT>
+static hipError_t launch_chunk_state(const RecurArgs& a, const RecurChunk* chunks, int n_chunks, float* U, float* D, hipStream_t st) {
+    static bool done = false;
+    const size_t lds = rc_state_lds(C, a.dim, a.vdim);
+    if (hipError_t e = rc_allow_lds(&recur_chunk_state_kernel<T, C, VT>, lds, done)) return e;
+    recur_chunk_state_kernel<T, C, VT><<<dim3(a.H, n_chunks), 512, lds, st>>>(a, chunks, U, D);
+    return hipGetLastError();
+}
+
 template <class T, int C>
 static pgk_status recur_chunked_t(const RecurArgs& a, const RecurChunk* chunks, int n_chunks, const int32_t* chunk_of_seq, void* ws, hipStream_t st) {
     float *U = (float*)ws, *D = U + (size_t)n_chunks * a.H * a.dim * a.vdim;
-    static bool done = false;
-    const size_t lds = rc_state_lds(C, a.dim, a.vdim);
-    PGK_CHECK_HIP(rc_allow_lds(&recur_chunk_state_kernel<T, C>, lds, done));
-    recur_chunk_state_kernel<T, C><<<dim3(a.H, n_chunks), 256, lds, st>>>(a, chunks, U, D);
-    PGK_LAUNCH_CHECK();
+    if (a.vdim % 128 == 0) PGK_CHECK_HIP((launch_chunk_state<T, C, 8>(a, chunks, n_chunks, U, D, st)));
+    else if (a.vdim % 64 == 0) PGK_CHECK_HIP((launch_chunk_state<T, C, 4>(a, chunks, n_chunks, U, D, st)));
+    else PGK_CHECK_HIP((launch_chunk_state<T, C, 1>(a, chunks, n_chunks, U, D, st)));
     recur_chunk_scan_kernel<<<dim3(ceil_div(a.dim * a.vdim / 4, 256), a.H, a.n_seqs), 256, 0, st>>>(a, chunk_of_seq, U, D);
     PGK_LAUNCH_CHECK();
     if (a.vdim <= 128) PGK_CHECK_HIP((launch_chunk_out<T, C, 1>(a, chunks, n_chunks, U, st)));

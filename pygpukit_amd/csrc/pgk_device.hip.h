@@ -39,6 +39,12 @@ template <> __device__ __forceinline__ float from_f<float>(float f) { return f; 
 template <> __device__ __forceinline__ f16 from_f<f16>(float f) { return f16{static_cast<_Float16>(f)}; }
 template <> __device__ __forceinline__ bf16 from_f<bf16>(float f) { return bf16{f_to_bf16_bits(f)}; }
 
+// xIELU with its two softplus'ed factors: z > 0: a z^2 + z / 2,  z <= 0: b (exp(z) - 1 - z) + z / 2  (EXACT: the fp32 engines' form)
+template <bool EXACT> __device__ __forceinline__ float xielu(float z, float a, float b) {
+    const float n = fminf(z, 0.f), e = EXACT ? expm1f(n) : __expf(n) - 1.0f;
+    return fmaf(0.5f, z, z > 0.f ? a * z * z : b * (e - n));
+}
+
 // ---- 16-byte vectors ----------------------------------------------------------------------
 // Vec<T>::N elements of T in one 16-byte access: 4 x fp32 or 8 x 16-bit.
 template <class T> struct Vec {
