@@ -412,7 +412,7 @@ pgk_status pgk_engine_create(const pgk_model_config_t* cfg, const void* embed, c
                              const void* final_norm, const pgk_layer_weights_t* layers, pgk_engine* out);
 /* Layer-list decoders (csrc/engine_stack.hip): fp32 residual stream, a norm after each sublayer and optionally before it, one of
  * several mixers per layer, dense SwiGLU / xIELU or no feed-forward; every layer has its own sizes.  dtype PGK_BF16 or PGK_F32 is the
- * element type of the tables, matrices, activations and caches; norm weights, biases, taps and gates' constants are fp32 with any
+ * element type of the tables, matrices, taps, activations and caches; norm weights, biases and gates' constants are fp32 with any
  * offset applied.  Caller pads with zeros: Wp = width up to a multiple of 64; n_in, n_att and ff_pad multiples of 64 (ff_pad 0: the
  * layer has no feed-forward).
  * PGK_MIX_LATENT     latent attention over a sliding window with a per-head output gate.  head_pad >= dim and vdim: 64, 128 or a
@@ -440,7 +440,8 @@ typedef struct {
     const float *norm1, *norm1b, *norm2, *norm2b;  /* [Wp]; norm1 / norm2 NULL: the sublayer reads the stream itself */
     const void* w_in;                              /* [n_in, Wp] */
     const float* b_in;                             /* [n_in] or NULL */
-    const float *conv, *q_norm, *k_norm, *slopes;  /* attention */
+    const void* conv;                              /* attention */
+    const float *q_norm, *k_norm, *slopes;
     const float *lower, *o_norm;                   /* hgrn2: [heads * head_pad], [vhead_pad] */
     const float* c_norm;                           /* latent: [rank_pad] */
     const void* w_ukv;                             /* latent: [2 heads head_pad, rank_pad]: key rows, then value rows */
@@ -474,8 +475,8 @@ pgk_status pgk_engine_set_state(pgk_engine e, const int32_t* h_tokens, const int
  * token log.  No host interaction: any number of steps can be queued back to back. */
 pgk_status pgk_engine_decode_step(pgk_engine e, int batch, pgk_stream s);
 /* Eager steps whose every launch carries its own start/stop hipEvent (hipExtLaunchKernelGGL: the dispatch's begin -> end
- * interval, what rocprofv3 --kernel-trace reports): per-kernel-class time sums (ms) and launch counts for the 8 classes
- * embed, norm_qkv, attn, oproj, gateup, down, lmhead, argmax (in that order).  Advances the decode state like n_iters
+ * interval, what rocprofv3 --kernel-trace reports): per-kernel-class time sums (ms) and launch counts for the 9 classes
+ * embed, norm_qkv, attn, oproj, gateup, down, lmhead, argmax, recur (in that order).  Advances the decode state like n_iters
  * ordinary steps.  (Measurement only: the reference's counterpart is its KernelProfiler, native/core/profiler.hpp.) */
 pgk_status pgk_engine_profile_step(pgk_engine e, int batch, int n_iters, float* h_ms_sum, int* h_count, pgk_stream s);
 /* Timeline of ONE graph-replayed step (diagnostic): every workgroup of every kernel stamps the 100 MHz s_memrealtime

@@ -38,7 +38,8 @@ __device__ __forceinline__ void split_range(int n, int nsplit, int s, int& k0, i
 // the cache [slot][k, v][head][R][D].
 struct ConvArgs {
     const void* in; int ld_in;
-    const float *bias, *conv;             // [channels] or null; [taps][channels] or null (no taps)
+    const float* bias;                    // [channels] or null
+    const void* conv;                     // [taps][channels] (element type) or null (no taps)
     int taps, n_q, n_kv, D, n, R;
     const float *q_norm, *k_norm;         // [n_q], [n_kv]; null: no norm
     int q_true, k_true;                   // channels that are not padding

@@ -12,9 +12,9 @@ constexpr float GA_LOG2E = 1.4426950408889634f;
 // -------------------------------------------------------------------------------------------- short convolution, norms
 // Where the channels c .. c + 3 (all of q, of k or of v) of one row go: normalised values to q_out, or to the scratch row and the cache.
 template <class T, class QT>
-__device__ __forceinline__ void conv_store(const ConvArgs& a, int row, int pos, int slot, int c, float4 y, float inv_q, float inv_k) {
+__device__ __forceinline__ void conv_store(const ConvArgs& a, int row, int pos, int slot, int c, float4 y, float inv) {
     if (c < a.n_q) {
-        const float s = a.q_norm ? inv_q * a.q_mult : a.q_mult;
+        const float s = a.q_norm ? inv * a.q_mult : a.q_mult;
         const float4 g = a.q_norm ? *reinterpret_cast<const float4*>(a.q_norm + c) : make_float4(1.f, 1.f, 1.f, 1.f);
         y.x *= s * g.x; y.y *= s * g.y; y.z *= s * g.z; y.w *= s * g.w;
         store4<QT>(reinterpret_cast<QT*>(a.q_out) + (size_t)row * a.ld_q + c, y);
@@ -24,7 +24,7 @@ __device__ __forceinline__ void conv_store(const ConvArgs& a, int row, int pos, 
     const int kc = c - a.n_q - (is_k ? 0 : a.n_kv);
     if (is_k && a.k_norm) {
         const float4 g = *reinterpret_cast<const float4*>(a.k_norm + kc);
-        y.x *= inv_k * g.x; y.y *= inv_k * g.y; y.z *= inv_k * g.z; y.w *= inv_k * g.w;
+        y.x *= inv * g.x; y.y *= inv * g.y; y.z *= inv * g.z; y.w *= inv * g.w;
     }
     if (a.place) {
         const RowPlace p = a.place[row];
@@ -34,20 +34,24 @@ __device__ __forceinline__ void conv_store(const ConvArgs& a, int row, int pos, 
     store4<T>(reinterpret_cast<T*>(a.cache) + ((((size_t)slot * 2 + (is_k ? 0 : 1)) * (a.n_kv / a.D) + kc / a.D) * a.R + pos % a.R) * a.D + kc % a.D, y);
 }
 
-// Per-row scales of q and k from per-thread sums of squares (q, k of every row in turn)
+// blockIdx.y: 0 works on q, 1 on k and v.  Per-row scale of the part's norm from per-thread sums of squares
+__device__ __forceinline__ void conv_part(const ConvArgs& a, int& c0, int& c1) {
+    c0 = blockIdx.y ? a.n_q : 0;
+    c1 = blockIdx.y ? a.n_q + 2 * a.n_kv : a.n_q;
+}
 template <int RB>
-__device__ __forceinline__ void conv_scales(const ConvArgs& a, float (&ss)[2 * RB], float (&red)[16][2 * RB], float (&inv)[2 * RB]) {
+__device__ __forceinline__ void conv_scales(const ConvArgs& a, float (&ss)[RB], float (&red)[16][RB], float (&inv)[RB]) {
 #pragma unroll
-    for (int i = 0; i < 2 * RB; ++i) {
+    for (int i = 0; i < RB; ++i) {
         const float t = wave_sum(ss[i]);
         if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6][i] = t;
     }
     __syncthreads();
 #pragma unroll
-    for (int i = 0; i < 2 * RB; ++i) {
+    for (int i = 0; i < RB; ++i) {
         float t = 0.f;
         for (int w = 0; w < (int)(blockDim.x >> 6); ++w) t += red[w][i];
-        inv[i] = 1.0f / sqrtf(t / ((i & 1) ? max(a.k_true, 1) : a.q_true) + a.eps);
+        inv[i] = 1.0f / sqrtf(t / (blockIdx.y ? a.k_true : a.q_true) + a.eps);
     }
 }
 
@@ -55,102 +59,112 @@ __device__ __forceinline__ RowSrc conv_row(const ConvArgs& a, int r) {
     return a.rows ? a.rows[r] : RowSrc{max(a.positions[r], 0), r, r};
 }
 
-// Up to four taps: RB rows and QPT groups of four channels per thread, everything requested up front and kept in registers.  Rows of one
-// portion share the rows above them (a window of RB + 3 loads); a workgroup that spans two portions loads each row's taps by itself.
+// four elements as they come from memory
+template <class T> struct Raw4;
+template <> struct Raw4<float> {
+    float4 v;
+    __device__ __forceinline__ void load(const float* p) { v = *reinterpret_cast<const float4*>(p); }
+    __device__ __forceinline__ float4 get() const { return v; }
+};
+template <> struct Raw4<bf16> {
+    uint2 v;
+    __device__ __forceinline__ void load(const bf16* p) { v = *reinterpret_cast<const uint2*>(p); }
+    __device__ __forceinline__ float4 get() const {
+        return make_float4(__uint_as_float(v.x << 16), __uint_as_float(v.x & 0xFFFF0000u), __uint_as_float(v.y << 16), __uint_as_float(v.y & 0xFFFF0000u));
+    }
+};
+
+// Up to four taps.  A workgroup walks `span` rows, RB at a time, QPT groups of four channels per thread: the taps' weights and the last
+// three rows stay in registers, the next RB rows travel while these are normalised and stored.  At a portion's first row (and the
+// workgroup's) the rows above come from the slot's ring or the rows above.
 constexpr int CONV_MT = 4;
 template <class T, class IT, class QT, int RB, int QPT>
-__global__ __launch_bounds__(1024, RB * QPT <= 2 ? 8 : 4) void conv_rows_kernel(unsigned long long* tl, ConvArgs a) {
+__global__ __launch_bounds__(1024) void conv_rows_kernel(unsigned long long* tl, ConvArgs a, int span) {
     const TLStamp tls(tl);
-    __shared__ float red[16][2 * RB];
-    constexpr int NW = RB + CONV_MT - 1;
-    const int taps = a.taps, nc = a.n_q + 2 * a.n_kv, nt = blockDim.x, r0 = blockIdx.x * RB, last = a.n - 1;
+    __shared__ float red[2][16][RB];
+    const int taps = a.taps, nc = a.n_q + 2 * a.n_kv, nt = blockDim.x, begin = blockIdx.x * span, end = min(begin + span, a.n);
+    int c0, c1;
+    conv_part(a, c0, c1);
+    const int normed = blockIdx.y ? a.n_q + a.n_kv : a.n_q;
+    const T* conv = reinterpret_cast<const T*>(a.conv);
     const IT* in = reinterpret_cast<const IT*>(a.in);
     T* ring = reinterpret_cast<T*>(a.tap_ring);
-    RowSrc src[RB];
-#pragma unroll
-    for (int m = 0; m < RB; ++m) src[m] = conv_row(a, min(r0 + m, last));
-    int c[QPT];
-    float4 b[QPT], w[QPT][CONV_MT], y[QPT][RB];
     const float4 zero = {0.f, 0.f, 0.f, 0.f};
-    // the projected values of position pos - back for the row `r` of portion s (zero before the sequence's start, bias included)
-    auto fetch = [&](const RowSrc& s, int r, int back, int cc) -> float4 {
-        const int p = s.pos - back;
-        if (p < 0 || back >= taps) return zero;
-        return r - back >= s.first ? load4<IT>(in + (size_t)(r - back) * a.ld_in + cc) : load4<T>(ring + ((size_t)s.slot * taps + p % taps) * nc + cc);
-    };
+    int c[QPT], cc[QPT];
+    float4 b[QPT], w[QPT][CONV_MT], h[QPT][CONV_MT - 1];          // h[k]: the row k + 1 above
+    Raw4<IT> next[QPT][RB];
+#pragma unroll
+    for (int q = 0; q < QPT; ++q) {
+        c[q] = c0 + 4 * (threadIdx.x + q * nt);
+        cc[q] = min(c[q], c1 - 4);
+#pragma unroll
+        for (int m = 0; m < RB; ++m) next[q][m].load(in + (size_t)min(begin + m, end - 1) * a.ld_in + cc[q]);
+        b[q] = a.bias ? *reinterpret_cast<const float4*>(a.bias + cc[q]) : zero;
+#pragma unroll
+        for (int k = 0; k < CONV_MT; ++k)
+            w[q][k] = k >= taps ? zero : conv ? load4<T>(conv + (size_t)(taps - 1 - k) * nc + cc[q]) : make_float4(1.f, 1.f, 1.f, 1.f);
+    }
     auto add = [](float4 u, const float4& v) { u.x += v.x; u.y += v.y; u.z += v.z; u.w += v.w; return u; };
     auto fma4 = [](const float4& x, const float4& u, float4 acc) {
         acc.x = fmaf(x.x, u.x, acc.x); acc.y = fmaf(x.y, u.y, acc.y); acc.z = fmaf(x.z, u.z, acc.z); acc.w = fmaf(x.w, u.w, acc.w);
         return acc;
     };
-    const bool whole = src[RB - 1].first == src[0].first;          // workgroup-uniform
-    if (whole) {
-        float4 u[QPT][NW];
+    for (int r0 = begin, pass = 0; r0 < end; r0 += RB, pass ^= 1) {
+        Raw4<IT> raw[QPT][RB];
+        RowSrc src[RB];
+        float4 y[QPT][RB];
+        float ss[RB], inv[RB];
 #pragma unroll
-        for (int q = 0; q < QPT; ++q) {
-            c[q] = 4 * (threadIdx.x + q * nt);
-            const int cc = min(c[q], nc - 4);
+        for (int m = 0; m < RB; ++m) { src[m] = conv_row(a, min(r0 + m, end - 1)); ss[m] = 0.f; }
 #pragma unroll
-            for (int i = 0; i < NW; ++i) {
-                const int back = CONV_MT - 1 - i;                  // of row r0: negative for the rows below it
-                u[q][i] = back > 0 ? fetch(src[0], r0, back, cc) : load4<IT>(in + (size_t)min(r0 - back, last) * a.ld_in + cc);
-            }
-            b[q] = a.bias ? *reinterpret_cast<const float4*>(a.bias + cc) : zero;
+        for (int q = 0; q < QPT; ++q)
 #pragma unroll
-            for (int k = 0; k < CONV_MT; ++k)
-                w[q][k] = k >= taps ? zero : a.conv ? *reinterpret_cast<const float4*>(a.conv + (size_t)(taps - 1 - k) * nc + cc) : make_float4(1.f, 1.f, 1.f, 1.f);
+            for (int m = 0; m < RB; ++m) raw[q][m] = next[q][m];
+        if (r0 + RB < end) {
+#pragma unroll
+            for (int q = 0; q < QPT; ++q)
+#pragma unroll
+                for (int m = 0; m < RB; ++m) next[q][m].load(in + (size_t)min(r0 + RB + m, end - 1) * a.ld_in + cc[q]);
         }
 #pragma unroll
-        for (int q = 0; q < QPT; ++q)
+        for (int m = 0; m < RB; ++m) {
+            const int r = min(r0 + m, end - 1);
+            if (r == begin || r == src[m].first) {                 // workgroup-uniform
 #pragma unroll
-            for (int i = 0; i < NW; ++i)
-                if (src[0].pos - (CONV_MT - 1 - i) >= 0) u[q][i] = add(u[q][i], b[q]);
+                for (int k = 0; k < CONV_MT - 1; ++k) {
+                    const int p = src[m].pos - 1 - k;
+                    const bool live = p >= 0 && k + 1 < taps;      // before the sequence's start: zero, bias included
 #pragma unroll
-        for (int q = 0; q < QPT; ++q)
-#pragma unroll
-            for (int m = 0; m < RB; ++m) {
-                y[q][m] = zero;
-#pragma unroll
-                for (int k = 0; k < CONV_MT; ++k) y[q][m] = fma4(w[q][k], u[q][m + CONV_MT - 1 - k], y[q][m]);
-            }
-    } else {
-#pragma unroll
-        for (int q = 0; q < QPT; ++q) {
-            c[q] = 4 * (threadIdx.x + q * nt);
-            const int cc = min(c[q], nc - 4);
-            b[q] = a.bias ? *reinterpret_cast<const float4*>(a.bias + cc) : zero;
-#pragma unroll
-            for (int m = 0; m < RB; ++m) {
-                const int r = min(r0 + m, last);
-                y[q][m] = zero;
-                for (int k = 0; k < taps; ++k) {
-                    if (src[m].pos - k < 0) break;
-                    const float4 x = a.conv ? *reinterpret_cast<const float4*>(a.conv + (size_t)(taps - 1 - k) * nc + cc) : make_float4(1.f, 1.f, 1.f, 1.f);
-                    y[q][m] = fma4(x, add(fetch(src[m], r, k, cc), b[q]), y[q][m]);
+                    for (int q = 0; q < QPT; ++q) {
+                        h[q][k] = zero;
+                        if (live) h[q][k] = add(b[q], r - 1 - k >= src[m].first ? load4<IT>(in + (size_t)(r - 1 - k) * a.ld_in + cc[q])
+                                                                                : load4<T>(ring + ((size_t)src[m].slot * taps + p % taps) * nc + cc[q]));
+                    }
                 }
             }
+#pragma unroll
+            for (int q = 0; q < QPT; ++q) {
+                const float4 u = add(raw[q][m].get(), b[q]);
+                float4 t = fma4(w[q][0], u, zero);
+#pragma unroll
+                for (int k = 0; k < CONV_MT - 1; ++k) t = fma4(w[q][k + 1], h[q][k], t);
+                y[q][m] = t;
+#pragma unroll
+                for (int k = CONV_MT - 2; k > 0; --k) h[q][k] = h[q][k - 1];
+                h[q][0] = u;
+                ss[m] += c[q] < normed ? t.x * t.x + t.y * t.y + t.z * t.z + t.w * t.w : 0.f;
+            }
         }
-    }
-    float ss[2 * RB], inv[2 * RB];
+        conv_scales<RB>(a, ss, red[pass], inv);                    // (one barrier: the other half of `red` is the next pass's)
 #pragma unroll
-    for (int i = 0; i < 2 * RB; ++i) ss[i] = 0.f;
+        for (int q = 0; q < QPT; ++q) {
+            if (c[q] >= c1) break;
 #pragma unroll
-    for (int q = 0; q < QPT; ++q)
-#pragma unroll
-        for (int m = 0; m < RB; ++m) {
-            const float t = y[q][m].x * y[q][m].x + y[q][m].y * y[q][m].y + y[q][m].z * y[q][m].z + y[q][m].w * y[q][m].w;
-            ss[2 * m] += c[q] < a.n_q ? t : 0.f;
-            ss[2 * m + 1] += c[q] >= a.n_q && c[q] < a.n_q + a.n_kv ? t : 0.f;
-        }
-    conv_scales<RB>(a, ss, red, inv);
-#pragma unroll
-    for (int q = 0; q < QPT; ++q) {
-        if (c[q] >= nc) break;
-#pragma unroll
-        for (int m = 0; m < RB; ++m) {
-            if (r0 + m > last) break;
-            conv_store<T, QT>(a, r0 + m, src[m].pos, src[m].slot, c[q], y[q][m], inv[2 * m], inv[2 * m + 1]);
-            if (!a.rows && a.conv) store4<T>(ring + ((size_t)src[m].slot * taps + src[m].pos % taps) * nc + c[q], load4<IT>(in + (size_t)(r0 + m) * a.ld_in + c[q]));
+            for (int m = 0; m < RB; ++m) {
+                if (r0 + m >= end) break;
+                conv_store<T, QT>(a, r0 + m, src[m].pos, src[m].slot, c[q], y[q][m], inv[m]);
+                if (!a.rows && a.conv) store4<T>(ring + ((size_t)src[m].slot * taps + src[m].pos % taps) * nc + c[q], raw[q][m].get());
+            }
         }
     }
     tls.end();
@@ -160,8 +174,11 @@ __global__ __launch_bounds__(1024, RB * QPT <= 2 ? 8 : 4) void conv_rows_kernel(
 template <class T, class IT, class QT>
 __global__ __launch_bounds__(256) void conv_rows_any_kernel(unsigned long long* tl, ConvArgs a) {
     const TLStamp tls(tl);
-    __shared__ float red[16][2];
+    __shared__ float red[16][1];
     const int taps = a.taps, nc = a.n_q + 2 * a.n_kv, r = blockIdx.x;
+    int c0, c1;
+    conv_part(a, c0, c1);
+    const T* conv = reinterpret_cast<const T*>(a.conv);
     const IT* in = reinterpret_cast<const IT*>(a.in);
     T* ring = reinterpret_cast<T*>(a.tap_ring);
     const RowSrc s = conv_row(a, r);
@@ -169,47 +186,57 @@ __global__ __launch_bounds__(256) void conv_rows_any_kernel(unsigned long long* 
         const float4 b = a.bias ? *reinterpret_cast<const float4*>(a.bias + c) : make_float4(0.f, 0.f, 0.f, 0.f);
         float4 y = {0.f, 0.f, 0.f, 0.f};
         for (int back = 0; back < taps && s.pos - back >= 0; ++back) {
-            const float4 w = a.conv ? *reinterpret_cast<const float4*>(a.conv + (size_t)(taps - 1 - back) * nc + c) : make_float4(1.f, 1.f, 1.f, 1.f);
+            const float4 w = conv ? load4<T>(conv + (size_t)(taps - 1 - back) * nc + c) : make_float4(1.f, 1.f, 1.f, 1.f);
             const float4 u = r - back >= s.first ? load4<IT>(in + (size_t)(r - back) * a.ld_in + c) : load4<T>(ring + ((size_t)s.slot * taps + (s.pos - back) % taps) * nc + c);
             y.x = fmaf(w.x, u.x + b.x, y.x); y.y = fmaf(w.y, u.y + b.y, y.y); y.z = fmaf(w.z, u.z + b.z, y.z); y.w = fmaf(w.w, u.w + b.w, y.w);
         }
         return y;
     };
-    float ss[2] = {0.f, 0.f}, inv[2];
-    for (int c = 4 * threadIdx.x; c < a.n_q + a.n_kv; c += 1024) {
+    float ss[1] = {0.f}, inv[1];
+    for (int c = c0 + 4 * threadIdx.x; c < (blockIdx.y ? a.n_q + a.n_kv : a.n_q); c += 1024) {
         const float4 y = conv4(c);
-        ss[c < a.n_q ? 0 : 1] += y.x * y.x + y.y * y.y + y.z * y.z + y.w * y.w;
+        ss[0] += y.x * y.x + y.y * y.y + y.z * y.z + y.w * y.w;
     }
     conv_scales<1>(a, ss, red, inv);
-    for (int c = 4 * threadIdx.x; c < nc; c += 1024) {
-        conv_store<T, QT>(a, r, s.pos, s.slot, c, conv4(c), inv[0], inv[1]);
+    for (int c = c0 + 4 * threadIdx.x; c < c1; c += 1024) {
+        conv_store<T, QT>(a, r, s.pos, s.slot, c, conv4(c), inv[0]);
         // (the row written is read by no tap of this step, and its channels by this thread only)
         if (!a.rows && a.conv) store4<T>(ring + ((size_t)s.slot * taps + s.pos % taps) * nc + c, load4<IT>(in + (size_t)r * a.ld_in + c));
     }
     tls.end();
 }
 
-template <class T, class IT, class QT, int RB>
+template <class T, class IT, class QT, bool PROMPT>
 static hipError_t conv_rows_launch(const ConvArgs& a, hipStream_t st) {
-    const int quads = (a.n_q + 2 * a.n_kv) / 4;
+    const int quads = (a.n_q > 2 * a.n_kv ? a.n_q : 2 * a.n_kv) / 4, parts = a.n_kv ? 2 : 1;     // of the longer part
     auto waves = [](int t) { return (t + 63) / 64 * 64; };
-    if (a.taps > CONV_MT || quads > 4096 || (RB > 1 && quads > 2048)) return launch_k(&conv_rows_any_kernel<T, IT, QT>, dim3(a.n), dim3(256), 0, st, a);
-    if (quads <= 1024) return launch_k(&conv_rows_kernel<T, IT, QT, RB, 1>, dim3(ceil_div(a.n, RB)), dim3(waves(quads)), 0, st, a);
-    if (quads <= 2048) return launch_k(&conv_rows_kernel<T, IT, QT, RB, 2>, dim3(ceil_div(a.n, RB)), dim3(waves((quads + 1) / 2)), 0, st, a);
-    return launch_k(&conv_rows_kernel<T, IT, QT, 1, 4>, dim3(a.n), dim3(waves((quads + 3) / 4)), 0, st, a);
+    if (a.taps > CONV_MT || quads > 4096 || (PROMPT && quads > 2048)) return launch_k(&conv_rows_any_kernel<T, IT, QT>, dim3(a.n, parts), dim3(256), 0, st, a);
+    // prompts: about a workgroup per CU and part, whole batches of rows each
+    auto go = [&](auto kfn, int rb, int qpt) {
+        const int span = PROMPT ? ceil_div(ceil_div(a.n, 256), rb) * rb : 1;
+        return launch_k(kfn, dim3(ceil_div(a.n, span), parts), dim3(waves((quads + qpt - 1) / qpt)), 0, st, a, span);
+    };
+    if constexpr (PROMPT) {
+        if (a.n <= 512) return quads <= 1024 ? go(&conv_rows_kernel<T, IT, QT, 1, 1>, 1, 1) : go(&conv_rows_kernel<T, IT, QT, 1, 2>, 1, 2);
+        return quads <= 1024 ? go(&conv_rows_kernel<T, IT, QT, 4, 1>, 4, 1) : go(&conv_rows_kernel<T, IT, QT, 2, 2>, 2, 2);
+    } else {
+        if (quads <= 1024) return go(&conv_rows_kernel<T, IT, QT, 1, 1>, 1, 1);
+        if (quads <= 2048) return go(&conv_rows_kernel<T, IT, QT, 1, 2>, 1, 2);
+        return go(&conv_rows_kernel<T, IT, QT, 1, 4>, 1, 4);
+    }
 }
 
 pgk_status conv_rows(const ConvArgs& a, pgk_dtype dt, bool in32, bool q32, hipStream_t st) {
     PGK_REQUIRE(a.n >= 1 && a.n_q % 4 == 0 && a.n_kv % 4 == 0 && a.D % 4 == 0 && (a.n_kv == 0 || a.n_kv % a.D == 0) && a.ld_in % 4 == 0 && a.ld_q % 4 == 0 && a.taps >= 1,
                 "conv_rows: %d rows of %d + 2 x %d channels, heads of %d, %d taps", a.n, a.n_q, a.n_kv, a.D, a.taps);
     if (a.rows) {                                                  // prompt: rows and q in the element type
-        if (dt == PGK_F32) PGK_CHECK_HIP((a.n > 512 ? conv_rows_launch<float, float, float, 2>(a, st) : conv_rows_launch<float, float, float, 1>(a, st)));
-        else PGK_CHECK_HIP((a.n > 512 ? conv_rows_launch<bf16, bf16, bf16, 2>(a, st) : conv_rows_launch<bf16, bf16, bf16, 1>(a, st)));
+        if (dt == PGK_F32) PGK_CHECK_HIP((conv_rows_launch<float, float, float, true>(a, st)));
+        else PGK_CHECK_HIP((conv_rows_launch<bf16, bf16, bf16, true>(a, st)));
         return PGK_OK;
     }
-    if (dt == PGK_F32) PGK_CHECK_HIP((conv_rows_launch<float, float, float, 1>(a, st)));
-    else if (in32) PGK_CHECK_HIP((q32 ? conv_rows_launch<bf16, float, float, 1>(a, st) : conv_rows_launch<bf16, float, bf16, 1>(a, st)));
-    else PGK_CHECK_HIP((q32 ? conv_rows_launch<bf16, bf16, float, 1>(a, st) : conv_rows_launch<bf16, bf16, bf16, 1>(a, st)));
+    if (dt == PGK_F32) PGK_CHECK_HIP((conv_rows_launch<float, float, float, false>(a, st)));
+    else if (in32) PGK_CHECK_HIP((q32 ? conv_rows_launch<bf16, float, float, false>(a, st) : conv_rows_launch<bf16, float, bf16, false>(a, st)));
+    else PGK_CHECK_HIP((q32 ? conv_rows_launch<bf16, bf16, float, false>(a, st) : conv_rows_launch<bf16, bf16, bf16, false>(a, st)));
     return PGK_OK;
 }
 

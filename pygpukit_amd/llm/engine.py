@@ -148,7 +148,8 @@ class Engine:
         ms = (C.c_float * len(self.KERNEL_CLASSES))()
         cnt = (C.c_int * len(self.KERNEL_CLASSES))()
         _hip.call("pgk_engine_profile_step", self.handle, batch, n_iters, ms, cnt, None)
-        return {name: ((ms[i] * 1e3 / cnt[i]) if cnt[i] else 0.0, cnt[i] // n_iters) for i, name in enumerate(self.KERNEL_CLASSES)}
+        return {name: ((ms[i] * 1e3 / cnt[i]) if cnt[i] else 0.0, cnt[i] // n_iters) for i, name in enumerate(self.KERNEL_CLASSES)
+                if cnt[i] or name != "recur"}      # (recur: layer-list models only)
 
     def timeline(self, batch: int = 1, warm: int = 2) -> list[dict]:
         """One graph-replayed step as a list of launches in order: kernel class, workgroups, and the first/last start and
@@ -378,7 +379,7 @@ class StackEngine(Engine):
             if lw["mixer"] == _hip.MIX_LATENT:
                 want.update(c_norm=((1, rp), float32, False), w_ukv=((2 * hd, rp), dt, False))
             elif lw["mixer"] == _hip.MIX_ATTENTION:
-                want.update(conv=((lw["taps"], hd + 2 * gd), float32, True), q_norm=((1, hd), float32, True), k_norm=((1, gd), float32, True),
+                want.update(conv=((lw["taps"], hd + 2 * gd), dt, True), q_norm=((1, hd), float32, True), k_norm=((1, gd), float32, True),
                             slopes=((1, lw["heads"]), float32, True))
             else:
                 want.update(lower=((1, hd), float32, False), o_norm=((1, lw["vhead_pad"]), float32, False))
@@ -463,7 +464,8 @@ class StackEngine(Engine):
             b[0, :rows] = channels(biases)
             b_in = from_numpy(b)
         if convs[0] is not None:
-            conv = from_numpy(np.ascontiguousarray(channels(convs)))
+            c = np.ascontiguousarray(channels(convs))          # (bfloat16 values: the upper halves are exact)
+            conv = from_numpy((c.view(np.uint32) >> 16).astype(np.uint16) if q.dtype == bfloat16 else c)
         vec = lambda a, n: None if a is None else from_numpy(_pad_heads(_host_f32(a).reshape(1, -1), n, hp))  # noqa: E731
         out.update(mixer=_hip.MIX_ATTENTION, heads=heads, kv_heads=kv_heads, dim=dim, vdim=vdim, window=window, scale=scale, head_pad=hp, vhead_pad=hp, n_att=heads * hp,
                    kv_from=-1 if kv_from is None else kv_from, taps=1 if conv is None else conv.shape[0], w_in=w_in, b_in=b_in, conv=conv, q_norm=vec(q_norm, heads),
