@@ -514,11 +514,13 @@ def test_deep_windows_in_batches(models, dtype, batch):
 
 
 @gpu
-@pytest.mark.parametrize("packed", ["0", "1"])
+@pytest.mark.parametrize("packed,big_tiles", [("0", "0"), ("1", "0"), ("1", "1")])
 @pytest.mark.parametrize("name", ["long", "tiles"])
-def test_projection_routes_agree(models, name, packed, monkeypatch):
-    """Fragment-major copies on and off: prompts of 2..300 rows and batches take other kernels, the logits stay the same."""
+def test_projection_routes_agree(models, name, packed, big_tiles, monkeypatch):
+    """Fragment-major copies on and off, 128- and 256-row tiles: prompts of 2..300 rows and batches take other kernels, the logits stay
+    the same."""
     monkeypatch.setenv("PGK_PACKED_PREFILL", packed)
+    monkeypatch.setenv("PGK_GEMM256", big_tiles)
     cfg, W, model = models(name, "bfloat16")
     t, want = reference(name, 400)
     e = model.build_engine(max_seq_len=310, max_batch=12)
