@@ -410,44 +410,69 @@ typedef struct {
 
 pgk_status pgk_engine_create(const pgk_model_config_t* cfg, const void* embed, const void* lm_head,
                              const void* final_norm, const pgk_layer_weights_t* layers, pgk_engine* out);
-/* Layer-list decoders (csrc/engine_stack.hip): fp32 residual stream, a norm after each sublayer and optionally before it, one of
- * several mixers per layer, dense SwiGLU / xIELU or no feed-forward; every layer has its own sizes.  dtype PGK_BF16 or PGK_F32 is the
+/* Layer-list decoders (csrc/engine_stack.hip): fp32 residual stream, one of several mixers per layer, SwiGLU / xIELU, a mixture of
+ * experts or no feed-forward; every layer has its own sizes.  A layer is a sandwich (mixer, then feed-forward, a norm after each and
+ * optionally before it) or parallel (one norm, mixer and feed-forward read its output, both results are added).  A run of layers may
+ * be passed several times with the same weights, each pass with caches of its own; a pass starts with
+ * x <- loop_in [x; embedding row] + loop_step[pass].  dtype PGK_BF16 or PGK_F32 is the
  * element type of the tables, matrices, taps, activations and caches; norm weights, biases and gates' constants are fp32 with any
  * offset applied.  Caller pads with zeros: Wp = width up to a multiple of 64; n_in, n_att and ff_pad multiples of 64 (ff_pad 0: the
  * layer has no feed-forward).
- * PGK_MIX_LATENT     latent attention over a sliding window with a per-head output gate.  head_pad >= dim and vdim: 64, 128 or a
- *                    larger multiple of 64; rank_pad a multiple of 64.  w_in rows: heads x head_pad queries | rank_pad latents |
- *                    heads gates.
+ * PGK_MIX_LATENT     latent attention over a sliding window, with a per-head output gate or (gated 0) without.  head_pad >= dim and
+ *                    vdim: 64, 128 or a larger multiple of 64; rank_pad a multiple of 64.  w_in rows: heads x head_pad queries |
+ *                    rank_pad latents | heads gates.  rot > 0: the last rot of the dim query columns and rot latent columns behind the
+ *                    first `rank` (which are not normed) are turned by position x rot_freq[i] in neighbouring pairs, and w_ukv's key rows pass
+ *                    them on.
  * PGK_MIX_ATTENTION  grouped heads over a K/V ring: q, k, v = taps over time of (w_in x + b_in), RMS norm over the whole q and k
  *                    rows, distance bias, elementwise output gate.  head_pad as above (at most 1024).  w_in rows: heads x head_pad q |
  *                    kv_heads x head_pad k | the same v | heads x head_pad gates; with kv_from >= 0 (that layer's keys and values)
  *                    q | gates.  conv [taps][q, k, v rows] or NULL, slopes [heads] or NULL.
  * PGK_MIX_HGRN2      gated linear recurrence (pgk_gated_recurrence).  head_pad, vhead_pad: dim, vdim up to multiples of 16.  w_in
- *                    rows: heads x head_pad q | the same f | heads x vhead_pad v. */
-typedef enum { PGK_MIX_LATENT = 0, PGK_MIX_ATTENTION = 1, PGK_MIX_HGRN2 = 2 } pgk_mixer;
-typedef enum { PGK_FF_SWIGLU = 0, PGK_FF_XIELU = 1 } pgk_ff;
+ *                    rows: heads x head_pad q | the same f | heads x vhead_pad v.
+ * PGK_MIX_DELTA      gated delta rule with a decay per key channel (pgk_delta_rule) after taps over time and SiLU on q, k, v.  head_pad,
+ *                    vhead_pad: up to multiples of 16 (32, 64 or 128 for head_pad: the chunked prompt form); rank_a, rank_g: ranks of
+ *                    decay and gate up to multiples of 64.  w_in rows: kv_heads x head_pad q | the same k | heads x vhead_pad v |
+ *                    heads strengths, up to a multiple of 64 | rank_a | rank_g.  decay [heads], dt_bias [heads x head_pad].
+ * PGK_MIX_SSD        state-space duality (pgk_state_space) after taps with bias and SiLU on x, B, C; the result times silu(z) and normed in
+ *                    norm_parts equal parts of its heads x vdim elements.  dim: the state's; kv_heads: the groups.  w_in rows: heads x vhead_pad
+ *                    x | kv_heads x head_pad B | the same C | heads x vhead_pad z | heads dt.  decay, dt_bias, skip [heads].
+ * PGK_FF_MOE         experts of ff_pad, `top` of them per token (see pgk_moe); behind w_in's n_in rows stand the router's, up to a
+ *                    multiple of 64.  Parallel layers only; SANDWICH layers take the dense forms. */
+typedef enum { PGK_MIX_LATENT = 0, PGK_MIX_ATTENTION = 1, PGK_MIX_HGRN2 = 2, PGK_MIX_DELTA = 3, PGK_MIX_SSD = 4 } pgk_mixer;
+typedef enum { PGK_FF_SWIGLU = 0, PGK_FF_XIELU = 1, PGK_FF_MOE = 2 } pgk_ff;
+typedef enum { PGK_BLOCK_SANDWICH = 0, PGK_BLOCK_PARALLEL = 1 } pgk_block;
 typedef struct {
     int vocab_size, width, num_layers, max_positions, max_seq_len, max_batch;
     float norm_eps, residual_mult;
     pgk_dtype dtype;
+    int block, layer_norm;                         /* pgk_block; parallel layers: norms subtract the mean */
+    int loop_start, loop_stop, loop_times;         /* layers loop_start .. loop_stop - 1 run loop_times times (0: no loop) */
+    const void* loop_in;                           /* [Wp, 2 Wp] */
+    const float* loop_step;                        /* [loop_times, Wp] */
 } pgk_stack_config_t;
 typedef struct {
     int mixer, ff;                                 /* pgk_mixer, pgk_ff */
     int heads, kv_heads, dim, vdim, rank;          /* true sizes */
     int window, taps, kv_from;                     /* window: keys a query sees, itself included; kv_from: -1 or an earlier layer */
     int head_pad, vhead_pad, rank_pad, n_in, n_att, ff_pad;
-    float scale, act_pos, act_neg;                 /* act_*: pgk_xielu's a and b */
+    int gated, rot, norm_parts, rank_a, rank_g;
+    int experts, top, groups, keep;                /* PGK_FF_MOE; groups 0: none */
+    float scale, act_pos, act_neg, router_scale;   /* act_*: pgk_xielu's a and b */
     const float *norm1, *norm1b, *norm2, *norm2b;  /* [Wp]; norm1 / norm2 NULL: the sublayer reads the stream itself */
     const void* w_in;                              /* [n_in, Wp] */
     const float* b_in;                             /* [n_in] or NULL */
     const void* conv;                              /* attention */
     const float *q_norm, *k_norm, *slopes;
-    const float *lower, *o_norm;                   /* hgrn2: [heads * head_pad], [vhead_pad] */
+    const float *lower, *o_norm;                   /* hgrn2: [heads * head_pad]; hgrn2, delta: [vhead_pad], ssd: [heads * vhead_pad] */
     const float* c_norm;                           /* latent: [rank_pad] */
     const void* w_ukv;                             /* latent: [2 heads head_pad, rank_pad]: key rows, then value rows */
     const void* w_o;                               /* [Wp, n_att] */
-    const void* w_gate_up;                         /* [2 ff_pad, Wp]; xIELU: [ff_pad, Wp] */
-    const void* w_down;                            /* [Wp, ff_pad] */
+    const void* w_gate_up;                         /* [2 ff_pad, Wp]; xIELU: [ff_pad, Wp]; MoE: [experts, 2 ff_pad, Wp] */
+    const void* w_down;                            /* [Wp, ff_pad]; MoE: [experts, Wp, ff_pad] */
+    const float* rot_freq;                         /* latent: [rot / 2] */
+    const float *decay, *dt_bias, *skip, *conv_bias;
+    const void *w_a2, *w_g2;                       /* delta: [heads head_pad, rank_a], [heads vhead_pad, rank_g] */
+    const float* correction;                       /* MoE: [experts] */
 } pgk_stack_layer_t;
 /* embed [vocab, width], pos_embed [max_positions, width] or NULL, head [vocab, Wp], final_norm [Wp] */
 pgk_status pgk_engine_create_stack(const pgk_stack_config_t* cfg, const void* embed, const void* pos_embed, const void* head,

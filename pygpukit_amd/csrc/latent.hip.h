@@ -37,6 +37,13 @@ struct RowsNormArgs {
     int store_h;
     int nslabs;               // > 0: y is fp32 split-K slabs, slab i at y + i * slab_stride (elements); the sublayer output is their sum
     long long slab_stride;
+    // plain: the sublayer output is added as it is, h = (base or h) + mult * (y + sum of e_top rows of e); y and e may be null
+    int plain, layer_norm;    // layer_norm: gamma's norm subtracts the mean
+    const float* base;        // [ld] or null
+    const void* e;            // [*][e_top][ld], element type
+    int e_top;
+    const void* embed;        // given: no norm, out rows (2 ld wide) are [h | embed[tok[row]]] (table rows of W)
+    const int32_t* tok;
 };
 pgk_status rows_norm(const RowsNormArgs& a, int n, pgk_dtype dt, hipStream_t st);
 

@@ -1,6 +1,6 @@
 // Sequence mixers of the layer-list engine beside latent attention (engine_stack.hip): short causal convolutions with norms over whole
-// projections, attention over a K/V ring with distance bias and elementwise gate (ops_gated_attn.hip), and a gated linear recurrence
-// whose forget gate also decides what is written (ops_recurrence.hip).
+// projections, attention over a K/V ring with distance bias and elementwise gate (ops_gated_attn.hip), linear recurrences whose decay
+// also decides what is written or stands beside it (ops_recurrence.hip), and the gated delta rule with a decay per channel (ops_delta.hip).
 #pragma once
 
 #include "engine_common.hip.h"
@@ -73,13 +73,58 @@ bool kv_attn_q32(int D, pgk_dtype dt);
 int kv_attn_splits(int B, int H, int G, int keys, int cus);
 pgk_status kv_attn_decode(const KvAttnArgs& a, pgk_dtype dt, bool io32, hipStream_t st, int* launches);
 
-// ---- gated linear recurrence ----
-//   q = silu(z_q),  f = lower + (1 - lower) sigmoid(z_f + bias),  S <- diag(f) S + (1 - f) v^T,  o = S^T q;  norm given: o / rms(o) * norm
-// Rows of `in`: z_q at q_off + head * dim, z_f at f_off + head * dim, v at v_off + head * vdim.
+// ---- taps over time and SiLU ----
+// y_t = silu(bias + sum_j w_j u_(t - taps + 1 + j)) per channel, zero before a sequence's start.  Ring [slot][taps][channels] of u: position p
+// in row p % taps (`taps` rows, so that writing a position touches no row the same step reads).
+struct ConvSiluArgs {
+    const void* in; int ld_in;            // the first channel of every row
+    const void* conv; const float* bias;  // [taps][channels] (element type), [channels] or null
+    int taps, channels, n;                // channels: a multiple of 4
+    const void* ring; const RowSrc* rows;
+    void* out; int ld_out;
+};
+pgk_status conv_silu_rows(const ConvSiluArgs& a, pgk_dtype dt, hipStream_t st);
+
+// One channel of the next token in a decode step (a kernel that needs a few channels per workgroup convolves them itself); `write`: the new
+// row goes to the ring, once per channel.
+struct ConvStep { const void* conv; const float* bias; int taps, channels; void* ring; };
+template <bool EXACT> __device__ __forceinline__ float silu_f(float z) { return z / (1.0f + (EXACT ? expf(-z) : __expf(-z))); }
+template <class T, class IT, bool EXACT>
+__device__ __forceinline__ float conv_step(const ConvStep& cs, const IT* in, int c, int slot, int pos, bool write) {
+    const T* w = reinterpret_cast<const T*>(cs.conv);
+    T* ring = reinterpret_cast<T*>(cs.ring) + (size_t)slot * cs.taps * cs.channels + c;
+    const float u = to_f(in[c]);
+    float y = fmaf(to_f(w[(size_t)(cs.taps - 1) * cs.channels + c]), u, cs.bias ? cs.bias[c] : 0.f);
+    float x[3], g[3];
+#pragma unroll
+    for (int k = 0; k < 3; ++k) {                                  // three taps back in flight, masked
+        const int b = min(k + 1, cs.taps - 1), p = max(pos - b, 0);
+        x[k] = to_f(ring[(size_t)(p % cs.taps) * cs.channels]);
+        g[k] = k + 1 < cs.taps && pos - b >= 0 ? to_f(w[(size_t)(cs.taps - 1 - b) * cs.channels + c]) : 0.f;
+    }
+#pragma unroll
+    for (int k = 0; k < 3; ++k) y = g[k] != 0.f ? fmaf(g[k], x[k], y) : y;      // (an unread ring row may hold anything)
+    for (int b = 4; b < cs.taps && pos - b >= 0; ++b) y = fmaf(to_f(w[(size_t)(cs.taps - 1 - b) * cs.channels + c]), to_f(ring[(size_t)((pos - b) % cs.taps) * cs.channels]), y);
+    if (write) ring[(size_t)(pos % cs.taps) * cs.channels] = from_f<T>(u);
+    return silu_f<EXACT>(y);
+}
+
+// ---- linear recurrences S <- diag(f) S + k v^T, o = S^T q ----
+// RECUR_HGRN2: q = silu(z_q),  f = lower + (1 - lower) sigmoid(z_f + bias),  k = 1 - f;  norm given: o / rms(o) * norm.
+//   Rows of `in`: z_q at q_off + head * dim, z_f at f_off + head * dim, v at v_off + head * vdim.
+// RECUR_SSD: t = softplus(dt + dt_bias), f = exp(-decay t) for every channel, k = t B, q = C, v = x;  (o + skip v) silu(z).
+//   x at v_off + head * vdim, B at f_off + group * dim, C at q_off + group * dim: channels of `rows` (prompts: after taps and SiLU) or of `in`
+//   (decode: before them, `conv`); z at z_off + head * vdim, dt at dt_off + head of `in`.  Group of a head: head / (H / G).
+enum { RECUR_HGRN2 = 0, RECUR_SSD = 1 };
 struct RecurArgs {
+    int kind;
     const void* in; int ld_in, q_off, f_off, v_off;
     const float *bias, *lower;            // [H * dim]; bias may be null
     const float* norm;                    // [vdim] or null
+    const void* rows; int ld_rows;
+    int G, z_off, dt_off;
+    const float *dt_bias, *decay, *skip;  // [H]
+    ConvStep conv;
     int H, dim, vdim, vdim_true, n;       // n: rows (decode: sequences)
     float eps;
     float* state;                         // [slots][H][dim][vdim] fp32
@@ -94,5 +139,38 @@ constexpr int RECUR_CHUNKED_FROM = 16;                                          
 int recur_chunk_rows(int dim, int vdim);                                                        // rows per chunk; 0: sizes the chunked form does not take
 // the chunked form: chunks in order, sequence by sequence (chunk_of_seq[i] .. chunk_of_seq[i + 1] are sequence i's)
 pgk_status recur_chunked(const RecurArgs& a, const RecurChunk* chunks, int n_chunks, const int32_t* chunk_of_seq, void* ws, pgk_dtype dt, hipStream_t st);
+
+// x / rms(x) * norm in `parts` equal parts of each row's heads x vdim_true elements (heads vdim apart), in place
+pgk_status parts_norm(void* x, int ld, int n, int heads, int vdim, int vdim_true, int parts, const float* norm, float eps, pgk_dtype dt, hipStream_t st);
+
+// ---- gated delta rule with a decay per key channel ----
+//   q, k of unit length (q times dim_true^-1/2),  b = sigmoid(beta),  g = exp(-decay softplus(z + dt_bias));
+//   S <- diag(g) S,  u = b (v - S^T k),  S <- S + k u^T,  o = S^T q;  o / rms(o) * norm * sigmoid(gate)
+// Channels q (G x dim) | k (G x dim) | v (H x vdim) of `rows` (prompts: after taps and SiLU) or of `in` (decode: before them).
+struct DeltaArgs {
+    const void* in; int ld_in, b_off;     // beta of head h at b_off + h
+    const void* rows; int ld_rows;
+    const float* z; int ld_z;             // [n][H * dim]
+    const void* gate; int ld_gate;        // [n][H * vdim], typed as the projection rows
+    ConvStep conv;
+    const float *decay, *dt_bias, *norm;  // [H], [H * dim], [vdim]
+    int H, G, dim, vdim, dim_true, vdim_true, n;
+    float eps;
+    float* state;                         // [slots][H][dim][vdim] fp32
+    const SeqSpan* seqs; int n_seqs;      // null: row b is the next token of slot b at positions[b]
+    const int32_t* positions;
+    void* out; int ld_out;                // head h at h * vdim; columns H * vdim .. ld_out are zeroed
+};
+pgk_status delta_rows(const DeltaArgs& a, pgk_dtype dt, bool io32, hipStream_t st);
+constexpr int DELTA_CHUNK = 64;                                                                 // rows per chunk of the chunked form
+bool delta_chunk_ok(int dim, int vdim);
+size_t delta_chunk_bytes(const DeltaArgs& a, int n_chunks);
+pgk_status delta_chunked(const DeltaArgs& a, const RecurChunk* chunks, int n_chunks, const int32_t* chunk_of_seq, void* ws, pgk_dtype dt, hipStream_t st);
+
+// z = A x_a (fp32 [n][na]) and g = G x_g (IT [n][ng]) for a few rows: x_a, x_g are columns of the projection rows, ka and kg of them
+pgk_status lowrank_rows(const void* in, int ld_in, int n, int a_off, int ka, const void* wa, float* z, int na, int g_off, int kg, const void* wg, void* g, int ng,
+                        pgk_dtype dt, bool io32, hipStream_t st);
+// columns off .. off + cols of rows -> dense rows
+pgk_status rows_slice(const void* in, int ld_in, int off, int cols, void* out, int n, pgk_dtype dt, hipStream_t st);
 
 }  // namespace pgk

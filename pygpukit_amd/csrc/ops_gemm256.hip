@@ -18,6 +18,7 @@
 
 #include "gemm_epilogues.hip.h"
 #include "gemv_core.hip.h"
+#include "moe.hip.h"
 #include "pgk_internal.h"
 
 namespace pgk {
@@ -467,22 +468,39 @@ __global__ __launch_bounds__(G2_THREADS) void gemm256s_bf16_kernel(const bf16* A
 // back as rows - 32 lanes x 16 B = one 512-byte row segment per instruction - for coalesced stores (EPI 1: float4
 // read-modify-write of the residual stream, all loads issued before the first store).
 constexpr int G1_THREADS = 256, G1_HALF = 128 * 64;
-template <int EPI>   // 0: bf16 C store (+bias); 1: fp32 C +=; 2: fp32 split-K slab; 3: QKV heads (QkvHeadArgs: tile column = head slot);
-                     // 4: SwiGLU (W = fused gate / up rows, N = I act columns, C = bf16 act [M][I]; tile tn = act columns [64 tn, +64)); 5: xIELU, bf16 store
-__global__ __launch_bounds__(G1_THREADS, 2) void gemm128s_bf16_kernel(const bf16* A, const bf16* W, const bf16* bias, void* Cv,
-                                                                       int M, int N, int K, int ntm, int ntn, int kps, QkvHeadArgs hd, int packed, XieluArgs xa = XieluArgs{}) {
+// EPI 0: bf16 C store (+bias); 1: fp32 C +=; 2: fp32 split-K slab; 3: QKV heads (QkvHeadArgs: tile column = head slot);
+// 4: SwiGLU (W = fused gate / up rows, N = I act columns, C = bf16 act [M][I]; tile tn = act columns [64 tn, +64)); 5: xIELU, bf16 store
+// GRP: rows sorted by expert (GroupArgs), every tile with its expert's weight; EPI 4, or 6: bf16 rows times their weight, each at its place
+template <int EPI, bool GRP>
+__device__ __forceinline__ void gemm128s_body(const bf16* A, const bf16* W, const bf16* bias, void* Cv,
+                                              int M, int N, int K, int ntm, int ntn, int kps, const QkvHeadArgs& hd, int packed, const XieluArgs& xa, const GroupArgs& ga) {
     extern __shared__ __attribute__((aligned(16))) char g2_smem[];   // 4 stages x (A 8 KiB | W 8 KiB)
     const int tid = threadIdx.x, lane = tid & 63, wid = tid >> 6;
     const int wr = wid >> 1, wc = wid & 1, q = lane >> 4, l15 = lane & 15;
-    int tm, tn;
+    int tm, tn, m0;
+    if constexpr (GRP) {
+        ntm = *ga.n_tiles;
+        if ((int)blockIdx.x >= ntm * ntn) return;            // (the grid is sized for the worst distribution)
+    }
     g2_tile_of(blockIdx.x, ntm * ntn, ntm, ntn, tm, tn);
-    const int m0 = tm * 128, n0 = tn * 128;
+    if constexpr (GRP) {
+        const MoeTile t = ga.tiles[tm];
+        m0 = t.row0;
+        M = t.row0 + t.rows;
+        W += t.expert * ga.w_stride;
+    } else m0 = tm * 128;
+    const int n0 = tn * 128;
     const int kbeg = (int)blockIdx.y * kps, kend = min(K, kbeg + kps);
 
     const int drow = wid * 32 + (lane >> 2);                 // one DMA instruction = 16 rows x 64 B
     const int dchunk = (lane & 3) ^ ((lane >> 4) & 2);
-    const bf16* a_src0 = A + (size_t)min(m0 + drow, M - 1) * K + kbeg + dchunk * 8;
-    const bf16* a_src1 = A + (size_t)min(m0 + drow + 16, M - 1) * K + kbeg + dchunk * 8;
+    auto a_row = [&](int r) -> int {
+        r = min(r, M - 1);
+        if constexpr (GRP) return ga.div > 0 ? ga.order[r] / ga.div : r;
+        else return r;
+    };
+    const bf16* a_src0 = A + (size_t)a_row(m0 + drow) * K + kbeg + dchunk * 8;
+    const bf16* a_src1 = A + (size_t)a_row(m0 + drow + 16) * K + kbeg + dchunk * 8;
     // EPI 4: B-tile rows 0-63 = gate rows 64 tn .., rows 64-127 = the matching up rows N + 64 tn .. (N = I); a wave's 32 rows stay in one half
     const int wrow = (EPI == 4) ? (drow < 64 ? tn * 64 + drow : N + tn * 64 + drow - 64) : n0 + drow;
     const int wlast = (EPI == 4) ? 2 * N - 1 : N - 1;
@@ -601,6 +619,21 @@ __global__ __launch_bounds__(G1_THREADS, 2) void gemm128s_bf16_kernel(const bf16
             raw.to_float(x);
             qkv_head_finish(x, c, tn, m0 + row, M, hd, reinterpret_cast<bf16*>(Cv), N);
         }
+    } else if constexpr (EPI == 6) {
+#pragma unroll
+        for (int it = 0; it < 8; ++it) {
+            const int item = it * G1_THREADS + tid, row = item >> 4, c = item & 15, sw = ((row >> 2) & 3) << 6;
+            const float4 v0 = *reinterpret_cast<const float4*>(g2_smem + row * 512 + ((c * 32) ^ sw));
+            const float4 v1 = *reinterpret_cast<const float4*>(g2_smem + row * 512 + ((c * 32 + 16) ^ sw));
+            const int grow = m0 + row, gcol = n0 + c * 8;
+            if (grow >= M || gcol >= N) continue;
+            const int place = ga.order[grow];
+            const float w = ga.wts[place];
+            const float f[8] = {v0.x * w, v0.y * w, v0.z * w, v0.w * w, v1.x * w, v1.y * w, v1.z * w, v1.w * w};
+            Vec<bf16> o;
+            o.from_float(f);
+            o.store(reinterpret_cast<bf16*>(Cv) + (size_t)place * N + gcol);
+        }
     } else if constexpr (EPI == 0 || EPI == 5) {
         // 8 columns per lane: two float4 -> 16 bytes of bf16
 #pragma unroll
@@ -644,6 +677,15 @@ __global__ __launch_bounds__(G1_THREADS, 2) void gemm128s_bf16_kernel(const bf16
             *reinterpret_cast<float4*>(C + (size_t)grow * N + gcol) = v;
         }
     }
+}
+template <int EPI>
+__global__ __launch_bounds__(G1_THREADS, 2) void gemm128s_bf16_kernel(const bf16* A, const bf16* W, const bf16* bias, void* Cv,
+                                                                       int M, int N, int K, int ntm, int ntn, int kps, QkvHeadArgs hd, int packed, XieluArgs xa = XieluArgs{}) {
+    gemm128s_body<EPI, false>(A, W, bias, Cv, M, N, K, ntm, ntn, kps, hd, packed, xa, GroupArgs{});
+}
+template <int EPI>
+__global__ __launch_bounds__(G1_THREADS, 2) void gemm128s_grouped_kernel(const bf16* A, const bf16* W, bf16* C, int N, int K, int ntn, GroupArgs ga) {
+    gemm128s_body<EPI, true>(A, W, nullptr, C, 0, N, K, 0, ntn, K, QkvHeadArgs{}, 0, XieluArgs{}, ga);
 }
 
 // ---- fp8 x fp8 with 128-wide block scales on the same structure --------------------------------------------
@@ -1040,6 +1082,22 @@ pgk_status gemm128s_bf16_nt(const bf16* A, const bf16* W, const bf16* bias, void
     else if (mode == 2) gemm128s_bf16_kernel<2><<<grid, G1_THREADS, LDS, st>>>(A, W, nullptr, C, M, N, K, ntm, ntn, kps, hd, pk, XieluArgs{});
     else if (mode == 3) gemm128s_bf16_kernel<3><<<grid, G1_THREADS, LDS, st>>>(A, W, nullptr, C, M, N, K, ntm, ntn, kps, hd, pk, XieluArgs{});
     else gemm128s_bf16_kernel<4><<<grid, G1_THREADS, LDS, st>>>(A, W, nullptr, C, M, N, K, ntm, ntn, kps, hd, pk, XieluArgs{});
+    PGK_CHECK_HIP(hipGetLastError());
+    return PGK_OK;
+}
+
+pgk_status gemm128s_grouped(const bf16* A, const bf16* W, bf16* C, bool down, const GroupArgs& g, int max_tiles, int rows, int N, int K, hipStream_t st) {
+    PGK_REQUIRE(K % 64 == 0 && N % 64 == 0 && max_tiles >= 1 && g.tiles && g.n_tiles && g.order && g.wts, "gemm128s_grouped: N=%d K=%d", N, K);
+    constexpr size_t LDS = 8 * (size_t)G1_HALF;
+    static bool attr_done = false;
+    if (!attr_done) {
+        PGK_CHECK_HIP(hipFuncSetAttribute(reinterpret_cast<const void*>(&gemm128s_grouped_kernel<4>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)LDS));
+        PGK_CHECK_HIP(hipFuncSetAttribute(reinterpret_cast<const void*>(&gemm128s_grouped_kernel<6>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)LDS));
+        attr_done = true;
+    }
+    const int ntn = down ? ceil_div(N, 128) : N / 64;
+    if (down) gemm128s_grouped_kernel<6><<<max_tiles * ntn, G1_THREADS, LDS, st>>>(A, W, C, N, K, ntn, g);
+    else gemm128s_grouped_kernel<4><<<max_tiles * ntn, G1_THREADS, LDS, st>>>(A, W, C, N, K, ntn, g);
     PGK_CHECK_HIP(hipGetLastError());
     return PGK_OK;
 }

@@ -91,6 +91,79 @@ __global__ __launch_bounds__(256) void rows_norm_kernel(RowsNormArgs a) {
     }
 }
 
+// The plain form: y (or its slabs) and the experts' rows are added, then layer norm or RMS norm, or the row beside its embedding
+template <class T, class YT, int NT>
+__global__ __launch_bounds__(256) void rows_add_kernel(RowsNormArgs a) {
+    __shared__ float red[16];
+    const int row = a.rows ? a.rows[blockIdx.x] : blockIdx.x, nt = a.ld;
+    float* hr = a.h + (size_t)row * a.ld;
+    const float* from = a.base ? a.base : hr;
+    const YT* yr = reinterpret_cast<const YT*>(a.y) + (size_t)row * a.ldy;
+    const T* er = reinterpret_cast<const T*>(a.e) + (size_t)row * a.e_top * a.ld;
+    float4 v[NT];
+    float s1 = 0.f;
+#pragma unroll
+    for (int t = 0; t < NT; ++t) {
+        const int i = min((int)(threadIdx.x + 256 * t) * 4, nt - 4);
+        float4 x = *reinterpret_cast<const float4*>(from + i), y = {0.f, 0.f, 0.f, 0.f};
+        auto add = [&](const float4& q) { y.x += q.x; y.y += q.y; y.z += q.z; y.w += q.w; };
+        if (a.y) add(load4<YT>(yr + i));
+#pragma unroll 4
+        for (int s = 1; s < a.nslabs; ++s) add(load4<YT>(yr + s * a.slab_stride + i));
+        if (a.e) {
+#pragma unroll 4
+            for (int k = 0; k < a.e_top; ++k) add(load4<T>(er + (size_t)k * a.ld + i));
+        }
+        x.x = fmaf(a.mult, y.x, x.x); x.y = fmaf(a.mult, y.y, x.y); x.z = fmaf(a.mult, y.z, x.z); x.w = fmaf(a.mult, y.w, x.w);
+        const bool in = (int)(threadIdx.x + 256 * t) * 4 < nt;
+        if (in && a.store_h) *reinterpret_cast<float4*>(hr + i) = x;
+        v[t] = in ? x : make_float4(0.f, 0.f, 0.f, 0.f);
+        s1 += v[t].x + v[t].y + v[t].z + v[t].w;                   // (columns W .. ld are zero)
+    }
+    if (!a.out) return;
+    if (a.embed) {
+        const T* er0 = reinterpret_cast<const T*>(a.embed) + (size_t)a.tok[row] * a.W;
+        T* o = reinterpret_cast<T*>(a.out) + (size_t)blockIdx.x * 2 * a.ld;
+#pragma unroll
+        for (int t = 0; t < NT; ++t) {
+            const int i = (threadIdx.x + 256 * t) * 4;
+            if (i < nt) store4<T>(o + i, v[t]);
+        }
+        for (int i = threadIdx.x; i < nt; i += 256) o[nt + i] = i < a.W ? er0[i] : from_f<T>(0.f);
+        return;
+    }
+    const float mean = a.layer_norm ? block_sum(s1, red) / a.W : 0.f;
+    float ss = 0.f;
+#pragma unroll
+    for (int t = 0; t < NT; ++t) {
+        const int i = (threadIdx.x + 256 * t) * 4;
+        v[t].x -= mean; v[t].y -= mean; v[t].z -= mean; v[t].w -= mean;
+        ss += (i < a.W ? v[t].x * v[t].x : 0.f) + (i + 1 < a.W ? v[t].y * v[t].y : 0.f) + (i + 2 < a.W ? v[t].z * v[t].z : 0.f) + (i + 3 < a.W ? v[t].w * v[t].w : 0.f);
+    }
+    const float inv = 1.0f / sqrtf(block_sum(ss, red) / a.W + a.eps);
+    T* o = reinterpret_cast<T*>(a.out) + (size_t)blockIdx.x * a.ld;
+#pragma unroll
+    for (int t = 0; t < NT; ++t) {
+        const int i = (threadIdx.x + 256 * t) * 4;
+        if (i < nt) {
+            const float4 g = *reinterpret_cast<const float4*>(a.gamma + i);      // zero in columns W .. ld
+            store4<T>(o + i, make_float4(v[t].x * inv * g.x, v[t].y * inv * g.y, v[t].z * inv * g.z, v[t].w * inv * g.w));
+        }
+    }
+}
+
+template <class T, class YT>
+static pgk_status rows_add_t(const RowsNormArgs& a, int n, hipStream_t st) {
+    PGK_REQUIRE(a.ld % 4 == 0 && a.W <= a.ld && (!a.out || a.embed || a.gamma) && !(a.e && a.e_top < 1), "rows_norm: row stride %d / width %d", a.ld, a.W);
+    if (a.ld <= 1024) rows_add_kernel<T, YT, 1><<<n, 256, 0, st>>>(a);
+    else if (a.ld <= 2048) rows_add_kernel<T, YT, 2><<<n, 256, 0, st>>>(a);
+    else if (a.ld <= 4096) rows_add_kernel<T, YT, 4><<<n, 256, 0, st>>>(a);
+    else if (a.ld <= 16384) rows_add_kernel<T, YT, 16><<<n, 256, 0, st>>>(a);
+    else return set_error(PGK_ERR_UNSUPPORTED, "rows_norm: width %d beyond 16384", a.W);
+    PGK_LAUNCH_CHECK();
+    return PGK_OK;
+}
+
 template <class T, class YT>
 static pgk_status rows_norm_t(const RowsNormArgs& a, int n, hipStream_t st) {
     PGK_REQUIRE(a.ld % 4 == 0 && a.W <= a.ld, "rows_norm: row stride %d / width %d", a.ld, a.W);
@@ -104,6 +177,10 @@ static pgk_status rows_norm_t(const RowsNormArgs& a, int n, hipStream_t st) {
 }
 
 pgk_status rows_norm(const RowsNormArgs& a, int n, pgk_dtype dt, hipStream_t st) {
+    if (a.plain) {
+        if (dt == PGK_BF16) return a.nslabs > 0 ? rows_add_t<bf16, float>(a, n, st) : rows_add_t<bf16, bf16>(a, n, st);
+        if (dt == PGK_F32) return rows_add_t<float, float>(a, n, st);
+    }
     if (dt == PGK_BF16) return a.nslabs > 0 ? rows_norm_t<bf16, float>(a, n, st) : rows_norm_t<bf16, bf16>(a, n, st);
     if (dt == PGK_F32) return rows_norm_t<float, float>(a, n, st);
     return set_error(PGK_ERR_UNSUPPORTED, "rows_norm: dtype %d", (int)dt);

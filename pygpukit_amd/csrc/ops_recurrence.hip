@@ -1,5 +1,5 @@
-// Gated linear recurrence (mixers.hip.h): per head a state S [dim][vdim] in fp32, S <- diag(f) S + (1 - f) v^T, o = S^T q.
-// Gates, state and the head norm are fp32 whatever the element type.
+// Linear recurrences (mixers.hip.h): per head a state S [dim][vdim] in fp32, S <- diag(f) S + k v^T, o = S^T q.
+// Gates, decays, state and norms are fp32 whatever the element type.  SRC: where f, k, q, v come from (RECUR_HGRN2, RECUR_SSD).
 //
 // Two forms.  Token by token (decode, short portions): one workgroup per sequence and head walks its rows.  Chunked (prompts): rows in
 // chunks of C, all chunks at once -
@@ -29,10 +29,17 @@ template <bool EXACT> __device__ __forceinline__ void rc_gate(float z, float low
     k = (1.0f - lower) * (z >= 0.f ? small : big);
 }
 
+// step size and decay of a state-space row (both forms: a scalar per head and row)
+__device__ __forceinline__ void ssd_step(float dt, float bias, float decay, float& step, float& fade) {
+    const float z = dt + bias;
+    step = z > 20.f ? z : log1pf(expf(z));
+    fade = expf(-decay * step);
+}
+
 // -------------------------------------------------------------------------------------------- token by token
 // One workgroup per (sequence, head).  A thread owns VEC columns of every NG-th state row (VEC = 4: one 16-byte access each); a
 // sequence that starts (position 0) begins with a zero state without reading the slot.
-template <class IT, bool EXACT, int VEC>
+template <class T, class IT, bool EXACT, int VEC, int SRC>
 __global__ __launch_bounds__(512) void recur_scan_kernel(unsigned long long* tl, RecurArgs a) {
     const TLStamp tls(tl);
     extern __shared__ float sm[];
@@ -47,12 +54,25 @@ __global__ __launch_bounds__(512) void recur_scan_kernel(unsigned long long* tl,
     for (int t = 0; t < s.len; ++t) {
         const IT* in = reinterpret_cast<const IT*>(a.in) + (size_t)(s.row0 + t) * a.ld_in;
         const bool fresh = s.start + t == 0;
+        if constexpr (SRC == RECUR_SSD) {
+            const int rep = a.H / a.G, grp = h / rep, pos = s.start + t;
+            float step, fade;
+            ssd_step(to_f(in[a.dt_off + h]), a.dt_bias[h], a.decay[h], step, fade);
+            const T* row = reinterpret_cast<const T*>(a.rows) + (size_t)(s.row0 + t) * a.ld_rows;
+            auto channel = [&](int c, bool own) { return a.seqs ? to_f(row[c]) : conv_step<T, IT, EXACT>(a.conv, in, c, s.slot, pos, own); };
+            for (int i = tid; i < 2 * dim + vdim; i += NT) {
+                if (i < dim) q[i] = channel(a.q_off + grp * dim + i, h % rep == 0);
+                else if (i < 2 * dim) { k[i - dim] = step * channel(a.f_off + grp * dim + i - dim, h % rep == 0); f[i - dim] = fade; }
+                else v[i - 2 * dim] = channel(a.v_off + h * vdim + i - 2 * dim, true);
+            }
+        } else {
         for (int d = tid; d < dim; d += NT) {
             const float zq = to_f(in[a.q_off + h * dim + d]), zf = to_f(in[a.f_off + h * dim + d]) + (a.bias ? a.bias[h * dim + d] : 0.f);
             q[d] = rc_silu<EXACT>(zq);
             rc_gate<EXACT>(zf, a.lower[h * dim + d], f[d], k[d]);
         }
         for (int i = tid; i < vdim; i += NT) v[i] = to_f(in[a.v_off + h * vdim + i]);
+        }
         __syncthreads();
         if (g < NG) {
             for (int cc = c; cc < NC; cc += NT) {                  // (one trip unless a head has more columns than the workgroup threads)
@@ -95,6 +115,7 @@ __global__ __launch_bounds__(512) void recur_scan_kernel(unsigned long long* tl,
         for (int i = tid; i < vdim; i += NT) {
             float o = 0.f;
             for (int j = 0; j < NG; ++j) o += po[j * vdim + i];
+            if constexpr (SRC == RECUR_SSD) o = fmaf(a.skip[h], v[i], o) * silu_f<EXACT>(to_f(in[a.z_off + h * vdim + i]));
             v[i] = o;                                              // the column's own thread: read again below
             ss = fmaf(o, o, ss);
         }
@@ -109,22 +130,27 @@ __global__ __launch_bounds__(512) void recur_scan_kernel(unsigned long long* tl,
     tls.end();
 }
 
-template <class IT, bool EXACT>
+template <class T, class IT, bool EXACT, int SRC>
 static pgk_status recur_scan(const RecurArgs& a, hipStream_t st) {
     const int B = a.seqs ? a.n_seqs : a.n, threads = a.dim * a.vdim >= 8192 ? 512 : 256;
     const bool vec = a.vdim % 4 == 0;
     const int cols = vec ? a.vdim / 4 : a.vdim, groups = threads / cols > 0 ? threads / cols : 1;
     const size_t lds = (size_t)(3 * a.dim + a.vdim + groups * a.vdim) * 4;
     PGK_REQUIRE(lds <= 64 * 1024, "recurrence: head widths %d / %d do not fit LDS", a.dim, a.vdim);
-    if (vec) PGK_CHECK_HIP(launch_k(&recur_scan_kernel<IT, EXACT, 4>, dim3(a.H, B), dim3(threads), lds, st, a));
-    else PGK_CHECK_HIP(launch_k(&recur_scan_kernel<IT, EXACT, 1>, dim3(a.H, B), dim3(threads), lds, st, a));
+    if (vec) PGK_CHECK_HIP(launch_k(&recur_scan_kernel<T, IT, EXACT, 4, SRC>, dim3(a.H, B), dim3(threads), lds, st, a));
+    else PGK_CHECK_HIP(launch_k(&recur_scan_kernel<T, IT, EXACT, 1, SRC>, dim3(a.H, B), dim3(threads), lds, st, a));
     return PGK_OK;
 }
 
 pgk_status recur_rows(const RecurArgs& a, pgk_dtype dt, bool io32, hipStream_t st) {
     PGK_REQUIRE(a.H >= 1 && a.dim >= 1 && a.vdim >= 1 && a.ld_out >= a.H * a.vdim && (a.seqs || a.positions), "recurrence: bad sizes");
-    if (dt == PGK_F32) return recur_scan<float, true>(a, st);
-    return io32 ? recur_scan<float, false>(a, st) : recur_scan<bf16, false>(a, st);
+    if (a.kind == RECUR_SSD) {
+        PGK_REQUIRE(a.G >= 1 && a.H % a.G == 0 && (a.seqs ? a.rows != nullptr : a.conv.taps >= 1 && a.conv.ring), "recurrence: bad state-space arguments");
+        if (dt == PGK_F32) return recur_scan<float, float, true, RECUR_SSD>(a, st);
+        return io32 ? recur_scan<bf16, float, false, RECUR_SSD>(a, st) : recur_scan<bf16, bf16, false, RECUR_SSD>(a, st);
+    }
+    if (dt == PGK_F32) return recur_scan<float, float, true, RECUR_HGRN2>(a, st);
+    return io32 ? recur_scan<bf16, float, false, RECUR_HGRN2>(a, st) : recur_scan<bf16, bf16, false, RECUR_HGRN2>(a, st);
 }
 
 // -------------------------------------------------------------------------------------------- chunks
@@ -140,8 +166,8 @@ __device__ __forceinline__ float4 mul4(const float4& a, const float4& b) { retur
 __host__ __device__ constexpr int rc_col_stride(int w) { return (w / 16) % 2 ? w : w + 16; }
 __host__ __device__ constexpr int rc_row_stride(int w) { return w + 4; }
 
-static size_t rc_state_lds(int C, int dim, int vdim) { return ((size_t)C * (rc_col_stride(dim) + rc_col_stride(vdim)) + (C / 16) * dim) * 4; }
-static size_t rc_out_lds(int C, int dim) { return ((size_t)3 * C * rc_row_stride(dim) + C * rc_row_stride(C) + (C / 16) * dim + 8 * C) * 4; }
+static size_t rc_state_lds(int C, int dim, int vdim) { return ((size_t)C * (rc_col_stride(dim) + rc_col_stride(vdim)) + (C / 16) * dim + 2 * C) * 4; }
+static size_t rc_out_lds(int C, int dim) { return ((size_t)3 * C * rc_row_stride(dim) + C * rc_row_stride(C) + (C / 16) * dim + 10 * C) * 4; }
 constexpr size_t RC_LDS_MAX = 156 * 1024;
 
 int recur_chunk_rows(int dim, int vdim) {
@@ -153,36 +179,44 @@ int recur_chunk_rows(int dim, int vdim) {
 size_t recur_chunk_bytes(const RecurArgs& a, int n_chunks) { return (size_t)n_chunks * a.H * ((size_t)a.dim * a.vdim + a.dim) * 4; }
 
 // 1: U [chunk][head][dim][vdim], D [chunk][head][dim].  Eight waves; VT column tiles of 16 at a time (vdim is a multiple of 16 VT).
-template <class T, int C, int VT>
+template <class T, int C, int VT, int SRC>
 __global__ __launch_bounds__(512) void recur_chunk_state_kernel(RecurArgs a, const RecurChunk* chunks, float* U, float* D) {
     extern __shared__ __attribute__((aligned(16))) float sm[];
     constexpr int NS = C / 16, VB = 4;
     constexpr bool EXACT = std::is_same<T, float>::value;
     const int dim = a.dim, vdim = a.vdim, ks = rc_col_stride(dim), vs = rc_col_stride(vdim), h = blockIdx.x;
-    float *kr = sm, *v = kr + C * ks, *F = v + C * vs;
+    float *kr = sm, *v = kr + C * ks, *F = v + C * vs, *step = F + NS * dim, *fade = step + C;
     const RecurChunk ch = chunks[blockIdx.y];
     const int tid = threadIdx.x, lane = tid & 63, wid = tid >> 6, l15 = lane & 15, q4 = lane >> 4, last = ch.len - 1;
     const T* in = reinterpret_cast<const T*>(a.in) + (size_t)ch.row0 * a.ld_in;
-    const T* vin = in + a.v_off + h * vdim;
+    const int ld = SRC == RECUR_SSD ? a.ld_rows : a.ld_in, kh = SRC == RECUR_SSD ? h / (a.H / a.G) : h;
+    const T* ch_in = SRC == RECUR_SSD ? reinterpret_cast<const T*>(a.rows) + (size_t)ch.row0 * ld : in;
+    const T* vin = ch_in + a.v_off + h * vdim;
+    if constexpr (SRC == RECUR_SSD) {
+        if (tid < C) ssd_step(to_f(in[(size_t)min(tid, last) * a.ld_in + a.dt_off + h]), a.dt_bias[h], a.decay[h], step[tid], fade[tid]);
+        __syncthreads();
+    }
     const int nv = C * vdim / 4, v4 = vdim / 4;
     // k times the decay to the end of its block of 16 rows, and the blocks' decays; the first values travel with the first gates
     float4 vv[VB];
     for (int t = tid, t0 = 0; t < NS * dim || t0 == 0; t += 512, t0 = 1) {
         const int b = min(t / dim, NS - 1), d = t % dim;
-        const T* z = in + a.f_off + h * dim + d;
+        const T* z = ch_in + a.f_off + kh * dim + d;
         float zf[16];
 #pragma unroll
-        for (int r = 0; r < 16; ++r) zf[r] = to_f(z[(size_t)min(16 * b + r, last) * a.ld_in]);
-        const float bias = a.bias ? a.bias[h * dim + d] : 0.f, low = a.lower[h * dim + d];
+        for (int r = 0; r < 16; ++r) zf[r] = to_f(z[(size_t)min(16 * b + r, last) * ld]);
+        float bias = 0.f, low = 0.f;
+        if constexpr (SRC == RECUR_HGRN2) { bias = a.bias ? a.bias[h * dim + d] : 0.f; low = a.lower[h * dim + d]; }
         if (t0 == 0) {
 #pragma unroll
-            for (int i = 0; i < VB; ++i) { const int e = min(tid + 512 * i, nv - 1); vv[i] = load4<T>(vin + (size_t)min(e / v4, last) * a.ld_in + e % v4 * 4); }
+            for (int i = 0; i < VB; ++i) { const int e = min(tid + 512 * i, nv - 1); vv[i] = load4<T>(vin + (size_t)min(e / v4, last) * ld + e % v4 * 4); }
         }
         float run = 1.f;
 #pragma unroll
         for (int r = 15; r >= 0; --r) {
             float f, k;
-            rc_gate<EXACT>(zf[r] + bias, low, f, k);
+            if constexpr (SRC == RECUR_SSD) { f = fade[16 * b + r]; k = step[16 * b + r] * zf[r]; }
+            else rc_gate<EXACT>(zf[r] + bias, low, f, k);
             const bool live = 16 * b + r <= last;
             if (t < NS * dim) kr[(16 * b + r) * ks + d] = live ? k * run : 0.f;
             run *= live ? f : 1.f;
@@ -191,7 +225,7 @@ __global__ __launch_bounds__(512) void recur_chunk_state_kernel(RecurArgs a, con
     }
 #pragma unroll
     for (int i = 0; i < VB; ++i) { const int e = tid + 512 * i; if (e < nv) *reinterpret_cast<float4*>(v + e / v4 * vs + e % v4 * 4) = vv[i]; }
-    for (int e = tid + 512 * VB; e < nv; e += 512) *reinterpret_cast<float4*>(v + e / v4 * vs + e % v4 * 4) = load4<T>(vin + (size_t)min(e / v4, last) * a.ld_in + e % v4 * 4);
+    for (int e = tid + 512 * VB; e < nv; e += 512) *reinterpret_cast<float4*>(v + e / v4 * vs + e % v4 * 4) = load4<T>(vin + (size_t)min(e / v4, last) * ld + e % v4 * 4);
     __syncthreads();
     const size_t rec = (size_t)blockIdx.y * a.H + h;
     for (int d = tid; d < dim; d += 512) {
@@ -260,24 +294,26 @@ __global__ __launch_bounds__(256) void recur_chunk_scan_kernel(RecurArgs a, cons
 
 // 3: output rows.  Eight waves; NVT column tiles of 16 per wave.  The values and the first rows of the state travel while the gates and
 // the decays are worked out.
-template <class T, int C, int NVT>
+template <class T, int C, int NVT, int SRC>
 __global__ __launch_bounds__(512) void recur_chunk_out_kernel(RecurArgs a, const RecurChunk* chunks, const float* U) {
     extern __shared__ __attribute__((aligned(16))) float sm[];
     constexpr int NS = C / 16, AS = rc_row_stride(C);
     constexpr bool EXACT = std::is_same<T, float>::value;
     const int dim = a.dim, vdim = a.vdim, S = rc_row_stride(dim), h = blockIdx.x;
-    float *q = sm, *f = q + C * S, *k = f + C * S, *A = k + C * S, *F = A + C * AS, *red = F + NS * dim;
+    float *q = sm, *f = q + C * S, *k = f + C * S, *A = k + C * S, *F = A + C * AS, *red = F + NS * dim, *step = red + 8 * C, *fade = step + C;
     const RecurChunk ch = chunks[blockIdx.y];
     const int tid = threadIdx.x, lane = tid & 63, wid = tid >> 6, l15 = lane & 15, q4 = lane >> 4;
     const T* in = reinterpret_cast<const T*>(a.in) + (size_t)ch.row0 * a.ld_in;
     const int nz = C * dim / 4, d4 = dim / 4, last = ch.len - 1;
+    const int ld = SRC == RECUR_SSD ? a.ld_rows : a.ld_in, kh = SRC == RECUR_SSD ? h / (a.H / a.G) : h;
+    const T* ch_in = SRC == RECUR_SSD ? reinterpret_cast<const T*>(a.rows) + (size_t)ch.row0 * ld : in;
     const float* st = U + ((size_t)blockIdx.y * a.H + h) * dim * vdim;
     constexpr int ZB = 4, PRE = 8 / NVT;                           // pieces of the rows requested first; blocks of 16 state rows requested ahead
     float4 pq[ZB], pf[ZB];
 #pragma unroll
     for (int i = 0; i < ZB; ++i) {
         const int t = min(tid + 512 * i, nz - 1);
-        const T* row = in + (size_t)min(t / d4, last) * a.ld_in + h * dim + t % d4 * 4;
+        const T* row = ch_in + (size_t)min(t / d4, last) * ld + kh * dim + t % d4 * 4;
         pq[i] = load4<T>(row + a.q_off);
         pf[i] = load4<T>(row + a.f_off);
     }
@@ -285,20 +321,32 @@ __global__ __launch_bounds__(512) void recur_chunk_out_kernel(RecurArgs a, const
 #pragma unroll
     for (int t = 0; t < NVT; ++t) col[t] = min(16 * (wid + 8 * t), vdim - 16) + l15;
     float pv[NVT][NS][4], ps[NVT][PRE][4];
-    const T* v = in + a.v_off + h * vdim;
+    const T* v = ch_in + a.v_off + h * vdim;
 #pragma unroll
     for (int t = 0; t < NVT; ++t) {
 #pragma unroll
         for (int b = 0; b < NS; ++b)
 #pragma unroll
-            for (int u = 0; u < 4; ++u) pv[t][b][u] = to_f(v[(size_t)min(16 * b + 4 * q4 + u, last) * a.ld_in + col[t]]);
+            for (int u = 0; u < 4; ++u) pv[t][b][u] = to_f(v[(size_t)min(16 * b + 4 * q4 + u, last) * ld + col[t]]);
 #pragma unroll
         for (int b = 0; b < PRE; ++b)
 #pragma unroll
             for (int u = 0; u < 4; ++u) ps[t][b][u] = st[(size_t)min(16 * b + 4 * q4 + u, dim - 1) * vdim + col[t]];
     }
+    if constexpr (SRC == RECUR_SSD) {
+        if (tid < C) ssd_step(to_f(in[(size_t)min(tid, last) * a.ld_in + a.dt_off + h]), a.dt_bias[h], a.decay[h], step[tid], fade[tid]);
+        __syncthreads();
+    }
     auto gates = [&](int t, const float4& zq, const float4& zf) {
         const int r = t / d4, c = t % d4 * 4;
+        if constexpr (SRC == RECUR_SSD) {
+            const bool live = r < ch.len;
+            const float fr = live ? fade[r] : 1.f, sr = live ? step[r] : 0.f;
+            *reinterpret_cast<float4*>(q + r * S + c) = live ? zq : make_float4(0.f, 0.f, 0.f, 0.f);
+            *reinterpret_cast<float4*>(f + r * S + c) = make_float4(fr, fr, fr, fr);
+            *reinterpret_cast<float4*>(k + r * S + c) = make_float4(sr * zf.x, sr * zf.y, sr * zf.z, sr * zf.w);
+            return;
+        }
         const float4 b = a.bias ? *reinterpret_cast<const float4*>(a.bias + h * dim + c) : make_float4(0.f, 0.f, 0.f, 0.f);
         const float4 low = *reinterpret_cast<const float4*>(a.lower + h * dim + c);
         float4 qq = {rc_silu<EXACT>(zq.x), rc_silu<EXACT>(zq.y), rc_silu<EXACT>(zq.z), rc_silu<EXACT>(zq.w)}, ff, kk;
@@ -312,7 +360,7 @@ __global__ __launch_bounds__(512) void recur_chunk_out_kernel(RecurArgs a, const
 #pragma unroll
     for (int i = 0; i < ZB; ++i) if (tid + 512 * i < nz) gates(tid + 512 * i, pq[i], pf[i]);
     for (int t = tid + 512 * ZB; t < nz; t += 512) {
-        const T* row = in + (size_t)min(t / d4, last) * a.ld_in + h * dim + t % d4 * 4;
+        const T* row = ch_in + (size_t)min(t / d4, last) * ld + kh * dim + t % d4 * 4;
         gates(t, load4<T>(row + a.q_off), load4<T>(row + a.f_off));
     }
     __syncthreads();
@@ -468,6 +516,15 @@ __global__ __launch_bounds__(512) void recur_chunk_out_kernel(RecurArgs a, const
                 for (int t = 0; t < NVT; ++t) o[t][b] = mfma4(u == 0 ? y.x : u == 1 ? y.y : u == 2 ? y.z : y.w, pv[t][bj][u], o[t][b]);
         }
     // lane: rows 16 b + 4 q4 + r, column l15 of each tile
+    if constexpr (SRC == RECUR_SSD) {
+        const float skip = a.skip[h];
+#pragma unroll
+        for (int t = 0; t < NVT; ++t)
+#pragma unroll
+            for (int b = 0; b < NS; ++b)
+#pragma unroll
+                for (int r = 0; r < 4; ++r) o[t][b][r] = fmaf(skip, pv[t][b][r], o[t][b][r]);
+    }
     float inv[NS][4];
 #pragma unroll
     for (int b = 0; b < NS; ++b)
@@ -507,14 +564,23 @@ __global__ __launch_bounds__(512) void recur_chunk_out_kernel(RecurArgs a, const
                 const int row = 16 * b + 4 * q4 + r;
                 const float y = o[t][b][r] * inv[b][r] * g;
                 if (staged) q[row * ys + c] = y;
-                else if (row < ch.len) out[(size_t)row * a.ld_out + h * vdim + c] = from_f<T>(y);
+                else if (row < ch.len) {
+                    float w = y;
+                    if constexpr (SRC == RECUR_SSD) w *= silu_f<EXACT>(to_f(in[(size_t)row * a.ld_in + a.z_off + h * vdim + c]));
+                    out[(size_t)row * a.ld_out + h * vdim + c] = from_f<T>(w);
+                }
             }
     }
     if (staged) {
         __syncthreads();
         for (int t = tid; t < ch.len * (vdim / 4); t += 512) {
             const int r = t / (vdim / 4), c = t % (vdim / 4) * 4;
-            store4<T>(out + (size_t)r * a.ld_out + h * vdim + c, ld4(q + r * ys + c));
+            float4 y = ld4(q + r * ys + c);
+            if constexpr (SRC == RECUR_SSD) {
+                const float4 z = load4<T>(in + (size_t)r * a.ld_in + a.z_off + h * vdim + c);
+                y = mul4(y, make_float4(silu_f<EXACT>(z.x), silu_f<EXACT>(z.y), silu_f<EXACT>(z.z), silu_f<EXACT>(z.w)));
+            }
+            store4<T>(out + (size_t)r * a.ld_out + h * vdim + c, y);
         }
     }
     if (h == a.H - 1 && a.ld_out > a.H * vdim) {
@@ -530,35 +596,35 @@ static hipError_t rc_allow_lds(K kfn, size_t lds, bool& done) {
     return hipFuncSetAttribute(reinterpret_cast<const void*>(kfn), hipFuncAttributeMaxDynamicSharedMemorySize, (int)RC_LDS_MAX);
 }
 
-template <class T, int C, int NVT>
+template <class T, int C, int NVT, int SRC>
 static hipError_t launch_chunk_out(const RecurArgs& a, const RecurChunk* chunks, int n_chunks, const float* U, hipStream_t st) {
     static bool done = false;
     const size_t lds = rc_out_lds(C, a.dim);
-    if (hipError_t e = rc_allow_lds(&recur_chunk_out_kernel<T, C, NVT>, lds, done)) return e;
-    recur_chunk_out_kernel<T, C, NVT><<<dim3(a.H, n_chunks), 512, lds, st>>>(a, chunks, U);
+    if (hipError_t e = rc_allow_lds(&recur_chunk_out_kernel<T, C, NVT, SRC>, lds, done)) return e;
+    recur_chunk_out_kernel<T, C, NVT, SRC><<<dim3(a.H, n_chunks), 512, lds, st>>>(a, chunks, U);
     return hipGetLastError();
 }
 
-template <class T, int C, int VT>
+template <class T, int C, int VT, int SRC>
 static hipError_t launch_chunk_state(const RecurArgs& a, const RecurChunk* chunks, int n_chunks, float* U, float* D, hipStream_t st) {
     static bool done = false;
     const size_t lds = rc_state_lds(C, a.dim, a.vdim);
-    if (hipError_t e = rc_allow_lds(&recur_chunk_state_kernel<T, C, VT>, lds, done)) return e;
-    recur_chunk_state_kernel<T, C, VT><<<dim3(a.H, n_chunks), 512, lds, st>>>(a, chunks, U, D);
+    if (hipError_t e = rc_allow_lds(&recur_chunk_state_kernel<T, C, VT, SRC>, lds, done)) return e;
+    recur_chunk_state_kernel<T, C, VT, SRC><<<dim3(a.H, n_chunks), 512, lds, st>>>(a, chunks, U, D);
     return hipGetLastError();
 }
 
-template <class T, int C>
+template <class T, int C, int SRC>
 static pgk_status recur_chunked_t(const RecurArgs& a, const RecurChunk* chunks, int n_chunks, const int32_t* chunk_of_seq, void* ws, hipStream_t st) {
     float *U = (float*)ws, *D = U + (size_t)n_chunks * a.H * a.dim * a.vdim;
-    if (a.vdim % 128 == 0) PGK_CHECK_HIP((launch_chunk_state<T, C, 8>(a, chunks, n_chunks, U, D, st)));
-    else if (a.vdim % 64 == 0) PGK_CHECK_HIP((launch_chunk_state<T, C, 4>(a, chunks, n_chunks, U, D, st)));
-    else PGK_CHECK_HIP((launch_chunk_state<T, C, 1>(a, chunks, n_chunks, U, D, st)));
+    if (a.vdim % 128 == 0) PGK_CHECK_HIP((launch_chunk_state<T, C, 8, SRC>(a, chunks, n_chunks, U, D, st)));
+    else if (a.vdim % 64 == 0) PGK_CHECK_HIP((launch_chunk_state<T, C, 4, SRC>(a, chunks, n_chunks, U, D, st)));
+    else PGK_CHECK_HIP((launch_chunk_state<T, C, 1, SRC>(a, chunks, n_chunks, U, D, st)));
     recur_chunk_scan_kernel<<<dim3(ceil_div(a.dim * a.vdim / 4, 256), a.H, a.n_seqs), 256, 0, st>>>(a, chunk_of_seq, U, D);
     PGK_LAUNCH_CHECK();
-    if (a.vdim <= 128) PGK_CHECK_HIP((launch_chunk_out<T, C, 1>(a, chunks, n_chunks, U, st)));
-    else if (a.vdim <= 256) PGK_CHECK_HIP((launch_chunk_out<T, C, 2>(a, chunks, n_chunks, U, st)));
-    else PGK_CHECK_HIP((launch_chunk_out<T, C, 4>(a, chunks, n_chunks, U, st)));
+    if (a.vdim <= 128) PGK_CHECK_HIP((launch_chunk_out<T, C, 1, SRC>(a, chunks, n_chunks, U, st)));
+    else if (a.vdim <= 256) PGK_CHECK_HIP((launch_chunk_out<T, C, 2, SRC>(a, chunks, n_chunks, U, st)));
+    else PGK_CHECK_HIP((launch_chunk_out<T, C, 4, SRC>(a, chunks, n_chunks, U, st)));
     return PGK_OK;
 }
 
@@ -566,8 +632,13 @@ pgk_status recur_chunked(const RecurArgs& a, const RecurChunk* chunks, int n_chu
     const int C = recur_chunk_rows(a.dim, a.vdim);
     PGK_REQUIRE(C && a.seqs && chunks && n_chunks >= 1 && n_chunks <= 65535 && a.H * a.vdim <= a.ld_out && a.ld_in % 4 == 0 && a.q_off % 4 == 0 && a.f_off % 4 == 0 && a.v_off % 4 == 0,
                 "recurrence: %d chunks of head widths %d / %d", n_chunks, a.dim, a.vdim);
-    if (dt == PGK_F32) return C == 64 ? recur_chunked_t<float, 64>(a, chunks, n_chunks, chunk_of_seq, ws, st) : recur_chunked_t<float, 32>(a, chunks, n_chunks, chunk_of_seq, ws, st);
-    return C == 64 ? recur_chunked_t<bf16, 64>(a, chunks, n_chunks, chunk_of_seq, ws, st) : recur_chunked_t<bf16, 32>(a, chunks, n_chunks, chunk_of_seq, ws, st);
+    PGK_REQUIRE(a.kind != RECUR_SSD || (a.rows && a.ld_rows % 4 == 0 && a.z_off % 4 == 0 && a.G >= 1 && a.H % a.G == 0), "recurrence: bad state-space arguments");
+    auto go = [&](auto src) -> pgk_status {
+        constexpr int SRC = decltype(src)::value;
+        if (dt == PGK_F32) return C == 64 ? recur_chunked_t<float, 64, SRC>(a, chunks, n_chunks, chunk_of_seq, ws, st) : recur_chunked_t<float, 32, SRC>(a, chunks, n_chunks, chunk_of_seq, ws, st);
+        return C == 64 ? recur_chunked_t<bf16, 64, SRC>(a, chunks, n_chunks, chunk_of_seq, ws, st) : recur_chunked_t<bf16, 32, SRC>(a, chunks, n_chunks, chunk_of_seq, ws, st);
+    };
+    return a.kind == RECUR_SSD ? go(std::integral_constant<int, RECUR_SSD>{}) : go(std::integral_constant<int, RECUR_HGRN2>{});
 }
 
 }  // namespace pgk
