@@ -375,9 +375,42 @@ pgk_status pgk_xielu(const void* x, void* y, size_t n, float a, float b, pgk_dty
 pgk_status pgk_gated_recurrence(const void* q, const void* f, const void* v, const float* f_bias, const float* lower,
                                 const float* norm, float* state, void* out, int n, int fresh, int heads, int dim, int vdim,
                                 float eps, pgk_dtype dt, pgk_stream s);
+/* silu of the short convolution: u [n, channels], w [taps, channels] (the last row multiplies the token itself), bias fp32 [channels]
+ * or NULL, past as for pgk_short_conv.  channels: a multiple of 4.  dt: PGK_BF16 or PGK_F32 */
+pgk_status pgk_conv_silu(const void* u, const void* past, const void* w, const float* bias, void* out, int n, int channels, int taps,
+                         pgk_dtype dt, pgk_stream s);
+/* Gated delta rule over n rows of one sequence: q, k [n, kv_heads * dim], v [n, heads * vdim] (after taps and activation), decay logits z
+ * [n, heads * dim], strengths [n, heads] and gates [n, heads * vdim] before their sigmoid; fp32 decay [heads], step_bias [heads * dim],
+ * norm [vdim].  q, k of unit length per head (q also times dim^-1/2), b = sigmoid(strength), g = exp(-decay softplus(z + step_bias)):
+ * S <- diag(g) S, u = b (v - S^T k), S <- S + k u^T, o = S^T q; out = o / rms(o) * norm * sigmoid(gate).  state: fp32 [heads, dim, vdim],
+ * read unless `fresh`, updated.  dim, vdim: multiples of 4.  dt (all but z, which is fp32): PGK_BF16 or PGK_F32 */
+pgk_status pgk_delta_rule(const void* q, const void* k, const void* v, const float* z, const void* strength, const void* gate,
+                          const float* decay, const float* step_bias, const float* norm, float* state, void* out, int n, int fresh,
+                          int heads, int kv_heads, int dim, int vdim, float eps, pgk_dtype dt, pgk_stream s);
+/* State-space duality over n rows of one sequence: xbc [n, heads * vdim | groups * dim | groups * dim] (x, B, C after taps and activation), z
+ * [n, heads * vdim], t [n, heads]; fp32 decay, step_bias, skip [heads], norm [heads * vdim].  t <- softplus(t + step_bias),
+ * S <- exp(-decay t) S + t B x^T, y = S^T C + skip x; out = (y silu(z)) / rms * norm in norm_parts equal parts.  state: fp32
+ * [heads, dim, vdim], read unless `fresh`, updated.  dim, vdim: multiples of 4.  dt: PGK_BF16 or PGK_F32 */
+pgk_status pgk_state_space(const void* xbc, const void* z, const void* t, const float* decay, const float* step_bias, const float* skip,
+                           const float* norm, float* state, void* out, int n, int fresh, int heads, int groups, int dim, int vdim,
+                           int norm_parts, float eps, pgk_dtype dt, pgk_stream s);
+/* Mixture of experts: x [n, width], router [experts up to a multiple of 64, width], correction fp32 [experts], w_up [experts, 2 ff, width]
+ * (gate rows, up rows), w_down [experts, width, ff], out fp32 [n, width].  s = sigmoid(router x); the `top` largest s + correction are
+ * chosen, with groups > 0 among the experts of the `keep` groups of neighbours whose two largest values have the largest sum; the chosen
+ * experts' SwiGLU outputs are summed with weights scale * s / (sum of the chosen s).  width, ff: multiples of 64.  dt: PGK_BF16 or PGK_F32 */
+pgk_status pgk_moe(const void* x, const void* router, const float* correction, const void* w_up, const void* w_down, float* out, int n,
+                   int width, int ff, int experts, int top, int groups, int keep, float scale, pgk_dtype dt, pgk_stream s);
+/* out[row] = (x - mean) / sqrt(mean((x - mean)^2) + eps) * weight: fp32 rows and weight, result in out_dt */
+pgk_status pgk_layernorm_f32(const float* x, const float* weight, void* out, int rows, int cols, float eps, pgk_dtype out_dt, pgk_stream s);
+/* Rows of a latent cache: x [n, rank + rot] -> [c / rms(c) * norm | r turned], c the first rank columns, r the last rot; row i is position
+ * first + i, columns (2j, 2j + 1) of r turn by position * freq[j].  norm fp32 [rank], freq fp32 [rot / 2] */
+pgk_status pgk_latent_rows(const void* x, const float* norm, const float* freq, void* out, int n, int rank, int rot, int first, float eps,
+                           pgk_dtype dt, pgk_stream s);
+/* x [n, heads, dim]: the last rot columns of every head are turned as in pgk_latent_rows, in place */
+pgk_status pgk_rotate_pairs(void* x, const float* freq, int n, int heads, int dim, int rot, int first, pgk_dtype dt, pgk_stream s);
 /* x[row][head][:] *= sigmoid(gate[row][head]) in place */
 pgk_status pgk_head_gate(void* x, const void* gate, int rows, int heads, int d, int64_t gate_stride, pgk_dtype dt, pgk_stream s);
-/* dst [dst_rows, dst_cols] = src [rows, cols] with zeros around it */
+/* dst [dst_rows, dst_cols] = src [rows, cols] with zeros around it (dst_cols < cols: its first columns) */
 pgk_status pgk_pad_2d(const void* src, void* dst, int rows, int cols, int dst_rows, int dst_cols, pgk_dtype dt, pgk_stream s);
 
 /* ---------------------------------------------------------------------- engine ------ */

@@ -48,19 +48,21 @@ class LayerWeights(C.Structure):
 
 class StackConfig(C.Structure):
     _fields_ = [(n, C.c_int) for n in ("vocab_size", "width", "num_layers", "max_positions", "max_seq_len", "max_batch")] + \
-               [("norm_eps", C.c_float), ("residual_mult", C.c_float), ("dtype", C.c_int)]
+               [("norm_eps", C.c_float), ("residual_mult", C.c_float), ("dtype", C.c_int)] + \
+               [(n, C.c_int) for n in ("block", "layer_norm", "loop_start", "loop_stop", "loop_times")] + [("loop_in", C.c_void_p), ("loop_step", C.c_void_p)]
 
 
 class StackLayer(C.Structure):
     _fields_ = [(n, C.c_int) for n in ("mixer", "ff", "heads", "kv_heads", "dim", "vdim", "rank", "window", "taps", "kv_from", "head_pad", "vhead_pad", "rank_pad",
-                                       "n_in", "n_att", "ff_pad")] + \
-               [(n, C.c_float) for n in ("scale", "act_pos", "act_neg")] + \
+                                       "n_in", "n_att", "ff_pad", "gated", "rot", "norm_parts", "rank_a", "rank_g", "experts", "top", "groups", "keep")] + \
+               [(n, C.c_float) for n in ("scale", "act_pos", "act_neg", "router_scale")] + \
                [(n, C.c_void_p) for n in ("norm1", "norm1b", "norm2", "norm2b", "w_in", "b_in", "conv", "q_norm", "k_norm", "slopes", "lower", "o_norm", "c_norm",
-                                          "w_ukv", "w_o", "w_gate_up", "w_down")]
+                                          "w_ukv", "w_o", "w_gate_up", "w_down", "rot_freq", "decay", "dt_bias", "skip", "conv_bias", "w_a2", "w_g2", "correction")]
 
 
-MIX_LATENT, MIX_ATTENTION, MIX_HGRN2 = 0, 1, 2      # pgk_mixer
-FF_SWIGLU, FF_XIELU = 0, 1                          # pgk_ff
+MIX_LATENT, MIX_ATTENTION, MIX_HGRN2, MIX_DELTA, MIX_SSD = 0, 1, 2, 3, 4      # pgk_mixer
+FF_SWIGLU, FF_XIELU, FF_MOE = 0, 1, 2                                           # pgk_ff
+BLOCK_SANDWICH, BLOCK_PARALLEL = 0, 1                                           # pgk_block
 
 
 # name -> (argtypes); every function returns pgk_status (int) unless listed in _NON_STATUS
@@ -123,6 +125,10 @@ _PROTOS = {
     "pgk_rmsnorm_f32": [_V, _V, _V, _I, _I, _F, _I, _V], "pgk_rmsnorm_add_f32": [_V, _V, _V, _I, _I, _F, _F, _I, _V],
     "pgk_window_attention": [_V, _V, _V, _V, _I, _I, _I, _I, _I, _I, _F, _I, _V, _I64, _I, _V, _I, _V],
     "pgk_short_conv": [_V, _V, _V, _V, _I, _I, _I, _I, _V], "pgk_sigmoid_mul": [_V, _V, _Z, _I, _V], "pgk_xielu": [_V, _V, _Z, _F, _F, _I, _V],
+    "pgk_conv_silu": [_V, _V, _V, _V, _V, _I, _I, _I, _I, _V],
+    "pgk_delta_rule": [_V] * 11 + [_I] * 6 + [_F, _I, _V], "pgk_state_space": [_V] * 9 + [_I] * 7 + [_F, _I, _V],
+    "pgk_moe": [_V] * 6 + [_I] * 7 + [_F, _I, _V], "pgk_layernorm_f32": [_V, _V, _V, _I, _I, _F, _I, _V],
+    "pgk_latent_rows": [_V, _V, _V, _V, _I, _I, _I, _I, _F, _I, _V], "pgk_rotate_pairs": [_V, _V, _I, _I, _I, _I, _I, _I, _V],
     "pgk_gated_recurrence": [_V, _V, _V, _V, _V, _V, _V, _V, _I, _I, _I, _I, _I, _F, _I, _V],
     "pgk_head_gate": [_V, _V, _I, _I, _I, _I64, _I, _V], "pgk_pad_2d": [_V, _V, _I, _I, _I, _I, _I, _V],
     "pgk_engine_set_state": [_V, c_i32_p, c_i32_p, _I, _V], "pgk_engine_decode_step": [_V, _I, _V],

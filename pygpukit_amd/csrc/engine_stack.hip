@@ -1,16 +1,22 @@
-// Native engine for layer-list decoders: an fp32 residual stream, RMSNorm after each sublayer and, where a layer has one, before it;
-// a dense feed-forward (SwiGLU or xIELU) or none.  Every layer has its own mixer and its own sizes.  Elements are bf16 (fp32 stream, norms,
-// scores, softmax, recurrent states) or fp32 throughout.
+// Native engine for layer-list decoders: an fp32 residual stream; every layer has its own mixer and its own sizes.  Elements are bf16
+// (fp32 stream, norms, scores, softmax, routers, recurrent states) or fp32 throughout.
 //
+// Sandwich layers: RMSNorm rho after each sublayer and, where a layer has one, before it; a dense feed-forward (SwiGLU or xIELU) or none
 //   x   <- x + m * rho(O mixer(h); n1b),            h = rho(x; n1) or x
 //   x   <- x + m * rho(W_d act(W_u h); n2b),        h = rho(x; n2) or x
+// Parallel layers: one norm (RMS or layer norm), a mixture of experts (moe.hip.h) or no feed-forward
+//   x   <- x + m * (O mixer(h) + moe(h)),           h = nu(x; n1)
+// A stretch of layers may run several times over with the same weights (`Run`: one pass of one layer, with a cache of its own); pass t
+// starts with  x <- L [x; embedding] + s_t.
 //
 // Mixers (pgk_mixer):
 //   latent attention  sigmoid(G h) * attention(Q h, c),  c = rms(D h) * w_c,  k = U_k c,  v = U_v c: over a sliding window; the cache holds
-//                     one normalised latent row per token, not keys and values.  The kernels are in this file.
+//                     one normalised latent row per token, not keys and values.  A latent row may end in columns that are turned by the
+//                     position instead (the rotary part of the key, one for all heads).  The kernels are in this file.
 //   attention         taps over time and norms on q, k, v, a K/V ring (which another layer may own), distance bias, elementwise gate:
 //                     ops_gated_attn.hip
-//   hgrn2             gated linear recurrence with an fp32 state per sequence and head: ops_recurrence.hip
+//   hgrn2, ssd        linear recurrences with an fp32 state per sequence and head: ops_recurrence.hip
+//   delta             gated delta rule with a decay per key channel: ops_delta.hip
 // In a step a mixer takes the in-projection row(s) and leaves the rows that the out-projection multiplies.
 //
 // Latent cache: per layer [slot][R][rank] latents, R = min(window, max_seq_len); position p lives in row p mod R, so a full ring IS the
@@ -27,6 +33,8 @@
 //   down       y = W_d act
 // The reduction a post-norm needs over the whole sublayer output is done in the NEXT kernel's prologue, by every workgroup for itself
 // (one row: a few KB from L2), so it costs no launch.
+// A parallel layer, one sequence: in_proj (pending add, norm; router logits are rows of the same matrix), the mixer, moe_up (choice,
+// SwiGLU of the chosen experts), out (W_o and the chosen experts' down projections as one product).
 // Several sequences and prompts: the same kernels on rows, the norms as a launch of their own and the projections on the GEMM family
 // (pgk_gemm_nt: GEMV up to 8 rows, weight-streaming MFMA up to 128, tiled MFMA beyond).
 // All widths are padded with zeros by the caller: every K is a multiple of 64, head widths are 64, 128 or a larger multiple of 64.
@@ -36,6 +44,7 @@
 #include "engine_state.hip.h"
 #include "latent.hip.h"
 #include "mixers.hip.h"
+#include "moe.hip.h"
 #include "pkgemm.hip.h"
 
 namespace pgk {
@@ -55,7 +64,7 @@ pgk_status engine_gemm_nt_slabs(const bf16* A, const void* W, float* slabs, int 
 constexpr float LOG2E = 1.4426950408889634f;
 
 // -------------------------------------------------------------------------------------------- one-row projection
-enum { SP_NORM = 0, SP_PLAIN = 1 };
+enum { SP_NORM = 0, SP_PLAIN = 1, SP_ADD = 2, SP_CAT = 3 };
 enum { SE_STORE = 0, SE_SWIGLU = 1, SE_LOGITS = 2, SE_XIELU = 3 };
 
 struct StackGemvArgs {
@@ -66,11 +75,28 @@ struct StackGemvArgs {
     const float* g_post;      // its post-norm weight
     float* x_out;             // where workgroup 0 writes the updated residual row (another buffer than x; null: nowhere)
     const float* gamma;       // null: the row is taken as it is
+    // SP_ADD: v = (base or x) + mult * y, then the norm (layer_norm: the mean is taken off); h_out: where workgroup 0 writes the normed row.
+    // SP_CAT: the input is [v | row *tok of the embedding table], K / 2 elements each
+    const float* base;
+    int layer_norm;
+    float* h_out;
+    const void* embed; const int32_t* tok;
     float eps, mult;
     float* out;               // [N]
     float* amax_val; int* amax_idx;
     float act_pos, act_neg;   // SE_XIELU
 };
+
+// s + 16 bytes of a weight row . the same piece of the LDS row
+template <class WT>
+__device__ __forceinline__ float dot_piece(const uint4& raw, const WT* xp, float s) {
+    if constexpr (std::is_same<WT, bf16>::value) return dot8_bf16(raw, *reinterpret_cast<const uint4*>(xp), s);
+    else {
+        const float4 x4 = *reinterpret_cast<const float4*>(xp);
+        s = fmaf(__uint_as_float(raw.x), x4.x, s); s = fmaf(__uint_as_float(raw.y), x4.y, s);
+        s = fmaf(__uint_as_float(raw.z), x4.z, s); return fmaf(__uint_as_float(raw.w), x4.w, s);
+    }
+}
 
 // 256 threads; a wave owns R weight rows per trip.  C > 0: the first trip's C chunks of every row are requested before the prologue
 // touches the activations (which were requested before them: vector memory returns in order), K <= C * 64 * NW; C == 0: any K.
@@ -92,13 +118,31 @@ __global__ __launch_bounds__(256) void stack_gemv_kernel(unsigned long long* tl,
         else return min(n0 + r, N - 1);
     };
     uint4 pre[R][C > 0 ? C : 1];
-    if constexpr (C > 0) {
+    if constexpr (PRO == SP_CAT) {
+        const WT* er = reinterpret_cast<const WT*>(a.embed) + (size_t)*a.tok * a.W;
+        const float* from = a.base ? a.base : a.x;
+        const int half = K / 2, pad = (K + CH - 1) / CH * CH;
+        for (int i = threadIdx.x; i < pad; i += 256)
+            xs[i] = i < half ? from_f<WT>(a.y ? fmaf(a.mult, a.y[i], from[i]) : from[i]) : i - half < a.W ? er[i - half] : from_f<WT>(0.f);
+        if constexpr (C > 0) {
+            const int nf = min(wave * OUT, N - 1);
+#pragma unroll
+            for (int r = 0; r < R; ++r)
+#pragma unroll
+                for (int c = 0; c < C; ++c) pre[r][c] = load_nt16(w + (size_t)row_of(nf, r) * K + min(c * CH + lane * NW, K - NW));
+            for (int i = pad + threadIdx.x; i < C * CH; i += 256) xs[i] = from_f<WT>(0.f);
+        }
+    } else if constexpr (C > 0) {
         constexpr int NT = (C * CH + 1023) / 1024;                // float4 per thread
         float4 v[NT], y[NT], gp[NT], gm[NT];
 #pragma unroll
         for (int t = 0; t < NT; ++t) {
             const int i = min((int)(threadIdx.x + 256 * t) * 4, K - 4);
-            v[t] = *reinterpret_cast<const float4*>(a.x + i);
+            v[t] = *reinterpret_cast<const float4*>((PRO == SP_ADD && a.base ? a.base : a.x) + i);
+            if constexpr (PRO == SP_ADD) {
+                y[t] = *reinterpret_cast<const float4*>((a.y ? a.y : a.x) + i);
+                gm[t] = *reinterpret_cast<const float4*>(a.gamma + i);
+            }
             if constexpr (PRO == SP_NORM) {
                 const float* yp = a.y ? a.y : a.x;                // unconditional loads; masked below
                 const float* gm_p = a.gamma ? a.gamma : a.x;
@@ -116,6 +160,38 @@ __global__ __launch_bounds__(256) void stack_gemv_kernel(unsigned long long* tl,
             for (int c = 0; c < C; ++c) pre[r][c] = load_nt16(w + (size_t)row_of(nf, r) * K + min(c * CH + lane * NW, K - NW));
         __builtin_amdgcn_sched_barrier(0);
         float ss = 0.f;
+        if constexpr (PRO == SP_ADD) {
+            if (a.y) {
+#pragma unroll
+                for (int t = 0; t < NT; ++t) {
+                    const int i = (threadIdx.x + 256 * t) * 4;
+                    v[t].x = fmaf(a.mult, y[t].x, v[t].x); v[t].y = fmaf(a.mult, y[t].y, v[t].y);
+                    v[t].z = fmaf(a.mult, y[t].z, v[t].z); v[t].w = fmaf(a.mult, y[t].w, v[t].w);
+                    if (a.x_out && blockIdx.x == 0 && i < K) *reinterpret_cast<float4*>(a.x_out + i) = v[t];
+                }
+            }
+            float mean = 0.f;
+            if (a.layer_norm) {                                    // (columns W .. K are zero)
+                float s1 = 0.f;
+#pragma unroll
+                for (int t = 0; t < NT; ++t)
+                    if ((int)(threadIdx.x + 256 * t) * 4 < K) s1 += (v[t].x + v[t].y) + (v[t].z + v[t].w);
+                mean = block_sum(s1, red) / a.W;
+            }
+#pragma unroll
+            for (int t = 0; t < NT; ++t) {
+                const int i = (threadIdx.x + 256 * t) * 4;
+                v[t].x -= mean; v[t].y -= mean; v[t].z -= mean; v[t].w -= mean;
+                ss += (i < a.W ? v[t].x * v[t].x : 0.f) + (i + 1 < a.W ? v[t].y * v[t].y : 0.f) + (i + 2 < a.W ? v[t].z * v[t].z : 0.f) + (i + 3 < a.W ? v[t].w * v[t].w : 0.f);
+            }
+            const float inv = 1.0f / sqrtf(block_sum(ss, red) / a.W + a.eps);
+#pragma unroll
+            for (int t = 0; t < NT; ++t) {
+                const int i = (threadIdx.x + 256 * t) * 4;
+                v[t].x *= inv * gm[t].x; v[t].y *= inv * gm[t].y; v[t].z *= inv * gm[t].z; v[t].w *= inv * gm[t].w;
+                if (a.h_out && blockIdx.x == 0 && i < K) *reinterpret_cast<float4*>(a.h_out + i) = v[t];
+            }
+        }
         if constexpr (PRO == SP_NORM) {
             if (a.y) {
 #pragma unroll
@@ -166,6 +242,23 @@ __global__ __launch_bounds__(256) void stack_gemv_kernel(unsigned long long* tl,
             }
             const float inv = a.gamma ? 1.0f / sqrtf(block_sum(ss, red) / a.W + a.eps) : 1.0f;
             for (int i = threadIdx.x; i < K; i += 256) xs[i] = from_f<WT>(a.gamma ? xin(i) * inv * a.gamma[i] : xin(i));
+        } else if constexpr (PRO == SP_ADD) {
+            const float* from = a.base ? a.base : a.x;
+            auto xin = [&](int i) -> float { return a.y ? fmaf(a.mult, a.y[i], from[i]) : from[i]; };
+            float s1 = 0.f, ss = 0.f;
+            for (int i = threadIdx.x; i < K; i += 256) {
+                const float v = xin(i);
+                if (a.y && a.x_out && blockIdx.x == 0) a.x_out[i] = v;
+                s1 += v;
+            }
+            const float mean = a.layer_norm ? block_sum(s1, red) / a.W : 0.f;
+            for (int i = threadIdx.x; i < a.W; i += 256) { const float v = xin(i) - mean; ss = fmaf(v, v, ss); }
+            const float inv = 1.0f / sqrtf(block_sum(ss, red) / a.W + a.eps);
+            for (int i = threadIdx.x; i < K; i += 256) {
+                const float v = (xin(i) - mean) * inv * a.gamma[i];
+                xs[i] = from_f<WT>(v);
+                if (a.h_out && blockIdx.x == 0) a.h_out[i] = v;
+            }
         } else {
             for (int i = threadIdx.x; i < K; i += 256) xs[i] = from_f<WT>(a.x[i]);
         }
@@ -178,14 +271,6 @@ __global__ __launch_bounds__(256) void stack_gemv_kernel(unsigned long long* tl,
         float acc[R][1];
 #pragma unroll
         for (int r = 0; r < R; ++r) acc[r][0] = 0.f;
-        auto dot = [&](const uint4& raw, const WT* xp, float s) -> float {
-            if constexpr (std::is_same<WT, bf16>::value) return dot8_bf16(raw, *reinterpret_cast<const uint4*>(xp), s);
-            else {
-                const float4 x4 = *reinterpret_cast<const float4*>(xp);
-                s = fmaf(__uint_as_float(raw.x), x4.x, s); s = fmaf(__uint_as_float(raw.y), x4.y, s);
-                s = fmaf(__uint_as_float(raw.z), x4.z, s); return fmaf(__uint_as_float(raw.w), x4.w, s);
-            }
-        };
         if (C > 0) {
             if (g != wave) {
 #pragma unroll
@@ -196,7 +281,7 @@ __global__ __launch_bounds__(256) void stack_gemv_kernel(unsigned long long* tl,
 #pragma unroll
             for (int c = 0; c < (C > 0 ? C : 1); ++c)
 #pragma unroll
-                for (int r = 0; r < R; ++r) acc[r][0] = dot(pre[r][c], xs + c * CH + lane * NW, acc[r][0]);
+                for (int r = 0; r < R; ++r) acc[r][0] = dot_piece<WT>(pre[r][c], xs + c * CH + lane * NW, acc[r][0]);
         } else {
             const WT* wrow[R];
 #pragma unroll
@@ -278,19 +363,30 @@ static pgk_status stack_gemv(const StackGemvArgs& a, hipStream_t st, int force_g
 // -------------------------------------------------------------------------------------------- latent attention, decode
 struct LatentArgs {
     const void* in;           // [B][ld_in] (IT): q at h * D, latent at qn, head gates at qn + rank
-    int ld_in, qn, g_off;
+    int ld_in, qn, g_off;     // g_off < 0: no gates
     const void *w_uk, *w_uv;  // [H * D][rank] (T)
     const float* c_norm;      // [rank]
     void* cache;              // [slots][R][rank] (T)
     const int32_t* positions; // [B]
     int B, H, D, dim, vdim, rank, rank_true, R, nsplit, vc;
     float eps, scale;         // scale already times log2e
+    int rot;                  // the last rot of a head's dim query columns and the rot latent columns behind rank_true are turned by the position
+    const float* rot_freq;    // [rot / 2]
     void* qlat;               // [B][H][rank], float or bf16
     float* po;                // [B][H][nsplit][rank]
     float* pml;               // [B][H][nsplit][2]
     void* out;                // [B][ld_out] (IT): head h at h * D
     int ld_out;
 };
+
+// Column i of n rotated ones (neighbours 2j, 2j + 1 are a pair): x points at column 0
+template <class T>
+__device__ __forceinline__ float rotated(const T* x, int i, int pos, const float* freq) {
+    float s, c;
+    sincosf((float)pos * freq[i >> 1], &s, &c);
+    const float u = to_f(x[i & ~1]), v = to_f(x[i | 1]);
+    return i & 1 ? fmaf(v, c, u * s) : fmaf(u, c, -v * s);
+}
 
 // q_lat[b][h][r] = scale * sum_d U_k[h D + d][r] q[b][h][d]: workgroup = (head, 128 columns) x MB sequences, the four waves split d
 // in runs of four; 128 rows of U_k are requested before the queries are staged.  QT: element type of q_lat (bf16 for the MFMA kernel).
@@ -305,10 +401,12 @@ __global__ __launch_bounds__(256) void latent_absorb_kernel(unsigned long long* 
             const int b = b0 + m;
             const IT* c = in + (size_t)b * a.ld_in + a.qn;
             float ss = 0.f;
-            for (int r = lane; r < a.rank; r += 64) { const float v = to_f(c[r]); ss = fmaf(v, v, ss); }
+            for (int r = lane; r < a.rank_true; r += 64) { const float v = to_f(c[r]); ss = fmaf(v, v, ss); }
             const float inv = 1.0f / sqrtf(wave_sum(ss) / a.rank_true + a.eps);
-            T* row = reinterpret_cast<T*>(a.cache) + ((size_t)b * a.R + max(a.positions[b], 0) % a.R) * a.rank;
-            for (int r = lane; r < a.rank; r += 64) row[r] = from_f<T>(to_f(c[r]) * inv * a.c_norm[r]);
+            const int pos = max(a.positions[b], 0);
+            T* row = reinterpret_cast<T*>(a.cache) + ((size_t)b * a.R + pos % a.R) * a.rank;
+            for (int r = lane; r < a.rank; r += 64)
+                row[r] = from_f<T>(r >= a.rank_true && r < a.rank_true + a.rot ? rotated(c + a.rank_true, r - a.rank_true, pos, a.rot_freq) : to_f(c[r]) * inv * a.c_norm[r]);
         }
         tls.end();
         return;
@@ -333,7 +431,9 @@ __global__ __launch_bounds__(256) void latent_absorb_kernel(unsigned long long* 
         __syncthreads();
         for (int i = threadIdx.x; i < MB * 128; i += 256) {
             const int m = i >> 7, d = i & 127;
-            qs[m][d] = d < dn ? to_f(in[(size_t)min(b0 + m, a.B - 1) * a.ld_in + h * a.D + d0 + d]) : 0.f;
+            const int b = min(b0 + m, a.B - 1), at = d0 + d - (a.dim - a.rot);
+            const IT* q = in + (size_t)b * a.ld_in + h * a.D;
+            qs[m][d] = d >= dn ? 0.f : at < 0 ? to_f(q[d0 + d]) : rotated(q + a.dim - a.rot, at, max(a.positions[b], 0), a.rot_freq);
         }
         __syncthreads();
 #pragma unroll
@@ -681,13 +781,146 @@ __global__ __launch_bounds__(256) void latent_merge_uv_kernel(unsigned long long
             for (int m = 0; m < MB; ++m) {
                 const float y = group16_sum(acc[m]);
                 if (sub == 0 && v < a.vdim && b0 + m < a.B) {
-                    const float g = to_f(reinterpret_cast<const IT*>(a.in)[(size_t)(b0 + m) * a.ld_in + a.g_off + h]);
-                    reinterpret_cast<IT*>(a.out)[(size_t)(b0 + m) * a.ld_out + h * a.D + v] = from_f<IT>(y / (1.0f + expf(-g)));
+                    const float g = a.g_off < 0 ? 1.f : 1.0f / (1.0f + expf(-to_f(reinterpret_cast<const IT*>(a.in)[(size_t)(b0 + m) * a.ld_in + a.g_off + h])));
+                    reinterpret_cast<IT*>(a.out)[(size_t)(b0 + m) * a.ld_out + h * a.D + v] = from_f<IT>(y * g);
                 }
             }
         }
     }
     tls.end();
+}
+
+// -------------------------------------------------------------------------------------------- experts of one row
+struct MoeOneArgs {
+    RouterCfg r;
+    const float *logits, *h;              // [E], [W] (normed row)
+    const void *w_up, *w_down;            // [E][2 ff][W], [E][N][ff]
+    int W, ff;
+    float* act;                           // [top][ff], times the choice's weight
+    int32_t* ids;                         // [top]
+    const void* w_o; const float* a; int n_att;
+    float* y; int N;
+};
+
+// Every workgroup chooses for itself (a few hundred operations); a wave owns R / 2 outputs of one expert per trip.
+template <class WT, int R>
+__global__ __launch_bounds__(256) void moe_up_one_kernel(unsigned long long* tl, MoeOneArgs a) {
+    const TLStamp tls(tl);
+    constexpr int NW = WTraits<WT>::NW, CH = 64 * NW, OUT = R / 2, U = 4;
+    extern __shared__ __attribute__((aligned(16))) char smem[];
+    const int W = a.W, padded = (W + CH - 1) / CH * CH, lane = threadIdx.x & 63, wid = threadIdx.x >> 6, top = a.r.top;
+    WT* xs = reinterpret_cast<WT*>(smem);                         // [padded]
+    float* rf = reinterpret_cast<float*>(xs + padded);
+    float* wts = rf + route_floats(a.r);
+    int32_t* ids = reinterpret_cast<int32_t*>(wts + top);
+    for (int i = threadIdx.x; i < padded; i += 256) xs[i] = from_f<WT>(i < W ? a.h[i] : 0.f);
+    route_row<256>(a.r, rf, threadIdx.x, [&](int e) { return a.logits[e]; }, ids, wts, []() { __syncthreads(); });
+    if (blockIdx.x == 0)
+        for (int i = threadIdx.x; i < top; i += 256) a.ids[i] = ids[i];
+    const int total = top * a.ff;
+    for (int o = (blockIdx.x * 4 + wid) * OUT; o < total; o += gridDim.x * 4 * OUT) {
+        const int k = o / a.ff, j = o - k * a.ff;                 // (ff is a multiple of 64: all OUT outputs are one expert's)
+        const WT* w = reinterpret_cast<const WT*>(a.w_up) + (size_t)ids[k] * 2 * a.ff * W;
+        float acc[R];
+#pragma unroll
+        for (int r = 0; r < R; ++r) acc[r] = 0.f;
+        for (int c0 = 0; c0 < padded; c0 += U * CH) {
+            uint4 raw[R][U];
+#pragma unroll
+            for (int u = 0; u < U; ++u)
+#pragma unroll
+                for (int r = 0; r < R; ++r)
+                    raw[r][u] = load_nt16(w + (size_t)((r / OUT) * a.ff + j + r % OUT) * W + min(c0 + u * CH + lane * NW, W - NW));
+#pragma unroll
+            for (int u = 0; u < U; ++u) {
+                if (c0 + u * CH >= padded) break;                  // (uniform)
+                const WT* xp = xs + c0 + u * CH + lane * NW;
+#pragma unroll
+                for (int r = 0; r < R; ++r) acc[r] = dot_piece<WT>(raw[r][u], xp, acc[r]);
+            }
+        }
+#pragma unroll
+        for (int r = 0; r < R; ++r) acc[r] = wave_sum(acc[r]);
+        if (lane == 0) {
+#pragma unroll
+            for (int r = 0; r < OUT; ++r) a.act[o + r] = silu_f<std::is_same<WT, float>::value>(acc[r]) * acc[r + OUT] * wts[k];
+        }
+    }
+    tls.end();
+}
+
+// y = W_o a + sum over the chosen experts of W_down act: one row of 16-byte pieces that starts in W_o and goes on through the experts'
+template <class WT, int R>
+__global__ __launch_bounds__(256) void moe_out_one_kernel(unsigned long long* tl, MoeOneArgs a) {
+    const TLStamp tls(tl);
+    constexpr int NW = WTraits<WT>::NW, U = R >= 4 ? 4 : 8;
+    extern __shared__ __attribute__((aligned(16))) char smem[];
+    __shared__ int32_t ids[MOE_MAX_TOP];
+    WT* xs = reinterpret_cast<WT*>(smem);                         // [n_att + top ff, one piece of zeros]
+    const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6, top = a.r.top, na = a.n_att / NW, nf = a.ff / NW, np = na + top * nf, len = np * NW;
+    if ((int)threadIdx.x < top) ids[threadIdx.x] = a.ids[threadIdx.x];
+    for (int i = threadIdx.x; i < len + NW; i += 256) xs[i] = from_f<WT>(i < a.n_att ? a.a[i] : i < len ? a.act[i - a.n_att] : 0.f);
+    __syncthreads();
+    for (int n0 = (blockIdx.x * 4 + wid) * R; n0 < a.N; n0 += gridDim.x * 4 * R) {
+        float acc[R];
+#pragma unroll
+        for (int r = 0; r < R; ++r) acc[r] = 0.f;
+        for (int p0 = lane; p0 - lane < np; p0 += 64 * U) {
+            uint4 raw[U][R];
+#pragma unroll
+            for (int u = 0; u < U; ++u) {
+                const int p = min(p0 + 64 * u, np - 1), q = max(p - na, 0), k = q / (nf > 0 ? nf : 1);
+                const WT* at = p < na ? reinterpret_cast<const WT*>(a.w_o) + p * NW : reinterpret_cast<const WT*>(a.w_down) + (size_t)ids[k] * a.N * a.ff + (q - k * nf) * NW;
+                const size_t ld = p < na ? a.n_att : a.ff;
+#pragma unroll
+                for (int r = 0; r < R; ++r) raw[u][r] = load_nt16(at + min(n0 + r, a.N - 1) * ld);
+            }
+#pragma unroll
+            for (int u = 0; u < U; ++u) {
+                const WT* xp = xs + min(p0 + 64 * u, np) * NW;
+#pragma unroll
+                for (int r = 0; r < R; ++r) acc[r] = dot_piece<WT>(raw[u][r], xp, acc[r]);
+            }
+        }
+#pragma unroll
+        for (int r = 0; r < R; ++r) {
+            const float y = wave_sum(acc[r]);
+            if (lane == 0 && n0 + r < a.N) a.y[n0 + r] = y;
+        }
+    }
+    tls.end();
+}
+
+template <class T>
+static pgk_status moe_up_one(const MoeOneArgs& a, hipStream_t st) {
+    constexpr int CH = 64 * WTraits<T>::NW;
+    const size_t lds = (size_t)ceil_div(a.W, CH) * CH * sizeof(T) + (size_t)(route_floats(a.r) + 2 * a.r.top) * 4;
+    PGK_REQUIRE(lds <= 64 * 1024, "engine: a row of %d and %d experts do not fit LDS", a.W, a.r.E);
+    const int total = a.r.top * a.ff;
+    auto go = [&](auto rows) -> pgk_status {
+        constexpr int R = decltype(rows)::value;
+        const int grid = ceil_div(total, 2 * R);
+        PGK_CHECK_HIP(launch_k(&moe_up_one_kernel<T, R>, dim3(grid < 1024 ? grid : 1024), dim3(256), lds, st, a));
+        return PGK_OK;
+    };
+    return total >= 8192 ? go(std::integral_constant<int, 4>{}) : go(std::integral_constant<int, 2>{});
+}
+template <class T>
+static pgk_status moe_out_one(const MoeOneArgs& a, hipStream_t st) {
+    const size_t lds = (size_t)(a.n_att + a.r.top * a.ff + WTraits<T>::NW) * sizeof(T);
+    PGK_REQUIRE(lds <= 144 * 1024, "engine: %d mixer columns and %d experts of %d do not fit LDS", a.n_att, a.r.top, a.ff);
+    auto go = [&](auto rows) -> pgk_status {
+        constexpr int R = decltype(rows)::value;
+        auto kfn = &moe_out_one_kernel<T, R>;
+        static bool done = false;
+        if (lds > 48 * 1024 && !done) {
+            PGK_CHECK_HIP(hipFuncSetAttribute(reinterpret_cast<const void*>(kfn), hipFuncAttributeMaxDynamicSharedMemorySize, 144 * 1024));
+            done = true;
+        }
+        PGK_CHECK_HIP(launch_k(kfn, dim3(ceil_div(a.N, 4 * R)), dim3(256), lds, st, a));
+        return PGK_OK;
+    };
+    return a.N >= 4096 ? go(std::integral_constant<int, 2>{}) : go(std::integral_constant<int, 1>{});
 }
 
 // -------------------------------------------------------------------------------------------- rows (prompts, batches)
@@ -715,20 +948,30 @@ __global__ void latent_gather_kernel(const RowPlace* pl, const T* cache, T* c_al
     for (int r = threadIdx.x; r < rank; r += blockDim.x) c_all[(size_t)p.kv * rank + r] = src[r];
 }
 
-// new rows: normalise the latent part of the in-projection -> scratch row and, for the last R positions of a sequence, ring row
+// new rows: normalise (and turn) the latent part of the in-projection -> scratch row and, for the last R positions of a sequence, ring
+// row; turn the rotated columns of the queries in place
 template <class T>
-__global__ __launch_bounds__(256) void latent_rows_kernel(const RowPlace* pl, const T* in, int ld_in, int off, const float* c_norm, T* cache, T* c_all, int n,
-                                                          int R, int rank, int rank_true, float eps) {
+__global__ __launch_bounds__(256) void latent_rows_kernel(const RowPlace* pl, T* in, int ld_in, int off, const float* c_norm, T* cache, T* c_all, int n,
+                                                          int R, int rank, int rank_true, float eps, int heads, int D, int dim, int rot, const float* rot_freq) {
     const int i = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
     if (i >= n) return;
     const T* c = in + (size_t)i * ld_in + off;
     float ss = 0.f;
-    for (int r = lane; r < rank; r += 64) { const float v = to_f(c[r]); ss = fmaf(v, v, ss); }
+    for (int r = lane; r < rank_true; r += 64) { const float v = to_f(c[r]); ss = fmaf(v, v, ss); }
     const float inv = 1.0f / sqrtf(wave_sum(ss) / rank_true + eps);
     const RowPlace p = pl[i];
     T* ring = cache + ((size_t)p.slot * R + p.pos % R) * rank;
+    const int pairs = rot / 2;
+    for (int t = lane; t < heads * pairs; t += 64) {
+        T* q = in + (size_t)i * ld_in + (t / pairs) * D + dim - rot + 2 * (t % pairs);
+        float sn, cs;
+        sincosf((float)p.pos * rot_freq[t % pairs], &sn, &cs);
+        const float u = to_f(q[0]), v = to_f(q[1]);
+        q[0] = from_f<T>(fmaf(u, cs, -v * sn));
+        q[1] = from_f<T>(fmaf(v, cs, u * sn));
+    }
     for (int r = lane; r < rank; r += 64) {
-        const T v = from_f<T>(to_f(c[r]) * inv * c_norm[r]);
+        const T v = from_f<T>(r >= rank_true && r < rank_true + rot ? rotated(c + rank_true, r - rank_true, p.pos, rot_freq) : to_f(c[r]) * inv * c_norm[r]);
         c_all[(size_t)p.kv * rank + r] = v;
         if (p.store) ring[r] = v;
     }
@@ -761,13 +1004,20 @@ __global__ __launch_bounds__(256) void rows_argmax_kernel(unsigned long long* tl
 }
 
 // -------------------------------------------------------------------------------------------- engine state
+static RouterCfg router_of(const pgk_stack_layer_t& L) { return RouterCfg{L.correction, L.experts, L.top, L.groups, L.keep, L.router_scale}; }
+static int router_rows(const pgk_stack_layer_t& L) { return L.ff_pad && L.ff == PGK_FF_MOE ? ceil_div(L.experts, 64) * 64 : 0; }
+struct Run { int layer, pass; };          // one pass of one layer; pass >= 0: the loop's pass `pass` starts with it
+
 struct Stack {
     pgk_stack_config_t cfg;
     std::vector<pgk_stack_layer_t> layers;
+    std::vector<Run> runs;                 // in the order they are run; without a loop run i is layer i
+    int n_runs() const { return (int)runs.size(); }
+    const pgk_stack_layer_t& at(int run) const { return layers[runs[run].layer]; }
     const void *embed = nullptr, *pos = nullptr, *head = nullptr;
     const float* final_norm = nullptr;
-    int Wp = 0, max_in = 0, max_att = 0, max_ff = 0, max_q = 0;
-    // per layer: latent rows [max_batch][R][rank] or K/V rows [max_batch][k, v][kv heads][R][head width] (a layer that takes another
+    int Wp = 0, max_in = 0, max_att = 0, max_ff = 0, max_q = 0, max_top = 0, max_conv = 0, max_z = 0, max_gate = 0, max_low = 0;
+    // per run: latent rows [max_batch][R][rank] or K/V rows [max_batch][k, v][kv heads][R][head width] (a layer that takes another
     // one's: that one's pointer) or recurrent states [max_batch][heads][dim][vdim] in fp32
     std::vector<void*> cache;
     std::vector<int> ring, reach;          // R; keys the cache has to keep (the largest window of the layers that read it).  0: no ring
@@ -777,10 +1027,19 @@ struct Stack {
     float *in32 = nullptr, *a32 = nullptr, *y32 = nullptr, *act32 = nullptr, *po = nullptr, *pml = nullptr;
     void *qlat = nullptr, *qx = nullptr, *x16 = nullptr, *in16 = nullptr, *a16 = nullptr, *y16 = nullptr, *gu16 = nullptr, *act16 = nullptr;
     float* slabs16 = nullptr;              // split-K slabs of a batch step's projections
+    float *y32b = nullptr, *h32 = nullptr, *z32 = nullptr;                          // one row: input of a pass, normed row; rows: decay projections
+    int32_t* ids = nullptr;
+    void *gate = nullptr, *cat16 = nullptr, *e16 = nullptr, *moe16 = nullptr;       // rows: gates, [x | embedding], experts' rows and workspace
     // fragment-major copies of the layer matrices for 2..128 rows (ops_pkgemm.hip), where its shapes allow; null entries: row-major kernels
     struct Packed { bf16 *in = nullptr, *o = nullptr, *gate_up = nullptr, *down = nullptr; };
     std::vector<Packed> packed;
     size_t slab_elems(int n, bool f32) const;   // fp32 elements the projections of n rows may need
+    size_t moe_ws(int n) const {           // workspace of the experts for n rows
+        size_t m = 0;
+        for (const auto& L : layers)
+            if (router_rows(L)) { const size_t z = moe_bytes(n, Wp, L.ff_pad, router_of(L), cfg.dtype); m = z > m ? z : m; }
+        return m;
+    }
     // prompt buffers, grown on demand outside capture
     void* pf = nullptr; size_t pf_bytes = 0;
     void* tab = nullptr; size_t tab_bytes = 0;
@@ -788,6 +1047,13 @@ struct Stack {
 };
 static Stack* stack_of(const Engine* e) { return (Stack*)e->kind_state; }
 static int kv_source(const pgk_stack_layer_t& L, int l) { return L.kv_from >= 0 ? L.kv_from : l; }
+static bool recurrent(const pgk_stack_layer_t& L) { return L.mixer == PGK_MIX_HGRN2 || L.mixer == PGK_MIX_DELTA || L.mixer == PGK_MIX_SSD; }
+// channels that pass taps over time before a recurrence, and where the delta rule's projections stand in a row
+static int conv_channels(const pgk_stack_layer_t& L) {
+    const int V = L.heads * L.vhead_pad, G = L.kv_heads * L.head_pad;
+    return L.mixer == PGK_MIX_DELTA || L.mixer == PGK_MIX_SSD ? V + 2 * G : 0;
+}
+static int delta_a_off(const pgk_stack_layer_t& L) { return ceil_div(conv_channels(L) + L.heads, 64) * 64; }
 static int up_rows(const pgk_stack_layer_t& L) { return (L.ff == PGK_FF_SWIGLU ? 2 : 1) * L.ff_pad; }     // rows of the first feed-forward matrix
 
 static int pick_nsplit(const Engine* e, int B, const pgk_stack_layer_t& L, int R) {
@@ -834,10 +1100,10 @@ static hipError_t launch_absorb(const LatentArgs& a, hipStream_t st) {
 template <class T, class IT>
 static pgk_status latent_decode(Engine* e, int l, int B, const void* in, void* out, hipStream_t st, int* launches) {
     Stack* s = stack_of(e);
-    const auto& L = s->layers[l];
+    const auto& L = s->at(l);
     constexpr bool F32 = std::is_same<T, float>::value;
     LatentArgs a{};
-    a.in = in; a.ld_in = L.n_in; a.qn = L.heads * L.head_pad; a.g_off = a.qn + L.rank_pad;
+    a.in = in; a.ld_in = L.n_in; a.qn = L.heads * L.head_pad; a.g_off = L.gated ? a.qn + L.rank_pad : -1; a.rot = L.rot; a.rot_freq = L.rot_freq;
     a.w_uk = L.w_ukv; a.w_uv = (const char*)L.w_ukv + (size_t)L.heads * L.head_pad * L.rank_pad * sizeof(T);
     a.c_norm = L.c_norm; a.cache = s->cache[l]; a.positions = e->positions;
     a.B = B; a.H = L.heads; a.D = L.head_pad; a.dim = L.dim; a.vdim = L.vdim; a.rank = L.rank_pad; a.rank_true = L.rank; a.R = s->ring[l];
@@ -878,7 +1144,7 @@ static pgk_status latent_decode(Engine* e, int l, int B, const void* in, void* o
 template <class T, class IT>
 static pgk_status attention_decode(Engine* e, int l, int B, const void* in, void* out, hipStream_t st, int* launches) {
     Stack* s = stack_of(e);
-    const auto& L = s->layers[l];
+    const auto& L = s->at(l);
     const int src = kv_source(L, l), HD = L.heads * L.head_pad, GD = L.kv_from >= 0 ? 0 : L.kv_heads * L.head_pad;
     constexpr pgk_dtype DT = std::is_same<T, float>::value ? PGK_F32 : PGK_BF16;
     constexpr bool IO32 = std::is_same<IT, float>::value;
@@ -897,11 +1163,34 @@ static pgk_status attention_decode(Engine* e, int l, int B, const void* in, void
 }
 
 static RecurArgs recur_args(const Stack* s, int l, const void* in, void* out, int n) {
-    const auto& L = s->layers[l];
+    const auto& L = s->at(l);
     RecurArgs a{};
-    a.in = in; a.ld_in = L.n_in; a.f_off = L.heads * L.head_pad; a.v_off = 2 * a.f_off;
+    a.in = in; a.ld_in = L.n_in; a.H = L.heads; a.dim = L.head_pad; a.vdim = L.vhead_pad; a.vdim_true = L.vdim; a.n = n; a.eps = s->cfg.norm_eps;
+    a.state = (float*)s->cache[l]; a.out = out; a.ld_out = L.n_att;
+    if (L.mixer == PGK_MIX_SSD) {          // x | B | C | z | dt; the norm in parts is a launch of its own
+        const int V = L.heads * L.vhead_pad, G = L.kv_heads * L.head_pad;
+        a.kind = RECUR_SSD; a.G = L.kv_heads; a.f_off = V; a.q_off = V + G; a.z_off = V + 2 * G; a.dt_off = a.z_off + V;
+        a.dt_bias = L.dt_bias; a.decay = L.decay; a.skip = L.skip;
+        a.conv = ConvStep{L.conv, L.conv_bias, L.taps, conv_channels(L), s->taps[l]};
+        return a;
+    }
+    a.f_off = L.heads * L.head_pad; a.v_off = 2 * a.f_off;
     a.bias = L.b_in ? L.b_in + a.f_off : nullptr; a.lower = L.lower; a.norm = L.o_norm;
-    a.H = L.heads; a.dim = L.head_pad; a.vdim = L.vhead_pad; a.vdim_true = L.vdim; a.n = n; a.eps = s->cfg.norm_eps;
+    return a;
+}
+static pgk_status ssd_norm(const Stack* s, int l, void* rows, int n, pgk_dtype dt, hipStream_t st) {
+    const auto& L = s->at(l);
+    return parts_norm(rows, L.n_att, n, L.heads, L.vhead_pad, L.vdim, L.norm_parts, L.o_norm, s->cfg.norm_eps, dt, st);
+}
+
+static DeltaArgs delta_args(const Stack* s, int l, const void* in, const float* z, const void* gate, void* out, int n) {
+    const auto& L = s->at(l);
+    DeltaArgs a{};
+    a.in = in; a.ld_in = L.n_in; a.b_off = conv_channels(L);
+    a.z = z; a.ld_z = L.heads * L.head_pad; a.gate = gate; a.ld_gate = L.heads * L.vhead_pad;
+    a.conv = ConvStep{L.conv, nullptr, L.taps, conv_channels(L), s->taps[l]};
+    a.decay = L.decay; a.dt_bias = L.dt_bias; a.norm = L.o_norm;
+    a.H = L.heads; a.G = L.kv_heads; a.dim = L.head_pad; a.vdim = L.vhead_pad; a.dim_true = L.dim; a.vdim_true = L.vdim; a.n = n; a.eps = s->cfg.norm_eps;
     a.state = (float*)s->cache[l]; a.out = out; a.ld_out = L.n_att;
     return a;
 }
@@ -910,16 +1199,96 @@ static RecurArgs recur_args(const Stack* s, int l, const void* in, void* out, in
 template <class T, class IT>
 static pgk_status mix_decode(Engine* e, int l, int B, const void* in, void* out, hipStream_t st, int* launches) {
     Stack* s = stack_of(e);
-    switch (s->layers[l].mixer) {
+    const auto& L = s->at(l);
+    constexpr pgk_dtype DT = std::is_same<T, float>::value ? PGK_F32 : PGK_BF16, IDT = std::is_same<IT, float>::value ? PGK_F32 : PGK_BF16;
+    constexpr bool IO32 = std::is_same<IT, float>::value;
+    switch (L.mixer) {
         case PGK_MIX_LATENT: return latent_decode<T, IT>(e, l, B, in, out, st, launches);
         case PGK_MIX_ATTENTION: return attention_decode<T, IT>(e, l, B, in, out, st, launches);
+        case PGK_MIX_DELTA: {
+            const int a_off = delta_a_off(L);
+            if (pgk_status r = lowrank_rows(in, L.n_in, B, a_off, L.rank_a, L.w_a2, s->z32, L.heads * L.head_pad, a_off + L.rank_a, L.rank_g, L.w_g2, s->gate, L.heads * L.vhead_pad,
+                                            DT, IO32, st))
+                return r;
+            DeltaArgs a = delta_args(s, l, in, s->z32, s->gate, out, B);
+            a.positions = e->positions;
+            *launches += 2;
+            return delta_rows(a, DT, IO32, st);
+        }
         default: {
             RecurArgs a = recur_args(s, l, in, out, B);
             a.positions = e->positions;
             *launches += 1;
-            return recur_rows(a, std::is_same<T, float>::value ? PGK_F32 : PGK_BF16, std::is_same<IT, float>::value, st);
+            if (pgk_status r = recur_rows(a, DT, IO32, st)) return r;
+            if (L.mixer != PGK_MIX_SSD) return PGK_OK;
+            *launches += 1;
+            return ssd_norm(s, l, out, B, IDT, st);
         }
     }
+}
+
+// Parallel layers, one sequence
+template <class T>
+static pgk_status step_parallel(Engine* e, hipStream_t st, int* launches) {
+    Stack* s = stack_of(e);
+    const auto& c = s->cfg;
+    float *x = e->h, *xn = e->h2;
+    const float *pend = nullptr, *base = nullptr;      // what is still to be added to the stream (or to the vector that takes its place)
+    auto input = [&](StackGemvArgs& a, int K) {
+        a.K = K; a.W = c.width; a.x = x; a.eps = c.norm_eps; a.mult = base ? 1.f : c.residual_mult; a.y = pend; a.base = base;
+    };
+    auto norm_in = [&](StackGemvArgs& a, const float* gamma) {
+        input(a, s->Wp);
+        a.gamma = gamma; a.layer_norm = c.layer_norm;
+        a.x_out = pend ? xn : nullptr;
+    };
+    for (int l = 0; l < s->n_runs(); ++l) {
+        const auto& L = s->at(l);
+        const int er = router_rows(L);
+        StackGemvArgs a{};
+        mark(KC_NORM_QKV);
+        if (s->runs[l].pass >= 0) {
+            input(a, 2 * s->Wp);
+            a.embed = s->embed; a.tok = e->tokens; a.w = c.loop_in; a.N = s->Wp; a.out = s->y32b;
+            if (pgk_status r = stack_gemv<T, SP_CAT, SE_STORE>(a, st)) return r;
+            pend = s->y32b;
+            base = c.loop_step + (size_t)s->runs[l].pass * s->Wp;
+            *launches += 1;
+            a = StackGemvArgs{};
+        }
+        norm_in(a, L.norm1);
+        a.h_out = er ? s->h32 : nullptr;
+        a.w = L.w_in; a.N = L.n_in + er; a.out = s->in32;
+        if (pgk_status r = stack_gemv<T, SP_ADD, SE_STORE>(a, st)) return r;
+        if (pend) { float* t = x; x = xn; xn = t; }
+        mark(recurrent(L) ? KC_RECUR : KC_ATTN);
+        if (pgk_status r = mix_decode<T, float>(e, l, 1, s->in32, s->a32, st, launches)) return r;
+        MoeOneArgs m{};
+        m.r = router_of(L); m.W = s->Wp; m.ff = L.ff_pad; m.logits = s->in32 + L.n_in; m.h = s->h32; m.w_up = L.w_gate_up; m.w_down = L.w_down; m.act = s->act32; m.ids = s->ids;
+        m.w_o = L.w_o; m.a = s->a32; m.n_att = L.n_att; m.y = s->y32; m.N = s->Wp;
+        if (er) {
+            mark(KC_GATEUP);
+            if (pgk_status r = moe_up_one<T>(m, st)) return r;
+            mark(KC_DOWN);
+            if (pgk_status r = moe_out_one<T>(m, st)) return r;
+            *launches += 1;
+        } else {
+            mark(KC_OPROJ);
+            a = StackGemvArgs{};
+            a.w = L.w_o; a.N = s->Wp; a.K = L.n_att; a.x = s->a32; a.out = s->y32;
+            if (pgk_status r = stack_gemv<T, SP_PLAIN, SE_STORE>(a, st)) return r;
+        }
+        pend = s->y32; base = nullptr;
+        *launches += 2;
+    }
+    mark(KC_LMHEAD);
+    StackGemvArgs a{};
+    norm_in(a, s->final_norm);
+    a.x_out = nullptr;
+    a.w = s->head; a.N = c.vocab_size; a.out = e->logits; a.amax_val = e->amax_val; a.amax_idx = e->amax_idx;
+    if (pgk_status r = stack_gemv<T, SP_ADD, SE_LOGITS>(a, st, e->lm_blocks)) return r;
+    *launches += 1;
+    return PGK_OK;
 }
 
 // ---- one sequence: fused steps, fp32 between kernels ----
@@ -942,7 +1311,7 @@ static pgk_status step_one(Engine* e, hipStream_t st, int* launches) {
         a.w = L.w_in; a.N = L.n_in; a.out = s->in32;
         if (pgk_status r = stack_gemv<T, SP_NORM, SE_STORE>(a, st)) return r;
         settle();
-        mark(L.mixer == PGK_MIX_HGRN2 ? KC_RECUR : KC_ATTN);
+        mark(recurrent(L) ? KC_RECUR : KC_ATTN);
         if (pgk_status r = mix_decode<T, float>(e, l, 1, s->in32, s->a32, st, launches)) return r;
         mark(KC_OPROJ);
         a = StackGemvArgs{};
@@ -987,7 +1356,10 @@ static pgk_status head_rows(Stack* s, const T* x, float* logits, int n, hipStrea
     return PGK_OK;
 }
 
-struct RowBufs { float* h; void *x, *in, *a, *y, *gu, *act; float* slabs; void* q; };
+struct RowBufs {
+    float* h; void *x, *in, *a, *y, *gu, *act; float* slabs; void* q;
+    void *cat, *e, *moe; const int32_t* tok;      // parallel layers: [x | embedding] rows, experts' rows, their workspace, the rows' tokens
+};
 
 // How a [N, K] projection of n bf16 rows runs: fragment-major copy (<= 128 rows), weight-streaming kernel (<= 128 rows) or tiled
 // MFMA, and over how many split-K slabs its result is left (0: one bf16 result).
@@ -1001,14 +1373,21 @@ static ProjPlan plan_proj(const bf16* packed, int n, int N, int K, bool split) {
     const int s = split ? engine_gemm_pick_splits(n, N, K) : 1;
     return {false, s > 1 ? s : 0};
 }
+// fp32 results of n bf16 rows, as one or more slabs
+static int plan_f32(int n, int N, int K) { return n <= 128 ? wsgemm_pick_splits(N, K, true) : engine_gemm_pick_splits(n, N, K); }
+static pgk_status gemm_f32(const void* x, const void* w, float* out, int splits, int n, int N, int K, hipStream_t st) {
+    if (n <= 128) return wsgemm_nt((const bf16*)x, K, w, nullptr, false, out, nullptr, 1, splits, n, N, K, st);
+    return engine_gemm_nt_slabs((const bf16*)x, w, out, splits, n, N, K, st);
+}
 size_t Stack::slab_elems(int n, bool f32) const {
     size_t m = 64;
     if (f32) return m;
+    if (cfg.loop_times) m = (size_t)plan_f32(n, Wp, 2 * Wp) * n * Wp;
     for (size_t l = 0; l < layers.size(); ++l) {
         const auto& L = layers[l];
         const Packed P = packed.empty() ? Packed{} : packed[l];
         const size_t need[] = {(size_t)plan_proj(P.o, n, Wp, L.n_att, true).slabs * n * Wp,
-                               L.ff_pad ? (size_t)plan_proj(P.down, n, Wp, L.ff_pad, true).slabs * n * Wp : 0,
+                               L.ff_pad && L.ff != PGK_FF_MOE ? (size_t)plan_proj(P.down, n, Wp, L.ff_pad, true).slabs * n * Wp : 0,
                                P.in || n > 128 ? 0 : (size_t)plan_proj(nullptr, n, L.n_in, Wp, true).slabs * n * L.n_in};
         for (size_t z : need) m = z > m ? z : m;
     }
@@ -1098,7 +1477,7 @@ static pgk_status rows_layers(Stack* s, const RowBufs& b, int n, hipStream_t st,
         mark(KC_NORM_QKV);
         if (pgk_status r = rows_norm(norm_args(s, b, n, *pend, L.norm1, b.x), n, DT, st)) return r;
         if (pgk_status r = rows_in_proj<T>(s, L, P.in, b, n, st)) return r;
-        mark(L.mixer == PGK_MIX_HGRN2 ? KC_RECUR : KC_ATTN);
+        mark(recurrent(L) ? KC_RECUR : KC_ATTN);
         if (pgk_status r = mix(l)) return r;
         mark(KC_OPROJ);
         if (pgk_status r = rows_out_proj<T>(s, b, b.a, L.w_o, P.o, n, L.n_att, &pend->slabs, st)) return r;
@@ -1114,6 +1493,73 @@ static pgk_status rows_layers(Stack* s, const RowBufs& b, int n, hipStream_t st,
     return PGK_OK;
 }
 
+// Parallel layers: what is still to be added to the stream, y rows (or slabs) on the stream or on `base`, and the experts' rows
+struct PendingAdd { bool y = false; int slabs = 0, top = 0; const float* base = nullptr; };
+
+static RowsNormArgs add_args(const Stack* s, const RowBufs& b, int n, const PendingAdd& p, const float* gamma, void* out) {
+    RowsNormArgs a{};
+    a.plain = 1; a.layer_norm = s->cfg.layer_norm;
+    a.h = b.h; a.y = !p.y ? nullptr : p.slabs ? (const void*)b.slabs : b.y; a.ldy = s->Wp; a.mult = p.base ? 1.f : s->cfg.residual_mult;
+    a.gamma = gamma; a.out = out; a.W = s->cfg.width; a.ld = s->Wp; a.eps = s->cfg.norm_eps; a.store_h = p.y;
+    a.nslabs = p.y ? p.slabs : 0; a.slab_stride = (long long)n * s->Wp;
+    a.base = p.base; a.e = p.top ? b.e : nullptr; a.e_top = p.top;
+    return a;
+}
+
+template <class T, class Mix>
+static pgk_status rows_parallel(Stack* s, const RowBufs& b, int n, hipStream_t st, PendingAdd* pend, Mix mix) {
+    constexpr pgk_dtype DT = std::is_same<T, float>::value ? PGK_F32 : PGK_BF16;
+    const auto& c = s->cfg;
+    *pend = PendingAdd{};
+    for (int l = 0; l < s->n_runs(); ++l) {
+        const auto& L = s->at(l);
+        const Stack::Packed P = s->packed.empty() ? Stack::Packed{} : s->packed[s->runs[l].layer];
+        mark(KC_NORM_QKV);
+        if (s->runs[l].pass >= 0) {
+            RowsNormArgs a = add_args(s, b, n, *pend, nullptr, b.cat);
+            a.embed = s->embed; a.tok = b.tok; a.store_h = 0;      // (`base` takes the stream's place)
+            if (pgk_status r = rows_norm(a, n, DT, st)) return r;
+            *pend = PendingAdd{};
+            pend->y = true;
+            pend->base = c.loop_step + (size_t)s->runs[l].pass * s->Wp;
+            if (DT == PGK_F32) { if (pgk_status r = pgk_gemm_nt(b.cat, c.loop_in, nullptr, b.y, n, s->Wp, 2 * s->Wp, PGK_F32, st)) return r; }
+            else {
+                pend->slabs = plan_f32(n, s->Wp, 2 * s->Wp);
+                if (pgk_status r = gemm_f32(b.cat, c.loop_in, b.slabs, pend->slabs, n, s->Wp, 2 * s->Wp, st)) return r;
+            }
+        }
+        if (pgk_status r = rows_norm(add_args(s, b, n, *pend, L.norm1, b.x), n, DT, st)) return r;
+        *pend = PendingAdd{};
+        if (pgk_status r = rows_in_proj<T>(s, L, P.in, b, n, st)) return r;
+        mark(recurrent(L) ? KC_RECUR : KC_ATTN);
+        if (pgk_status r = mix(l)) return r;
+        mark(KC_OPROJ);
+        if (pgk_status r = rows_out_proj<T>(s, b, b.a, L.w_o, P.o, n, L.n_att, &pend->slabs, st)) return r;
+        pend->y = true;
+        if (!L.ff_pad) continue;
+        mark(KC_GATEUP);
+        MoeArgs m{b.x, n, s->Wp, L.ff_pad, router_of(L), (const T*)L.w_in + (size_t)L.n_in * s->Wp, L.w_gate_up, L.w_down, b.e, b.moe};
+        if (pgk_status r = moe_rows(m, DT, st)) return r;
+        pend->top = L.top;
+    }
+    return PGK_OK;
+}
+
+// All layers on n rows of b.h (embedded tokens); `last`: the launch of rows_norm that completes the stream and leaves normed rows in b.x
+template <class T, class Mix>
+static pgk_status rows_model(Stack* s, const RowBufs& b, int n, hipStream_t st, Mix mix, RowsNormArgs* last) {
+    if (s->cfg.block == PGK_BLOCK_PARALLEL) {
+        PendingAdd p;
+        if (pgk_status r = rows_parallel<T>(s, b, n, st, &p, mix)) return r;
+        *last = add_args(s, b, n, p, s->final_norm, b.x);
+        return PGK_OK;
+    }
+    Pending p;
+    if (pgk_status r = rows_layers<T>(s, b, n, st, &p, mix)) return r;
+    *last = norm_args(s, b, n, p, s->final_norm, b.x);
+    return PGK_OK;
+}
+
 constexpr int ROWS_ARGMAX_BLOCKS = 64;
 
 template <class T>
@@ -1121,15 +1567,15 @@ static pgk_status step_rows(Engine* e, int B, hipStream_t st, int* launches) {
     Stack* s = stack_of(e);
     constexpr pgk_dtype DT = std::is_same<T, float>::value ? PGK_F32 : PGK_BF16;
     const auto& c = s->cfg;
-    const RowBufs b{e->h, s->x16, s->in16, s->a16, s->y16, s->gu16, s->act16, s->slabs16, nullptr};
-    Pending pend;
-    if (pgk_status r = rows_layers<T>(s, b, B, st, &pend, [&](int l) { return mix_decode<T, T>(e, l, B, b.in, b.a, st, launches); })) return r;
+    const RowBufs b{e->h, s->x16, s->in16, s->a16, s->y16, s->gu16, s->act16, s->slabs16, nullptr, s->cat16, s->e16, s->moe16, e->tokens};
+    RowsNormArgs last;
+    if (pgk_status r = rows_model<T>(s, b, B, st, [&](int l) { return mix_decode<T, T>(e, l, B, b.in, b.a, st, launches); }, &last)) return r;
     mark(KC_LMHEAD);
-    if (pgk_status r = rows_norm(norm_args(s, b, B, pend, s->final_norm, b.x), B, DT, st)) return r;
+    if (pgk_status r = rows_norm(last, B, DT, st)) return r;
     if (pgk_status r = head_rows<T>(s, (const T*)b.x, e->logits, B, st)) return r;
     PGK_CHECK_HIP(launch_k(rows_argmax_kernel, dim3(ROWS_ARGMAX_BLOCKS, B), dim3(256), 0, st, e->logits, c.vocab_size, e->amax_val, e->amax_idx));
     *launches += 3;
-    for (const auto& L : s->layers) *launches += 3 + (L.ff_pad ? 3 : 0);     // (one more where a projection's slabs or SwiGLU take a launch of their own)
+    for (const auto& r : s->runs) *launches += 3 + (s->layers[r.layer].ff_pad ? 3 : 0);     // (one more where a projection's slabs or SwiGLU take a launch of their own)
     return PGK_OK;
 }
 
@@ -1139,7 +1585,7 @@ static pgk_status stack_step(Engine* e, int batch, hipStream_t st, int* launches
     int nblk = ROWS_ARGMAX_BLOCKS;
     if (batch == 1) {
         nblk = e->lm_blocks;
-        if (pgk_status r = step_one<T>(e, st, launches)) return r;
+        if (pgk_status r = s->cfg.block == PGK_BLOCK_PARALLEL ? step_parallel<T>(e, st, launches) : step_one<T>(e, st, launches)) return r;
     } else if (pgk_status r = step_rows<T>(e, batch, st, launches)) return r;
     mark(KC_ARGMAX);
     const int32_t* sampled = nullptr;
@@ -1175,9 +1621,9 @@ static pgk_status check_position(const Engine* e, int slot, int pos) {
     const int len = s->len[slot];
     PGK_REQUIRE(pos <= len, "engine: slot %d holds %d positions, cannot go on at position %d", slot, len, pos);
     if (pos == 0 || pos == len) return PGK_OK;
-    for (int l = 0; l < s->cfg.num_layers; ++l) {
-        const auto& L = s->layers[l];
-        PGK_REQUIRE(L.mixer != PGK_MIX_HGRN2, "engine: slot %d has moved on to position %d; its recurrent state cannot go back to position %d", slot, len, pos);
+    for (int l = 0; l < s->n_runs(); ++l) {
+        const auto& L = s->at(l);
+        PGK_REQUIRE(!recurrent(L), "engine: slot %d has moved on to position %d; its recurrent state cannot go back to position %d", slot, len, pos);
         auto kept = [&](int back, int R) { return (pos - back > 0 ? pos - back : 0) + R >= len; };
         PGK_REQUIRE(kept(L.window - 1, s->ring[kv_source(L, l)]) && (L.mixer != PGK_MIX_ATTENTION || !L.conv || kept(L.taps - 1, L.taps)),
                     "engine: slot %d has moved on to position %d; the window of position %d is no longer in its ring", slot, len, pos);
@@ -1208,12 +1654,13 @@ static pgk_status stack_prefill_t(Engine* e, int n_seqs, const int32_t* slots, c
     for (int i = 0; i < n_seqs; ++i) n += lens[i];
     // per layer with a ring: which cached rows a sequence's queries reach (its own and up to reach - 1 before them)
     struct LayerRows { size_t past0 = 0; int n_past = 0, n_kv = 0; };
-    std::vector<LayerRows> lr(c.num_layers);
+    const int n_runs = s->n_runs();
+    std::vector<LayerRows> lr(n_runs);
     std::vector<RowPlace> place;                        // per layer: n_past gathered rows, then n new rows (equal layers share them)
-    std::vector<int> share(c.num_layers, -1);
+    std::vector<int> share(n_runs, -1);
     int max_kv = 0;
     auto past_of = [&](int l, int i) { return starts[i] < s->reach[l] - 1 ? starts[i] : s->reach[l] - 1; };
-    for (int l = 0; l < c.num_layers; ++l) {
+    for (int l = 0; l < n_runs; ++l) {
         if (!s->reach[l]) continue;
         for (int k = 0; k < l && share[l] < 0; ++k)
             if (share[k] < 0 && s->ring[k] == s->ring[l] && s->reach[k] == s->reach[l]) share[l] = k;
@@ -1233,11 +1680,11 @@ static pgk_status stack_prefill_t(Engine* e, int n_seqs, const int32_t* slots, c
     }
     // K/V scratch: one region that the layers use in turn, and one of its own for every layer whose keys others take
     size_t kv_elems = 0, c_elems = 0, own_elems = 0;
-    std::vector<size_t> own(c.num_layers, 0);           // 1 + offset
-    for (int l = 0; l < c.num_layers; ++l)
-        if (s->layers[l].kv_from >= 0) own[s->layers[l].kv_from] = 1;
-    for (int l = 0; l < c.num_layers; ++l) {
-        const auto& L = s->layers[l];
+    std::vector<size_t> own(n_runs, 0);           // 1 + offset
+    for (int l = 0; l < n_runs; ++l)
+        if (s->at(l).kv_from >= 0) own[s->at(l).kv_from] = 1;
+    for (int l = 0; l < n_runs; ++l) {
+        const auto& L = s->at(l);
         if (!s->reach[l]) continue;
         const size_t ke = (size_t)lr[l].n_kv * 2 * L.kv_heads * L.head_pad, ce = (size_t)lr[l].n_kv * L.rank_pad;
         if (own[l]) { own[l] = 1 + own_elems; own_elems += (ke + 127) & ~(size_t)127; }
@@ -1249,11 +1696,11 @@ static pgk_status stack_prefill_t(Engine* e, int n_seqs, const int32_t* slots, c
     for (int i = 0; i < n_seqs; ++i) longest = lens[i] > longest ? lens[i] : longest;
     struct Chunks { int rows = 0; std::vector<RecurChunk> list; std::vector<int32_t> of_seq; size_t o_list = 0, o_seq = 0; };
     std::vector<Chunks> chunkings;
-    std::vector<int> chunking(c.num_layers, -1);
+    std::vector<int> chunking(n_runs, -1);
     size_t chunk_ws = 0, chunk_tab = 0;
-    for (int l = 0; l < c.num_layers; ++l) {
-        const auto& L = s->layers[l];
-        const int C = L.mixer == PGK_MIX_HGRN2 && longest >= RECUR_CHUNKED_FROM ? recur_chunk_rows(L.head_pad, L.vhead_pad) : 0;
+    for (int l = 0; l < n_runs; ++l) {
+        const auto& L = s->at(l);
+        const int C = !recurrent(L) || longest < RECUR_CHUNKED_FROM ? 0 : L.mixer != PGK_MIX_DELTA ? recur_chunk_rows(L.head_pad, L.vhead_pad) : delta_chunk_ok(L.head_pad, L.vhead_pad) ? DELTA_CHUNK : 0;
         if (!C) continue;
         for (size_t k = 0; k < chunkings.size(); ++k) if (chunkings[k].rows == C) chunking[l] = (int)k;
         if (chunking[l] < 0) {
@@ -1267,7 +1714,8 @@ static pgk_status stack_prefill_t(Engine* e, int n_seqs, const int32_t* slots, c
             chunking[l] = (int)chunkings.size();
             chunkings.push_back(t);
         }
-        const size_t need = recur_chunk_bytes(recur_args(s, l, nullptr, nullptr, n), (int)chunkings[chunking[l]].list.size());
+        const int n_chunks = (int)chunkings[chunking[l]].list.size();
+        const size_t need = L.mixer == PGK_MIX_DELTA ? delta_chunk_bytes(delta_args(s, l, nullptr, nullptr, nullptr, nullptr, n), n_chunks) : recur_chunk_bytes(recur_args(s, l, nullptr, nullptr, n), n_chunks);
         if (need > chunk_ws) chunk_ws = need;
     }
     const int wrows = n_want < 128 ? n_want : 128;
@@ -1275,7 +1723,8 @@ static pgk_status stack_prefill_t(Engine* e, int n_seqs, const int32_t* slots, c
     const size_t E = sizeof(T);
     const size_t sizes[] = {(size_t)n * s->Wp * 4, (size_t)n * s->Wp * E, (size_t)n * s->max_in * E, (size_t)n * s->max_att * E, (size_t)n * s->Wp * E,
                             (size_t)n * 2 * s->max_ff * E, (size_t)n * s->max_ff * E, c_elems * E, kv_elems * E, (size_t)wrows * s->Wp * E, (size_t)wrows * c.vocab_size * 4,
-                            s->slab_elems(n, DT == PGK_F32) * 4, (size_t)n * s->max_q * E, own_elems * E, chunk_ws};
+                            s->slab_elems(n, DT == PGK_F32) * 4, (size_t)n * s->max_q * E, own_elems * E, chunk_ws, (size_t)n * s->max_conv * E, (size_t)n * s->max_z * 4,
+                            (size_t)n * s->max_gate * E, (size_t)n * s->max_low * E, c.loop_times ? (size_t)n * 2 * s->Wp * E : 0, (size_t)n * s->max_top * s->Wp * E, s->moe_ws(n)};
     for (auto& t : chunkings) {
         t.o_list = chunk_tab;
         t.o_seq = t.o_list + up(t.list.size() * sizeof(RecurChunk));
@@ -1308,6 +1757,10 @@ static pgk_status stack_prefill_t(Engine* e, int n_seqs, const int32_t* slots, c
     b.q = take(sizes[12]);
     T* kv_own = (T*)take(sizes[13]);
     void* ws_chunk = take(sizes[14]);
+    void* conv_rows_buf = take(sizes[15]);
+    float* z_rows = (float*)take(sizes[16]);
+    void *gate_rows = take(sizes[17]), *low_rows = take(sizes[18]);
+    b.cat = take(sizes[19]); b.e = take(sizes[20]); b.moe = take(sizes[21]);
     // one host image of the index tables, one copy
     std::vector<char> img(tab_need, 0);
     const size_t o_pos = up((size_t)n * 4), o_place = 2 * o_pos, o_want = o_place + up(place.size() * sizeof(RowPlace)),
@@ -1329,6 +1782,7 @@ static pgk_status stack_prefill_t(Engine* e, int n_seqs, const int32_t* slots, c
     PGK_CHECK_HIP(hipMemcpyAsync(s->tab, img.data(), tab_need, hipMemcpyHostToDevice, st));
     PGK_CHECK_HIP(hipStreamSynchronize(st));      // the image is pageable host memory
     const int32_t* d_tok = (const int32_t*)s->tab;
+    b.tok = d_tok;
     const int32_t* d_pos = (const int32_t*)((char*)s->tab + o_pos);
     const RowPlace* d_place = (const RowPlace*)((char*)s->tab + o_place);
     const int32_t* d_want = (const int32_t*)((char*)s->tab + o_want);
@@ -1337,15 +1791,15 @@ static pgk_status stack_prefill_t(Engine* e, int n_seqs, const int32_t* slots, c
     stack_embed_kernel<T><<<n, 256, 0, st>>>((const T*)s->embed, (const T*)s->pos, d_tok, d_pos, b.h, c.width, s->Wp, c.max_positions);
     PGK_LAUNCH_CHECK();
     auto latent = [&](int l) -> pgk_status {
-        const auto& L = s->layers[l];
+        const auto& L = s->at(l);
         const LayerRows& w = lr[l];
         const int HD = L.heads * L.head_pad, R = s->ring[l];
         if (w.n_past) {
             latent_gather_kernel<T><<<w.n_past, 64, 0, st>>>(d_place + w.past0, (const T*)s->cache[l], c_all, R, L.rank_pad);
             PGK_LAUNCH_CHECK();
         }
-        latent_rows_kernel<T><<<ceil_div(n, 4), 256, 0, st>>>(d_place + w.past0 + w.n_past, (const T*)b.in, L.n_in, HD, L.c_norm, (T*)s->cache[l], c_all, n, R,
-                                                              L.rank_pad, L.rank, c.norm_eps);
+        latent_rows_kernel<T><<<ceil_div(n, 4), 256, 0, st>>>(d_place + w.past0 + w.n_past, (T*)b.in, L.n_in, HD, L.c_norm, (T*)s->cache[l], c_all, n, R,
+                                                              L.rank_pad, L.rank, c.norm_eps, L.heads, L.head_pad, L.dim, L.rot, L.rot_freq);
         PGK_LAUNCH_CHECK();
         if (pgk_status r = pgk_gemm_nt(c_all, L.w_ukv, nullptr, kv, w.n_kv, 2 * HD, L.rank_pad, DT, st)) return r;
         int row = 0, kv0 = 0;
@@ -1355,7 +1809,7 @@ static pgk_status stack_prefill_t(Engine* e, int n_seqs, const int32_t* slots, c
             const T* q = (const T*)b.in + (size_t)row * L.n_in;
             const T* k = kv + (size_t)kv0 * 2 * HD;
             if (pgk_status r = window_attention(q, k, k + HD, (T*)b.a + (size_t)row * HD, L.heads, L.heads, lens[i], klen, L.head_pad, L.head_pad, L.scale, L.window, sd,
-                                                OutGate{q + HD + L.rank_pad, L.n_in, 1, 0}, nullptr, DT, st))
+                                                OutGate{L.gated ? q + HD + L.rank_pad : nullptr, L.n_in, 1, 0}, nullptr, DT, st))
                 return r;
             row += lens[i];
             kv0 += klen;
@@ -1363,7 +1817,7 @@ static pgk_status stack_prefill_t(Engine* e, int n_seqs, const int32_t* slots, c
         return PGK_OK;
     };
     auto attention = [&](int l) -> pgk_status {
-        const auto& L = s->layers[l];
+        const auto& L = s->at(l);
         const int src = kv_source(L, l), HD = L.heads * L.head_pad, GD = L.kv_heads * L.head_pad, R = s->ring[src];
         const bool mine = src == l;
         const LayerRows& w = lr[src];
@@ -1392,29 +1846,62 @@ static pgk_status stack_prefill_t(Engine* e, int n_seqs, const int32_t* slots, c
         }
         return PGK_OK;
     };
+    // taps over time and SiLU on the projected channels; then the rings take the last rows
+    auto convolve = [&](int l) -> pgk_status {
+        const auto& L = s->at(l);
+        const int ch = conv_channels(L);
+        if (pgk_status r = conv_silu_rows(ConvSiluArgs{b.in, L.n_in, L.conv, L.conv_bias, L.taps, ch, n, s->taps[l], d_rows, conv_rows_buf, ch}, DT, st)) return r;
+        return conv_save(b.in, L.n_in, d_seqs, n_seqs, s->taps[l], L.taps, ch, DT, st);
+    };
+    auto in_chunks = [&](int l, auto go) -> pgk_status {           // go(chunk list, its length, first chunk of every sequence)
+        const Chunks& t = chunkings[chunking[l]];
+        const char* tab = (const char*)s->tab + o_chunk;
+        return go((const RecurChunk*)(tab + t.o_list), (int)t.list.size(), (const int32_t*)(tab + t.o_seq));
+    };
     auto recurrence = [&](int l) -> pgk_status {
         RecurArgs a = recur_args(s, l, b.in, b.a, n);
         a.seqs = d_seqs; a.n_seqs = n_seqs;
-        if (chunking[l] >= 0) {
-            const Chunks& t = chunkings[chunking[l]];
-            const char* tab = (const char*)s->tab + o_chunk;
-            return recur_chunked(a, (const RecurChunk*)(tab + t.o_list), (int)t.list.size(), (const int32_t*)(tab + t.o_seq), ws_chunk, DT, st);
+        if (a.kind == RECUR_SSD) {
+            if (pgk_status r = convolve(l)) return r;
+            a.rows = conv_rows_buf; a.ld_rows = conv_channels(s->at(l));
         }
-        return recur_rows(a, DT, DT == PGK_F32, st);
+        if (pgk_status r = chunking[l] < 0 ? recur_rows(a, DT, DT == PGK_F32, st)
+                                           : in_chunks(l, [&](const RecurChunk* ch, int nc, const int32_t* of) { return recur_chunked(a, ch, nc, of, ws_chunk, DT, st); }))
+            return r;
+        return a.kind == RECUR_SSD ? ssd_norm(s, l, b.a, n, DT, st) : PGK_OK;
+    };
+    auto delta = [&](int l) -> pgk_status {
+        const auto& L = s->at(l);
+        const int a_off = delta_a_off(L), g_off = a_off + L.rank_a, NZ = L.heads * L.head_pad, NG = L.heads * L.vhead_pad;
+        if (pgk_status r = convolve(l)) return r;
+        if (n <= 16) {
+            if (pgk_status r = lowrank_rows(b.in, L.n_in, n, a_off, L.rank_a, L.w_a2, z_rows, NZ, g_off, L.rank_g, L.w_g2, gate_rows, NG, DT, DT == PGK_F32, st)) return r;
+        } else {
+            if (pgk_status r = rows_slice(b.in, L.n_in, a_off, L.rank_a, low_rows, n, DT, st)) return r;
+            if (pgk_status r = DT == PGK_F32 ? pgk_gemm_nt(low_rows, L.w_a2, nullptr, z_rows, n, NZ, L.rank_a, PGK_F32, st) : gemm_f32(low_rows, L.w_a2, z_rows, 1, n, NZ, L.rank_a, st)) return r;
+            if (pgk_status r = rows_slice(b.in, L.n_in, g_off, L.rank_g, low_rows, n, DT, st)) return r;
+            if (pgk_status r = pgk_gemm_nt(low_rows, L.w_g2, nullptr, gate_rows, n, NG, L.rank_g, DT, st)) return r;
+        }
+        DeltaArgs a = delta_args(s, l, b.in, z_rows, gate_rows, b.a, n);
+        a.rows = conv_rows_buf; a.ld_rows = conv_channels(L); a.seqs = d_seqs; a.n_seqs = n_seqs;
+        if (chunking[l] < 0) return delta_rows(a, DT, DT == PGK_F32, st);
+        return in_chunks(l, [&](const RecurChunk* ch, int nc, const int32_t* of) { return delta_chunked(a, ch, nc, of, ws_chunk, DT, st); });
     };
     auto mix = [&](int l) -> pgk_status {
-        switch (s->layers[l].mixer) {
+        switch (s->at(l).mixer) {
             case PGK_MIX_LATENT: return latent(l);
             case PGK_MIX_ATTENTION: return attention(l);
+            case PGK_MIX_DELTA: return delta(l);
             default: return recurrence(l);
         }
     };
-    Pending pend;
-    if (pgk_status r = rows_layers<T>(s, b, n, st, &pend, mix)) return r;
+    RowsNormArgs last;
+    if (pgk_status r = rows_model<T>(s, b, n, st, mix, &last)) return r;
     for (int i = 0; i < n_seqs; ++i) s->len[slots[i]] = starts[i] + lens[i];
     for (int w0 = 0; w0 < n_want; w0 += 128) {
         const int m = n_want - w0 < 128 ? n_want - w0 : 128;
-        RowsNormArgs a = norm_args(s, b, n, pend, s->final_norm, xw);
+        RowsNormArgs a = last;
+        a.out = xw;
         a.rows = d_want + w0;
         a.store_h = 0;                        // a wanted row may be asked for twice
         if (pgk_status r = rows_norm(a, m, DT, st)) return r;
@@ -1434,7 +1921,7 @@ static pgk_status stack_prefill(Engine* e, int n_seqs, const int32_t* slots, con
 // layer l's latent ring, K/V ring (values after the keys of a slot: v points at the first slot's) or recurrent states
 static pgk_status stack_kv_ptr(Engine* e, int layer, void** k, void** v) {
     const Stack* s = stack_of(e);
-    const auto& L = s->layers[layer];
+    const auto& L = s->at(layer);
     *k = s->cache[layer];
     *v = L.mixer == PGK_MIX_ATTENTION ? (char*)s->cache[layer] + (size_t)L.kv_heads * s->ring[kv_source(L, layer)] * L.head_pad * s->esize() : nullptr;
     return PGK_OK;
@@ -1466,12 +1953,31 @@ pgk_status pgk_engine_create_stack(const pgk_stack_config_t* cfg, const void* em
     const int Wp = ceil_div(c.width, 64) * 64;
     for (int l = 0; l < c.num_layers; ++l) {
         const auto& L = layers[l];
-        PGK_REQUIRE(L.mixer >= PGK_MIX_LATENT && L.mixer <= PGK_MIX_HGRN2 && (L.ff == PGK_FF_SWIGLU || L.ff == PGK_FF_XIELU), "pgk_engine_create_stack: layer %d: mixer %d, feed-forward %d", l, L.mixer, L.ff);
+        PGK_REQUIRE(L.mixer >= PGK_MIX_LATENT && L.mixer <= PGK_MIX_SSD && L.ff >= PGK_FF_SWIGLU && L.ff <= PGK_FF_MOE, "pgk_engine_create_stack: layer %d: mixer %d, feed-forward %d", l, L.mixer, L.ff);
         PGK_REQUIRE(L.heads >= 1 && L.dim >= 1 && L.vdim >= 1, "pgk_engine_create_stack: layer %d: bad mixer sizes", l);
         PGK_REQUIRE(L.ff_pad % 64 == 0 && L.ff_pad >= 0, "pgk_engine_create_stack: layer %d: feed-forward pad %d", l, L.ff_pad);
         PGK_REQUIRE(L.n_in % 64 == 0 && L.n_att % 64 == 0, "pgk_engine_create_stack: layer %d: %d in-projection rows, %d out-projection columns", l, L.n_in, L.n_att);
-        PGK_REQUIRE(L.norm1b && L.w_in && L.w_o && (!L.ff_pad || (L.norm2b && L.w_gate_up && L.w_down)), "pgk_engine_create_stack: layer %d: missing weights", l);
+        PGK_REQUIRE(L.w_in && L.w_o && (!L.ff_pad || (L.w_gate_up && L.w_down)), "pgk_engine_create_stack: layer %d: missing weights", l);
+        if (c.block == PGK_BLOCK_PARALLEL) {
+            PGK_REQUIRE(L.norm1 && (!L.ff_pad || (L.ff == PGK_FF_MOE && L.correction)), "pgk_engine_create_stack: layer %d: a parallel layer has one norm and experts or no feed-forward", l);
+            if (L.ff_pad)
+                PGK_REQUIRE(L.experts >= 1 && L.experts <= MOE_MAX_EXPERTS && L.top >= 1 && L.top <= L.experts && L.top <= MOE_MAX_TOP && L.groups >= 0 &&
+                                (L.groups == 0 || (L.experts % L.groups == 0 && L.keep >= 1 && L.keep <= L.groups && L.keep * (L.experts / L.groups) >= L.top)),
+                            "pgk_engine_create_stack: layer %d: %d experts, top %d, %d of %d groups", l, L.experts, L.top, L.keep, L.groups);
+        } else {
+            PGK_REQUIRE(L.norm1b && (!L.ff_pad || (L.ff != PGK_FF_MOE && L.norm2b)), "pgk_engine_create_stack: layer %d: missing norms", l);
+        }
         const int HD = L.heads * L.head_pad;
+        if (L.mixer == PGK_MIX_DELTA || L.mixer == PGK_MIX_SSD) {
+            const bool delta = L.mixer == PGK_MIX_DELTA;
+            PGK_REQUIRE(L.kv_heads >= 1 && L.heads % L.kv_heads == 0 && L.head_pad % 16 == 0 && L.vhead_pad % 16 == 0 && L.head_pad >= L.dim && L.vhead_pad >= L.vdim && L.taps >= 1 && L.kv_from < 0 &&
+                            L.n_att >= L.heads * L.vhead_pad && L.n_in >= (delta ? delta_a_off(L) + L.rank_a + L.rank_g : conv_channels(L) + L.heads * L.vhead_pad + L.heads),
+                        "pgk_engine_create_stack: layer %d: %d / %d heads of %d / %d padded to %d / %d, %d taps", l, L.heads, L.kv_heads, L.dim, L.vdim, L.head_pad, L.vhead_pad, L.taps);
+            PGK_REQUIRE(L.conv && L.o_norm && L.decay && L.dt_bias && (delta ? L.w_a2 && L.w_g2 : L.skip != nullptr), "pgk_engine_create_stack: layer %d: missing weights", l);
+            PGK_REQUIRE(delta ? L.rank_a % 64 == 0 && L.rank_a >= 64 && L.rank_g % 64 == 0 && L.rank_g >= 64 : L.norm_parts >= 1 && L.heads * L.vdim % L.norm_parts == 0,
+                        "pgk_engine_create_stack: layer %d: ranks %d / %d, %d norm parts", l, L.rank_a, L.rank_g, L.norm_parts);
+            continue;
+        }
         if (L.mixer == PGK_MIX_HGRN2) {
             PGK_REQUIRE(L.head_pad % 16 == 0 && L.vhead_pad % 16 == 0 && L.head_pad >= L.dim && L.vhead_pad >= L.vdim && L.n_in >= 2 * HD + L.heads * L.vhead_pad && L.n_att >= L.heads * L.vhead_pad,
                         "pgk_engine_create_stack: layer %d: head widths %d / %d padded to %d / %d", l, L.dim, L.vdim, L.head_pad, L.vhead_pad);
@@ -1480,8 +1986,8 @@ pgk_status pgk_engine_create_stack(const pgk_stack_config_t* cfg, const void* em
         }
         PGK_REQUIRE(L.window >= 1 && L.head_pad % 64 == 0 && L.head_pad >= L.dim && L.head_pad >= L.vdim && L.n_att == HD, "pgk_engine_create_stack: layer %d: window %d, head pad %d for widths %d / %d", l, L.window, L.head_pad, L.dim, L.vdim);
         if (L.mixer == PGK_MIX_LATENT) {
-            PGK_REQUIRE(L.rank >= 1 && L.rank_pad % 64 == 0 && L.rank_pad >= L.rank && L.rank_pad <= 2048, "pgk_engine_create_stack: layer %d: latent size %d padded to %d (at most 2048)", l, L.rank, L.rank_pad);
-            PGK_REQUIRE(L.n_in >= HD + L.rank_pad + L.heads && L.kv_heads == L.heads && L.kv_from < 0, "pgk_engine_create_stack: layer %d: in-projection rows %d", l, L.n_in);
+            PGK_REQUIRE(L.rank >= 1 && L.rank_pad % 64 == 0 && L.rank_pad >= L.rank + L.rot && L.rank_pad <= 2048 && L.rot >= 0 && L.rot % 2 == 0 && L.rot <= L.dim && (!L.rot || L.rot_freq), "pgk_engine_create_stack: layer %d: latent size %d padded to %d (at most 2048)", l, L.rank, L.rank_pad);
+            PGK_REQUIRE(L.n_in >= HD + L.rank_pad + (L.gated ? L.heads : 0) && L.kv_heads == L.heads && L.kv_from < 0, "pgk_engine_create_stack: layer %d: in-projection rows %d", l, L.n_in);
             PGK_REQUIRE(L.norm1 && L.c_norm && L.w_ukv, "pgk_engine_create_stack: layer %d: missing weights", l);
         } else {
             PGK_REQUIRE(L.kv_heads >= 1 && L.heads % L.kv_heads == 0 && L.head_pad <= 1024 && L.taps >= 1, "pgk_engine_create_stack: layer %d: %d / %d heads of %d, %d taps", l, L.heads, L.kv_heads, L.head_pad, L.taps);
@@ -1492,6 +1998,8 @@ pgk_status pgk_engine_create_stack(const pgk_stack_config_t* cfg, const void* em
             }
         }
     }
+    PGK_REQUIRE(c.loop_times >= 0 && (!c.loop_times || (c.block == PGK_BLOCK_PARALLEL && c.loop_start >= 0 && c.loop_start < c.loop_stop && c.loop_stop <= c.num_layers && c.loop_in && c.loop_step)),
+                "pgk_engine_create_stack: layers %d .. %d of %d, %d times", c.loop_start, c.loop_stop - 1, c.num_layers, c.loop_times);
     Engine* e = new Engine();
     Stack* s = new Stack();
     e->kind = &STACK_KIND;
@@ -1499,11 +2007,20 @@ pgk_status pgk_engine_create_stack(const pgk_stack_config_t* cfg, const void* em
     e->one_sequence = true;
     s->cfg = c;
     s->layers.assign(layers, layers + c.num_layers);
+    for (int l = 0; l < c.num_layers; ++l) {
+        if (c.loop_times && l == c.loop_start) {
+            for (int t = 0; t < c.loop_times; ++t)
+                for (int k = c.loop_start; k < c.loop_stop; ++k) s->runs.push_back(Run{k, k == c.loop_start ? t : -1});
+            l = c.loop_stop - 1;
+        } else s->runs.push_back(Run{l, -1});
+    }
+    for (int l = 0; l < c.num_layers; ++l)
+        if (c.loop_times && layers[l].kv_from >= 0) { delete s; delete e; return set_error(PGK_ERR_UNSUPPORTED, "pgk_engine_create_stack: layer %d takes another layer's keys in a model with a loop", l); }
     s->embed = embed; s->pos = pos_embed; s->head = head; s->final_norm = final_norm;
     s->Wp = Wp;
     s->len.assign(c.max_batch, 0);
     e->cfg = pgk_model_config_t{};
-    e->cfg.vocab_size = c.vocab_size; e->cfg.hidden_size = c.width; e->cfg.num_layers = c.num_layers;
+    e->cfg.vocab_size = c.vocab_size; e->cfg.hidden_size = c.width; e->cfg.num_layers = s->n_runs();
     e->cfg.max_seq_len = c.max_seq_len; e->cfg.max_batch = c.max_batch; e->cfg.norm_eps = c.norm_eps;
     {
         int dev = 0;
@@ -1520,17 +2037,28 @@ pgk_status pgk_engine_create_stack(const pgk_stack_config_t* cfg, const void* em
     };
     const size_t B = c.max_batch, E = s->esize();
     size_t part = 0, ml = 0, ql = 0;
+    int max_router = 0, max_act = 0;
     auto most = [](auto& m, auto v) { if (v > m) m = v; };
-    s->reach.assign(c.num_layers, 0);
-    for (int l = 0; l < c.num_layers; ++l)
-        if (s->layers[l].mixer != PGK_MIX_HGRN2) most(s->reach[kv_source(s->layers[l], l)], s->layers[l].window);
-    for (int l = 0; l < c.num_layers; ++l) {
-        const auto& L = s->layers[l];
+    s->reach.assign(s->n_runs(), 0);
+    for (int l = 0; l < s->n_runs(); ++l)
+        if (!recurrent(s->at(l))) most(s->reach[kv_source(s->at(l), l)], s->at(l).window);
+    for (int l = 0; l < s->n_runs(); ++l) {
+        const auto& L = s->at(l);
         const int R = s->reach[l] < c.max_seq_len ? s->reach[l] : c.max_seq_len, HD = L.heads * L.head_pad;
         s->ring.push_back(R);
         void *p = nullptr, *t = nullptr;
         if (L.mixer == PGK_MIX_LATENT) A(&p, B * R * L.rank_pad * E, &e->kv_bytes, true);
-        else if (L.mixer == PGK_MIX_HGRN2) A(&p, B * HD * L.vhead_pad * 4, &e->kv_bytes, true);
+        else if (recurrent(L)) {
+            A(&p, B * HD * L.vhead_pad * 4, &e->kv_bytes, true);
+            const int ch = conv_channels(L);
+            if (ch) A(&t, B * L.taps * ch * E, &e->kv_bytes, true);
+            most(s->max_conv, ch);
+            if (L.mixer == PGK_MIX_DELTA) {
+                most(s->max_z, HD);
+                most(s->max_gate, L.heads * L.vhead_pad);
+                most(s->max_low, L.rank_a > L.rank_g ? L.rank_a : L.rank_g);
+            }
+        }
         else {
             const int GD = L.kv_heads * L.head_pad;
             if (L.kv_from < 0) A(&p, B * 2 * R * GD * E, &e->kv_bytes, true);
@@ -1542,8 +2070,9 @@ pgk_status pgk_engine_create_stack(const pgk_stack_config_t* cfg, const void* em
         s->taps.push_back(t);
         most(s->max_in, L.n_in);
         most(s->max_att, L.n_att);
-        most(s->max_ff, L.ff_pad);
-        for (int m = 1; m <= c.max_batch && L.mixer != PGK_MIX_HGRN2; ++m) {
+        if (router_rows(L)) { most(s->max_top, L.top); most(max_router, router_rows(L)); most(max_act, L.top * L.ff_pad); }
+        else { most(s->max_ff, L.ff_pad); most(max_act, L.ff_pad); }
+        for (int m = 1; m <= c.max_batch && !recurrent(L); ++m) {
             const int src = kv_source(L, l), keys = L.window < s->ring[src] ? L.window : s->ring[src];
             const size_t ns = (size_t)(L.mixer == PGK_MIX_LATENT ? pick_nsplit(e, m, L, R) : kv_attn_splits(m, L.heads, L.kv_heads, keys, e->cu_count)) * m * L.heads;
             most(part, ns * (L.mixer == PGK_MIX_LATENT ? L.rank_pad : L.head_pad));
@@ -1561,10 +2090,24 @@ pgk_status pgk_engine_create_stack(const pgk_stack_config_t* cfg, const void* em
     A((void**)&e->amax_val, B * e->lm_cap * 4, &e->ws_bytes);
     A((void**)&e->amax_idx, B * e->lm_cap * 4, &e->ws_bytes);
     A((void**)&e->clk_log, (size_t)e->log_cap * 16, &e->ws_bytes);
-    A((void**)&s->in32, (size_t)s->max_in * 4, &e->ws_bytes);
+    A((void**)&s->in32, (size_t)(s->max_in + max_router) * 4, &e->ws_bytes);
     A((void**)&s->a32, (size_t)s->max_att * 4, &e->ws_bytes, true);     // padding columns of a head are never written: zero
     A((void**)&s->y32, (size_t)Wp * 4, &e->ws_bytes, true);
-    A((void**)&s->act32, (size_t)(s->max_ff ? s->max_ff : 64) * 4, &e->ws_bytes);
+    A((void**)&s->act32, (size_t)(max_act ? max_act : 64) * 4, &e->ws_bytes);
+    if (c.block == PGK_BLOCK_PARALLEL) {
+        A((void**)&s->y32b, (size_t)Wp * 4, &e->ws_bytes, true);
+        A((void**)&s->h32, (size_t)Wp * 4, &e->ws_bytes, true);
+        A((void**)&s->ids, MOE_MAX_TOP * 4, &e->ws_bytes, true);
+        if (c.loop_times) A(&s->cat16, B * 2 * Wp * E, &e->ws_bytes);
+        if (s->max_top) A(&s->e16, B * s->max_top * Wp * E, &e->ws_bytes);
+        size_t ws = 0;
+        for (int m = 2; m <= c.max_batch; ++m) most(ws, s->moe_ws(m));
+        if (ws) A(&s->moe16, ws, &e->ws_bytes);
+    }
+    if (s->max_z) {
+        A((void**)&s->z32, B * s->max_z * 4, &e->ws_bytes);
+        A(&s->gate, B * s->max_gate * 4, &e->ws_bytes);
+    }
     auto some = [](size_t v) { return v ? v : (size_t)64; };
     A(&s->qlat, some(ql) * 4, &e->ws_bytes);
     A(&s->qx, some(B * s->max_q) * 4, &e->ws_bytes);
@@ -1588,7 +2131,7 @@ pgk_status pgk_engine_create_stack(const pgk_stack_config_t* cfg, const void* em
                 auto& P = s->packed[l];
                 if (pkgemm_shape_ok(L.n_in, Wp, false)) fn(&P.in, L.w_in, L.n_in, Wp);
                 if (pkgemm_shape_ok(Wp, L.n_att, true)) fn(&P.o, L.w_o, Wp, L.n_att);
-                if (!L.ff_pad) continue;
+                if (!L.ff_pad || L.ff == PGK_FF_MOE) continue;
                 if (pkgemm_shape_ok(up_rows(L), Wp, false)) fn(&P.gate_up, L.w_gate_up, up_rows(L), Wp);
                 if (pkgemm_shape_ok(Wp, L.ff_pad, true)) fn(&P.down, L.w_down, Wp, L.ff_pad);
             }

@@ -13,6 +13,7 @@
 // block substitution with the 16 x 16 inverses.  All products are fp32 (v_mfma_f32_16x16x4_f32).
 
 #include <type_traits>
+#include <vector>
 
 #include "mixers.hip.h"
 
@@ -619,3 +620,46 @@ pgk_status lowrank_rows(const void* in, int ld_in, int n, int a_off, int ka, con
 }
 
 }  // namespace pgk
+
+using namespace pgk;
+
+extern "C" {
+
+pgk_status pgk_delta_rule(const void* q, const void* k, const void* v, const float* z, const void* strength, const void* gate, const float* decay, const float* step_bias,
+                          const float* norm, float* state, void* out, int n, int fresh, int heads, int kv_heads, int dim, int vdim, float eps, pgk_dtype dt, pgk_stream s) {
+    PGK_REQUIRE(q && k && v && z && strength && gate && decay && step_bias && norm && state && out, "pgk_delta_rule: null pointer");
+    PGK_REQUIRE(n >= 1 && heads >= 1 && kv_heads >= 1 && heads % kv_heads == 0 && dim >= 4 && dim % 4 == 0 && vdim >= 4 && vdim % 4 == 0, "pgk_delta_rule: bad shape %d / %d x %d x %d, %d rows",
+                heads, kv_heads, dim, vdim, n);
+    PGK_REQUIRE(dt == PGK_BF16 || dt == PGK_F32, "pgk_delta_rule: dtype %d (bf16 or f32)", (int)dt);
+    hipStream_t st = resolve_stream(s);
+    const size_t E = dtype_size(dt), wq = (size_t)kv_heads * dim * E, wv = (size_t)heads * vdim * E, row = 2 * wq + wv;
+    auto up = [](size_t b) { return (b + 255) & ~(size_t)255; };
+    DeltaArgs a{};
+    a.in = strength; a.ld_in = heads; a.ld_rows = (int)(row / E); a.z = z; a.ld_z = heads * dim; a.gate = gate; a.ld_gate = heads * vdim;
+    a.decay = decay; a.dt_bias = step_bias; a.norm = norm; a.H = heads; a.G = kv_heads; a.dim = a.dim_true = dim; a.vdim = a.vdim_true = vdim; a.n = n; a.eps = eps;
+    a.state = state; a.n_seqs = 1; a.out = out; a.ld_out = heads * vdim;
+    const int C = n >= RECUR_CHUNKED_FROM && delta_chunk_ok(dim, vdim) ? DELTA_CHUNK : 0, nch = C ? ceil_div(n, C) : 0;
+    std::vector<RecurChunk> chunks;
+    for (int c = 0; c < nch; ++c) chunks.push_back(RecurChunk{c * C, n - c * C < C ? n - c * C : C});
+    const int32_t of_seq[2] = {0, nch};
+    const SeqSpan span{0, n, fresh ? 0 : 1, 0};
+    const size_t o_span = up(n * row), o_of = o_span + up(sizeof(span)), o_ch = o_of + up(sizeof(of_seq)), o_ws = o_ch + up(nch * sizeof(RecurChunk));
+    char* ws = nullptr;
+    if (pgk_status r = pgk_malloc((void**)&ws, o_ws + (nch ? delta_chunk_bytes(a, nch) : 0) + 256)) return r;
+    hipError_t e = hipMemcpy2DAsync(ws, row, q, wq, wq, n, hipMemcpyDeviceToDevice, st);
+    if (e == hipSuccess) e = hipMemcpy2DAsync(ws + wq, row, k, wq, wq, n, hipMemcpyDeviceToDevice, st);
+    if (e == hipSuccess) e = hipMemcpy2DAsync(ws + 2 * wq, row, v, wv, wv, n, hipMemcpyDeviceToDevice, st);
+    if (e == hipSuccess) e = hipMemcpyAsync(ws + o_span, &span, sizeof(span), hipMemcpyHostToDevice, st);
+    if (e == hipSuccess) e = hipMemcpyAsync(ws + o_of, of_seq, sizeof(of_seq), hipMemcpyHostToDevice, st);
+    if (e == hipSuccess && nch) e = hipMemcpyAsync(ws + o_ch, chunks.data(), nch * sizeof(RecurChunk), hipMemcpyHostToDevice, st);
+    if (e == hipSuccess) e = hipStreamSynchronize(st);
+    a.rows = ws; a.seqs = (const SeqSpan*)(ws + o_span);
+    pgk_status r;
+    if (e != hipSuccess) r = set_error(PGK_ERR_HIP, "pgk_delta_rule: %s", hipGetErrorString(e));
+    else if (nch) r = delta_chunked(a, (const RecurChunk*)(ws + o_ch), nch, (const int32_t*)(ws + o_of), ws + o_ws, dt, st);
+    else r = delta_rows(a, dt, dt == PGK_F32, st);
+    pgk_free(ws);       // stream-ordered reuse
+    return r;
+}
+
+}  // extern "C"

@@ -399,7 +399,7 @@ int engine_gemm_pick_splits(int M, int N, int K) {
     return s < 1 ? 1 : s;
 }
 pgk_status engine_gemm_nt_slabs(const bf16* A, const void* W, float* slabs, int splits, int M, int N, int K, hipStream_t st, bool packed) {
-    PGK_REQUIRE(splits >= 2 && K % 8 == 0, "engine_gemm_nt_slabs: splits=%d K=%d", splits, K);
+    PGK_REQUIRE(splits >= 1 && K % 8 == 0, "engine_gemm_nt_slabs: splits=%d K=%d", splits, K);
     if (gemm128s_ok(M, N, K) && K % (64 * splits) == 0) return gemm128s_bf16_nt(A, (const bf16*)W, nullptr, slabs, 2, splits, M, N, K, st, nullptr, packed);
     PGK_REQUIRE(!packed, "engine_gemm_nt_slabs: M=%d N=%d K=%d splits=%d has no kernel that reads the fragment-major copy", M, N, K, splits);
     return launch_mfma<bf16, 128, 128, B_NT, 2>(A, W, nullptr, nullptr, slabs, M, N, K, st, splits);

@@ -318,7 +318,71 @@ pgk_status window_attention(const void* q, const void* k, const void* v, void* o
 
 using namespace pgk;
 
+// One wave per row: layer norm, latent rows, rotation of query columns
+template <class T>
+__global__ __launch_bounds__(256) void layernorm_f32_kernel(const float* x, const float* w, T* out, int rows, int cols, float eps) {
+    const int row = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
+    if (row >= rows) return;
+    const float* r = x + (size_t)row * cols;
+    float s = 0.f, ss = 0.f;
+    for (int i = lane; i < cols; i += 64) s += r[i];
+    const float mean = wave_sum(s) / cols;
+    for (int i = lane; i < cols; i += 64) ss = fmaf(r[i] - mean, r[i] - mean, ss);
+    const float inv = 1.0f / sqrtf(wave_sum(ss) / cols + eps);
+    for (int i = lane; i < cols; i += 64) out[(size_t)row * cols + i] = from_f<T>((r[i] - mean) * inv * w[i]);
+}
+template <class T>
+__device__ __forceinline__ void turn_pair(const T* src, T* dst, float angle) {
+    float s, c;
+    sincosf(angle, &s, &c);
+    const float u = to_f(src[0]), v = to_f(src[1]);
+    dst[0] = from_f<T>(fmaf(u, c, -v * s));
+    dst[1] = from_f<T>(fmaf(v, c, u * s));
+}
+template <class T>
+__global__ __launch_bounds__(256) void latent_cache_rows_kernel(const T* x, const float* norm, const float* freq, T* out, int n, int rank, int rot, int first, float eps) {
+    const int row = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
+    if (row >= n) return;
+    const T* r = x + (size_t)row * (rank + rot);
+    T* o = out + (size_t)row * (rank + rot);
+    float ss = 0.f;
+    for (int i = lane; i < rank; i += 64) { const float v = to_f(r[i]); ss = fmaf(v, v, ss); }
+    const float inv = 1.0f / sqrtf(wave_sum(ss) / rank + eps);
+    for (int i = lane; i < rank; i += 64) o[i] = from_f<T>(to_f(r[i]) * inv * norm[i]);
+    for (int i = lane; i < rot / 2; i += 64) turn_pair<T>(r + rank + 2 * i, o + rank + 2 * i, (float)(first + row) * freq[i]);
+}
+template <class T>
+__global__ __launch_bounds__(256) void rotate_pairs_kernel(T* x, const float* freq, int total, int heads, int dim, int rot, int first) {
+    const int i = blockIdx.x * 256 + threadIdx.x, pairs = rot / 2;
+    if (i >= total) return;
+    T* p = x + (size_t)(i / pairs) * dim + dim - rot + 2 * (i % pairs);
+    turn_pair<T>(p, p, (float)(first + i / pairs / heads) * freq[i % pairs]);
+}
+
 extern "C" {
+
+pgk_status pgk_layernorm_f32(const float* x, const float* weight, void* out, int rows, int cols, float eps, pgk_dtype out_dt, pgk_stream s) {
+    PGK_REQUIRE(x && weight && out && rows >= 0 && cols >= 1, "pgk_layernorm_f32: %d x %d", rows, cols);
+    if (!rows) return PGK_OK;
+    PGK_DISPATCH_FLOAT(out_dt, "pgk_layernorm_f32", (layernorm_f32_kernel<T><<<ceil_div(rows, 4), 256, 0, resolve_stream(s)>>>(x, weight, (T*)out, rows, cols, eps)));
+    PGK_LAUNCH_CHECK();
+    return PGK_OK;
+}
+
+pgk_status pgk_latent_rows(const void* x, const float* norm, const float* freq, void* out, int n, int rank, int rot, int first, float eps, pgk_dtype dt, pgk_stream s) {
+    PGK_REQUIRE(x && norm && freq && out && n >= 1 && rank >= 1 && rot >= 2 && rot % 2 == 0 && first >= 0, "pgk_latent_rows: %d rows of %d + %d", n, rank, rot);
+    PGK_DISPATCH_FLOAT(dt, "pgk_latent_rows", (latent_cache_rows_kernel<T><<<ceil_div(n, 4), 256, 0, resolve_stream(s)>>>((const T*)x, norm, freq, (T*)out, n, rank, rot, first, eps)));
+    PGK_LAUNCH_CHECK();
+    return PGK_OK;
+}
+
+pgk_status pgk_rotate_pairs(void* x, const float* freq, int n, int heads, int dim, int rot, int first, pgk_dtype dt, pgk_stream s) {
+    PGK_REQUIRE(x && freq && n >= 1 && heads >= 1 && rot >= 2 && rot % 2 == 0 && rot <= dim && first >= 0 && (long long)n * heads * rot < (1LL << 31), "pgk_rotate_pairs: %d x %d x %d, %d turned", n, heads, dim, rot);
+    const int total = n * heads * (rot / 2);
+    PGK_DISPATCH_FLOAT(dt, "pgk_rotate_pairs", (rotate_pairs_kernel<T><<<ceil_div(total, 256), 256, 0, resolve_stream(s)>>>((T*)x, freq, total, heads, dim, rot, first)));
+    PGK_LAUNCH_CHECK();
+    return PGK_OK;
+}
 
 pgk_status pgk_rmsnorm_f32(const float* x, const float* weight, void* out, int rows, int cols, float eps, pgk_dtype out_dt, pgk_stream s) {
     PGK_REQUIRE(x && weight && out && rows >= 0 && cols > 0, "pgk_rmsnorm_f32: bad arguments [%d, %d]", rows, cols);
@@ -366,7 +430,7 @@ pgk_status pgk_head_gate(void* x, const void* gate, int rows, int heads, int d, 
 }
 
 pgk_status pgk_pad_2d(const void* src, void* dst, int rows, int cols, int dst_rows, int dst_cols, pgk_dtype dt, pgk_stream s) {
-    PGK_REQUIRE(src && dst && rows >= 1 && cols >= 1 && dst_rows >= rows && dst_cols >= cols, "pgk_pad_2d: [%d, %d] into [%d, %d]", rows, cols, dst_rows, dst_cols);
+    PGK_REQUIRE(src && dst && rows >= 1 && cols >= 1 && dst_rows >= rows && dst_cols >= 1, "pgk_pad_2d: [%d, %d] into [%d, %d]", rows, cols, dst_rows, dst_cols);
     const size_t total = (size_t)dst_rows * dst_cols;
     const int grid = ceil_div((long long)total, 256) > 8192 ? 8192 : ceil_div((long long)total, 256);
     hipStream_t st = resolve_stream(s);

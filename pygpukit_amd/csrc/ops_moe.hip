@@ -301,4 +301,40 @@ pgk_status moe_rows(const MoeArgs& a, pgk_dtype dt, hipStream_t st) {
     return PGK_OK;
 }
 
+template <class T>
+__global__ __launch_bounds__(256) void moe_sum_kernel(const T* e, float* out, int W, int top) {
+    const size_t row = blockIdx.x;
+    for (int i = threadIdx.x; i < W; i += 256) {
+        float s = 0.f;
+        for (int k = 0; k < top; ++k) s += to_f(e[(row * top + k) * W + i]);
+        out[row * W + i] = s;
+    }
+}
+
 }  // namespace pgk
+
+using namespace pgk;
+
+extern "C" {
+
+pgk_status pgk_moe(const void* x, const void* router, const float* correction, const void* w_up, const void* w_down, float* out, int n, int width, int ff, int experts, int top, int groups,
+                   int keep, float scale, pgk_dtype dt, pgk_stream s) {
+    PGK_REQUIRE(x && router && correction && w_up && w_down && out && n >= 1 && top >= 1, "pgk_moe: null pointer or empty");
+    PGK_REQUIRE(dt == PGK_BF16 || dt == PGK_F32, "pgk_moe: dtype %d (bf16 or f32)", (int)dt);
+    PGK_REQUIRE(width >= 64 && width % 64 == 0 && ff >= 64 && ff % 64 == 0 && experts >= 1, "pgk_moe: %d experts of %d x %d", experts, width, ff);
+    hipStream_t st = resolve_stream(s);
+    const RouterCfg r{correction, experts, top, groups, keep, scale};
+    const size_t rows = (((size_t)n * top * width * dtype_size(dt)) + 255) & ~(size_t)255;
+    char* ws = nullptr;
+    if (pgk_status q = pgk_malloc((void**)&ws, rows + moe_bytes(n, width, ff, r, dt))) return q;
+    pgk_status q = moe_rows(MoeArgs{x, n, width, ff, r, router, w_up, w_down, ws, ws + rows}, dt, st);
+    if (q == PGK_OK) {
+        if (dt == PGK_F32) moe_sum_kernel<float><<<n, 256, 0, st>>>((const float*)ws, out, width, top);
+        else moe_sum_kernel<bf16><<<n, 256, 0, st>>>((const bf16*)ws, out, width, top);
+        if (hipError_t e = hipGetLastError()) q = set_error(PGK_ERR_HIP, "pgk_moe: %s", hipGetErrorString(e));
+    }
+    pgk_free(ws);       // stream-ordered reuse
+    return q;
+}
+
+}  // extern "C"

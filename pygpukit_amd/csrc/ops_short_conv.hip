@@ -2,6 +2,7 @@
 // mixers.hip.h), RMS norm in equal parts of a row, column slices.
 
 #include <type_traits>
+#include <vector>
 
 #include "mixers.hip.h"
 
@@ -144,3 +145,30 @@ pgk_status rows_slice(const void* in, int ld_in, int off, int cols, void* out, i
 }
 
 }  // namespace pgk
+
+using namespace pgk;
+
+extern "C" {
+
+pgk_status pgk_conv_silu(const void* u, const void* past, const void* w, const float* bias, void* out, int n, int channels, int taps, pgk_dtype dt, pgk_stream s) {
+    PGK_REQUIRE(u && w && out && n >= 1 && taps >= 1, "pgk_conv_silu: %d rows of %d channels, %d taps", n, channels, taps);
+    PGK_REQUIRE(dt == PGK_BF16 || dt == PGK_F32, "pgk_conv_silu: dtype %d (bf16 or f32)", (int)dt);
+    hipStream_t st = resolve_stream(s);
+    // the past as ring rows of positions 1 .. taps - 1, the rows are positions taps, taps + 1, ...
+    const size_t E = dtype_size(dt), row = (size_t)channels * E, o_rows = ((size_t)taps * row + 255) & ~(size_t)255;
+    const bool goes_on = past && taps > 1;
+    std::vector<RowSrc> src(n);
+    for (int i = 0; i < n; ++i) src[i] = RowSrc{(goes_on ? taps : 0) + i, 0, 0};
+    char* ws = nullptr;
+    if (pgk_status r = pgk_malloc((void**)&ws, o_rows + n * sizeof(RowSrc))) return r;
+    hipError_t e = hipSuccess;
+    if (goes_on) e = hipMemcpyAsync(ws + row, past, (taps - 1) * row, hipMemcpyDeviceToDevice, st);
+    if (e == hipSuccess) e = hipMemcpyAsync(ws + o_rows, src.data(), n * sizeof(RowSrc), hipMemcpyHostToDevice, st);
+    if (e == hipSuccess) e = hipStreamSynchronize(st);
+    const pgk_status r = e != hipSuccess ? set_error(PGK_ERR_HIP, "pgk_conv_silu: %s", hipGetErrorString(e))
+                                         : conv_silu_rows(ConvSiluArgs{u, channels, w, bias, taps, channels, n, ws, (const RowSrc*)(ws + o_rows), out, channels}, dt, st);
+    pgk_free(ws);       // stream-ordered reuse
+    return r;
+}
+
+}  // extern "C"

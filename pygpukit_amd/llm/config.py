@@ -2,8 +2,8 @@
 
 TransformerConfig carries the dimensions; ModelSpec is the data-only description of one
 architecture family (HF tensor-name patterns + architecture flags + default hyper-parameters).
-Dense families are described: GPT-2, Llama, Qwen2, Qwen3 and the layer-list families Totolorn and Malasun (MoE families are
-not).  A layer-list model's config.json spells out every layer: LayerConfig."""
+Described are the dense families GPT-2, Llama, Qwen2, Qwen3 and the layer-list families Totolorn, Malasun and Ratasun (whose
+feed-forwards are mixtures of experts).  A layer-list model's config.json spells out every layer: LayerConfig."""
 
 from __future__ import annotations
 
@@ -76,6 +76,23 @@ class ModelSpec:
     norm_scalar: bool = False              # a norm's weight is one number
     norm_weight_offset: float = 0.0        # norms multiply by offset + weight (1: weights stored around zero)
     residual_f32: bool = False             # the residual stream stays fp32 whatever the element type
+    parallel: bool = False                 # mixer and feed-forward read one norm, both results are added
+    strength: str | None = None            # delta rule: write strength, the two maps of the decay and of the output gate
+    decay_down: str | None = None
+    decay_up: str | None = None
+    gate_down: str | None = None
+    gate_up: str | None = None
+    decay_log: str | None = None           # recurrences: logarithm of the decay rate, bias of its step
+    step_bias: str | None = None
+    in_proj: str | None = None             # state space: all projections in one matrix, taps and their bias, skip, norm of the output
+    conv: str | None = None
+    conv_bias: str | None = None
+    skip: str | None = None
+    out_norm: str | None = None
+    router: str | None = None              # experts: router, correction of the choice
+    router_correction: str | None = None
+    loop_in: str | None = None             # passes over a stretch of layers: map of [stream; embedding], one vector per pass
+    loop_step: str | None = None
 
 
 def _hf_decoder_spec(name: str, *, qk_norm: bool, qkv_bias: bool, eps: float, theta: float) -> ModelSpec:
@@ -136,8 +153,21 @@ MALASUN_SPEC = ModelSpec(
     v_conv=_T + "mix.v.conv", out_gate=_T + "mix.g", forget_proj=_T + "mix.f", forget_bias=_T + "mix.f.b", forget_lower=_T + "mix.lower",
     head_norm=_T + "mix.norm", act_params=_T + "mlp.act", norm_scalar=True, residual_f32=True)
 
+RATASUN_SPEC = ModelSpec(
+    name="ratasun", embed_tokens="embed", position_embed=None, lm_head="head", final_norm="final.norm", final_norm_bias=None,
+    attn_norm=_T + "norm1", attn_norm_bias=None, q_proj=_T + "mix.q", k_proj=_T + "mix.k", v_proj=_T + "mix.v", o_proj=_T + "mix.o",
+    q_bias=None, k_bias=None, v_bias=None, o_bias=None, q_norm=None, k_norm=None, mlp_norm=None, mlp_norm_bias=None,
+    fc1=None, fc1_bias=None, fc2=None, fc2_bias=None, gate_proj=None, up_proj=None, down_proj=None,
+    expert_gate_proj=_T + "mlp.e{expert}.gate", expert_up_proj=_T + "mlp.e{expert}.up", expert_down_proj=_T + "mlp.e{expert}.down",
+    norm_type="layernorm", activation="silu", use_rope=True, is_moe=True, architecture="Ratasun", parallel=True, residual_f32=True,
+    kv_down_proj=_T + "mix.dkv", kv_down_norm=_T + "mix.dkv.norm", k_up_proj=_T + "mix.uk", v_up_proj=_T + "mix.uv",
+    q_conv=_T + "mix.q.conv", k_conv=_T + "mix.k.conv", v_conv=_T + "mix.v.conv", head_norm=_T + "mix.norm", strength=_T + "mix.b",
+    decay_down=_T + "mix.a1", decay_up=_T + "mix.a2", gate_down=_T + "mix.g1", gate_up=_T + "mix.g2", decay_log=_T + "mix.A_log",
+    step_bias=_T + "mix.dt_bias", in_proj=_T + "mix.in", conv=_T + "mix.conv", conv_bias=_T + "mix.conv.b", skip=_T + "mix.D", out_norm=_T + "mix.norm",
+    router=_T + "mlp.router", router_correction=_T + "mlp.correction", loop_in="loop.in", loop_step="loop.step")
+
 MODEL_SPECS: dict[str, ModelSpec] = {"gpt2": GPT2_SPEC, "llama": LLAMA_SPEC, "qwen3": QWEN3_SPEC, "qwen2": QWEN2_SPEC,
-                                     "totolorn": TOTOLORN_SPEC, "malasun": MALASUN_SPEC}
+                                     "totolorn": TOTOLORN_SPEC, "malasun": MALASUN_SPEC, "ratasun": RATASUN_SPEC}
 
 
 def detect_model_spec(tensor_names: list[str], config: dict | None = None) -> ModelSpec:
@@ -152,7 +182,7 @@ def detect_model_spec(tensor_names: list[str], config: dict | None = None) -> Mo
         raise ValueError(f"unknown architecture {arch!r} (known: {[s.architecture for s in MODEL_SPECS.values() if s.architecture]})")
     names = set(tensor_names)
     if any("block_sparse_moe" in n or "mlp.experts" in n for n in names):
-        raise ValueError("MoE checkpoints are not supported by pygpukit_amd")
+        raise ValueError("MoE checkpoints of the Hugging Face families are not supported by pygpukit_amd")
     if any("q_norm" in n for n in names):
         return QWEN3_SPEC
     if "model.embed_tokens.weight" in names:
@@ -163,10 +193,36 @@ def detect_model_spec(tensor_names: list[str], config: dict | None = None) -> Mo
 
 
 @dataclass(frozen=True)
+class ExpertsConfig:
+    """A layer's mixture of experts; with groups > 0 only experts of the `keep` best groups of neighbours can be chosen."""
+
+    count: int
+    top: int
+    groups: int
+    keep: int
+    scale: float                      # of the chosen experts' weights, which sum to it
+
+
+@dataclass(frozen=True)
+class LoopConfig:
+    """Layers start .. stop - 1 run `times` times with the same weights, every pass with caches of its own."""
+
+    start: int
+    stop: int
+    times: int
+
+    def runs(self, num_layers: int) -> list[tuple[int, int | None]]:
+        """(layer, number of the pass that starts with it or None) in the order they run."""
+        head = [(i, None) for i in range(self.start)]
+        body = [(i, t if i == self.start else None) for t in range(self.times) for i in range(self.start, self.stop)]
+        return head + body + [(i, None) for i in range(self.stop, num_layers)]
+
+
+@dataclass(frozen=True)
 class LayerConfig:
     """One layer of a layer-list model."""
 
-    mixer: Literal["latent_attention", "attention", "hgrn2"]
+    mixer: Literal["latent_attention", "attention", "hgrn2", "channel_delta", "mamba2"]
     num_heads: int
     head_dim: int                     # query / key width of a head
     v_head_dim: int                   # value width of a head
@@ -177,23 +233,48 @@ class LayerConfig:
     num_kv_heads: int = 0             # attention: key / value heads
     conv_taps: int | None = None      # attention: taps over time on q, k, v (None: no convolution)
     kv_from: int | None = None        # attention: the layer whose keys and values this one uses (None: its own)
+    # latent attention: rotated query / key columns beside head_dim's (0: none); pair i turns by position * base^(-2i / rot_dim)
+    rot_dim: int = 0
+    rot_base: float = 10000.0
+    norm_groups: int = 1              # state space: equal parts of the output that are normed on their own
+    experts: ExpertsConfig | None = None
+
+
+def parse_experts(i: int, mlp: dict) -> tuple[ExpertsConfig, int]:
+    r = mlp["router"]
+    g = r.get("groups")
+    e = ExpertsConfig(int(r["experts"]), int(r["top"]), int(g["count"]) if g else 0, int(g["keep"]) if g else 0, float(r.get("scale", 1.0)))
+    if not 1 <= e.top <= e.count or (e.groups and (e.count % e.groups or not 1 <= e.keep <= e.groups or e.keep * (e.count // e.groups) < e.top)):
+        raise ValueError(f"layer {i}: cannot choose {e.top} of {e.count} experts in {e.keep} of {e.groups} groups")
+    return e, int(mlp["expert"]["ff"])
 
 
 def parse_layer(i: int, entry: dict) -> LayerConfig:
     kind, mlp = entry.get("type"), entry.get("mlp")
-    if kind not in ("latent_attention", "attention", "hgrn2"):
+    if kind not in ("latent_attention", "attention", "hgrn2", "channel_delta", "mamba2"):
         raise ValueError(f"layer {i}: unknown mixer {kind!r}")
     m = entry["mixer"]
-    if mlp is not None and mlp.get("kind") != "dense":
+    if mlp is not None and mlp.get("kind") not in ("dense", "moe"):
         raise ValueError(f"layer {i}: unknown feed-forward {mlp.get('kind')!r}")
-    ff = int(mlp["ff"]) if mlp is not None else None
-    heads, dim, vdim = int(m["heads"]), int(m["dim"]), int(m["vdim"])
+    experts, ff = (None, None) if mlp is None else parse_experts(i, mlp) if mlp["kind"] == "moe" else (None, int(mlp["ff"]))
+    heads, vdim = int(m["heads"]), int(m["vdim"])
+    dim = int(m["state"] if kind == "mamba2" else m["dim"])
     if kind == "hgrn2":
-        return LayerConfig(kind, heads, dim, vdim, 0, None, 1.0, ff)
+        return LayerConfig(kind, heads, dim, vdim, 0, None, 1.0, ff, experts=experts)
+    if kind in ("channel_delta", "mamba2"):
+        lc = LayerConfig(kind, heads, dim, vdim, 0, None, 1.0, ff, int(m["kv_heads" if kind == "channel_delta" else "groups"]), int(m["conv"]),
+                         norm_groups=int(m.get("norm_groups", 1)), experts=experts)
+        if lc.num_kv_heads < 1 or heads % lc.num_kv_heads or heads * vdim % lc.norm_groups or lc.conv_taps < 1:
+            raise ValueError(f"layer {i}: {heads} heads of {vdim} over {lc.num_kv_heads} key heads, {lc.conv_taps} taps, {lc.norm_groups} norm groups")
+        return lc
     mask = m.get("mask")
     window = int(mask["size"]) if mask else None
     if kind == "latent_attention":
-        return LayerConfig(kind, heads, dim, vdim, int(m["kv_rank"]), window, float(m["scale"]), ff)
+        rot, rd = m.get("rot"), int(m.get("rot_dim", 0))
+        if rd % 2 or (rot is not None and int(rot["dims"]) != rd):
+            raise ValueError(f"layer {i}: {rd} rotated columns, rotation of {rot}")
+        return LayerConfig(kind, heads, dim, vdim, int(m["kv_rank"]), window, float(m["scale"]), ff, rot_dim=rd, rot_base=float(rot["base"]) if rot else 10000.0,
+                           experts=experts)
     taps, src = m.get("conv"), m.get("kv_from")
     return LayerConfig(kind, heads, dim, vdim, 0, window, float(m["scale"]), ff, int(m["kv_heads"]), int(taps) if taps is not None else None,
                        int(src) if src is not None else None)
@@ -220,10 +301,16 @@ def layer_list_config(config: dict) -> "TransformerConfig":
             if s is None or s.mixer != "attention" or s.kv_from is not None or (s.num_kv_heads, s.head_dim, s.v_head_dim) != (l.num_kv_heads, l.head_dim, l.v_head_dim):
                 raise ValueError(f"layer {i}: cannot take the keys and values of layer {l.kv_from}")
     first = layers[0]
+    loop = config.get("loop")
+    if loop is not None:
+        loop = LoopConfig(int(loop["start"]), int(loop["stop"]), int(loop["times"]))
+        if not 0 <= loop.start < loop.stop <= len(layers) or loop.times < 1 or any(l.kv_from is not None for l in layers):
+            raise ValueError(f"cannot run layers {loop.start} .. {loop.stop - 1} of {len(layers)} {loop.times} times")
     spec = next((s for s in MODEL_SPECS.values() if s.architecture == config.get("architecture")), TOTOLORN_SPEC)
     return TransformerConfig(vocab_size=int(config["vocab"]), hidden_size=int(config["width"]), num_layers=len(layers), num_heads=first.num_heads,
                              num_kv_heads=first.num_kv_heads or first.num_heads, intermediate_size=max([l.intermediate_size or 0 for l in layers]),
-                             _head_dim=first.head_dim, norm_type="rmsnorm", activation=spec.activation, use_rope=False,
+                             _head_dim=first.head_dim, norm_type=spec.norm_type, activation=spec.activation, use_rope=spec.use_rope, loop=loop,
+                             logit_scale=float(config.get("logit_scale", 1.0)),
                              max_position_embeddings=int(config["max_positions"]) if spec.use_position_embed else NO_POSITION_LIMIT,
                              norm_eps=float(config["norm"]["eps"]), tie_word_embeddings=False, layers=layers, residual_mult=float(config.get("residual_mult", 1.0)))
 
@@ -253,6 +340,8 @@ class TransformerConfig:
     tie_word_embeddings: bool = True
     layers: tuple[LayerConfig, ...] | None = None    # layer-list models: every layer's own sizes
     residual_mult: float = 1.0                       # factor of every sublayer's contribution to the residual stream
+    loop: LoopConfig | None = None                   # layer-list models: a stretch of layers that runs several times
+    logit_scale: float = 1.0                         # factor of the logits (the loader multiplies the output norm's weight by it)
 
     def __post_init__(self):
         if self.num_kv_heads is None:

@@ -15,6 +15,7 @@ from pygpukit_amd import _hip
 from pygpukit_amd.core.array import GPUArray
 from pygpukit_amd.core.dtypes import bfloat16, float32
 from pygpukit_amd.core.factory import from_numpy, zeros
+from pygpukit_amd.llm.config import LoopConfig
 from pygpukit_amd.ops.tensor import concat_axis0, pad_2d
 
 
@@ -338,20 +339,29 @@ def _pad_heads(v: np.ndarray, heads: int, pad: int, fill: float = 0.0) -> np.nda
     return out.reshape(*v.shape[:-1], heads * pad)
 
 
+def _pad_taps(taps: tuple[GPUArray, ...], heads: tuple[tuple[int, int], ...]) -> GPUArray:
+    """[taps, heads * d] each -> one [taps, all padded channels]"""
+    c = np.ascontiguousarray(np.concatenate([_pad_heads(_host_f32(t), h, p) for t, (h, p) in zip(taps, heads)], axis=1))
+    return from_numpy((c.view(np.uint32) >> 16).astype(np.uint16) if taps[0].dtype == bfloat16 else c)      # (bfloat16 values: the upper halves are exact)
+
+
 class StackEngine(Engine):
-    """The native engine for layer-list models (csrc/engine_stack.hip): fp32 residual stream, a norm after each sublayer and optionally
-    before it, a mixer per layer (latent attention, attention over a K/V ring, gated linear recurrence), every layer with its own
-    sizes.  State, graphs, sampling and generation are Engine's.
+    """The native engine for layer-list models (csrc/engine_stack.hip): fp32 residual stream, sandwich layers (a norm after each sublayer
+    and optionally before it) or parallel ones (one norm, mixer beside experts), a mixer per layer (latent attention, attention over
+    a K/V ring, linear recurrences, gated delta rule), every layer with its own sizes, possibly a stretch of layers that runs several
+    times.  State, graphs, sampling and generation are Engine's.
 
     The cache of an attention layer is a ring of min(window, max_seq_len) rows per sequence slot, that of a recurrent one a state: a
     sequence goes on where it stopped (or starts again at position 0); a position whose window or state has been overwritten is refused."""
 
     _SIZES = ("mixer", "ff", "heads", "kv_heads", "dim", "vdim", "rank", "window", "taps", "kv_from", "head_pad", "vhead_pad", "rank_pad", "n_att", "ff_pad")
+    _MORE = dict(gated=0, rot=0, norm_parts=1, rank_a=0, rank_g=0, experts=0, top=0, groups=0, keep=0)       # sizes of some layers, and their defaults
 
     def __init__(self, config: dict, embed: GPUArray, position_embed: GPUArray | None, head: GPUArray, final_norm: GPUArray, layers: list[dict], *,
                  max_seq_len: int = 512, max_batch: int = 1):
-        """config: vocab_size, width, max_positions, norm_eps, residual_mult.  layers[i]: the sizes and packed arrays of pack_layer(),
-        pack_attention() or pack_recurrence()."""
+        """config: vocab_size, width, max_positions, norm_eps, residual_mult; for parallel layers block and layer_norm, with a loop `loop`
+        (start, stop, times) and its arrays loop_in [wp, 2 wp], loop_step [times, wp].  layers[i]: the sizes and packed arrays of
+        pack_layer(), pack_attention(), pack_recurrence(), pack_delta() or pack_state_space()."""
         _hip.require_device()
         dt = embed.dtype
         if dt not in (bfloat16, float32):
@@ -366,18 +376,29 @@ class StackEngine(Engine):
             raise ValueError("StackEngine: embedding / head / final norm shapes do not match the configuration")
         if position_embed is not None and position_embed.shape != (config["max_positions"], config["width"]):
             raise ValueError(f"StackEngine: position table {position_embed.shape}")
+        parallel, loop = config.get("block", _hip.BLOCK_SANDWICH) == _hip.BLOCK_PARALLEL, config.get("loop")
+        self._runs = [i for i, _ in LoopConfig(*loop).runs(len(layers))] if loop else list(range(len(layers)))
         arr = (_hip.StackLayer * len(layers))()
         for i, lw in enumerate(layers):
             hd, gd = lw["heads"] * lw["head_pad"], 0 if lw["kv_from"] >= 0 else lw["kv_heads"] * lw["head_pad"]
-            ff, rp, n_in, n_att = lw["ff_pad"], lw["rank_pad"], lw["w_in"].shape[0], lw["n_att"]
+            moe, E = lw["ff_pad"] and lw["ff"] == _hip.FF_MOE, lw.get("experts", 0)
+            ff, rp, n_att, n_in = lw["ff_pad"], lw["rank_pad"], lw["n_att"], lw["w_in"].shape[0] - (_up64(E) if moe else 0)
             up = 2 * ff if lw["ff"] == _hip.FF_SWIGLU else ff
             # name -> (shape, dtype, may be absent)
-            want = {"norm1": ((1, wp), float32, True), "norm1b": ((1, wp), float32, False), "w_in": ((n_in, wp), dt, False), "w_o": ((wp, n_att), dt, False),
-                    "b_in": ((1, n_in), float32, True)}
-            if ff:
+            want = {"norm1": ((1, wp), float32, not parallel), "norm1b": ((1, wp), float32, parallel), "w_in": ((n_in + (_up64(E) if moe else 0), wp), dt, False),
+                    "w_o": ((wp, n_att), dt, False), "b_in": ((1, n_in), float32, True)}
+            if moe:
+                want.update(w_gate_up=((E, 2 * ff, wp), dt, False), w_down=((E, wp, ff), dt, False), correction=((E,), float32, False))
+            elif ff:
                 want.update(norm2=((1, wp), float32, True), norm2b=((1, wp), float32, False), w_gate_up=((up, wp), dt, False), w_down=((wp, ff), dt, False))
             if lw["mixer"] == _hip.MIX_LATENT:
-                want.update(c_norm=((1, rp), float32, False), w_ukv=((2 * hd, rp), dt, False))
+                want.update(c_norm=((1, rp), float32, False), w_ukv=((2 * hd, rp), dt, False), rot_freq=((lw.get("rot", 0) // 2,), float32, not lw.get("rot", 0)))
+            elif lw["mixer"] in (_hip.MIX_DELTA, _hip.MIX_SSD):
+                delta, hv = lw["mixer"] == _hip.MIX_DELTA, lw["heads"] * lw["vhead_pad"]
+                want.update(conv=((lw["taps"], hv + 2 * gd), dt, False), conv_bias=((1, hv + 2 * gd), float32, delta), decay=((lw["heads"],), float32, False),
+                            dt_bias=((1, hd if delta else lw["heads"]), float32, False), skip=((1, lw["heads"]), float32, delta),
+                            o_norm=((1, lw["vhead_pad"] if delta else hv), float32, False), w_a2=((hd, lw.get("rank_a", 0)), dt, not delta),
+                            w_g2=((hv, lw.get("rank_g", 0)), dt, not delta))
             elif lw["mixer"] == _hip.MIX_ATTENTION:
                 want.update(conv=((lw["taps"], hd + 2 * gd), dt, True), q_norm=((1, hd), float32, True), k_norm=((1, gd), float32, True),
                             slopes=((1, lw["heads"]), float32, True))
@@ -392,10 +413,18 @@ class StackEngine(Engine):
                 setattr(arr[i], name, t.data_ptr())
             for name in self._SIZES:
                 setattr(arr[i], name, lw[name])
-            arr[i].n_in, arr[i].scale = n_in, lw["scale"]
+            for name, default in self._MORE.items():
+                setattr(arr[i], name, lw.get(name, default))
+            arr[i].n_in, arr[i].scale, arr[i].router_scale = n_in, lw["scale"], lw.get("router_scale", 1.0)
             arr[i].act_pos, arr[i].act_neg = lw.get("act_params", (0.0, 0.0))
         sc = _hip.StackConfig(config["vocab_size"], config["width"], len(layers), config["max_positions"], max_seq_len, max_batch, config["norm_eps"],
-                              config["residual_mult"], dt.code)
+                              config["residual_mult"], dt.code, int(parallel), int(config.get("layer_norm", 0)))
+        if loop:
+            lin, step = config["loop_in"], config["loop_step"]
+            if lin.shape != (wp, 2 * wp) or lin.dtype != dt or step.shape != (loop[2], wp) or step.dtype != float32:
+                raise ValueError(f"StackEngine: loop input {lin.shape}, steps {step.shape}")
+            self._keep += [lin, step]
+            sc.loop_start, sc.loop_stop, sc.loop_times, sc.loop_in, sc.loop_step = *loop, lin.data_ptr(), step.data_ptr()
         h = C.c_void_p()
         _hip.call("pgk_engine_create_stack", C.byref(sc), embed._p, position_embed._p if position_embed is not None else None, head._p, final_norm._p,
                   arr, C.byref(h))
@@ -404,12 +433,12 @@ class StackEngine(Engine):
         self.last_prefill_logits = None
 
     @staticmethod
-    def _pack_common(width: int, norm1: GPUArray | None, norm1b: GPUArray, gate_up: GPUArray | None, down: GPUArray | None, norm2: GPUArray | None,
+    def _pack_common(width: int, norm1: GPUArray | None, norm1b: GPUArray | None, gate_up: GPUArray | None, down: GPUArray | None, norm2: GPUArray | None,
                      norm2b: GPUArray | None, act_params: tuple[float, float] | None) -> dict:
         """Norms and feed-forward of a layer.  gate_up: the SwiGLU matrix [2 ff, width], or with act_params (xIELU's two factors)
         the up-projection [ff, width]."""
         wp = _up64(width)
-        out = dict(norm1=None if norm1 is None else _row(norm1, wp), norm1b=_row(norm1b, wp), ff_pad=0, ff=_hip.FF_SWIGLU if act_params is None else _hip.FF_XIELU,
+        out = dict(norm1=None if norm1 is None else _row(norm1, wp), norm1b=None if norm1b is None else _row(norm1b, wp), ff_pad=0, ff=_hip.FF_SWIGLU if act_params is None else _hip.FF_XIELU,
                    rank=0, rank_pad=0, kv_from=-1, taps=1, window=NO_WINDOW, scale=1.0)
         if act_params is not None:
             out["act_params"] = act_params
@@ -424,18 +453,21 @@ class StackEngine(Engine):
         return out
 
     @classmethod
-    def pack_layer(cls, q: GPUArray, kv_down: GPUArray, head_gate: GPUArray, kv_norm: GPUArray, k_up: GPUArray, v_up: GPUArray, o: GPUArray, norm1: GPUArray,
-                   norm1b: GPUArray, *, heads: int, dim: int, vdim: int, window: int, scale: float, gate_up: GPUArray | None = None,
+    def pack_layer(cls, q: GPUArray, kv_down: GPUArray, head_gate: GPUArray | None, kv_norm: GPUArray, k_up: GPUArray, v_up: GPUArray, o: GPUArray, norm1: GPUArray,
+                   norm1b: GPUArray | None, *, rot_freq: GPUArray | None = None, heads: int, dim: int, vdim: int, window: int, scale: float, gate_up: GPUArray | None = None,
                    down: GPUArray | None = None, norm2: GPUArray | None = None, norm2b: GPUArray | None = None,
                    act_params: tuple[float, float] | None = None) -> dict:
         """One latent-attention layer's matrices ([out, in]; norms fp32 with offsets applied) -> the engine's padded layout: head widths to
-        64 / 128 / a multiple of 64, every other width to a multiple of 64.  Arrays that already fit are used as they are."""
-        width, rank = q.shape[1], kv_down.shape[0]
-        wp, rp, hp = _up64(width), _up64(rank), _attention_pad(dim, vdim)
+        64 / 128 / a multiple of 64, every other width to a multiple of 64.  Arrays that already fit are used as they are.  rot_freq [rot / 2]:
+        the last rot of the dim query columns, and of kv_down's rows, are the rotated part (k_up and v_up take all of a cached row)."""
+        rot = 0 if rot_freq is None else 2 * rot_freq.size
+        width, rank = q.shape[1], kv_down.shape[0] - rot
+        wp, rp, hp = _up64(width), _up64(rank + rot), _attention_pad(dim, vdim)
         hd = heads * hp
         out = cls._pack_common(width, norm1, norm1b, gate_up, down, norm2, norm2b, act_params)
         out.update(mixer=_hip.MIX_LATENT, heads=heads, kv_heads=heads, dim=dim, vdim=vdim, rank=rank, window=window, scale=scale, head_pad=hp, vhead_pad=hp, rank_pad=rp,
-                   n_att=hd, w_in=_stack_rows([_head_rows(q, heads, dim, hp, wp), pad_2d(kv_down, rp, wp), pad_2d(head_gate, heads, wp)]), c_norm=_row(kv_norm, rp),
+                   gated=int(head_gate is not None), rot=rot, rot_freq=rot_freq, n_att=hd,
+                   w_in=_stack_rows([_head_rows(q, heads, dim, hp, wp), pad_2d(kv_down, rp, wp)] + ([] if head_gate is None else [pad_2d(head_gate, heads, wp)])), c_norm=_row(kv_norm, rp),
                    w_ukv=concat_axis0(_head_rows(k_up, heads, dim, hp, rp), _head_rows(v_up, heads, vdim, hp, rp)), w_o=_head_cols(o, heads, vdim, hp, wp, hd))
         return out
 
@@ -492,9 +524,94 @@ class StackEngine(Engine):
         return out
 
     @classmethod
-    def _pack_block(cls, b, c) -> dict:
-        from pygpukit_amd.llm.layers import GatedRecurrence, GatedWindowAttention, LatentAttention
+    def pack_delta(cls, q: GPUArray, k: GPUArray, v: GPUArray, strength: GPUArray, decay_maps: tuple[GPUArray, GPUArray], gate_maps: tuple[GPUArray, GPUArray], o: GPUArray,
+                   taps: tuple[GPUArray, GPUArray, GPUArray], decay: GPUArray, step_bias: GPUArray, head_norm: GPUArray, norm1: GPUArray | None,
+                   norm1b: GPUArray | None = None, *, heads: int, kv_heads: int, dim: int, vdim: int) -> dict:
+        """One layer of the gated delta rule: matrices [out, in], taps of q, k, v [taps, channels]; fp32 decay [heads], step_bias [heads * dim],
+        head_norm [vdim].  Head widths up to 32 / 64 / 128 / a multiple of 16 (keys) and of 16 (values); padding channels stay zero."""
+        width = q.shape[1]
+        wp, vp = _up64(width), _up(vdim, 16)
+        dp = next((p for p in (32, 64, 128) if dim <= p), _up(dim, 16))
+        ra, rg = (_up64(m[0].shape[0]) for m in (decay_maps, gate_maps))
+        channels = 2 * kv_heads * dp + heads * vp
+        w_in = _stack_rows([_head_rows(q, kv_heads, dim, dp, wp), _head_rows(k, kv_heads, dim, dp, wp), _head_rows(v, heads, vdim, vp, wp),
+                            pad_2d(strength, _up64(channels + heads) - channels, wp), pad_2d(decay_maps[0], ra, wp), pad_2d(gate_maps[0], rg, wp)])
+        n_att = _up64(heads * vp)
+        out = cls._pack_common(width, norm1, norm1b, None, None, None, None, None)
+        out.update(mixer=_hip.MIX_DELTA, heads=heads, kv_heads=kv_heads, dim=dim, vdim=vdim, head_pad=dp, vhead_pad=vp, rank_a=ra, rank_g=rg, n_att=n_att, w_in=w_in,
+                   taps=taps[0].shape[0], conv=_pad_taps(taps, ((kv_heads, dp), (kv_heads, dp), (heads, vp))), decay=decay,
+                   dt_bias=from_numpy(_pad_heads(_host_f32(step_bias).reshape(1, -1), heads, dp)), o_norm=_row(head_norm, vp),
+                   w_a2=_head_rows(decay_maps[1], heads, dim, dp, ra), w_g2=_head_rows(gate_maps[1], heads, vdim, vp, rg), w_o=_head_cols(o, heads, vdim, vp, wp, n_att))
+        return out
 
+    @classmethod
+    def pack_state_space(cls, z: GPUArray, xbc: GPUArray, t: GPUArray, o: GPUArray, taps: GPUArray, taps_bias: GPUArray, decay: GPUArray, step_bias: GPUArray, skip: GPUArray,
+                         out_norm: GPUArray, norm1: GPUArray | None, norm1b: GPUArray | None = None, *, heads: int, groups: int, dim: int, vdim: int, norm_parts: int) -> dict:
+        """One state-space layer: rows of z [heads * vdim, width], x | B | C and t [heads, width]; taps [taps, channels of x | B | C]; fp32 taps_bias,
+        decay, step_bias, skip [heads], out_norm [heads * vdim]."""
+        width = z.shape[1]
+        wp, dp, vp = _up64(width), _up(dim, 16), _up(vdim, 16)
+        v, g = heads * vdim, groups * dim
+        sizes, heads_of = (v, g, g), ((heads, vp), (groups, dp), (groups, dp))
+        at = (0, v, v + g)
+        cut = lambda i: xbc._view(at[i] * width, (sizes[i], width))  # noqa: E731
+        w_in = _stack_rows([_head_rows(cut(0), heads, vdim, vp, wp), _head_rows(cut(1), groups, dim, dp, wp), _head_rows(cut(2), groups, dim, dp, wp),
+                            _head_rows(z, heads, vdim, vp, wp), pad_2d(t, heads, wp)])
+        n_att = _up64(heads * vp)
+        host = taps.to_numpy()
+        parts = tuple(from_numpy(host[:, a:a + n]) for a, n in zip(at, sizes))
+        bias = _host_f32(taps_bias).reshape(1, -1)
+        out = cls._pack_common(width, norm1, norm1b, None, None, None, None, None)
+        out.update(mixer=_hip.MIX_SSD, heads=heads, kv_heads=groups, dim=dim, vdim=vdim, head_pad=dp, vhead_pad=vp, n_att=n_att, w_in=w_in, norm_parts=norm_parts,
+                   taps=taps.shape[0], conv=_pad_taps(parts, heads_of), decay=decay, dt_bias=step_bias.view((1, heads)), skip=skip.view((1, heads)),
+                   conv_bias=from_numpy(np.concatenate([_pad_heads(bias[:, a:a + n], h, p) for a, n, (h, p) in zip(at, sizes, heads_of)], axis=1)),
+                   o_norm=from_numpy(_pad_heads(_host_f32(out_norm).reshape(1, -1), heads, vp)), w_o=_head_cols(o, heads, vdim, vp, wp, n_att))
+        return out
+
+    @staticmethod
+    def add_experts(layer: dict, width: int, router: GPUArray, correction: GPUArray, gate_up: GPUArray, down: GPUArray, *, top: int, groups: int = 0, keep: int = 0,
+                    scale: float = 1.0) -> dict:
+        """A packed mixer plus its layer's experts: router [E, width], gate_up [E, 2 ff, width], down [E, width, ff], correction fp32 [E].  The
+        router's rows go behind the mixer's in w_in."""
+        E, two_ff, _ = gate_up.shape
+        ff, wp = two_ff // 2, _up64(width)
+        fp = _up64(ff)
+        layer.update(ff=_hip.FF_MOE, ff_pad=fp, experts=E, top=top, groups=groups, keep=keep, router_scale=scale, correction=correction,
+                     w_in=concat_axis0(layer["w_in"], pad_2d(router, _up64(E), wp)),
+                     w_gate_up=_head_rows(gate_up.view((2 * E * ff, width)), 2 * E, ff, fp, wp).view((E, 2 * fp, wp)),
+                     w_down=_head_rows(down.view((E * width, ff)), E, width, wp, fp).view((E, wp, fp)))
+        return layer
+
+    @classmethod
+    def _pack_parallel(cls, b) -> dict:
+        from pygpukit_amd.llm.layers import ChannelDelta, LatentAttention, StateSpace
+
+        a, norm = b.attn, b.attn_norm.weight
+        if isinstance(a, LatentAttention):
+            out = cls.pack_layer(a.q_proj.weight, a.kv_down.weight, None if a.head_gate is None else a.head_gate.weight, a.kv_norm.weight, a.k_up.weight, a.v_up.weight,
+                                 a.o_proj.weight, norm, None, heads=a.num_heads, dim=a.head_dim + a.rot_dim, vdim=a.v_head_dim, window=a.window, scale=a.scale, rot_freq=a.rot_freq)
+        elif isinstance(a, ChannelDelta):
+            w = lambda maps: tuple(m.weight for m in maps)  # noqa: E731
+            out = cls.pack_delta(a.q_proj.weight, a.k_proj.weight, a.v_proj.weight, a.strength.weight, w(a.decay_maps), w(a.gate_maps), a.o_proj.weight, a.taps, a.decay, a.step_bias,
+                                 a.head_norm, norm, heads=a.num_heads, kv_heads=a.num_kv_heads, dim=a.head_dim, vdim=a.v_head_dim)
+        elif isinstance(a, StateSpace):
+            out = cls.pack_state_space(a.z_proj.weight, a.xbc_proj.weight, a.t_proj.weight, a.o_proj.weight, a.taps, a.taps_bias, a.decay, a.step_bias, a.skip, a.out_norm, norm,
+                                       heads=a.num_heads, groups=a.num_groups, dim=a.head_dim, vdim=a.v_head_dim, norm_parts=a.norm_groups)
+        else:
+            raise NotImplementedError(f"the layer-list engine has no parallel layer of {type(a).__name__}")
+        m = b.mlp
+        if m is not None:
+            cls.add_experts(out, m.router.shape[1], m.router, m.correction, m.gate_up, m.down, top=m.top, groups=m.groups, keep=m.keep, scale=m.scale)
+        return out
+
+    @classmethod
+    def _pack_block(cls, b, c) -> dict:
+        from pygpukit_amd.llm.layers import GatedRecurrence, GatedWindowAttention, LatentAttention, ParallelBlock
+
+        if isinstance(b, ParallelBlock):
+            if b.attn_norm.eps != c.norm_eps or b.attn_norm.norm_type != c.norm_type:
+                raise NotImplementedError("the layer-list engine takes one kind of norm and one epsilon for all layers")
+            return cls._pack_parallel(b)
         a = b.attn
         if b.post_attn_norm is None or (b.mlp is not None and b.post_mlp_norm is None):
             raise NotImplementedError("the layer-list engine needs a norm after each sublayer")
@@ -513,7 +630,7 @@ class StackEngine(Engine):
             if a.head_gate is None or b.attn_norm is None:
                 raise NotImplementedError("the layer-list engine needs a norm before gated latent attention")
             return cls.pack_layer(a.q_proj.weight, a.kv_down.weight, a.head_gate.weight, a.kv_norm.weight, a.k_up.weight, a.v_up.weight, a.o_proj.weight, *norms,
-                                  heads=a.num_heads, dim=a.head_dim, vdim=a.v_head_dim, window=a.window, scale=a.scale, **common)
+                                  rot_freq=a.rot_freq, heads=a.num_heads, dim=a.head_dim + a.rot_dim, vdim=a.v_head_dim, window=a.window, scale=a.scale, **common)
         if isinstance(a, GatedWindowAttention):
             own = a.source is None
             return cls.pack_attention(a.q_proj.weight, a.k_proj.weight if own else None, a.v_proj.weight if own else None, a.out_gate.weight, a.o_proj.weight, *norms,
@@ -537,10 +654,27 @@ class StackEngine(Engine):
             wp = _up64(width)
             model._stack_layers = packed
             model._stack_head = (pad_2d(head, head.shape[0], wp), _row(model.final_norm.weight, wp))
+            model._stack_more = cls._pack_more(model, width)
         head, fnorm = model._stack_head
         cfg = dict(vocab_size=model.embed_tokens.shape[0], width=width, hidden_size=width, max_positions=c.max_position_embeddings, norm_eps=c.norm_eps,
-                   residual_mult=c.residual_mult)
+                   residual_mult=c.residual_mult, **model._stack_more)
         return cls(cfg, model.embed_tokens, model.position_embed, head, fnorm, packed, max_seq_len=max_seq_len, max_batch=max_batch)
+
+    @staticmethod
+    def _pack_more(model, width: int) -> dict:
+        """What parallel layers and a loop add to the engine's configuration."""
+        from pygpukit_amd.llm.layers import ParallelBlock
+
+        parallel = [isinstance(b, ParallelBlock) for b in model.blocks]
+        if not any(parallel):
+            return {}
+        if not all(parallel):
+            raise NotImplementedError("the layer-list engine takes parallel or sandwich layers, not both")
+        out: dict = dict(block=_hip.BLOCK_PARALLEL, layer_norm=int(model.final_norm.norm_type == "layernorm"))
+        if model.loop is not None:
+            l, wp = model.config.loop, _up64(width)
+            out.update(loop=(l.start, l.stop, l.times), loop_in=_head_cols(model.loop.weight, 2, width, wp, wp, 2 * wp), loop_step=pad_2d(model.loop.step, l.times, wp))
+        return out
 
     def _layer_memory(self, layer: int, shape: tuple[int, ...], dtype) -> GPUArray:
         p, none = C.c_void_p(), C.c_void_p()
@@ -550,16 +684,17 @@ class StackEngine(Engine):
         return a
 
     def latent_cache(self, layer: int) -> GPUArray:
-        """[max_batch, R, rank_pad] view of layer `layer`'s latent rings: position p of a sequence is row p % R, R = min(window, max_seq_len)."""
-        lw = self.layers[layer]
+        """[max_batch, R, rank_pad] view of layer `layer`'s latent rings: position p of a sequence is row p % R, R = min(window, max_seq_len).
+        (With a loop, here and below: of run `layer`, one pass of one layer in the order they run.)"""
+        lw = self.layers[self._runs[layer]]
         if lw["mixer"] != _hip.MIX_LATENT:
             raise ValueError(f"layer {layer} caches no latents")
         return self._layer_memory(layer, (self.max_batch, min(lw["window"], self.max_seq_len), lw["rank_pad"]), self.dtype)
 
     def recurrent_state(self, layer: int) -> GPUArray:
         """float32 [max_batch, heads, dim, vdim] (widths padded) view of layer `layer`'s states."""
-        lw = self.layers[layer]
-        if lw["mixer"] != _hip.MIX_HGRN2:
+        lw = self.layers[self._runs[layer]]
+        if lw["mixer"] not in (_hip.MIX_HGRN2, _hip.MIX_DELTA, _hip.MIX_SSD):
             raise ValueError(f"layer {layer} has no recurrent state")
         return self._layer_memory(layer, (self.max_batch, lw["heads"], lw["head_pad"], lw["vhead_pad"]), float32)
 

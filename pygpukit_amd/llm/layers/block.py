@@ -1,21 +1,34 @@
 """Transformer block (reference: src/pygpukit/llm/layers/block.py:18-57): pre-norm attention and MLP with
 residual adds.  Layer-list models add a norm on each sublayer's output (with or without one on its input), a factor on its
-contribution and layers without MLP."""
+contribution and layers without MLP, or run mixer and experts side by side (ParallelBlock)."""
 
 from __future__ import annotations
 
 from pygpukit_amd.core.array import GPUArray
 from pygpukit_amd.core.dtypes import float16, float32
-from pygpukit_amd.ops.basic import add, cast_f32_to_bf16, cast_f32_to_f16
+from pygpukit_amd.core.factory import from_numpy
+from pygpukit_amd.ops.basic import add, add_inplace, bias_add_inplace, cast_bf16_to_f32, cast_f16_to_f32, cast_f32_to_bf16, cast_f32_to_f16
 
 from .attention import Attention
+from .delta import ChannelDelta
+from .experts import MixtureOfExperts
 from .latent_attention import LatentAttention
+from .linear import LinearBF16
 from .mlp import MLP
 from .norm import Norm
 from .recurrence import GatedRecurrence
+from .state_space import StateSpace
 from .window_attention import GatedWindowAttention
 
-Mixer = Attention | LatentAttention | GatedWindowAttention | GatedRecurrence
+Mixer = Attention | LatentAttention | GatedWindowAttention | GatedRecurrence | ChannelDelta | StateSpace
+
+
+def _narrow(x: GPUArray, dtype) -> GPUArray:
+    return x if dtype == float32 else cast_f32_to_f16(x) if dtype == float16 else cast_f32_to_bf16(x)
+
+
+def _wide(x: GPUArray) -> GPUArray:
+    return x if x.dtype == float32 else cast_f16_to_f32(x) if x.dtype == float16 else cast_bf16_to_f32(x)
 
 
 class TransformerBlock:
@@ -28,8 +41,7 @@ class TransformerBlock:
         """What a sublayer reads: the norm of the stream, or without a norm the stream itself in the sublayer's element type."""
         if norm is not None:
             return norm(x)
-        dt = post.stream_dtype
-        return x if dt == float32 else cast_f32_to_f16(x) if dt == float16 else cast_f32_to_bf16(x)
+        return _narrow(x, post.stream_dtype)
 
     def add_attn(self, x: GPUArray, y: GPUArray) -> GPUArray:
         return add(x, y) if self.post_attn_norm is None else self.post_attn_norm.add_to(x, y, self.residual_mult)
@@ -54,4 +66,51 @@ class TransformerBlock:
         return self.add_mlp(self.add_attn(x, attn(self._enter(self.attn_norm, x, self.post_attn_norm), position, context_len)))
 
 
-__all__ = ["TransformerBlock"]
+class ParallelBlock:
+    """x += mixer(h) + experts(h) with h = norm(x): one norm, an fp32 stream, experts or none."""
+
+    residual_mult = 1.0
+
+    def __init__(self, norm: Norm, attn: Mixer, mlp: MixtureOfExperts | None):
+        self.attn_norm, self.attn, self.mlp = norm, attn, mlp
+
+    def _add(self, x: GPUArray, h: GPUArray, y: GPUArray) -> GPUArray:
+        y = _wide(y)
+        if self.mlp is not None:
+            add_inplace(y, self.mlp(h))
+        return add(x, y)
+
+    def __call__(self, x: GPUArray, position_ids: list[int] | None = None, past_kv: tuple | None = None,
+                 use_cache: bool = False, source_kv: tuple | None = None) -> tuple[GPUArray, tuple | None]:
+        h = self.attn_norm(x)
+        y, present_kv = self.attn(h, position_ids, past_kv, use_cache)
+        return self._add(x, h, y), present_kv
+
+    def forward_fixed_cache(self, x: GPUArray, position: int, context_len: int) -> GPUArray:
+        h = self.attn_norm(x)
+        return self._add(x, h, self.attn.forward_fixed_cache_batch(h, position, context_len))
+
+
+class LoopInput:
+    """What a pass of a looped stretch starts with: x <- W_x x + W_e e + step[pass], e the embedding rows."""
+
+    def __init__(self, weight: GPUArray, step: GPUArray):
+        """weight [hidden, 2 hidden]; step float32 [passes, hidden]."""
+        hidden = weight.shape[0]
+        if weight.shape != (hidden, 2 * hidden) or step.ndim != 2 or step.shape[1] != hidden or step.dtype != float32:
+            raise ValueError(f"LoopInput: weight {weight.shape}, step {step.shape}")
+        self.weight, self.step = weight, step
+        self._halves: tuple[LinearBF16, LinearBF16] | None = None
+
+    def __call__(self, x: GPUArray, e: GPUArray, t: int) -> GPUArray:
+        hidden, dt = x.shape[1], self.weight.dtype
+        if self._halves is None:
+            w = self.weight.to_numpy()
+            self._halves = tuple(LinearBF16(from_numpy(w[:, i * hidden:(i + 1) * hidden])) for i in (0, 1))
+        y = _wide(self._halves[0](_narrow(x, dt)))
+        add_inplace(y, _wide(self._halves[1](_narrow(e, dt))))
+        bias_add_inplace(y, self.step._view(t * hidden, (hidden,)))
+        return y
+
+
+__all__ = ["TransformerBlock", "ParallelBlock", "LoopInput"]

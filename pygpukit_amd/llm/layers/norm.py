@@ -6,7 +6,7 @@ from typing import Literal
 
 from pygpukit_amd.core.array import GPUArray
 from pygpukit_amd.core.dtypes import DataType, float32
-from pygpukit_amd.ops.basic import layernorm, rmsnorm, rmsnorm_add_f32, rmsnorm_f32
+from pygpukit_amd.ops.basic import layernorm, layernorm_f32, rmsnorm, rmsnorm_add_f32, rmsnorm_f32
 
 
 class Norm:
@@ -17,15 +17,19 @@ class Norm:
                  norm_type: Literal["rmsnorm", "layernorm"] = "rmsnorm", eps: float = 1e-5, stream_dtype: DataType | None = None):
         self.weight, self.bias, self.norm_type, self.eps = weight, bias, norm_type, eps
         self.stream_dtype = stream_dtype
-        if stream_dtype is not None and (norm_type != "rmsnorm" or weight.dtype != float32):
-            raise ValueError("an fp32-stream norm is an RMSNorm with a float32 weight")
+        if stream_dtype is not None and (bias is not None or weight.dtype != float32):
+            raise ValueError("an fp32-stream norm has a float32 weight and no bias")
 
     def add_to(self, stream: GPUArray, y: GPUArray, mult: float = 1.0) -> GPUArray:
         """stream += mult * norm(y), in place."""
+        if self.norm_type != "rmsnorm":
+            raise NotImplementedError("a layer norm of a sublayer's output")
         return rmsnorm_add_f32(stream, y, self.weight, self.eps, mult)
 
     def __call__(self, x: GPUArray, *, out: GPUArray | None = None) -> GPUArray:
         if self.stream_dtype is not None:
+            if self.norm_type == "layernorm":
+                return layernorm_f32(x, self.weight, self.eps, dtype=self.stream_dtype, out=out)
             return rmsnorm_f32(x, self.weight, self.eps, dtype=self.stream_dtype, out=out)
         if self.norm_type == "rmsnorm":
             return rmsnorm(x, self.weight, self.eps, out=out)

@@ -2,22 +2,25 @@
 CausalTransformerModel, architecture and dimensions inferred from tensor names and shapes exactly as the reference does
 (detect_model_spec; head_dim from the QK-norm weight or the 128/64/256 probe; rope_theta / rms_norm_eps and the FP8
 `quantization_config` from a sibling config.json).  Tensors whose stored dtype equals the target dtype go from the file
-mapping straight to device memory; others are converted on the host first.  MoE checkpoints are out of scope."""
+mapping straight to device memory; others are converted on the host first.  Experts are served in the layer-list families only."""
 
 from __future__ import annotations
 
+import ctypes as C
 import json
 import os
 from dataclasses import dataclass
 
 import numpy as np
 
+from pygpukit_amd import _hip
 from pygpukit_amd.core.array import GPUArray
 from pygpukit_amd.core.dtypes import bfloat16, float16, float32, uint8
 from pygpukit_amd.core.factory import from_numpy
-from pygpukit_amd.llm.config import (GPT2_SPEC, LLAMA_SPEC, MALASUN_SPEC, QWEN3_SPEC, TOTOLORN_SPEC, LayerConfig, ModelSpec, TransformerConfig,
+from pygpukit_amd.llm.config import (GPT2_SPEC, LLAMA_SPEC, MALASUN_SPEC, QWEN3_SPEC, RATASUN_SPEC, TOTOLORN_SPEC, LayerConfig, ModelSpec, TransformerConfig,
                                      detect_model_spec, distance_slopes, layer_list_config)
-from pygpukit_amd.llm.layers import MLP, Attention, GatedRecurrence, GatedWindowAttention, LatentAttention, Norm, TransformerBlock
+from pygpukit_amd.llm.layers import (MLP, Attention, ChannelDelta, GatedRecurrence, GatedWindowAttention, LatentAttention, LoopInput, MixtureOfExperts, Norm,
+                                     ParallelBlock, StateSpace, TransformerBlock)
 from pygpukit_amd.llm.layers.linear import LinearBF16, LinearFP8
 from pygpukit_amd.llm.models.causal import CausalTransformerModel
 from pygpukit_amd.llm.safetensors import Dtype, load_safetensors
@@ -219,19 +222,22 @@ def _load_layer_list(st, spec: ModelSpec, config: dict, dtype, load_tensor, try_
             raise ValueError(f"{name}: missing or not of {size} elements")
         return np.ascontiguousarray(st.tensor_as_f32(name), dtype=np.float32).reshape(size)
 
-    def norm(name: str, width: int, offset: float, scalar: bool = False) -> Norm:
+    def norm(name: str, width: int, offset: float, scalar: bool = False, kind: str = "rmsnorm", mult: float = 1.0) -> Norm:
         w = np.repeat(fp32(name, 1), width) if scalar else fp32(name, width)
-        return Norm(from_numpy(w + np.float32(offset)), None, "rmsnorm", cfg.norm_eps, stream_dtype=dtype)
+        return Norm(from_numpy((w + np.float32(offset)) * np.float32(mult)), None, kind, cfg.norm_eps, stream_dtype=dtype)
 
     H, off, one = cfg.hidden_size, spec.norm_weight_offset, spec.norm_scalar
     blocks: list[TransformerBlock] = []
 
     def latent_mixer(lc: LayerConfig, nm) -> LatentAttention:
-        return LatentAttention(tensor(nm(spec.q_proj), (lc.num_heads * lc.head_dim, H)), tensor(nm(spec.kv_down_proj), (lc.kv_rank, H)),
+        rot = lc.rot_dim
+        freq = from_numpy((lc.rot_base ** (-2.0 * np.arange(rot // 2) / rot)).astype(np.float32)) if rot else None
+        gate = tensor(nm(spec.head_gate), (lc.num_heads, H)) if spec.head_gate else None
+        return LatentAttention(tensor(nm(spec.q_proj), (lc.num_heads * (lc.head_dim + rot), H)), tensor(nm(spec.kv_down_proj), (lc.kv_rank + rot, H)),
                                norm(nm(spec.kv_down_norm), lc.kv_rank, 0.0), tensor(nm(spec.k_up_proj), (lc.num_heads * lc.head_dim, lc.kv_rank)),
                                tensor(nm(spec.v_up_proj), (lc.num_heads * lc.v_head_dim, lc.kv_rank)),
                                tensor(nm(spec.o_proj), (H, lc.num_heads * lc.v_head_dim)), num_heads=lc.num_heads, head_dim=lc.head_dim,
-                               v_head_dim=lc.v_head_dim, scale=lc.scale, window=lc.window, head_gate=tensor(nm(spec.head_gate), (lc.num_heads, H)))
+                               v_head_dim=lc.v_head_dim, scale=lc.scale, window=lc.window, head_gate=gate, rot_dim=rot, rot_freq=freq)
 
     def attention_mixer(lc: LayerConfig, nm) -> GatedWindowAttention:
         q, k, v = lc.num_heads * lc.head_dim, lc.num_kv_heads * lc.head_dim, lc.num_kv_heads * lc.v_head_dim
@@ -257,14 +263,63 @@ def _load_layer_list(st, spec: ModelSpec, config: dict, dtype, load_tensor, try_
                                from_numpy(fp32(nm(spec.forget_bias), qk)), from_numpy(fp32(nm(spec.forget_lower), qk)), from_numpy(fp32(nm(spec.head_norm), lc.v_head_dim)),
                                num_heads=lc.num_heads, head_dim=lc.head_dim, v_head_dim=lc.v_head_dim, eps=cfg.norm_eps)
 
-    mixers = {"latent_attention": (latent_mixer, spec.kv_down_proj), "attention": (attention_mixer, spec.out_gate), "hgrn2": (recurrent_mixer, spec.forget_proj)}
+    def decay_rates(name: str, heads: int) -> GPUArray:
+        return from_numpy(np.exp(fp32(name, heads).astype(np.float64)).astype(np.float32))
+
+    def rows_of(name: str) -> int:
+        if name not in st or len(st.tensor_info(name).shape) != 2:
+            raise ValueError(f"checkpoint has no matrix {name!r}")
+        return int(st.tensor_info(name).shape[0])
+
+    def taps(name: str, channels: int, n: int) -> GPUArray:
+        return _transposed(tensor(name, (channels, n)))
+
+    def delta_mixer(lc: LayerConfig, nm) -> ChannelDelta:
+        k, q, v, n = lc.num_kv_heads * lc.head_dim, lc.num_heads * lc.head_dim, lc.num_heads * lc.v_head_dim, lc.conv_taps
+
+        def maps(down: str, up: str, rows: int) -> tuple[GPUArray, GPUArray]:
+            rank = rows_of(nm(down))
+            return tensor(nm(down), (rank, H)), tensor(nm(up), (rows, rank))
+
+        return ChannelDelta(tensor(nm(spec.q_proj), (k, H)), tensor(nm(spec.k_proj), (k, H)), tensor(nm(spec.v_proj), (v, H)), tensor(nm(spec.o_proj), (H, v)),
+                            tensor(nm(spec.strength), (lc.num_heads, H)), maps(spec.decay_down, spec.decay_up, q), maps(spec.gate_down, spec.gate_up, v),
+                            (taps(nm(spec.q_conv), k, n), taps(nm(spec.k_conv), k, n), taps(nm(spec.v_conv), v, n)), decay_rates(nm(spec.decay_log), lc.num_heads),
+                            from_numpy(fp32(nm(spec.step_bias), q)), from_numpy(fp32(nm(spec.head_norm), lc.v_head_dim)), num_heads=lc.num_heads,
+                            num_kv_heads=lc.num_kv_heads, head_dim=lc.head_dim, v_head_dim=lc.v_head_dim, eps=cfg.norm_eps)
+
+    def state_space_mixer(lc: LayerConfig, nm) -> StateSpace:
+        v, ch, heads = lc.num_heads * lc.v_head_dim, lc.num_heads * lc.v_head_dim + 2 * lc.num_kv_heads * lc.head_dim, lc.num_heads
+        w = tensor(nm(spec.in_proj), (v + ch + heads, H))
+        parts = (w._view(0, (v, H)), w._view(v * H, (ch, H)), w._view((v + ch) * H, (heads, H)))
+        return StateSpace(parts, tensor(nm(spec.o_proj), (H, v)), taps(nm(spec.conv), ch, lc.conv_taps), from_numpy(fp32(nm(spec.conv_bias), ch)),
+                          decay_rates(nm(spec.decay_log), heads), from_numpy(fp32(nm(spec.step_bias), heads)), from_numpy(fp32(nm(spec.skip), heads)),
+                          from_numpy(fp32(nm(spec.out_norm), v)), num_heads=heads, num_groups=lc.num_kv_heads, state_dim=lc.head_dim, v_head_dim=lc.v_head_dim,
+                          norm_groups=lc.norm_groups, eps=cfg.norm_eps)
+
+    def expert_mlp(lc: LayerConfig, nm) -> MixtureOfExperts:
+        e, I = lc.experts, lc.intermediate_size
+        gate_up, down = GPUArray((e.count, 2 * I, H), dtype), GPUArray((e.count, H, I), dtype)
+        for k in range(e.count):
+            for out, at, pattern, shape in ((gate_up, 2 * k, spec.expert_gate_proj, (I, H)), (gate_up, 2 * k + 1, spec.expert_up_proj, (I, H)), (down, k, spec.expert_down_proj, (H, I))):
+                w = tensor(nm(pattern, expert=k), shape)
+                _hip.call("pgk_memcpy_d2d", C.c_void_p(out.data_ptr() + at * w.nbytes), w._p, w.nbytes, None)
+        return MixtureOfExperts(tensor(nm(spec.router), (e.count, H)), from_numpy(fp32(nm(spec.router_correction), e.count)), gate_up, down, top=e.top, groups=e.groups,
+                                keep=e.keep, scale=e.scale)
+
+    mixers = {"latent_attention": (latent_mixer, spec.kv_down_proj), "attention": (attention_mixer, spec.out_gate), "hgrn2": (recurrent_mixer, spec.forget_proj),
+              "channel_delta": (delta_mixer, spec.decay_down), "mamba2": (state_space_mixer, spec.in_proj)}
     for i, lc in enumerate(cfg.layers):
-        nm = lambda pattern: pattern.format(layer=i)  # noqa: E731, B023
+        nm = lambda pattern, **kw: pattern.format(layer=i, **kw)  # noqa: E731, B023
         make, known = mixers[lc.mixer]
         if known is None:
             raise ValueError(f"layer {i}: {spec.name} models have no {lc.mixer} layers")
         mlp = mlp_norm = post_mlp = None
         attn = make(lc, nm)
+        if (lc.experts is not None) != (spec.is_moe and lc.intermediate_size is not None):
+            raise ValueError(f"layer {i}: {spec.name} models have {'no dense feed-forwards' if spec.is_moe else 'no experts'}")
+        if spec.parallel:
+            blocks.append(ParallelBlock(norm(nm(spec.attn_norm), H, off, one, spec.norm_type), attn, None if lc.experts is None else expert_mlp(lc, nm)))
+            continue
         if lc.intermediate_size is not None:
             I = lc.intermediate_size
             if spec.activation == "xielu":
@@ -278,7 +333,16 @@ def _load_layer_list(st, spec: ModelSpec, config: dict, dtype, load_tensor, try_
                                        norm(nm(spec.post_attn_norm), H, off, one), post_mlp, cfg.residual_mult))
     lm_head = tensor(spec.lm_head, (cfg.vocab_size, H)) if spec.lm_head in st else None
     pos = tensor(spec.position_embed, (cfg.max_position_embeddings, H)) if spec.use_position_embed else None
-    return CausalTransformerModel(cfg, tensor(spec.embed_tokens, (cfg.vocab_size, H)), blocks, norm(spec.final_norm, H, off, one), lm_head, pos, spec)
+    loop = None
+    if cfg.loop is not None:
+        if spec.loop_in is None:
+            raise ValueError(f"{spec.name} models have no loop")
+        loop = LoopInput(tensor(spec.loop_in, (H, 2 * H)), from_numpy(fp32(spec.loop_step, cfg.loop.times * H).reshape(cfg.loop.times, H)))
+    return CausalTransformerModel(cfg, tensor(spec.embed_tokens, (cfg.vocab_size, H)), blocks, norm(spec.final_norm, H, off, one, spec.norm_type, cfg.logit_scale), lm_head, pos, spec, loop)
+
+
+def _transposed(w: GPUArray) -> GPUArray:
+    return from_numpy(np.ascontiguousarray(w.to_numpy().T))
 
 
 def _bf16_array(bits: np.ndarray) -> GPUArray:
@@ -314,5 +378,9 @@ def load_malasun_from_safetensors(model_path: str, dtype: str = "bfloat16") -> C
     return load_model_from_safetensors(model_path, dtype=dtype, spec=MALASUN_SPEC)
 
 
-__all__ = ["load_malasun_from_safetensors", "load_totolorn_from_safetensors", "load_model_from_safetensors", "load_gpt2_from_safetensors", "load_llama_from_safetensors", "load_qwen3_from_safetensors",
+def load_ratasun_from_safetensors(model_path: str, dtype: str = "bfloat16") -> CausalTransformerModel:
+    return load_model_from_safetensors(model_path, dtype=dtype, spec=RATASUN_SPEC)
+
+
+__all__ = ["load_ratasun_from_safetensors", "load_malasun_from_safetensors", "load_totolorn_from_safetensors", "load_model_from_safetensors", "load_gpt2_from_safetensors", "load_llama_from_safetensors", "load_qwen3_from_safetensors",
            "FP8QuantConfig"]

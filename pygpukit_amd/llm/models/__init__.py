@@ -1,3 +1,3 @@
-from .causal import CausalTransformerModel, GPT2Model, LlamaModel, QwenModel, TotolornModel, MalasunModel
+from .causal import CausalTransformerModel, GPT2Model, LlamaModel, QwenModel, TotolornModel, MalasunModel, RatasunModel
 
-__all__ = ["CausalTransformerModel", "GPT2Model", "LlamaModel", "QwenModel", "TotolornModel", "MalasunModel"]
+__all__ = ["CausalTransformerModel", "GPT2Model", "LlamaModel", "QwenModel", "TotolornModel", "MalasunModel", "RatasunModel"]

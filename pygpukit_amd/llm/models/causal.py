@@ -17,7 +17,7 @@ from pygpukit_amd.core.dtypes import bfloat16
 from pygpukit_amd.core.factory import from_numpy
 from pygpukit_amd.llm.buffers import DecodeBuffers
 from pygpukit_amd.llm.config import ModelSpec, TransformerConfig
-from pygpukit_amd.llm.layers import MLP, Attention, Norm, TransformerBlock
+from pygpukit_amd.llm.layers import MLP, Attention, LoopInput, Norm, TransformerBlock
 from pygpukit_amd.llm.sampling import sample_token
 from pygpukit_amd.ops.basic import (add_inplace, cast_bf16_to_f32, embedding_lookup_batch, glu_packed, matmul_nt,
                                    rmsnorm, sample_token_gpu)
@@ -32,7 +32,9 @@ def _to_float32_logits(logits_np: np.ndarray) -> np.ndarray:
 
 class CausalTransformerModel:
     def __init__(self, config: TransformerConfig, embed_tokens: GPUArray, blocks: list[TransformerBlock], final_norm: Norm,
-                 lm_head: GPUArray | None = None, position_embed: GPUArray | None = None, spec: ModelSpec | None = None):
+                 lm_head: GPUArray | None = None, position_embed: GPUArray | None = None, spec: ModelSpec | None = None,
+                 loop: LoopInput | None = None):
+        """loop: what the passes of config.loop start with."""
         self.config = config
         self.embed_tokens = embed_tokens
         self.blocks = blocks
@@ -40,6 +42,11 @@ class CausalTransformerModel:
         self._lm_head = lm_head
         self.position_embed = position_embed
         self.spec = spec
+        self.loop = loop
+
+    def _runs(self) -> list[tuple[int, int | None]]:
+        """(block, number of the pass that starts with it or None) in the order they run."""
+        return [(i, None) for i in range(len(self.blocks))] if self.loop is None else self.config.loop.runs(len(self.blocks))
 
     @property
     def lm_head(self) -> GPUArray | None:
@@ -72,13 +79,16 @@ class CausalTransformerModel:
         if position_ids is None:
             past_len = 0
             if past_key_values is not None:
-                past_len = next((p[0].shape[0] for b, p in zip(self.blocks, past_key_values) if p is not None and getattr(b.attn, "cache_rows", True)), 0)
+                past_len = next((p[0].shape[0] for (i, _), p in zip(self._runs(), past_key_values) if p is not None and getattr(self.blocks[i].attn, "cache_rows", True)), 0)
             position_ids = list(range(past_len, past_len + seq_len))
-        hidden = self._embed(input_ids, position_ids)
+        hidden = embedded = self._embed(input_ids, position_ids)
         present = []
         sources = {getattr(b.attn, "kv_from", None) for b in self.blocks}
-        for i, block in enumerate(self.blocks):
-            past_kv = past_key_values[i] if past_key_values else None
+        for run, (i, start) in enumerate(self._runs()):
+            block = self.blocks[i]
+            if start is not None:
+                hidden = self.loop(hidden, embedded, start)
+            past_kv = past_key_values[run] if past_key_values else None
             src = getattr(block.attn, "kv_from", None)
             hidden, kv = block(hidden, position_ids, past_kv, use_cache or i in sources, None if src is None else present[src])
             present.append(kv)
@@ -143,6 +153,8 @@ class CausalTransformerModel:
     # ------------------------------------------------------------------ fixed-cache decode (eager ops path)
     def init_fixed_cache(self, max_seq_len: int, dtype: str | None = None) -> None:
         dt = dtype or str(self.embed_tokens.dtype)
+        if self.loop is not None:
+            raise NotImplementedError("the fixed caches hold one pass of every block: use past_key_values or build_engine()")
         for block in self.blocks:
             block.attn.init_fixed_cache(max_seq_len, dt)
 
@@ -226,5 +238,6 @@ LlamaModel = CausalTransformerModel
 QwenModel = CausalTransformerModel
 TotolornModel = CausalTransformerModel
 MalasunModel = CausalTransformerModel
+RatasunModel = CausalTransformerModel
 
-__all__ = ["CausalTransformerModel", "GPT2Model", "LlamaModel", "QwenModel", "TotolornModel", "MalasunModel"]
+__all__ = ["CausalTransformerModel", "GPT2Model", "LlamaModel", "QwenModel", "TotolornModel", "MalasunModel", "RatasunModel"]

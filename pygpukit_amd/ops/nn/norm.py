@@ -35,6 +35,16 @@ def rmsnorm_f32(input: GPUArray, weight: GPUArray, eps: float = 1e-5, *, dtype=f
     return o
 
 
+def layernorm_f32(input: GPUArray, weight: GPUArray, eps: float = 1e-5, *, dtype=float32, out: GPUArray | None = None) -> GPUArray:
+    """Layer norm (no bias) of an fp32 stream with an fp32 weight; the result leaves in `dtype`."""
+    _check(input, weight, "layernorm_f32")
+    if input.dtype != float32:
+        raise ValueError("layernorm_f32: input and weight must be float32")
+    o = check_out(out, input.shape, dtype, "layernorm_f32")
+    call("pgk_layernorm_f32", input._p, weight._p, o._p, input.shape[0], input.shape[1], eps, o.dtype.code, None)
+    return o
+
+
 def rmsnorm_add_f32(stream: GPUArray, y: GPUArray, weight: GPUArray, eps: float = 1e-5, mult: float = 1.0) -> GPUArray:
     """stream += mult * rmsnorm(y) * weight in place (fp32 stream and weight, y in any float type)."""
     validate_float(y, "rmsnorm_add_f32")
