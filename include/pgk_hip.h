@@ -383,14 +383,14 @@ pgk_status pgk_conv_silu(const void* u, const void* past, const void* w, const f
  * [n, heads * dim], strengths [n, heads] and gates [n, heads * vdim] before their sigmoid; fp32 decay [heads], step_bias [heads * dim],
  * norm [vdim].  q, k of unit length per head (q also times dim^-1/2), b = sigmoid(strength), g = exp(-decay softplus(z + step_bias)):
  * S <- diag(g) S, u = b (v - S^T k), S <- S + k u^T, o = S^T q; out = o / rms(o) * norm * sigmoid(gate).  state: fp32 [heads, dim, vdim],
- * read unless `fresh`, updated.  dim, vdim: multiples of 4.  dt (all but z, which is fp32): PGK_BF16 or PGK_F32 */
+ * read unless `fresh`, updated.  dt (all but z, which is fp32): PGK_BF16 or PGK_F32 */
 pgk_status pgk_delta_rule(const void* q, const void* k, const void* v, const float* z, const void* strength, const void* gate,
                           const float* decay, const float* step_bias, const float* norm, float* state, void* out, int n, int fresh,
                           int heads, int kv_heads, int dim, int vdim, float eps, pgk_dtype dt, pgk_stream s);
 /* State-space duality over n rows of one sequence: xbc [n, heads * vdim | groups * dim | groups * dim] (x, B, C after taps and activation), z
  * [n, heads * vdim], t [n, heads]; fp32 decay, step_bias, skip [heads], norm [heads * vdim].  t <- softplus(t + step_bias),
  * S <- exp(-decay t) S + t B x^T, y = S^T C + skip x; out = (y silu(z)) / rms * norm in norm_parts equal parts.  state: fp32
- * [heads, dim, vdim], read unless `fresh`, updated.  dim, vdim: multiples of 4.  dt: PGK_BF16 or PGK_F32 */
+ * [heads, dim, vdim], read unless `fresh`, updated.  dt: PGK_BF16 or PGK_F32 */
 pgk_status pgk_state_space(const void* xbc, const void* z, const void* t, const float* decay, const float* step_bias, const float* skip,
                            const float* norm, float* state, void* out, int n, int fresh, int heads, int groups, int dim, int vdim,
                            int norm_parts, float eps, pgk_dtype dt, pgk_stream s);

@@ -173,4 +173,15 @@ pgk_status lowrank_rows(const void* in, int ld_in, int n, int a_off, int ka, con
 // columns off .. off + cols of rows -> dense rows
 pgk_status rows_slice(const void* in, int ld_in, int off, int cols, void* out, int n, pgk_dtype dt, hipStream_t st);
 
+// Device copies of rows [rows][heads * d] to or from rows whose heads are `p` elements apart (bytes throughout; the ends of wider heads are
+// left alone).
+inline hipError_t copy_heads(void* dst, size_t ld_dst, size_t p_dst, const void* src, size_t ld_src, size_t p_src, size_t rows, int heads, hipStream_t st) {
+    if (p_dst == p_src) return hipMemcpy2DAsync(dst, ld_dst, src, ld_src, heads * p_dst, rows, hipMemcpyDeviceToDevice, st);
+    const size_t w = p_dst < p_src ? p_dst : p_src;
+    hipError_t e = hipSuccess;
+    for (int h = 0; h < heads && e == hipSuccess; ++h)
+        e = hipMemcpy2DAsync((char*)dst + h * p_dst, ld_dst, (const char*)src + h * p_src, ld_src, w, rows, hipMemcpyDeviceToDevice, st);
+    return e;
+}
+
 }  // namespace pgk

@@ -628,36 +628,61 @@ extern "C" {
 pgk_status pgk_delta_rule(const void* q, const void* k, const void* v, const float* z, const void* strength, const void* gate, const float* decay, const float* step_bias,
                           const float* norm, float* state, void* out, int n, int fresh, int heads, int kv_heads, int dim, int vdim, float eps, pgk_dtype dt, pgk_stream s) {
     PGK_REQUIRE(q && k && v && z && strength && gate && decay && step_bias && norm && state && out, "pgk_delta_rule: null pointer");
-    PGK_REQUIRE(n >= 1 && heads >= 1 && kv_heads >= 1 && heads % kv_heads == 0 && dim >= 4 && dim % 4 == 0 && vdim >= 4 && vdim % 4 == 0, "pgk_delta_rule: bad shape %d / %d x %d x %d, %d rows",
+    PGK_REQUIRE(n >= 1 && heads >= 1 && kv_heads >= 1 && heads % kv_heads == 0 && dim >= 1 && vdim >= 1, "pgk_delta_rule: bad shape %d / %d x %d x %d, %d rows",
                 heads, kv_heads, dim, vdim, n);
     PGK_REQUIRE(dt == PGK_BF16 || dt == PGK_F32, "pgk_delta_rule: dtype %d (bf16 or f32)", (int)dt);
     hipStream_t st = resolve_stream(s);
-    const size_t E = dtype_size(dt), wq = (size_t)kv_heads * dim * E, wv = (size_t)heads * vdim * E, row = 2 * wq + wv;
+    // one row buffer q | k | v, the tables and the chunked form's workspace behind it; head widths that are no multiple of 4 run as copies
+    // with zeros behind every head
+    const int dp = ceil_div(dim, 4) * 4, vp = ceil_div(vdim, 4) * 4;
+    const bool pad = dp != dim || vp != vdim;
+    const size_t E = dtype_size(dt), wq = (size_t)kv_heads * dp * E, wv = (size_t)heads * vp * E, row = 2 * wq + wv, wz = (size_t)heads * dp * 4;
+    const size_t d = (size_t)dim * E, v1 = (size_t)vdim * E;
     auto up = [](size_t b) { return (b + 255) & ~(size_t)255; };
     DeltaArgs a{};
-    a.in = strength; a.ld_in = heads; a.ld_rows = (int)(row / E); a.z = z; a.ld_z = heads * dim; a.gate = gate; a.ld_gate = heads * vdim;
-    a.decay = decay; a.dt_bias = step_bias; a.norm = norm; a.H = heads; a.G = kv_heads; a.dim = a.dim_true = dim; a.vdim = a.vdim_true = vdim; a.n = n; a.eps = eps;
-    a.state = state; a.n_seqs = 1; a.out = out; a.ld_out = heads * vdim;
-    const int C = n >= RECUR_CHUNKED_FROM && delta_chunk_ok(dim, vdim) ? DELTA_CHUNK : 0, nch = C ? ceil_div(n, C) : 0;
+    a.in = strength; a.ld_in = heads; a.ld_rows = (int)(row / E); a.z = z; a.ld_z = heads * dp; a.gate = gate; a.ld_gate = heads * vp;
+    a.decay = decay; a.dt_bias = step_bias; a.norm = norm; a.H = heads; a.G = kv_heads; a.dim = dp; a.dim_true = dim; a.vdim = vp; a.vdim_true = vdim; a.n = n; a.eps = eps;
+    a.state = state; a.n_seqs = 1; a.out = out; a.ld_out = heads * vp;
+    const int C = n >= RECUR_CHUNKED_FROM && delta_chunk_ok(dp, vp) ? DELTA_CHUNK : 0, nch = C ? ceil_div(n, C) : 0;
     std::vector<RecurChunk> chunks;
     for (int c = 0; c < nch; ++c) chunks.push_back(RecurChunk{c * C, n - c * C < C ? n - c * C : C});
     const int32_t of_seq[2] = {0, nch};
     const SeqSpan span{0, n, fresh ? 0 : 1, 0};
-    const size_t o_span = up(n * row), o_of = o_span + up(sizeof(span)), o_ch = o_of + up(sizeof(of_seq)), o_ws = o_ch + up(nch * sizeof(RecurChunk));
+    size_t at = 0;
+    auto take = [&](size_t b) { const size_t o = at; at += up(b); return o; };
+    const size_t o_rows = take(n * row), o_z = take(pad ? n * wz : 0), o_gate = take(pad ? n * wv : 0), o_out = take(pad ? n * wv : 0), o_bias = take(pad ? wz : 0), o_norm = take(pad ? vp * 4 : 0),
+                 o_state = take(pad ? wz * vp : 0), zeroed = at, o_span = take(sizeof(span)), o_of = take(sizeof(of_seq)), o_ch = take(nch * sizeof(RecurChunk)), o_ws = take(nch ? delta_chunk_bytes(a, nch) : 0);
     char* ws = nullptr;
-    if (pgk_status r = pgk_malloc((void**)&ws, o_ws + (nch ? delta_chunk_bytes(a, nch) : 0) + 256)) return r;
-    hipError_t e = hipMemcpy2DAsync(ws, row, q, wq, wq, n, hipMemcpyDeviceToDevice, st);
-    if (e == hipSuccess) e = hipMemcpy2DAsync(ws + wq, row, k, wq, wq, n, hipMemcpyDeviceToDevice, st);
-    if (e == hipSuccess) e = hipMemcpy2DAsync(ws + 2 * wq, row, v, wv, wv, n, hipMemcpyDeviceToDevice, st);
+    if (pgk_status r = pgk_malloc((void**)&ws, at + 256)) return r;
+    hipError_t e = pad ? hipMemsetAsync(ws, 0, zeroed, st) : hipSuccess;
+    const size_t fd = (size_t)dim * 4, fv = (size_t)vdim * 4, fdp = (size_t)dp * 4, fvp = (size_t)vp * 4;
+    auto copy = [&](size_t dst, size_t ld_dst, size_t p_dst, const void* src, size_t p_src, size_t rows, int nh) {
+        if (e == hipSuccess) e = copy_heads(ws + dst, ld_dst, p_dst, src, nh * p_src, p_src, rows, nh, st);
+    };
+    copy(o_rows, row, dp * E, q, d, n, kv_heads);
+    copy(o_rows + wq, row, dp * E, k, d, n, kv_heads);
+    copy(o_rows + 2 * wq, row, vp * E, v, v1, n, heads);
+    if (pad) {
+        copy(o_z, wz, fdp, z, fd, n, heads);
+        copy(o_gate, wv, vp * E, gate, v1, n, heads);
+        copy(o_bias, wz, fdp, step_bias, fd, 1, heads);
+        copy(o_norm, fvp, fvp, norm, fv, 1, 1);
+        for (int h = 0; h < heads; ++h) copy(o_state + h * dp * fvp, fvp, fvp, state + (size_t)h * dim * vdim, fv, dim, 1);
+        a.z = (const float*)(ws + o_z); a.gate = ws + o_gate; a.dt_bias = (const float*)(ws + o_bias); a.norm = (const float*)(ws + o_norm);
+        a.state = (float*)(ws + o_state); a.out = ws + o_out;
+    }
     if (e == hipSuccess) e = hipMemcpyAsync(ws + o_span, &span, sizeof(span), hipMemcpyHostToDevice, st);
     if (e == hipSuccess) e = hipMemcpyAsync(ws + o_of, of_seq, sizeof(of_seq), hipMemcpyHostToDevice, st);
     if (e == hipSuccess && nch) e = hipMemcpyAsync(ws + o_ch, chunks.data(), nch * sizeof(RecurChunk), hipMemcpyHostToDevice, st);
     if (e == hipSuccess) e = hipStreamSynchronize(st);
-    a.rows = ws; a.seqs = (const SeqSpan*)(ws + o_span);
-    pgk_status r;
+    a.rows = ws + o_rows; a.seqs = (const SeqSpan*)(ws + o_span);
+    pgk_status r = PGK_OK;
+    if (e == hipSuccess) r = nch ? delta_chunked(a, (const RecurChunk*)(ws + o_ch), nch, (const int32_t*)(ws + o_of), ws + o_ws, dt, st) : delta_rows(a, dt, dt == PGK_F32, st);
+    if (pad && e == hipSuccess && r == PGK_OK) {
+        e = copy_heads(out, heads * v1, v1, ws + o_out, wv, vp * E, n, heads, st);
+        for (int h = 0; h < heads && e == hipSuccess; ++h) e = copy_heads(state + (size_t)h * dim * vdim, fv, fv, ws + o_state + h * dp * fvp, fvp, fvp, dim, 1, st);
+    }
     if (e != hipSuccess) r = set_error(PGK_ERR_HIP, "pgk_delta_rule: %s", hipGetErrorString(e));
-    else if (nch) r = delta_chunked(a, (const RecurChunk*)(ws + o_ch), nch, (const int32_t*)(ws + o_of), ws + o_ws, dt, st);
-    else r = delta_rows(a, dt, dt == PGK_F32, st);
     pgk_free(ws);       // stream-ordered reuse
     return r;
 }

@@ -688,38 +688,58 @@ pgk_status pgk_gated_recurrence(const void* q, const void* f, const void* v, con
 pgk_status pgk_state_space(const void* xbc, const void* z, const void* t, const float* decay, const float* step_bias, const float* skip, const float* norm, float* state, void* out,
                            int n, int fresh, int heads, int groups, int dim, int vdim, int norm_parts, float eps, pgk_dtype dt, pgk_stream s) {
     PGK_REQUIRE(xbc && z && t && decay && step_bias && skip && norm && state && out, "pgk_state_space: null pointer");
-    PGK_REQUIRE(n >= 1 && heads >= 1 && groups >= 1 && heads % groups == 0 && dim >= 4 && dim % 4 == 0 && vdim >= 4 && vdim % 4 == 0 && norm_parts >= 1 && heads * vdim % norm_parts == 0,
+    PGK_REQUIRE(n >= 1 && heads >= 1 && groups >= 1 && heads % groups == 0 && dim >= 1 && vdim >= 1 && norm_parts >= 1 && heads * vdim % norm_parts == 0,
                 "pgk_state_space: bad shape %d / %d x %d x %d, %d norm parts, %d rows", heads, groups, dim, vdim, norm_parts, n);
     PGK_REQUIRE(dt == PGK_BF16 || dt == PGK_F32, "pgk_state_space: dtype %d (bf16 or f32)", (int)dt);
     hipStream_t st = resolve_stream(s);
-    // one row buffer z | t, the tables and the chunked form's workspace behind it
-    const int V = heads * vdim, ld = (V + heads + 3) / 4 * 4;
-    const size_t E = dtype_size(dt), row = (size_t)ld * E, wz = (size_t)V * E, wt = (size_t)heads * E;
+    // one row buffer z | t, the tables and the chunked form's workspace behind it; head widths that are no multiple of 4 run as copies with
+    // zeros behind every head
+    const int dp = ceil_div(dim, 4) * 4, vp = ceil_div(vdim, 4) * 4, V = heads * vp, ld = (V + heads + 3) / 4 * 4, ld_x = V + 2 * groups * dp;
+    const bool pad = dp != dim || vp != vdim;
+    const size_t E = dtype_size(dt), row = (size_t)ld * E, wz = (size_t)V * E, wt = (size_t)heads * E, v1 = (size_t)vdim * E, d = (size_t)dim * E, fv = (size_t)vdim * 4, fvp = (size_t)vp * 4;
     auto up = [](size_t b) { return (b + 255) & ~(size_t)255; };
     RecurArgs a{};
-    a.kind = RECUR_SSD; a.ld_in = ld; a.rows = xbc; a.ld_rows = V + 2 * groups * dim; a.G = groups; a.f_off = V; a.q_off = V + groups * dim; a.z_off = 0; a.dt_off = V;
-    a.dt_bias = step_bias; a.decay = decay; a.skip = skip; a.H = heads; a.dim = dim; a.vdim = a.vdim_true = vdim; a.n = n; a.eps = eps;
+    a.kind = RECUR_SSD; a.ld_in = ld; a.rows = xbc; a.ld_rows = ld_x; a.G = groups; a.f_off = V; a.q_off = V + groups * dp; a.z_off = 0; a.dt_off = V;
+    a.dt_bias = step_bias; a.decay = decay; a.skip = skip; a.H = heads; a.dim = dp; a.vdim = vp; a.vdim_true = vdim; a.n = n; a.eps = eps;
     a.state = state; a.n_seqs = 1; a.out = out; a.ld_out = V;
-    const int C = n >= RECUR_CHUNKED_FROM ? recur_chunk_rows(dim, vdim) : 0, nch = C ? ceil_div(n, C) : 0;
+    const int C = n >= RECUR_CHUNKED_FROM ? recur_chunk_rows(dp, vp) : 0, nch = C ? ceil_div(n, C) : 0;
     std::vector<RecurChunk> chunks;
     for (int c = 0; c < nch; ++c) chunks.push_back(RecurChunk{c * C, n - c * C < C ? n - c * C : C});
     const int32_t of_seq[2] = {0, nch};
     const SeqSpan span{0, n, fresh ? 0 : 1, 0};
-    const size_t o_span = up(n * row), o_of = o_span + up(sizeof(span)), o_ch = o_of + up(sizeof(of_seq)), o_ws = o_ch + up(nch * sizeof(RecurChunk));
+    size_t at = 0;
+    auto take = [&](size_t b) { const size_t o = at; at += up(b); return o; };
+    const size_t o_in = take(n * row), o_x = take(pad ? (size_t)n * ld_x * E : 0), o_out = take(pad ? n * wz : 0), o_norm = take(pad ? heads * fvp : 0), o_state = take(pad ? heads * dp * fvp : 0), zeroed = at,
+                 o_span = take(sizeof(span)), o_of = take(sizeof(of_seq)), o_ch = take(nch * sizeof(RecurChunk)), o_ws = take(nch ? recur_chunk_bytes(a, nch) : 0);
     char* ws = nullptr;
-    if (pgk_status r = pgk_malloc((void**)&ws, o_ws + (nch ? recur_chunk_bytes(a, nch) : 0) + 256)) return r;
-    hipError_t e = hipMemcpy2DAsync(ws, row, z, wz, wz, n, hipMemcpyDeviceToDevice, st);
-    if (e == hipSuccess) e = hipMemcpy2DAsync(ws + wz, row, t, wt, wt, n, hipMemcpyDeviceToDevice, st);
+    if (pgk_status r = pgk_malloc((void**)&ws, at + 256)) return r;
+    hipError_t e = pad ? hipMemsetAsync(ws, 0, zeroed, st) : hipSuccess;
+    auto copy = [&](size_t dst, size_t ld_dst, size_t p_dst, const void* src, size_t ld_src, size_t p_src, size_t rows, int nh) {
+        if (e == hipSuccess) e = copy_heads(ws + dst, ld_dst, p_dst, src, ld_src, p_src, rows, nh, st);
+    };
+    copy(o_in, row, vp * E, z, heads * v1, v1, n, heads);
+    copy(o_in + wz, row, wt, t, wt, wt, n, 1);
+    if (pad) {
+        const size_t lx = heads * v1 + 2 * groups * d, lp = (size_t)ld_x * E;
+        copy(o_x, lp, vp * E, xbc, lx, v1, n, heads);
+        copy(o_x + V * E, lp, dp * E, (const char*)xbc + heads * v1, lx, d, n, 2 * groups);
+        copy(o_norm, heads * fvp, fvp, norm, heads * fv, fv, 1, heads);
+        for (int h = 0; h < heads; ++h) copy(o_state + h * dp * fvp, fvp, fvp, state + (size_t)h * dim * vdim, fv, fv, dim, 1);
+        a.rows = ws + o_x; a.state = (float*)(ws + o_state); a.out = ws + o_out; norm = (const float*)(ws + o_norm);
+    }
     if (e == hipSuccess) e = hipMemcpyAsync(ws + o_span, &span, sizeof(span), hipMemcpyHostToDevice, st);
     if (e == hipSuccess) e = hipMemcpyAsync(ws + o_of, of_seq, sizeof(of_seq), hipMemcpyHostToDevice, st);
     if (e == hipSuccess && nch) e = hipMemcpyAsync(ws + o_ch, chunks.data(), nch * sizeof(RecurChunk), hipMemcpyHostToDevice, st);
     if (e == hipSuccess) e = hipStreamSynchronize(st);
-    a.in = ws; a.seqs = (const SeqSpan*)(ws + o_span);
-    pgk_status r;
+    a.in = ws + o_in; a.seqs = (const SeqSpan*)(ws + o_span);
+    pgk_status r = PGK_OK;
+    if (e == hipSuccess) r = nch ? recur_chunked(a, (const RecurChunk*)(ws + o_ch), nch, (const int32_t*)(ws + o_of), ws + o_ws, dt, st) : recur_rows(a, dt, dt == PGK_F32, st);
+    if (r == PGK_OK && e == hipSuccess) r = parts_norm(a.out, V, n, heads, vp, vdim, norm_parts, norm, eps, dt, st);
+    if (pad && e == hipSuccess && r == PGK_OK) {
+        e = copy_heads(out, heads * v1, v1, ws + o_out, wz, vp * E, n, heads, st);
+        for (int h = 0; h < heads && e == hipSuccess; ++h) e = copy_heads(state + (size_t)h * dim * vdim, fv, fv, ws + o_state + h * dp * fvp, fvp, fvp, dim, 1, st);
+    }
     if (e != hipSuccess) r = set_error(PGK_ERR_HIP, "pgk_state_space: %s", hipGetErrorString(e));
-    else if (nch) r = recur_chunked(a, (const RecurChunk*)(ws + o_ch), nch, (const int32_t*)(ws + o_of), ws + o_ws, dt, st);
-    else r = recur_rows(a, dt, dt == PGK_F32, st);
-    if (r == PGK_OK) r = parts_norm(out, V, n, heads, vdim, vdim, norm_parts, norm, eps, dt, st);
     pgk_free(ws);       // stream-ordered reuse
     return r;
 }

@@ -5,7 +5,7 @@ from __future__ import annotations
 from pygpukit_amd.core.array import GPUArray
 from pygpukit_amd.core.dtypes import bfloat16, float32
 from pygpukit_amd.ops._common import call, check_out, validate_float
-from pygpukit_amd.ops.tensor import cast_bf16_to_f32
+from pygpukit_amd.ops.tensor import cast_bf16_to_f32, pad_2d
 
 
 def short_conv(u: GPUArray, weight: GPUArray, past: GPUArray | None = None, *, out: GPUArray | None = None) -> GPUArray:
@@ -54,6 +54,13 @@ def conv_silu(u: GPUArray, taps: GPUArray, past: GPUArray | None = None, *, bias
     if bias is not None and (bias.size != u.shape[1] or bias.dtype != float32):
         raise ValueError(f"conv_silu: bias must be float32 of {u.shape[1]} elements")
     o = check_out(out, u.shape, u.dtype, "conv_silu")
+    n, ch = u.shape
+    if ch % 4:                                                 # the kernel takes four channels at a time
+        p = -(-ch // 4) * 4
+        y = conv_silu(pad_2d(u, n, p), pad_2d(taps, taps.shape[0], p), None if past is None else pad_2d(past, past.shape[0], p),
+                      bias=None if bias is None else pad_2d(bias.view((1, ch)), 1, p))
+        call("pgk_pad_2d", y._p, o._p, n, p, n, ch, u.dtype.code, None)
+        return o
     call("pgk_conv_silu", u._p, _opt(past), taps._p, _opt(bias), o._p, u.shape[0], u.shape[1], taps.shape[0], u.dtype.code, None)
     return o
 
