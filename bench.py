@@ -124,10 +124,84 @@ DESIGN_SIZES = {
 }
 
 
+DESIGN_VOCAB = 32000
+
+
+def dense_config(z: dict) -> dict:
+    return dict(vocab_size=DESIGN_VOCAB, hidden_size=z["width"], num_layers=z["layers"], num_heads=z["heads"], num_kv_heads=z["kv_heads"], head_dim=z["dim"],
+                intermediate_size=z["ff"], norm_eps=1e-5, rope_theta=1e6)
+
+
+# Ratasun at those sizes: its three mixers in turn with heads of the others' widths, in every layer experts of which each token uses as much
+# feed-forward width as the others have
+RATASUN_EXPERTS = {"experts": 16, "top": 4, "split": 4, "groups": 4, "keep": 3}
+RATASUN_RANK = 128
+RATASUN_MIXERS = ("latent_attention", "channel_delta", "mamba2")
+
+
+def ratasun_layer(i: int) -> str:
+    return RATASUN_MIXERS[i % len(RATASUN_MIXERS)]
+
+
+def ratasun_model(z: dict, vocab: int, embed, head, draw, feed_forward):
+    """A Ratasun of the sizes `z`; feed_forward(i): gate | up [2 ff, width] and down [width, ff] of layer i, whose copies are its experts."""
+    from pygpukit_amd import _hip
+    from pygpukit_amd.core.array import GPUArray
+    from pygpukit_amd.core.factory import from_numpy
+    from pygpukit_amd.llm import (RATASUN_SPEC, CausalTransformerModel, ChannelDelta, LatentAttention, MixtureOfExperts, Norm, ParallelBlock, StateSpace, layer_list_config)
+
+    W, F, H, G, D, r, L = (z[k] for k in ("width", "ff", "heads", "kv_heads", "dim", "rank", "layers"))
+    x, rot, hd, lr = RATASUN_EXPERTS, D // 4, H * D, RATASUN_RANK
+    f, E = F // x["split"], x["experts"]
+    mixers = {"latent_attention": {"heads": H, "dim": D - rot, "rot_dim": rot, "vdim": D, "kv_rank": r, "scale": D**-0.5, "rot": {"base": 1e4, "dims": rot}},
+              "channel_delta": {"heads": H, "kv_heads": H, "dim": D, "vdim": D, "conv": 4},
+              "mamba2": {"heads": 2 * H, "groups": G, "state": D, "vdim": D // 2, "conv": 4, "norm_groups": G}}
+    moe = {"kind": "moe", "expert": {"ff": f}, "router": {"experts": E, "top": x["top"], "groups": {"count": x["groups"], "keep": x["keep"]}}}
+    cfg = layer_list_config({"architecture": "Ratasun", "vocab": vocab, "width": W, "norm": {"eps": 1e-5},
+                             "layers": [{"type": ratasun_layer(i), "mixer": mixers[ratasun_layer(i)], "mlp": moe} for i in range(L)]})
+    full = lambda n, v=1.0: from_numpy(np.full(n, v, np.float32))  # noqa: E731
+    dt = embed.dtype
+    norm = lambda n, kind="layernorm": Norm(full(n), None, kind, 1e-5, stream_dtype=dt)  # noqa: E731
+
+    def copies(w, n, shape):
+        out = GPUArray(shape, w.dtype)
+        for i in range(out.nbytes // (w.nbytes // n)):
+            _hip.call("pgk_memcpy_d2d", out.data_ptr() + i * (w.nbytes // n), w.data_ptr() + i % n * (w.nbytes // n), w.nbytes // n, None)
+        return out
+
+    def block(i):
+        gu, dn = feed_forward(i)
+        kind, o = ratasun_layer(i), draw(W, hd)
+        if kind == "latent_attention":
+            mix = LatentAttention(draw(hd, W), draw(r + rot, W), norm(r, "rmsnorm"), draw(H * (D - rot), r), draw(hd, r), o, num_heads=H, head_dim=D - rot, v_head_dim=D, scale=D**-0.5,
+                                  rot_dim=rot, rot_freq=from_numpy((1e4 ** (-2.0 * np.arange(rot // 2) / rot)).astype(np.float32)))
+        elif kind == "channel_delta":
+            mix = ChannelDelta(draw(hd, W), draw(hd, W), draw(hd, W), o, draw(H, W), (draw(lr, W), draw(hd, lr)), (draw(lr, W), draw(hd, lr)), tuple(draw(4, hd) for _ in range(3)),
+                               full(H), full(hd, -3.0), full(D), num_heads=H, num_kv_heads=H, head_dim=D, v_head_dim=D, eps=1e-5)
+        else:
+            ch = hd + 2 * G * D
+            mix = StateSpace((draw(hd, W), draw(ch, W), draw(2 * H, W)), o, draw(4, ch), full(ch, 0.1), full(2 * H), full(2 * H, -3.0), full(2 * H), full(hd), num_heads=2 * H, num_groups=G,
+                             state_dim=D, v_head_dim=D // 2, norm_groups=G, eps=1e-5)
+        experts = MixtureOfExperts(draw(E, W), full(E, 0.0), copies(gu, x["split"], (E, 2 * f, W)), copies(dn, x["split"], (E, W, f)), top=x["top"], groups=x["groups"], keep=x["keep"])
+        return ParallelBlock(norm(W), mix, experts)
+
+    return CausalTransformerModel(cfg, embed, [block(i) for i in range(L)], norm(W), head, None, RATASUN_SPEC)
+
+
 def stack_kernel_bytes(kind: str, z: dict, vocab: int, ctx: int, B: int) -> dict:
     """Algorithmic bytes of ONE decode step of a layer-list engine by kernel class (bf16 weights and caches, fp32 rows and states)."""
     W, F, H, D, L, n = z["width"], z["ff"], z["heads"], z["dim"], z["layers"], min(ctx, z["window"])
     hd, gd, r = H * D, z["kv_heads"] * D, z["rank"]
+    if kind == "ratasun":              # experts of one sequence: the chosen ones; `down` is out-projection and experts in one launch
+        x, kinds = RATASUN_EXPERTS, [ratasun_layer(i) for i in range(L)]
+        E, top, f, rot, lr = x["experts"], x["top"], F // x["split"], D // 4, RATASUN_RANK
+        n_in = {"latent_attention": hd + r + rot, "channel_delta": 3 * hd + H + 2 * lr, "mamba2": 2 * hd + 2 * gd + 2 * H}
+        state = B * (2 * hd * D * 4 + 4 * 4 * hd)
+        return {"norm_qkv": sum((n_in[k] + E) * W * 2 + B * 4 * (2 * W + n_in[k] + E) for k in kinds),
+                "attn": kinds.count("latent_attention") * (2 * hd * r * 2 + B * (ctx * (r + rot) * 2 + 8 * hd + 4 * r)),
+                "recur": sum(state + (2 * hd * lr * 2 if k == "channel_delta" else 0) for k in kinds if k != "latent_attention"),
+                "gateup": L * (2 * top * f * W * 2 + B * 4 * (W + top * f)), "down": L * ((hd + top * f) * W * 2 + B * 4 * (hd + top * f + W)),
+                "lmhead": vocab * W * 2 + B * 4 * (W + vocab)}
     out = {"oproj": L * (hd * W * 2 + B * 4 * (hd + W)), "down": L * (F * W * 2 + B * 4 * (F + W)), "lmhead": vocab * W * 2 + B * 4 * (W + vocab)}
     if kind == "totolorn":
         out.update(norm_qkv=L * ((hd + r + H) * W * 2 + B * 4 * (2 * W + hd + r)), attn=L * (2 * hd * r * 2 + B * (n * r * 2 + 8 * hd + 4 * r)),
@@ -140,17 +214,67 @@ def stack_kernel_bytes(kind: str, z: dict, vocab: int, ctx: int, B: int) -> dict
     return out
 
 
-def design_leg(name: str, sizes: list[str], seed: int) -> dict:
-    """--design totolorn | malasun: prefill and decode of the layer-list engine at sizes that resemble a real model's layers (random
-    weights), beside its closest relatives here at equal width, heads, feed-forward width, depth and vocabulary: the dense QKV + RoPE
-    engine, and for Malasun (every other layer attention, the others recurrent) Totolorn too."""
-    from pygpukit_amd import _hip
+def design_engines(name: str, size: str, seed: int) -> tuple[dict, dict]:
+    """(sizes, kind -> engine constructor (max_seq_len, max_batch)) of a design and its relatives."""
     from pygpukit_amd.core.factory import from_numpy
     from pygpukit_amd.llm import synthetic as S
     from pygpukit_amd.llm.config import distance_slopes
     from pygpukit_amd.llm.engine import Engine, StackEngine
 
-    V = 32000
+    V, z = DESIGN_VOCAB, DESIGN_SIZES[size]
+    W, H, G, D, r, F, L = z["width"], z["heads"], z["kv_heads"], z["dim"], z["rank"], z["ff"], z["layers"]
+    rng = np.random.default_rng(seed)
+
+    def draw(*shape):
+        w = rng.standard_normal(shape, dtype=np.float32)
+        w *= np.float32(0.02)
+        return from_numpy(S.f32_to_bf16_bits(w).reshape(shape))
+
+    def ones(*shape):
+        return from_numpy(np.ones(shape, np.float32))
+
+    embed, head, pos = draw(V, W), draw(V, W), draw(4400, W)
+    one = ones(1, W)
+    b16 = S._bf16(np.ones(W, np.float32))
+    totolorn, malasun, dense, feed_forwards = [], [], [], []
+    for l in range(L):
+        gu, dn, o = draw(2 * F, W), draw(W, F), draw(W, H * D)
+        dense.append(dict(attn_norm=b16, mlp_norm=b16, q_norm=None, k_norm=None, w_qkv=draw((H + 2 * G) * D, W), w_o=o, w_gate_up=gu, w_down=dn))
+        totolorn.append(StackEngine.pack_layer(draw(H * D, W), draw(r, W), draw(H, W), ones(r), draw(H * D, r), draw(H * D, r), o, one, one, heads=H, dim=D, vdim=D,
+                                               window=z["window"], scale=D**-0.5, gate_up=gu, down=dn, norm2=one, norm2b=one))
+        feed_forwards.append((gu, dn))
+        if name == "totolorn":
+            continue
+        ff = dict(gate_up=gu._view(0, (F, W)), down=dn, norm2b=one, act_params=(0.8, 1.2))
+        if l % 2 == 0:
+            widths = (H * D, G * D, G * D)
+            malasun.append(StackEngine.pack_attention(*(draw(w, W) for w in widths), draw(H * D, W), o, None, one, heads=H, kv_heads=G, dim=D, vdim=D,
+                                                      window=z["window"], scale=D**-0.5, biases=tuple(draw(w) for w in widths), convs=tuple(draw(w, 4) for w in widths),
+                                                      q_norm=ones(H * D), k_norm=ones(G * D), slopes=from_numpy(np.asarray(distance_slopes(H), np.float32)), **ff))
+        else:
+            malasun.append(StackEngine.pack_recurrence(*(draw(H * D, W) for _ in range(3)), o, from_numpy(np.full(H * D, 3.0, np.float32)),
+                                                       from_numpy(np.full(H * D, 0.2, np.float32)), ones(D), None, one, heads=H, dim=D, vdim=D, **ff))
+    dcfg = dense_config(z)
+    scfg = dict(vocab_size=V, width=W, max_positions=4400, norm_eps=1e-5, residual_mult=0.7)
+    make = {"malasun": lambda ms, mb: StackEngine(dict(scfg, residual_mult=1.0), embed, None, head, one, malasun, max_seq_len=ms, max_batch=mb),
+            "totolorn": lambda ms, mb: StackEngine(scfg, embed, pos, head, one, totolorn, max_seq_len=ms, max_batch=mb),
+            "dense": lambda ms, mb: Engine(dcfg, embed, dense, b16, head, max_seq_len=ms, max_batch=mb, use_qk_norm=False)}
+    if name == "ratasun":
+        model = ratasun_model(z, V, embed, head, draw, lambda i: feed_forwards[i])
+        make = {"ratasun": lambda ms, mb: model.build_engine(max_seq_len=ms, max_batch=mb), "malasun": make["malasun"], "totolorn": make["totolorn"]}
+    elif name != "malasun":
+        del make["malasun"]
+    return z, make
+
+
+def design_leg(name: str, sizes: list[str], seed: int) -> dict:
+    """--design totolorn | malasun | ratasun: prefill and decode of the layer-list engine at sizes that resemble a real model's layers (random
+    weights), beside its closest relatives here at equal width, heads, feed-forward width, depth and vocabulary: the dense QKV + RoPE
+    engine, and for Malasun (every other layer attention, the others recurrent) Totolorn too; for Ratasun (three mixers in turn, experts)
+    Malasun and Totolorn."""
+    from pygpukit_amd import _hip
+
+    V = DESIGN_VOCAB
     out = {"design": name, "vocab": V, "dtype": "bf16", "data": "synthetic", "sizes": {}}
 
     def sync():
@@ -168,45 +292,9 @@ def design_leg(name: str, sizes: list[str], seed: int) -> dict:
         return float(np.median(best))
 
     for size in sizes:
-        z = DESIGN_SIZES[size]
-        W, H, G, D, r, F, L = z["width"], z["heads"], z["kv_heads"], z["dim"], z["rank"], z["ff"], z["layers"]
-        rng = np.random.default_rng(seed)
-
-        def draw(*shape):
-            w = rng.standard_normal(shape, dtype=np.float32)
-            w *= np.float32(0.02)
-            return from_numpy(S.f32_to_bf16_bits(w).reshape(shape))
-
-        def ones(*shape):
-            return from_numpy(np.ones(shape, np.float32))
-
-        embed, head, pos = draw(V, W), draw(V, W), draw(4400, W)
-        one = ones(1, W)
-        b16 = S._bf16(np.ones(W, np.float32))
-        totolorn, malasun, dense = [], [], []
-        for l in range(L):
-            gu, dn, o = draw(2 * F, W), draw(W, F), draw(W, H * D)
-            dense.append(dict(attn_norm=b16, mlp_norm=b16, q_norm=None, k_norm=None, w_qkv=draw((H + 2 * G) * D, W), w_o=o, w_gate_up=gu, w_down=dn))
-            totolorn.append(StackEngine.pack_layer(draw(H * D, W), draw(r, W), draw(H, W), ones(r), draw(H * D, r), draw(H * D, r), o, one, one, heads=H, dim=D, vdim=D,
-                                                   window=z["window"], scale=D**-0.5, gate_up=gu, down=dn, norm2=one, norm2b=one))
-            if name != "malasun":
-                continue
-            ff = dict(gate_up=gu._view(0, (F, W)), down=dn, norm2b=one, act_params=(0.8, 1.2))
-            if l % 2 == 0:
-                widths = (H * D, G * D, G * D)
-                malasun.append(StackEngine.pack_attention(*(draw(w, W) for w in widths), draw(H * D, W), o, None, one, heads=H, kv_heads=G, dim=D, vdim=D,
-                                                          window=z["window"], scale=D**-0.5, biases=tuple(draw(w) for w in widths), convs=tuple(draw(w, 4) for w in widths),
-                                                          q_norm=ones(H * D), k_norm=ones(G * D), slopes=from_numpy(np.asarray(distance_slopes(H), np.float32)), **ff))
-            else:
-                malasun.append(StackEngine.pack_recurrence(*(draw(H * D, W) for _ in range(3)), o, from_numpy(np.full(H * D, 3.0, np.float32)),
-                                                           from_numpy(np.full(H * D, 0.2, np.float32)), ones(D), None, one, heads=H, dim=D, vdim=D, **ff))
-        scfg = dict(vocab_size=V, width=W, max_positions=4400, norm_eps=1e-5, residual_mult=0.7)
-        dcfg = dict(vocab_size=V, hidden_size=W, num_layers=L, num_heads=H, num_kv_heads=G, head_dim=D, intermediate_size=F, norm_eps=1e-5, rope_theta=1e6)
-        make = {"malasun": lambda ms, mb: StackEngine(dict(scfg, residual_mult=1.0), embed, None, head, one, malasun, max_seq_len=ms, max_batch=mb),
-                "totolorn": lambda ms, mb: StackEngine(scfg, embed, pos, head, one, totolorn, max_seq_len=ms, max_batch=mb),
-                "dense": lambda ms, mb: Engine(dcfg, embed, dense, b16, head, max_seq_len=ms, max_batch=mb, use_qk_norm=False)}
-        if name != "malasun":
-            del make["malasun"]
+        z, make = design_engines(name, size, seed)
+        L = z["layers"]
+        dcfg = dense_config(z)
         res = {"config": z}
         for kind, new in make.items():
             rec = {"prefill": {}, "decode": {}}
@@ -217,10 +305,10 @@ def design_leg(name: str, sizes: list[str], seed: int) -> dict:
                 rec["prefill"][n] = {"ms": round(ms, 3), "tokens_per_s": round(n / ms * 1e3)}
             for B, ctx in ((1, 512), (1, 2048), (8, 512), (32, 512), (64, 512)):
                 e = new(ctx + 96, B)
-                toks = [int(t) for t in np.random.default_rng(ctx).integers(0, V, ctx)]
+                toks = np.random.default_rng(ctx).integers(0, V, (B, ctx + 1)).tolist()      # (unlike prompts: they choose unlike experts)
                 for b in range(B):
-                    e.prefill(toks, seq=b, want_last_logits=False)
-                e.set_state([1] * B, [ctx] * B)
+                    e.prefill(toks[b][:ctx], seq=b, want_last_logits=False)
+                e.set_state([t[ctx] for t in toks], [ctx] * B)
                 try:
                     e.capture(B)
                 except _hip.PgkError as err:          # the dense engine has no batch decode at these sizes
@@ -232,10 +320,11 @@ def design_leg(name: str, sizes: list[str], seed: int) -> dict:
                 if B == 1 or kind != "dense":
                     prof = e.profile_step(B, 8)
                     nb = stack_kernel_bytes(kind, z, V, ctx, B) if kind != "dense" else {k: v * (1 if k == "lmhead" else L) for k, v in kernel_bytes_per_launch(dcfg, ctx, B).items()}
-                    per = {"lmhead": 1, "attn": L // 2 if kind == "malasun" else L, "recur": L // 2}      # layers that have the class
+                    n_attn = {"malasun": L // 2, "ratasun": -(-L // 3)}.get(kind, L)
+                    per = {"lmhead": 1, "attn": n_attn, "recur": max(1, L - n_attn)}      # layers that have the class
                     rec["decode"][f"b{B}_ctx{ctx}"]["kernels"] = {
                         k: {"us_per_layer": round(us * n / per.get(k, L), 2), "hbm_frac": round(nb[k] / (us * n) / 1e3 / HBM_PEAK_GBS, 3)}
-                        for k, (us, n) in prof.items() if n and k in nb and k != "argmax"}
+                        for k, (us, n) in prof.items() if n and k in nb and k != "argmax" and (B == 1 or kind != "ratasun" or k in ("attn", "recur"))}
                 del e
             res[kind] = rec
         out["sizes"][size] = res
@@ -264,7 +353,7 @@ def main() -> None:
                     help="skip every extra leg (config 4 weak/strong; at N = 1 also context 2048 in bf16 and w8a16, config 5)")
     ap.add_argument("--config4-steps", type=int, default=32)
     ap.add_argument("--layers", type=int, default=0, help="debug only: override the layer count (result is then INVALID)")
-    ap.add_argument("--design", choices=["totolorn", "malasun"], help="instead of the headline: prefill / decode of a layer-list design beside its relatives")
+    ap.add_argument("--design", choices=["totolorn", "malasun", "ratasun"], help="instead of the headline: prefill / decode of a layer-list design beside its relatives")
     ap.add_argument("--design-sizes", default="w1024,w2048,w4096", help="with --design: which sizes")
     args = ap.parse_args()
 

@@ -334,7 +334,7 @@ def delta_oracle(rows, consts, heads, dim, vdim, eps=1e-4):
 
 @gpu
 @both
-@pytest.mark.parametrize("heads,kv,dim,vdim", [(2, 2, 64, 64), (4, 2, 32, 48), (2, 1, 128, 128), (3, 1, 24, 40), (1, 1, 144, 272), (2, 1, 16, 16), (1, 1, 4, 4), (1, 1, 64, 512)])
+@pytest.mark.parametrize("heads,kv,dim,vdim", [(3, 3, 64, 80), (4, 2, 32, 48), (2, 1, 128, 128), (3, 1, 24, 40), (1, 1, 144, 272), (2, 1, 16, 16), (1, 1, 4, 4), (1, 1, 64, 512)])
 def test_delta_rule(heads, kv, dim, vdim, dtype):
     """Both forms, lengths around their blocks and chunks; portions continue the state."""
     from pygpukit_amd.ops.basic import delta_rule
@@ -389,7 +389,7 @@ def test_a_write_far_back_is_still_there():
 
 @gpu
 @both
-@pytest.mark.parametrize("heads,groups,dim,vdim,parts", [(2, 1, 64, 64, 1), (6, 2, 24, 20, 3), (4, 4, 128, 128, 2), (1, 1, 256, 64, 1), (3, 3, 48, 144, 1), (1, 1, 6, 10, 1), (8, 2, 32, 48, 2),
+@pytest.mark.parametrize("heads,groups,dim,vdim,parts", [(2, 1, 64, 64, 1), (6, 2, 24, 20, 3), (4, 4, 128, 128, 2), (1, 1, 256, 64, 1), (3, 3, 48, 144, 1), (1, 1, 6, 10, 1), (6, 2, 32, 80, 2),
                                                          (2, 2, 16, 512, 4)])
 def test_state_space(heads, groups, dim, vdim, parts, dtype):
     from pygpukit_amd.ops.basic import state_space
@@ -420,7 +420,7 @@ def test_state_space(heads, groups, dim, vdim, parts, dtype):
 @gpu
 @both
 @pytest.mark.parametrize("n", [1, 3, 40, 130, 700])
-@pytest.mark.parametrize("E,top,groups,keep,ff,H", [(12, 3, 4, 3, 96, 256), (8, 2, 0, 0, 50, 90), (1, 1, 0, 0, 64, 64), (5, 5, 5, 5, 30, 200), (200, 8, 10, 4, 64, 192), (16, 1, 8, 2, 320, 576)])
+@pytest.mark.parametrize("E,top,groups,keep,ff,H", [(15, 4, 5, 3, 80, 320), (8, 2, 0, 0, 50, 90), (1, 1, 0, 0, 64, 64), (5, 5, 5, 5, 30, 200), (200, 8, 10, 4, 64, 192), (16, 1, 8, 2, 320, 576)])
 def test_experts(n, E, top, groups, keep, ff, H, dtype):
     """Routing by whole random rows, negative choices among them; one row, few rows per expert, and tiles of them."""
     from pygpukit_amd.ops.basic import mixture_of_experts
