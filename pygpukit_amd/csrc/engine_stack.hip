@@ -1575,7 +1575,10 @@ static pgk_status step_rows(Engine* e, int B, hipStream_t st, int* launches) {
     if (pgk_status r = head_rows<T>(s, (const T*)b.x, e->logits, B, st)) return r;
     PGK_CHECK_HIP(launch_k(rows_argmax_kernel, dim3(ROWS_ARGMAX_BLOCKS, B), dim3(256), 0, st, e->logits, c.vocab_size, e->amax_val, e->amax_idx));
     *launches += 3;
-    for (const auto& r : s->runs) *launches += 3 + (s->layers[r.layer].ff_pad ? 3 : 0);     // (one more where a projection's slabs or SwiGLU take a launch of their own)
+    for (const auto& r : s->runs) {                    // (one more where a projection's slabs or SwiGLU take a launch of their own)
+        const auto& L = s->layers[r.layer];
+        *launches += 3 + (!L.ff_pad ? 0 : L.ff == PGK_FF_MOE ? 5 : 3) + (r.pass >= 0 ? 2 : 0);
+    }
     return PGK_OK;
 }
 
