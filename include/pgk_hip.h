@@ -443,9 +443,35 @@ typedef struct {
 
 pgk_status pgk_engine_create(const pgk_model_config_t* cfg, const void* embed, const void* lm_head,
                              const void* final_norm, const pgk_layer_weights_t* layers, pgk_engine* out);
+/* Experts without a router: row tokens[i] of table [vocab, top] names those of row i, each weighted 1 / top; w_down gelu(w_up x) with the
+ * exact gelu, w_up [experts, ff, width], w_down [experts, width, ff]; widths multiples of 64, entries below `experts`. */
+pgk_status pgk_table_moe(const void* x, const int32_t* table, const int32_t* tokens, const void* w_up, const void* w_down, float* out, int n,
+                         int width, int ff, int experts, int top, pgk_dtype dt, pgk_stream s);
+/* Hyper-connections on fp32 streams x [n][streams][width]: u = sum_a in[a] x_a (in NULL: plain sum), and in place
+ * x_b <- sum_a mix[a][b] x_a + out[b] y with y rows of y_dt; at most 8 streams. */
+pgk_status pgk_hyper_read(const float* x, const float* in, float* u, int n, int streams, int width, pgk_stream s);
+pgk_status pgk_hyper_write(float* x, const void* y, const float* out, const float* mix, int n, int streams, int width, pgk_dtype y_dt, pgk_stream s);
+/* RMS norm of fp32 rows in `groups` equal parts, each over its own root mean square; weight fp32 [cols] */
+pgk_status pgk_group_norm_f32(const float* x, const float* weight, void* out, int rows, int cols, int groups, float eps, pgk_dtype out_dt, pgk_stream s);
+/* a r(z) + b r(z^2) + c r(z^3) + e per row, r(z) = z / sqrt(mean(z^2) + eps); act fp32 (a, b, c, e) on the device; bf16 or fp32 */
+pgk_status pgk_poly_norm(const void* z, void* out, int rows, int cols, const float* act, float eps, pgk_dtype dt, pgk_stream s);
+pgk_status pgk_gelu_erf(const void* x, void* y, size_t n, pgk_dtype dt, pgk_stream s);              /* z / 2 (1 + erf(z / sqrt 2)) */
+pgk_status pgk_soft_cap(const void* x, void* y, size_t n, float cap, pgk_dtype dt, pgk_stream s);  /* cap tanh(x / cap) */
+/* Heads x [n][heads][dim] -> out: RMS norm per head (norm fp32 [dim] or NULL), then columns i and i + rot / 2 turned by
+ * (first + row) * freq[i]; columns from rot on pass. */
+pgk_status pgk_head_norm_rope(const void* x, const float* norm, const float* freq, void* out, int n, int heads, int dim, int rot, int first,
+                              float eps, pgk_dtype dt, pgk_stream s);
+/* q [q_len][hq][dk], k [kv_len][hkv][dk], v [kv_len][hkv][dv], the queries being the last positions; row t of k is position first + t.
+ * score_h = sum_g talk[h][g] scale q_g . k (talk fp32 [hq][hq] or NULL) over the last `window` keys, or (chunked) those of the query's own
+ * chunk of `window` positions; softmax whose denominator also holds exp(sink[h]) (fp32 [hq] or NULL).  bf16 or fp32. */
+pgk_status pgk_talk_attention(const void* q, const void* k, const void* v, const float* talk, const float* sink, void* out, int hq, int hkv,
+                              int q_len, int kv_len, int first, int dk, int dv, float scale, int window, int chunked, pgk_dtype dt, pgk_stream s);
+
 /* Layer-list decoders (csrc/engine_stack.hip): fp32 residual stream, one of several mixers per layer, SwiGLU / xIELU, a mixture of
  * experts or no feed-forward; every layer has its own sizes.  A layer is a sandwich (mixer, then feed-forward, a norm after each and
- * optionally before it) or parallel (one norm, mixer and feed-forward read its output, both results are added).  A run of layers may
+ * optionally before it), parallel (one norm, mixer and feed-forward read its output, both results are added) or hyper-connected
+ * (PGK_BLOCK_HYPER: `streams` residual streams; a sublayer reads the norm of a combination of them and its output goes to all of them
+ * while they mix; norms in norm_groups equal parts of the width).  A run of layers may
  * be passed several times with the same weights, each pass with caches of its own; a pass starts with
  * x <- loop_in [x; embedding row] + loop_step[pass].  dtype PGK_BF16 or PGK_F32 is the
  * element type of the tables, matrices, taps, activations and caches; norm weights, biases and gates' constants are fp32 with any
@@ -469,11 +495,19 @@ pgk_status pgk_engine_create(const pgk_model_config_t* cfg, const void* embed, c
  * PGK_MIX_SSD        state-space duality (pgk_state_space) after taps with bias and SiLU on x, B, C; the result times silu(z) and normed in
  *                    norm_parts equal parts of its heads x vdim elements.  dim: the state's; kv_heads: the groups.  w_in rows: heads x vhead_pad
  *                    x | kv_heads x head_pad B | the same C | heads x vhead_pad z | heads dt.  decay, dt_bias, skip [heads].
+ * PGK_MIX_TALK       grouped heads over a K/V ring: q, k, v = w_in x + b_in, RMS norm per head (q_norm, k_norm [head_pad]), the first rot
+ *                    columns of q and k turned by position x rot_freq[i], i with i + rot / 2; the heads' scores are mixed by talk
+ *                    [heads][heads] (NULL: not); softmax with exp(sink[h]) in the denominator (NULL: without); window as a sliding
+ *                    window, or chunked: only keys of the query's own chunk of `window` positions.  w_in rows: heads x head_pad q |
+ *                    kv_heads x head_pad k | the same v; with kv_from >= 0 only q.  b_o [Wp] is added to the out-projection.
+ * PGK_FF_POLY        w_down p(w_gate_up x), p(z) = a r(z) + b r(z^2) + c r(z^3) + e with r the RMS norm over the row; act [4].  Hyper only.
+ * PGK_FF_TABLE       row `token` of table [vocab][top] names experts w_down gelu(w_gate_up x), each weighted 1 / top; shared_pad > 0: one more
+ *                    for all tokens, w_shared_down gelu(w_shared_up x), times sigmoid(w_shared_gate . x).  Hyper only.
  * PGK_FF_MOE         experts of ff_pad, `top` of them per token (see pgk_moe); behind w_in's n_in rows stand the router's, up to a
  *                    multiple of 64.  Parallel layers only; SANDWICH layers take the dense forms. */
-typedef enum { PGK_MIX_LATENT = 0, PGK_MIX_ATTENTION = 1, PGK_MIX_HGRN2 = 2, PGK_MIX_DELTA = 3, PGK_MIX_SSD = 4 } pgk_mixer;
-typedef enum { PGK_FF_SWIGLU = 0, PGK_FF_XIELU = 1, PGK_FF_MOE = 2 } pgk_ff;
-typedef enum { PGK_BLOCK_SANDWICH = 0, PGK_BLOCK_PARALLEL = 1 } pgk_block;
+typedef enum { PGK_MIX_LATENT = 0, PGK_MIX_ATTENTION = 1, PGK_MIX_HGRN2 = 2, PGK_MIX_DELTA = 3, PGK_MIX_SSD = 4, PGK_MIX_TALK = 5 } pgk_mixer;
+typedef enum { PGK_FF_SWIGLU = 0, PGK_FF_XIELU = 1, PGK_FF_MOE = 2, PGK_FF_POLY = 3, PGK_FF_TABLE = 4 } pgk_ff;
+typedef enum { PGK_BLOCK_SANDWICH = 0, PGK_BLOCK_PARALLEL = 1, PGK_BLOCK_HYPER = 2 } pgk_block;
 typedef struct {
     int vocab_size, width, num_layers, max_positions, max_seq_len, max_batch;
     float norm_eps, residual_mult;
@@ -482,6 +516,8 @@ typedef struct {
     int loop_start, loop_stop, loop_times;         /* layers loop_start .. loop_stop - 1 run loop_times times (0: no loop) */
     const void* loop_in;                           /* [Wp, 2 Wp] */
     const float* loop_step;                        /* [loop_times, Wp] */
+    int streams, norm_groups;                      /* hyper-connected layers (others: 1, 1) */
+    float logit_cap;                               /* > 0: logits become cap * tanh(logits / cap) */
 } pgk_stack_config_t;
 typedef struct {
     int mixer, ff;                                 /* pgk_mixer, pgk_ff */
@@ -489,7 +525,8 @@ typedef struct {
     int window, taps, kv_from;                     /* window: keys a query sees, itself included; kv_from: -1 or an earlier layer */
     int head_pad, vhead_pad, rank_pad, n_in, n_att, ff_pad;
     int gated, rot, norm_parts, rank_a, rank_g;
-    int experts, top, groups, keep;                /* PGK_FF_MOE; groups 0: none */
+    int experts, top, groups, keep;                /* PGK_FF_MOE (groups 0: none), PGK_FF_TABLE */
+    int chunked, ff_dim, shared_pad;               /* ff_dim: PGK_FF_POLY, the true feed-forward width */
     float scale, act_pos, act_neg, router_scale;   /* act_*: pgk_xielu's a and b */
     const float *norm1, *norm1b, *norm2, *norm2b;  /* [Wp]; norm1 / norm2 NULL: the sublayer reads the stream itself */
     const void* w_in;                              /* [n_in, Wp] */
@@ -500,12 +537,17 @@ typedef struct {
     const float* c_norm;                           /* latent: [rank_pad] */
     const void* w_ukv;                             /* latent: [2 heads head_pad, rank_pad]: key rows, then value rows */
     const void* w_o;                               /* [Wp, n_att] */
-    const void* w_gate_up;                         /* [2 ff_pad, Wp]; xIELU: [ff_pad, Wp]; MoE: [experts, 2 ff_pad, Wp] */
-    const void* w_down;                            /* [Wp, ff_pad]; MoE: [experts, Wp, ff_pad] */
-    const float* rot_freq;                         /* latent: [rot / 2] */
+    const void* w_gate_up;                         /* [2 ff_pad, Wp]; xIELU, poly: [ff_pad, Wp]; MoE: [experts, 2 ff_pad, Wp]; table: [experts, ff_pad, Wp] */
+    const void* w_down;                            /* [Wp, ff_pad]; MoE, table: [experts, Wp, ff_pad] */
+    const float* rot_freq;                         /* latent, talk: [rot / 2] */
     const float *decay, *dt_bias, *skip, *conv_bias;
     const void *w_a2, *w_g2;                       /* delta: [heads head_pad, rank_a], [heads vhead_pad, rank_g] */
     const float* correction;                       /* MoE: [experts] */
+    const float *b_o, *talk, *sink;                /* talk: [Wp], [heads, heads], [heads] */
+    const float *hyper1, *hyper2;                  /* in [streams] | out [streams] | mix [streams from][streams to], of mixer and feed-forward */
+    const float* act;                              /* PGK_FF_POLY: [4] */
+    const int32_t* table;                          /* PGK_FF_TABLE: [vocab, top] */
+    const void *w_shared_up, *w_shared_down, *w_shared_gate;  /* [shared_pad, Wp], [Wp, shared_pad], [Wp] */
 } pgk_stack_layer_t;
 /* embed [vocab, width], pos_embed [max_positions, width] or NULL, head [vocab, Wp], final_norm [Wp] */
 pgk_status pgk_engine_create_stack(const pgk_stack_config_t* cfg, const void* embed, const void* pos_embed, const void* head,

@@ -49,20 +49,21 @@ class LayerWeights(C.Structure):
 class StackConfig(C.Structure):
     _fields_ = [(n, C.c_int) for n in ("vocab_size", "width", "num_layers", "max_positions", "max_seq_len", "max_batch")] + \
                [("norm_eps", C.c_float), ("residual_mult", C.c_float), ("dtype", C.c_int)] + \
-               [(n, C.c_int) for n in ("block", "layer_norm", "loop_start", "loop_stop", "loop_times")] + [("loop_in", C.c_void_p), ("loop_step", C.c_void_p)]
+               [(n, C.c_int) for n in ("block", "layer_norm", "loop_start", "loop_stop", "loop_times")] + [("loop_in", C.c_void_p), ("loop_step", C.c_void_p), ("streams", C.c_int), ("norm_groups", C.c_int), ("logit_cap", C.c_float)]
 
 
 class StackLayer(C.Structure):
     _fields_ = [(n, C.c_int) for n in ("mixer", "ff", "heads", "kv_heads", "dim", "vdim", "rank", "window", "taps", "kv_from", "head_pad", "vhead_pad", "rank_pad",
-                                       "n_in", "n_att", "ff_pad", "gated", "rot", "norm_parts", "rank_a", "rank_g", "experts", "top", "groups", "keep")] + \
+                                       "n_in", "n_att", "ff_pad", "gated", "rot", "norm_parts", "rank_a", "rank_g", "experts", "top", "groups", "keep", "chunked", "ff_dim", "shared_pad")] + \
                [(n, C.c_float) for n in ("scale", "act_pos", "act_neg", "router_scale")] + \
                [(n, C.c_void_p) for n in ("norm1", "norm1b", "norm2", "norm2b", "w_in", "b_in", "conv", "q_norm", "k_norm", "slopes", "lower", "o_norm", "c_norm",
-                                          "w_ukv", "w_o", "w_gate_up", "w_down", "rot_freq", "decay", "dt_bias", "skip", "conv_bias", "w_a2", "w_g2", "correction")]
+                                          "w_ukv", "w_o", "w_gate_up", "w_down", "rot_freq", "decay", "dt_bias", "skip", "conv_bias", "w_a2", "w_g2", "correction", "b_o", "talk", "sink",
+                                          "hyper1", "hyper2", "act", "table", "w_shared_up", "w_shared_down", "w_shared_gate")]
 
 
-MIX_LATENT, MIX_ATTENTION, MIX_HGRN2, MIX_DELTA, MIX_SSD = 0, 1, 2, 3, 4      # pgk_mixer
-FF_SWIGLU, FF_XIELU, FF_MOE = 0, 1, 2                                           # pgk_ff
-BLOCK_SANDWICH, BLOCK_PARALLEL = 0, 1                                           # pgk_block
+MIX_LATENT, MIX_ATTENTION, MIX_HGRN2, MIX_DELTA, MIX_SSD, MIX_TALK = 0, 1, 2, 3, 4, 5      # pgk_mixer
+FF_SWIGLU, FF_XIELU, FF_MOE, FF_POLY, FF_TABLE = 0, 1, 2, 3, 4                                           # pgk_ff
+BLOCK_SANDWICH, BLOCK_PARALLEL, BLOCK_HYPER = 0, 1, 2                                           # pgk_block
 
 
 # name -> (argtypes); every function returns pgk_status (int) unless listed in _NON_STATUS
@@ -128,6 +129,10 @@ _PROTOS = {
     "pgk_conv_silu": [_V, _V, _V, _V, _V, _I, _I, _I, _I, _V],
     "pgk_delta_rule": [_V] * 11 + [_I] * 6 + [_F, _I, _V], "pgk_state_space": [_V] * 9 + [_I] * 7 + [_F, _I, _V],
     "pgk_moe": [_V] * 6 + [_I] * 7 + [_F, _I, _V], "pgk_layernorm_f32": [_V, _V, _V, _I, _I, _F, _I, _V],
+    "pgk_table_moe": [_V] * 6 + [_I] * 6 + [_V], "pgk_hyper_read": [_V, _V, _V, _I, _I, _I, _V], "pgk_hyper_write": [_V] * 4 + [_I] * 4 + [_V],
+    "pgk_group_norm_f32": [_V, _V, _V, _I, _I, _I, _F, _I, _V], "pgk_poly_norm": [_V, _V, _I, _I, _V, _F, _I, _V], "pgk_gelu_erf": [_V, _V, _Z, _I, _V],
+    "pgk_soft_cap": [_V, _V, _Z, _F, _I, _V], "pgk_head_norm_rope": [_V] * 4 + [_I] * 5 + [_F, _I, _V],
+    "pgk_talk_attention": [_V] * 6 + [_I] * 7 + [_F, _I, _I, _I, _V],
     "pgk_latent_rows": [_V, _V, _V, _V, _I, _I, _I, _I, _F, _I, _V], "pgk_rotate_pairs": [_V, _V, _I, _I, _I, _I, _I, _I, _V],
     "pgk_gated_recurrence": [_V, _V, _V, _V, _V, _V, _V, _V, _I, _I, _I, _I, _I, _F, _I, _V],
     "pgk_head_gate": [_V, _V, _I, _I, _I, _I64, _I, _V], "pgk_pad_2d": [_V, _V, _I, _I, _I, _I, _I, _V],

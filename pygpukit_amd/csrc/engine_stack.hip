@@ -6,6 +6,9 @@
 //   x   <- x + m * rho(W_d act(W_u h); n2b),        h = rho(x; n2) or x
 // Parallel layers: one norm (RMS or layer norm), a mixture of experts (moe.hip.h) or no feed-forward
 //   x   <- x + m * (O mixer(h) + moe(h)),           h = nu(x; n1)
+// Hyper-connected layers: s streams instead of one (hyper.hip.h), norms in groups; dense feed-forwards with a polynomial-norm activation
+// (W_d p(W_u h)) or experts that a table of token ids chooses, beside a gated shared one
+//   u = sum_a c_a x_a,   y = F(nu(u)),   x_b <- sum_a M_ab x_a + d_b y      for F the mixer, then the feed-forward
 // A stretch of layers may run several times over with the same weights (`Run`: one pass of one layer, with a cache of its own); pass t
 // starts with  x <- L [x; embedding] + s_t.
 //
@@ -15,6 +18,7 @@
 //                     position instead (the rotary part of the key, one for all heads).  The kernels are in this file.
 //   attention         taps over time and norms on q, k, v, a K/V ring (which another layer may own), distance bias, elementwise gate:
 //                     ops_gated_attn.hip
+//   talk              norms per head and rotation, a K/V ring over a window or chunk, mixed scores, a sink: ops_talk.hip
 //   hgrn2, ssd        linear recurrences with an fp32 state per sequence and head: ops_recurrence.hip
 //   delta             gated delta rule with a decay per key channel: ops_delta.hip
 // In a step a mixer takes the in-projection row(s) and leaves the rows that the out-projection multiplies.
@@ -35,13 +39,18 @@
 // (one row: a few KB from L2), so it costs no launch.
 // A parallel layer, one sequence: in_proj (pending add, norm; router logits are rows of the same matrix), the mixer, moe_up (choice,
 // SwiGLU of the chosen experts), out (W_o and the chosen experts' down projections as one product).
+// A hyper-connected layer, one sequence: in_proj (pending update of the streams, their combination and norm in the prologue), head norms and
+// rotation, attn, merge, oproj (+ bias), up, down (activation in the prologue; experts: the chosen ones and the shared one in one launch).
 // Several sequences and prompts: the same kernels on rows, the norms as a launch of their own and the projections on the GEMM family
 // (pgk_gemm_nt: GEMV up to 8 rows, weight-streaming MFMA up to 128, tiled MFMA beyond).
 // All widths are padded with zeros by the caller: every K is a multiple of 64, head widths are 64, 128 or a larger multiple of 64.
 
+#include <algorithm>
 #include <cstring>
 
 #include "engine_state.hip.h"
+#include "gemm_epilogues.hip.h"
+#include "hyper.hip.h"
 #include "latent.hip.h"
 #include "mixers.hip.h"
 #include "moe.hip.h"
@@ -54,8 +63,8 @@ pgk_status wsgemm_nt(const bf16* a, int lda, const void* w, const bf16* wscale, 
 bool engine_gemm_swiglu_ok(int M, int I, int K, bool fp8);     // ops_gemm.hip
 pgk_status engine_gemm_swiglu_nt(const bf16* A, const void* W, const bf16* wscale, bool fp8, bf16* act, int M, int I, int K, hipStream_t st, bool packed = false);
 
-bool engine_gemm_xielu_ok(int M, int N, int K);                // ops_gemm.hip
-pgk_status engine_gemm_xielu_nt(const bf16* A, const bf16* W, bf16* act, int M, int N, int K, float pos, float neg, hipStream_t st);
+bool engine_gemm_act_ok(int M, int N, int K);                  // ops_gemm.hip
+pgk_status engine_gemm_act_nt(const bf16* A, const bf16* W, bf16* act, int M, int N, int K, const ActArgs& xa, hipStream_t st);
 
 int wsgemm_pick_splits(int N, int K, bool allow_split);        // ops_wsgemm.hip
 int engine_gemm_pick_splits(int M, int N, int K);              // ops_gemm.hip: split-K slabs for prompts whose tiles do not cover the chip
@@ -64,8 +73,8 @@ pgk_status engine_gemm_nt_slabs(const bf16* A, const void* W, float* slabs, int 
 constexpr float LOG2E = 1.4426950408889634f;
 
 // -------------------------------------------------------------------------------------------- one-row projection
-enum { SP_NORM = 0, SP_PLAIN = 1, SP_ADD = 2, SP_CAT = 3 };
-enum { SE_STORE = 0, SE_SWIGLU = 1, SE_LOGITS = 2, SE_XIELU = 3 };
+enum { SP_NORM = 0, SP_PLAIN = 1, SP_ADD = 2, SP_CAT = 3, SP_HYPER = 4, SP_POLY = 5 };
+enum { SE_STORE = 0, SE_SWIGLU = 1, SE_LOGITS = 2, SE_XIELU = 3, SE_TABLE = 4 };
 
 struct StackGemvArgs {
     const void* w;            // [N][K] (SE_SWIGLU: [2 N][K], gate rows then up rows)
@@ -85,6 +94,18 @@ struct StackGemvArgs {
     float* out;               // [N]
     float* amax_val; int* amax_idx;
     float act_pos, act_neg;   // SE_XIELU
+    const float* bias;        // SE_STORE: added to the result (null: none)
+    float cap;                // SE_LOGITS: soft cap (0: none)
+    // SP_HYPER: stream s at x + s * x_stream, y with `upd` the pending sublayer output, `in` the combination (null: sum), norm in groups;
+    // x_out: [S][K].  SP_POLY: the input is the polynomial-norm activation of x, W true columns, act [4]
+    int S, x_stream, groups;
+    const float *upd, *in, *act;
+    // SE_TABLE: rows of the shared expert (fs of them, w), then of the token's `top` experts (ff each, w2 [E][ff][K]), then the shared one's gate
+    // (w3); gelu, gelu / top, sigmoid.  ids: where workgroup 0 writes the experts
+    const void *w2, *w3;
+    const int32_t* table;
+    int fs, top, ff;
+    int32_t* ids;
 };
 
 // s + 16 bytes of a weight row . the same piece of the LDS row
@@ -117,8 +138,158 @@ __global__ __launch_bounds__(256) void stack_gemv_kernel(unsigned long long* tl,
         if constexpr (EPI == SE_SWIGLU) return r < R / 2 ? min(n0 + r, N - 1) : N + min(n0 + r - R / 2, N - 1);
         else return min(n0 + r, N - 1);
     };
+    const int32_t* chosen = nullptr;
+    if constexpr (EPI == SE_TABLE) {
+        chosen = a.table + (size_t)*a.tok * a.top;
+        if (blockIdx.x == 0) for (int i = threadIdx.x; i < a.top; i += 256) a.ids[i] = chosen[i];
+    }
+    auto row_at = [&](int n0, int r) -> const WT* {
+        if constexpr (EPI == SE_TABLE) {
+            const int n = min(n0 + r, N - 1), j = n - a.fs;
+            if (j < 0) return w + (size_t)n * K;
+            if (j >= a.top * a.ff) return reinterpret_cast<const WT*>(a.w3);
+            const int k = j / a.ff;
+            return reinterpret_cast<const WT*>(a.w2) + ((size_t)chosen[k] * a.ff + (j - k * a.ff)) * K;
+        } else return w + (size_t)row_of(n0, r) * K;
+    };
     uint4 pre[R][C > 0 ? C : 1];
-    if constexpr (PRO == SP_CAT) {
+    if constexpr (PRO == SP_HYPER) {
+        float* xf = reinterpret_cast<float*>(smem + (size_t)((K + CH - 1) / CH * CH > C * CH ? (K + CH - 1) / CH * CH : C * CH) * sizeof(WT));   // [K], [groups]
+        const int S = a.S;
+        auto in_of = [&](int s) { return a.in ? a.in[s] : 1.0f; };
+        auto coef_x = [&](int s) {
+            if (!a.y) return in_of(s);
+            float c = 0.f;
+            for (int t = 0; t < S; ++t) c = fmaf(a.upd[2 * S + s * S + t], in_of(t), c);
+            return c;
+        };
+        float cy = 0.f;
+        if (a.y) for (int t = 0; t < S; ++t) cy = fmaf(a.upd[S + t], in_of(t), cy);
+        if constexpr (C > 0) {                                     // S <= 4
+            constexpr int NT = (C * CH + 1023) / 1024;
+            const float4 zero = {0.f, 0.f, 0.f, 0.f};
+            float4 x[NT][4], y[NT], gm[NT], v[NT];
+#pragma unroll
+            for (int t = 0; t < NT; ++t) {
+                const int i = min((int)(threadIdx.x + 256 * t) * 4, K - 4);
+#pragma unroll
+                for (int s = 0; s < 4; ++s) {
+                    x[t][s] = zero;
+                    if (s < S) x[t][s] = *reinterpret_cast<const float4*>(a.x + (size_t)s * a.x_stream + i);
+                }
+                y[t] = zero;
+                if (a.y) y[t] = *reinterpret_cast<const float4*>(a.y + i);
+                gm[t] = *reinterpret_cast<const float4*>(a.gamma + i);
+            }
+            __builtin_amdgcn_sched_barrier(0);
+            const int nf = min(wave * OUT, N - 1);
+#pragma unroll
+            for (int r = 0; r < R; ++r) {
+                const WT* wr = row_at(nf, r);
+#pragma unroll
+                for (int c = 0; c < C; ++c) pre[r][c] = load_nt16(wr + min(c * CH + lane * NW, K - NW));
+            }
+            __builtin_amdgcn_sched_barrier(0);
+            float cx[4];
+#pragma unroll
+            for (int s = 0; s < 4; ++s) cx[s] = s < S ? coef_x(s) : 0.f;
+            auto mul = [](float c, const float4& p, const float4& q) { return make_float4(fmaf(c, p.x, q.x), fmaf(c, p.y, q.y), fmaf(c, p.z, q.z), fmaf(c, p.w, q.w)); };
+            float ss = 0.f;
+#pragma unroll
+            for (int t = 0; t < NT; ++t) {
+                const int i = (threadIdx.x + 256 * t) * 4;
+                v[t] = mul(cy, y[t], zero);
+#pragma unroll
+                for (int s = 0; s < 4; ++s) v[t] = mul(cx[s], x[t][s], v[t]);
+                if (i >= K) v[t] = zero;
+                ss += v[t].x * v[t].x + v[t].y * v[t].y + v[t].z * v[t].z + v[t].w * v[t].w;
+                if (a.y && a.x_out && blockIdx.x == t % gridDim.x && i < K)         // the new streams, a piece per workgroup
+                    for (int o = 0; o < S; ++o) {
+                        float4 z = mul(a.upd[S + o], y[t], zero);
+#pragma unroll
+                        for (int s = 0; s < 4; ++s) if (s < S) z = mul(a.upd[2 * S + s * S + o], x[t][s], z);
+                        *reinterpret_cast<float4*>(a.x_out + (size_t)o * K + i) = z;
+                    }
+                if (a.groups > 1 && i < K) *reinterpret_cast<float4*>(xf + i) = v[t];
+            }
+            if (a.groups == 1) {
+                const float inv = 1.0f / sqrtf(block_sum(ss, red) / a.W + a.eps);
+#pragma unroll
+                for (int t = 0; t < NT; ++t) { v[t].x *= inv; v[t].y *= inv; v[t].z *= inv; v[t].w *= inv; }
+            } else {
+                __syncthreads();
+                group_rstd(xf, a.W, a.groups, a.eps, xf + K);
+                const int gs = a.W / a.groups;
+                const float* rs = xf + K;
+#pragma unroll
+                for (int t = 0; t < NT; ++t) {
+                    const int i = min((int)(threadIdx.x + 256 * t) * 4, K - 4), top = a.groups - 1;
+                    if ((gs & 3) == 0) { const float q = rs[min(i / gs, top)]; v[t].x *= q; v[t].y *= q; v[t].z *= q; v[t].w *= q; }
+                    else { v[t].x *= rs[min(i / gs, top)]; v[t].y *= rs[min((i + 1) / gs, top)]; v[t].z *= rs[min((i + 2) / gs, top)]; v[t].w *= rs[min((i + 3) / gs, top)]; }
+                }
+            }
+#pragma unroll
+            for (int t = 0; t < NT; ++t) {
+                const int i = (threadIdx.x + 256 * t) * 4;
+                if (i < C * CH) store4<WT>(xs + i, i < K ? make_float4(v[t].x * gm[t].x, v[t].y * gm[t].y, v[t].z * gm[t].z, v[t].w * gm[t].w) : zero);
+            }
+        } else {
+            for (int i = threadIdx.x; i < K; i += 256) {
+                const float y = a.y ? a.y[i] : 0.f;
+                float u = cy * y;
+                for (int s = 0; s < S; ++s) u = fmaf(coef_x(s), a.x[(size_t)s * a.x_stream + i], u);
+                xf[i] = u;
+                if (a.y && a.x_out && blockIdx.x == (i >> 10) % gridDim.x)
+                    for (int o = 0; o < S; ++o) {
+                        float z = a.upd[S + o] * y;
+                        for (int s = 0; s < S; ++s) z = fmaf(a.upd[2 * S + s * S + o], a.x[(size_t)s * a.x_stream + i], z);
+                        a.x_out[(size_t)o * K + i] = z;
+                    }
+            }
+            __syncthreads();
+            group_rstd(xf, a.W, a.groups, a.eps, xf + K);
+            const int gs = a.W / a.groups;
+            for (int i = threadIdx.x; i < K; i += 256) xs[i] = from_f<WT>(i < a.W ? xf[i] * xf[K + i / gs] * a.gamma[i] : 0.f);
+        }
+    } else if constexpr (PRO == SP_POLY) {
+        float s2 = 0.f, s4 = 0.f, s6 = 0.f;
+        auto add = [&](float z) { const float z2 = z * z, z4 = z2 * z2; s2 += z2; s4 += z4; s6 = fmaf(z4, z2, s6); };
+        if constexpr (C > 0) {
+            constexpr int NT = (C * CH + 1023) / 1024;
+            float4 v[NT];
+#pragma unroll
+            for (int t = 0; t < NT; ++t) v[t] = *reinterpret_cast<const float4*>(a.x + min((int)(threadIdx.x + 256 * t) * 4, K - 4));
+            __builtin_amdgcn_sched_barrier(0);
+            const int nf = min(wave * OUT, N - 1);
+#pragma unroll
+            for (int r = 0; r < R; ++r)
+#pragma unroll
+                for (int c = 0; c < C; ++c) pre[r][c] = load_nt16(row_at(nf, r) + min(c * CH + lane * NW, K - NW));
+            __builtin_amdgcn_sched_barrier(0);
+#pragma unroll
+            for (int t = 0; t < NT; ++t)
+                if ((int)(threadIdx.x + 256 * t) * 4 < K) { add(v[t].x); add(v[t].y); add(v[t].z); add(v[t].w); }      // (columns W .. K are zero)
+            s2 = block_sum(s2, red); s4 = block_sum(s4, red); s6 = block_sum(s6, red);
+            const float3 cf = poly_coef(a.act, s2, s4, s6, a.W, a.eps);
+            const float e = a.act[3];
+#pragma unroll
+            for (int t = 0; t < NT; ++t) {
+                const int i = (threadIdx.x + 256 * t) * 4;
+                auto at = [&](int j, float z) { return j < a.W ? poly_at(cf, e, z) : 0.f; };
+                if (i < C * CH) store4<WT>(xs + i, make_float4(at(i, v[t].x), at(i + 1, v[t].y), at(i + 2, v[t].z), at(i + 3, v[t].w)));
+            }
+        } else {
+            for (int i = threadIdx.x * 4; i < K; i += 1024) { const float4 q = *reinterpret_cast<const float4*>(a.x + i); add(q.x); add(q.y); add(q.z); add(q.w); }
+            s2 = block_sum(s2, red); s4 = block_sum(s4, red); s6 = block_sum(s6, red);
+            const float3 cf = poly_coef(a.act, s2, s4, s6, a.W, a.eps);
+            const float e = a.act[3];
+            auto at = [&](int j, float z) { return j < a.W ? poly_at(cf, e, z) : 0.f; };
+            for (int i = threadIdx.x * 4; i < K; i += 1024) {
+                const float4 q = *reinterpret_cast<const float4*>(a.x + i);
+                store4<WT>(xs + i, make_float4(at(i, q.x), at(i + 1, q.y), at(i + 2, q.z), at(i + 3, q.w)));
+            }
+        }
+    } else if constexpr (PRO == SP_CAT) {
         const WT* er = reinterpret_cast<const WT*>(a.embed) + (size_t)*a.tok * a.W;
         const float* from = a.base ? a.base : a.x;
         const int half = K / 2, pad = (K + CH - 1) / CH * CH;
@@ -274,9 +445,11 @@ __global__ __launch_bounds__(256) void stack_gemv_kernel(unsigned long long* tl,
         if (C > 0) {
             if (g != wave) {
 #pragma unroll
-                for (int r = 0; r < R; ++r)
+                for (int r = 0; r < R; ++r) {
+                    const WT* wr = row_at(n0, r);
 #pragma unroll
-                    for (int c = 0; c < C; ++c) pre[r][c] = load_nt16(w + (size_t)row_of(n0, r) * K + min(c * CH + lane * NW, K - NW));
+                    for (int c = 0; c < C; ++c) pre[r][c] = load_nt16(wr + min(c * CH + lane * NW, K - NW));
+                }
             }
 #pragma unroll
             for (int c = 0; c < (C > 0 ? C : 1); ++c)
@@ -285,7 +458,7 @@ __global__ __launch_bounds__(256) void stack_gemv_kernel(unsigned long long* tl,
         } else {
             const WT* wrow[R];
 #pragma unroll
-            for (int r = 0; r < R; ++r) wrow[r] = w + (size_t)row_of(n0, r) * K;
+            for (int r = 0; r < R; ++r) wrow[r] = row_at(n0, r);
             gemv_rows<WT, WT, 1, R>(wrow, xs, K, K, lane, acc);
         }
 #pragma unroll
@@ -297,6 +470,12 @@ __global__ __launch_bounds__(256) void stack_gemv_kernel(unsigned long long* tl,
                     float o = acc[r][0];
                     if constexpr (EPI == SE_SWIGLU) o = o / (1.0f + (std::is_same<WT, float>::value ? expf(-o) : __expf(-o))) * acc[r + R / 2][0];
                     if constexpr (EPI == SE_XIELU) o = xielu<std::is_same<WT, float>::value>(o, a.act_pos, a.act_neg);
+                    if constexpr (EPI == SE_STORE) { if (a.bias) o += a.bias[n0 + r]; }
+                    if constexpr (EPI == SE_LOGITS) { if (a.cap > 0.f) o = soft_cap(o, a.cap); }
+                    if constexpr (EPI == SE_TABLE) {
+                        const int j = n0 + r - a.fs;
+                        o = j >= a.top * a.ff ? 1.0f / (1.0f + expf(-o)) : j < 0 ? gelu_erf(o) : gelu_erf(o) / a.top;
+                    }
                     a.out[n0 + r] = o;
                     if constexpr (EPI == SE_LOGITS) { if (o > best_v) { best_v = o; best_i = n0 + r; } }
                 }
@@ -320,7 +499,8 @@ __global__ __launch_bounds__(256) void stack_gemv_kernel(unsigned long long* tl,
 template <class WT, int R, int PRO, int EPI, int C>
 static pgk_status stack_gemv_c(const StackGemvArgs& a, int grid, hipStream_t st) {
     constexpr int CH = 64 * WTraits<WT>::NW;
-    const size_t lds = (size_t)ceil_div(a.K, CH) * CH * sizeof(WT) > (size_t)C * CH * sizeof(WT) ? (size_t)ceil_div(a.K, CH) * CH * sizeof(WT) : (size_t)C * CH * sizeof(WT);
+    size_t lds = (size_t)ceil_div(a.K, CH) * CH * sizeof(WT) > (size_t)C * CH * sizeof(WT) ? (size_t)ceil_div(a.K, CH) * CH * sizeof(WT) : (size_t)C * CH * sizeof(WT);
+    if (PRO == SP_HYPER && (C == 0 || a.groups > 1)) lds += (size_t)(a.K + a.groups) * 4;
     auto kfn = &stack_gemv_kernel<WT, R, PRO, EPI, C>;
     PGK_REQUIRE(lds <= 156 * 1024, "engine: a row of %d does not fit LDS", a.K);
     static bool attr_done = false;
@@ -338,7 +518,7 @@ static pgk_status stack_gemv_r(const StackGemvArgs& a, hipStream_t st, int force
     int grid = force_grid ? force_grid : ceil_div(a.N, OUT * 4);
     if (grid > 1024) grid = 1024;
     if constexpr (std::is_same<WT, bf16>::value) {
-        const int c = ceil_div(a.K, 512);
+        const int c = PRO == SP_HYPER && a.S > 4 ? 99 : ceil_div(a.K, 512);
         if constexpr (R * 2 <= 16) { if (c <= 2) return stack_gemv_c<WT, R, PRO, EPI, 2>(a, grid, st); }
         if constexpr (R * 4 <= 16) { if (c <= 4) return stack_gemv_c<WT, R, PRO, EPI, 4>(a, grid, st); }
         if constexpr (R * 8 <= 16) { if (c <= 8) return stack_gemv_c<WT, R, PRO, EPI, 8>(a, grid, st); }
@@ -799,6 +979,7 @@ struct MoeOneArgs {
     float* act;                           // [top][ff], times the choice's weight
     int32_t* ids;                         // [top]
     const void* w_o; const float* a; int n_att;
+    const float* gate;                    // moe_out_one: a is multiplied by *gate (null: not)
     float* y; int N;
 };
 
@@ -849,7 +1030,7 @@ __global__ __launch_bounds__(256) void moe_up_one_kernel(unsigned long long* tl,
     tls.end();
 }
 
-// y = W_o a + sum over the chosen experts of W_down act: one row of 16-byte pieces that starts in W_o and goes on through the experts'
+// y = W_o (gate a) + sum over the chosen experts of W_down act: one row of 16-byte pieces that starts in W_o and goes on through the experts'
 template <class WT, int R>
 __global__ __launch_bounds__(256) void moe_out_one_kernel(unsigned long long* tl, MoeOneArgs a) {
     const TLStamp tls(tl);
@@ -859,7 +1040,8 @@ __global__ __launch_bounds__(256) void moe_out_one_kernel(unsigned long long* tl
     WT* xs = reinterpret_cast<WT*>(smem);                         // [n_att + top ff, one piece of zeros]
     const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6, top = a.r.top, na = a.n_att / NW, nf = a.ff / NW, np = na + top * nf, len = np * NW;
     if ((int)threadIdx.x < top) ids[threadIdx.x] = a.ids[threadIdx.x];
-    for (int i = threadIdx.x; i < len + NW; i += 256) xs[i] = from_f<WT>(i < a.n_att ? a.a[i] : i < len ? a.act[i - a.n_att] : 0.f);
+    const float gate = a.gate ? *a.gate : 1.0f;
+    for (int i = threadIdx.x; i < len + NW; i += 256) xs[i] = from_f<WT>(i < a.n_att ? gate * a.a[i] : i < len ? a.act[i - a.n_att] : 0.f);
     __syncthreads();
     for (int n0 = (blockIdx.x * 4 + wid) * R; n0 < a.N; n0 += gridDim.x * 4 * R) {
         float acc[R];
@@ -977,15 +1159,19 @@ __global__ __launch_bounds__(256) void latent_rows_kernel(const RowPlace* pl, T*
     }
 }
 
-// argmax partials of fp32 logit rows: grid (nblk, rows)
-__global__ __launch_bounds__(256) void rows_argmax_kernel(unsigned long long* tl, const float* logits, int V, float* amax_val, int* amax_idx) {
+// argmax partials of fp32 logit rows, which are soft-capped on the way (cap 0: not): grid (nblk, rows)
+__global__ __launch_bounds__(256) void rows_argmax_kernel(unsigned long long* tl, float* logits, int V, float cap, float* amax_val, int* amax_idx) {
     const TLStamp tls(tl);
     __shared__ float sv[4];
     __shared__ int si[4];
-    const float* l = logits + (size_t)blockIdx.y * V;
+    float* l = logits + (size_t)blockIdx.y * V;
     float bv = -INFINITY;
     int bi = 0x7FFFFFFF;
-    for (int i = blockIdx.x * 256 + threadIdx.x; i < V; i += gridDim.x * 256) if (l[i] > bv) { bv = l[i]; bi = i; }
+    for (int i = blockIdx.x * 256 + threadIdx.x; i < V; i += gridDim.x * 256) {
+        float v = l[i];
+        if (cap > 0.f) l[i] = v = soft_cap(v, cap);
+        if (v > bv) { bv = v; bi = i; }
+    }
 #pragma unroll
     for (int off = 32; off >= 1; off >>= 1) {
         const float ov = __shfl_xor(bv, off, 64);
@@ -1004,7 +1190,8 @@ __global__ __launch_bounds__(256) void rows_argmax_kernel(unsigned long long* tl
 }
 
 // -------------------------------------------------------------------------------------------- engine state
-static RouterCfg router_of(const pgk_stack_layer_t& L) { return RouterCfg{L.correction, L.experts, L.top, L.groups, L.keep, L.router_scale}; }
+static RouterCfg router_of(const pgk_stack_layer_t& L) { return RouterCfg{L.correction, L.experts, L.top, L.groups, L.keep, L.router_scale, L.table}; }
+static bool has_experts(const pgk_stack_layer_t& L) { return L.ff_pad && (L.ff == PGK_FF_MOE || L.ff == PGK_FF_TABLE); }
 static int router_rows(const pgk_stack_layer_t& L) { return L.ff_pad && L.ff == PGK_FF_MOE ? ceil_div(L.experts, 64) * 64 : 0; }
 struct Run { int layer, pass; };          // one pass of one layer; pass >= 0: the loop's pass `pass` starts with it
 
@@ -1021,6 +1208,13 @@ struct Stack {
     // one's: that one's pointer) or recurrent states [max_batch][heads][dim][vdim] in fp32
     std::vector<void*> cache;
     std::vector<int> ring, reach;          // R; keys the cache has to keep (the largest window of the layers that read it).  0: no ring
+    std::vector<std::vector<std::pair<int, int>>> readers;        // (window, chunked) of the layers that read it, sorted, each once
+    // positions before `pos` that a query at `pos` or later may reach through the cache of run `run`
+    int past(int run, int pos) const {
+        int m = 0;
+        for (const auto& r : readers[run]) { const int k = span_keys(pos, r.first, r.second) - 1; m = k > m ? k : m; }
+        return m;
+    }
     std::vector<void*> taps;               // rings of projected values [max_batch][taps][channels], or null
     std::vector<int32_t> len;              // per slot: positions held (host side; advanced with every step enqueued)
     // decode buffers (rows = max_batch)
@@ -1029,6 +1223,7 @@ struct Stack {
     float* slabs16 = nullptr;              // split-K slabs of a batch step's projections
     float *y32b = nullptr, *h32 = nullptr, *z32 = nullptr;                          // one row: input of a pass, normed row; rows: decay projections
     int32_t* ids = nullptr;
+    float *xs[2] = {nullptr, nullptr}, *xrows = nullptr, *ygate = nullptr;          // hyper-connected layers: streams of one row (two copies), of rows, rows' gates
     void *gate = nullptr, *cat16 = nullptr, *e16 = nullptr, *moe16 = nullptr;       // rows: gates, [x | embedding], experts' rows and workspace
     // fragment-major copies of the layer matrices for 2..128 rows (ops_pkgemm.hip), where its shapes allow; null entries: row-major kernels
     struct Packed { bf16 *in = nullptr, *o = nullptr, *gate_up = nullptr, *down = nullptr; };
@@ -1037,7 +1232,7 @@ struct Stack {
     size_t moe_ws(int n) const {           // workspace of the experts for n rows
         size_t m = 0;
         for (const auto& L : layers)
-            if (router_rows(L)) { const size_t z = moe_bytes(n, Wp, L.ff_pad, router_of(L), cfg.dtype); m = z > m ? z : m; }
+            if (has_experts(L)) { const size_t z = moe_bytes(n, Wp, L.ff_pad, router_of(L), cfg.dtype); m = z > m ? z : m; }
         return m;
     }
     // prompt buffers, grown on demand outside capture
@@ -1054,7 +1249,11 @@ static int conv_channels(const pgk_stack_layer_t& L) {
     return L.mixer == PGK_MIX_DELTA || L.mixer == PGK_MIX_SSD ? V + 2 * G : 0;
 }
 static int delta_a_off(const pgk_stack_layer_t& L) { return ceil_div(conv_channels(L) + L.heads, 64) * 64; }
-static int up_rows(const pgk_stack_layer_t& L) { return (L.ff == PGK_FF_SWIGLU ? 2 : 1) * L.ff_pad; }     // rows of the first feed-forward matrix
+// the feed-forward that runs for every token (of experts: the shared one): its width and matrices, rows of the first one
+static int dense_ff(const pgk_stack_layer_t& L) { return L.ff == PGK_FF_MOE ? 0 : L.ff == PGK_FF_TABLE ? L.shared_pad : L.ff_pad; }
+static const void* dense_up(const pgk_stack_layer_t& L) { return L.ff == PGK_FF_TABLE ? L.w_shared_up : L.w_gate_up; }
+static const void* dense_down(const pgk_stack_layer_t& L) { return L.ff == PGK_FF_TABLE ? L.w_shared_down : L.w_down; }
+static int up_rows(const pgk_stack_layer_t& L) { return (L.ff == PGK_FF_SWIGLU ? 2 : 1) * dense_ff(L); }
 
 static int pick_nsplit(const Engine* e, int B, const pgk_stack_layer_t& L, int R) {
     const int htiles = ceil_div(L.heads, 16);
@@ -1162,6 +1361,40 @@ static pgk_status attention_decode(Engine* e, int l, int B, const void* in, void
     return kv_attn_decode(a, DT, IO32, st, launches);
 }
 
+static HeadRowsArgs head_args(const Stack* s, int l, const void* in, int n) {
+    const auto& L = s->at(l);
+    HeadRowsArgs a{};
+    a.in = in; a.ld_in = L.n_in; a.bias = L.b_in; a.q_norm = L.q_norm; a.k_norm = L.k_norm; a.H = L.heads; a.G = L.kv_from >= 0 ? 0 : L.kv_heads; a.D = L.head_pad; a.dim = L.dim;
+    a.rot = L.rot; a.rot_freq = L.rot_freq; a.n = n; a.R = s->ring[kv_source(L, l)]; a.eps = s->cfg.norm_eps; a.ld_q = L.heads * L.head_pad; a.cache = s->cache[kv_source(L, l)];
+    return a;
+}
+static TalkArgs talk_args(const Stack* s, int l, int n, void* out) {
+    const auto& L = s->at(l);
+    TalkArgs a{};
+    a.ld_q = L.heads * L.head_pad; a.talk = L.talk; a.sink = L.sink; a.H = L.heads; a.G = L.kv_heads; a.D = L.head_pad; a.n = n; a.window = L.window; a.chunked = L.chunked;
+    a.scale = L.scale; a.nsplit = 1; a.out = out; a.ld_out = L.n_att;
+    return a;
+}
+
+// norms and rotation, new k and v -> ring -> attention over it (split) -> combine
+template <class T, class IT>
+static pgk_status talk_decode(Engine* e, int l, int B, const void* in, void* out, hipStream_t st, int* launches) {
+    Stack* s = stack_of(e);
+    const auto& L = s->at(l);
+    const int src = kv_source(L, l);
+    constexpr pgk_dtype DT = std::is_same<T, float>::value ? PGK_F32 : PGK_BF16;
+    constexpr bool IO32 = std::is_same<IT, float>::value;
+    HeadRowsArgs h = head_args(s, l, in, B);
+    h.positions = e->positions; h.q_out = s->qx;
+    if (pgk_status r = head_rows(h, DT, IO32, st)) return r;
+    TalkArgs a = talk_args(s, l, B, out);
+    a.q = s->qx; a.cache = s->cache[src]; a.positions = e->positions; a.R = s->ring[src];
+    a.nsplit = talk_splits(B, L.heads, L.kv_heads, L.window < a.R ? L.window : a.R, e->cu_count);
+    a.po = s->po; a.pml = s->pml;
+    *launches += 1;
+    return talk_attention(a, DT, IO32, st, launches);
+}
+
 static RecurArgs recur_args(const Stack* s, int l, const void* in, void* out, int n) {
     const auto& L = s->at(l);
     RecurArgs a{};
@@ -1205,6 +1438,7 @@ static pgk_status mix_decode(Engine* e, int l, int B, const void* in, void* out,
     switch (L.mixer) {
         case PGK_MIX_LATENT: return latent_decode<T, IT>(e, l, B, in, out, st, launches);
         case PGK_MIX_ATTENTION: return attention_decode<T, IT>(e, l, B, in, out, st, launches);
+        case PGK_MIX_TALK: return talk_decode<T, IT>(e, l, B, in, out, st, launches);
         case PGK_MIX_DELTA: {
             const int a_off = delta_a_off(L);
             if (pgk_status r = lowrank_rows(in, L.n_in, B, a_off, L.rank_a, L.w_a2, s->z32, L.heads * L.head_pad, a_off + L.rank_a, L.rank_g, L.w_g2, s->gate, L.heads * L.vhead_pad,
@@ -1291,6 +1525,76 @@ static pgk_status step_parallel(Engine* e, hipStream_t st, int* launches) {
     return PGK_OK;
 }
 
+// Hyper-connected layers, one sequence
+template <class T>
+static pgk_status step_hyper(Engine* e, hipStream_t st, int* launches) {
+    Stack* s = stack_of(e);
+    const auto& c = s->cfg;
+    const float *x = e->h, *pend = nullptr;   // the streams (at first all the embedded row), the numbers of the sublayer whose output waits in y32
+    int stream = 0, buf = 0;
+    auto input = [&](StackGemvArgs& a, const float* in, const float* gamma) {
+        a.K = s->Wp; a.W = c.width; a.x = x; a.x_stream = stream; a.S = c.streams; a.groups = c.norm_groups; a.in = in; a.gamma = gamma; a.eps = c.norm_eps;
+        if (pend) { a.y = s->y32; a.upd = pend; a.x_out = s->xs[buf]; }
+    };
+    auto settle = [&]() {
+        if (!pend) return;
+        x = s->xs[buf]; stream = s->Wp; buf ^= 1;
+        pend = nullptr;
+    };
+    for (int l = 0; l < c.num_layers; ++l) {
+        const auto& L = s->layers[l];
+        StackGemvArgs a{};
+        mark(KC_NORM_QKV);
+        input(a, L.hyper1, L.norm1);
+        a.w = L.w_in; a.N = L.n_in; a.out = s->in32;
+        if (pgk_status r = stack_gemv<T, SP_HYPER, SE_STORE>(a, st)) return r;
+        settle();
+        mark(KC_ATTN);
+        if (pgk_status r = mix_decode<T, float>(e, l, 1, s->in32, s->a32, st, launches)) return r;
+        mark(KC_OPROJ);
+        a = StackGemvArgs{};
+        a.w = L.w_o; a.N = s->Wp; a.K = L.n_att; a.x = s->a32; a.out = s->y32; a.bias = L.b_o;
+        if (pgk_status r = stack_gemv<T, SP_PLAIN, SE_STORE>(a, st)) return r;
+        pend = L.hyper1;
+        *launches += 2;
+        if (!L.ff_pad) continue;
+        mark(KC_GATEUP);
+        a = StackGemvArgs{};
+        input(a, L.hyper2, L.norm2);
+        a.out = s->act32;
+        if (L.ff == PGK_FF_TABLE) {
+            a.w = L.w_shared_up; a.w2 = L.w_gate_up; a.w3 = L.w_shared_gate; a.table = L.table; a.tok = e->tokens; a.fs = L.shared_pad; a.top = L.top; a.ff = L.ff_pad; a.ids = s->ids;
+            a.N = L.shared_pad + L.top * L.ff_pad + (L.shared_pad ? 1 : 0);
+            if (pgk_status r = stack_gemv<T, SP_HYPER, SE_TABLE>(a, st)) return r;
+        } else {
+            a.w = L.w_gate_up; a.N = L.ff_pad;
+            if (pgk_status r = stack_gemv<T, SP_HYPER, SE_STORE>(a, st)) return r;
+        }
+        settle();
+        mark(KC_DOWN);
+        if (L.ff == PGK_FF_TABLE) {
+            MoeOneArgs m{};
+            m.r = router_of(L); m.ff = L.ff_pad; m.w_down = L.w_down; m.act = s->act32 + L.shared_pad; m.ids = s->ids; m.w_o = L.w_shared_down; m.a = s->act32; m.n_att = L.shared_pad;
+            m.gate = L.shared_pad ? s->act32 + L.shared_pad + L.top * L.ff_pad : nullptr; m.y = s->y32; m.N = s->Wp;
+            if (pgk_status r = moe_out_one<T>(m, st)) return r;
+        } else {
+            a = StackGemvArgs{};
+            a.w = L.w_down; a.N = s->Wp; a.K = L.ff_pad; a.W = L.ff_dim; a.eps = c.norm_eps; a.act = L.act; a.x = s->act32; a.out = s->y32;
+            if (pgk_status r = stack_gemv<T, SP_POLY, SE_STORE>(a, st)) return r;
+        }
+        pend = L.hyper2;
+        *launches += 2;
+    }
+    mark(KC_LMHEAD);
+    StackGemvArgs a{};
+    input(a, nullptr, s->final_norm);
+    a.x_out = nullptr;
+    a.w = s->head; a.N = c.vocab_size; a.out = e->logits; a.cap = c.logit_cap; a.amax_val = e->amax_val; a.amax_idx = e->amax_idx;
+    if (pgk_status r = stack_gemv<T, SP_HYPER, SE_LOGITS>(a, st, e->lm_blocks)) return r;
+    *launches += 1;
+    return PGK_OK;
+}
+
 // ---- one sequence: fused steps, fp32 between kernels ----
 template <class T>
 static pgk_status step_one(Engine* e, hipStream_t st, int* launches) {
@@ -1344,9 +1648,9 @@ static pgk_status step_one(Engine* e, hipStream_t st, int* launches) {
     return PGK_OK;
 }
 
-// fp32 logits of `n` normalised rows (element type T, row stride Wp)
+// fp32 logits of `n` normalised rows (element type T, row stride Wp), before any soft cap
 template <class T>
-static pgk_status head_rows(Stack* s, const T* x, float* logits, int n, hipStream_t st) {
+static pgk_status logit_rows(Stack* s, const T* x, float* logits, int n, hipStream_t st) {
     const int V = s->cfg.vocab_size;
     if constexpr (std::is_same<T, float>::value) return pgk_gemm_nt(x, s->head, nullptr, logits, n, V, s->Wp, PGK_F32, st);
     for (int r = 0; r < n; r += 128) {
@@ -1359,6 +1663,7 @@ static pgk_status head_rows(Stack* s, const T* x, float* logits, int n, hipStrea
 struct RowBufs {
     float* h; void *x, *in, *a, *y, *gu, *act; float* slabs; void* q;
     void *cat, *e, *moe; const int32_t* tok;      // parallel layers: [x | embedding] rows, experts' rows, their workspace, the rows' tokens
+    float *xs, *ygate;                            // hyper-connected layers: streams [n][S][Wp], gates of the shared experts
 };
 
 // How a [N, K] projection of n bf16 rows runs: fragment-major copy (<= 128 rows), weight-streaming kernel (<= 128 rows) or tiled
@@ -1387,8 +1692,9 @@ size_t Stack::slab_elems(int n, bool f32) const {
         const auto& L = layers[l];
         const Packed P = packed.empty() ? Packed{} : packed[l];
         const size_t need[] = {(size_t)plan_proj(P.o, n, Wp, L.n_att, true).slabs * n * Wp,
-                               L.ff_pad && L.ff != PGK_FF_MOE ? (size_t)plan_proj(P.down, n, Wp, L.ff_pad, true).slabs * n * Wp : 0,
-                               P.in || n > 128 ? 0 : (size_t)plan_proj(nullptr, n, L.n_in, Wp, true).slabs * n * L.n_in};
+                               dense_ff(L) ? (size_t)plan_proj(P.down, n, Wp, dense_ff(L), true).slabs * n * Wp : 0,
+                               P.in || n > 128 ? 0 : (size_t)plan_proj(nullptr, n, L.n_in, Wp, true).slabs * n * L.n_in,
+                               L.ff != PGK_FF_POLY || P.gate_up || n > 128 ? 0 : (size_t)plan_proj(nullptr, n, L.ff_pad, Wp, true).slabs * n * L.ff_pad};
         for (size_t z : need) m = z > m ? z : m;
     }
     return m;
@@ -1420,33 +1726,41 @@ static pgk_status rows_out_proj(Stack* s, const RowBufs& b, const void* x, const
     return engine_gemm_nt_slabs((const bf16*)x, w, b.slabs, p.slabs, n, s->Wp, K, st);
 }
 
+// out = x W^T in the element type, K = Wp
 template <class T>
-static pgk_status rows_in_proj(Stack* s, const pgk_stack_layer_t& L, const bf16* packed, const RowBufs& b, int n, hipStream_t st) {
-    if constexpr (std::is_same<T, float>::value) return pgk_gemm_nt(b.x, L.w_in, nullptr, b.in, n, L.n_in, s->Wp, PGK_F32, st);
-    if (n <= 128 && packed) return pkgemm_nt((const bf16*)b.x, s->Wp, packed, b.in, L.n_in, PK_EPI_BF16, 1, n, L.n_in, s->Wp, nullptr, st);
-    const int slabs = n <= 128 ? plan_proj(nullptr, n, L.n_in, s->Wp, true).slabs : 0;
-    if (!slabs) return pgk_gemm_nt(b.x, L.w_in, nullptr, b.in, n, L.n_in, s->Wp, PGK_BF16, st);
-    if (pgk_status r = wsgemm_nt((const bf16*)b.x, s->Wp, L.w_in, nullptr, false, b.slabs, nullptr, 1, slabs, n, L.n_in, s->Wp, st)) return r;
-    const size_t n4 = (size_t)n * L.n_in / 4;
-    slab_rows_kernel<<<(unsigned)(n4 / 256 > 2048 ? 2048 : (n4 + 255) / 256), 256, 0, st>>>(b.slabs, slabs, (bf16*)b.in, n4);
+static pgk_status rows_proj(Stack* s, const RowBufs& b, const void* w, const bf16* packed, void* out, int n, int N, hipStream_t st) {
+    if constexpr (std::is_same<T, float>::value) return pgk_gemm_nt(b.x, w, nullptr, out, n, N, s->Wp, PGK_F32, st);
+    if (n <= 128 && packed) return pkgemm_nt((const bf16*)b.x, s->Wp, packed, out, N, PK_EPI_BF16, 1, n, N, s->Wp, nullptr, st);
+    const int slabs = n <= 128 ? plan_proj(nullptr, n, N, s->Wp, true).slabs : 0;
+    if (!slabs) return pgk_gemm_nt(b.x, w, nullptr, out, n, N, s->Wp, PGK_BF16, st);
+    if (pgk_status r = wsgemm_nt((const bf16*)b.x, s->Wp, w, nullptr, false, b.slabs, nullptr, 1, slabs, n, N, s->Wp, st)) return r;
+    const size_t n4 = (size_t)n * N / 4;
+    slab_rows_kernel<<<(unsigned)(n4 / 256 > 2048 ? 2048 : (n4 + 255) / 256), 256, 0, st>>>(b.slabs, slabs, (bf16*)out, n4);
     PGK_LAUNCH_CHECK();
     return PGK_OK;
 }
+template <class T>
+static pgk_status rows_in_proj(Stack* s, const pgk_stack_layer_t& L, const bf16* packed, const RowBufs& b, int n, hipStream_t st) {
+    return rows_proj<T>(s, b, L.w_in, packed, b.in, n, L.n_in, st);
+}
 
-// first feed-forward projection of n rows: act = silu(x W_g) * (x W_u), or xIELU(x W_u)
+// first feed-forward projection of n rows: act = silu(x W_g) * (x W_u), xIELU(x W_u), or (a shared expert) gelu(x W_u)
 template <class T>
 static pgk_status rows_gate_up(Stack* s, const pgk_stack_layer_t& L, const bf16* packed, const RowBufs& b, int n, hipStream_t st) {
     constexpr pgk_dtype DT = std::is_same<T, float>::value ? PGK_F32 : PGK_BF16;
-    if (L.ff == PGK_FF_XIELU) {
+    if (L.ff == PGK_FF_XIELU || L.ff == PGK_FF_TABLE) {
+        const bool gelu = L.ff == PGK_FF_TABLE;
+        const int ff = dense_ff(L);
+        const void* w = dense_up(L);
         if (DT == PGK_BF16 && n <= 128 && packed) {
             PkArgs g{};
             g.act_pos = L.act_pos; g.act_neg = L.act_neg;
-            return pkgemm_nt((const bf16*)b.x, s->Wp, packed, b.act, L.ff_pad, PK_EPI_XIELU, 1, n, L.ff_pad, s->Wp, &g, st);
+            return pkgemm_nt((const bf16*)b.x, s->Wp, packed, b.act, ff, gelu ? PK_EPI_GELU : PK_EPI_XIELU, 1, n, ff, s->Wp, &g, st);
         }
-        if (DT == PGK_BF16 && engine_gemm_xielu_ok(n, L.ff_pad, s->Wp))
-            return engine_gemm_xielu_nt((const bf16*)b.x, (const bf16*)L.w_gate_up, (bf16*)b.act, n, L.ff_pad, s->Wp, L.act_pos, L.act_neg, st);
-        if (pgk_status r = pgk_gemm_nt(b.x, L.w_gate_up, nullptr, b.act, n, L.ff_pad, s->Wp, DT, st)) return r;
-        return pgk_xielu(b.act, b.act, (size_t)n * L.ff_pad, L.act_pos, L.act_neg, DT, st);
+        if (DT == PGK_BF16 && engine_gemm_act_ok(n, ff, s->Wp))
+            return engine_gemm_act_nt((const bf16*)b.x, (const bf16*)w, (bf16*)b.act, n, ff, s->Wp, ActArgs{L.act_pos, L.act_neg, gelu}, st);
+        if (pgk_status r = pgk_gemm_nt(b.x, w, nullptr, b.act, n, ff, s->Wp, DT, st)) return r;
+        return gelu ? pgk_gelu_erf(b.act, b.act, (size_t)n * ff, DT, st) : pgk_xielu(b.act, b.act, (size_t)n * ff, L.act_pos, L.act_neg, DT, st);
     }
     if (DT == PGK_BF16 && n <= 128 && packed)
         return pkgemm_nt((const bf16*)b.x, s->Wp, packed, b.act, L.ff_pad, PK_EPI_SWIGLU, 1, n, 2 * L.ff_pad, s->Wp, nullptr, st);
@@ -1545,18 +1859,98 @@ static pgk_status rows_parallel(Stack* s, const RowBufs& b, int n, hipStream_t s
     return PGK_OK;
 }
 
-// All layers on n rows of b.h (embedded tokens); `last`: the launch of rows_norm that completes the stream and leaves normed rows in b.x
+// Hyper-connected layers: the sublayer output that is still to go into the streams (its numbers `upd`; null: none)
+struct PendingHyper { const float *upd = nullptr, *bias = nullptr; int slabs = 0, top = 0; bool y = true, gated = false, spread = false; };
+
+static HyperArgs hyper_args(const Stack* s, const RowBufs& b, int n, const PendingHyper& p, const float* in, const float* gamma, void* out) {
+    HyperArgs a{};
+    const int ld = s->Wp;
+    a.S = s->cfg.streams; a.W = s->cfg.width; a.ld = ld; a.groups = s->cfg.norm_groups; a.eps = s->cfg.norm_eps;
+    a.src = p.spread ? b.xs : b.h; a.src_row = p.spread ? (long long)a.S * ld : ld; a.src_stream = p.spread ? ld : 0;
+    a.in = in; a.gamma = gamma; a.out = out;
+    if (!p.upd) return a;
+    a.dst = b.xs; a.upd = p.upd; a.y = !p.y ? nullptr : p.slabs ? (const void*)b.slabs : b.y; a.ldy = ld; a.nslabs = p.slabs; a.slab_stride = (long long)n * ld;
+    a.y_bias = p.bias; a.y_gate = p.gated ? b.ygate : nullptr; a.e = p.top ? b.e : nullptr; a.e_top = p.top;
+    return a;
+}
+
 template <class T, class Mix>
-static pgk_status rows_model(Stack* s, const RowBufs& b, int n, hipStream_t st, Mix mix, RowsNormArgs* last) {
+static pgk_status rows_hyper(Stack* s, const RowBufs& b, int n, hipStream_t st, PendingHyper* pend, Mix mix) {
+    constexpr pgk_dtype DT = std::is_same<T, float>::value ? PGK_F32 : PGK_BF16;
+    *pend = PendingHyper{};
+    auto settle = [&]() {
+        const bool spread = pend->spread || pend->upd;
+        *pend = PendingHyper{};
+        pend->spread = spread;
+    };
+    for (int l = 0; l < s->cfg.num_layers; ++l) {
+        const auto& L = s->layers[l];
+        const Stack::Packed P = s->packed.empty() ? Stack::Packed{} : s->packed[l];
+        mark(KC_NORM_QKV);
+        if (pgk_status r = hyper_rows(hyper_args(s, b, n, *pend, L.hyper1, L.norm1, b.x), n, DT, st)) return r;
+        settle();
+        if (pgk_status r = rows_in_proj<T>(s, L, P.in, b, n, st)) return r;
+        mark(KC_ATTN);
+        if (pgk_status r = mix(l)) return r;
+        mark(KC_OPROJ);
+        if (pgk_status r = rows_out_proj<T>(s, b, b.a, L.w_o, P.o, n, L.n_att, &pend->slabs, st)) return r;
+        pend->upd = L.hyper1; pend->bias = L.b_o;
+        if (!L.ff_pad) continue;
+        mark(KC_GATEUP);
+        HyperArgs h = hyper_args(s, b, n, *pend, L.hyper2, L.norm2, b.x);
+        const bool shared = L.ff == PGK_FF_TABLE && L.shared_pad;
+        if (shared) { h.gate_w = L.w_shared_gate; h.gate_out = b.ygate; }
+        if (pgk_status r = hyper_rows(h, n, DT, st)) return r;
+        settle();
+        if (L.ff == PGK_FF_TABLE) {
+            MoeArgs m{b.x, n, s->Wp, L.ff_pad, router_of(L), nullptr, L.w_gate_up, L.w_down, b.e, b.moe, true, b.tok};
+            if (pgk_status r = moe_rows(m, DT, st)) return r;
+            pend->top = L.top;
+            if (shared) { if (pgk_status r = rows_gate_up<T>(s, L, P.gate_up, b, n, st)) return r; }
+        } else {
+            if (pgk_status r = rows_proj<T>(s, b, L.w_gate_up, P.gate_up, b.gu, n, L.ff_pad, st)) return r;
+            if (pgk_status r = poly_rows(b.gu, b.act, n, L.ff_dim, L.ff_pad, L.act, s->cfg.norm_eps, DT, st)) return r;
+        }
+        mark(KC_DOWN);
+        if (dense_ff(L)) { if (pgk_status r = rows_out_proj<T>(s, b, b.act, dense_down(L), P.down, n, dense_ff(L), &pend->slabs, st)) return r; }
+        pend->upd = L.hyper2; pend->gated = shared; pend->y = dense_ff(L) > 0;
+    }
+    return PGK_OK;
+}
+
+// The launch that completes the stream and leaves normed rows
+struct LastRows { bool hyper = false; RowsNormArgs norm; HyperArgs streams; };
+// ... for n rows (`rows`: which, null: the first n) into `out`; the stream itself stays as it is
+static pgk_status last_rows(const LastRows& l, void* out, const int32_t* rows, int n, pgk_dtype dt, hipStream_t st) {
+    if (l.hyper) {
+        HyperArgs a = l.streams;
+        a.out = out; a.rows = rows; a.dst = nullptr;
+        return hyper_rows(a, n, dt, st);
+    }
+    RowsNormArgs a = l.norm;
+    a.out = out; a.rows = rows; a.store_h = 0;
+    return rows_norm(a, n, dt, st);
+}
+
+// All layers on n rows of b.h (embedded tokens)
+template <class T, class Mix>
+static pgk_status rows_model(Stack* s, const RowBufs& b, int n, hipStream_t st, Mix mix, LastRows* last) {
+    if (s->cfg.block == PGK_BLOCK_HYPER) {
+        PendingHyper p;
+        if (pgk_status r = rows_hyper<T>(s, b, n, st, &p, mix)) return r;
+        last->hyper = true;
+        last->streams = hyper_args(s, b, n, p, nullptr, s->final_norm, b.x);
+        return PGK_OK;
+    }
     if (s->cfg.block == PGK_BLOCK_PARALLEL) {
         PendingAdd p;
         if (pgk_status r = rows_parallel<T>(s, b, n, st, &p, mix)) return r;
-        *last = add_args(s, b, n, p, s->final_norm, b.x);
+        last->norm = add_args(s, b, n, p, s->final_norm, b.x);
         return PGK_OK;
     }
     Pending p;
     if (pgk_status r = rows_layers<T>(s, b, n, st, &p, mix)) return r;
-    *last = norm_args(s, b, n, p, s->final_norm, b.x);
+    last->norm = norm_args(s, b, n, p, s->final_norm, b.x);
     return PGK_OK;
 }
 
@@ -1567,17 +1961,17 @@ static pgk_status step_rows(Engine* e, int B, hipStream_t st, int* launches) {
     Stack* s = stack_of(e);
     constexpr pgk_dtype DT = std::is_same<T, float>::value ? PGK_F32 : PGK_BF16;
     const auto& c = s->cfg;
-    const RowBufs b{e->h, s->x16, s->in16, s->a16, s->y16, s->gu16, s->act16, s->slabs16, nullptr, s->cat16, s->e16, s->moe16, e->tokens};
-    RowsNormArgs last;
+    const RowBufs b{e->h, s->x16, s->in16, s->a16, s->y16, s->gu16, s->act16, s->slabs16, nullptr, s->cat16, s->e16, s->moe16, e->tokens, s->xrows, s->ygate};
+    LastRows last;
     if (pgk_status r = rows_model<T>(s, b, B, st, [&](int l) { return mix_decode<T, T>(e, l, B, b.in, b.a, st, launches); }, &last)) return r;
     mark(KC_LMHEAD);
-    if (pgk_status r = rows_norm(last, B, DT, st)) return r;
-    if (pgk_status r = head_rows<T>(s, (const T*)b.x, e->logits, B, st)) return r;
-    PGK_CHECK_HIP(launch_k(rows_argmax_kernel, dim3(ROWS_ARGMAX_BLOCKS, B), dim3(256), 0, st, e->logits, c.vocab_size, e->amax_val, e->amax_idx));
+    if (pgk_status r = last_rows(last, b.x, nullptr, B, DT, st)) return r;
+    if (pgk_status r = logit_rows<T>(s, (const T*)b.x, e->logits, B, st)) return r;
+    PGK_CHECK_HIP(launch_k(rows_argmax_kernel, dim3(ROWS_ARGMAX_BLOCKS, B), dim3(256), 0, st, e->logits, c.vocab_size, c.logit_cap, e->amax_val, e->amax_idx));
     *launches += 3;
     for (const auto& r : s->runs) {                    // (one more where a projection's slabs or SwiGLU take a launch of their own)
         const auto& L = s->layers[r.layer];
-        *launches += 3 + (!L.ff_pad ? 0 : L.ff == PGK_FF_MOE ? 5 : 3) + (r.pass >= 0 ? 2 : 0);
+        *launches += 3 + (!L.ff_pad ? 0 : L.ff == PGK_FF_MOE ? 5 : L.ff == PGK_FF_TABLE ? (L.shared_pad ? 7 : 5) : L.ff == PGK_FF_POLY ? 4 : 3) + (r.pass >= 0 ? 2 : 0);
     }
     return PGK_OK;
 }
@@ -1588,7 +1982,7 @@ static pgk_status stack_step(Engine* e, int batch, hipStream_t st, int* launches
     int nblk = ROWS_ARGMAX_BLOCKS;
     if (batch == 1) {
         nblk = e->lm_blocks;
-        if (pgk_status r = s->cfg.block == PGK_BLOCK_PARALLEL ? step_parallel<T>(e, st, launches) : step_one<T>(e, st, launches)) return r;
+        if (pgk_status r = s->cfg.block == PGK_BLOCK_HYPER ? step_hyper<T>(e, st, launches) : s->cfg.block == PGK_BLOCK_PARALLEL ? step_parallel<T>(e, st, launches) : step_one<T>(e, st, launches)) return r;
     } else if (pgk_status r = step_rows<T>(e, batch, st, launches)) return r;
     mark(KC_ARGMAX);
     const int32_t* sampled = nullptr;
@@ -1628,7 +2022,7 @@ static pgk_status check_position(const Engine* e, int slot, int pos) {
         const auto& L = s->at(l);
         PGK_REQUIRE(!recurrent(L), "engine: slot %d has moved on to position %d; its recurrent state cannot go back to position %d", slot, len, pos);
         auto kept = [&](int back, int R) { return (pos - back > 0 ? pos - back : 0) + R >= len; };
-        PGK_REQUIRE(kept(L.window - 1, s->ring[kv_source(L, l)]) && (L.mixer != PGK_MIX_ATTENTION || !L.conv || kept(L.taps - 1, L.taps)),
+        PGK_REQUIRE(kept(span_keys(pos, L.window, L.chunked) - 1, s->ring[kv_source(L, l)]) && (L.mixer != PGK_MIX_ATTENTION || !L.conv || kept(L.taps - 1, L.taps)),
                     "engine: slot %d has moved on to position %d; the window of position %d is no longer in its ring", slot, len, pos);
     }
     return PGK_OK;
@@ -1655,18 +2049,18 @@ static pgk_status stack_prefill_t(Engine* e, int n_seqs, const int32_t* slots, c
         if (pgk_status r = check_position(e, slots[i], starts[i])) return r;
     int n = 0;
     for (int i = 0; i < n_seqs; ++i) n += lens[i];
-    // per layer with a ring: which cached rows a sequence's queries reach (its own and up to reach - 1 before them)
+    // per layer with a ring: which cached rows a sequence's queries reach (its own and those before them in a window or chunk)
     struct LayerRows { size_t past0 = 0; int n_past = 0, n_kv = 0; };
     const int n_runs = s->n_runs();
     std::vector<LayerRows> lr(n_runs);
     std::vector<RowPlace> place;                        // per layer: n_past gathered rows, then n new rows (equal layers share them)
     std::vector<int> share(n_runs, -1);
     int max_kv = 0;
-    auto past_of = [&](int l, int i) { return starts[i] < s->reach[l] - 1 ? starts[i] : s->reach[l] - 1; };
+    auto past_of = [&](int l, int i) { return s->past(l, starts[i]); };
     for (int l = 0; l < n_runs; ++l) {
         if (!s->reach[l]) continue;
         for (int k = 0; k < l && share[l] < 0; ++k)
-            if (share[k] < 0 && s->ring[k] == s->ring[l] && s->reach[k] == s->reach[l]) share[l] = k;
+            if (share[k] < 0 && s->ring[k] == s->ring[l] && s->readers[k] == s->readers[l]) share[l] = k;
         if (share[l] >= 0) { lr[l] = lr[share[l]]; continue; }
         lr[l].past0 = place.size();
         int kv = 0;
@@ -1727,7 +2121,8 @@ static pgk_status stack_prefill_t(Engine* e, int n_seqs, const int32_t* slots, c
     const size_t sizes[] = {(size_t)n * s->Wp * 4, (size_t)n * s->Wp * E, (size_t)n * s->max_in * E, (size_t)n * s->max_att * E, (size_t)n * s->Wp * E,
                             (size_t)n * 2 * s->max_ff * E, (size_t)n * s->max_ff * E, c_elems * E, kv_elems * E, (size_t)wrows * s->Wp * E, (size_t)wrows * c.vocab_size * 4,
                             s->slab_elems(n, DT == PGK_F32) * 4, (size_t)n * s->max_q * E, own_elems * E, chunk_ws, (size_t)n * s->max_conv * E, (size_t)n * s->max_z * 4,
-                            (size_t)n * s->max_gate * E, (size_t)n * s->max_low * E, c.loop_times ? (size_t)n * 2 * s->Wp * E : 0, (size_t)n * s->max_top * s->Wp * E, s->moe_ws(n)};
+                            (size_t)n * s->max_gate * E, (size_t)n * s->max_low * E, c.loop_times ? (size_t)n * 2 * s->Wp * E : 0, (size_t)n * s->max_top * s->Wp * E, s->moe_ws(n),
+                            c.block == PGK_BLOCK_HYPER ? (size_t)n * c.streams * s->Wp * 4 : 0, c.block == PGK_BLOCK_HYPER ? (size_t)n * 4 : 0};
     for (auto& t : chunkings) {
         t.o_list = chunk_tab;
         t.o_seq = t.o_list + up(t.list.size() * sizeof(RecurChunk));
@@ -1763,7 +2158,7 @@ static pgk_status stack_prefill_t(Engine* e, int n_seqs, const int32_t* slots, c
     void* conv_rows_buf = take(sizes[15]);
     float* z_rows = (float*)take(sizes[16]);
     void *gate_rows = take(sizes[17]), *low_rows = take(sizes[18]);
-    b.cat = take(sizes[19]); b.e = take(sizes[20]); b.moe = take(sizes[21]);
+    b.cat = take(sizes[19]); b.e = take(sizes[20]); b.moe = take(sizes[21]); b.xs = (float*)take(sizes[22]); b.ygate = (float*)take(sizes[23]);
     // one host image of the index tables, one copy
     std::vector<char> img(tab_need, 0);
     const size_t o_pos = up((size_t)n * 4), o_place = 2 * o_pos, o_want = o_place + up(place.size() * sizeof(RowPlace)),
@@ -1849,6 +2244,28 @@ static pgk_status stack_prefill_t(Engine* e, int n_seqs, const int32_t* slots, c
         }
         return PGK_OK;
     };
+    auto talk = [&](int l) -> pgk_status {
+        const auto& L = s->at(l);
+        const int src = kv_source(L, l), HD = L.heads * L.head_pad, GD = L.kv_heads * L.head_pad;
+        const LayerRows& w = lr[src];
+        T* rows = own[src] ? kv_own + (own[src] - 1) : kv;
+        if (src == l)
+            if (pgk_status r = kv_gather(d_place + w.past0, w.n_past, s->cache[l], rows, 2 * GD, GD, L.head_pad, s->ring[l], DT, st)) return r;
+        HeadRowsArgs h = head_args(s, l, b.in, n);
+        h.rows = d_rows; h.place = d_place + w.past0 + w.n_past; h.q_out = b.q; h.kv_rows = rows; h.ld_kv = 2 * GD;
+        if (pgk_status r = head_rows(h, DT, DT == PGK_F32, st)) return r;
+        int none = 0;
+        for (int i = 0, row = 0, kv0 = 0; i < n_seqs; ++i) {
+            const int past = past_of(src, i);
+            TalkArgs a = talk_args(s, l, lens[i], (T*)b.a + (size_t)row * HD);
+            a.q = (const T*)b.q + (size_t)row * HD; a.k = rows + (size_t)kv0 * 2 * GD; a.v = (const T*)a.k + GD; a.ld_kv = 2 * GD;
+            a.kv_len = past + lens[i]; a.pos0 = starts[i] - past;
+            if (pgk_status r = talk_attention(a, DT, DT == PGK_F32, st, &none)) return r;
+            row += lens[i];
+            kv0 += past + lens[i];
+        }
+        return PGK_OK;
+    };
     // taps over time and SiLU on the projected channels; then the rings take the last rows
     auto convolve = [&](int l) -> pgk_status {
         const auto& L = s->at(l);
@@ -1894,21 +2311,19 @@ static pgk_status stack_prefill_t(Engine* e, int n_seqs, const int32_t* slots, c
         switch (s->at(l).mixer) {
             case PGK_MIX_LATENT: return latent(l);
             case PGK_MIX_ATTENTION: return attention(l);
+            case PGK_MIX_TALK: return talk(l);
             case PGK_MIX_DELTA: return delta(l);
             default: return recurrence(l);
         }
     };
-    RowsNormArgs last;
+    LastRows last;
     if (pgk_status r = rows_model<T>(s, b, n, st, mix, &last)) return r;
     for (int i = 0; i < n_seqs; ++i) s->len[slots[i]] = starts[i] + lens[i];
     for (int w0 = 0; w0 < n_want; w0 += 128) {
         const int m = n_want - w0 < 128 ? n_want - w0 : 128;
-        RowsNormArgs a = last;
-        a.out = xw;
-        a.rows = d_want + w0;
-        a.store_h = 0;                        // a wanted row may be asked for twice
-        if (pgk_status r = rows_norm(a, m, DT, st)) return r;
-        if (pgk_status r = head_rows<T>(s, (const T*)xw, lg, m, st)) return r;
+        if (pgk_status r = last_rows(last, xw, d_want + w0, m, DT, st)) return r;      // (a wanted row may be asked for twice)
+        if (pgk_status r = logit_rows<T>(s, (const T*)xw, lg, m, st)) return r;
+        if (c.logit_cap > 0.f) { if (pgk_status r = soft_cap_rows(lg, (size_t)m * c.vocab_size, c.logit_cap, st)) return r; }
         PGK_CHECK_HIP(hipMemcpyAsync(h_logits + (size_t)w0 * c.vocab_size, lg, (size_t)m * c.vocab_size * 4, hipMemcpyDeviceToHost, st));
         PGK_CHECK_HIP(hipStreamSynchronize(st));
     }
@@ -1926,7 +2341,7 @@ static pgk_status stack_kv_ptr(Engine* e, int layer, void** k, void** v) {
     const Stack* s = stack_of(e);
     const auto& L = s->at(layer);
     *k = s->cache[layer];
-    *v = L.mixer == PGK_MIX_ATTENTION ? (char*)s->cache[layer] + (size_t)L.kv_heads * s->ring[kv_source(L, layer)] * L.head_pad * s->esize() : nullptr;
+    *v = L.mixer == PGK_MIX_ATTENTION || L.mixer == PGK_MIX_TALK ? (char*)s->cache[layer] + (size_t)L.kv_heads * s->ring[kv_source(L, layer)] * L.head_pad * s->esize() : nullptr;
     return PGK_OK;
 }
 
@@ -1956,19 +2371,26 @@ pgk_status pgk_engine_create_stack(const pgk_stack_config_t* cfg, const void* em
     const int Wp = ceil_div(c.width, 64) * 64;
     for (int l = 0; l < c.num_layers; ++l) {
         const auto& L = layers[l];
-        PGK_REQUIRE(L.mixer >= PGK_MIX_LATENT && L.mixer <= PGK_MIX_SSD && L.ff >= PGK_FF_SWIGLU && L.ff <= PGK_FF_MOE, "pgk_engine_create_stack: layer %d: mixer %d, feed-forward %d", l, L.mixer, L.ff);
+        PGK_REQUIRE(L.mixer >= PGK_MIX_LATENT && L.mixer <= PGK_MIX_TALK && L.ff >= PGK_FF_SWIGLU && L.ff <= PGK_FF_TABLE, "pgk_engine_create_stack: layer %d: mixer %d, feed-forward %d", l, L.mixer, L.ff);
         PGK_REQUIRE(L.heads >= 1 && L.dim >= 1 && L.vdim >= 1, "pgk_engine_create_stack: layer %d: bad mixer sizes", l);
         PGK_REQUIRE(L.ff_pad % 64 == 0 && L.ff_pad >= 0, "pgk_engine_create_stack: layer %d: feed-forward pad %d", l, L.ff_pad);
         PGK_REQUIRE(L.n_in % 64 == 0 && L.n_att % 64 == 0, "pgk_engine_create_stack: layer %d: %d in-projection rows, %d out-projection columns", l, L.n_in, L.n_att);
         PGK_REQUIRE(L.w_in && L.w_o && (!L.ff_pad || (L.w_gate_up && L.w_down)), "pgk_engine_create_stack: layer %d: missing weights", l);
-        if (c.block == PGK_BLOCK_PARALLEL) {
+        PGK_REQUIRE((c.block == PGK_BLOCK_HYPER) == (L.mixer == PGK_MIX_TALK), "pgk_engine_create_stack: layer %d: mixer %d in block kind %d", l, L.mixer, c.block);
+        if (c.block == PGK_BLOCK_HYPER) {
+            PGK_REQUIRE(L.norm1 && L.hyper1 && (!L.ff_pad || (L.norm2 && L.hyper2)), "pgk_engine_create_stack: layer %d: missing norms or stream weights", l);
+            PGK_REQUIRE(!L.ff_pad || (L.ff == PGK_FF_POLY ? L.act && L.ff_dim >= 1 && L.ff_dim <= L.ff_pad
+                                                         : L.ff == PGK_FF_TABLE && L.table && L.experts >= 1 && L.experts <= MOE_MAX_EXPERTS && L.top >= 1 && L.top <= L.experts && L.top <= MOE_MAX_TOP &&
+                                                               L.shared_pad >= 0 && L.shared_pad % 64 == 0 && (!L.shared_pad || (L.w_shared_up && L.w_shared_down && L.w_shared_gate))),
+                        "pgk_engine_create_stack: layer %d: feed-forward %d of %d, %d experts, top %d, shared %d", l, L.ff, L.ff_pad, L.experts, L.top, L.shared_pad);
+        } else if (c.block == PGK_BLOCK_PARALLEL) {
             PGK_REQUIRE(L.norm1 && (!L.ff_pad || (L.ff == PGK_FF_MOE && L.correction)), "pgk_engine_create_stack: layer %d: a parallel layer has one norm and experts or no feed-forward", l);
             if (L.ff_pad)
                 PGK_REQUIRE(L.experts >= 1 && L.experts <= MOE_MAX_EXPERTS && L.top >= 1 && L.top <= L.experts && L.top <= MOE_MAX_TOP && L.groups >= 0 &&
                                 (L.groups == 0 || (L.experts % L.groups == 0 && L.keep >= 1 && L.keep <= L.groups && L.keep * (L.experts / L.groups) >= L.top)),
                             "pgk_engine_create_stack: layer %d: %d experts, top %d, %d of %d groups", l, L.experts, L.top, L.keep, L.groups);
         } else {
-            PGK_REQUIRE(L.norm1b && (!L.ff_pad || (L.ff != PGK_FF_MOE && L.norm2b)), "pgk_engine_create_stack: layer %d: missing norms", l);
+            PGK_REQUIRE(L.norm1b && (!L.ff_pad || (L.ff <= PGK_FF_XIELU && L.norm2b)), "pgk_engine_create_stack: layer %d: missing norms", l);
         }
         const int HD = L.heads * L.head_pad;
         if (L.mixer == PGK_MIX_DELTA || L.mixer == PGK_MIX_SSD) {
@@ -1992,6 +2414,12 @@ pgk_status pgk_engine_create_stack(const pgk_stack_config_t* cfg, const void* em
             PGK_REQUIRE(L.rank >= 1 && L.rank_pad % 64 == 0 && L.rank_pad >= L.rank + L.rot && L.rank_pad <= 2048 && L.rot >= 0 && L.rot % 2 == 0 && L.rot <= L.dim && (!L.rot || L.rot_freq), "pgk_engine_create_stack: layer %d: latent size %d padded to %d (at most 2048)", l, L.rank, L.rank_pad);
             PGK_REQUIRE(L.n_in >= HD + L.rank_pad + (L.gated ? L.heads : 0) && L.kv_heads == L.heads && L.kv_from < 0, "pgk_engine_create_stack: layer %d: in-projection rows %d", l, L.n_in);
             PGK_REQUIRE(L.norm1 && L.c_norm && L.w_ukv, "pgk_engine_create_stack: layer %d: missing weights", l);
+        } else if (L.mixer == PGK_MIX_TALK) {
+            PGK_REQUIRE(L.kv_heads >= 1 && L.heads % L.kv_heads == 0 && L.head_pad <= 1024 && L.rot >= 0 && L.rot % 2 == 0 && L.rot <= L.dim && (!L.rot || L.rot_freq) && L.q_norm && (L.kv_from >= 0 || L.k_norm) &&
+                            L.n_in >= HD + (L.kv_from < 0 ? 2 * L.kv_heads * L.head_pad : 0),
+                        "pgk_engine_create_stack: layer %d: %d / %d heads of %d, %d turned, in-projection rows %d", l, L.heads, L.kv_heads, L.head_pad, L.rot, L.n_in);
+            PGK_REQUIRE(L.kv_from < 0 || (L.kv_from < l && layers[L.kv_from].mixer == PGK_MIX_TALK && layers[L.kv_from].kv_from < 0 && layers[L.kv_from].kv_heads == L.kv_heads && layers[L.kv_from].head_pad == L.head_pad),
+                        "pgk_engine_create_stack: layer %d cannot take the keys and values of layer %d", l, L.kv_from);
         } else {
             PGK_REQUIRE(L.kv_heads >= 1 && L.heads % L.kv_heads == 0 && L.head_pad <= 1024 && L.taps >= 1, "pgk_engine_create_stack: layer %d: %d / %d heads of %d, %d taps", l, L.heads, L.kv_heads, L.head_pad, L.taps);
             PGK_REQUIRE(L.n_in >= 2 * HD + (L.kv_from < 0 ? 2 * L.kv_heads * L.head_pad : 0), "pgk_engine_create_stack: layer %d: in-projection rows %d", l, L.n_in);
@@ -2001,6 +2429,9 @@ pgk_status pgk_engine_create_stack(const pgk_stack_config_t* cfg, const void* em
             }
         }
     }
+    PGK_REQUIRE(c.block != PGK_BLOCK_HYPER || (c.streams >= 1 && c.streams <= HYPER_MAX_STREAMS && c.norm_groups >= 1 && c.norm_groups <= NORM_MAX_GROUPS && c.width % c.norm_groups == 0),
+                "pgk_engine_create_stack: %d streams, %d norm groups of %d", c.streams, c.norm_groups, c.width);
+    PGK_REQUIRE(c.block == PGK_BLOCK_HYPER || (c.norm_groups <= 1 && !(c.logit_cap > 0.f)), "pgk_engine_create_stack: norms in groups and capped logits belong to hyper-connected layers");
     PGK_REQUIRE(c.loop_times >= 0 && (!c.loop_times || (c.block == PGK_BLOCK_PARALLEL && c.loop_start >= 0 && c.loop_start < c.loop_stop && c.loop_stop <= c.num_layers && c.loop_in && c.loop_step)),
                 "pgk_engine_create_stack: layers %d .. %d of %d, %d times", c.loop_start, c.loop_stop - 1, c.num_layers, c.loop_times);
     Engine* e = new Engine();
@@ -2043,8 +2474,16 @@ pgk_status pgk_engine_create_stack(const pgk_stack_config_t* cfg, const void* em
     int max_router = 0, max_act = 0;
     auto most = [](auto& m, auto v) { if (v > m) m = v; };
     s->reach.assign(s->n_runs(), 0);
-    for (int l = 0; l < s->n_runs(); ++l)
-        if (!recurrent(s->at(l))) most(s->reach[kv_source(s->at(l), l)], s->at(l).window);
+    s->readers.resize(s->n_runs());
+    for (int l = 0; l < s->n_runs(); ++l) {
+        const auto& L = s->at(l);
+        if (recurrent(L)) continue;
+        auto& rd = s->readers[kv_source(L, l)];
+        const std::pair<int, int> span{L.window, L.chunked ? 1 : 0};
+        most(s->reach[kv_source(L, l)], L.window);
+        const auto at = std::lower_bound(rd.begin(), rd.end(), span);
+        if (at == rd.end() || *at != span) rd.insert(at, span);
+    }
     for (int l = 0; l < s->n_runs(); ++l) {
         const auto& L = s->at(l);
         const int R = s->reach[l] < c.max_seq_len ? s->reach[l] : c.max_seq_len, HD = L.heads * L.head_pad;
@@ -2073,11 +2512,12 @@ pgk_status pgk_engine_create_stack(const pgk_stack_config_t* cfg, const void* em
         s->taps.push_back(t);
         most(s->max_in, L.n_in);
         most(s->max_att, L.n_att);
-        if (router_rows(L)) { most(s->max_top, L.top); most(max_router, router_rows(L)); most(max_act, L.top * L.ff_pad); }
-        else { most(s->max_ff, L.ff_pad); most(max_act, L.ff_pad); }
+        if (has_experts(L)) { most(s->max_top, L.top); most(max_router, router_rows(L)); most(max_act, L.top * L.ff_pad + L.shared_pad + 64); }
+        else most(max_act, L.ff_pad);
+        most(s->max_ff, dense_ff(L));
         for (int m = 1; m <= c.max_batch && !recurrent(L); ++m) {
             const int src = kv_source(L, l), keys = L.window < s->ring[src] ? L.window : s->ring[src];
-            const size_t ns = (size_t)(L.mixer == PGK_MIX_LATENT ? pick_nsplit(e, m, L, R) : kv_attn_splits(m, L.heads, L.kv_heads, keys, e->cu_count)) * m * L.heads;
+            const size_t ns = (size_t)(L.mixer == PGK_MIX_LATENT ? pick_nsplit(e, m, L, R) : L.mixer == PGK_MIX_TALK ? talk_splits(m, L.heads, L.kv_heads, keys, e->cu_count) : kv_attn_splits(m, L.heads, L.kv_heads, keys, e->cu_count)) * m * L.heads;
             most(part, ns * (L.mixer == PGK_MIX_LATENT ? L.rank_pad : L.head_pad));
             most(ml, ns * 2);
         }
@@ -2097,7 +2537,12 @@ pgk_status pgk_engine_create_stack(const pgk_stack_config_t* cfg, const void* em
     A((void**)&s->a32, (size_t)s->max_att * 4, &e->ws_bytes, true);     // padding columns of a head are never written: zero
     A((void**)&s->y32, (size_t)Wp * 4, &e->ws_bytes, true);
     A((void**)&s->act32, (size_t)(max_act ? max_act : 64) * 4, &e->ws_bytes);
-    if (c.block == PGK_BLOCK_PARALLEL) {
+    if (c.block == PGK_BLOCK_HYPER) {
+        for (auto& x : s->xs) A((void**)&x, (size_t)c.streams * Wp * 4, &e->ws_bytes, true);
+        A((void**)&s->xrows, B * c.streams * Wp * 4, &e->ws_bytes, true);
+        A((void**)&s->ygate, B * 4, &e->ws_bytes, true);
+    }
+    if (c.block == PGK_BLOCK_PARALLEL || c.block == PGK_BLOCK_HYPER) {
         A((void**)&s->y32b, (size_t)Wp * 4, &e->ws_bytes, true);
         A((void**)&s->h32, (size_t)Wp * 4, &e->ws_bytes, true);
         A((void**)&s->ids, MOE_MAX_TOP * 4, &e->ws_bytes, true);
@@ -2134,9 +2579,9 @@ pgk_status pgk_engine_create_stack(const pgk_stack_config_t* cfg, const void* em
                 auto& P = s->packed[l];
                 if (pkgemm_shape_ok(L.n_in, Wp, false)) fn(&P.in, L.w_in, L.n_in, Wp);
                 if (pkgemm_shape_ok(Wp, L.n_att, true)) fn(&P.o, L.w_o, Wp, L.n_att);
-                if (!L.ff_pad || L.ff == PGK_FF_MOE) continue;
-                if (pkgemm_shape_ok(up_rows(L), Wp, false)) fn(&P.gate_up, L.w_gate_up, up_rows(L), Wp);
-                if (pkgemm_shape_ok(Wp, L.ff_pad, true)) fn(&P.down, L.w_down, Wp, L.ff_pad);
+                if (!dense_ff(L)) continue;
+                if (pkgemm_shape_ok(up_rows(L), Wp, false)) fn(&P.gate_up, dense_up(L), up_rows(L), Wp);
+                if (pkgemm_shape_ok(Wp, dense_ff(L), true)) fn(&P.down, dense_down(L), Wp, dense_ff(L));
             }
         };
         s->packed.resize(c.num_layers);

@@ -14,7 +14,7 @@ struct QkvHeadArgs {
     bf16 *kcache, *vcache;                // this layer's, this sequence's: [Hkv][max_seq][128]
     int hq, hkv, max_seq, start_pos;
 };
-struct XieluArgs { float pos, neg; };     // pgk_device.hip.h: xielu's factors
+struct ActArgs { float pos, neg; bool gelu; };     // pgk_device.hip.h: xielu's factors, or gelu_erf
 
 // The 16 lanes that hold one (token row, head slot) of the bf16-rounded QKV projection, 8 dims each (sub = lane's chunk):
 // the arithmetic of qknorm_rope_kvwrite_kernel, operation for operation, then the store.  All 16 lanes must be active.

@@ -15,10 +15,12 @@ struct SeqSpan { int32_t row0, len, start, slot; };
 // A prompt row's place: position, cache slot, row in the prompt's K/V (or latent) scratch, and whether the ring keeps it
 struct RowPlace { int32_t pos, slot, kv, store; };
 
-// Keys of a query at position `pos` with window `window` in a ring of R rows (position p in row p % R): n keys, oldest first, key t in
-// ring row lo + t (minus R past the end) at distance n - 1 - t.
-__device__ __forceinline__ void ring_window(int pos, int window, int R, int& n, int& lo) {
-    n = min(pos + 1, min(window, R));
+// How many keys a query at position `pos` sees: a sliding window, or its own chunk of `window` positions, itself included
+__host__ __device__ __forceinline__ int span_keys(int pos, int window, int chunked) { return chunked ? pos % window + 1 : pos < window ? pos + 1 : window; }
+// The keys of that query in a ring of R rows (position p in row p % R): n keys, oldest first, key t in ring row lo + t (minus R past the
+// end) at distance n - 1 - t.
+__device__ __forceinline__ void ring_window(int pos, int window, int R, int& n, int& lo, int chunked = 0) {
+    n = min(span_keys(pos, window, chunked), R);
     lo = (pos - n + 1) % R;
 }
 __device__ __forceinline__ int ring_row(int lo, int t, int R) { const int r = lo + t; return r >= R ? r - R : r; }
@@ -68,10 +70,51 @@ struct KvAttnArgs {
     float *po, *pml;                      // records [B][H][nsplit][D] and [B][H][nsplit][2]
     const void* gate; int ld_gate;        // rows like `out`: the result is multiplied by its sigmoid; null: none
     void* out; int ld_out;                // head h at h * D
+    const float* sink;                    // [H]: exp(sink) stands in the denominator (kv_merge only; null: none)
+    int chunked;
 };
+// combine the split records po, pml -> out (gate, sink)
+pgk_status kv_merge(const KvAttnArgs& a, bool io32, hipStream_t st);
 bool kv_attn_q32(int D, pgk_dtype dt);
 int kv_attn_splits(int B, int H, int G, int keys, int cus);
 pgk_status kv_attn_decode(const KvAttnArgs& a, pgk_dtype dt, bool io32, hipStream_t st, int* launches);
+
+// ---- projection rows -> q, k, v heads: bias, RMS norm per head, rotation of the first columns by the position (ops_talk.hip) ----
+// Heads q (H) | k (G) | v (G) of width D, `dim` of them true; G 0: only q.  Column i < rot / 2 turns with column i + rot / 2.  Rows, k and v go
+// where conv_rows puts them; everything but `in` is in the element type.
+struct HeadRowsArgs {
+    const void* in; int ld_in;
+    const float* bias;                    // [(H + 2 G) * D] or null
+    const float *q_norm, *k_norm;         // [D] or null
+    int H, G, D, dim, rot, n, R;
+    const float* rot_freq;                // [rot / 2]
+    float eps;
+    const int32_t* positions;
+    const RowSrc* rows; const RowPlace* place;
+    void* q_out; int ld_q;
+    void* kv_rows; int ld_kv;
+    void* cache;
+};
+pgk_status head_rows(const HeadRowsArgs& a, pgk_dtype dt, bool in32, hipStream_t st);
+
+// ---- attention whose heads mix their scores, with a sink (ops_talk.hip) ----
+// raw_h = scale q_h . k,  score_h = sum_g talk[h][g] raw_g,  weights exp(score_h) / (sum over the keys + exp(sink_h))
+struct TalkArgs {
+    const void* q; int ld_q;              // rows, head h at h * D
+    const float *talk, *sink;             // [H][H] or null (no mixing), [H] or null (no sink)
+    int H, G, D, n, window, chunked;      // n: rows
+    float scale;
+    // decode (cache given): row b is the next token of slot b at positions[b], over the ring [slots][k, v][G][R][D] in nsplit splits
+    const void* cache; const int32_t* positions;
+    int R, nsplit;
+    float *po, *pml;
+    // prompt: kv_len rows of k and v (head g at g * D), row t is position pos0 + t; the queries are the last n of them
+    const void *k, *v; int ld_kv, kv_len, pos0;
+    void* out; int ld_out;                // head h at h * D
+    int Dv, ld_v;                         // value heads of another width, rows ld_v apart, heads of `out` too (0: D, ld_kv); prompts only
+};
+int talk_splits(int B, int H, int G, int keys, int cus);
+pgk_status talk_attention(const TalkArgs& a, pgk_dtype dt, bool io32, hipStream_t st, int* launches);   // io32: `out` is fp32 (else dt)
 
 // ---- taps over time and SiLU ----
 // y_t = silu(bias + sum_j w_j u_(t - taps + 1 + j)) per channel, zero before a sequence's start.  Ring [slot][taps][channels] of u: position p

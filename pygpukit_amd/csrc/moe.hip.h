@@ -1,5 +1,5 @@
-// Mixture of experts (ops_moe.hip; the one-row kernels of a decode step are in engine_stack.hip): a router picks `top` of E experts per
-// row, every expert is a SwiGLU feed-forward.
+// Mixture of experts (ops_moe.hip; the one-row kernels of a decode step are in engine_stack.hip): a router, or a table of token ids, picks
+// `top` of E experts per row; every expert is a SwiGLU or a gelu feed-forward.
 #pragma once
 
 #include "engine_common.hip.h"
@@ -10,7 +10,8 @@ namespace pgk {
 // Choice: s = sigmoid(z), c = s + correction.  With groups > 0 only experts of the `keep` groups of neighbours with the largest sum of
 // their two largest c can be chosen.  The `top` experts with the largest c (lowest index on ties), weights s / (sum of the chosen s + 1e-20)
 // * scale.
-struct RouterCfg { const float* correction; int E, top, groups, keep; float scale; };
+// With a table [tokens][top] there is no router: its row of the token names the experts, each with weight 1 / top.
+struct RouterCfg { const float* correction; int E, top, groups, keep; float scale; const int32_t* table; };
 
 constexpr int MOE_MAX_EXPERTS = 1024, MOE_MAX_TOP = 64;
 struct RouteScratch { float *s, *c, *g, *w; };                     // LDS: [E], [E], [2 groups], [top]
@@ -64,19 +65,24 @@ struct MoeTile { int32_t expert, row0, rows, pad; };
 // between two experts' matrices.  A's row of sorted row p is place / div (div > 0) or p.
 struct GroupArgs { const MoeTile* tiles; const int32_t* n_tiles; const int32_t* order; const float* wts; long long w_stride; int div; };
 
+// What a product over rows sorted by expert leaves: SwiGLU rows of fused gate | up matrices, gelu rows, or weighted rows at their places
+enum MoeProduct { MOE_SWIGLU = 0, MOE_GELU = 1, MOE_DOWN = 2 };
+
 struct MoeArgs {
     const void* x;                        // [n][W], element type; W a multiple of 64
     int n, W, ff;                         // ff: a multiple of 64
     RouterCfg router;
-    const void *w_router, *w_up, *w_down; // [E up to a multiple of 64][W], [E][2 ff][W] (gate rows, up rows), [E][W][ff]
+    const void *w_router, *w_up, *w_down; // [E up to a multiple of 64][W] (with a table: unused), [E][2 ff][W] (gate rows, up rows; gelu: [E][ff][W]), [E][W][ff]
     void* out;                            // [n][top][W], element type: weighted expert outputs
     void* ws;                             // moe_bytes(...)
+    bool gelu = false;
+    const int32_t* tok = nullptr;         // with a table: the rows' tokens
 };
 size_t moe_bytes(int n, int W, int ff, const RouterCfg& r, pgk_dtype dt);
 pgk_status moe_rows(const MoeArgs& a, pgk_dtype dt, hipStream_t st);
 
 // ops_gemm256.hip: 128 x 128 tiles over rows sorted by expert (tile list of runs of up to 128 rows): SwiGLU rows act [p][N] from fused
-// gate | up matrices [2 N, K], or (down) weighted rows C [place][N]
-pgk_status gemm128s_grouped(const bf16* A, const bf16* W, bf16* C, bool down, const GroupArgs& g, int max_tiles, int rows, int N, int K, hipStream_t st);
+// gate | up matrices [2 N, K], gelu rows from [N, K], or (down) weighted rows C [place][N]
+pgk_status gemm128s_grouped(const bf16* A, const bf16* W, bf16* C, MoeProduct what, const GroupArgs& g, int max_tiles, int rows, int N, int K, hipStream_t st);
 
 }  // namespace pgk

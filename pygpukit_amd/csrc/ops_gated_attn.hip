@@ -529,11 +529,16 @@ __global__ __launch_bounds__(128) void kv_merge_kernel(unsigned long long* tl, K
     const size_t rec = ((size_t)b * a.H + h) * a.nsplit;
     const float mm = lane < a.nsplit ? a.pml[(rec + lane) * 2] : -INFINITY, ll = lane < a.nsplit ? a.pml[(rec + lane) * 2 + 1] : 0.f;
     const float top = wave_max(ll > 0.f ? mm : -INFINITY), f = ll > 0.f ? exp2f(mm - top) : 0.f;
-    const float den = wave_sum(f * ll);
-    if (threadIdx.x < 64) sw[lane] = f / den;
+    float den = wave_sum(f * ll), more = 1.0f;
+    if (a.sink) {                                                  // (no value: it only takes its share)
+        const float sk = a.sink[h] * GA_LOG2E, t2 = fmaxf(top, sk);
+        more = exp2f(top - t2);
+        den = fmaf(den, more, exp2f(sk - t2));
+    }
+    if (threadIdx.x < 64) sw[lane] = f * more / den;
     __syncthreads();
     int n, lo;
-    ring_window(max(a.positions[b], 0), a.window, a.R, n, lo);
+    ring_window(max(a.positions[b], 0), a.window, a.R, n, lo, a.chunked);
     const int per = split_rows(n, a.nsplit), used = (n + per - 1) / per;
     for (int c = 2 * threadIdx.x; c < a.D; c += 256) {
         float x = 0.f, y = 0.f;
@@ -549,6 +554,13 @@ __global__ __launch_bounds__(128) void kv_merge_kernel(unsigned long long* tl, K
         out[1] = from_f<IT>(y * gate_at<IT>(a, b, oc + 1));
     }
     tls.end();
+}
+
+pgk_status kv_merge(const KvAttnArgs& a, bool io32, hipStream_t st) {
+    PGK_REQUIRE(a.D % 64 == 0 && a.nsplit >= 1 && a.nsplit <= 64, "kv_merge: head width %d, %d splits", a.D, a.nsplit);
+    if (io32) PGK_CHECK_HIP(launch_k(&kv_merge_kernel<float>, dim3(a.H, a.B), dim3(128), 0, st, a));
+    else PGK_CHECK_HIP(launch_k(&kv_merge_kernel<bf16>, dim3(a.H, a.B), dim3(128), 0, st, a));
+    return PGK_OK;
 }
 
 bool kv_attn_q32(int D, pgk_dtype dt) { return dt == PGK_F32 || D > 256; }

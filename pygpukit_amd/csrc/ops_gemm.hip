@@ -23,11 +23,11 @@ pgk_status wsgemm_nt(const bf16* a, int lda, const void* w, const bf16* wscale, 
 // (packed: W is the fragment-major bf16 copy of ops_pkgemm.hip instead of the row-major weight - the staged kernels' DMA
 // instruction moves 16 rows x 32 k, which is one block of that layout)
 pgk_status gemm256_bf16_nt(const bf16* A, const bf16* W, const bf16* bias, void* C, bool accum_f32, int M, int N, int K,
-                           hipStream_t st, bool packed = false, const XieluArgs* act = nullptr);
+                           hipStream_t st, bool packed = false, const ActArgs* act = nullptr);
 pgk_status gemm256_bf16_swiglu_nt(const bf16* A, const bf16* W, bf16* act, int M, int I, int K, hipStream_t st, bool packed = false);
 bool gemm128s_ok(int M, int N, int K);    // ops_gemm256.hip: 128 x 128 tiles on the staged LDS-DMA pipeline (bf16, M > 128, K % 64 == 0, N % 8 == 0)
 pgk_status gemm128s_bf16_nt(const bf16* A, const bf16* W, const bf16* bias, void* C, int mode, int splits, int M, int N, int K, hipStream_t st,
-                            const QkvHeadArgs* heads = nullptr, bool packed = false, const XieluArgs* act = nullptr);
+                            const QkvHeadArgs* heads = nullptr, bool packed = false, const ActArgs* act = nullptr);
 // the 256 x 256 structure needs enough tiles to fill the chip and whole 128-byte K rows
 // PGK_GEMM256 = 0 / 1 forces the choice (read per call: tests flip it to drive small shapes through both kernels); shared
 // with the fp8 x fp8 GEMM (ops_fp8_gemm.hip)
@@ -439,11 +439,10 @@ pgk_status engine_gemm_nt(const bf16* A, const void* W, const bf16* wscale, bool
     return dispatch_mfma<bf16, B_NT, 0>(A, W, nullptr, nullptr, C, M, N, K, st);
 }
 
-// internal (engine prefill): act[M][N] = bf16(xIELU(A . W^T)) in the product's epilogue, for the shapes the staged kernels take
-bool engine_gemm_xielu_ok(int M, int N, int K) { return M > 128 && (use_gemm256(M, N, K) || gemm128s_ok(M, N, K)); }
-pgk_status engine_gemm_xielu_nt(const bf16* A, const bf16* W, bf16* act, int M, int N, int K, float pos, float neg, hipStream_t st) {
-    PGK_REQUIRE(engine_gemm_xielu_ok(M, N, K), "engine_gemm_xielu: M=%d N=%d K=%d outside the fused kernels' shapes", M, N, K);
-    const XieluArgs xa{pos, neg};
+// internal (engine prefill): act[M][N] = bf16(act(A . W^T)), xIELU or gelu, in the product's epilogue, for the shapes the staged kernels take
+bool engine_gemm_act_ok(int M, int N, int K) { return M > 128 && (use_gemm256(M, N, K) || gemm128s_ok(M, N, K)); }
+pgk_status engine_gemm_act_nt(const bf16* A, const bf16* W, bf16* act, int M, int N, int K, const ActArgs& xa, hipStream_t st) {
+    PGK_REQUIRE(engine_gemm_act_ok(M, N, K), "engine_gemm_act: M=%d N=%d K=%d outside the fused kernels' shapes", M, N, K);
     if (use_gemm256(M, N, K)) return gemm256_bf16_nt(A, W, nullptr, act, false, M, N, K, st, false, &xa);
     return gemm128s_bf16_nt(A, W, nullptr, act, 0, 1, M, N, K, st, nullptr, false, &xa);
 }

@@ -318,10 +318,10 @@ __global__ __launch_bounds__(G2_THREADS) void gemm256_bf16_kernel(const bf16* A,
 // half-empty last round: Llama's QKV (4096 x 6144) is 384 tiles = 1.5 rounds of the 256 CUs, 512 tiles of 256 x 192 are two
 // full rounds of three quarters the work.  The W stage then has 192 rows = 12 DMA instructions: waves 0-3 move two (rows 0-127),
 // waves 4-7 one (rows 128-191), so the "two younger stages in flight" count is vmcnt(8) for the former, vmcnt(6) for the latter.
-template <int EPI, int TN = 4>   // EPI 0: bf16 C store (+bias); 1: fp32 C +=; 2: SwiGLU (W = fused gate / up rows, N = I act columns, C = bf16 act [M][I]); 3: xIELU, bf16 store
+template <int EPI, int TN = 4>   // EPI 0: bf16 C store (+bias); 1: fp32 C +=; 2: SwiGLU (W = fused gate / up rows, N = I act columns, C = bf16 act [M][I]); 3: xIELU, 4: gelu, bf16 store
 __global__ __launch_bounds__(G2_THREADS) void gemm256s_bf16_kernel(const bf16* A, const bf16* W, const bf16* bias, void* Cv,
-                                                                    int M, int N, int K, int ntm, int ntn, int packed, XieluArgs xa = XieluArgs{}) {
-    static_assert(TN == 4 || (TN == 3 && (EPI == 0 || EPI == 2 || EPI == 3)), "192-column tiles: bf16 store and SwiGLU only");
+                                                                    int M, int N, int K, int ntm, int ntn, int packed, ActArgs xa = ActArgs{}) {
+    static_assert(TN == 4 || (TN == 3 && (EPI == 0 || EPI >= 2)), "192-column tiles: bf16 store and SwiGLU only");
     extern __shared__ __attribute__((aligned(16))) char g2_smem[];   // 4 stages x (A 16 KiB | W 16 KiB)
     constexpr int HALF = 256 * 64, BN = TN * 64, WN = TN * 16;
     const int tid = threadIdx.x, lane = tid & 63, wid = tid >> 6;
@@ -451,6 +451,7 @@ __global__ __launch_bounds__(G2_THREADS) void gemm256s_bf16_kernel(const bf16* A
                 if (row >= M) continue;
                 if constexpr (EPI == 0) reinterpret_cast<bf16*>(Cv)[(size_t)row * N + col] = from_f<bf16>(acc[i][j][r] + b);
                 else if constexpr (EPI == 3) reinterpret_cast<bf16*>(Cv)[(size_t)row * N + col] = from_f<bf16>(xielu<false>(acc[i][j][r], xa.pos, xa.neg));
+                else if constexpr (EPI == 4) reinterpret_cast<bf16*>(Cv)[(size_t)row * N + col] = from_f<bf16>(gelu_erf(acc[i][j][r]));
                 else reinterpret_cast<float*>(Cv)[(size_t)row * N + col] += acc[i][j][r];
             }
     }
@@ -469,11 +470,11 @@ __global__ __launch_bounds__(G2_THREADS) void gemm256s_bf16_kernel(const bf16* A
 // read-modify-write of the residual stream, all loads issued before the first store).
 constexpr int G1_THREADS = 256, G1_HALF = 128 * 64;
 // EPI 0: bf16 C store (+bias); 1: fp32 C +=; 2: fp32 split-K slab; 3: QKV heads (QkvHeadArgs: tile column = head slot);
-// 4: SwiGLU (W = fused gate / up rows, N = I act columns, C = bf16 act [M][I]; tile tn = act columns [64 tn, +64)); 5: xIELU, bf16 store
-// GRP: rows sorted by expert (GroupArgs), every tile with its expert's weight; EPI 4, or 6: bf16 rows times their weight, each at its place
+// 4: SwiGLU (W = fused gate / up rows, N = I act columns, C = bf16 act [M][I]; tile tn = act columns [64 tn, +64)); 5: xIELU, 7: gelu, bf16 store
+// GRP: rows sorted by expert (GroupArgs), every tile with its expert's weight; EPI 4, 7, or 6: bf16 rows times their weight, each at its place
 template <int EPI, bool GRP>
 __device__ __forceinline__ void gemm128s_body(const bf16* A, const bf16* W, const bf16* bias, void* Cv,
-                                              int M, int N, int K, int ntm, int ntn, int kps, const QkvHeadArgs& hd, int packed, const XieluArgs& xa, const GroupArgs& ga) {
+                                              int M, int N, int K, int ntm, int ntn, int kps, const QkvHeadArgs& hd, int packed, const ActArgs& xa, const GroupArgs& ga) {
     extern __shared__ __attribute__((aligned(16))) char g2_smem[];   // 4 stages x (A 8 KiB | W 8 KiB)
     const int tid = threadIdx.x, lane = tid & 63, wid = tid >> 6;
     const int wr = wid >> 1, wc = wid & 1, q = lane >> 4, l15 = lane & 15;
@@ -634,7 +635,7 @@ __device__ __forceinline__ void gemm128s_body(const bf16* A, const bf16* W, cons
             o.from_float(f);
             o.store(reinterpret_cast<bf16*>(Cv) + (size_t)place * N + gcol);
         }
-    } else if constexpr (EPI == 0 || EPI == 5) {
+    } else if constexpr (EPI == 0 || EPI == 5 || EPI == 7) {
         // 8 columns per lane: two float4 -> 16 bytes of bf16
 #pragma unroll
         for (int it = 0; it < 8; ++it) {
@@ -651,6 +652,10 @@ __device__ __forceinline__ void gemm128s_body(const bf16* A, const bf16* W, cons
             if constexpr (EPI == 5) {
 #pragma unroll
                 for (int e = 0; e < 8; ++e) f[e] = xielu<false>(f[e], xa.pos, xa.neg);
+            }
+            if constexpr (EPI == 7) {
+#pragma unroll
+                for (int e = 0; e < 8; ++e) f[e] = gelu_erf(f[e]);
             }
             Vec<bf16> o;
             o.from_float(f);
@@ -680,12 +685,12 @@ __device__ __forceinline__ void gemm128s_body(const bf16* A, const bf16* W, cons
 }
 template <int EPI>
 __global__ __launch_bounds__(G1_THREADS, 2) void gemm128s_bf16_kernel(const bf16* A, const bf16* W, const bf16* bias, void* Cv,
-                                                                       int M, int N, int K, int ntm, int ntn, int kps, QkvHeadArgs hd, int packed, XieluArgs xa = XieluArgs{}) {
+                                                                       int M, int N, int K, int ntm, int ntn, int kps, QkvHeadArgs hd, int packed, ActArgs xa = ActArgs{}) {
     gemm128s_body<EPI, false>(A, W, bias, Cv, M, N, K, ntm, ntn, kps, hd, packed, xa, GroupArgs{});
 }
 template <int EPI>
 __global__ __launch_bounds__(G1_THREADS, 2) void gemm128s_grouped_kernel(const bf16* A, const bf16* W, bf16* C, int N, int K, int ntn, GroupArgs ga) {
-    gemm128s_body<EPI, true>(A, W, nullptr, C, 0, N, K, 0, ntn, K, QkvHeadArgs{}, 0, XieluArgs{}, ga);
+    gemm128s_body<EPI, true>(A, W, nullptr, C, 0, N, K, 0, ntn, K, QkvHeadArgs{}, 0, ActArgs{}, ga);
 }
 
 // ---- fp8 x fp8 with 128-wide block scales on the same structure --------------------------------------------
@@ -978,7 +983,7 @@ pgk_status gemm256_fp8_swiglu_nt(const uint8_t* a, const float* sa, const uint8_
 
 // bf16 NT on the 256^2 structure; caller guarantees K % 64 == 0 and 16-byte aligned rows
 pgk_status gemm256_bf16_nt(const bf16* A, const bf16* W, const bf16* bias, void* C, bool accum_f32, int M, int N, int K,
-                           hipStream_t st, bool packed, const XieluArgs* act) {
+                           hipStream_t st, bool packed, const ActArgs* act) {
     PGK_REQUIRE(K % 64 == 0 && K >= 64, "gemm256: K=%d must be a multiple of 64", K);
     PGK_REQUIRE(!packed || N % 16 == 0, "gemm256: the fragment-major weight copy has whole 16-row tiles (N=%d)", N);
     constexpr size_t LDS = 4 * (size_t)G2_TILE;
@@ -1008,18 +1013,20 @@ pgk_status gemm256_bf16_nt(const bf16* A, const bf16* W, const bf16* bias, void*
                 attr_n = true;
             }
             if (act) {
-                static bool attr_x = false;
-                if (!attr_x) PGK_CHECK_HIP(hipFuncSetAttribute(reinterpret_cast<const void*>(&gemm256s_bf16_kernel<3, 3>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)LDS));
-                attr_x = true;
-                gemm256s_bf16_kernel<3, 3><<<ntm * ntn3, G2_THREADS, LDS, st>>>(A, W, nullptr, C, M, N, K, ntm, ntn3, packed ? 1 : 0, *act);
-            } else gemm256s_bf16_kernel<0, 3><<<ntm * ntn3, G2_THREADS, LDS, st>>>(A, W, bias, C, M, N, K, ntm, ntn3, packed ? 1 : 0, XieluArgs{});
+                auto kfn = act->gelu ? &gemm256s_bf16_kernel<4, 3> : &gemm256s_bf16_kernel<3, 3>;
+                static bool attr_x[2] = {false, false};
+                if (!attr_x[act->gelu]) PGK_CHECK_HIP(hipFuncSetAttribute(reinterpret_cast<const void*>(kfn), hipFuncAttributeMaxDynamicSharedMemorySize, (int)LDS));
+                attr_x[act->gelu] = true;
+                kfn<<<ntm * ntn3, G2_THREADS, LDS, st>>>(A, W, nullptr, C, M, N, K, ntm, ntn3, packed ? 1 : 0, *act);
+            } else gemm256s_bf16_kernel<0, 3><<<ntm * ntn3, G2_THREADS, LDS, st>>>(A, W, bias, C, M, N, K, ntm, ntn3, packed ? 1 : 0, ActArgs{});
         } else if (act) {
-            static bool attr_x = false;
-            if (!attr_x) PGK_CHECK_HIP(hipFuncSetAttribute(reinterpret_cast<const void*>(&gemm256s_bf16_kernel<3>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)LDS));
-            attr_x = true;
-            gemm256s_bf16_kernel<3><<<ntm * ntn, G2_THREADS, LDS, st>>>(A, W, nullptr, C, M, N, K, ntm, ntn, packed ? 1 : 0, *act);
-        } else if (accum_f32) gemm256s_bf16_kernel<1><<<ntm * ntn, G2_THREADS, LDS, st>>>(A, W, nullptr, C, M, N, K, ntm, ntn, packed ? 1 : 0, XieluArgs{});
-        else gemm256s_bf16_kernel<0><<<ntm * ntn, G2_THREADS, LDS, st>>>(A, W, bias, C, M, N, K, ntm, ntn, packed ? 1 : 0, XieluArgs{});
+            auto kfn = act->gelu ? &gemm256s_bf16_kernel<4> : &gemm256s_bf16_kernel<3>;
+            static bool attr_x[2] = {false, false};
+            if (!attr_x[act->gelu]) PGK_CHECK_HIP(hipFuncSetAttribute(reinterpret_cast<const void*>(kfn), hipFuncAttributeMaxDynamicSharedMemorySize, (int)LDS));
+            attr_x[act->gelu] = true;
+            kfn<<<ntm * ntn, G2_THREADS, LDS, st>>>(A, W, nullptr, C, M, N, K, ntm, ntn, packed ? 1 : 0, *act);
+        } else if (accum_f32) gemm256s_bf16_kernel<1><<<ntm * ntn, G2_THREADS, LDS, st>>>(A, W, nullptr, C, M, N, K, ntm, ntn, packed ? 1 : 0, ActArgs{});
+        else gemm256s_bf16_kernel<0><<<ntm * ntn, G2_THREADS, LDS, st>>>(A, W, bias, C, M, N, K, ntm, ntn, packed ? 1 : 0, ActArgs{});
         PGK_CHECK_HIP(hipGetLastError());
         return PGK_OK;
     }
@@ -1043,18 +1050,18 @@ pgk_status gemm256_bf16_swiglu_nt(const bf16* A, const bf16* W, bf16* act, int M
     // 96 act columns per tile (192-column B tiles) when that fills the rounds of the chip better: Qwen3-0.6B at S = 2048 is
     // 8 x 24 = 192 tiles of 128 (three quarters of the CUs, one round) or 8 x 32 = 256 tiles of 96 (all of them)
     if (I % 96 == 0 && 0.75 * ceil_div(ntm * (I / 96), 256) < (double)ceil_div(ntm * ntn, 256) - 0.01) {
-        gemm256s_bf16_kernel<2, 3><<<ntm * (I / 96), G2_THREADS, LDS, st>>>(A, W, nullptr, act, M, I, K, ntm, I / 96, packed ? 1 : 0, XieluArgs{});
+        gemm256s_bf16_kernel<2, 3><<<ntm * (I / 96), G2_THREADS, LDS, st>>>(A, W, nullptr, act, M, I, K, ntm, I / 96, packed ? 1 : 0, ActArgs{});
     } else {
-        gemm256s_bf16_kernel<2><<<ntm * ntn, G2_THREADS, LDS, st>>>(A, W, nullptr, act, M, I, K, ntm, ntn, packed ? 1 : 0, XieluArgs{});
+        gemm256s_bf16_kernel<2><<<ntm * ntn, G2_THREADS, LDS, st>>>(A, W, nullptr, act, M, I, K, ntm, ntn, packed ? 1 : 0, ActArgs{});
     }
     PGK_CHECK_HIP(hipGetLastError());
     return PGK_OK;
 }
 
-// 128 x 128 tiles; mode 0: bf16 C (+bias, or with `act` its xIELU), 1: fp32 C +=, 2: fp32 slabs [splits][M][N] (K split into `splits` runs of whole 64-k steps)
+// 128 x 128 tiles; mode 0: bf16 C (+bias, or with `act` its activation), 1: fp32 C +=, 2: fp32 slabs [splits][M][N] (K split into `splits` runs of whole 64-k steps)
 bool gemm128s_ok(int M, int N, int K) { return M > 128 && K % 64 == 0 && N % 8 == 0 && N >= 8; }
 pgk_status gemm128s_bf16_nt(const bf16* A, const bf16* W, const bf16* bias, void* C, int mode, int splits, int M, int N, int K, hipStream_t st,
-                            const QkvHeadArgs* heads, bool packed, const XieluArgs* act) {
+                            const QkvHeadArgs* heads, bool packed, const ActArgs* act) {
     PGK_REQUIRE(!packed || N % 16 == 0, "gemm128s: the fragment-major weight copy has whole 16-row tiles (N=%d)", N);
     const int pk = packed ? 1 : 0;
     PGK_REQUIRE(gemm128s_ok(M, N, K) && mode >= 0 && mode <= 4 && splits >= 1 && (splits == 1 || mode == 2), "gemm128s: M=%d N=%d K=%d mode=%d splits=%d", M, N, K, mode, splits);
@@ -1070,33 +1077,37 @@ pgk_status gemm128s_bf16_nt(const bf16* A, const bf16* W, const bf16* bias, void
         PGK_CHECK_HIP(hipFuncSetAttribute(reinterpret_cast<const void*>(&gemm128s_bf16_kernel<3>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)LDS));
         PGK_CHECK_HIP(hipFuncSetAttribute(reinterpret_cast<const void*>(&gemm128s_bf16_kernel<4>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)LDS));
         PGK_CHECK_HIP(hipFuncSetAttribute(reinterpret_cast<const void*>(&gemm128s_bf16_kernel<5>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)LDS));
+        PGK_CHECK_HIP(hipFuncSetAttribute(reinterpret_cast<const void*>(&gemm128s_bf16_kernel<7>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)LDS));
         attr_done = true;
     }
     const int ntm = ceil_div(M, 128), ntn = mode == 4 ? N / 64 : ceil_div(N, 128);      // SwiGLU: N = I act columns, 64 per tile
     const int kps = ceil_div(ceil_div(K, splits), 64) * 64;
     const dim3 grid(ntm * ntn, ceil_div(K, kps));
     PGK_REQUIRE((int)grid.y == splits, "gemm128s: K=%d does not split into %d runs of whole 64-k steps", K, splits);
-    if (mode == 0 && act) gemm128s_bf16_kernel<5><<<grid, G1_THREADS, LDS, st>>>(A, W, nullptr, C, M, N, K, ntm, ntn, kps, hd, pk, *act);
-    else if (mode == 0) gemm128s_bf16_kernel<0><<<grid, G1_THREADS, LDS, st>>>(A, W, bias, C, M, N, K, ntm, ntn, kps, hd, pk, XieluArgs{});
-    else if (mode == 1) gemm128s_bf16_kernel<1><<<grid, G1_THREADS, LDS, st>>>(A, W, nullptr, C, M, N, K, ntm, ntn, kps, hd, pk, XieluArgs{});
-    else if (mode == 2) gemm128s_bf16_kernel<2><<<grid, G1_THREADS, LDS, st>>>(A, W, nullptr, C, M, N, K, ntm, ntn, kps, hd, pk, XieluArgs{});
-    else if (mode == 3) gemm128s_bf16_kernel<3><<<grid, G1_THREADS, LDS, st>>>(A, W, nullptr, C, M, N, K, ntm, ntn, kps, hd, pk, XieluArgs{});
-    else gemm128s_bf16_kernel<4><<<grid, G1_THREADS, LDS, st>>>(A, W, nullptr, C, M, N, K, ntm, ntn, kps, hd, pk, XieluArgs{});
+    if (mode == 0 && act && act->gelu) gemm128s_bf16_kernel<7><<<grid, G1_THREADS, LDS, st>>>(A, W, nullptr, C, M, N, K, ntm, ntn, kps, hd, pk, *act);
+    else if (mode == 0 && act) gemm128s_bf16_kernel<5><<<grid, G1_THREADS, LDS, st>>>(A, W, nullptr, C, M, N, K, ntm, ntn, kps, hd, pk, *act);
+    else if (mode == 0) gemm128s_bf16_kernel<0><<<grid, G1_THREADS, LDS, st>>>(A, W, bias, C, M, N, K, ntm, ntn, kps, hd, pk, ActArgs{});
+    else if (mode == 1) gemm128s_bf16_kernel<1><<<grid, G1_THREADS, LDS, st>>>(A, W, nullptr, C, M, N, K, ntm, ntn, kps, hd, pk, ActArgs{});
+    else if (mode == 2) gemm128s_bf16_kernel<2><<<grid, G1_THREADS, LDS, st>>>(A, W, nullptr, C, M, N, K, ntm, ntn, kps, hd, pk, ActArgs{});
+    else if (mode == 3) gemm128s_bf16_kernel<3><<<grid, G1_THREADS, LDS, st>>>(A, W, nullptr, C, M, N, K, ntm, ntn, kps, hd, pk, ActArgs{});
+    else gemm128s_bf16_kernel<4><<<grid, G1_THREADS, LDS, st>>>(A, W, nullptr, C, M, N, K, ntm, ntn, kps, hd, pk, ActArgs{});
     PGK_CHECK_HIP(hipGetLastError());
     return PGK_OK;
 }
 
-pgk_status gemm128s_grouped(const bf16* A, const bf16* W, bf16* C, bool down, const GroupArgs& g, int max_tiles, int rows, int N, int K, hipStream_t st) {
+pgk_status gemm128s_grouped(const bf16* A, const bf16* W, bf16* C, MoeProduct what, const GroupArgs& g, int max_tiles, int rows, int N, int K, hipStream_t st) {
     PGK_REQUIRE(K % 64 == 0 && N % 64 == 0 && max_tiles >= 1 && g.tiles && g.n_tiles && g.order && g.wts, "gemm128s_grouped: N=%d K=%d", N, K);
     constexpr size_t LDS = 8 * (size_t)G1_HALF;
     static bool attr_done = false;
     if (!attr_done) {
         PGK_CHECK_HIP(hipFuncSetAttribute(reinterpret_cast<const void*>(&gemm128s_grouped_kernel<4>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)LDS));
         PGK_CHECK_HIP(hipFuncSetAttribute(reinterpret_cast<const void*>(&gemm128s_grouped_kernel<6>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)LDS));
+        PGK_CHECK_HIP(hipFuncSetAttribute(reinterpret_cast<const void*>(&gemm128s_grouped_kernel<7>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)LDS));
         attr_done = true;
     }
-    const int ntn = down ? ceil_div(N, 128) : N / 64;
-    if (down) gemm128s_grouped_kernel<6><<<max_tiles * ntn, G1_THREADS, LDS, st>>>(A, W, C, N, K, ntn, g);
+    const int ntn = what == MOE_SWIGLU ? N / 64 : ceil_div(N, 128);
+    if (what == MOE_GELU) gemm128s_grouped_kernel<7><<<max_tiles * ntn, G1_THREADS, LDS, st>>>(A, W, C, N, K, ntn, g);
+    else if (what == MOE_DOWN) gemm128s_grouped_kernel<6><<<max_tiles * ntn, G1_THREADS, LDS, st>>>(A, W, C, N, K, ntn, g);
     else gemm128s_grouped_kernel<4><<<max_tiles * ntn, G1_THREADS, LDS, st>>>(A, W, C, N, K, ntn, g);
     PGK_CHECK_HIP(hipGetLastError());
     return PGK_OK;

@@ -1,4 +1,4 @@
-// Mixture of experts over rows (moe.hip.h): router logits (fp32) -> choice -> rows sorted by expert -> grouped SwiGLU -> grouped down
+// Mixture of experts over rows (moe.hip.h): router logits (fp32) -> choice, or a table of tokens -> rows sorted by expert -> grouped SwiGLU or gelu -> grouped down
 // projection, each result weighted and stored at [row][k].  The rows' sum over k is left to the norm that follows (rows_norm).
 // Nothing about the distribution is known on the host: grids are sized for the worst case, a tile list says what a workgroup does.
 
@@ -13,9 +13,9 @@ pgk_status wsgemm_nt(const bf16* a, int lda, const void* w, const bf16* wscale, 
 int wsgemm_pick_splits(int N, int K, bool allow_split);
 bool gemm128s_ok(int M, int N, int K);
 struct QkvHeadArgs;
-struct XieluArgs;
+struct ActArgs;
 pgk_status gemm128s_bf16_nt(const bf16* A, const bf16* W, const bf16* bias, void* C, int mode, int splits, int M, int N, int K, hipStream_t st,
-                            const QkvHeadArgs* heads, bool packed, const XieluArgs* act);
+                            const QkvHeadArgs* heads, bool packed, const ActArgs* act);
 
 // -------------------------------------------------------------------------------------------- choice and sorting
 // A wave per row; logits are the sum of `slabs` fp32 slabs
@@ -30,6 +30,13 @@ __global__ __launch_bounds__(256) void moe_route_kernel(RouterCfg r, const float
     };
     auto sync = []() { __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront"); __builtin_amdgcn_wave_barrier(); __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront"); };
     route_row<64>(r, rt_smem + wid * route_floats(r), threadIdx.x & 63, logit, ids + (size_t)row * r.top, wts + (size_t)row * r.top, sync);
+}
+
+__global__ __launch_bounds__(256) void moe_table_kernel(const int32_t* table, const int32_t* tok, int total, int top, int32_t* ids, float* wts) {
+    const int i = blockIdx.x * 256 + threadIdx.x;
+    if (i >= total) return;
+    ids[i] = table[(size_t)tok[i / top] * top + i % top];
+    wts[i] = 1.0f / top;
 }
 
 // Workgroup e writes expert e's places in ascending order and its runs of `tm` rows to the tile list
@@ -82,19 +89,19 @@ __global__ __launch_bounds__(1024) void moe_sort_kernel(const int32_t* ids, int 
 }
 
 // -------------------------------------------------------------------------------------------- few rows per expert, bf16
-// The weight-streaming product of ops_wsgemm.hip on a tile list: a wave has 16 weight rows (UP: 16 gate rows and the matching up rows),
+// The weight-streaming product of ops_wsgemm.hip on a tile list: a wave has 16 weight rows (SwiGLU: 16 gate rows and the matching up rows),
 // which are read once from memory as the MFMA operand; the tile's rows (up to 16 MT) pass through LDS in pieces of 256 k.
 typedef __bf16 bf16x8_me __attribute__((ext_vector_type(8)));
 typedef float f32x4_me __attribute__((ext_vector_type(4)));
 constexpr int ME_KT = 256;
 __device__ __forceinline__ int me_off(int r, int c) { return r * (ME_KT * 2) + (((c & ~15) | ((c ^ r) & 15)) << 4); }
 
-template <int MT, bool UP>
+template <int MT, MoeProduct P>
 __global__ __launch_bounds__(256) void moe_stream_kernel(const bf16* A, const bf16* W, bf16* C, int N, int K, GroupArgs ga) {
     __shared__ __attribute__((aligned(16))) char a_lds[MT * 16 * ME_KT * 2];
     if ((int)blockIdx.y >= *ga.n_tiles) return;
     const MoeTile t = ga.tiles[blockIdx.y];
-    constexpr int NB = UP ? 2 : 1;
+    constexpr int NB = P == MOE_SWIGLU ? 2 : 1;
     const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6, l15 = lane & 15, q4 = lane >> 4, n0 = (blockIdx.x * 4 + wid) * 16, kl = 8 * q4;
     const bf16* wr[NB];
 #pragma unroll
@@ -159,9 +166,11 @@ __global__ __launch_bounds__(256) void moe_stream_kernel(const bf16* A, const bf
         for (int r = 0; r < 4; ++r) {
             const int row = 16 * m + 4 * q4 + r;
             if (row >= t.rows) continue;
-            if constexpr (UP) {
+            if constexpr (P == MOE_SWIGLU) {
                 const float g = acc[0][m][r];
                 C[(size_t)(t.row0 + row) * N + n] = from_f<bf16>(g / (1.0f + __expf(-g)) * acc[NB - 1][m][r]);
+            } else if constexpr (P == MOE_GELU) {
+                C[(size_t)(t.row0 + row) * N + n] = from_f<bf16>(gelu_erf(acc[0][m][r]));
             } else {
                 const int place = ga.order[t.row0 + row];
                 C[(size_t)place * N + n] = from_f<bf16>(acc[0][m][r] * ga.wts[place]);
@@ -170,9 +179,9 @@ __global__ __launch_bounds__(256) void moe_stream_kernel(const bf16* A, const bf
 }
 
 // -------------------------------------------------------------------------------------------- fp32
-template <bool UP>
+template <MoeProduct P>
 __global__ __launch_bounds__(256) void moe_f32_kernel(const float* A, const float* W, float* C, int N, int K, GroupArgs ga) {
-    constexpr int NB = UP ? 2 : 1, TM = 32, TN = 64, TK = 16;
+    constexpr int NB = P == MOE_SWIGLU ? 2 : 1, TM = 32, TN = 64, TK = 16;
     __shared__ float As[TK][TM + 1], Bs[NB][TK][TN + 1];
     if ((int)blockIdx.y >= *ga.n_tiles) return;
     const MoeTile t = ga.tiles[blockIdx.y];
@@ -204,9 +213,11 @@ __global__ __launch_bounds__(256) void moe_f32_kernel(const float* A, const floa
         for (int j = 0; j < 4; ++j) {
             const int row = 2 * ty + i, n = n0 + 4 * tx + j;
             if (row >= t.rows || n >= N) continue;
-            if constexpr (UP) {
+            if constexpr (P == MOE_SWIGLU) {
                 const float g = acc[0][i][j];
                 C[(size_t)(t.row0 + row) * N + n] = g / (1.0f + expf(-g)) * acc[NB - 1][i][j];
+            } else if constexpr (P == MOE_GELU) {
+                C[(size_t)(t.row0 + row) * N + n] = gelu_erf(acc[0][i][j]);
             } else {
                 const int place = ga.order[t.row0 + row];
                 C[(size_t)place * N + n] = acc[0][i][j] * ga.wts[place];
@@ -263,42 +274,48 @@ pgk_status moe_rows(const MoeArgs& a, pgk_dtype dt, hipStream_t st) {
     float *logits = (float*)(ws + p.logits), *wts = (float*)(ws + p.wts);
     int32_t *ids = (int32_t*)(ws + p.ids), *order = (int32_t*)(ws + p.order), *count = (int32_t*)(ws + p.count);
     MoeTile* tiles = (MoeTile*)(ws + p.tiles);
-    if (dt == PGK_F32) { if (pgk_status q = pgk_gemm_nt(a.x, a.w_router, nullptr, logits, a.n, p.Ep, a.W, PGK_F32, st)) return q; }
-    else if (a.n <= 128) { if (pgk_status q = wsgemm_nt((const bf16*)a.x, a.W, a.w_router, nullptr, false, logits, nullptr, 1, p.slabs, a.n, p.Ep, a.W, st)) return q; }
-    else if (pgk_status q = gemm128s_bf16_nt((const bf16*)a.x, (const bf16*)a.w_router, nullptr, logits, 2, p.slabs, a.n, p.Ep, a.W, st, nullptr, false, nullptr)) return q;
-    const size_t lds = (size_t)4 * route_floats(r) * 4;
-    PGK_REQUIRE(lds <= 60 * 1024, "moe: %d experts", r.E);
-    moe_route_kernel<<<ceil_div(a.n, 4), 256, lds, st>>>(r, logits, p.Ep, p.slabs, (size_t)a.n * p.Ep, a.n, ids, wts);
+    if (r.table) {
+        PGK_REQUIRE(a.tok, "moe: a table of experts needs the rows' tokens");
+        moe_table_kernel<<<ceil_div(p.total, 256), 256, 0, st>>>(r.table, a.tok, p.total, r.top, ids, wts);
+    } else {
+        if (dt == PGK_F32) { if (pgk_status q = pgk_gemm_nt(a.x, a.w_router, nullptr, logits, a.n, p.Ep, a.W, PGK_F32, st)) return q; }
+        else if (a.n <= 128) { if (pgk_status q = wsgemm_nt((const bf16*)a.x, a.W, a.w_router, nullptr, false, logits, nullptr, 1, p.slabs, a.n, p.Ep, a.W, st)) return q; }
+        else if (pgk_status q = gemm128s_bf16_nt((const bf16*)a.x, (const bf16*)a.w_router, nullptr, logits, 2, p.slabs, a.n, p.Ep, a.W, st, nullptr, false, nullptr)) return q;
+        const size_t lds = (size_t)4 * route_floats(r) * 4;
+        PGK_REQUIRE(lds <= 60 * 1024, "moe: %d experts", r.E);
+        moe_route_kernel<<<ceil_div(a.n, 4), 256, lds, st>>>(r, logits, p.Ep, p.slabs, (size_t)a.n * p.Ep, a.n, ids, wts);
+    }
     PGK_LAUNCH_CHECK();
     moe_sort_kernel<<<r.E, p.total > 2048 ? 1024 : 256, 0, st>>>(ids, p.total, r.E, p.tm, order, tiles, count);
     PGK_LAUNCH_CHECK();
-    const GroupArgs up{tiles, count, order, wts, (long long)2 * a.ff * a.W, r.top}, down{tiles, count, order, wts, (long long)a.ff * a.W, 0};
+    const GroupArgs up{tiles, count, order, wts, (long long)(a.gelu ? 1 : 2) * a.ff * a.W, r.top}, down{tiles, count, order, wts, (long long)a.ff * a.W, 0};
     const int tn_up = ceil_div(a.ff, 64), tn_down = ceil_div(a.W, 64);
     if (dt == PGK_F32) {
-        moe_f32_kernel<true><<<dim3(tn_up, p.max_tiles), 256, 0, st>>>((const float*)a.x, (const float*)a.w_up, (float*)(ws + p.act), a.ff, a.W, up);
+        const float *x = (const float*)a.x, *wu = (const float*)a.w_up;
+        if (a.gelu) moe_f32_kernel<MOE_GELU><<<dim3(tn_up, p.max_tiles), 256, 0, st>>>(x, wu, (float*)(ws + p.act), a.ff, a.W, up);
+        else moe_f32_kernel<MOE_SWIGLU><<<dim3(tn_up, p.max_tiles), 256, 0, st>>>(x, wu, (float*)(ws + p.act), a.ff, a.W, up);
         PGK_LAUNCH_CHECK();
-        moe_f32_kernel<false><<<dim3(tn_down, p.max_tiles), 256, 0, st>>>((const float*)(ws + p.act), (const float*)a.w_down, (float*)a.out, a.W, a.ff, down);
+        moe_f32_kernel<MOE_DOWN><<<dim3(tn_down, p.max_tiles), 256, 0, st>>>((const float*)(ws + p.act), (const float*)a.w_down, (float*)a.out, a.W, a.ff, down);
         PGK_LAUNCH_CHECK();
         return PGK_OK;
     }
     const bf16 *x = (const bf16*)a.x, *wu = (const bf16*)a.w_up, *wd = (const bf16*)a.w_down;
     bf16 *act = (bf16*)(ws + p.act), *out = (bf16*)a.out;
     if (p.tm == 128) {
-        if (pgk_status q = gemm128s_grouped(x, wu, act, false, up, p.max_tiles, p.total, a.ff, a.W, st)) return q;
-        return gemm128s_grouped(act, wd, out, true, down, p.max_tiles, p.total, a.W, a.ff, st);
+        if (pgk_status q = gemm128s_grouped(x, wu, act, a.gelu ? MOE_GELU : MOE_SWIGLU, up, p.max_tiles, p.total, a.ff, a.W, st)) return q;
+        return gemm128s_grouped(act, wd, out, MOE_DOWN, down, p.max_tiles, p.total, a.W, a.ff, st);
     }
     PGK_REQUIRE(p.max_tiles <= 65535, "moe: %d tiles", p.max_tiles);
-    if (p.tm == 32) {
-        moe_stream_kernel<2, true><<<dim3(tn_up, p.max_tiles), 256, 0, st>>>(x, wu, act, a.ff, a.W, up);
+    auto go = [&](auto mt) -> pgk_status {
+        constexpr int MT = decltype(mt)::value;
+        if (a.gelu) moe_stream_kernel<MT, MOE_GELU><<<dim3(tn_up, p.max_tiles), 256, 0, st>>>(x, wu, act, a.ff, a.W, up);
+        else moe_stream_kernel<MT, MOE_SWIGLU><<<dim3(tn_up, p.max_tiles), 256, 0, st>>>(x, wu, act, a.ff, a.W, up);
         PGK_LAUNCH_CHECK();
-        moe_stream_kernel<2, false><<<dim3(tn_down, p.max_tiles), 256, 0, st>>>(act, wd, out, a.W, a.ff, down);
-    } else {
-        moe_stream_kernel<1, true><<<dim3(tn_up, p.max_tiles), 256, 0, st>>>(x, wu, act, a.ff, a.W, up);
+        moe_stream_kernel<MT, MOE_DOWN><<<dim3(tn_down, p.max_tiles), 256, 0, st>>>(act, wd, out, a.W, a.ff, down);
         PGK_LAUNCH_CHECK();
-        moe_stream_kernel<1, false><<<dim3(tn_down, p.max_tiles), 256, 0, st>>>(act, wd, out, a.W, a.ff, down);
-    }
-    PGK_LAUNCH_CHECK();
-    return PGK_OK;
+        return PGK_OK;
+    };
+    return p.tm == 32 ? go(std::integral_constant<int, 2>{}) : go(std::integral_constant<int, 1>{});
 }
 
 template <class T>
@@ -315,6 +332,23 @@ __global__ __launch_bounds__(256) void moe_sum_kernel(const T* e, float* out, in
 
 using namespace pgk;
 
+// rows through `m` (out and ws are set here), summed over the chosen experts
+static pgk_status moe_op(MoeArgs m, float* out, pgk_dtype dt, hipStream_t st) {
+    const size_t rows = (((size_t)m.n * m.router.top * m.W * dtype_size(dt)) + 255) & ~(size_t)255;
+    char* ws = nullptr;
+    if (pgk_status q = pgk_malloc((void**)&ws, rows + moe_bytes(m.n, m.W, m.ff, m.router, dt))) return q;
+    m.out = ws;
+    m.ws = ws + rows;
+    pgk_status q = moe_rows(m, dt, st);
+    if (q == PGK_OK) {
+        if (dt == PGK_F32) moe_sum_kernel<float><<<m.n, 256, 0, st>>>((const float*)ws, out, m.W, m.router.top);
+        else moe_sum_kernel<bf16><<<m.n, 256, 0, st>>>((const bf16*)ws, out, m.W, m.router.top);
+        if (hipError_t e = hipGetLastError()) q = set_error(PGK_ERR_HIP, "pgk_moe: %s", hipGetErrorString(e));
+    }
+    pgk_free(ws);       // stream-ordered reuse
+    return q;
+}
+
 extern "C" {
 
 pgk_status pgk_moe(const void* x, const void* router, const float* correction, const void* w_up, const void* w_down, float* out, int n, int width, int ff, int experts, int top, int groups,
@@ -322,19 +356,16 @@ pgk_status pgk_moe(const void* x, const void* router, const float* correction, c
     PGK_REQUIRE(x && router && correction && w_up && w_down && out && n >= 1 && top >= 1, "pgk_moe: null pointer or empty");
     PGK_REQUIRE(dt == PGK_BF16 || dt == PGK_F32, "pgk_moe: dtype %d (bf16 or f32)", (int)dt);
     PGK_REQUIRE(width >= 64 && width % 64 == 0 && ff >= 64 && ff % 64 == 0 && experts >= 1, "pgk_moe: %d experts of %d x %d", experts, width, ff);
-    hipStream_t st = resolve_stream(s);
-    const RouterCfg r{correction, experts, top, groups, keep, scale};
-    const size_t rows = (((size_t)n * top * width * dtype_size(dt)) + 255) & ~(size_t)255;
-    char* ws = nullptr;
-    if (pgk_status q = pgk_malloc((void**)&ws, rows + moe_bytes(n, width, ff, r, dt))) return q;
-    pgk_status q = moe_rows(MoeArgs{x, n, width, ff, r, router, w_up, w_down, ws, ws + rows}, dt, st);
-    if (q == PGK_OK) {
-        if (dt == PGK_F32) moe_sum_kernel<float><<<n, 256, 0, st>>>((const float*)ws, out, width, top);
-        else moe_sum_kernel<bf16><<<n, 256, 0, st>>>((const bf16*)ws, out, width, top);
-        if (hipError_t e = hipGetLastError()) q = set_error(PGK_ERR_HIP, "pgk_moe: %s", hipGetErrorString(e));
-    }
-    pgk_free(ws);       // stream-ordered reuse
-    return q;
+    const RouterCfg r{correction, experts, top, groups, keep, scale, nullptr};
+    return moe_op(MoeArgs{x, n, width, ff, r, router, w_up, w_down, nullptr, nullptr}, out, dt, resolve_stream(s));
+}
+
+pgk_status pgk_table_moe(const void* x, const int32_t* table, const int32_t* tokens, const void* w_up, const void* w_down, float* out, int n, int width, int ff, int experts, int top,
+                         pgk_dtype dt, pgk_stream s) {
+    PGK_REQUIRE(x && table && tokens && w_up && w_down && out && n >= 1 && top >= 1, "pgk_table_moe: null pointer or empty");
+    PGK_REQUIRE(dt == PGK_BF16 || dt == PGK_F32, "pgk_table_moe: dtype %d (bf16 or f32)", (int)dt);
+    PGK_REQUIRE(width >= 64 && width % 64 == 0 && ff >= 64 && ff % 64 == 0 && experts >= 1, "pgk_table_moe: %d experts of %d x %d", experts, width, ff);
+    return moe_op(MoeArgs{x, n, width, ff, RouterCfg{nullptr, experts, top, 0, 0, 1.0f, table}, nullptr, w_up, w_down, nullptr, nullptr, true, tokens}, out, dt, resolve_stream(s));
 }
 
 }  // extern "C"

@@ -286,7 +286,7 @@ __global__ __launch_bounds__(PK_THREADS) void pkgemm_kernel(PkArgs g) {
             }
     }
     // C/D map: column (weight row) = l15 of the tile, row m = mt * 16 + 4 q + r
-    if constexpr (EPI == PK_EPI_BF16 || EPI == PK_EPI_XIELU || EPI == PK_EPI_SLAB || EPI == PK_EPI_ACCUM) {
+    if constexpr (EPI == PK_EPI_BF16 || EPI == PK_EPI_XIELU || EPI == PK_EPI_GELU || EPI == PK_EPI_SLAB || EPI == PK_EPI_ACCUM) {
 #pragma unroll
         for (int t = 0; t < NTW; ++t) {
             const int n = (tile_a + t * g.tile_b_off) * 16 + l15;
@@ -313,6 +313,7 @@ __global__ __launch_bounds__(PK_THREADS) void pkgemm_kernel(PkArgs g) {
                         if (m < g.M) {
                             if constexpr (EPI == PK_EPI_BF16) reinterpret_cast<bf16*>(g.c)[(size_t)m * g.ldc + n] = from_f<bf16>(acc[t][mt][r]);
                             else if constexpr (EPI == PK_EPI_XIELU) reinterpret_cast<bf16*>(g.c)[(size_t)m * g.ldc + n] = from_f<bf16>(xielu<false>(acc[t][mt][r], g.act_pos, g.act_neg));
+                            else if constexpr (EPI == PK_EPI_GELU) reinterpret_cast<bf16*>(g.c)[(size_t)m * g.ldc + n] = from_f<bf16>(gelu_erf(acc[t][mt][r]));
                             else (reinterpret_cast<float*>(g.c) + (size_t)sp * g.M * g.ldc)[(size_t)m * g.ldc + n] = acc[t][mt][r];
                         }
                     }
@@ -664,6 +665,7 @@ pgk_status pkgemm_nt(const bf16* a, int lda, const void* wp, void* c, int ldc, i
     switch (epi) {
         case PK_EPI_BF16: PGK_PK_LAUNCH(1, PK_EPI_BF16) break;
         case PK_EPI_XIELU: PGK_PK_LAUNCH(1, PK_EPI_XIELU) break;
+        case PK_EPI_GELU: PGK_PK_LAUNCH(1, PK_EPI_GELU) break;
         case PK_EPI_SLAB: PGK_PK_LAUNCH(1, PK_EPI_SLAB) break;
         case PK_EPI_ACCUM: PGK_PK_LAUNCH(1, PK_EPI_ACCUM) break;
         case PK_EPI_SWIGLU: PGK_PK_LAUNCH(2, PK_EPI_SWIGLU) break;

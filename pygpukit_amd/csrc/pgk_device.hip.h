@@ -45,6 +45,8 @@ template <bool EXACT> __device__ __forceinline__ float xielu(float z, float a, f
     return fmaf(0.5f, z, z > 0.f ? a * z * z : b * (e - n));
 }
 
+__device__ __forceinline__ float gelu_erf(float z) { return 0.5f * z * (1.0f + erff(z * 0.70710678118654752f)); }
+
 // ---- 16-byte vectors ----------------------------------------------------------------------
 // Vec<T>::N elements of T in one 16-byte access: 4 x fp32 or 8 x 16-bit.
 template <class T> struct Vec {

@@ -6,7 +6,7 @@
 
 namespace pgk {
 
-enum { PK_EPI_BF16 = 0, PK_EPI_SLAB = 1, PK_EPI_ACCUM = 2, PK_EPI_SWIGLU = 3, PK_EPI_QKV = 4, PK_EPI_XIELU = 5 };
+enum { PK_EPI_BF16 = 0, PK_EPI_SLAB = 1, PK_EPI_ACCUM = 2, PK_EPI_SWIGLU = 3, PK_EPI_QKV = 4, PK_EPI_XIELU = 5, PK_EPI_GELU = 6 };
 
 struct PkArgs {
     const bf16* a;
@@ -31,7 +31,7 @@ struct PkArgs {
     const float* ss_in;
     int ss_n;
     float ss_eps;
-    float act_pos, act_neg;   // PK_EPI_XIELU: bf16 rows of xIELU of the result
+    float act_pos, act_neg;   // PK_EPI_XIELU: bf16 rows of xIELU of the result (PK_EPI_GELU: of its gelu)
 };
 
 constexpr int PK_SS_LD = 64;    // floats per row of a sum-of-squares table

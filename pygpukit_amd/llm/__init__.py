@@ -1,15 +1,16 @@
 """LLM layer of pygpukit_amd: config, layers, CausalTransformerModel, decode strategies, native engine."""
 
 from pygpukit_amd.llm.buffers import DecodeBuffers, PrefillBuffers
-from pygpukit_amd.llm.config import (GPT2_SPEC, LLAMA_SPEC, MODEL_SPECS, QWEN2_SPEC, QWEN3_SPEC, TOTOLORN_SPEC, MALASUN_SPEC, RATASUN_SPEC, ExpertsConfig, GPT2Config, LayerConfig, LlamaConfig, LoopConfig, ModelSpec,
+from pygpukit_amd.llm.config import (FETEZEN_SPEC, GPT2_SPEC, LLAMA_SPEC, MODEL_SPECS, QWEN2_SPEC, QWEN3_SPEC, TOTOLORN_SPEC, MALASUN_SPEC, RATASUN_SPEC, ExpertsConfig, GPT2Config, LayerConfig, LlamaConfig, LoopConfig, ModelSpec,
                                     Qwen3Config, TransformerConfig, detect_model_spec, layer_list_config)
 from pygpukit_amd.llm.decode import DecodeBatch, DecodeM1, DecodeM1Graph, DecodeStrategy
 from pygpukit_amd.llm.engine import Engine, StackEngine
-from pygpukit_amd.llm.layers import (MLP, Attention, ChannelDelta, GatedRecurrence, GatedWindowAttention, LatentAttention, Linear, LinearBF16, LinearFP8, MixtureOfExperts, Norm, ParallelBlock,
-                                    StateSpace, TransformerBlock, apply_rotary_pos_emb_numpy, precompute_freqs_cis)
-from pygpukit_amd.llm.models import CausalTransformerModel, GPT2Model, LlamaModel, MalasunModel, QwenModel, RatasunModel, TotolornModel
+from pygpukit_amd.llm.layers import (MLP, Attention, ChannelDelta, GatedRecurrence, GatedWindowAttention, HyperBlock, HyperConnection, LatentAttention, Linear, LinearBF16, LinearFP8, MixtureOfExperts, Norm, ParallelBlock,
+                                    StateSpace, TableExperts, TalkingAttention, TransformerBlock, apply_rotary_pos_emb_numpy, precompute_freqs_cis)
+from pygpukit_amd.llm.models import CausalTransformerModel, FetezenModel, GPT2Model, LlamaModel, MalasunModel, QwenModel, RatasunModel, TotolornModel
 from pygpukit_amd.llm.loader import (FP8QuantConfig, load_gpt2_from_safetensors, load_llama_from_safetensors,  # noqa: E402
-                                     load_model_from_safetensors, load_qwen3_from_safetensors, load_totolorn_from_safetensors, load_malasun_from_safetensors, load_ratasun_from_safetensors)
+                                     load_model_from_safetensors, load_qwen3_from_safetensors, load_totolorn_from_safetensors, load_malasun_from_safetensors, load_ratasun_from_safetensors,
+                                     load_fetezen_from_safetensors)
 from pygpukit_amd.llm.scheduler import BatchScheduler  # noqa: E402
 from pygpukit_amd.llm.safetensors import Dtype, SafeTensorsFile, ShardedSafeTensorsFile, TensorInfo, load_safetensors  # noqa: E402
 from pygpukit_amd.llm.sampling import sample_token
@@ -30,4 +31,5 @@ __all__ = ["load_model_from_safetensors", "load_qwen3_from_safetensors", "load_l
            "CausalSelfAttention", "LlamaMLP", "LlamaBlock", "TOTOLORN_SPEC", "LayerConfig", "layer_list_config", "StackEngine", "LatentAttention", "TotolornModel",
            "load_totolorn_from_safetensors", "BatchScheduler", "MALASUN_SPEC", "MalasunModel", "GatedWindowAttention", "GatedRecurrence",
            "load_malasun_from_safetensors", "RATASUN_SPEC", "RatasunModel", "ExpertsConfig", "LoopConfig", "ChannelDelta", "StateSpace", "MixtureOfExperts",
-           "ParallelBlock", "load_ratasun_from_safetensors"]
+           "ParallelBlock", "load_ratasun_from_safetensors", "FETEZEN_SPEC", "FetezenModel", "HyperBlock", "HyperConnection", "TableExperts", "TalkingAttention",
+           "load_fetezen_from_safetensors"]

@@ -2,8 +2,8 @@
 
 TransformerConfig carries the dimensions; ModelSpec is the data-only description of one
 architecture family (HF tensor-name patterns + architecture flags + default hyper-parameters).
-Described are the dense families GPT-2, Llama, Qwen2, Qwen3 and the layer-list families Totolorn, Malasun and Ratasun (whose
-feed-forwards are mixtures of experts).  A layer-list model's config.json spells out every layer: LayerConfig."""
+Described are the dense families GPT-2, Llama, Qwen2, Qwen3 and the layer-list families Totolorn, Malasun, Ratasun (whose
+feed-forwards are mixtures of experts) and Fetezen (dense layers beside experts that a table of tokens chooses).  A layer-list model's config.json spells out every layer: LayerConfig."""
 
 from __future__ import annotations
 
@@ -45,7 +45,7 @@ class ModelSpec:
     expert_up_proj: str | None = None
     expert_down_proj: str | None = None
     norm_type: Literal["rmsnorm", "layernorm"] = "rmsnorm"
-    activation: Literal["gelu", "silu", "xielu"] = "silu"
+    activation: Literal["gelu", "silu", "xielu", "poly_norm"] = "silu"
     use_rope: bool = True
     use_qk_norm: bool = False
     use_position_embed: bool = False
@@ -93,6 +93,14 @@ class ModelSpec:
     router_correction: str | None = None
     loop_in: str | None = None             # passes over a stretch of layers: map of [stream; embedding], one vector per pass
     loop_step: str | None = None
+    talk: str | None = None                # attention: mix of the heads' scores, sinks
+    sink: str | None = None
+    chunked: bool = False                  # an attention mask's size is a chunk, not a sliding window
+    hyper: str | None = None               # hyper-connections of sublayer {sublayer}: prefix of its in, out and mix
+    expert_table: str | None = None        # experts: table of tokens instead of a router; the shared expert and its gate
+    shared_up_proj: str | None = None
+    shared_down_proj: str | None = None
+    shared_gate: str | None = None
 
 
 def _hf_decoder_spec(name: str, *, qk_norm: bool, qkv_bias: bool, eps: float, theta: float) -> ModelSpec:
@@ -166,8 +174,17 @@ RATASUN_SPEC = ModelSpec(
     step_bias=_T + "mix.dt_bias", in_proj=_T + "mix.in", conv=_T + "mix.conv", conv_bias=_T + "mix.conv.b", skip=_T + "mix.D", out_norm=_T + "mix.norm",
     router=_T + "mlp.router", router_correction=_T + "mlp.correction", loop_in="loop.in", loop_step="loop.step")
 
+FETEZEN_SPEC = ModelSpec(
+    name="fetezen", embed_tokens="embed", position_embed=None, lm_head="head", final_norm="final.norm", final_norm_bias=None,
+    attn_norm=_T + "norm1", attn_norm_bias=None, q_proj=_T + "mix.q", k_proj=_T + "mix.k", v_proj=_T + "mix.v", o_proj=_T + "mix.o",
+    q_bias=_T + "mix.q.b", k_bias=_T + "mix.k.b", v_bias=_T + "mix.v.b", o_bias=_T + "mix.o.b", q_norm=_T + "mix.q.norm", k_norm=_T + "mix.k.norm",
+    mlp_norm=_T + "norm2", mlp_norm_bias=None, fc1=_T + "mlp.up", fc1_bias=None, fc2=_T + "mlp.down", fc2_bias=None, gate_proj=None, up_proj=None, down_proj=None,
+    expert_up_proj=_T + "mlp.e{expert}.up", expert_down_proj=_T + "mlp.e{expert}.down", norm_type="rmsnorm", activation="poly_norm", use_rope=True, use_qk_norm=True,
+    is_moe=True, architecture="Fetezen", act_params=_T + "mlp.act", residual_f32=True, talk=_T + "mix.talk", sink=_T + "mix.sink", chunked=True, hyper=_T + "hc{sublayer}.",
+    expert_table=_T + "mlp.table", shared_up_proj=_T + "mlp.shared.up", shared_down_proj=_T + "mlp.shared.down", shared_gate=_T + "mlp.shared.sg")
+
 MODEL_SPECS: dict[str, ModelSpec] = {"gpt2": GPT2_SPEC, "llama": LLAMA_SPEC, "qwen3": QWEN3_SPEC, "qwen2": QWEN2_SPEC,
-                                     "totolorn": TOTOLORN_SPEC, "malasun": MALASUN_SPEC, "ratasun": RATASUN_SPEC}
+                                     "totolorn": TOTOLORN_SPEC, "malasun": MALASUN_SPEC, "ratasun": RATASUN_SPEC, "fetezen": FETEZEN_SPEC}
 
 
 def detect_model_spec(tensor_names: list[str], config: dict | None = None) -> ModelSpec:
@@ -194,13 +211,16 @@ def detect_model_spec(tensor_names: list[str], config: dict | None = None) -> Mo
 
 @dataclass(frozen=True)
 class ExpertsConfig:
-    """A layer's mixture of experts; with groups > 0 only experts of the `keep` best groups of neighbours can be chosen."""
+    """A layer's mixture of experts; with groups > 0 only experts of the `keep` best groups of neighbours can be chosen.  With `table` a
+    table of token ids chooses; shared_size: width of one more expert that every token runs (None: none)."""
 
     count: int
     top: int
     groups: int
     keep: int
     scale: float                      # of the chosen experts' weights, which sum to it
+    table: bool = False
+    shared_size: int | None = None
 
 
 @dataclass(frozen=True)
@@ -233,30 +253,33 @@ class LayerConfig:
     num_kv_heads: int = 0             # attention: key / value heads
     conv_taps: int | None = None      # attention: taps over time on q, k, v (None: no convolution)
     kv_from: int | None = None        # attention: the layer whose keys and values this one uses (None: its own)
-    # latent attention: rotated query / key columns beside head_dim's (0: none); pair i turns by position * base^(-2i / rot_dim)
+    # rotated query / key columns (0: none), pair i turns by position * base^(-2i / rot_dim): latent attention: beside head_dim's, neighbours
+    # are a pair; attention: the first of head_dim's, i and i + rot_dim / 2 are a pair
     rot_dim: int = 0
     rot_base: float = 10000.0
     norm_groups: int = 1              # state space: equal parts of the output that are normed on their own
     experts: ExpertsConfig | None = None
+    chunked: bool = False             # attention: `window` is the size of the chunks of positions that see only themselves
 
 
-def parse_experts(i: int, mlp: dict) -> tuple[ExpertsConfig, int]:
-    r = mlp["router"]
+def parse_experts(i: int, mlp: dict, table: bool = False) -> tuple[ExpertsConfig, int]:
+    r, shared = mlp["router"], mlp.get("shared")
     g = r.get("groups")
-    e = ExpertsConfig(int(r["experts"]), int(r["top"]), int(g["count"]) if g else 0, int(g["keep"]) if g else 0, float(r.get("scale", 1.0)))
+    e = ExpertsConfig(int(r["experts"]), int(r["top"]), int(g["count"]) if g else 0, int(g["keep"]) if g else 0, float(r.get("scale", 1.0)), table,
+                      int(shared["ff"]) if shared else None)
     if not 1 <= e.top <= e.count or (e.groups and (e.count % e.groups or not 1 <= e.keep <= e.groups or e.keep * (e.count // e.groups) < e.top)):
         raise ValueError(f"layer {i}: cannot choose {e.top} of {e.count} experts in {e.keep} of {e.groups} groups")
     return e, int(mlp["expert"]["ff"])
 
 
-def parse_layer(i: int, entry: dict) -> LayerConfig:
+def parse_layer(i: int, entry: dict, spec: ModelSpec | None = None) -> LayerConfig:
     kind, mlp = entry.get("type"), entry.get("mlp")
     if kind not in ("latent_attention", "attention", "hgrn2", "channel_delta", "mamba2"):
         raise ValueError(f"layer {i}: unknown mixer {kind!r}")
     m = entry["mixer"]
     if mlp is not None and mlp.get("kind") not in ("dense", "moe"):
         raise ValueError(f"layer {i}: unknown feed-forward {mlp.get('kind')!r}")
-    experts, ff = (None, None) if mlp is None else parse_experts(i, mlp) if mlp["kind"] == "moe" else (None, int(mlp["ff"]))
+    experts, ff = (None, None) if mlp is None else parse_experts(i, mlp, spec is not None and spec.expert_table is not None) if mlp["kind"] == "moe" else (None, int(mlp["ff"]))
     heads, vdim = int(m["heads"]), int(m["vdim"])
     dim = int(m["state"] if kind == "mamba2" else m["dim"])
     if kind == "hgrn2":
@@ -275,9 +298,13 @@ def parse_layer(i: int, entry: dict) -> LayerConfig:
             raise ValueError(f"layer {i}: {rd} rotated columns, rotation of {rot}")
         return LayerConfig(kind, heads, dim, vdim, int(m["kv_rank"]), window, float(m["scale"]), ff, rot_dim=rd, rot_base=float(rot["base"]) if rot else 10000.0,
                            experts=experts)
-    taps, src = m.get("conv"), m.get("kv_from")
+    taps, src, rot = m.get("conv"), m.get("kv_from"), m.get("rot") if spec is not None and spec.use_rope else None
+    rd = int(rot["dims"]) if rot else 0
+    if rd % 2 or not 0 <= rd <= dim or (window is not None and window < 1):
+        raise ValueError(f"layer {i}: {rd} rotated columns of {dim}, mask of {window}")
     return LayerConfig(kind, heads, dim, vdim, 0, window, float(m["scale"]), ff, int(m["kv_heads"]), int(taps) if taps is not None else None,
-                       int(src) if src is not None else None)
+                       int(src) if src is not None else None, rot_dim=rd, rot_base=float(rot["base"]) if rot else 10000.0, experts=experts,
+                       chunked=window is not None and spec is not None and spec.chunked)
 
 
 def distance_slopes(heads: int) -> list[float]:
@@ -290,7 +317,8 @@ NO_POSITION_LIMIT = 2**30       # models without learned positions
 
 def layer_list_config(config: dict) -> "TransformerConfig":
     """config.json of a layer-list model -> TransformerConfig.  The per-model head fields take the first layer's values."""
-    layers = tuple(parse_layer(i, e) for i, e in enumerate(config["layers"]))
+    found = next((s for s in MODEL_SPECS.values() if s.architecture and s.architecture == config.get("architecture")), None)
+    layers = tuple(parse_layer(i, e, found) for i, e in enumerate(config["layers"]))
     if not layers:
         raise ValueError("config.json lists no layers")
     for i, l in enumerate(layers):
@@ -306,13 +334,17 @@ def layer_list_config(config: dict) -> "TransformerConfig":
         loop = LoopConfig(int(loop["start"]), int(loop["stop"]), int(loop["times"]))
         if not 0 <= loop.start < loop.stop <= len(layers) or loop.times < 1 or any(l.kv_from is not None for l in layers):
             raise ValueError(f"cannot run layers {loop.start} .. {loop.stop - 1} of {len(layers)} {loop.times} times")
-    spec = next((s for s in MODEL_SPECS.values() if s.architecture == config.get("architecture")), TOTOLORN_SPEC)
-    return TransformerConfig(vocab_size=int(config["vocab"]), hidden_size=int(config["width"]), num_layers=len(layers), num_heads=first.num_heads,
+    spec = found or TOTOLORN_SPEC
+    width, streams, groups, cap = int(config["width"]), int(config.get("streams", 1)), int(config["norm"].get("groups", 1)), config.get("logit_softcap")
+    if groups < 1 or width % groups or streams < 1 or (cap is not None and not float(cap) > 0) or (spec.hyper is None and (streams, groups, cap) != (1, 1, None)):
+        raise ValueError(f"{spec.name}: width {width} in {groups} norm groups, {streams} streams, logits capped at {cap}")
+    return TransformerConfig(vocab_size=int(config["vocab"]), hidden_size=width, num_layers=len(layers), num_heads=first.num_heads,
                              num_kv_heads=first.num_kv_heads or first.num_heads, intermediate_size=max([l.intermediate_size or 0 for l in layers]),
                              _head_dim=first.head_dim, norm_type=spec.norm_type, activation=spec.activation, use_rope=spec.use_rope, loop=loop,
                              logit_scale=float(config.get("logit_scale", 1.0)),
                              max_position_embeddings=int(config["max_positions"]) if spec.use_position_embed else NO_POSITION_LIMIT,
-                             norm_eps=float(config["norm"]["eps"]), tie_word_embeddings=False, layers=layers, residual_mult=float(config.get("residual_mult", 1.0)))
+                             norm_eps=float(config["norm"]["eps"]), tie_word_embeddings=False, layers=layers, residual_mult=float(config.get("residual_mult", 1.0)),
+                             streams=streams, norm_groups=groups, logit_softcap=None if cap is None else float(cap))
 
 
 @dataclass
@@ -331,7 +363,7 @@ class TransformerConfig:
     num_experts_per_tok: int = 2
     moe_intermediate_size: int | None = None
     norm_type: Literal["rmsnorm", "layernorm"] = "rmsnorm"
-    activation: Literal["gelu", "silu", "xielu"] = "silu"
+    activation: Literal["gelu", "silu", "xielu", "poly_norm"] = "silu"
     use_rope: bool = True
     causal: bool = True
     max_position_embeddings: int = 2048
@@ -342,6 +374,9 @@ class TransformerConfig:
     residual_mult: float = 1.0                       # factor of every sublayer's contribution to the residual stream
     loop: LoopConfig | None = None                   # layer-list models: a stretch of layers that runs several times
     logit_scale: float = 1.0                         # factor of the logits (the loader multiplies the output norm's weight by it)
+    streams: int = 1                                 # hyper-connected models: residual streams
+    norm_groups: int = 1                             # equal parts of the width that the norms treat on their own
+    logit_softcap: float | None = None               # logits become cap * tanh(logits / cap)
 
     def __post_init__(self):
         if self.num_kv_heads is None:

@@ -16,7 +16,7 @@ class DecodeM1(DecodeStrategy):
         if model.config.layers is not None:      # fp32 residual stream, per-layer sizes: the block runs its own sequence of ops
             hidden = model._decode_step_fixed_cache(token_id, position, context_len)
             matmul_nt(hidden, model._lm_head if model._lm_head is not None else model.embed_tokens, out=buffers.logits)
-            return buffers.logits
+            return model.cap_logits(buffers.logits)
         embedding_lookup(model.embed_tokens, buffers.hidden, token_id)
         for block in model.blocks:
             rmsnorm(buffers.hidden, block.attn_norm.weight, block.attn_norm.eps, out=buffers.norm_out)

@@ -13,7 +13,7 @@ import numpy as np
 
 from pygpukit_amd import _hip
 from pygpukit_amd.core.array import GPUArray
-from pygpukit_amd.core.dtypes import bfloat16, float32
+from pygpukit_amd.core.dtypes import bfloat16, float32, int32
 from pygpukit_amd.core.factory import from_numpy, zeros
 from pygpukit_amd.llm.config import LoopConfig
 from pygpukit_amd.ops.tensor import concat_axis0, pad_2d
@@ -347,21 +347,22 @@ def _pad_taps(taps: tuple[GPUArray, ...], heads: tuple[tuple[int, int], ...]) ->
 
 class StackEngine(Engine):
     """The native engine for layer-list models (csrc/engine_stack.hip): fp32 residual stream, sandwich layers (a norm after each sublayer
-    and optionally before it) or parallel ones (one norm, mixer beside experts), a mixer per layer (latent attention, attention over
-    a K/V ring, linear recurrences, gated delta rule), every layer with its own sizes, possibly a stretch of layers that runs several
+    and optionally before it) parallel ones (one norm, mixer beside experts) or hyper-connected ones (several streams), a mixer per layer (latent attention, attention
+    over a K/V ring, with mixed scores or without, linear recurrences, gated delta rule), every layer with its own sizes, possibly a stretch of layers that runs several
     times.  State, graphs, sampling and generation are Engine's.
 
-    The cache of an attention layer is a ring of min(window, max_seq_len) rows per sequence slot, that of a recurrent one a state: a
+    The cache of an attention layer is a ring of min(window or chunk, max_seq_len) rows per sequence slot, that of a recurrent one a state: a
     sequence goes on where it stopped (or starts again at position 0); a position whose window or state has been overwritten is refused."""
 
     _SIZES = ("mixer", "ff", "heads", "kv_heads", "dim", "vdim", "rank", "window", "taps", "kv_from", "head_pad", "vhead_pad", "rank_pad", "n_att", "ff_pad")
-    _MORE = dict(gated=0, rot=0, norm_parts=1, rank_a=0, rank_g=0, experts=0, top=0, groups=0, keep=0)       # sizes of some layers, and their defaults
+    _MORE = dict(gated=0, rot=0, norm_parts=1, rank_a=0, rank_g=0, experts=0, top=0, groups=0, keep=0, chunked=0, ff_dim=0, shared_pad=0)       # sizes of some layers, and their defaults
 
     def __init__(self, config: dict, embed: GPUArray, position_embed: GPUArray | None, head: GPUArray, final_norm: GPUArray, layers: list[dict], *,
                  max_seq_len: int = 512, max_batch: int = 1):
         """config: vocab_size, width, max_positions, norm_eps, residual_mult; for parallel layers block and layer_norm, with a loop `loop`
-        (start, stop, times) and its arrays loop_in [wp, 2 wp], loop_step [times, wp].  layers[i]: the sizes and packed arrays of
-        pack_layer(), pack_attention(), pack_recurrence(), pack_delta() or pack_state_space()."""
+        (start, stop, times) and its arrays loop_in [wp, 2 wp], loop_step [times, wp]; for hyper-connected ones block, streams, norm_groups,
+        logit_cap.  layers[i]: the sizes and packed arrays of pack_layer(), pack_attention(), pack_recurrence(), pack_delta(),
+        pack_state_space() or pack_talking()."""
         _hip.require_device()
         dt = embed.dtype
         if dt not in (bfloat16, float32):
@@ -376,22 +377,35 @@ class StackEngine(Engine):
             raise ValueError("StackEngine: embedding / head / final norm shapes do not match the configuration")
         if position_embed is not None and position_embed.shape != (config["max_positions"], config["width"]):
             raise ValueError(f"StackEngine: position table {position_embed.shape}")
-        parallel, loop = config.get("block", _hip.BLOCK_SANDWICH) == _hip.BLOCK_PARALLEL, config.get("loop")
+        block, loop = config.get("block", _hip.BLOCK_SANDWICH), config.get("loop")
+        parallel, hyper, streams = block == _hip.BLOCK_PARALLEL, block == _hip.BLOCK_HYPER, config.get("streams", 1)
         self._runs = [i for i, _ in LoopConfig(*loop).runs(len(layers))] if loop else list(range(len(layers)))
         arr = (_hip.StackLayer * len(layers))()
         for i, lw in enumerate(layers):
             hd, gd = lw["heads"] * lw["head_pad"], 0 if lw["kv_from"] >= 0 else lw["kv_heads"] * lw["head_pad"]
             moe, E = lw["ff_pad"] and lw["ff"] == _hip.FF_MOE, lw.get("experts", 0)
             ff, rp, n_att, n_in = lw["ff_pad"], lw["rank_pad"], lw["n_att"], lw["w_in"].shape[0] - (_up64(E) if moe else 0)
-            up = 2 * ff if lw["ff"] == _hip.FF_SWIGLU else ff
+            up, table = 2 * ff if lw["ff"] == _hip.FF_SWIGLU else ff, ff and lw["ff"] == _hip.FF_TABLE
             # name -> (shape, dtype, may be absent)
-            want = {"norm1": ((1, wp), float32, not parallel), "norm1b": ((1, wp), float32, parallel), "w_in": ((n_in + (_up64(E) if moe else 0), wp), dt, False),
+            want = {"norm1": ((1, wp), float32, not parallel and not hyper), "norm1b": ((1, wp), float32, parallel or hyper), "w_in": ((n_in + (_up64(E) if moe else 0), wp), dt, False),
                     "w_o": ((wp, n_att), dt, False), "b_in": ((1, n_in), float32, True)}
             if moe:
                 want.update(w_gate_up=((E, 2 * ff, wp), dt, False), w_down=((E, wp, ff), dt, False), correction=((E,), float32, False))
+            elif table:
+                sp = lw["shared_pad"]
+                want.update(w_gate_up=((E, ff, wp), dt, False), w_down=((E, wp, ff), dt, False), table=((config["vocab_size"], lw["top"]), int32, False),
+                            w_shared_up=((sp, wp), dt, not sp), w_shared_down=((wp, sp), dt, not sp), w_shared_gate=((1, wp), dt, not sp))
+            elif ff and hyper:
+                want.update(w_gate_up=((ff, wp), dt, False), w_down=((wp, ff), dt, False), act=((4,), float32, False))
             elif ff:
                 want.update(norm2=((1, wp), float32, True), norm2b=((1, wp), float32, False), w_gate_up=((up, wp), dt, False), w_down=((wp, ff), dt, False))
-            if lw["mixer"] == _hip.MIX_LATENT:
+            if hyper:
+                want.update(hyper1=((streams * (streams + 2),), float32, False), hyper2=((streams * (streams + 2),), float32, not ff), norm2=((1, wp), float32, not ff))
+            if lw["mixer"] == _hip.MIX_TALK:
+                hp = lw["head_pad"]
+                want.update(q_norm=((1, hp), float32, False), k_norm=((1, hp), float32, lw["kv_from"] >= 0), rot_freq=((lw["rot"] // 2,), float32, not lw["rot"]),
+                            talk=((lw["heads"], lw["heads"]), float32, True), sink=((lw["heads"],), float32, True), b_o=((1, wp), float32, True))
+            elif lw["mixer"] == _hip.MIX_LATENT:
                 want.update(c_norm=((1, rp), float32, False), w_ukv=((2 * hd, rp), dt, False), rot_freq=((lw.get("rot", 0) // 2,), float32, not lw.get("rot", 0)))
             elif lw["mixer"] in (_hip.MIX_DELTA, _hip.MIX_SSD):
                 delta, hv = lw["mixer"] == _hip.MIX_DELTA, lw["heads"] * lw["vhead_pad"]
@@ -418,7 +432,8 @@ class StackEngine(Engine):
             arr[i].n_in, arr[i].scale, arr[i].router_scale = n_in, lw["scale"], lw.get("router_scale", 1.0)
             arr[i].act_pos, arr[i].act_neg = lw.get("act_params", (0.0, 0.0))
         sc = _hip.StackConfig(config["vocab_size"], config["width"], len(layers), config["max_positions"], max_seq_len, max_batch, config["norm_eps"],
-                              config["residual_mult"], dt.code, int(parallel), int(config.get("layer_norm", 0)))
+                              config["residual_mult"], dt.code, block, int(config.get("layer_norm", 0)))
+        sc.streams, sc.norm_groups, sc.logit_cap = streams, config.get("norm_groups", 1), config.get("logit_cap") or 0.0
         if loop:
             lin, step = config["loop_in"], config["loop_step"]
             if lin.shape != (wp, 2 * wp) or lin.dtype != dt or step.shape != (loop[2], wp) or step.dtype != float32:
@@ -568,6 +583,80 @@ class StackEngine(Engine):
                    o_norm=from_numpy(_pad_heads(_host_f32(out_norm).reshape(1, -1), heads, vp)), w_o=_head_cols(o, heads, vdim, vp, wp, n_att))
         return out
 
+    @classmethod
+    def pack_talking(cls, q: GPUArray, k: GPUArray | None, v: GPUArray | None, o: GPUArray, norm1: GPUArray, *, heads: int, kv_heads: int, dim: int, vdim: int, window: int,
+                     chunked: bool, scale: float, biases: tuple, o_bias: GPUArray | None, q_norm: GPUArray, k_norm: GPUArray | None, rot_freq: GPUArray | None = None,
+                     talk: GPUArray | None = None, sink: GPUArray | None = None, kv_from: int | None = None) -> dict:
+        """The mixer of one hyper-connected layer: q, k, v, o [out, in] (k, v None with kv_from) and their biases; fp32 norms over a head's dim,
+        rot_freq [rot / 2], talk [heads, heads], sink [heads]."""
+        width = q.shape[1]
+        wp, hp = _up64(width), _attention_pad(dim, vdim)
+        parts = [(q, heads, dim)] + ([] if kv_from is not None else [(k, kv_heads, dim), (v, kv_heads, vdim)])
+        w_in = _stack_rows([_head_rows(w, n, d, hp, wp) for w, n, d in parts])
+        b = np.zeros((1, w_in.shape[0]), np.float32)
+        flat = np.concatenate([_pad_heads(_host_f32(a).reshape(-1), n, hp) for a, (_, n, _) in zip(biases, parts)])
+        b[0, :flat.size] = flat
+        out = cls._pack_common(width, norm1, None, None, None, None, None, None)
+        out.update(mixer=_hip.MIX_TALK, heads=heads, kv_heads=kv_heads, dim=dim, vdim=vdim, window=window, chunked=int(chunked), scale=scale, head_pad=hp, vhead_pad=hp, n_att=heads * hp,
+                   kv_from=-1 if kv_from is None else kv_from, w_in=w_in, b_in=from_numpy(b), q_norm=_row(q_norm, hp), k_norm=None if k_norm is None else _row(k_norm, hp),
+                   rot=0 if rot_freq is None else 2 * rot_freq.size, rot_freq=rot_freq, talk=talk, sink=sink,
+                   b_o=None if o_bias is None else _row(from_numpy(_host_f32(o_bias)), wp), w_o=_head_cols(o, heads, vdim, hp, wp, heads * hp))
+        return out
+
+    @staticmethod
+    def pack_hyper(read: GPUArray, write: GPUArray, mix: GPUArray) -> GPUArray:
+        """A sublayer's numbers as the kernels read them: read | write | mix [from][to]"""
+        return from_numpy(np.concatenate([a.to_numpy().reshape(-1) for a in (read, write, mix)]))
+
+    @staticmethod
+    def add_poly_mlp(layer: dict, width: int, up: GPUArray, down: GPUArray, act: GPUArray) -> dict:
+        """A packed mixer plus a dense feed-forward with a polynomial-norm activation: up [ff, width], down [width, ff], act fp32 [4]."""
+        ff, wp = up.shape[0], _up64(width)
+        fp = _up64(ff)
+        layer.update(ff=_hip.FF_POLY, ff_pad=fp, ff_dim=ff, w_gate_up=pad_2d(up, fp, wp), w_down=pad_2d(down, wp, fp), act=act)
+        return layer
+
+    @staticmethod
+    def add_table_experts(layer: dict, width: int, table: GPUArray, up: GPUArray, down: GPUArray, shared: tuple[GPUArray, GPUArray, GPUArray] | None) -> dict:
+        """A packed mixer plus experts that a table chooses: table int32 [vocab, top], up [E, ff, width], down [E, width, ff]; shared: the shared
+        expert's up [ff', width], down [width, ff'] and gate [1, width]."""
+        E, ff, _ = up.shape
+        wp, fp = _up64(width), _up64(ff)
+        layer.update(ff=_hip.FF_TABLE, ff_pad=fp, experts=E, top=table.shape[1], table=table, shared_pad=0,
+                     w_gate_up=_head_rows(up.view((E * ff, width)), E, ff, fp, wp).view((E, fp, wp)), w_down=_head_rows(down.view((E * width, ff)), E, width, wp, fp).view((E, wp, fp)))
+        if shared is not None:
+            sp = _up64(shared[0].shape[0])
+            layer.update(shared_pad=sp, w_shared_up=pad_2d(shared[0], sp, wp), w_shared_down=pad_2d(shared[1], wp, sp), w_shared_gate=pad_2d(shared[2], 1, wp))
+        return layer
+
+    @classmethod
+    def _pack_hyper_block(cls, b, c) -> dict:
+        from pygpukit_amd.llm.layers import TableExperts, TalkingAttention
+
+        a = b.attn
+        if not isinstance(a, TalkingAttention):
+            raise NotImplementedError(f"the layer-list engine has no hyper-connected layer of {type(a).__name__}")
+        norms = [n for n in (b.attn_norm, b.mlp_norm, a.q_norm, a.k_norm) if n is not None]
+        if any(n.eps != c.norm_eps for n in norms) or any(n.groups != c.norm_groups for n in norms[:1 if b.mlp_norm is None else 2]):
+            raise NotImplementedError("the layer-list engine takes one epsilon and one number of norm groups for all layers")
+        own = a.source is None
+        out = cls.pack_talking(a.q_proj.weight, a.k_proj.weight if own else None, a.v_proj.weight if own else None, a.o_proj.weight, b.attn_norm.weight, heads=a.num_heads,
+                               kv_heads=a.num_kv_heads, dim=a.head_dim, vdim=a.v_head_dim, window=a.window, chunked=a.chunked, scale=a.scale,
+                               biases=tuple(p.bias for p in ((a.q_proj, a.k_proj, a.v_proj) if own else (a.q_proj,))), o_bias=a.o_proj.bias, q_norm=a.q_norm.weight,
+                               k_norm=a.k_norm.weight if own else None, rot_freq=a.rot_freq, talk=a.talk, sink=a.sink, kv_from=a.kv_from)
+        h, m, width = b.attn_hyper, b.mlp, a.q_proj.weight.shape[1]
+        out["hyper1"] = cls.pack_hyper(h.read, h.write, h.mix)
+        if m is None:
+            return out
+        h = b.mlp_hyper
+        out.update(hyper2=cls.pack_hyper(h.read, h.write, h.mix), norm2=_row(b.mlp_norm.weight, _up64(width)))
+        if isinstance(m, TableExperts):
+            shared = None if m.shared_up is None else (m.shared_up.weight, m.shared_down.weight, m.shared_gate.weight)
+            return cls.add_table_experts(out, width, m.table, m.up, m.down, shared)
+        if m.activation != "poly_norm" or m.act_eps != c.norm_eps:
+            raise NotImplementedError("hyper-connected layers have polynomial-norm feed-forwards or experts chosen by a table")
+        return cls.add_poly_mlp(out, width, m.fc1.weight, m.fc2.weight, m.act_params)
+
     @staticmethod
     def add_experts(layer: dict, width: int, router: GPUArray, correction: GPUArray, gate_up: GPUArray, down: GPUArray, *, top: int, groups: int = 0, keep: int = 0,
                     scale: float = 1.0) -> dict:
@@ -606,8 +695,10 @@ class StackEngine(Engine):
 
     @classmethod
     def _pack_block(cls, b, c) -> dict:
-        from pygpukit_amd.llm.layers import GatedRecurrence, GatedWindowAttention, LatentAttention, ParallelBlock
+        from pygpukit_amd.llm.layers import GatedRecurrence, GatedWindowAttention, HyperBlock, LatentAttention, ParallelBlock
 
+        if isinstance(b, HyperBlock):
+            return cls._pack_hyper_block(b, c)
         if isinstance(b, ParallelBlock):
             if b.attn_norm.eps != c.norm_eps or b.attn_norm.norm_type != c.norm_type:
                 raise NotImplementedError("the layer-list engine takes one kind of norm and one epsilon for all layers")
@@ -662,8 +753,14 @@ class StackEngine(Engine):
 
     @staticmethod
     def _pack_more(model, width: int) -> dict:
-        """What parallel layers and a loop add to the engine's configuration."""
-        from pygpukit_amd.llm.layers import ParallelBlock
+        """What parallel or hyper-connected layers and a loop add to the engine's configuration."""
+        from pygpukit_amd.llm.layers import HyperBlock, ParallelBlock
+
+        c, hyper = model.config, [isinstance(b, HyperBlock) for b in model.blocks]
+        if any(hyper):
+            if not all(hyper):
+                raise NotImplementedError("the layer-list engine takes hyper-connected layers or others, not both")
+            return dict(block=_hip.BLOCK_HYPER, streams=c.streams, norm_groups=c.norm_groups, logit_cap=c.logit_softcap)
 
         parallel = [isinstance(b, ParallelBlock) for b in model.blocks]
         if not any(parallel):

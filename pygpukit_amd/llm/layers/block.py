@@ -1,26 +1,27 @@
 """Transformer block (reference: src/pygpukit/llm/layers/block.py:18-57): pre-norm attention and MLP with
 residual adds.  Layer-list models add a norm on each sublayer's output (with or without one on its input), a factor on its
-contribution and layers without MLP, or run mixer and experts side by side (ParallelBlock)."""
+contribution and layers without MLP, run mixer and experts side by side (ParallelBlock), or keep several residual streams (HyperBlock)."""
 
 from __future__ import annotations
 
 from pygpukit_amd.core.array import GPUArray
 from pygpukit_amd.core.dtypes import float16, float32
 from pygpukit_amd.core.factory import from_numpy
-from pygpukit_amd.ops.basic import add, add_inplace, bias_add_inplace, cast_bf16_to_f32, cast_f16_to_f32, cast_f32_to_bf16, cast_f32_to_f16
+from pygpukit_amd.ops.basic import add, add_inplace, bias_add_inplace, cast_bf16_to_f32, cast_f16_to_f32, cast_f32_to_bf16, cast_f32_to_f16, hyper_read, hyper_write
 
 from .attention import Attention
 from .delta import ChannelDelta
-from .experts import MixtureOfExperts
+from .experts import MixtureOfExperts, TableExperts
 from .latent_attention import LatentAttention
 from .linear import LinearBF16
 from .mlp import MLP
 from .norm import Norm
 from .recurrence import GatedRecurrence
 from .state_space import StateSpace
+from .talking_attention import TalkingAttention
 from .window_attention import GatedWindowAttention
 
-Mixer = Attention | LatentAttention | GatedWindowAttention | GatedRecurrence | ChannelDelta | StateSpace
+Mixer = Attention | LatentAttention | GatedWindowAttention | GatedRecurrence | ChannelDelta | StateSpace | TalkingAttention
 
 
 def _narrow(x: GPUArray, dtype) -> GPUArray:
@@ -91,6 +92,50 @@ class ParallelBlock:
         return self._add(x, h, self.attn.forward_fixed_cache_batch(h, position, context_len))
 
 
+class HyperConnection:
+    """How a sublayer is tied to the residual streams: reads sum_a read[a] x_a, writes x_b <- sum_a mix[a, b] x_a + write[b] y (float32)."""
+
+    def __init__(self, read: GPUArray, write: GPUArray, mix: GPUArray):
+        n = read.size
+        if read.shape != (n,) or write.shape != (n,) or mix.shape != (n, n) or any(w.dtype != float32 for w in (read, write, mix)):
+            raise ValueError(f"HyperConnection: {read.shape}, {write.shape}, {mix.shape}")
+        self.read, self.write, self.mix = read, write, mix
+
+
+class HyperBlock:
+    """Mixer, then feed-forward (an MLP, experts chosen by token, or none), each with a norm of its own and a HyperConnection, on float32
+    streams [n, streams, hidden]."""
+
+    residual_mult = 1.0
+
+    def __init__(self, attn_norm: Norm, attn: Mixer, attn_hyper: HyperConnection, mlp_norm: Norm | None, mlp: MLP | TableExperts | None, mlp_hyper: HyperConnection | None):
+        self.attn_norm, self.attn, self.attn_hyper, self.mlp_norm, self.mlp, self.mlp_hyper = attn_norm, attn, attn_hyper, mlp_norm, mlp, mlp_hyper
+
+    @property
+    def needs_tokens(self) -> bool:
+        return getattr(self.mlp, "needs_tokens", False)
+
+    @staticmethod
+    def _write(x: GPUArray, y: GPUArray, h: HyperConnection) -> GPUArray:
+        return hyper_write(x, y, h.write, h.mix)
+
+    def _feed_forward(self, x: GPUArray, tokens: GPUArray | None) -> GPUArray:
+        if self.mlp is None:
+            return x
+        h = self.mlp_norm(hyper_read(x, self.mlp_hyper.read))
+        return self._write(x, self.mlp(h, tokens) if self.needs_tokens else self.mlp(h), self.mlp_hyper)
+
+    def __call__(self, x: GPUArray, position_ids: list[int] | None = None, past_kv: tuple | None = None, use_cache: bool = False,
+                 source_kv: tuple | None = None, tokens: GPUArray | None = None) -> tuple[GPUArray, tuple | None]:
+        extra = {} if source_kv is None else {"source_kv": source_kv}
+        y, present_kv = self.attn(self.attn_norm(hyper_read(x, self.attn_hyper.read)), position_ids, past_kv, use_cache, **extra)
+        return self._feed_forward(self._write(x, y, self.attn_hyper), tokens), present_kv
+
+    def forward_fixed_cache(self, x: GPUArray, position: int, context_len: int, tokens: GPUArray | None = None) -> GPUArray:
+        y = self.attn.forward_fixed_cache_batch(self.attn_norm(hyper_read(x, self.attn_hyper.read)), position, context_len)
+        return self._feed_forward(self._write(x, y, self.attn_hyper), tokens)
+
+
 class LoopInput:
     """What a pass of a looped stretch starts with: x <- W_x x + W_e e + step[pass], e the embedding rows."""
 
@@ -113,4 +158,4 @@ class LoopInput:
         return y
 
 
-__all__ = ["TransformerBlock", "ParallelBlock", "LoopInput"]
+__all__ = ["TransformerBlock", "ParallelBlock", "HyperBlock", "HyperConnection", "LoopInput"]

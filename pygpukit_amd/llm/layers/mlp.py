@@ -1,4 +1,4 @@
-"""MLP layer (reference: src/pygpukit/llm/layers/mlp.py:25-98): GELU (fc1 -> gelu -> fc2), xIELU in its place, or SwiGLU
+"""MLP layer (reference: src/pygpukit/llm/layers/mlp.py:25-98): GELU (fc1 -> gelu -> fc2), xIELU or PolyNorm in its place, or SwiGLU
 (silu(gate) * up -> down).  With raw bf16 weights gate and up are fused into ONE [2I, H] weight
 (mlp.py:84-86); here gate_proj / up_proj are zero-copy row views of that fused weight, so the bytes exist
 once, and the forward is one projection + one packed GLU kernel + the down projection."""
@@ -8,7 +8,7 @@ from __future__ import annotations
 from typing import TYPE_CHECKING
 
 from pygpukit_amd.core.array import GPUArray
-from pygpukit_amd.ops.basic import concat_axis0, gelu, glu_packed, swiglu, xielu
+from pygpukit_amd.ops.basic import concat_axis0, gelu, glu_packed, poly_norm, swiglu, xielu
 
 from .linear import LinearBF16, LinearFP8
 
@@ -25,17 +25,17 @@ def _wrap(proj, bias=None):
 class MLP:
     def __init__(self, config: "TransformerConfig", fc1_weight=None, fc1_bias: GPUArray | None = None, fc2_weight=None,
                  fc2_bias: GPUArray | None = None, gate_proj=None, up_proj=None, down_proj=None,
-                 act_params: tuple[float, float] | None = None):
-        """act_params: xIELU's two factors (of z^2 and of exp(z) - 1 - z)."""
+                 act_params: tuple[float, float] | GPUArray | None = None, act_eps: float = 1e-5):
+        """act_params: xIELU's two factors (of z^2 and of exp(z) - 1 - z), or PolyNorm's four numbers (float32; act_eps in its norms)."""
         self.config = config
         self.activation = config.activation
         self.gate_up_proj: LinearBF16 | None = None
-        if config.activation in ("gelu", "xielu"):
+        if config.activation in ("gelu", "xielu", "poly_norm"):
             if fc1_weight is None or fc2_weight is None:
                 raise ValueError(f"{config.activation} MLP requires fc1_weight and fc2_weight")
-            if (act_params is not None) != (config.activation == "xielu"):
-                raise ValueError("act_params are xIELU's")
-            self.act_params = act_params
+            if (act_params is not None) != (config.activation != "gelu"):
+                raise ValueError("act_params are xIELU's or PolyNorm's")
+            self.act_params, self.act_eps = act_params, act_eps
             self.fc1, self.fc2 = _wrap(fc1_weight, fc1_bias), _wrap(fc2_weight, fc2_bias)
             return
         if gate_proj is None or up_proj is None or down_proj is None:
@@ -59,6 +59,9 @@ class MLP:
         if self.activation == "xielu":
             h = self.fc1(x)
             return self.fc2(xielu(h, *self.act_params, out=h))
+        if self.activation == "poly_norm":
+            h = self.fc1(x)
+            return self.fc2(poly_norm(h, self.act_params, self.act_eps, out=h))
         if self.gate_up_proj is not None:
             act = glu_packed(self.gate_up_proj(x), self.intermediate_size)
         else:

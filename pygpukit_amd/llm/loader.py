@@ -17,10 +17,10 @@ from pygpukit_amd import _hip
 from pygpukit_amd.core.array import GPUArray
 from pygpukit_amd.core.dtypes import bfloat16, float16, float32, uint8
 from pygpukit_amd.core.factory import from_numpy
-from pygpukit_amd.llm.config import (GPT2_SPEC, LLAMA_SPEC, MALASUN_SPEC, QWEN3_SPEC, RATASUN_SPEC, TOTOLORN_SPEC, LayerConfig, ModelSpec, TransformerConfig,
+from pygpukit_amd.llm.config import (FETEZEN_SPEC, GPT2_SPEC, LLAMA_SPEC, MALASUN_SPEC, QWEN3_SPEC, RATASUN_SPEC, TOTOLORN_SPEC, LayerConfig, ModelSpec, TransformerConfig,
                                      detect_model_spec, distance_slopes, layer_list_config)
-from pygpukit_amd.llm.layers import (MLP, Attention, ChannelDelta, GatedRecurrence, GatedWindowAttention, LatentAttention, LoopInput, MixtureOfExperts, Norm,
-                                     ParallelBlock, StateSpace, TransformerBlock)
+from pygpukit_amd.llm.layers import (MLP, Attention, ChannelDelta, GatedRecurrence, GatedWindowAttention, HyperBlock, HyperConnection, LatentAttention, LoopInput,
+                                     MixtureOfExperts, Norm, ParallelBlock, StateSpace, TableExperts, TalkingAttention, TransformerBlock)
 from pygpukit_amd.llm.layers.linear import LinearBF16, LinearFP8
 from pygpukit_amd.llm.models.causal import CausalTransformerModel
 from pygpukit_amd.llm.safetensors import Dtype, load_safetensors
@@ -224,7 +224,7 @@ def _load_layer_list(st, spec: ModelSpec, config: dict, dtype, load_tensor, try_
 
     def norm(name: str, width: int, offset: float, scalar: bool = False, kind: str = "rmsnorm", mult: float = 1.0) -> Norm:
         w = np.repeat(fp32(name, 1), width) if scalar else fp32(name, width)
-        return Norm(from_numpy((w + np.float32(offset)) * np.float32(mult)), None, kind, cfg.norm_eps, stream_dtype=dtype)
+        return Norm(from_numpy((w + np.float32(offset)) * np.float32(mult)), None, kind, cfg.norm_eps, stream_dtype=dtype, groups=cfg.norm_groups if width == cfg.hidden_size and spec.hyper else 1)
 
     H, off, one = cfg.hidden_size, spec.norm_weight_offset, spec.norm_scalar
     blocks: list[TransformerBlock] = []
@@ -255,6 +255,24 @@ def _load_layer_list(st, spec: ModelSpec, config: dict, dtype, load_tensor, try_
             num_kv_heads=lc.num_kv_heads, head_dim=lc.head_dim, v_head_dim=lc.v_head_dim, scale=lc.scale, window=lc.window, q_norm=norm(nm(spec.q_norm), q, 0.0),
             k_norm=norm(nm(spec.k_norm), k, 0.0) if own else None, q_conv=conv(spec.q_conv, q), k_conv=conv(spec.k_conv, k) if own else None,
             v_conv=conv(spec.v_conv, v) if own else None, slopes=from_numpy(np.asarray(distance_slopes(lc.num_heads), np.float32)),
+            source=None if own else blocks[lc.kv_from].attn, kv_from=lc.kv_from)
+
+    def talking_mixer(lc: LayerConfig, nm) -> TalkingAttention:
+        q, k, v = lc.num_heads * lc.head_dim, lc.num_kv_heads * lc.head_dim, lc.num_kv_heads * lc.v_head_dim
+        own, rot = lc.kv_from is None, lc.rot_dim
+        freq = from_numpy((lc.rot_base ** (-2.0 * np.arange(rot // 2) / rot)).astype(np.float32)) if rot else None
+
+        def proj(weight: str, bias: str, rows: int, cols: int = H) -> LinearBF16:
+            return LinearBF16(tensor(nm(weight), (rows, cols)), tensor(nm(bias), (rows,)))
+
+        def head_norm(name: str) -> Norm:
+            return Norm(from_numpy(fp32(nm(name), lc.head_dim)), None, "rmsnorm", cfg.norm_eps, stream_dtype=dtype)
+
+        return TalkingAttention(
+            proj(spec.q_proj, spec.q_bias, q), proj(spec.k_proj, spec.k_bias, k) if own else None, proj(spec.v_proj, spec.v_bias, v) if own else None,
+            proj(spec.o_proj, spec.o_bias, H, lc.num_heads * lc.v_head_dim), num_heads=lc.num_heads, num_kv_heads=lc.num_kv_heads, head_dim=lc.head_dim,
+            v_head_dim=lc.v_head_dim, scale=lc.scale, window=lc.window, chunked=lc.chunked, q_norm=head_norm(spec.q_norm), k_norm=head_norm(spec.k_norm) if own else None,
+            rot_freq=freq, talk=from_numpy(fp32(nm(spec.talk), lc.num_heads ** 2).reshape(lc.num_heads, lc.num_heads)), sink=from_numpy(fp32(nm(spec.sink), lc.num_heads)),
             source=None if own else blocks[lc.kv_from].attn, kv_from=lc.kv_from)
 
     def recurrent_mixer(lc: LayerConfig, nm) -> GatedRecurrence:
@@ -306,7 +324,39 @@ def _load_layer_list(st, spec: ModelSpec, config: dict, dtype, load_tensor, try_
         return MixtureOfExperts(tensor(nm(spec.router), (e.count, H)), from_numpy(fp32(nm(spec.router_correction), e.count)), gate_up, down, top=e.top, groups=e.groups,
                                 keep=e.keep, scale=e.scale)
 
-    mixers = {"latent_attention": (latent_mixer, spec.kv_down_proj), "attention": (attention_mixer, spec.out_gate), "hgrn2": (recurrent_mixer, spec.forget_proj),
+    def table_mlp(i: int, lc: LayerConfig, nm) -> TableExperts:
+        e, I = lc.experts, lc.intermediate_size
+        name = nm(spec.expert_table)
+        if name not in st or tuple(st.tensor_info(name).shape) != (cfg.vocab_size, e.top) or st.tensor_info(name).dtype not in (Dtype.Int32, Dtype.Int64):
+            raise ValueError(f"{name}: missing, or not integers [{cfg.vocab_size}, {e.top}]")
+        table = np.ascontiguousarray(st.tensor_numpy(name))
+        if table.min() < 0 or table.max() >= e.count:
+            raise ValueError(f"{name}: names experts outside [0, {e.count})")
+        up, down = GPUArray((e.count, I, H), dtype), GPUArray((e.count, H, I), dtype)
+        for k in range(e.count):
+            for out, pattern, shape in ((up, spec.expert_up_proj, (I, H)), (down, spec.expert_down_proj, (H, I))):
+                w = tensor(nm(pattern, expert=k), shape)
+                _hip.call("pgk_memcpy_d2d", C.c_void_p(out.data_ptr() + k * w.nbytes), w._p, w.nbytes, None)
+        shared = {}
+        if e.shared_size is not None:
+            shared = dict(shared_up=tensor(nm(spec.shared_up_proj), (e.shared_size, H)), shared_down=tensor(nm(spec.shared_down_proj), (H, e.shared_size)),
+                          shared_gate=tensor(nm(spec.shared_gate), (1, H)))
+        return TableExperts(from_numpy(table.astype(np.int32)), up, down, **shared)
+
+    def hyper(nm, sublayer: int) -> HyperConnection:
+        p, n = nm(spec.hyper, sublayer=sublayer), cfg.streams
+        return HyperConnection(from_numpy(fp32(p + "in", n)), from_numpy(fp32(p + "out", n)), from_numpy(fp32(p + "mix", n * n).reshape(n, n)))
+
+    def hyper_block(i: int, lc: LayerConfig, nm, attn) -> HyperBlock:
+        mlp = None
+        if lc.experts is not None:
+            mlp = table_mlp(i, lc, nm)
+        elif lc.intermediate_size is not None:
+            I = lc.intermediate_size
+            mlp = MLP(cfg, fc1_weight=tensor(nm(spec.fc1), (I, H)), fc2_weight=tensor(nm(spec.fc2), (H, I)), act_params=from_numpy(fp32(nm(spec.act_params), 4)), act_eps=cfg.norm_eps)
+        return HyperBlock(norm(nm(spec.attn_norm), H, off), attn, hyper(nm, 1), None if mlp is None else norm(nm(spec.mlp_norm), H, off), mlp, None if mlp is None else hyper(nm, 2))
+
+    mixers = {"latent_attention": (latent_mixer, spec.kv_down_proj), "attention": (talking_mixer, spec.talk) if spec.talk else (attention_mixer, spec.out_gate), "hgrn2": (recurrent_mixer, spec.forget_proj),
               "channel_delta": (delta_mixer, spec.decay_down), "mamba2": (state_space_mixer, spec.in_proj)}
     for i, lc in enumerate(cfg.layers):
         nm = lambda pattern, **kw: pattern.format(layer=i, **kw)  # noqa: E731, B023
@@ -315,6 +365,9 @@ def _load_layer_list(st, spec: ModelSpec, config: dict, dtype, load_tensor, try_
             raise ValueError(f"layer {i}: {spec.name} models have no {lc.mixer} layers")
         mlp = mlp_norm = post_mlp = None
         attn = make(lc, nm)
+        if spec.hyper:
+            blocks.append(hyper_block(i, lc, nm, attn))
+            continue
         if (lc.experts is not None) != (spec.is_moe and lc.intermediate_size is not None):
             raise ValueError(f"layer {i}: {spec.name} models have {'no dense feed-forwards' if spec.is_moe else 'no experts'}")
         if spec.parallel:
@@ -378,9 +431,13 @@ def load_malasun_from_safetensors(model_path: str, dtype: str = "bfloat16") -> C
     return load_model_from_safetensors(model_path, dtype=dtype, spec=MALASUN_SPEC)
 
 
+def load_fetezen_from_safetensors(model_path: str, dtype: str = "bfloat16") -> CausalTransformerModel:
+    return load_model_from_safetensors(model_path, dtype=dtype, spec=FETEZEN_SPEC)
+
+
 def load_ratasun_from_safetensors(model_path: str, dtype: str = "bfloat16") -> CausalTransformerModel:
     return load_model_from_safetensors(model_path, dtype=dtype, spec=RATASUN_SPEC)
 
 
-__all__ = ["load_ratasun_from_safetensors", "load_malasun_from_safetensors", "load_totolorn_from_safetensors", "load_model_from_safetensors", "load_gpt2_from_safetensors", "load_llama_from_safetensors", "load_qwen3_from_safetensors",
+__all__ = ["load_fetezen_from_safetensors", "load_ratasun_from_safetensors", "load_malasun_from_safetensors", "load_totolorn_from_safetensors", "load_model_from_safetensors", "load_gpt2_from_safetensors", "load_llama_from_safetensors", "load_qwen3_from_safetensors",
            "FP8QuantConfig"]

@@ -1,3 +1,3 @@
-from .causal import CausalTransformerModel, GPT2Model, LlamaModel, QwenModel, TotolornModel, MalasunModel, RatasunModel
+from .causal import CausalTransformerModel, GPT2Model, LlamaModel, QwenModel, TotolornModel, MalasunModel, RatasunModel, FetezenModel
 
-__all__ = ["CausalTransformerModel", "GPT2Model", "LlamaModel", "QwenModel", "TotolornModel", "MalasunModel", "RatasunModel"]
+__all__ = ["CausalTransformerModel", "GPT2Model", "LlamaModel", "QwenModel", "TotolornModel", "MalasunModel", "RatasunModel", "FetezenModel"]

@@ -20,7 +20,7 @@ from pygpukit_amd.llm.config import ModelSpec, TransformerConfig
 from pygpukit_amd.llm.layers import MLP, Attention, LoopInput, Norm, TransformerBlock
 from pygpukit_amd.llm.sampling import sample_token
 from pygpukit_amd.ops.basic import (add_inplace, cast_bf16_to_f32, embedding_lookup_batch, glu_packed, matmul_nt,
-                                   rmsnorm, sample_token_gpu)
+                                   hyper_read, repeat_interleave_axis1, rmsnorm, sample_token_gpu, soft_cap)
 
 
 def _to_float32_logits(logits_np: np.ndarray) -> np.ndarray:
@@ -73,6 +73,23 @@ class CausalTransformerModel:
             add_inplace(hidden, rows(self.position_embed, pos))
         return hidden
 
+    def _enter(self, hidden: GPUArray) -> GPUArray:
+        """What the first block reads: the embedded rows, or as many equal streams of them as the blocks connect."""
+        if self.config.layers is None or self.spec is None or self.spec.hyper is None:
+            return hidden
+        n, w = hidden.shape
+        return repeat_interleave_axis1(hidden.view((n, 1, w)), self.config.streams)
+
+    def _leave(self, hidden: GPUArray) -> GPUArray:
+        return self.final_norm(hyper_read(hidden) if hidden.ndim == 3 else hidden)
+
+    def _tokens_for(self, block, input_ids) -> dict:
+        return {"tokens": from_numpy(np.asarray(input_ids, np.int32))} if getattr(block, "needs_tokens", False) else {}
+
+    def cap_logits(self, logits: GPUArray) -> GPUArray:
+        """The model's soft cap, in place."""
+        return logits if self.config.logit_softcap is None else soft_cap(logits, self.config.logit_softcap, out=logits)
+
     def __call__(self, input_ids: list[int], position_ids: list[int] | None = None,
                  past_key_values: list[tuple | None] | None = None, use_cache: bool = False):
         seq_len = len(input_ids)
@@ -81,7 +98,8 @@ class CausalTransformerModel:
             if past_key_values is not None:
                 past_len = next((p[0].shape[0] for (i, _), p in zip(self._runs(), past_key_values) if p is not None and getattr(self.blocks[i].attn, "cache_rows", True)), 0)
             position_ids = list(range(past_len, past_len + seq_len))
-        hidden = embedded = self._embed(input_ids, position_ids)
+        embedded = self._embed(input_ids, position_ids)
+        hidden = self._enter(embedded)
         present = []
         sources = {getattr(b.attn, "kv_from", None) for b in self.blocks}
         for run, (i, start) in enumerate(self._runs()):
@@ -90,9 +108,9 @@ class CausalTransformerModel:
                 hidden = self.loop(hidden, embedded, start)
             past_kv = past_key_values[run] if past_key_values else None
             src = getattr(block.attn, "kv_from", None)
-            hidden, kv = block(hidden, position_ids, past_kv, use_cache or i in sources, None if src is None else present[src])
+            hidden, kv = block(hidden, position_ids, past_kv, use_cache or i in sources, None if src is None else present[src], **self._tokens_for(block, input_ids))
             present.append(kv)
-        hidden = self.final_norm(hidden)
+        hidden = self._leave(hidden)
         return (hidden, present) if use_cache else (hidden, None)
 
     forward = __call__  # the "QwenModel.forward()" spelling of the docs
@@ -100,7 +118,7 @@ class CausalTransformerModel:
     def get_logits(self, hidden: GPUArray) -> GPUArray:
         """[seq, hidden] -> [seq, vocab]: hidden @ lm_head^T (tied to embed_tokens when lm_head is None)."""
         head = self._lm_head if self._lm_head is not None else self.embed_tokens
-        return matmul_nt(hidden, head)
+        return self.cap_logits(matmul_nt(hidden, head))
 
     # ------------------------------------------------------------------ generation
     def _sample(self, logits: GPUArray, temperature, top_k, top_p, gpu_sampling) -> int:
@@ -175,10 +193,10 @@ class CausalTransformerModel:
 
     def _decode_step_fixed_cache_batch(self, token_ids: list[int], start_position: int, context_len: int) -> GPUArray:
         """M consecutive tokens of one sequence (speculative verify, causal.py:842-891) -> hidden [M, H]."""
-        hidden = self._embed(token_ids, list(range(start_position, start_position + len(token_ids))))
+        hidden = self._enter(self._embed(token_ids, list(range(start_position, start_position + len(token_ids)))))
         for block in self.blocks:
-            hidden = block.forward_fixed_cache(hidden, start_position, context_len)
-        return self.final_norm(hidden)
+            hidden = block.forward_fixed_cache(hidden, start_position, context_len, **self._tokens_for(block, token_ids))
+        return self._leave(hidden)
 
     def prefill_fixed_cache(self, input_ids: list[int]) -> GPUArray:
         """Prefill that leaves K/V in the fixed caches (the chat flow's prefill + kv_cache_prefill_gqa,
@@ -239,5 +257,6 @@ QwenModel = CausalTransformerModel
 TotolornModel = CausalTransformerModel
 MalasunModel = CausalTransformerModel
 RatasunModel = CausalTransformerModel
+FetezenModel = CausalTransformerModel
 
-__all__ = ["CausalTransformerModel", "GPT2Model", "LlamaModel", "QwenModel", "TotolornModel", "MalasunModel", "RatasunModel"]
+__all__ = ["CausalTransformerModel", "GPT2Model", "LlamaModel", "QwenModel", "TotolornModel", "MalasunModel", "RatasunModel", "FetezenModel"]

@@ -9,7 +9,8 @@ from pygpukit_amd.ops.matmul import (batched_matmul, gemm_w8a16_init_lut, gemv_b
 from pygpukit_amd.ops.matmul.fp8 import *  # noqa: F401,F403
 from pygpukit_amd.ops.nn import (bias_add_inplace, conv_silu, delta_rule, gated_recurrence, geglu, gelu, glu_packed, latent_rows, layernorm, layernorm_f32, mixture_of_experts, relu2, rmsnorm, rmsnorm_residual, rope_inplace,
                                 rope_inplace_f32table, sdpa_causal, sdpa_causal_fixed_cache, sdpa_causal_fixed_cache_ptr,
-                                sdpa_causal_strided, rotate_pairs, state_space, window_attention, head_gate, rmsnorm_f32, rmsnorm_add_f32, short_conv, sigmoid, sigmoid_mul, silu, slice_rows_range_ptr, split_qkv_batch, swiglu, tanh, xielu)
+                                sdpa_causal_strided, rotate_pairs, state_space, window_attention, head_gate, rmsnorm_f32, rmsnorm_add_f32, short_conv, sigmoid, sigmoid_mul, silu, slice_rows_range_ptr, split_qkv_batch, swiglu, tanh, xielu,
+                                gelu_erf, group_norm_f32, head_norm_rope, hyper_read, hyper_write, poly_norm, soft_cap, table_experts, talk_attention)
 from pygpukit_amd.ops.reduction import argmax, argmax_int, argmax_rows, max, mean, min, softmax, sum, sum_axis
 from pygpukit_amd.ops.unary import abs, cos, exp, log, neg, relu, rsqrt, sin, sqrt
 from pygpukit_amd.ops.sampling import (sample_greedy, sample_multinomial, sample_token_gpu, sample_topk, sample_topk_to_buf_ptr,

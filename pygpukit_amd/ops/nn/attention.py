@@ -7,7 +7,7 @@ import ctypes as C
 
 from pygpukit_amd import _hip
 from pygpukit_amd.core.array import GPUArray
-from pygpukit_amd.core.dtypes import float32, int32
+from pygpukit_amd.core.dtypes import bfloat16, float32, int32
 from pygpukit_amd.ops._common import call, check_out, validate_float
 
 _ws_cache: dict[tuple[int, int, int], GPUArray] = {}
@@ -102,6 +102,38 @@ def window_attention(q: GPUArray, k: GPUArray, v: GPUArray, scale: float, window
     o = check_out(out, (q_len, hq, dv), q.dtype, "window_attention")
     call("pgk_window_attention", q._p, k._p, v._p, o._p, hq, hkv, q_len, kv_len, dk, dv, float(scale), min(int(window), 2**30),
          gate._p if gate is not None else None, hq * dv if each else hq, int(each), slopes._p if slopes is not None else None, q.dtype.code, None)
+    return o
+
+
+def head_norm_rope(x: GPUArray, norm: GPUArray | None, freq: GPUArray | None, first: int, eps: float = 1e-5) -> GPUArray:
+    """x [n, heads, dim], row i at position first + i: RMS norm over every head (norm float32 [dim] or None), then columns i and
+    i + rot / 2 turned by position * freq[i] (freq float32 [rot / 2]); columns from rot on pass."""
+    validate_float(x, "head_norm_rope")
+    rot = 0 if freq is None else 2 * freq.size
+    if x.ndim != 3 or rot > x.shape[2] or first < 0 or (norm is not None and (norm.shape != (x.shape[2],) or norm.dtype != float32)) or (freq is not None and freq.dtype != float32):
+        raise ValueError(f"head_norm_rope: x {x.shape}, {rot} turned columns")
+    o = GPUArray(x.shape, x.dtype)
+    call("pgk_head_norm_rope", x._p, norm._p if norm is not None else None, freq._p if freq is not None else None, o._p, *x.shape, rot, first, float(eps), x.dtype.code, None)
+    return o
+
+
+def talk_attention(q: GPUArray, k: GPUArray, v: GPUArray, scale: float, window: int, *, chunked: bool = False, first: int = 0, talk: GPUArray | None = None,
+                   sink: GPUArray | None = None, out: GPUArray | None = None) -> GPUArray:
+    """q [q_len, Hq, dk], k [kv_len, Hkv, dk], v [kv_len, Hkv, dv] -> [q_len, Hq, dv]: row t of k is position first + t, the queries are the
+    last q_len positions.  A query sees the `window` positions that end with its own, or (chunked) those of its own chunk of
+    `window` positions, counted from position 0.  talk float32 [Hq, Hq] mixes the heads' scaled scores; exp(sink), float32 [Hq],
+    stands in the softmax's denominator."""
+    if q.ndim != 3 or k.ndim != 3 or v.ndim != 3 or q.dtype not in (float32, bfloat16) or k.dtype != q.dtype or v.dtype != q.dtype:
+        raise ValueError("talk_attention expects q, k, v as [seq, heads, width], float32 or bfloat16")
+    (q_len, hq, dk), (kv_len, hkv, dk2), (kv2, hkv2, dv) = q.shape, k.shape, v.shape
+    if dk != dk2 or kv_len != kv2 or hkv != hkv2 or hq % hkv or kv_len < q_len or window < 1 or first < 0:
+        raise ValueError(f"talk_attention: shapes {q.shape}, {k.shape}, {v.shape}, window {window}, first position {first}")
+    for a, shape in ((talk, (hq, hq)), (sink, (hq,))):
+        if a is not None and (a.shape != shape or a.dtype != float32):
+            raise ValueError(f"talk_attention: talk and sink are float32 [Hq, Hq] and [Hq], got {a.shape}")
+    o = check_out(out, (q_len, hq, dv), q.dtype, "talk_attention")
+    call("pgk_talk_attention", q._p, k._p, v._p, talk._p if talk is not None else None, sink._p if sink is not None else None, o._p, hq, hkv, q_len, kv_len, int(first), dk, dv,
+         float(scale), min(int(window), 2**30), int(chunked), q.dtype.code, None)
     return o
 
 

@@ -35,6 +35,16 @@ def rmsnorm_f32(input: GPUArray, weight: GPUArray, eps: float = 1e-5, *, dtype=f
     return o
 
 
+def group_norm_f32(input: GPUArray, weight: GPUArray, groups: int, eps: float = 1e-5, *, dtype=float32, out: GPUArray | None = None) -> GPUArray:
+    """RMS norm of an fp32 stream in `groups` equal consecutive parts, each over its own root mean square, with an fp32 weight."""
+    _check(input, weight, "group_norm_f32")
+    if input.dtype != float32 or groups < 1 or input.shape[1] % groups:
+        raise ValueError(f"group_norm_f32: float32 rows of {input.shape[1]} in {groups} groups")
+    o = check_out(out, input.shape, dtype, "group_norm_f32")
+    call("pgk_group_norm_f32", input._p, weight._p, o._p, input.shape[0], input.shape[1], int(groups), eps, o.dtype.code, None)
+    return o
+
+
 def layernorm_f32(input: GPUArray, weight: GPUArray, eps: float = 1e-5, *, dtype=float32, out: GPUArray | None = None) -> GPUArray:
     """Layer norm (no bias) of an fp32 stream with an fp32 weight; the result leaves in `dtype`."""
     _check(input, weight, "layernorm_f32")

@@ -83,7 +83,7 @@ def test_config_and_specs():
     assert d.head_dim == 64 and d.num_kv_heads == 12 and d.intermediate_size == 3072
     assert QWEN3_SPEC.use_qk_norm and QWEN3_SPEC.default_norm_eps == 1e-6 and QWEN3_SPEC.q_norm.format(layer=3).endswith("layers.3.self_attn.q_norm.weight")
     assert GPT2_SPEC.norm_type == "layernorm" and GPT2_SPEC.activation == "gelu" and not GPT2_SPEC.use_rope and GPT2_SPEC.qkv_combined
-    assert set(MODEL_SPECS) == {"gpt2", "llama", "qwen3", "qwen2", "totolorn", "malasun", "ratasun"}
+    assert set(MODEL_SPECS) == {"gpt2", "llama", "qwen3", "qwen2", "totolorn", "malasun", "ratasun", "fetezen"}
     assert detect_model_spec(["model.embed_tokens.weight", "model.layers.0.self_attn.q_norm.weight"]) is QWEN3_SPEC
     assert detect_model_spec(["model.embed_tokens.weight", "model.layers.0.self_attn.q_proj.bias"]) is QWEN2_SPEC
     assert detect_model_spec(["model.embed_tokens.weight"]) is LLAMA_SPEC
