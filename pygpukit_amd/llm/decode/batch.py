@@ -33,7 +33,7 @@ class DecodeBatch(DecodeStrategy):
         hidden = model._decode_step_fixed_cache_batch(list(token_ids), start_position, context_len)
         head = model._lm_head if model._lm_head is not None else model.embed_tokens
         out = buffers.logits_batch.slice_rows(len(token_ids)) if buffers is not None and buffers.logits_batch is not None else None
-        return matmul_nt(hidden, head, out=out)
+        return model.cap_logits(matmul_nt(hidden, head, out=out))
 
     def step_graph(self, token_ids: list[int], start_position: int, context_len: int):
         """batch.py:308-363: the verify step for exactly `batch_size` tokens after init_graph() -> logits

@@ -21,7 +21,8 @@ def save(folder, cfg, W):
 
     with open(os.path.join(folder, "config.json"), "w", encoding="utf-8") as f:
         json.dump(cfg, f)
-    save_safetensors(os.path.join(folder, "model.safetensors"), {k: (O.f32_to_bf16_bits(v).reshape(v.shape), "BF16") for k, v in W.items()})
+    save_safetensors(os.path.join(folder, "model.safetensors"), {k: (np.asarray(v, np.int32), "I32") if np.issubdtype(v.dtype, np.integer) else
+                                                                 (O.f32_to_bf16_bits(v).reshape(v.shape), "BF16") for k, v in W.items()})
     return str(folder)
 
 
