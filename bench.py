@@ -188,10 +188,60 @@ def ratasun_model(z: dict, vocab: int, embed, head, draw, feed_forward):
     return CausalTransformerModel(cfg, embed, [block(i) for i in range(L)], norm(W), head, None, RATASUN_SPEC)
 
 
+# Fetezen at those sizes: chunks as long as the others' windows; every other layer dense, the others experts of which each token uses, with the
+# shared one, as much feed-forward width as the dense layers have
+FETEZEN_EXPERTS = {"experts": 16, "top": 3, "split": 4}
+FETEZEN_STREAMS, FETEZEN_GROUPS = 2, 2
+
+
+def fetezen_layers(z: dict, vocab: int, draw, feed_forward, seed: int) -> list[dict]:
+    """Packed layers of a Fetezen of the sizes `z`; feed_forward(i): gate | up [2 ff, width] and down [width, ff] of layer i: its first half is a
+    dense layer's, its parts the experts'."""
+    from pygpukit_amd import _hip
+    from pygpukit_amd.core.array import GPUArray
+    from pygpukit_amd.core.factory import from_numpy
+    from pygpukit_amd.llm.engine import StackEngine, _row
+
+    W, F, H, G, D, L = (z[k] for k in ("width", "ff", "heads", "kv_heads", "dim", "layers"))
+    x, S, rng = FETEZEN_EXPERTS, FETEZEN_STREAMS, np.random.default_rng(seed + 1)
+    f, E = F // x["split"], x["experts"]
+    vec = lambda n, v=1.0: from_numpy(np.full(n, v, np.float32))  # noqa: E731
+
+    def copies(w, n, shape):
+        out = GPUArray(shape, w.dtype)
+        for i in range(out.nbytes // (w.nbytes // n)):
+            _hip.call("pgk_memcpy_d2d", out.data_ptr() + i * (w.nbytes // n), w.data_ptr() + i % n * (w.nbytes // n), w.nbytes // n, None)
+        return out
+
+    layers = []
+    for i in range(L):
+        gu, dn = feed_forward(i)
+        talk = from_numpy((np.eye(H) + 0.3 * rng.standard_normal((H, H)) / np.sqrt(H)).astype(np.float32))
+        lw = StackEngine.pack_talking(draw(H * D, W), draw(G * D, W), draw(G * D, W), draw(W, H * D), vec(W), heads=H, kv_heads=G, dim=D, vdim=D, window=z["window"], chunked=True,
+                                      scale=D**-0.5, biases=(draw(H * D), draw(G * D), draw(G * D)), o_bias=draw(W), q_norm=vec(D), k_norm=vec(D),
+                                      rot_freq=from_numpy((1e4 ** (-2.0 * np.arange(D // 2) / D)).astype(np.float32)), talk=talk, sink=vec(H))
+        hyper = StackEngine.pack_hyper(vec(S, 1.0 / S), vec(S), from_numpy((0.7 * np.eye(S) + 0.1).astype(np.float32)))
+        lw.update(hyper1=hyper, hyper2=hyper, norm2=_row(vec(W), W))
+        if i % 2 == 0:
+            StackEngine.add_poly_mlp(lw, W, gu._view(0, (F, W)), dn, vec(4, 0.5))
+        else:
+            table = from_numpy(np.argsort(rng.random((vocab, E)), axis=1)[:, :x["top"]].astype(np.int32))
+            StackEngine.add_table_experts(lw, W, table, copies(gu._view(0, (F, W)), x["split"], (E, f, W)), copies(dn, x["split"], (E, W, f)), (draw(f, W), draw(W, f), draw(1, W)))
+        layers.append(lw)
+    return layers
+
+
 def stack_kernel_bytes(kind: str, z: dict, vocab: int, ctx: int, B: int) -> dict:
     """Algorithmic bytes of ONE decode step of a layer-list engine by kernel class (bf16 weights and caches, fp32 rows and states)."""
     W, F, H, D, L, n = z["width"], z["ff"], z["heads"], z["dim"], z["layers"], min(ctx, z["window"])
     hd, gd, r = H * D, z["kv_heads"] * D, z["rank"]
+    if kind == "fetezen":              # experts of one sequence: the chosen ones
+        x, S, A = FETEZEN_EXPERTS, FETEZEN_STREAMS, L // 2
+        used = F // x["split"] * (x["top"] + 1)
+        n, n_in = ctx % z["window"] + 1, hd + 2 * gd
+        return {"norm_qkv": L * (n_in * W * 2 + B * 4 * ((S + 1) * W + n_in)), "attn": L * B * (n * gd * 2 * 2 + 4 * (n_in + hd)), "oproj": L * (hd * W * 2 + B * 4 * (hd + W)),
+                "gateup": (L - A) * (F * W * 2 + B * 4 * ((S + 1) * W + F)) + A * (used * W * 2 + B * 4 * ((S + 1) * W + used)),
+                "down": (L - A) * (F * W * 2 + B * 4 * (F + W)) + A * (used * W * 2 + B * 4 * (used + W)), "lmhead": vocab * W * 2 + B * 4 * (S * W + vocab)}
     if kind == "ratasun":              # experts of one sequence: the chosen ones; `down` is out-projection and experts in one launch
         x, kinds = RATASUN_EXPERTS, [ratasun_layer(i) for i in range(L)]
         E, top, f, rot, lr = x["experts"], x["top"], F // x["split"], D // 4, RATASUN_RANK
@@ -216,6 +266,7 @@ def stack_kernel_bytes(kind: str, z: dict, vocab: int, ctx: int, B: int) -> dict
 
 def design_engines(name: str, size: str, seed: int) -> tuple[dict, dict]:
     """(sizes, kind -> engine constructor (max_seq_len, max_batch)) of a design and its relatives."""
+    from pygpukit_amd import _hip
     from pygpukit_amd.core.factory import from_numpy
     from pygpukit_amd.llm import synthetic as S
     from pygpukit_amd.llm.config import distance_slopes
@@ -262,16 +313,22 @@ def design_engines(name: str, size: str, seed: int) -> tuple[dict, dict]:
     if name == "ratasun":
         model = ratasun_model(z, V, embed, head, draw, lambda i: feed_forwards[i])
         make = {"ratasun": lambda ms, mb: model.build_engine(max_seq_len=ms, max_batch=mb), "malasun": make["malasun"], "totolorn": make["totolorn"]}
+    elif name == "fetezen":
+        layers = fetezen_layers(z, V, draw, lambda i: feed_forwards[i], seed)
+        fcfg = dict(scfg, residual_mult=1.0, block=_hip.BLOCK_HYPER, streams=FETEZEN_STREAMS, norm_groups=FETEZEN_GROUPS, logit_cap=30.0)
+        model = ratasun_model(z, V, embed, head, draw, lambda i: feed_forwards[i])
+        make = {"fetezen": lambda ms, mb: StackEngine(fcfg, embed, None, head, one, layers, max_seq_len=ms, max_batch=mb), "malasun": make["malasun"],
+                "ratasun": lambda ms, mb: model.build_engine(max_seq_len=ms, max_batch=mb), "dense": make["dense"]}
     elif name != "malasun":
         del make["malasun"]
     return z, make
 
 
-def design_leg(name: str, sizes: list[str], seed: int) -> dict:
-    """--design totolorn | malasun | ratasun: prefill and decode of the layer-list engine at sizes that resemble a real model's layers (random
+def design_leg(name: str, sizes: list[str], seed: int, kinds: list[str] | None = None) -> dict:
+    """--design totolorn | malasun | ratasun | fetezen: prefill and decode of the layer-list engine at sizes that resemble a real model's layers (random
     weights), beside its closest relatives here at equal width, heads, feed-forward width, depth and vocabulary: the dense QKV + RoPE
     engine, and for Malasun (every other layer attention, the others recurrent) Totolorn too; for Ratasun (three mixers in turn, experts)
-    Malasun and Totolorn."""
+    Malasun and Totolorn; for Fetezen (attention everywhere, every other layer experts) Malasun, Ratasun and the dense engine."""
     from pygpukit_amd import _hip
 
     V = DESIGN_VOCAB
@@ -296,6 +353,7 @@ def design_leg(name: str, sizes: list[str], seed: int) -> dict:
         L = z["layers"]
         dcfg = dense_config(z)
         res = {"config": z}
+        make = {k: v for k, v in make.items() if kinds is None or k in kinds}
         for kind, new in make.items():
             rec = {"prefill": {}, "decode": {}}
             e = new(4200, 1)
@@ -324,7 +382,7 @@ def design_leg(name: str, sizes: list[str], seed: int) -> dict:
                     per = {"lmhead": 1, "attn": n_attn, "recur": max(1, L - n_attn)}      # layers that have the class
                     rec["decode"][f"b{B}_ctx{ctx}"]["kernels"] = {
                         k: {"us_per_layer": round(us * n / per.get(k, L), 2), "hbm_frac": round(nb[k] / (us * n) / 1e3 / HBM_PEAK_GBS, 3)}
-                        for k, (us, n) in prof.items() if n and k in nb and k != "argmax" and (B == 1 or kind != "ratasun" or k in ("attn", "recur"))}
+                        for k, (us, n) in prof.items() if n and k in nb and k != "argmax" and (B == 1 or kind not in ("ratasun", "fetezen") or k in ("attn", "recur"))}
                 del e
             res[kind] = rec
         out["sizes"][size] = res
@@ -353,8 +411,9 @@ def main() -> None:
                     help="skip every extra leg (config 4 weak/strong; at N = 1 also context 2048 in bf16 and w8a16, config 5)")
     ap.add_argument("--config4-steps", type=int, default=32)
     ap.add_argument("--layers", type=int, default=0, help="debug only: override the layer count (result is then INVALID)")
-    ap.add_argument("--design", choices=["totolorn", "malasun", "ratasun"], help="instead of the headline: prefill / decode of a layer-list design beside its relatives")
+    ap.add_argument("--design", choices=["totolorn", "malasun", "ratasun", "fetezen"], help="instead of the headline: prefill / decode of a layer-list design beside its relatives")
     ap.add_argument("--design-sizes", default="w1024,w2048,w4096", help="with --design: which sizes")
+    ap.add_argument("--design-kinds", default="", help="with --design: only these of the design and its relatives (default: all)")
     args = ap.parse_args()
 
     # ONE JSON line on stdout, whatever the libraries underneath print: RCCL writes a version banner to the process's stdout
@@ -368,7 +427,7 @@ def main() -> None:
         os.write(result_fd, (json.dumps(obj) + "\n").encode())
 
     if args.design:
-        emit(design_leg(args.design, args.design_sizes.split(","), args.seed))
+        emit(design_leg(args.design, args.design_sizes.split(","), args.seed, args.design_kinds.split(",") if args.design_kinds else None))
         return
 
     from pygpukit_amd import _hip

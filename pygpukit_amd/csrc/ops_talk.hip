@@ -235,6 +235,436 @@ static pgk_status talk_any(const TalkArgs& a, hipStream_t st) {
     return PGK_OK;
 }
 
+// -------------------------------------------------------------------------------------------- bf16 on the matrix pipe
+typedef __bf16 bf16x8_tk __attribute__((ext_vector_type(8)));
+typedef float f32x4_tk __attribute__((ext_vector_type(4)));
+typedef float f32x2_tk __attribute__((ext_vector_type(2)));
+typedef short v4s_tk __attribute__((ext_vector_type(4)));
+template <class A, class B>       // 16 bytes each
+__device__ __forceinline__ f32x4_tk mfma_tk(const A& a, const B& b, f32x4_tk c) {
+    return __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8_tk, a), __builtin_bit_cast(bf16x8_tk, b), c, 0, 0, 0);
+}
+// four rows' worth of a 16-column block, transposed: two reads make an operand whose k order is 16 (j >> 2) + 4 (lane >> 4) + (j & 3)
+__device__ __forceinline__ uint4 read_tr(const bf16* lo, const bf16* hi) {
+    const v4s_tk a = __builtin_amdgcn_ds_read_tr16_b64_v4i16((__attribute__((address_space(3))) v4s_tk*)lo);
+    const v4s_tk b = __builtin_amdgcn_ds_read_tr16_b64_v4i16((__attribute__((address_space(3))) v4s_tk*)hi);
+    const uint2 x = __builtin_bit_cast(uint2, a), y = __builtin_bit_cast(uint2, b);
+    return make_uint4(x.x, x.y, y.x, y.y);
+}
+
+// ---- decode: one query per sequence ----
+// A workgroup per (split, sequence), all heads, 32 keys at a time: raw scores [up to 16 heads of a key head][16 keys] by product (waves: two
+// halves of the keys x two halves of the key heads, keys straight from memory), scores meet in LDS, a thread mixes H / 8 heads of one
+// key, and O[heads][d] += P V goes with every wave taking a quarter of the columns of all heads.
+constexpr int TD_S = 33, TD_P = 36;                                // row strides of scores and weights
+static size_t talk_decode_lds(int H, int G, int D) {
+    return (size_t)32 * (G * D + 8) * 2 + (size_t)H * TD_S * 4 + (size_t)H * ((H + 7) / 8 * 8) * 4 + (size_t)H * TD_P * 2 + (size_t)H * 4 + 64;
+}
+template <class IT, int GM, int RT>
+__global__ __launch_bounds__(256) void talk_decode_kernel(unsigned long long* tl, TalkArgs a) {
+    const TLStamp tls(tl);
+    extern __shared__ __attribute__((aligned(16))) char td_smem[];
+    constexpr int CH = 2 * RT, HT = 8;                             // 32-wide pieces of a head, most heads per mixing thread
+    const int H = a.H, G = a.G, D = a.D, rep = H / G, GD = G * D, ldv = GD + 8, hpt = (H + 7) / 8;
+    bf16* vs = reinterpret_cast<bf16*>(td_smem);                  // [32][ldv]
+    float* sc = reinterpret_cast<float*>(td_smem + (size_t)32 * ldv * 2);      // [H][TD_S]
+    float* tt = sc + ((H * TD_S + 3) & ~3);                       // [H from][8][hpt]: head hg + 8 j at [hg][j]
+    bf16* ps = reinterpret_cast<bf16*>(tt + H * 8 * hpt);         // [H][TD_P]
+    float* al = reinterpret_cast<float*>(ps + ((H * TD_P + 1) & ~1));           // [H]
+    const int tid = threadIdx.x, lane = tid & 63, wid = __builtin_amdgcn_readfirstlane(tid >> 6), l15 = lane & 15, q4 = lane >> 4, s = blockIdx.x, b = blockIdx.y;
+    const int kh = wid & 1, uh = wid >> 1, key = tid & 31, hg = tid >> 5;
+    int n, lo, k0, k1;
+    ring_window(max(a.positions[b], 0), a.window, a.R, n, lo, a.chunked);
+    split_range(n, a.nsplit, s, k0, k1);
+    if (k0 >= k1) {                                                // an empty split: its record says so, the sums are never read
+        for (int h = tid; h < H; h += 256) {
+            float* ml = a.pml + (((size_t)b * H + h) * a.nsplit + s) * 2;
+            ml[0] = -INFINITY; ml[1] = 0.f;
+        }
+        tls.end();
+        return;
+    }
+    const bf16* kb = reinterpret_cast<const bf16*>(a.cache) + (size_t)b * 2 * G * a.R * D;
+    const bf16* vb = kb + (size_t)G * a.R * D;
+    const bf16* qb = reinterpret_cast<const bf16*>(a.q) + (size_t)b * a.ld_q;
+    constexpr int GW = (GM + 1) / 2, LPR = 8 * RT, RPP = 256 / LPR;               // key heads of a wave; lanes and rows of a pass over V (lanes past a row's end repeat its last piece)
+    u32x4 qf[GW][CH], kf[GW][CH], vr[GM][RT];
+    const int hl = min(l15, rep - 1), vrow = tid / LPR, vcol = min((tid % LPR) * 8, D - 8);
+    const size_t gstep = (size_t)a.R * D;
+    auto fetch = [&](int kt) {
+        const bf16* kr = kb + (size_t)ring_row(lo, min(kt + 16 * kh + l15, k1 - 1), a.R) * D + uh * gstep;
+#pragma unroll
+        for (int i = 0; i < GW; ++i) {
+            if (2 * i + uh < G) {                                  // wave-uniform
+#pragma unroll
+                for (int c = 0; c < CH; ++c) kf[i][c] = *reinterpret_cast<const u32x4*>(kr + min(32 * c + 8 * q4, D - 8));
+            }
+            kr += 2 * gstep;
+        }
+        const bf16* vp[RT];
+#pragma unroll
+        for (int t = 0; t < RT; ++t) vp[t] = vb + (size_t)ring_row(lo, min(kt + vrow + t * RPP, k1 - 1), a.R) * D + vcol;
+#pragma unroll
+        for (int g = 0; g < GM; ++g) {
+#pragma unroll
+            for (int t = 0; t < RT; ++t) { vr[g][t] = *reinterpret_cast<const u32x4*>(vp[t]); vp[t] += g + 1 < G ? gstep : 0; }      // (past the last: that one again)
+        }
+    };
+    {
+        const bf16* qr = qb + (size_t)(uh * rep + hl) * D;
+#pragma unroll
+        for (int i = 0; i < GW; ++i) {
+            if (2 * i + uh < G) {
+#pragma unroll
+                for (int c = 0; c < CH; ++c) qf[i][c] = *reinterpret_cast<const u32x4*>(qr + min(32 * c + 8 * q4, D - 8));
+            }
+            qr += (size_t)2 * rep * D;
+        }
+    }
+    fetch(k0);
+    const float mult = a.scale * TK_LOG2E;
+    if (a.talk)
+        for (int i = tid; i < H * H; i += 256) { const int h = i / H, g = i - h * H; tt[(g * 8 + (h & 7)) * hpt + (h >> 3)] = a.talk[i] * mult; }
+    float m_run[HT], l_run[HT];
+#pragma unroll
+    for (int j = 0; j < HT; ++j) { m_run[j] = -INFINITY; l_run[j] = 0.f; }
+    f32x4_tk o[GM][RT];
+#pragma unroll
+    for (int g = 0; g < GM; ++g)
+#pragma unroll
+        for (int t = 0; t < RT; ++t) o[g][t] = f32x4_tk{0.f, 0.f, 0.f, 0.f};
+    for (int kt = k0; kt < k1; kt += 32) {
+        if (kt != k0) __syncthreads();                             // the last step's reads of V and the weights are done
+#pragma unroll
+        for (int g = 0; g < GM; ++g) {
+#pragma unroll
+            for (int t = 0; t < RT; ++t)
+                if (g < G) *reinterpret_cast<u32x4*>(vs + (vrow + t * RPP) * ldv + g * D + vcol) = vr[g][t];
+        }
+        float* sw = sc + (uh * rep + 4 * q4) * TD_S + 16 * kh + l15;
+#pragma unroll
+        for (int i = 0; i < GW; ++i) {
+            if (2 * i + uh < G) {
+                f32x4_tk t = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+                for (int c = 0; c < CH; ++c) if (32 * c < D) t = mfma_tk(qf[i][c], kf[i][c], t);
+#pragma unroll
+                for (int r = 0; r < 4; ++r) if (4 * q4 + r < rep) sw[r * TD_S] = t[r];
+            }
+            sw += 2 * rep * TD_S;
+        }
+        if (kt + 32 < k1) fetch(kt + 32);                          // the next tile travels under the rest of this one
+        __syncthreads();
+        float x[HT];
+#pragma unroll
+        for (int j = 0; j < HT; ++j) x[j] = 0.f;
+        if (a.talk) {
+            for (int g = 0; g < H; ++g) {
+                const float r = sc[g * TD_S + key];
+                const float* tg = tt + (g * 8 + hg) * hpt;
+#pragma unroll
+                for (int j = 0; j < HT; ++j) if (j < hpt) x[j] = fmaf(tg[j], r, x[j]);
+            }
+        } else {
+#pragma unroll
+            for (int j = 0; j < HT; ++j) if (hg + 8 * j < H) x[j] = sc[(hg + 8 * j) * TD_S + key] * mult;
+        }
+#pragma unroll
+        for (int j = 0; j < HT; ++j) {
+            const int h = hg + 8 * j;
+            if (h >= H) continue;                                  // (uniform over the 32 lanes of a key row)
+            const float v = kt + key < k1 ? x[j] : -INFINITY;
+            float top = v;
+#pragma unroll
+            for (int off = 16; off >= 1; off >>= 1) top = fmaxf(top, __shfl_xor(top, off, 64));
+            const float mn = fmaxf(m_run[j], top), f = __builtin_amdgcn_exp2f(m_run[j] - mn), p = __builtin_amdgcn_exp2f(v - mn);     // mn is finite: kt < k1
+            m_run[j] = mn;
+            l_run[j] = fmaf(l_run[j], f, p);
+            ps[h * TD_P + key] = from_f<bf16>(p);
+            if (key == 0) al[h] = f;
+        }
+        __syncthreads();
+#pragma unroll
+        for (int g = 0; g < GM; ++g) {
+            if (g >= G) continue;
+            float f[4];
+#pragma unroll
+            for (int r = 0; r < 4; ++r) f[r] = al[g * rep + min(4 * q4 + r, rep - 1)];
+            const bf16* pr = ps + (g * rep + hl) * TD_P + 4 * q4;
+            const uint2 p0 = *reinterpret_cast<const uint2*>(pr), p1 = *reinterpret_cast<const uint2*>(pr + 16);
+            const uint4 pf = make_uint4(p0.x, p0.y, p1.x, p1.y);
+            const bf16* row = vs + (4 * q4 + (l15 >> 2)) * ldv + g * D + 4 * (l15 & 3);
+#pragma unroll
+            for (int t = 0; t < RT; ++t) {
+                const int dc = 16 * (wid + 4 * t);
+                if (dc < D) {                                      // wave-uniform
+#pragma unroll
+                    for (int r = 0; r < 4; ++r) o[g][t][r] *= f[r];
+                    o[g][t] = mfma_tk(pf, read_tr(row + dc, row + 16 * ldv + dc), o[g][t]);
+                }
+            }
+        }
+    }
+    __syncthreads();
+    float* fin = al;                                               // [H]: what the sums are multiplied by
+#pragma unroll
+    for (int j = 0; j < HT; ++j) {
+        const int h = hg + 8 * j;
+        if (h >= H) continue;
+        float l = l_run[j];
+#pragma unroll
+        for (int off = 16; off >= 1; off >>= 1) l += __shfl_xor(l, off, 64);
+        if (key != 0) continue;
+        if (a.nsplit > 1) {
+            float* ml = a.pml + (((size_t)b * H + h) * a.nsplit + s) * 2;
+            ml[0] = m_run[j]; ml[1] = l;
+        } else fin[h] = sink_scale(a.sink, h, m_run[j], l);
+    }
+    if (a.nsplit == 1) __syncthreads();
+#pragma unroll
+    for (int g = 0; g < GM; ++g) {
+        if (g >= G) continue;
+#pragma unroll
+        for (int t = 0; t < RT; ++t)
+#pragma unroll
+            for (int r = 0; r < 4; ++r) {
+                const int hh = 4 * q4 + r, dc = 16 * (wid + 4 * t) + l15, h = g * rep + hh;
+                if (hh >= rep || dc >= D) continue;
+                if (a.nsplit > 1) a.po[(((size_t)b * H + h) * a.nsplit + s) * D + dc] = o[g][t][r];
+                else reinterpret_cast<IT*>(a.out)[(size_t)b * a.ld_out + h * D + dc] = from_f<IT>(o[g][t][r] * fin[h]);
+            }
+    }
+    tls.end();
+}
+
+static bool talk_decode_ok(const TalkArgs& a) {
+    return a.cache && a.D <= 256 && a.H <= 64 && a.H / a.G <= 16 && a.ld_q % 8 == 0 && a.G * ceil_div(a.D, 64) <= 16 && talk_decode_lds(a.H, a.G, a.D) <= (size_t)TALK_LDS_MAX;
+}
+template <class IT>
+static pgk_status talk_decode_mfma(const TalkArgs& a, hipStream_t st) {
+    const size_t lds = talk_decode_lds(a.H, a.G, a.D);
+    auto go = [&](auto um, auto rt) -> pgk_status {
+        auto kfn = &talk_decode_kernel<IT, decltype(um)::value, decltype(rt)::value>;
+        static bool done = false;
+        if (lds > 48 * 1024 && !done) {
+            PGK_CHECK_HIP(hipFuncSetAttribute(reinterpret_cast<const void*>(kfn), hipFuncAttributeMaxDynamicSharedMemorySize, TALK_LDS_MAX));
+            done = true;
+        }
+        PGK_CHECK_HIP(launch_k(kfn, dim3(a.nsplit, a.n), dim3(256), lds, st, a));
+        return PGK_OK;
+    };
+    const int G = a.G;
+    using std::integral_constant;
+    auto pick = [&](auto rt) -> pgk_status {
+        constexpr int RT = decltype(rt)::value;
+        if (G <= 2) return go(integral_constant<int, 2>{}, rt);
+        if (G <= 4) return go(integral_constant<int, 4>{}, rt);
+        if constexpr (RT <= 2) { if (G <= 8) return go(integral_constant<int, 8>{}, rt); }
+        if constexpr (RT == 1) { if (G <= 16) return go(integral_constant<int, 16>{}, rt); }
+        return set_error(PGK_ERR_UNSUPPORTED, "talk_attention: %d key heads of width %d", G, a.D);
+    };
+    return a.D <= 64 ? pick(integral_constant<int, 1>{}) : a.D <= 128 ? pick(integral_constant<int, 2>{}) : pick(integral_constant<int, 4>{});
+}
+
+// ---- prompts: 16 queries x all heads per workgroup, 32 keys at a time ----
+// NW waves of up to HW heads.  (1) a wave's raw scores [32 keys][16 queries] per head go to LDS as S[head][query][key]; (2) a wave mixes the
+// heads of its 16 / NW queries in place, fp32 products T S of the matrix pipe; (3) a wave takes its heads' rows back, softmax in
+// registers (a lane per query and eighth of the keys), O^T[d][query] += V^T P^T with V of its key head in a part of LDS of its own.
+// V's rows of D columns lie in 16-byte pieces that are XOR-ed by the row, so that the transposing reads of 16 rows spread over the banks.
+constexpr int TF_Q = 36, TF_H = 16 * TF_Q;                         // floats per query and head of S
+static size_t talk_flash_lds(int NW, int HW, int D) { return (size_t)NW * HW * TF_H * 4 + (size_t)(NW * HW + 15) / 16 * 16 * (NW * HW + 4) * 4 + (size_t)NW * 32 * D * 2; }
+
+// ONE: the heads of a wave share a key head.  Waves and heads past the last repeat it and store nothing.
+template <int NW, int HW, int RT, bool ONE>
+__global__ __launch_bounds__(64 * NW, 2) void talk_flash_kernel(unsigned long long* tl, TalkArgs a, int tiles) {
+    const TLStamp tls(tl);
+    extern __shared__ __attribute__((aligned(16))) char tf_smem[];
+    constexpr bool FULL = HW * RT == 8;                            // queries and sums take most of the registers
+    constexpr int D = 64 * RT, CH = D / 32, DT = D / 16, HM = (NW * HW + 15) / 16, KS = NW * HW / 4, PC = D / 8;
+    float* S = reinterpret_cast<float*>(tf_smem);                 // [NW HW][16][TF_Q]
+    constexpr int TL = NW * HW + 4;
+    float* T = S + NW * HW * TF_H;                                 // [16 HM][TL], times the score factor, zero where there is no head
+    bf16* vs = reinterpret_cast<bf16*>(T + 16 * HM * TL) + (threadIdx.x >> 6) * 32 * D;       // [32][D] of this wave
+    const int H = a.H, rep = H / a.G, lane = threadIdx.x & 63, l15 = lane & 15, q4 = lane >> 4;
+    const int wid = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+    // tiles of 16 queries: a run of neighbours per die, longest first within it does not pay at one round
+    const int per = (tiles + 7) / 8, tile = (blockIdx.x & 7) * per + (blockIdx.x >> 3);
+    if (tile >= tiles) { tls.end(); return; }
+    const int q0 = tile * 16, nq = min(16, a.n - q0), past = a.kv_len - a.n;
+    auto first_key = [&](int q) { const int last = past + q; return last + 1 - min(span_keys(a.pos0 + last, a.window, a.chunked), last + 1); };
+    const int my_q = q0 + min(l15, nq - 1), my_lo = first_key(my_q), my_last = past + my_q;
+    const int k_begin = first_key(q0), k_end = past + q0 + nq, lo_max = first_key(q0 + nq - 1), last_min = past + q0;
+    const bf16 *kbase = reinterpret_cast<const bf16*>(a.k), *vbase = reinterpret_cast<const bf16*>(a.v);
+    auto head = [&](int i) { return min(wid * HW + i, H - 1); };
+    u32x4 qf[HW][CH];
+#pragma unroll
+    for (int i = 0; i < HW; ++i) {
+        const bf16* qr = reinterpret_cast<const bf16*>(a.q) + (size_t)my_q * a.ld_q + (size_t)head(i) * D + 8 * q4;
+#pragma unroll
+        for (int c = 0; c < CH; ++c) qf[i][c] = *reinterpret_cast<const u32x4*>(qr + 32 * c);
+    }
+    const float mult = a.scale * TK_LOG2E;
+    for (int i = threadIdx.x; i < 16 * HM * TL; i += 64 * NW) {
+        const int h = i / TL, g = i - h * TL;
+        T[i] = h < H && g < H ? (a.talk ? a.talk[h * H + g] : h == g ? 1.0f : 0.f) * mult : 0.f;
+    }
+    for (int i = H * TF_H + threadIdx.x; i < NW * HW * TF_H; i += 64 * NW) S[i] = 0.f;         // heads that do not exist
+    f32x4_tk o[HW][DT];
+    float m[HW], l[HW];
+#pragma unroll
+    for (int i = 0; i < HW; ++i) {
+        m[i] = -INFINITY; l[i] = 0.f;
+#pragma unroll
+        for (int t = 0; t < DT; ++t) o[i][t] = f32x4_tk{0.f, 0.f, 0.f, 0.f};
+    }
+    // V of key head g, keys kt ..: 16-byte pieces, piece c of row r at c ^ swizzle(r)
+    auto swz = [](int r) { return RT == 2 ? (r & 7) * 2 : ((r >> 1) & 3) * 2; };
+    const uint32_t vaddr = __builtin_amdgcn_readfirstlane((uint32_t)(uintptr_t)(__attribute__((address_space(3))) void*)vs);
+    auto load_v = [&](int g, int kt) {
+#pragma unroll
+        for (int i = 0; i < 32 * PC / 64; ++i) {
+            const int p = i * 64 + lane, r = p / PC, c = (p % PC) ^ swz(r);
+            const bf16* src = vbase + (size_t)min(kt + r, k_end - 1) * a.ld_kv + g * D + c * 8;
+            asm volatile("s_mov_b32 m0, %1\n\ts_nop 0\n\tglobal_load_lds_dwordx4 %0, off" ::"v"(src), "s"(vaddr + i * 1024) : "memory", "m0");
+        }
+    };
+    for (int kt = k_begin; kt < k_end; kt += 32) {
+#pragma unroll
+        for (int u = 0; u < 2; ++u) {
+            u32x4 kf[CH];
+            auto load_k = [&](int g) {
+                const bf16* kr = kbase + (size_t)min(kt + 16 * u + l15, k_end - 1) * a.ld_kv + g * D + 8 * q4;
+#pragma unroll
+                for (int c = 0; c < CH; ++c) kf[c] = *reinterpret_cast<const u32x4*>(kr + 32 * c);
+            };
+            if constexpr (ONE) load_k(head(0) / rep);
+            if (u == 0) load_v(head(0) / rep, kt);                 // (this wave's reads of the last tile's V are done: they fed its products)
+#pragma unroll
+            for (int i = 0; i < HW; ++i) {
+                if constexpr (!ONE) load_k(head(i) / rep);
+                f32x4_tk t = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+                for (int c = 0; c < CH; ++c) t = mfma_tk(kf[c], qf[i][c], t);
+                *reinterpret_cast<f32x4_tk*>(S + head(i) * TF_H + l15 * TF_Q + 16 * u + 4 * q4) = t;            // keys 16 u + 4 q4 .. of query l15
+                if (FULL && !ONE) __builtin_amdgcn_sched_barrier(0);
+            }
+            if (FULL) __builtin_amdgcn_sched_barrier(0);           // (registers: one half's keys at a time)
+        }
+        __syncthreads();
+#pragma unroll 1
+        for (int pass = 0; pass < 16 / NW; ++pass) {               // a query at a time: lane l15 has keys 2 l15 and 2 l15 + 1
+            float* at = S + (wid * (16 / NW) + pass) * TF_Q + 2 * l15;
+            f32x2_tk r[KS];
+#pragma unroll
+            for (int k = 0; k < KS; ++k) r[k] = *reinterpret_cast<const f32x2_tk*>(at + (4 * k + q4) * TF_H);
+            f32x4_tk x[HM][2];
+            const float* tp = T + l15 * TL + q4;                   // T as operand: row l15 of each 16 heads, columns 4 k + q4
+#pragma unroll
+            for (int mt = 0; mt < HM; ++mt)
+#pragma unroll
+                for (int j = 0; j < 2; ++j) {
+                    x[mt][j] = f32x4_tk{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+                    for (int k = 0; k < KS; ++k) x[mt][j] = __builtin_amdgcn_mfma_f32_16x16x4f32(tp[mt * 16 * TL + 4 * k], r[k][j], x[mt][j], 0, 0, 0);
+                }
+            // (every lane's reads of this query fed the products: the wave may write it)
+#pragma unroll
+            for (int mt = 0; mt < HM; ++mt)
+#pragma unroll
+                for (int e = 0; e < 4; ++e) {
+                    const int h = 16 * mt + 4 * q4 + e;
+                    if (h < NW * HW) *reinterpret_cast<f32x2_tk*>(at + h * TF_H) = f32x2_tk{x[mt][0][e], x[mt][1][e]};
+                }
+        }
+        __syncthreads();
+        {
+            const bool whole = kt >= lo_max && kt + 31 <= last_min;
+            asm volatile("s_waitcnt vmcnt(0)" ::: "memory");       // V has arrived
+#pragma unroll
+            for (int i = 0; i < HW; ++i) {
+                if (!ONE && i > 0) {
+                    asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");         // the last head's reads
+                    load_v(head(i) / rep, kt);
+                    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+                }
+                const float* sr = S + head(i) * TF_H + l15 * TF_Q + 4 * q4;
+                f32x4_tk s0 = *reinterpret_cast<const f32x4_tk*>(sr), s1 = *reinterpret_cast<const f32x4_tk*>(sr + 16);      // keys 4 q4 .., 16 + 4 q4 ..
+                if (!whole) {
+#pragma unroll
+                    for (int e = 0; e < 4; ++e) {
+                        const int k = kt + 4 * q4 + e;
+                        if (k < my_lo || k > my_last) s0[e] = -INFINITY;
+                        if (k + 16 < my_lo || k + 16 > my_last) s1[e] = -INFINITY;
+                    }
+                }
+                float top = fmaxf(fmaxf(fmaxf(s0[0], s0[1]), fmaxf(s0[2], s0[3])), fmaxf(fmaxf(s1[0], s1[1]), fmaxf(s1[2], s1[3])));
+                top = fmaxf(top, __shfl_xor(top, 16, 64));
+                top = fmaxf(top, __shfl_xor(top, 32, 64));
+                const float mn = fmaxf(m[i], top), ref = mn == -INFINITY ? 0.f : mn, f = __builtin_amdgcn_exp2f(m[i] - ref);
+                m[i] = mn;
+                float sum = 0.f;
+#pragma unroll
+                for (int e = 0; e < 4; ++e) {
+                    s0[e] = __builtin_amdgcn_exp2f(s0[e] - ref);
+                    s1[e] = __builtin_amdgcn_exp2f(s1[e] - ref);
+                    sum += s0[e] + s1[e];
+                }
+                l[i] = fmaf(l[i], f, sum);
+                const uint4 pf = make_uint4(pack_bf16x2(s0[0], s0[1]), pack_bf16x2(s0[2], s0[3]), pack_bf16x2(s1[0], s1[1]), pack_bf16x2(s1[2], s1[3]));
+                const int r0 = 4 * q4 + (l15 >> 2), sz = swz(r0);              // rows r0 and r0 + 16 have the same swizzle
+#pragma unroll
+                for (int t = 0; t < DT; ++t) {
+                    const bf16* row = vs + r0 * D + (((2 * t + ((l15 & 3) >> 1)) ^ sz) << 3) + 4 * (l15 & 1);
+                    o[i][t] = mfma_tk(read_tr(row, row + 16 * D), pf, o[i][t] * f);
+                    if (FULL && (t & 1)) __builtin_amdgcn_sched_barrier(0);                // (no more reads in flight than two columns')
+                }
+            }
+        }
+        __syncthreads();                                           // the next tile's scores take S
+    }
+#pragma unroll
+    for (int i = 0; i < HW; ++i) {
+        float sum = l[i];
+        sum += __shfl_xor(sum, 16, 64);
+        sum += __shfl_xor(sum, 32, 64);
+        const float f = sink_scale(a.sink, head(i), m[i], sum);
+        if (l15 >= nq || wid * HW + i >= H) continue;
+        bf16* out = reinterpret_cast<bf16*>(a.out) + (size_t)(q0 + l15) * a.ld_out + (size_t)(wid * HW + i) * D + 4 * q4;
+#pragma unroll
+        for (int t = 0; t < DT; ++t) store4<bf16>(out + 16 * t, make_float4(o[i][t][0] * f, o[i][t][1] * f, o[i][t][2] * f, o[i][t][3] * f));
+    }
+    tls.end();
+}
+
+static bool talk_flash_ok(const TalkArgs& a) {
+    return !a.cache && !a.Dv && (a.D == 64 || a.D == 128) && a.H <= 32 && a.ld_q % 8 == 0 && a.ld_kv % 8 == 0 && a.ld_out % 4 == 0 && aligned16(a.q) && aligned16(a.k) && aligned16(a.v) &&
+           (reinterpret_cast<uintptr_t>(a.out) & 7u) == 0;
+}
+static pgk_status talk_flash(const TalkArgs& a, hipStream_t st) {
+    const int tiles = ceil_div(a.n, 16);
+    auto go = [&](auto nw, auto hw, auto rt) -> pgk_status {
+        constexpr int NW = decltype(nw)::value, HW = decltype(hw)::value, RT = decltype(rt)::value;
+        auto kfn = (a.H / a.G) % HW == 0 ? &talk_flash_kernel<NW, HW, RT, true> : &talk_flash_kernel<NW, HW, RT, HW == 1>;
+        const size_t lds = talk_flash_lds(NW, HW, 64 * RT);
+        static bool done[2] = {false, false};
+        bool& set = done[(a.H / a.G) % HW == 0];
+        if (lds > 48 * 1024 && !set) {
+            PGK_CHECK_HIP(hipFuncSetAttribute(reinterpret_cast<const void*>(kfn), hipFuncAttributeMaxDynamicSharedMemorySize, TALK_LDS_MAX));
+            set = true;
+        }
+        PGK_CHECK_HIP(launch_k(kfn, dim3(ceil_div(tiles, 8) * 8), dim3(64 * NW), lds, st, a, tiles));
+        return PGK_OK;
+    };
+    using std::integral_constant;
+    auto pick = [&](auto rt) -> pgk_status {
+        if (a.H <= 4) return go(integral_constant<int, 4>{}, integral_constant<int, 1>{}, rt);
+        if (a.H <= 8) return go(integral_constant<int, 4>{}, integral_constant<int, 2>{}, rt);
+        if (a.H <= 16) return go(integral_constant<int, 4>{}, integral_constant<int, 4>{}, rt);
+        return go(integral_constant<int, 8>{}, integral_constant<int, 4>{}, rt);
+    };
+    return a.D == 64 ? pick(integral_constant<int, 1>{}) : pick(integral_constant<int, 2>{});
+}
+
 int talk_splits(int B, int H, int G, int keys, int cus) {
     int s = ceil_div(keys, 32);
     const int want = ceil_div(2 * cus, B);
@@ -246,8 +676,12 @@ pgk_status talk_attention(const TalkArgs& a, pgk_dtype dt, bool io32, hipStream_
     PGK_REQUIRE(a.n >= 1 && a.H >= 1 && a.G >= 1 && a.H % a.G == 0 && a.window >= 1 && a.nsplit >= 1 && a.nsplit <= 64 && ((a.D % 64 == 0 && a.ld_q % 8 == 0) || a.Dv) && (!a.Dv || !a.cache) &&
                     (a.cache ? a.positions && a.R >= 1 && (a.nsplit == 1 || (a.po && a.pml)) : a.k && a.v && a.kv_len >= a.n && a.nsplit == 1),
                 "talk_attention: %d rows, %d / %d heads of %d, %d splits", a.n, a.H, a.G, a.D, a.nsplit);
-    if (dt == PGK_F32) { if (pgk_status r = talk_any<float, float>(a, st)) return r; }
-    else if (pgk_status r = io32 ? talk_any<bf16, float>(a, st) : talk_any<bf16, bf16>(a, st)) return r;
+    pgk_status r;
+    if (dt == PGK_F32) r = talk_any<float, float>(a, st);
+    else if (talk_decode_ok(a)) r = io32 ? talk_decode_mfma<float>(a, st) : talk_decode_mfma<bf16>(a, st);
+    else if (!io32 && talk_flash_ok(a)) r = talk_flash(a, st);
+    else r = io32 ? talk_any<bf16, float>(a, st) : talk_any<bf16, bf16>(a, st);
+    if (r) return r;
     *launches += 1;
     if (a.nsplit == 1) return PGK_OK;
     KvAttnArgs m{};
