@@ -466,57 +466,45 @@ static pgk_status talk_decode_mfma(const TalkArgs& a, hipStream_t st) {
     return a.D <= 64 ? pick(integral_constant<int, 1>{}) : a.D <= 128 ? pick(integral_constant<int, 2>{}) : pick(integral_constant<int, 4>{});
 }
 
-// ---- prompts: 16 queries x all heads per workgroup, 32 keys at a time ----
-// NW waves of up to HW heads.  (1) a wave's raw scores [32 keys][16 queries] per head go to LDS as S[head][query][key]; (2) a wave mixes the
-// heads of its 16 / NW queries in place, fp32 products T S of the matrix pipe; (3) a wave takes its heads' rows back, softmax in
-// registers (a lane per query and eighth of the keys), O^T[d][query] += V^T P^T with V of its key head in a part of LDS of its own.
-// V's rows of D columns lie in 16-byte pieces that are XOR-ed by the row, so that the transposing reads of 16 rows spread over the banks.
+// ---- prompts: 16 queries per workgroup, 32 keys at a time ----
+// NW waves.  (1) The raw scores [32 keys][16 queries] of HW heads per wave go to LDS as S[head][query][key]; (2) a wave mixes the heads of its
+// 16 / NW queries, fp32 products T S of the matrix pipe, into the NW HO output heads of this workgroup (blockIdx.y: which), in place;
+// (3) HO output heads per wave: their rows come back, softmax in registers (a lane per query and eighth of the keys), O^T[d][query] +=
+// V^T P^T with V of the key head in a part of LDS of the wave's own.  Keys of the next tile travel meanwhile; DB: S exists twice, so that no
+// wave waits for the others' step 3.  V's rows of D columns lie in 16-byte pieces that are XOR-ed by the row, so that the transposing
+// reads of 16 rows spread over the banks.  ONE: the heads of a wave share a key head.  Heads past the last repeat it and store nothing.
 constexpr int TF_Q = 36, TF_H = 16 * TF_Q;                         // floats per query and head of S
-static size_t talk_flash_lds(int NW, int HW, int D) { return (size_t)NW * HW * TF_H * 4 + (size_t)(NW * HW + 15) / 16 * 16 * (NW * HW + 4) * 4 + (size_t)NW * 32 * D * 2; }
+static size_t talk_flash_lds(int NW, int HW, int HO, int D, bool db) {
+    return (size_t)NW * HW * TF_H * 4 * (db ? 2 : 1) + (size_t)(NW * HO + 15) / 16 * 16 * (NW * HW + 4) * 4 + (size_t)NW * 32 * D * 2;
+}
 
-// ONE: the heads of a wave share a key head.  Waves and heads past the last repeat it and store nothing.
-template <int NW, int HW, int RT, bool ONE>
-__global__ __launch_bounds__(64 * NW, 2) void talk_flash_kernel(unsigned long long* tl, TalkArgs a, int tiles) {
+template <int NW, int HW, int HO, int RT, bool ONE, bool DB>
+__global__ __launch_bounds__(64 * NW, 2) void talk_flash_kernel(unsigned long long* tl, TalkArgs a, int tiles, int per) {
     const TLStamp tls(tl);
     extern __shared__ __attribute__((aligned(16))) char tf_smem[];
-    constexpr bool FULL = HW * RT == 8;                            // queries and sums take most of the registers
-    constexpr int D = 64 * RT, CH = D / 32, DT = D / 16, HM = (NW * HW + 15) / 16, KS = NW * HW / 4, PC = D / 8;
-    float* S = reinterpret_cast<float*>(tf_smem);                 // [NW HW][16][TF_Q]
-    constexpr int TL = NW * HW + 4;
-    float* T = S + NW * HW * TF_H;                                 // [16 HM][TL], times the score factor, zero where there is no head
+    constexpr int D = 64 * RT, CH = D / 32, DT = D / 16, HM = (NW * HO + 15) / 16, KS = NW * HW / 4, PC = D / 8, TL = NW * HW + 4, SN = NW * HW * TF_H;
+    constexpr bool FULL = (HW * CH + HO * DT) * 4 >= 128;          // queries and sums take most of the registers
+    float* S0 = reinterpret_cast<float*>(tf_smem);                // [NW HW][16][TF_Q]
+    float* T = S0 + SN * (DB ? 2 : 1);                             // [16 HM][TL], times the score factor, zero where there is no head
     bf16* vs = reinterpret_cast<bf16*>(T + 16 * HM * TL) + (threadIdx.x >> 6) * 32 * D;       // [32][D] of this wave
     const int H = a.H, rep = H / a.G, lane = threadIdx.x & 63, l15 = lane & 15, q4 = lane >> 4;
-    const int wid = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
-    // tiles of 16 queries: a run of neighbours per die, longest first within it does not pay at one round
-    const int per = (tiles + 7) / 8, tile = (blockIdx.x & 7) * per + (blockIdx.x >> 3);
+    const int wid = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), ho0 = (int)blockIdx.y * NW * HO;
+    // runs of `per` tiles (a chunk's), the last tiles of all runs first: they have the most keys
+    const int runs = (tiles + per - 1) / per, tile = (int)(blockIdx.x % runs) * per + per - 1 - (int)(blockIdx.x / runs);
     if (tile >= tiles) { tls.end(); return; }
     const int q0 = tile * 16, nq = min(16, a.n - q0), past = a.kv_len - a.n;
     auto first_key = [&](int q) { const int last = past + q; return last + 1 - min(span_keys(a.pos0 + last, a.window, a.chunked), last + 1); };
     const int my_q = q0 + min(l15, nq - 1), my_lo = first_key(my_q), my_last = past + my_q;
     const int k_begin = first_key(q0), k_end = past + q0 + nq, lo_max = first_key(q0 + nq - 1), last_min = past + q0;
-    const bf16 *kbase = reinterpret_cast<const bf16*>(a.k), *vbase = reinterpret_cast<const bf16*>(a.v);
+    const bf16 *kbase = reinterpret_cast<const bf16*>(a.k) + 8 * q4, *vbase = reinterpret_cast<const bf16*>(a.v);
     auto head = [&](int i) { return min(wid * HW + i, H - 1); };
-    u32x4 qf[HW][CH];
+    auto out_head = [&](int i) { return min(ho0 + wid * HO + i, H - 1); };
+    u32x4 qf[HW][CH], kf[2][CH];
+    auto load_k = [&](int u, int g, int kt) {
+        const bf16* kr = kbase + (size_t)min(kt + 16 * u + l15, k_end - 1) * a.ld_kv + g * D;
 #pragma unroll
-    for (int i = 0; i < HW; ++i) {
-        const bf16* qr = reinterpret_cast<const bf16*>(a.q) + (size_t)my_q * a.ld_q + (size_t)head(i) * D + 8 * q4;
-#pragma unroll
-        for (int c = 0; c < CH; ++c) qf[i][c] = *reinterpret_cast<const u32x4*>(qr + 32 * c);
-    }
-    const float mult = a.scale * TK_LOG2E;
-    for (int i = threadIdx.x; i < 16 * HM * TL; i += 64 * NW) {
-        const int h = i / TL, g = i - h * TL;
-        T[i] = h < H && g < H ? (a.talk ? a.talk[h * H + g] : h == g ? 1.0f : 0.f) * mult : 0.f;
-    }
-    for (int i = H * TF_H + threadIdx.x; i < NW * HW * TF_H; i += 64 * NW) S[i] = 0.f;         // heads that do not exist
-    f32x4_tk o[HW][DT];
-    float m[HW], l[HW];
-#pragma unroll
-    for (int i = 0; i < HW; ++i) {
-        m[i] = -INFINITY; l[i] = 0.f;
-#pragma unroll
-        for (int t = 0; t < DT; ++t) o[i][t] = f32x4_tk{0.f, 0.f, 0.f, 0.f};
-    }
+        for (int c = 0; c < CH; ++c) kf[u][c] = *reinterpret_cast<const u32x4*>(kr + 32 * c);
+    };
     // V of key head g, keys kt ..: 16-byte pieces, piece c of row r at c ^ swizzle(r)
     auto swz = [](int r) { return RT == 2 ? (r & 7) * 2 : ((r >> 1) & 3) * 2; };
     const uint32_t vaddr = __builtin_amdgcn_readfirstlane((uint32_t)(uintptr_t)(__attribute__((address_space(3))) void*)vs);
@@ -528,29 +516,48 @@ __global__ __launch_bounds__(64 * NW, 2) void talk_flash_kernel(unsigned long lo
             asm volatile("s_mov_b32 m0, %1\n\ts_nop 0\n\tglobal_load_lds_dwordx4 %0, off" ::"v"(src), "s"(vaddr + i * 1024) : "memory", "m0");
         }
     };
+#pragma unroll
+    for (int i = 0; i < HW; ++i) {
+        const bf16* qr = reinterpret_cast<const bf16*>(a.q) + (size_t)my_q * a.ld_q + (size_t)head(i) * D + 8 * q4;
+#pragma unroll
+        for (int c = 0; c < CH; ++c) qf[i][c] = *reinterpret_cast<const u32x4*>(qr + 32 * c);
+    }
+    if constexpr (ONE) { load_k(0, head(0) / rep, k_begin); load_k(1, head(0) / rep, k_begin); }
+    const float mult = a.scale * TK_LOG2E;
+    for (int i = threadIdx.x; i < 16 * HM * TL; i += 64 * NW) {
+        const int h = ho0 + i / TL, g = i % TL;
+        T[i] = h < H && g < H ? (a.talk ? a.talk[h * H + g] : h == g ? 1.0f : 0.f) * mult : 0.f;
+    }
+#pragma unroll
+    for (int d = 0; d < (DB ? 2 : 1); ++d)
+        for (int i = H * TF_H + threadIdx.x; i < SN; i += 64 * NW) S0[d * SN + i] = 0.f;      // heads that do not exist
+    f32x4_tk o[HO][DT];
+    float m[HO], l[HO];
+#pragma unroll
+    for (int i = 0; i < HO; ++i) {
+        m[i] = -INFINITY; l[i] = 0.f;
+#pragma unroll
+        for (int t = 0; t < DT; ++t) o[i][t] = f32x4_tk{0.f, 0.f, 0.f, 0.f};
+    }
+    float* S = S0;
     for (int kt = k_begin; kt < k_end; kt += 32) {
 #pragma unroll
-        for (int u = 0; u < 2; ++u) {
-            u32x4 kf[CH];
-            auto load_k = [&](int g) {
-                const bf16* kr = kbase + (size_t)min(kt + 16 * u + l15, k_end - 1) * a.ld_kv + g * D + 8 * q4;
+        for (int i = 0; i < HW; ++i) {
+            if constexpr (!ONE) { load_k(0, head(i) / rep, kt); load_k(1, head(i) / rep, kt); }
 #pragma unroll
-                for (int c = 0; c < CH; ++c) kf[c] = *reinterpret_cast<const u32x4*>(kr + 32 * c);
-            };
-            if constexpr (ONE) load_k(head(0) / rep);
-            if (u == 0) load_v(head(0) / rep, kt);                 // (this wave's reads of the last tile's V are done: they fed its products)
-#pragma unroll
-            for (int i = 0; i < HW; ++i) {
-                if constexpr (!ONE) load_k(head(i) / rep);
+            for (int u = 0; u < 2; ++u) {
                 f32x4_tk t = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-                for (int c = 0; c < CH; ++c) t = mfma_tk(kf[c], qf[i][c], t);
+                for (int c = 0; c < CH; ++c) t = mfma_tk(kf[u][c], qf[i][c], t);
                 *reinterpret_cast<f32x4_tk*>(S + head(i) * TF_H + l15 * TF_Q + 16 * u + 4 * q4) = t;            // keys 16 u + 4 q4 .. of query l15
-                if (FULL && !ONE) __builtin_amdgcn_sched_barrier(0);
             }
-            if (FULL) __builtin_amdgcn_sched_barrier(0);           // (registers: one half's keys at a time)
         }
-        __syncthreads();
+        // (behind the products that the compiler has made wait for the keys: it does not count these; the reads of the last tile's V are done)
+        load_v(out_head(0) / rep, kt);
+        if constexpr (ONE) { load_k(0, head(0) / rep, kt + 32); load_k(1, head(0) / rep, kt + 32); }
+        asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+        __builtin_amdgcn_s_barrier();                              // (loads stay in flight)
+        asm volatile("" ::: "memory");
 #pragma unroll 1
         for (int pass = 0; pass < 16 / NW; ++pass) {               // a query at a time: lane l15 has keys 2 l15 and 2 l15 + 1
             float* at = S + (wid * (16 / NW) + pass) * TF_Q + 2 * l15;
@@ -573,63 +580,68 @@ __global__ __launch_bounds__(64 * NW, 2) void talk_flash_kernel(unsigned long lo
 #pragma unroll
                 for (int e = 0; e < 4; ++e) {
                     const int h = 16 * mt + 4 * q4 + e;
-                    if (h < NW * HW) *reinterpret_cast<f32x2_tk*>(at + h * TF_H) = f32x2_tk{x[mt][0][e], x[mt][1][e]};
+                    if (h < NW * HO) *reinterpret_cast<f32x2_tk*>(at + h * TF_H) = f32x2_tk{x[mt][0][e], x[mt][1][e]};
                 }
         }
-        __syncthreads();
-        {
-            const bool whole = kt >= lo_max && kt + 31 <= last_min;
-            asm volatile("s_waitcnt vmcnt(0)" ::: "memory");       // V has arrived
+        asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+        __builtin_amdgcn_s_barrier();
+        const bool whole = kt >= lo_max && kt + 31 <= last_min;
+        if constexpr (ONE) asm volatile("s_waitcnt vmcnt(%0)" ::"n"(2 * CH) : "memory");       // V has arrived, the keys behind it may still travel
+        else asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
 #pragma unroll
-            for (int i = 0; i < HW; ++i) {
-                if (!ONE && i > 0) {
-                    asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");         // the last head's reads
-                    load_v(head(i) / rep, kt);
-                    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
-                }
-                const float* sr = S + head(i) * TF_H + l15 * TF_Q + 4 * q4;
-                f32x4_tk s0 = *reinterpret_cast<const f32x4_tk*>(sr), s1 = *reinterpret_cast<const f32x4_tk*>(sr + 16);      // keys 4 q4 .., 16 + 4 q4 ..
-                if (!whole) {
-#pragma unroll
-                    for (int e = 0; e < 4; ++e) {
-                        const int k = kt + 4 * q4 + e;
-                        if (k < my_lo || k > my_last) s0[e] = -INFINITY;
-                        if (k + 16 < my_lo || k + 16 > my_last) s1[e] = -INFINITY;
-                    }
-                }
-                float top = fmaxf(fmaxf(fmaxf(s0[0], s0[1]), fmaxf(s0[2], s0[3])), fmaxf(fmaxf(s1[0], s1[1]), fmaxf(s1[2], s1[3])));
-                top = fmaxf(top, __shfl_xor(top, 16, 64));
-                top = fmaxf(top, __shfl_xor(top, 32, 64));
-                const float mn = fmaxf(m[i], top), ref = mn == -INFINITY ? 0.f : mn, f = __builtin_amdgcn_exp2f(m[i] - ref);
-                m[i] = mn;
-                float sum = 0.f;
+        for (int i = 0; i < HO; ++i) {
+            if (!ONE && i > 0) {
+                asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");             // the last head's reads
+                load_v(out_head(i) / rep, kt);
+                asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+            }
+            const float* sr = S + min(wid * HO + i, NW * HW - 1) * TF_H + l15 * TF_Q + 4 * q4;
+            f32x4_tk s0 = *reinterpret_cast<const f32x4_tk*>(sr), s1 = *reinterpret_cast<const f32x4_tk*>(sr + 16);      // keys 4 q4 .., 16 + 4 q4 ..
+            if (!whole) {
 #pragma unroll
                 for (int e = 0; e < 4; ++e) {
-                    s0[e] = __builtin_amdgcn_exp2f(s0[e] - ref);
-                    s1[e] = __builtin_amdgcn_exp2f(s1[e] - ref);
-                    sum += s0[e] + s1[e];
-                }
-                l[i] = fmaf(l[i], f, sum);
-                const uint4 pf = make_uint4(pack_bf16x2(s0[0], s0[1]), pack_bf16x2(s0[2], s0[3]), pack_bf16x2(s1[0], s1[1]), pack_bf16x2(s1[2], s1[3]));
-                const int r0 = 4 * q4 + (l15 >> 2), sz = swz(r0);              // rows r0 and r0 + 16 have the same swizzle
-#pragma unroll
-                for (int t = 0; t < DT; ++t) {
-                    const bf16* row = vs + r0 * D + (((2 * t + ((l15 & 3) >> 1)) ^ sz) << 3) + 4 * (l15 & 1);
-                    o[i][t] = mfma_tk(read_tr(row, row + 16 * D), pf, o[i][t] * f);
-                    if (FULL && (t & 1)) __builtin_amdgcn_sched_barrier(0);                // (no more reads in flight than two columns')
+                    const int k = kt + 4 * q4 + e;
+                    if (k < my_lo || k > my_last) s0[e] = -INFINITY;
+                    if (k + 16 < my_lo || k + 16 > my_last) s1[e] = -INFINITY;
                 }
             }
-        }
-        __syncthreads();                                           // the next tile's scores take S
-    }
+            float top = fmaxf(fmaxf(fmaxf(s0[0], s0[1]), fmaxf(s0[2], s0[3])), fmaxf(fmaxf(s1[0], s1[1]), fmaxf(s1[2], s1[3])));
+            top = fmaxf(top, __shfl_xor(top, 16, 64));
+            top = fmaxf(top, __shfl_xor(top, 32, 64));
+            const float mn = fmaxf(m[i], top), ref = mn == -INFINITY ? 0.f : mn, f = __builtin_amdgcn_exp2f(m[i] - ref);
+            m[i] = mn;
+            float sum = 0.f;
 #pragma unroll
-    for (int i = 0; i < HW; ++i) {
+            for (int e = 0; e < 4; ++e) {
+                s0[e] = __builtin_amdgcn_exp2f(s0[e] - ref);
+                s1[e] = __builtin_amdgcn_exp2f(s1[e] - ref);
+                sum += s0[e] + s1[e];
+            }
+            l[i] = fmaf(l[i], f, sum);
+            const uint4 pf = make_uint4(pack_bf16x2(s0[0], s0[1]), pack_bf16x2(s0[2], s0[3]), pack_bf16x2(s1[0], s1[1]), pack_bf16x2(s1[2], s1[3]));
+            const int r0 = 4 * q4 + (l15 >> 2), sz = swz(r0);                  // rows r0 and r0 + 16 have the same swizzle
+#pragma unroll
+            for (int t = 0; t < DT; ++t) {
+                const bf16* row = vs + r0 * D + (((2 * t + ((l15 & 3) >> 1)) ^ sz) << 3) + 4 * (l15 & 1);
+                o[i][t] = mfma_tk(read_tr(row, row + 16 * D), pf, o[i][t] * f);
+                if (FULL && (t & 3) == 3) __builtin_amdgcn_sched_barrier(0);   // (registers: no more reads in flight than four columns')
+            }
+        }
+        if constexpr (DB) S = S == S0 ? S0 + SN : S0;
+        else {
+            asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+            __builtin_amdgcn_s_barrier();                          // the next tile's scores take S
+        }
+    }
+    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+#pragma unroll
+    for (int i = 0; i < HO; ++i) {
         float sum = l[i];
         sum += __shfl_xor(sum, 16, 64);
         sum += __shfl_xor(sum, 32, 64);
-        const float f = sink_scale(a.sink, head(i), m[i], sum);
-        if (l15 >= nq || wid * HW + i >= H) continue;
-        bf16* out = reinterpret_cast<bf16*>(a.out) + (size_t)(q0 + l15) * a.ld_out + (size_t)(wid * HW + i) * D + 4 * q4;
+        const float f = sink_scale(a.sink, out_head(i), m[i], sum);
+        if (l15 >= nq || ho0 + wid * HO + i >= H) continue;
+        bf16* out = reinterpret_cast<bf16*>(a.out) + (size_t)(q0 + l15) * a.ld_out + (size_t)(ho0 + wid * HO + i) * D + 4 * q4;
 #pragma unroll
         for (int t = 0; t < DT; ++t) store4<bf16>(out + 16 * t, make_float4(o[i][t][0] * f, o[i][t][1] * f, o[i][t][2] * f, o[i][t][3] * f));
     }
@@ -641,28 +653,34 @@ static bool talk_flash_ok(const TalkArgs& a) {
            (reinterpret_cast<uintptr_t>(a.out) & 7u) == 0;
 }
 static pgk_status talk_flash(const TalkArgs& a, hipStream_t st) {
-    const int tiles = ceil_div(a.n, 16);
-    auto go = [&](auto nw, auto hw, auto rt) -> pgk_status {
-        constexpr int NW = decltype(nw)::value, HW = decltype(hw)::value, RT = decltype(rt)::value;
-        auto kfn = (a.H / a.G) % HW == 0 ? &talk_flash_kernel<NW, HW, RT, true> : &talk_flash_kernel<NW, HW, RT, HW == 1>;
-        const size_t lds = talk_flash_lds(NW, HW, 64 * RT);
-        static bool done[2] = {false, false};
-        bool& set = done[(a.H / a.G) % HW == 0];
-        if (lds > 48 * 1024 && !set) {
-            PGK_CHECK_HIP(hipFuncSetAttribute(reinterpret_cast<const void*>(kfn), hipFuncAttributeMaxDynamicSharedMemorySize, TALK_LDS_MAX));
-            set = true;
+    const int tiles = ceil_div(a.n, 16), rep = a.H / a.G;
+    const int per = a.chunked && a.window / 16 >= 1 && a.window / 16 < tiles ? a.window / 16 : tiles, runs = ceil_div(tiles, per);
+    auto go = [&](auto nw, auto hw, auto ho, auto rt, auto one, auto db) -> pgk_status {
+        constexpr int NW = decltype(nw)::value, HW = decltype(hw)::value, HO = decltype(ho)::value, RT = decltype(rt)::value;
+        auto kfn = &talk_flash_kernel<NW, HW, HO, RT, decltype(one)::value, decltype(db)::value>;
+        const size_t lds = talk_flash_lds(NW, HW, HO, 64 * RT, decltype(db)::value);
+        static bool done = false;
+        if (lds > 48 * 1024 && !done) {
+            PGK_CHECK_HIP(hipFuncSetAttribute(reinterpret_cast<const void*>(kfn), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds));
+            done = true;
         }
-        PGK_CHECK_HIP(launch_k(kfn, dim3(ceil_div(tiles, 8) * 8), dim3(64 * NW), lds, st, a, tiles));
+        PGK_CHECK_HIP(launch_k(kfn, dim3(runs * per, ceil_div(a.H, NW * HO)), dim3(64 * NW), lds, st, a, tiles, per));
         return PGK_OK;
     };
     using std::integral_constant;
+    using std::true_type;
+    using std::false_type;
+    integral_constant<int, 1> one;
+    integral_constant<int, 2> two;
+    integral_constant<int, 4> four;
+    integral_constant<int, 8> eight;
     auto pick = [&](auto rt) -> pgk_status {
-        if (a.H <= 4) return go(integral_constant<int, 4>{}, integral_constant<int, 1>{}, rt);
-        if (a.H <= 8) return go(integral_constant<int, 4>{}, integral_constant<int, 2>{}, rt);
-        if (a.H <= 16) return go(integral_constant<int, 4>{}, integral_constant<int, 4>{}, rt);
-        return go(integral_constant<int, 8>{}, integral_constant<int, 4>{}, rt);
+        if (a.H <= 4) return go(four, one, one, rt, true_type{}, true_type{});
+        if (a.H <= 8) return rep % 2 ? go(eight, one, one, rt, true_type{}, true_type{}) : go(four, two, two, rt, true_type{}, true_type{});
+        if (a.H <= 16) return rep % 2 ? go(eight, two, two, rt, false_type{}, true_type{}) : go(eight, two, two, rt, true_type{}, true_type{});
+        return rep % 4 ? go(eight, four, two, rt, false_type{}, false_type{}) : go(eight, four, two, rt, true_type{}, false_type{});
     };
-    return a.D == 64 ? pick(integral_constant<int, 1>{}) : pick(integral_constant<int, 2>{});
+    return a.D == 64 ? pick(one) : pick(two);
 }
 
 int talk_splits(int B, int H, int G, int keys, int cus) {
