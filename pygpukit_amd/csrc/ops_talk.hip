@@ -466,13 +466,21 @@ static pgk_status talk_decode_mfma(const TalkArgs& a, hipStream_t st) {
     return a.D <= 64 ? pick(integral_constant<int, 1>{}) : a.D <= 128 ? pick(integral_constant<int, 2>{}) : pick(integral_constant<int, 4>{});
 }
 
+// over the four quarters of a wave, lane by lane
+__device__ __forceinline__ float max_of_quarters(float x) {
+    const auto a = __builtin_amdgcn_permlane16_swap(__float_as_uint(x), __float_as_uint(x), false, false);
+    x = fmaxf(__uint_as_float(a[0]), __uint_as_float(a[1]));
+    const auto b = __builtin_amdgcn_permlane32_swap(__float_as_uint(x), __float_as_uint(x), false, false);
+    return fmaxf(__uint_as_float(b[0]), __uint_as_float(b[1]));
+}
+
 // ---- prompts: 16 queries per workgroup, 32 keys at a time ----
 // NW waves.  (1) The raw scores [32 keys][16 queries] of HW heads per wave go to LDS as S[head][query][key]; (2) a wave mixes the heads of its
 // 16 / NW queries, fp32 products T S of the matrix pipe, into the NW HO output heads of this workgroup (blockIdx.y: which), in place;
 // (3) HO output heads per wave: their rows come back, softmax in registers (a lane per query and eighth of the keys), O^T[d][query] +=
-// V^T P^T with V of the key head in a part of LDS of the wave's own.  Keys of the next tile travel meanwhile; DB: S exists twice, so that no
-// wave waits for the others' step 3.  V's rows of D columns lie in 16-byte pieces that are XOR-ed by the row, so that the transposing
-// reads of 16 rows spread over the banks.  ONE: the heads of a wave share a key head.  Heads past the last repeat it and store nothing.
+// V^T P^T.  Keys, then values, of a wave's key head come as whole rows through registers (fetched a step ahead) into a part of LDS of the
+// wave's own, in 16-byte pieces that are XOR-ed by the row, so that operand reads of 16 rows spread over the banks.  DB: S exists twice, so
+// that no wave waits for the others' step 3.  ONE: the heads of a wave share a key head.  Heads past the last repeat it and store nothing.
 constexpr int TF_Q = 36, TF_H = 16 * TF_Q;                         // floats per query and head of S
 static size_t talk_flash_lds(int NW, int HW, int HO, int D, bool db) {
     return (size_t)NW * HW * TF_H * 4 * (db ? 2 : 1) + (size_t)(NW * HO + 15) / 16 * 16 * (NW * HW + 4) * 4 + (size_t)NW * 32 * D * 2;
@@ -486,7 +494,7 @@ __global__ __launch_bounds__(64 * NW, 2) void talk_flash_kernel(unsigned long lo
     constexpr bool FULL = (HW * CH + HO * DT) * 4 >= 128;          // queries and sums take most of the registers
     float* S0 = reinterpret_cast<float*>(tf_smem);                // [NW HW][16][TF_Q]
     float* T = S0 + SN * (DB ? 2 : 1);                             // [16 HM][TL], times the score factor, zero where there is no head
-    bf16* vs = reinterpret_cast<bf16*>(T + 16 * HM * TL) + (threadIdx.x >> 6) * 32 * D;       // [32][D] of this wave
+    bf16* kv = reinterpret_cast<bf16*>(T + 16 * HM * TL) + (threadIdx.x >> 6) * 32 * D;       // [32][D] of this wave
     const int H = a.H, rep = H / a.G, lane = threadIdx.x & 63, l15 = lane & 15, q4 = lane >> 4;
     const int wid = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), ho0 = (int)blockIdx.y * NW * HO;
     // runs of `per` tiles (a chunk's), the last tiles of all runs first: they have the most keys
@@ -496,25 +504,35 @@ __global__ __launch_bounds__(64 * NW, 2) void talk_flash_kernel(unsigned long lo
     auto first_key = [&](int q) { const int last = past + q; return last + 1 - min(span_keys(a.pos0 + last, a.window, a.chunked), last + 1); };
     const int my_q = q0 + min(l15, nq - 1), my_lo = first_key(my_q), my_last = past + my_q;
     const int k_begin = first_key(q0), k_end = past + q0 + nq, lo_max = first_key(q0 + nq - 1), last_min = past + q0;
-    const bf16 *kbase = reinterpret_cast<const bf16*>(a.k) + 8 * q4, *vbase = reinterpret_cast<const bf16*>(a.v);
+    const bf16 *kbase = reinterpret_cast<const bf16*>(a.k), *vbase = reinterpret_cast<const bf16*>(a.v);
     auto head = [&](int i) { return min(wid * HW + i, H - 1); };
     auto out_head = [&](int i) { return min(ho0 + wid * HO + i, H - 1); };
-    u32x4 qf[HW][CH], kf[2][CH];
-    auto load_k = [&](int u, int g, int kt) {
-        const bf16* kr = kbase + (size_t)min(kt + 16 * u + l15, k_end - 1) * a.ld_kv + g * D;
-#pragma unroll
-        for (int c = 0; c < CH; ++c) kf[u][c] = *reinterpret_cast<const u32x4*>(kr + 32 * c);
-    };
-    // V of key head g, keys kt ..: 16-byte pieces, piece c of row r at c ^ swizzle(r)
+    // 32 rows of a key head's keys or values pass through `st` into this wave's part of LDS: piece c of row r at c ^ swizzle(r)
+    constexpr int NV = 32 * PC / 64;
     auto swz = [](int r) { return RT == 2 ? (r & 7) * 2 : ((r >> 1) & 3) * 2; };
-    const uint32_t vaddr = __builtin_amdgcn_readfirstlane((uint32_t)(uintptr_t)(__attribute__((address_space(3))) void*)vs);
-    auto load_v = [&](int g, int kt) {
+    u32x4 qf[HW][CH], st[NV];
+    uint32_t off[NV];                                              // of this lane's pieces in 32 whole rows
 #pragma unroll
-        for (int i = 0; i < 32 * PC / 64; ++i) {
-            const int p = i * 64 + lane, r = p / PC, c = (p % PC) ^ swz(r);
-            const bf16* src = vbase + (size_t)min(kt + r, k_end - 1) * a.ld_kv + g * D + c * 8;
-            asm volatile("s_mov_b32 m0, %1\n\ts_nop 0\n\tglobal_load_lds_dwordx4 %0, off" ::"v"(src), "s"(vaddr + i * 1024) : "memory", "m0");
+    for (int i = 0; i < NV; ++i) off[i] = (uint32_t)((i * 64 + lane) / PC) * (uint32_t)a.ld_kv + (lane % PC) * 8;
+    auto fetch = [&](const bf16* base, int g, int kt) {
+        const bf16* at = base + (size_t)kt * a.ld_kv + g * D;      // (uniform)
+        if (kt + 32 <= k_end) {
+#pragma unroll
+            for (int i = 0; i < NV; ++i) st[i] = *reinterpret_cast<const u32x4*>(at + off[i]);
+        } else if (kt < k_end) {                                   // rows past the end repeat the last
+            const int back = k_end - 1 - kt;
+#pragma unroll
+            for (int i = 0; i < NV; ++i) st[i] = *reinterpret_cast<const u32x4*>(at + (size_t)min((i * 64 + lane) / PC, back) * a.ld_kv + (lane % PC) * 8);
         }
+    };
+    auto put = [&]() {                                             // (behind this wave's reads of what was there)
+        wave_sync();
+#pragma unroll
+        for (int i = 0; i < NV; ++i) {
+            const int p = i * 64 + lane, r = p / PC;
+            *reinterpret_cast<u32x4*>(kv + r * D + ((p % PC) ^ swz(r)) * 8) = st[i];
+        }
+        wave_sync();
     };
 #pragma unroll
     for (int i = 0; i < HW; ++i) {
@@ -522,7 +540,7 @@ __global__ __launch_bounds__(64 * NW, 2) void talk_flash_kernel(unsigned long lo
 #pragma unroll
         for (int c = 0; c < CH; ++c) qf[i][c] = *reinterpret_cast<const u32x4*>(qr + 32 * c);
     }
-    if constexpr (ONE) { load_k(0, head(0) / rep, k_begin); load_k(1, head(0) / rep, k_begin); }
+    fetch(kbase, head(0) / rep, k_begin);
     const float mult = a.scale * TK_LOG2E;
     for (int i = threadIdx.x; i < 16 * HM * TL; i += 64 * NW) {
         const int h = ho0 + i / TL, g = i % TL;
@@ -541,24 +559,32 @@ __global__ __launch_bounds__(64 * NW, 2) void talk_flash_kernel(unsigned long lo
     }
     float* S = S0;
     for (int kt = k_begin; kt < k_end; kt += 32) {
+        constexpr int KG = ONE ? 1 : HW, VG = ONE ? 1 : HO;        // key heads of the wave (those of the output heads: VG) and the heads of each
 #pragma unroll
-        for (int i = 0; i < HW; ++i) {
-            if constexpr (!ONE) { load_k(0, head(i) / rep, kt); load_k(1, head(i) / rep, kt); }
+        for (int gi = 0; gi < KG; ++gi) {
+            put();
+            if (gi + 1 < KG) fetch(kbase, head(gi + 1) / rep, kt);
+            else fetch(vbase, out_head(0) / rep, kt);
 #pragma unroll
             for (int u = 0; u < 2; ++u) {
-                f32x4_tk t = {0.f, 0.f, 0.f, 0.f};
+                u32x4 kf[CH];
 #pragma unroll
-                for (int c = 0; c < CH; ++c) t = mfma_tk(kf[u][c], qf[i][c], t);
-                *reinterpret_cast<f32x4_tk*>(S + head(i) * TF_H + l15 * TF_Q + 16 * u + 4 * q4) = t;            // keys 16 u + 4 q4 .. of query l15
+                for (int c = 0; c < CH; ++c) kf[c] = *reinterpret_cast<const u32x4*>(kv + (16 * u + l15) * D + (((4 * c + q4) ^ swz(l15)) << 3));
+#pragma unroll
+                for (int j = 0; j < HW / KG; ++j) {
+                    const int i = gi * (HW / KG) + j;
+                    f32x4_tk t = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+                    for (int c = 0; c < CH; ++c) t = mfma_tk(kf[c], qf[i][c], t);
+                    *reinterpret_cast<f32x4_tk*>(S + head(i) * TF_H + l15 * TF_Q + 16 * u + 4 * q4) = t;        // keys 16 u + 4 q4 .. of query l15
+                }
+                if (FULL) __builtin_amdgcn_sched_barrier(0);       // (registers: one half's keys at a time)
             }
         }
-        // (behind the products that the compiler has made wait for the keys: it does not count these; the reads of the last tile's V are done)
-        load_v(out_head(0) / rep, kt);
-        if constexpr (ONE) { load_k(0, head(0) / rep, kt + 32); load_k(1, head(0) / rep, kt + 32); }
         asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
         __builtin_amdgcn_s_barrier();                              // (loads stay in flight)
         asm volatile("" ::: "memory");
-#pragma unroll 1
+#pragma unroll (FULL ? 1 : 2)
         for (int pass = 0; pass < 16 / NW; ++pass) {               // a query at a time: lane l15 has keys 2 l15 and 2 l15 + 1
             float* at = S + (wid * (16 / NW) + pass) * TF_Q + 2 * l15;
             f32x2_tk r[KS];
@@ -586,45 +612,52 @@ __global__ __launch_bounds__(64 * NW, 2) void talk_flash_kernel(unsigned long lo
         asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
         __builtin_amdgcn_s_barrier();
         const bool whole = kt >= lo_max && kt + 31 <= last_min;
-        if constexpr (ONE) asm volatile("s_waitcnt vmcnt(%0)" ::"n"(2 * CH) : "memory");       // V has arrived, the keys behind it may still travel
-        else asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
 #pragma unroll
-        for (int i = 0; i < HO; ++i) {
-            if (!ONE && i > 0) {
-                asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");             // the last head's reads
-                load_v(out_head(i) / rep, kt);
-                asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
-            }
-            const float* sr = S + min(wid * HO + i, NW * HW - 1) * TF_H + l15 * TF_Q + 4 * q4;
-            f32x4_tk s0 = *reinterpret_cast<const f32x4_tk*>(sr), s1 = *reinterpret_cast<const f32x4_tk*>(sr + 16);      // keys 4 q4 .., 16 + 4 q4 ..
-            if (!whole) {
+        for (int gi = 0; gi < VG; ++gi) {
+            put();
+            if (gi + 1 < VG) fetch(vbase, out_head(gi + 1) / rep, kt);
+            else fetch(kbase, head(0) / rep, kt + 32);
+            constexpr int HG = HO / VG;
+            uint4 pf[HG];
+#pragma unroll
+            for (int j = 0; j < HG; ++j) {
+                const int i = gi * HG + j;
+                const float* sr = S + min(wid * HO + i, NW * HW - 1) * TF_H + l15 * TF_Q + 4 * q4;
+                f32x4_tk s0 = *reinterpret_cast<const f32x4_tk*>(sr), s1 = *reinterpret_cast<const f32x4_tk*>(sr + 16);      // keys 4 q4 .., 16 + 4 q4 ..
+                if (!whole) {
+#pragma unroll
+                    for (int e = 0; e < 4; ++e) {
+                        const uint32_t k = kt + 4 * q4 + e - my_lo, seen = my_last - my_lo;      // (unsigned: before the first is past the last)
+                        if (k > seen) s0[e] = -INFINITY;
+                        if (k + 16 > seen) s1[e] = -INFINITY;
+                    }
+                }
+                const float top = max_of_quarters(fmaxf(fmaxf(fmaxf(s0[0], s0[1]), fmaxf(s0[2], s0[3])), fmaxf(fmaxf(s1[0], s1[1]), fmaxf(s1[2], s1[3]))));
+                // the reference follows the maximum only when it is left behind by 2^8: until then the weights are as exact
+                if (__any(top > m[i] + 8.0f)) {
+                    const float mn = fmaxf(m[i], top), f = mn == -INFINITY ? 0.f : __builtin_amdgcn_exp2f(m[i] - mn);
+                    m[i] = mn;
+                    l[i] *= f;
+#pragma unroll
+                    for (int t = 0; t < DT; ++t) o[i][t] *= f;
+                }
+                const float ref = m[i] == -INFINITY ? 0.f : m[i];              // (a query that has seen no key yet)
 #pragma unroll
                 for (int e = 0; e < 4; ++e) {
-                    const int k = kt + 4 * q4 + e;
-                    if (k < my_lo || k > my_last) s0[e] = -INFINITY;
-                    if (k + 16 < my_lo || k + 16 > my_last) s1[e] = -INFINITY;
+                    s0[e] = __builtin_amdgcn_exp2f(s0[e] - ref);
+                    s1[e] = __builtin_amdgcn_exp2f(s1[e] - ref);
                 }
+                l[i] += ((s0[0] + s0[1]) + (s0[2] + s0[3])) + ((s1[0] + s1[1]) + (s1[2] + s1[3]));
+                pf[j] = make_uint4(pack_bf16x2(s0[0], s0[1]), pack_bf16x2(s0[2], s0[3]), pack_bf16x2(s1[0], s1[1]), pack_bf16x2(s1[2], s1[3]));
             }
-            float top = fmaxf(fmaxf(fmaxf(s0[0], s0[1]), fmaxf(s0[2], s0[3])), fmaxf(fmaxf(s1[0], s1[1]), fmaxf(s1[2], s1[3])));
-            top = fmaxf(top, __shfl_xor(top, 16, 64));
-            top = fmaxf(top, __shfl_xor(top, 32, 64));
-            const float mn = fmaxf(m[i], top), ref = mn == -INFINITY ? 0.f : mn, f = __builtin_amdgcn_exp2f(m[i] - ref);
-            m[i] = mn;
-            float sum = 0.f;
-#pragma unroll
-            for (int e = 0; e < 4; ++e) {
-                s0[e] = __builtin_amdgcn_exp2f(s0[e] - ref);
-                s1[e] = __builtin_amdgcn_exp2f(s1[e] - ref);
-                sum += s0[e] + s1[e];
-            }
-            l[i] = fmaf(l[i], f, sum);
-            const uint4 pf = make_uint4(pack_bf16x2(s0[0], s0[1]), pack_bf16x2(s0[2], s0[3]), pack_bf16x2(s1[0], s1[1]), pack_bf16x2(s1[2], s1[3]));
             const int r0 = 4 * q4 + (l15 >> 2), sz = swz(r0);                  // rows r0 and r0 + 16 have the same swizzle
 #pragma unroll
             for (int t = 0; t < DT; ++t) {
-                const bf16* row = vs + r0 * D + (((2 * t + ((l15 & 3) >> 1)) ^ sz) << 3) + 4 * (l15 & 1);
-                o[i][t] = mfma_tk(read_tr(row, row + 16 * D), pf, o[i][t] * f);
-                if (FULL && (t & 3) == 3) __builtin_amdgcn_sched_barrier(0);   // (registers: no more reads in flight than four columns')
+                const bf16* row = kv + r0 * D + (((2 * t + ((l15 & 3) >> 1)) ^ sz) << 3) + 4 * (l15 & 1);
+                const uint4 vt = read_tr(row, row + 16 * D);
+#pragma unroll
+                for (int j = 0; j < HG; ++j) o[gi * HG + j][t] = mfma_tk(vt, pf[j], o[gi * HG + j][t]);
+                if (FULL && (t & 3) == 3) __builtin_amdgcn_sched_barrier(0);   // (... and no more reads in flight than four columns')
             }
         }
         if constexpr (DB) S = S == S0 ? S0 + SN : S0;
@@ -633,7 +666,6 @@ __global__ __launch_bounds__(64 * NW, 2) void talk_flash_kernel(unsigned long lo
             __builtin_amdgcn_s_barrier();                          // the next tile's scores take S
         }
     }
-    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
 #pragma unroll
     for (int i = 0; i < HO; ++i) {
         float sum = l[i];
