@@ -252,226 +252,242 @@ __device__ __forceinline__ uint4 read_tr(const bf16* lo, const bf16* hi) {
     return make_uint4(x.x, x.y, y.x, y.y);
 }
 
-// ---- decode: one query per sequence ----
-// A workgroup per (split, sequence), all heads, 32 keys at a time: raw scores [up to 16 heads of a key head][16 keys] by product (waves: two
-// halves of the keys x two halves of the key heads, keys straight from memory), scores meet in LDS, a thread mixes H / 8 heads of one
-// key, and O[heads][d] += P V goes with every wave taking a quarter of the columns of all heads.
-constexpr int TD_S = 33, TD_P = 36;                                // row strides of scores and weights
-static size_t talk_decode_lds(int H, int G, int D) {
-    return (size_t)32 * (G * D + 8) * 2 + (size_t)H * TD_S * 4 + (size_t)H * ((H + 7) / 8 * 8) * 4 + (size_t)H * TD_P * 2 + (size_t)H * 4 + 64;
-}
-template <class IT, int GM, int RT>
-__global__ __launch_bounds__(256) void talk_decode_kernel(unsigned long long* tl, TalkArgs a) {
-    const TLStamp tls(tl);
-    extern __shared__ __attribute__((aligned(16))) char td_smem[];
-    constexpr int CH = 2 * RT, HT = 8;                             // 32-wide pieces of a head, most heads per mixing thread
-    const int H = a.H, G = a.G, D = a.D, rep = H / G, GD = G * D, ldv = GD + 8, hpt = (H + 7) / 8;
-    bf16* vs = reinterpret_cast<bf16*>(td_smem);                  // [32][ldv]
-    float* sc = reinterpret_cast<float*>(td_smem + (size_t)32 * ldv * 2);      // [H][TD_S]
-    float* tt = sc + ((H * TD_S + 3) & ~3);                       // [H from][8][hpt]: head hg + 8 j at [hg][j]
-    bf16* ps = reinterpret_cast<bf16*>(tt + H * 8 * hpt);         // [H][TD_P]
-    float* al = reinterpret_cast<float*>(ps + ((H * TD_P + 1) & ~1));           // [H]
-    const int tid = threadIdx.x, lane = tid & 63, wid = __builtin_amdgcn_readfirstlane(tid >> 6), l15 = lane & 15, q4 = lane >> 4, s = blockIdx.x, b = blockIdx.y;
-    const int kh = wid & 1, uh = wid >> 1, key = tid & 31, hg = tid >> 5;
-    int n, lo, k0, k1;
-    ring_window(max(a.positions[b], 0), a.window, a.R, n, lo, a.chunked);
-    split_range(n, a.nsplit, s, k0, k1);
-    if (k0 >= k1) {                                                // an empty split: its record says so, the sums are never read
-        for (int h = tid; h < H; h += 256) {
-            float* ml = a.pml + (((size_t)b * H + h) * a.nsplit + s) * 2;
-            ml[0] = -INFINITY; ml[1] = 0.f;
-        }
-        tls.end();
-        return;
-    }
-    const bf16* kb = reinterpret_cast<const bf16*>(a.cache) + (size_t)b * 2 * G * a.R * D;
-    const bf16* vb = kb + (size_t)G * a.R * D;
-    const bf16* qb = reinterpret_cast<const bf16*>(a.q) + (size_t)b * a.ld_q;
-    constexpr int GW = (GM + 1) / 2, LPR = 8 * RT, RPP = 256 / LPR;               // key heads of a wave; lanes and rows of a pass over V (lanes past a row's end repeat its last piece)
-    u32x4 qf[GW][CH], kf[GW][CH], vr[GM][RT];
-    const int hl = min(l15, rep - 1), vrow = tid / LPR, vcol = min((tid % LPR) * 8, D - 8);
-    const size_t gstep = (size_t)a.R * D;
-    auto fetch = [&](int kt) {
-        const bf16* kr = kb + (size_t)ring_row(lo, min(kt + 16 * kh + l15, k1 - 1), a.R) * D + uh * gstep;
-#pragma unroll
-        for (int i = 0; i < GW; ++i) {
-            if (2 * i + uh < G) {                                  // wave-uniform
-#pragma unroll
-                for (int c = 0; c < CH; ++c) kf[i][c] = *reinterpret_cast<const u32x4*>(kr + min(32 * c + 8 * q4, D - 8));
-            }
-            kr += 2 * gstep;
-        }
-        const bf16* vp[RT];
-#pragma unroll
-        for (int t = 0; t < RT; ++t) vp[t] = vb + (size_t)ring_row(lo, min(kt + vrow + t * RPP, k1 - 1), a.R) * D + vcol;
-#pragma unroll
-        for (int g = 0; g < GM; ++g) {
-#pragma unroll
-            for (int t = 0; t < RT; ++t) { vr[g][t] = *reinterpret_cast<const u32x4*>(vp[t]); vp[t] += g + 1 < G ? gstep : 0; }      // (past the last: that one again)
-        }
-    };
-    {
-        const bf16* qr = qb + (size_t)(uh * rep + hl) * D;
-#pragma unroll
-        for (int i = 0; i < GW; ++i) {
-            if (2 * i + uh < G) {
-#pragma unroll
-                for (int c = 0; c < CH; ++c) qf[i][c] = *reinterpret_cast<const u32x4*>(qr + min(32 * c + 8 * q4, D - 8));
-            }
-            qr += (size_t)2 * rep * D;
-        }
-    }
-    fetch(k0);
-    const float mult = a.scale * TK_LOG2E;
-    if (a.talk)
-        for (int i = tid; i < H * H; i += 256) { const int h = i / H, g = i - h * H; tt[(g * 8 + (h & 7)) * hpt + (h >> 3)] = a.talk[i] * mult; }
-    float m_run[HT], l_run[HT];
-#pragma unroll
-    for (int j = 0; j < HT; ++j) { m_run[j] = -INFINITY; l_run[j] = 0.f; }
-    f32x4_tk o[GM][RT];
-#pragma unroll
-    for (int g = 0; g < GM; ++g)
-#pragma unroll
-        for (int t = 0; t < RT; ++t) o[g][t] = f32x4_tk{0.f, 0.f, 0.f, 0.f};
-    for (int kt = k0; kt < k1; kt += 32) {
-        if (kt != k0) __syncthreads();                             // the last step's reads of V and the weights are done
-#pragma unroll
-        for (int g = 0; g < GM; ++g) {
-#pragma unroll
-            for (int t = 0; t < RT; ++t)
-                if (g < G) *reinterpret_cast<u32x4*>(vs + (vrow + t * RPP) * ldv + g * D + vcol) = vr[g][t];
-        }
-        float* sw = sc + (uh * rep + 4 * q4) * TD_S + 16 * kh + l15;
-#pragma unroll
-        for (int i = 0; i < GW; ++i) {
-            if (2 * i + uh < G) {
-                f32x4_tk t = {0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-                for (int c = 0; c < CH; ++c) if (32 * c < D) t = mfma_tk(qf[i][c], kf[i][c], t);
-#pragma unroll
-                for (int r = 0; r < 4; ++r) if (4 * q4 + r < rep) sw[r * TD_S] = t[r];
-            }
-            sw += 2 * rep * TD_S;
-        }
-        if (kt + 32 < k1) fetch(kt + 32);                          // the next tile travels under the rest of this one
-        __syncthreads();
-        float x[HT];
-#pragma unroll
-        for (int j = 0; j < HT; ++j) x[j] = 0.f;
-        if (a.talk) {
-            for (int g = 0; g < H; ++g) {
-                const float r = sc[g * TD_S + key];
-                const float* tg = tt + (g * 8 + hg) * hpt;
-#pragma unroll
-                for (int j = 0; j < HT; ++j) if (j < hpt) x[j] = fmaf(tg[j], r, x[j]);
-            }
-        } else {
-#pragma unroll
-            for (int j = 0; j < HT; ++j) if (hg + 8 * j < H) x[j] = sc[(hg + 8 * j) * TD_S + key] * mult;
-        }
-#pragma unroll
-        for (int j = 0; j < HT; ++j) {
-            const int h = hg + 8 * j;
-            if (h >= H) continue;                                  // (uniform over the 32 lanes of a key row)
-            const float v = kt + key < k1 ? x[j] : -INFINITY;
-            float top = v;
-#pragma unroll
-            for (int off = 16; off >= 1; off >>= 1) top = fmaxf(top, __shfl_xor(top, off, 64));
-            const float mn = fmaxf(m_run[j], top), f = __builtin_amdgcn_exp2f(m_run[j] - mn), p = __builtin_amdgcn_exp2f(v - mn);     // mn is finite: kt < k1
-            m_run[j] = mn;
-            l_run[j] = fmaf(l_run[j], f, p);
-            ps[h * TD_P + key] = from_f<bf16>(p);
-            if (key == 0) al[h] = f;
-        }
-        __syncthreads();
-#pragma unroll
-        for (int g = 0; g < GM; ++g) {
-            if (g >= G) continue;
-            float f[4];
-#pragma unroll
-            for (int r = 0; r < 4; ++r) f[r] = al[g * rep + min(4 * q4 + r, rep - 1)];
-            const bf16* pr = ps + (g * rep + hl) * TD_P + 4 * q4;
-            const uint2 p0 = *reinterpret_cast<const uint2*>(pr), p1 = *reinterpret_cast<const uint2*>(pr + 16);
-            const uint4 pf = make_uint4(p0.x, p0.y, p1.x, p1.y);
-            const bf16* row = vs + (4 * q4 + (l15 >> 2)) * ldv + g * D + 4 * (l15 & 3);
-#pragma unroll
-            for (int t = 0; t < RT; ++t) {
-                const int dc = 16 * (wid + 4 * t);
-                if (dc < D) {                                      // wave-uniform
-#pragma unroll
-                    for (int r = 0; r < 4; ++r) o[g][t][r] *= f[r];
-                    o[g][t] = mfma_tk(pf, read_tr(row + dc, row + 16 * ldv + dc), o[g][t]);
-                }
-            }
-        }
-    }
-    __syncthreads();
-    float* fin = al;                                               // [H]: what the sums are multiplied by
-#pragma unroll
-    for (int j = 0; j < HT; ++j) {
-        const int h = hg + 8 * j;
-        if (h >= H) continue;
-        float l = l_run[j];
-#pragma unroll
-        for (int off = 16; off >= 1; off >>= 1) l += __shfl_xor(l, off, 64);
-        if (key != 0) continue;
-        if (a.nsplit > 1) {
-            float* ml = a.pml + (((size_t)b * H + h) * a.nsplit + s) * 2;
-            ml[0] = m_run[j]; ml[1] = l;
-        } else fin[h] = sink_scale(a.sink, h, m_run[j], l);
-    }
-    if (a.nsplit == 1) __syncthreads();
-#pragma unroll
-    for (int g = 0; g < GM; ++g) {
-        if (g >= G) continue;
-#pragma unroll
-        for (int t = 0; t < RT; ++t)
-#pragma unroll
-            for (int r = 0; r < 4; ++r) {
-                const int hh = 4 * q4 + r, dc = 16 * (wid + 4 * t) + l15, h = g * rep + hh;
-                if (hh >= rep || dc >= D) continue;
-                if (a.nsplit > 1) a.po[(((size_t)b * H + h) * a.nsplit + s) * D + dc] = o[g][t][r];
-                else reinterpret_cast<IT*>(a.out)[(size_t)b * a.ld_out + h * D + dc] = from_f<IT>(o[g][t][r] * fin[h]);
-            }
-    }
-    tls.end();
-}
-
-static bool talk_decode_ok(const TalkArgs& a) {
-    return a.cache && a.D <= 256 && a.H <= 64 && a.H / a.G <= 16 && a.ld_q % 8 == 0 && a.G * ceil_div(a.D, 64) <= 16 && talk_decode_lds(a.H, a.G, a.D) <= (size_t)TALK_LDS_MAX;
-}
-template <class IT>
-static pgk_status talk_decode_mfma(const TalkArgs& a, hipStream_t st) {
-    const size_t lds = talk_decode_lds(a.H, a.G, a.D);
-    auto go = [&](auto um, auto rt) -> pgk_status {
-        auto kfn = &talk_decode_kernel<IT, decltype(um)::value, decltype(rt)::value>;
-        static bool done = false;
-        if (lds > 48 * 1024 && !done) {
-            PGK_CHECK_HIP(hipFuncSetAttribute(reinterpret_cast<const void*>(kfn), hipFuncAttributeMaxDynamicSharedMemorySize, TALK_LDS_MAX));
-            done = true;
-        }
-        PGK_CHECK_HIP(launch_k(kfn, dim3(a.nsplit, a.n), dim3(256), lds, st, a));
-        return PGK_OK;
-    };
-    const int G = a.G;
-    using std::integral_constant;
-    auto pick = [&](auto rt) -> pgk_status {
-        constexpr int RT = decltype(rt)::value;
-        if (G <= 2) return go(integral_constant<int, 2>{}, rt);
-        if (G <= 4) return go(integral_constant<int, 4>{}, rt);
-        if constexpr (RT <= 2) { if (G <= 8) return go(integral_constant<int, 8>{}, rt); }
-        if constexpr (RT == 1) { if (G <= 16) return go(integral_constant<int, 16>{}, rt); }
-        return set_error(PGK_ERR_UNSUPPORTED, "talk_attention: %d key heads of width %d", G, a.D);
-    };
-    return a.D <= 64 ? pick(integral_constant<int, 1>{}) : a.D <= 128 ? pick(integral_constant<int, 2>{}) : pick(integral_constant<int, 4>{});
-}
-
 // over the four quarters of a wave, lane by lane
 __device__ __forceinline__ float max_of_quarters(float x) {
     const auto a = __builtin_amdgcn_permlane16_swap(__float_as_uint(x), __float_as_uint(x), false, false);
     x = fmaxf(__uint_as_float(a[0]), __uint_as_float(a[1]));
     const auto b = __builtin_amdgcn_permlane32_swap(__float_as_uint(x), __float_as_uint(x), false, false);
     return fmaxf(__uint_as_float(b[0]), __uint_as_float(b[1]));
+}
+
+// ---- decode: one query per sequence ----
+// A workgroup per (split, sequence), all heads, 32 keys at a time.  A wave has GW key heads, or WPG waves share one.  Raw scores K q go to
+// LDS as S[head][key]; behind the barrier a wave mixes, in fp32 products S^T T^T of the matrix pipe, the heads of its key head, which
+// leaves a lane with one head and an eighth of the keys: softmax in registers, then O^T[d][head] += V^T P^T, the waves of a key head each
+// with their part of the columns.  Values pass through registers into a part of LDS of the wave's own; keys and values are fetched a step
+// ahead (AHEAD: where they fit the registers).  S exists twice, so one barrier a step is enough.
+constexpr int TD_S = 36;                                           // floats per head of S
+static size_t talk_decode_lds(int nw, int H, int GW, int DW) {
+    return (size_t)2 * ((H + 15) / 16 * 16) * TD_S * 4 + (size_t)nw * GW * 32 * (DW + 8) * 2;
+}
+template <class IT, int GW, int WPG, int RT>
+__global__ __launch_bounds__(512) void talk_decode_kernel(unsigned long long* tl, TalkArgs a) {
+    const TLStamp tls(tl);
+    extern __shared__ __attribute__((aligned(16))) char td_smem[];
+    constexpr int D = 64 * RT, CH = D / 32, DW = D / WPG, DT = DW / 16, PC = DW / 8, NV = 32 * PC / 64, UN = WPG == 1 ? 2 : 1, LDV = DW + 8, KM = 4;
+    constexpr bool AHEAD = GW * RT <= 2 * WPG;
+    constexpr int GB = AHEAD ? GW : 1;                             // key heads in the registers
+    const int H = a.H, G = a.G, rep = H / G, lane = threadIdx.x & 63, l15 = lane & 15, q4 = lane >> 4, s = blockIdx.x, b = blockIdx.y;
+    const int wid = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), nw = blockDim.x >> 6, sub = wid % WPG, gw = wid / WPG;     // the wave's key heads: gw + i nw / WPG
+    const int kmt = (H + 15) / 16, SN = kmt * 16 * TD_S;
+    float* S0 = reinterpret_cast<float*>(td_smem);                // [16 kmt][TD_S], twice
+    bf16* kv = reinterpret_cast<bf16*>(S0 + 2 * SN) + wid * GW * 32 * LDV;     // [GW][32][LDV]
+    int n, lo, k0, k1;
+    ring_window(max(a.positions[b], 0), a.window, a.R, n, lo, a.chunked);
+    split_range(n, a.nsplit, s, k0, k1);
+    if (k0 >= k1) {                                                // an empty split: its record says so, the sums are never read
+        for (int h = threadIdx.x; h < H; h += blockDim.x) {
+            float* ml = a.pml + (((size_t)b * H + h) * a.nsplit + s) * 2;
+            ml[0] = -INFINITY; ml[1] = 0.f;
+        }
+        tls.end();
+        return;
+    }
+    const size_t gstep = (size_t)a.R * D;
+    const bf16* kb = reinterpret_cast<const bf16*>(a.cache) + (size_t)b * 2 * G * gstep;
+    const bf16* vb = kb + G * gstep;
+    auto group = [&](int i) { return min(gw + i * (nw / WPG), G - 1); };       // (key heads past the last repeat it and store nothing)
+    u32x4 qf[GW][CH], kf[GB][UN][CH], st[GB][NV];
+    const int hl = min(l15, rep - 1), u0 = WPG == 1 ? 0 : sub & 1;
+    auto fetch_k = [&](int kt, int i0) {                           // key heads i0 .. i0 + GB
+#pragma unroll
+        for (int u = 0; u < UN; ++u) {
+            const bf16* kr = kb + (size_t)ring_row(lo, min(kt + 16 * (u0 + u) + l15, k1 - 1), a.R) * D + 8 * q4;
+#pragma unroll
+            for (int i = 0; i < GB; ++i)
+#pragma unroll
+                for (int c = 0; c < CH; ++c) kf[i][u][c] = *reinterpret_cast<const u32x4*>(kr + group(i0 + i) * gstep + 32 * c);
+        }
+    };
+    auto fetch_v = [&](int kt, int i0) {
+#pragma unroll
+        for (int v = 0; v < NV; ++v) {
+            const int p = v * 64 + lane;
+            const bf16* vr = vb + (size_t)ring_row(lo, min(kt + p / PC, k1 - 1), a.R) * D + sub * DW + p % PC * 8;
+#pragma unroll
+            for (int i = 0; i < GB; ++i) st[i][v] = *reinterpret_cast<const u32x4*>(vr + group(i0 + i) * gstep);
+        }
+    };
+    // T as operand: column l15 is the head's, steps go through the raw heads 16 k + 4 q4 + j; zero where there is none
+    f32x4_tk tf[GW][KM];
+#pragma unroll
+    for (int i = 0; i < GW; ++i) {
+        const int h = group(i) * rep + hl;
+#pragma unroll
+        for (int k = 0; k < KM; ++k) {
+            tf[i][k] = f32x4_tk{0.f, 0.f, 0.f, 0.f};
+            if (k >= kmt) continue;                                // uniform
+#pragma unroll
+            for (int j = 0; j < 4; ++j) {
+                const int g = 16 * k + 4 * q4 + j;
+                tf[i][k][j] = a.talk ? a.talk[(size_t)h * H + min(g, H - 1)] : h == g ? 1.0f : 0.f;
+            }
+        }
+    }
+    if (AHEAD) fetch_k(k0, 0);
+#pragma unroll
+    for (int i = 0; i < GW; ++i) {
+        const bf16* qr = reinterpret_cast<const bf16*>(a.q) + (size_t)b * a.ld_q + (size_t)(group(i) * rep + hl) * D + 8 * q4;
+#pragma unroll
+        for (int c = 0; c < CH; ++c) qf[i][c] = *reinterpret_cast<const u32x4*>(qr + 32 * c);
+    }
+    if (AHEAD) fetch_v(k0, 0);
+    const float mult = a.scale * TK_LOG2E;
+#pragma unroll
+    for (int i = 0; i < GW; ++i)
+#pragma unroll
+        for (int k = 0; k < KM; ++k)
+#pragma unroll
+            for (int j = 0; j < 4; ++j) tf[i][k][j] = 16 * k + 4 * q4 + j < H ? tf[i][k][j] * mult : 0.f;
+    for (int i = H * TD_S + threadIdx.x; i < SN; i += blockDim.x) { S0[i] = 0.f; S0[SN + i] = 0.f; }      // heads that do not exist
+    f32x4_tk o[GW][DT];
+    float m[GW], l[GW];
+#pragma unroll
+    for (int i = 0; i < GW; ++i) {
+        m[i] = -INFINITY; l[i] = 0.f;
+#pragma unroll
+        for (int t = 0; t < DT; ++t) o[i][t] = f32x4_tk{0.f, 0.f, 0.f, 0.f};
+    }
+    float* S = S0;
+    for (int kt = k0; kt < k1; kt += 32) {
+        if (WPG <= 2 || sub < 2) {                                 // uniform: two waves have the two halves of the keys
+#pragma unroll
+            for (int i = 0; i < GW; ++i) {
+                if (!AHEAD) fetch_k(kt, i);
+#pragma unroll
+                for (int u = 0; u < UN; ++u) {
+                    f32x4_tk t = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+                    for (int c = 0; c < CH; ++c) t = mfma_tk(kf[AHEAD ? i : 0][u][c], qf[i][c], t);
+                    if (l15 < rep) *reinterpret_cast<f32x4_tk*>(S + (group(i) * rep + l15) * TD_S + 16 * (u0 + u) + 4 * q4) = t;      // keys 16 u + 4 q4 .. of head l15
+                }
+                if (!AHEAD) __builtin_amdgcn_sched_barrier(0);
+            }
+        }
+        if (AHEAD && kt + 32 < k1) fetch_k(kt + 32, 0);            // the next tile travels under the rest of this one
+        wave_sync();                                               // (the last step's reads of the values)
+#pragma unroll
+        for (int i = 0; i < GW; ++i) {
+            if (!AHEAD) fetch_v(kt, i);
+#pragma unroll
+            for (int v = 0; v < NV; ++v) {
+                const int p = v * 64 + lane;
+                *reinterpret_cast<u32x4*>(kv + (i * 32 + p / PC) * LDV + p % PC * 8) = st[AHEAD ? i : 0][v];
+            }
+            if (!AHEAD) __builtin_amdgcn_sched_barrier(0);
+        }
+        if (AHEAD && kt + 32 < k1) fetch_v(kt + 32, 0);
+        asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+        __builtin_amdgcn_s_barrier();                              // (loads stay in flight)
+        asm volatile("" ::: "memory");
+        const float* sk = S + 4 * q4 * TD_S + l15;
+        f32x4_tk x[GW][2];
+#pragma unroll
+        for (int i = 0; i < GW; ++i) { x[i][0] = f32x4_tk{0.f, 0.f, 0.f, 0.f}; x[i][1] = x[i][0]; }
+#pragma unroll
+        for (int k = 0; k < KM; ++k) {
+            if (k >= kmt) continue;                                // uniform
+#pragma unroll
+            for (int j = 0; j < 4; ++j)
+#pragma unroll
+                for (int u = 0; u < 2; ++u) {
+                    const float r = sk[(16 * k + j) * TD_S + 16 * u];
+#pragma unroll
+                    for (int i = 0; i < GW; ++i) x[i][u] = __builtin_amdgcn_mfma_f32_16x16x4f32(r, tf[i][k][j], x[i][u], 0, 0, 0);
+                }
+        }
+        const int seen = k1 - kt - 4 * q4;
+#pragma unroll
+        for (int i = 0; i < GW; ++i) {
+            f32x4_tk s0 = x[i][0], s1 = x[i][1];
+            if (kt + 32 > k1) {
+#pragma unroll
+                for (int e = 0; e < 4; ++e) {
+                    if (e >= seen) s0[e] = -INFINITY;
+                    if (e + 16 >= seen) s1[e] = -INFINITY;
+                }
+            }
+            const float top = max_of_quarters(fmaxf(fmaxf(fmaxf(s0[0], s0[1]), fmaxf(s0[2], s0[3])), fmaxf(fmaxf(s1[0], s1[1]), fmaxf(s1[2], s1[3]))));
+            const float mn = fmaxf(m[i], top), f = __builtin_amdgcn_exp2f(m[i] - mn);        // mn is finite: kt < k1
+            m[i] = mn;
+#pragma unroll
+            for (int e = 0; e < 4; ++e) {
+                s0[e] = __builtin_amdgcn_exp2f(s0[e] - mn);
+                s1[e] = __builtin_amdgcn_exp2f(s1[e] - mn);
+            }
+            l[i] = fmaf(l[i], f, ((s0[0] + s0[1]) + (s0[2] + s0[3])) + ((s1[0] + s1[1]) + (s1[2] + s1[3])));
+            const uint4 pf = make_uint4(pack_bf16x2(s0[0], s0[1]), pack_bf16x2(s0[2], s0[3]), pack_bf16x2(s1[0], s1[1]), pack_bf16x2(s1[2], s1[3]));
+            const bf16* row = kv + (i * 32 + 4 * q4 + (l15 >> 2)) * LDV + 4 * (l15 & 3);
+#pragma unroll
+            for (int t = 0; t < DT; ++t) o[i][t] = mfma_tk(read_tr(row + 16 * t, row + 16 * LDV + 16 * t), pf, o[i][t] * f);
+        }
+        S = S == S0 ? S0 + SN : S0;
+    }
+#pragma unroll
+    for (int i = 0; i < GW; ++i) {
+        float sum = l[i];
+        sum += __shfl_xor(sum, 16, 64);
+        sum += __shfl_xor(sum, 32, 64);
+        const int g = gw + i * (nw / WPG), h = g * rep + l15, d0 = sub * DW + 4 * q4;
+        if (g >= G || l15 >= rep) continue;
+        if (a.nsplit > 1) {
+            const size_t rec = ((size_t)b * H + h) * a.nsplit + s;
+            if (sub == 0 && q4 == 0) *reinterpret_cast<float2*>(a.pml + rec * 2) = make_float2(m[i], sum);
+            float* po = a.po + rec * D + d0;
+#pragma unroll
+            for (int t = 0; t < DT; ++t) *reinterpret_cast<f32x4_tk*>(po + 16 * t) = o[i][t];
+        } else {
+            const float f = sink_scale(a.sink, h, m[i], sum);
+            IT* out = reinterpret_cast<IT*>(a.out) + (size_t)b * a.ld_out + h * D + d0;
+#pragma unroll
+            for (int t = 0; t < DT; ++t) store4<IT>(out + 16 * t, make_float4(o[i][t][0] * f, o[i][t][1] * f, o[i][t][2] * f, o[i][t][3] * f));
+        }
+    }
+    tls.end();
+}
+
+static bool talk_decode_ok(const TalkArgs& a) {
+    return a.cache && a.D % 64 == 0 && a.D <= (a.G > 8 ? 128 : 256) && a.H <= 64 && a.G <= 16 && a.H / a.G <= 16 && a.ld_q % 8 == 0 && a.ld_out % 4 == 0 && aligned16(a.q) && aligned16(a.out);
+}
+template <class IT>
+static pgk_status talk_decode_mfma(const TalkArgs& a, hipStream_t st) {
+    auto go = [&](auto gw, auto wpg, auto rt) -> pgk_status {
+        constexpr int GW = decltype(gw)::value, WPG = decltype(wpg)::value, RT = decltype(rt)::value;
+        auto kfn = &talk_decode_kernel<IT, GW, WPG, RT>;
+        const int nw = GW > 1 ? 8 : min(8, a.G * WPG);
+        const size_t lds = talk_decode_lds(nw, a.H, GW, 64 * RT / WPG);
+        static bool done = false;
+        if (lds > 48 * 1024 && !done) {
+            PGK_CHECK_HIP(hipFuncSetAttribute(reinterpret_cast<const void*>(kfn), hipFuncAttributeMaxDynamicSharedMemorySize, TALK_LDS_MAX + 8 * 1024));
+            done = true;
+        }
+        PGK_CHECK_HIP(launch_k(kfn, dim3(a.nsplit, a.n), dim3(64 * nw), lds, st, a));
+        return PGK_OK;
+    };
+    using std::integral_constant;
+    integral_constant<int, 1> one;
+    integral_constant<int, 2> two;
+    integral_constant<int, 4> four;
+    auto pick = [&](auto rt) -> pgk_status {
+        if constexpr (decltype(rt)::value <= 2) { if (a.G > 8) return go(two, one, rt); }
+        return a.G <= 2 ? go(one, four, rt) : a.G <= 4 ? go(one, two, rt) : go(one, one, rt);
+    };
+    switch (a.D / 64) {
+        case 1: return pick(one);
+        case 2: return pick(two);
+        case 3: return pick(integral_constant<int, 3>{});
+        default: return pick(four);
+    }
 }
 
 // ---- prompts: 16 queries per workgroup, 32 keys at a time ----
@@ -782,7 +798,7 @@ pgk_status pgk_talk_attention(const void* q, const void* k, const void* v, const
     PGK_REQUIRE(hq >= 1 && hkv >= 1 && kv_len >= q_len, "pgk_talk_attention: %d / %d heads, %d keys", hq, hkv, kv_len);
     TalkArgs a{};
     a.q = q; a.ld_q = hq * dk; a.talk = talk; a.sink = sink; a.H = hq; a.G = hkv; a.D = dk; a.n = q_len; a.window = window; a.chunked = chunked; a.scale = scale; a.nsplit = 1;
-    a.k = k; a.v = v; a.ld_kv = hkv * dk; a.kv_len = kv_len; a.pos0 = first; a.out = out; a.ld_out = hq * dv; a.Dv = dv; a.ld_v = hkv * dv;
+    a.k = k; a.v = v; a.ld_kv = hkv * dk; a.kv_len = kv_len; a.pos0 = first; a.out = out; a.ld_out = hq * dv; a.Dv = dk == dv && dk % 64 == 0 ? 0 : dv; a.ld_v = hkv * dv;      // (0: as wide, in the same rows)
     int launches = 0;
     return talk_attention(a, dt, dt == PGK_F32, resolve_stream(s), &launches);
 }
