@@ -234,16 +234,23 @@ __global__ __launch_bounds__(256) void stack_gemv_kernel(unsigned long long* tl,
                 if (i < C * CH) store4<WT>(xs + i, i < K ? make_float4(v[t].x * gm[t].x, v[t].y * gm[t].y, v[t].z * gm[t].z, v[t].w * gm[t].w) : zero);
             }
         } else {
-            for (int i = threadIdx.x; i < K; i += 256) {
-                const float y = a.y ? a.y[i] : 0.f;
-                float u = cy * y;
-                for (int s = 0; s < S; ++s) u = fmaf(coef_x(s), a.x[(size_t)s * a.x_stream + i], u);
-                xf[i] = u;
+            float* cx = xf + K + a.groups;                         // [S]
+            for (int s = threadIdx.x; s < S; s += 256) cx[s] = coef_x(s);
+            __syncthreads();
+            const float4 zero = {0.f, 0.f, 0.f, 0.f};
+            auto mul = [](float c, const float4& p, const float4& q) { return make_float4(fmaf(c, p.x, q.x), fmaf(c, p.y, q.y), fmaf(c, p.z, q.z), fmaf(c, p.w, q.w)); };
+            for (int i = threadIdx.x * 4; i < K; i += 1024) {
+                const float* xi = a.x + i;
+                const float4 y = a.y ? *reinterpret_cast<const float4*>(a.y + i) : zero;
+                float4 u = mul(cy, y, zero);
+#pragma unroll 4
+                for (int s = 0; s < S; ++s) u = mul(cx[s], *reinterpret_cast<const float4*>(xi + (size_t)s * a.x_stream), u);
+                *reinterpret_cast<float4*>(xf + i) = u;
                 if (a.y && a.x_out && blockIdx.x == (i >> 10) % gridDim.x)
                     for (int o = 0; o < S; ++o) {
-                        float z = a.upd[S + o] * y;
-                        for (int s = 0; s < S; ++s) z = fmaf(a.upd[2 * S + s * S + o], a.x[(size_t)s * a.x_stream + i], z);
-                        a.x_out[(size_t)o * K + i] = z;
+                        float4 z = mul(a.upd[S + o], y, zero);
+                        for (int s = 0; s < S; ++s) z = mul(a.upd[2 * S + s * S + o], *reinterpret_cast<const float4*>(xi + (size_t)s * a.x_stream), z);
+                        *reinterpret_cast<float4*>(a.x_out + (size_t)o * K + i) = z;
                     }
             }
             __syncthreads();
@@ -463,6 +470,16 @@ __global__ __launch_bounds__(256) void stack_gemv_kernel(unsigned long long* tl,
         }
 #pragma unroll
         for (int r = 0; r < R; ++r) acc[r][0] = wave_sum(acc[r][0]);
+        if constexpr (EPI == SE_LOGITS) {
+            if (a.cap > 0.f) {                                     // every lane has the sums: lane r caps row r's
+                float v = acc[0][0];
+#pragma unroll
+                for (int r = 1; r < R; ++r) if (lane == r) v = acc[r][0];
+                v = soft_cap(v, a.cap);
+#pragma unroll
+                for (int r = 0; r < R; ++r) acc[r][0] = __shfl(v, r, 64);
+            }
+        }
         if (lane == 0) {
 #pragma unroll
             for (int r = 0; r < OUT; ++r)
@@ -471,7 +488,6 @@ __global__ __launch_bounds__(256) void stack_gemv_kernel(unsigned long long* tl,
                     if constexpr (EPI == SE_SWIGLU) o = o / (1.0f + (std::is_same<WT, float>::value ? expf(-o) : __expf(-o))) * acc[r + R / 2][0];
                     if constexpr (EPI == SE_XIELU) o = xielu<std::is_same<WT, float>::value>(o, a.act_pos, a.act_neg);
                     if constexpr (EPI == SE_STORE) { if (a.bias) o += a.bias[n0 + r]; }
-                    if constexpr (EPI == SE_LOGITS) { if (a.cap > 0.f) o = soft_cap(o, a.cap); }
                     if constexpr (EPI == SE_TABLE) {
                         const int j = n0 + r - a.fs;
                         o = j >= a.top * a.ff ? 1.0f / (1.0f + expf(-o)) : j < 0 ? gelu_erf(o) : gelu_erf(o) / a.top;
@@ -500,7 +516,7 @@ template <class WT, int R, int PRO, int EPI, int C>
 static pgk_status stack_gemv_c(const StackGemvArgs& a, int grid, hipStream_t st) {
     constexpr int CH = 64 * WTraits<WT>::NW;
     size_t lds = (size_t)ceil_div(a.K, CH) * CH * sizeof(WT) > (size_t)C * CH * sizeof(WT) ? (size_t)ceil_div(a.K, CH) * CH * sizeof(WT) : (size_t)C * CH * sizeof(WT);
-    if (PRO == SP_HYPER && (C == 0 || a.groups > 1)) lds += (size_t)(a.K + a.groups) * 4;
+    if (PRO == SP_HYPER && (C == 0 || a.groups > 1)) lds += (size_t)(a.K + a.groups + a.S) * 4;
     auto kfn = &stack_gemv_kernel<WT, R, PRO, EPI, C>;
     PGK_REQUIRE(lds <= 156 * 1024, "engine: a row of %d does not fit LDS", a.K);
     static bool attr_done = false;
@@ -526,14 +542,22 @@ static pgk_status stack_gemv_r(const StackGemvArgs& a, hipStream_t st, int force
     return stack_gemv_c<WT, R, PRO, EPI, 0>(a, grid, st);
 }
 
+// A wide row of several streams: two rows a wave, so that the streams stay in registers, and no more workgroups than are resident, since
+// every one reads all streams
+constexpr int HYPER_WIDE_GRID = 512;
+static bool hyper_wide(int K) { return K > 2048 && K <= 4096; }
+
 template <class WT, int PRO, int EPI>
 static pgk_status stack_gemv(const StackGemvArgs& a, hipStream_t st, int force_grid = 0) {
     if constexpr (std::is_same<WT, float>::value) return stack_gemv_r<WT, EPI == SE_STORE || EPI == SE_XIELU ? 1 : 2, PRO, EPI>(a, st, force_grid);
     else if constexpr (EPI == SE_SWIGLU) {
         if (a.N >= 4096) return stack_gemv_r<WT, 4, PRO, EPI>(a, st);
         return stack_gemv_r<WT, 2, PRO, EPI>(a, st);
-    } else if constexpr (EPI == SE_LOGITS) return stack_gemv_r<WT, 4, PRO, EPI>(a, st, force_grid);
-    else {
+    } else if constexpr (EPI == SE_LOGITS) {
+        if constexpr (PRO == SP_HYPER) { if (hyper_wide(a.K)) return stack_gemv_r<WT, 2, PRO, EPI>(a, st, force_grid); }
+        return stack_gemv_r<WT, 4, PRO, EPI>(a, st, force_grid);
+    } else {
+        if (PRO == SP_HYPER && hyper_wide(a.K)) return stack_gemv_r<WT, 2, PRO, EPI>(a, st, min(ceil_div(a.N, 8), HYPER_WIDE_GRID));
         if (a.N >= 8192) return stack_gemv_r<WT, 4, PRO, EPI>(a, st);
         if (a.N >= 2048) return stack_gemv_r<WT, 2, PRO, EPI>(a, st);
         return stack_gemv_r<WT, 1, PRO, EPI>(a, st);
@@ -2462,6 +2486,7 @@ pgk_status pgk_engine_create_stack(const pgk_stack_config_t* cfg, const void* em
         if (hipGetDevice(&dev) == hipSuccess && hipGetDeviceProperties(&prop, dev) == hipSuccess && prop.multiProcessorCount > 0) e->cu_count = prop.multiProcessorCount;
     }
     e->lm_blocks = ceil_div(c.vocab_size, 16) < 1024 ? ceil_div(c.vocab_size, 16) : 1024;
+    if (c.block == PGK_BLOCK_HYPER && hyper_wide(s->Wp)) e->lm_blocks = min(e->lm_blocks, HYPER_WIDE_GRID);
     e->lm_cap = e->lm_blocks > ROWS_ARGMAX_BLOCKS ? e->lm_blocks : ROWS_ARGMAX_BLOCKS;
     pgk_status r = PGK_OK;
     std::vector<std::pair<void*, size_t>> clear;
