@@ -141,14 +141,15 @@ pgk_status hyper_rows(const HyperArgs& a, int n, pgk_dtype dt, hipStream_t st) {
 // NT groups of four per thread stay in registers; NT 0: any width, the row is read twice
 template <class T, int NT>
 __global__ __launch_bounds__(256) void poly_rows_kernel(const T* z, T* out, int W, int ld, const float* act, float eps) {
-    __shared__ float red[3][16];
+    __shared__ float red[3][4];
     const T* zr = z + (size_t)blockIdx.x * ld;
     T* o = out + (size_t)blockIdx.x * ld;
     float4 v[NT > 0 ? NT : 1];
     float s2 = 0.f, s4 = 0.f, s6 = 0.f;
     auto add = [&](float x) { const float x2 = x * x, x4 = x2 * x2; s2 += x2; s4 += x4; s6 = fmaf(x4, x2, s6); };
     auto put = [&](int i, const float4& q, const float3& c, float e) {
-        store4<T>(o + i, make_float4(i < W ? poly_at(c, e, q.x) : 0.f, i + 1 < W ? poly_at(c, e, q.y) : 0.f, i + 2 < W ? poly_at(c, e, q.z) : 0.f, i + 3 < W ? poly_at(c, e, q.w) : 0.f));
+        if (i + 3 < W) store4<T>(o + i, make_float4(poly_at(c, e, q.x), poly_at(c, e, q.y), poly_at(c, e, q.z), poly_at(c, e, q.w)));
+        else store4<T>(o + i, make_float4(i < W ? poly_at(c, e, q.x) : 0.f, i + 1 < W ? poly_at(c, e, q.y) : 0.f, i + 2 < W ? poly_at(c, e, q.z) : 0.f, i + 3 < W ? poly_at(c, e, q.w) : 0.f));
     };
     if constexpr (NT > 0) {
 #pragma unroll
@@ -160,7 +161,11 @@ __global__ __launch_bounds__(256) void poly_rows_kernel(const T* z, T* out, int 
     } else {
         for (int i = threadIdx.x; i < W; i += 256) add(to_f(zr[i]));
     }
-    s2 = block_sum(s2, red[0]); s4 = block_sum(s4, red[1]); s6 = block_sum(s6, red[2]);
+    s2 = wave_sum(s2); s4 = wave_sum(s4); s6 = wave_sum(s6);
+    if ((threadIdx.x & 63) == 0) { red[0][threadIdx.x >> 6] = s2; red[1][threadIdx.x >> 6] = s4; red[2][threadIdx.x >> 6] = s6; }
+    __syncthreads();
+    auto total = [&](int i) { return (red[i][0] + red[i][1]) + (red[i][2] + red[i][3]); };
+    s2 = total(0); s4 = total(1); s6 = total(2);
     const float3 c = poly_coef(act, s2, s4, s6, W, eps);
     const float e = act[3];
     if constexpr (NT > 0) {
@@ -177,6 +182,8 @@ template <class T>
 static void poly_rows_t(const T* z, T* out, int n, int W, int ld, const float* act, float eps, hipStream_t st) {
     if (ld % 4 != 0) poly_rows_kernel<T, 0><<<n, 256, 0, st>>>(z, out, W, ld, act, eps);
     else if (ld <= 4096) poly_rows_kernel<T, 4><<<n, 256, 0, st>>>(z, out, W, ld, act, eps);
+    else if (ld <= 8192) poly_rows_kernel<T, 8><<<n, 256, 0, st>>>(z, out, W, ld, act, eps);
+    else if (ld <= 12288) poly_rows_kernel<T, 12><<<n, 256, 0, st>>>(z, out, W, ld, act, eps);
     else if (ld <= 16384) poly_rows_kernel<T, 16><<<n, 256, 0, st>>>(z, out, W, ld, act, eps);
     else poly_rows_kernel<T, 0><<<n, 256, 0, st>>>(z, out, W, ld, act, eps);
 }

@@ -2,6 +2,7 @@
 // step before it: bias, norm per head and rotation of projection rows.
 
 #include <type_traits>
+#include <vector>
 
 #include "mixers.hip.h"
 
@@ -497,13 +498,21 @@ static pgk_status talk_decode_mfma(const TalkArgs& a, hipStream_t st) {
 // V^T P^T.  Keys, then values, of a wave's key head come as whole rows through registers (fetched a step ahead) into a part of LDS of the
 // wave's own, in 16-byte pieces that are XOR-ed by the row, so that operand reads of 16 rows spread over the banks.  DB: S exists twice, so
 // that no wave waits for the others' step 3.  ONE: the heads of a wave share a key head.  Heads past the last repeat it and store nothing.
+// blockIdx.z: which `part` tiles of 32 keys; queries with several such parts leave, per part, a normalised output and (m, l), which
+// talk_join_kernel combines.
 constexpr int TF_Q = 36, TF_H = 16 * TF_Q;                         // floats per query and head of S
 static size_t talk_flash_lds(int NW, int HW, int HO, int D, bool db) {
     return (size_t)NW * HW * TF_H * 4 * (db ? 2 : 1) + (size_t)(NW * HO + 15) / 16 * 16 * (NW * HW + 4) * 4 + (size_t)NW * 32 * D * 2;
 }
 
+struct TalkParts { int part; bf16* o; float2* ml; };               // o [parts][n][H D], ml [parts][n][H]
+__device__ __forceinline__ int talk_first_key(const TalkArgs& a, int q) {
+    const int last = a.kv_len - a.n + q;
+    return last + 1 - min(span_keys(a.pos0 + last, a.window, a.chunked), last + 1);
+}
+
 template <int NW, int HW, int HO, int RT, bool ONE, bool DB>
-__global__ __launch_bounds__(64 * NW, 2) void talk_flash_kernel(unsigned long long* tl, TalkArgs a, int tiles, int per) {
+__global__ __launch_bounds__(64 * NW, 2) void talk_flash_kernel(unsigned long long* tl, TalkArgs a, int tiles, int per, TalkParts pt) {
     const TLStamp tls(tl);
     extern __shared__ __attribute__((aligned(16))) char tf_smem[];
     constexpr int D = 64 * RT, CH = D / 32, DT = D / 16, HM = (NW * HO + 15) / 16, KS = NW * HW / 4, PC = D / 8, TL = NW * HW + 4, SN = NW * HW * TF_H;
@@ -517,9 +526,10 @@ __global__ __launch_bounds__(64 * NW, 2) void talk_flash_kernel(unsigned long lo
     const int runs = (tiles + per - 1) / per, tile = (int)(blockIdx.x % runs) * per + per - 1 - (int)(blockIdx.x / runs);
     if (tile >= tiles) { tls.end(); return; }
     const int q0 = tile * 16, nq = min(16, a.n - q0), past = a.kv_len - a.n;
-    auto first_key = [&](int q) { const int last = past + q; return last + 1 - min(span_keys(a.pos0 + last, a.window, a.chunked), last + 1); };
-    const int my_q = q0 + min(l15, nq - 1), my_lo = first_key(my_q), my_last = past + my_q;
-    const int k_begin = first_key(q0), k_end = past + q0 + nq, lo_max = first_key(q0 + nq - 1), last_min = past + q0;
+    const int my_q = q0 + min(l15, nq - 1), my_lo = talk_first_key(a, my_q), my_last = past + my_q;
+    const int k_first = talk_first_key(a, q0), k_last = past + q0 + nq, lo_max = talk_first_key(a, q0 + nq - 1), last_min = past + q0;
+    const int k_begin = k_first + (int)blockIdx.z * pt.part * 32, k_end = min(k_last, k_begin + pt.part * 32);
+    if (k_begin >= k_last) { tls.end(); return; }
     const bf16 *kbase = reinterpret_cast<const bf16*>(a.k), *vbase = reinterpret_cast<const bf16*>(a.v);
     auto head = [&](int i) { return min(wid * HW + i, H - 1); };
     auto out_head = [&](int i) { return min(ho0 + wid * HO + i, H - 1); };
@@ -687,12 +697,51 @@ __global__ __launch_bounds__(64 * NW, 2) void talk_flash_kernel(unsigned long lo
         float sum = l[i];
         sum += __shfl_xor(sum, 16, 64);
         sum += __shfl_xor(sum, 32, 64);
-        const float f = sink_scale(a.sink, out_head(i), m[i], sum);
-        if (l15 >= nq || ho0 + wid * HO + i >= H) continue;
-        bf16* out = reinterpret_cast<bf16*>(a.out) + (size_t)(q0 + l15) * a.ld_out + (size_t)(ho0 + wid * HO + i) * D + 4 * q4;
+        const bool join = k_last - k_first > pt.part * 32;         // uniform
+        const float f = join ? (sum > 0.f ? 1.0f / sum : 0.f) : sink_scale(a.sink, out_head(i), m[i], sum);
+        const int h = ho0 + wid * HO + i;
+        if (l15 >= nq || h >= H) continue;
+        bf16* out = reinterpret_cast<bf16*>(a.out) + (size_t)(q0 + l15) * a.ld_out + (size_t)h * D + 4 * q4;
+        if (join) {
+            const size_t row = (size_t)blockIdx.z * a.n + q0 + l15;
+            if (q4 == 0) pt.ml[row * H + h] = make_float2(m[i], sum);
+            out = pt.o + (row * H + h) * D + 4 * q4;
+        }
 #pragma unroll
         for (int t = 0; t < DT; ++t) store4<bf16>(out + 16 * t, make_float4(o[i][t][0] * f, o[i][t][1] * f, o[i][t][2] * f, o[i][t][3] * f));
     }
+    tls.end();
+}
+
+// A workgroup per query, eight columns per thread
+__global__ __launch_bounds__(256) void talk_join_kernel(unsigned long long* tl, TalkArgs a, TalkParts pt) {
+    const TLStamp tls(tl);
+    const int q = blockIdx.x, q0 = q / 16 * 16, n = (a.kv_len - a.n + min(q0 + 16, a.n) - talk_first_key(a, q0) + pt.part * 32 - 1) / (pt.part * 32);
+    if (n > 1)
+        for (int i = threadIdx.x; i < a.H * a.D / 8; i += 256) {
+            const int h = i * 8 / a.D;
+            const float2* ml = pt.ml + (size_t)q * a.H + h;
+            float m = -INFINITY;
+            for (int p = 0; p < n; ++p) m = fmaxf(m, ml[(size_t)p * a.n * a.H].x);
+            float l = 0.f, o[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
+#pragma unroll 4
+            for (int p = 0; p < n; ++p) {
+                const float2 r = ml[(size_t)p * a.n * a.H];
+                const float w = r.y * __builtin_amdgcn_exp2f(r.x - m);         // (every query sees itself: m is finite)
+                const uint4 v = *reinterpret_cast<const uint4*>(pt.o + ((size_t)p * a.n + q) * a.H * a.D + i * 8);
+                const uint32_t* u = &v.x;
+                l += w;
+#pragma unroll
+                for (int j = 0; j < 4; ++j) {
+                    o[2 * j] = fmaf(w, __uint_as_float(u[j] << 16), o[2 * j]);
+                    o[2 * j + 1] = fmaf(w, __uint_as_float(u[j] & 0xffff0000u), o[2 * j + 1]);
+                }
+            }
+            const float f = sink_scale(a.sink, h, m, l);
+            bf16* out = reinterpret_cast<bf16*>(a.out) + (size_t)q * a.ld_out + i * 8;
+            store4<bf16>(out, make_float4(o[0] * f, o[1] * f, o[2] * f, o[3] * f));
+            store4<bf16>(out + 4, make_float4(o[4] * f, o[5] * f, o[6] * f, o[7] * f));
+        }
     tls.end();
 }
 
@@ -700,7 +749,42 @@ static bool talk_flash_ok(const TalkArgs& a) {
     return !a.cache && !a.Dv && (a.D == 64 || a.D == 128) && a.H <= 32 && a.ld_q % 8 == 0 && a.ld_kv % 8 == 0 && a.ld_out % 4 == 0 && aligned16(a.q) && aligned16(a.k) && aligned16(a.v) &&
            (reinterpret_cast<uintptr_t>(a.out) & 7u) == 0;
 }
-static pgk_status talk_flash(const TalkArgs& a, hipStream_t st) {
+static int cu_count() {
+    static const int n = [] {
+        int dev = 0;
+        hipDeviceProp_t prop;
+        return hipGetDevice(&dev) == hipSuccess && hipGetDeviceProperties(&prop, dev) == hipSuccess && prop.multiProcessorCount > 0 ? prop.multiProcessorCount : 256;
+    }();
+    return n;
+}
+// Parts of the heaviest query tile's keys, and the 32-key tiles of one.  One workgroup fits a CU, so a launch ends with its longest
+// workgroup: where CUs idle or the heaviest tiles outlast the mean, more parts pay, until their overhead and the joining do not.  Counted in
+// times of a tile (about 3 us).
+static int plan_parts(const TalkArgs& a, int tiles, int groups, int cus, int* part) {
+    std::vector<int> keys(tiles);
+    int most = 1;
+    long long all = 0;
+    for (int t = 0; t < tiles; ++t) {
+        const int last = a.kv_len - a.n + 16 * t, seen = span_keys(a.pos0 + last, a.window, a.chunked), own = a.n - 16 * t < 16 ? a.n - 16 * t : 16;
+        keys[t] = ceil_div((seen < last + 1 ? seen : last + 1) + own - 1, 32);
+        all += keys[t];
+        if (keys[t] > most) most = keys[t];
+    }
+    int best = 1;
+    double best_cost = 0.0;
+    for (int k = 1; k <= 16 && k <= most; ++k) {
+        const int p = ceil_div(most, k);
+        long long wgs = 0, joined = 0;
+        for (int t : keys) { const int c = ceil_div(t, p); wgs += c; if (c > 1) joined += c; }
+        const double lead = 3.0, alone = p + lead, shared = wgs * groups <= cus ? 0.0 : (double)(all + lead * wgs) * groups / cus + 2.0;
+        const double join = k == 1 ? 0.0 : 1.7 + (double)joined * 16 * a.H * a.D * 4 / 12e6;
+        const double cost = (alone > shared ? alone : shared) + join;
+        if (k == 1 || cost < best_cost) { best = k; best_cost = cost; }
+    }
+    *part = ceil_div(most, best);
+    return ceil_div(most, *part);
+}
+static pgk_status talk_flash(const TalkArgs& a, hipStream_t st, int* launches) {
     const int tiles = ceil_div(a.n, 16), rep = a.H / a.G;
     const int per = a.chunked && a.window / 16 >= 1 && a.window / 16 < tiles ? a.window / 16 : tiles, runs = ceil_div(tiles, per);
     auto go = [&](auto nw, auto hw, auto ho, auto rt, auto one, auto db) -> pgk_status {
@@ -712,7 +796,21 @@ static pgk_status talk_flash(const TalkArgs& a, hipStream_t st) {
             PGK_CHECK_HIP(hipFuncSetAttribute(reinterpret_cast<const void*>(kfn), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds));
             done = true;
         }
-        PGK_CHECK_HIP(launch_k(kfn, dim3(runs * per, ceil_div(a.H, NW * HO)), dim3(64 * NW), lds, st, a, tiles, per));
+        TalkParts pt{};
+        const int groups = ceil_div(a.H, NW * HO), parts = plan_parts(a, tiles, groups, cu_count(), &pt.part);
+        void* ws = nullptr;
+        if (parts > 1) {
+            const size_t rows = (size_t)parts * a.n * a.H, o_bytes = (rows * a.D * 2 + 255) & ~(size_t)255;
+            if (pgk_status r = pgk_malloc(&ws, o_bytes + rows * sizeof(float2))) return r;
+            pt.o = (bf16*)ws; pt.ml = (float2*)((char*)ws + o_bytes);
+        }
+        hipError_t err = launch_k(kfn, dim3(runs * per, groups, parts), dim3(64 * NW), lds, st, a, tiles, per, pt);
+        if (ws) {
+            if (err == hipSuccess) err = launch_k(&talk_join_kernel, dim3(a.n), dim3(256), 0, st, a, pt);
+            *launches += 1;
+            pgk_free(ws);                                          // (what takes it next runs behind these kernels)
+        }
+        PGK_CHECK_HIP(err);
         return PGK_OK;
     };
     using std::integral_constant;
@@ -745,7 +843,7 @@ pgk_status talk_attention(const TalkArgs& a, pgk_dtype dt, bool io32, hipStream_
     pgk_status r;
     if (dt == PGK_F32) r = talk_any<float, float>(a, st);
     else if (talk_decode_ok(a)) r = io32 ? talk_decode_mfma<float>(a, st) : talk_decode_mfma<bf16>(a, st);
-    else if (!io32 && talk_flash_ok(a)) r = talk_flash(a, st);
+    else if (!io32 && talk_flash_ok(a)) r = talk_flash(a, st, launches);
     else r = io32 ? talk_any<bf16, float>(a, st) : talk_any<bf16, bf16>(a, st);
     if (r) return r;
     *launches += 1;
