@@ -70,8 +70,14 @@ CONFIGS = {
     # many heads and streams; near one-hot attention over hundreds of keys
     "deep": config(64, 90, [(attn(8, 4, 64, 64, 32, 300), moe(96, 6, 32, 40)), (attn(33, 3, 16, 48, 8, 350), None), (attn(24, 8, 64, 64, 64, 256), poly(90)), (attn(24, 8, 64, 64, 64, 500, kv_from=2), None)],
                    6, 2, cap=2.0),
+    # numbers of key heads and widths for every shape of the decode kernel, and past them
+    "heads": config(96, 110, [(attn(12, 12, 64, 64, 64, 48), None), (attn(16, 16, 128, 100, 32, 70), poly(64)), (attn(5, 5, 144, 180, 100, 40), None), (attn(8, 8, 200, 256, 200, 90), None),
+                              (attn(18, 18, 40, 64, 20, 30), None), (attn(24, 1, 64, 64, 64, 64), None), (attn(40, 4, 64, 64, 8, 77), moe(5, 2, 64)), (attn(9, 3, 192, 150, 64, 100), None)], 2, 3),
+    # one layer of near one-hot attention: what lies outside a chunk moves nothing
+    "edge37": config(64, 40, [(attn(8, 2, 64, 64, 32, 37), None)], 2, 2),
+    "edge64": config(64, 40, [(attn(6, 6, 48, 40, 32, 64), None)], 2, 2),
 }
-SHARP = {"deep": 6.0}
+SHARP = {"deep": 6.0, "edge37": 6.0, "edge64": 6.0}
 
 
 def weights(name, seed=0):
@@ -335,7 +341,7 @@ def test_table_experts(dtype):
 # ------------------------------------------------------------------------------------------------ GPU: whole models
 _models: dict = {}
 _refs: dict = {}
-every = pytest.mark.parametrize("name", list(CONFIGS))
+every = pytest.mark.parametrize("name", [c for c in CONFIGS if not c.startswith("edge")])
 
 
 @pytest.fixture(scope="module")
@@ -506,6 +512,39 @@ def test_unequal_batch_and_slots_used_again(models, name, dtype):
         for i in live:
             s.release((again, i))
     assert s.live == ()
+
+
+@gpu
+@both
+@pytest.mark.parametrize("name", ["edge37", "edge64"])
+def test_keys_at_chunk_edges(models, name, dtype):
+    """A token whose key stands out, put on a chunk's first position, moves the logits of the chunk's rows; put one before it, it moves none.
+    In prompts and in decoding over a ring that holds both sides of the edge."""
+    cfg, W, model = models(name, dtype)
+    C = cfg["layers"][0]["mixer"]["mask"]["size"]
+    t = tokens(cfg, 3 * C, 4)
+    base = R.forward(t, cfg, W)
+    rms = lambda a: np.sqrt(np.mean(np.square(a)))  # noqa: E731
+    e = model.build_engine(max_seq_len=3 * C, max_batch=1)
+
+    def both_ways(s, p):
+        """Row p of a prompt that goes on behind it, of one that ends there, and decoded."""
+        rows = [e.prefill_batch([s], want=[[p]])[0], e.prefill(s[:p + 1])]
+        e.prefill(s[:p], want_last_logits=False)
+        e.set_state([s[p]], [p])
+        e.decode_step(1)
+        return np.stack([*rows, e.logits(1).to_numpy()[0]])
+
+    for first in (C, 2 * C):
+        for p in (first + 1, first + C // 2, first + C - 1):
+            swap = lambda j, z: t[:j] + [z] + t[j + 1:]  # noqa: E731
+            z = max(range(cfg["vocab"]), key=lambda z: rms(R.forward(swap(first, z)[:p + 1], cfg, W)[p] - base[p]))
+            inside, outside = swap(first, z), swap(first - 1, z)
+            want = R.forward(inside, cfg, W)[p]
+            assert rms(want - base[p]) > 0.3 * rms(base)
+            assert rms(R.forward(outside, cfg, W)[p] - base[p]) == 0.0
+            assert near(both_ways(inside, p), np.stack([want] * 3), dtype, p), p
+            assert near(both_ways(outside, p), np.stack([base[p]] * 3), dtype, p), p
 
 
 @gpu
